@@ -13,9 +13,10 @@ Sampling defaults match the reference's hard-coded sampler
 from __future__ import annotations
 
 import dataclasses
+import math
 import os
 from dataclasses import dataclass, field
-from typing import Optional, Sequence, Tuple
+from typing import Optional, Sequence, Tuple, Union
 
 
 # ---------------------------------------------------------------------------
@@ -40,6 +41,163 @@ class LatentAttentionSpec:
         """Weight columns of `hidden` rows: q, out, and an own latent projection."""
         return self.heads * (self.dim + self.vdim) + (self.kv_rank if self.kv_from is None else 0)
 
+    @property
+    def cached_per_token(self) -> int:
+        return self.kv_rank if self.kv_from is None else 0
+
+    def params(self, hidden: int) -> int:
+        return hidden * self.params_per_hidden + self.heads * (self.dim + self.vdim) * self.kv_rank + self.cached_per_token
+
+    def check(self) -> None:
+        if min(self.heads, self.dim, self.vdim, self.kv_rank) < 1 or (self.window is not None and self.window < 1):
+            raise ValueError("attention sizes must be positive")
+
+
+@dataclass(frozen=True)
+class RopeScaling:
+    """Wavelengths above original / low are stretched by `factor`, those below
+    original / high stay, a linear ramp lies between."""
+
+    factor: float
+    low: float
+    high: float
+    original: float
+
+
+@dataclass(frozen=True)
+class RopeSpec:
+    """Rotation of the first `dims` dimensions of a head, pairs (i, i + dims / 2)."""
+
+    dims: int
+    base: float
+    scaling: Optional[RopeScaling] = None
+
+    def frequencies(self) -> list:
+        out = []
+        for i in range(self.dims // 2):
+            f = self.base ** (-2.0 * i / self.dims)
+            s = self.scaling
+            if s is not None:
+                turns = s.original * f / (2.0 * math.pi)  # original context in wavelengths
+                if turns < s.low:
+                    f /= s.factor
+                elif turns <= s.high:
+                    keep = (turns - s.low) / (s.high - s.low)
+                    f = (1.0 - keep) * f / s.factor + keep * f
+            out.append(f)
+        return out
+
+
+@dataclass(frozen=True)
+class AttentionSpec:
+    """Grouped-query attention over a paged K/V cache: partial rotation, capped
+    scores (softcap tanh(s / softcap)), and scores mixed over the heads by a
+    learned [heads, heads] matrix before the softmax (`talking`)."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: Optional[int] = None
+    rope: Optional[RopeSpec] = None
+    softcap: Optional[float] = None
+    talking: bool = True
+    kv_from: None = None
+
+    @property
+    def cached_per_token(self) -> int:
+        return self.kv_heads * (self.dim + self.vdim)
+
+    def params(self, hidden: int) -> int:
+        n = hidden * (self.heads * (self.dim + self.vdim) + self.kv_heads * (self.dim + self.vdim))
+        return n + (self.heads ** 2 if self.talking else 0)
+
+    def check(self) -> None:
+        if min(self.heads, self.kv_heads, self.dim, self.vdim) < 1 or (self.window is not None and self.window < 1):
+            raise ValueError("attention sizes must be positive")
+        if self.heads % self.kv_heads:
+            raise ValueError(f"{self.heads} heads cannot share {self.kv_heads} key / value heads evenly")
+        if self.rope is not None and (self.rope.dims % 2 or not 0 <= self.rope.dims <= self.dim):
+            raise ValueError(f"cannot rotate {self.rope.dims} of {self.dim} dimensions")
+        if self.softcap is not None and self.softcap <= 0:
+            raise ValueError("softcap must be positive")
+
+
+@dataclass(frozen=True)
+class ChannelDeltaSpec:
+    """Gated delta rule with one decay per head and key channel: a state
+    [dim, vdim] per head, a short convolution in front of q, k and v."""
+
+    heads: int
+    kv_heads: int                  # q / k heads; head h uses h // (heads / kv_heads)
+    dim: int
+    vdim: int
+    conv: int                      # taps
+    decay_rank: int                # inner width of the decay projection
+    gate_rank: int                 # ... and of the output gate's
+    kv_from: None = None
+    cached_per_token = 0
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+    def params(self, hidden: int) -> int:
+        o, hd = self.heads * self.vdim, self.heads * self.dim
+        n = hidden * (self.conv_channels + self.heads + self.decay_rank + self.gate_rank + o)
+        return n + self.conv_channels * self.conv + self.decay_rank * hd + self.gate_rank * o + hd + self.heads + self.vdim
+
+    def check(self) -> None:
+        if min(self.heads, self.kv_heads, self.dim, self.vdim, self.conv, self.decay_rank, self.gate_rank) < 1:
+            raise ValueError("delta rule sizes must be positive")
+        if self.heads % self.kv_heads:
+            raise ValueError(f"{self.heads} heads cannot share {self.kv_heads} key heads evenly")
+
+
+@dataclass(frozen=True)
+class SSMSpec:
+    """Mamba-2: a state [state, vdim] per head with one decay per head and
+    token; B and C shared by heads / groups heads, gated norm in norm_groups parts."""
+
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    norm_groups: int
+    conv: int
+    kv_from: None = None
+    cached_per_token = 0
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def conv_channels(self) -> int:
+        return self.inner + 2 * self.groups * self.state
+
+    def params(self, hidden: int) -> int:
+        n = hidden * (2 * self.inner + 2 * self.groups * self.state + self.heads + self.inner)
+        return n + self.conv_channels * (self.conv + 1) + 3 * self.heads + self.inner
+
+    def check(self) -> None:
+        if min(self.heads, self.vdim, self.state, self.groups, self.norm_groups, self.conv) < 1:
+            raise ValueError("state-space sizes must be positive")
+        if self.heads % self.groups or self.inner % self.norm_groups:
+            raise ValueError(f"{self.heads} heads in {self.groups} groups, width {self.inner} in "
+                             f"{self.norm_groups} norm groups: must divide evenly")
+
+
+@dataclass(frozen=True)
+class DenseSpec:
+    """Gated feed-forward W_down(gelu_tanh(W_gate h) * W_up h)."""
+
+    ff: int
+
+    def params(self, hidden: int) -> int:
+        return 3 * hidden * self.ff
+
 
 @dataclass(frozen=True)
 class ExpertSpec:
@@ -56,11 +214,25 @@ class MoESpec:
     expert: ExpertSpec
     shared: Optional[ExpertSpec] = None  # runs for every token
 
+    def params(self, hidden: int) -> int:
+        n = self.experts * (hidden + 1 + 3 * hidden * self.expert.ff)
+        return n + (3 * hidden * self.shared.ff if self.shared is not None else 0)
+
+
+MixerSpec = Union[LatentAttentionSpec, AttentionSpec, ChannelDeltaSpec, SSMSpec]
+
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: LatentAttentionSpec
-    mlp: Optional[MoESpec] = None
+    """One layer as it runs.  A loop over layers is written out: every pass has
+    entries of its own (and so its own cache or state), `weights` names the
+    layer whose tensors they share (None: its own), and `enter` is the pass
+    that begins in front of this entry (None: no pass begins here)."""
+
+    mixer: MixerSpec
+    mlp: Union[MoESpec, DenseSpec, None] = None
+    weights: Optional[int] = None
+    enter: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -69,11 +241,12 @@ class ModelConfig:
 
     GPT-2 and Llama have uniform layers: the scalar fields say everything.
     Models whose layers differ list them in `layers` (arch "timisun": parallel
-    blocks of latent attention and experts); the scalar head / ffn fields then
-    only describe the first layer."""
+    blocks of latent attention and experts; "vizalix": parallel blocks of
+    attention, delta rule or Mamba-2 and a dense feed-forward, some of them
+    looped); the scalar head / ffn fields then only describe the first layer."""
 
     name: str
-    arch: str  # "gpt2" | "llama" | "timisun"
+    arch: str  # "gpt2" | "llama" | "timisun" | "vizalix"
     vocab_size: int
     hidden: int
     n_layers: int
@@ -93,13 +266,35 @@ class ModelConfig:
     def parallel_block(self) -> bool:
         """Attention and MLP read the same normed input and are added together:
         a layer cannot be cut between them."""
-        return self.arch == "timisun"
+        return bool(self.layers)
 
     @property
     def paged_cache(self) -> bool:
         """The cache is a pool of token pages shared by the sequences
-        (runtime/kv_cache.py LatentCache) instead of a region per slot."""
-        return self.arch == "timisun"
+        (runtime/kv_cache.py PagedCache) instead of a region per slot."""
+        return bool(self.layers)
+
+    @property
+    def loop_times(self) -> int:
+        """Passes of the looped layers (0: no loop)."""
+        return max((l.enter + 1 for l in self.layers if l.enter is not None), default=0)
+
+    @property
+    def boundary(self) -> int:
+        """Columns a stage hands to the next: the residual, and the embedding
+        output where a loop's passes read it again."""
+        return self.hidden * (2 if self.loop_times else 1)
+
+    def weight_layer(self, i: int) -> int:
+        """The layer whose tensors layer i uses."""
+        return i if not self.layers or self.layers[i].weights is None else self.layers[i].weights
+
+    def stage_params(self, layers: Sequence[int]) -> int:
+        """Parameters a stage with these layers holds (shared ones once)."""
+        n = sum(self.layer_params(i) for i in {self.weight_layer(i): i for i in layers}.values())
+        if any(self.layers and self.layers[i].enter is not None for i in layers):
+            n += 2 * self.hidden * self.hidden + self.loop_times * self.hidden
+        return n
 
     def cache_layers(self, layers: Sequence[int]) -> list:
         """Those of `layers` that own a cache (others share an earlier one)."""
@@ -133,14 +328,8 @@ class ModelConfig:
         if not self.layers:
             return self.block_params()
         h, m, f = self.hidden, self.layers[i].mixer, self.layers[i].mlp
-        n = h + h * m.params_per_hidden + m.heads * (m.dim + m.vdim) * m.kv_rank
-        if m.kv_from is None:
-            n += m.kv_rank
-        if f is not None:
-            n += f.experts * (h + 1 + 3 * h * f.expert.ff)
-            if f.shared is not None:
-                n += 3 * h * f.shared.ff
-        return n
+        norms = h if self.arch == "timisun" else 1 + (f is not None)
+        return norms + m.params(h) + (f.params(h) if f is not None else 0)
 
     def block_params(self) -> int:
         """Parameters of a layer (of the mean layer when they differ)."""
@@ -162,8 +351,7 @@ class ModelConfig:
 
     def kv_bytes_per_token_per_layer(self, dtype_bytes: int = 2) -> int:
         if self.layers:
-            own = self.cache_layers(range(self.n_layers))
-            return sum(self.layers[i].mixer.kv_rank for i in own) * dtype_bytes // self.n_layers
+            return sum(l.mixer.cached_per_token for l in self.layers) * dtype_bytes // self.n_layers
         return 2 * self.kv_size * dtype_bytes
 
 
@@ -218,15 +406,19 @@ def check_layers(layers: Sequence[LayerSpec]) -> None:
         raise ValueError("a model needs at least one layer")
     for i, l in enumerate(layers):
         m, f = l.mixer, l.mlp
-        if min(m.heads, m.dim, m.vdim, m.kv_rank) < 1 or (m.window is not None and m.window < 1):
-            raise ValueError(f"layer {i}: attention sizes must be positive")
+        try:
+            m.check()
+        except ValueError as e:
+            raise ValueError(f"layer {i}: {e}") from None
         if m.kv_from is not None:
             j = m.kv_from
             if not 0 <= j < i or layers[j].mixer.kv_from is not None or layers[j].mixer.kv_rank != m.kv_rank:
                 raise ValueError(f"layer {i}: kv_from {j} must name an earlier layer with its own latents of "
                                  f"rank {m.kv_rank}")
-        if f is not None and not 1 <= f.top <= f.experts:
+        if isinstance(f, MoESpec) and not 1 <= f.top <= f.experts:
             raise ValueError(f"layer {i}: top must be in [1, experts]")
+        if isinstance(f, DenseSpec) and f.ff < 1:
+            raise ValueError(f"layer {i}: feed-forward width must be positive")
 
 
 def _timisun_layers(n: int, share: int = 2, experts: int = 16, **kw) -> list:
@@ -249,6 +441,54 @@ MODEL_PRESETS.update({
     "timisun-8b": _timisun("timisun-8b", 32000, 4096, _timisun_layers(
         6, heads=32, dim=128, vdim=128, kv_rank=256, scale=128 ** -0.5, window=1024, experts=32, top=4, ff=2048,
         shared_ff=4096)),
+})
+
+def unroll(layers: Sequence[LayerSpec], start: int, stop: int, times: int) -> list:
+    """Layers start .. stop - 1 run `times` times in a row, written out."""
+    if not (0 <= start < stop <= len(layers) and times >= 1):
+        raise ValueError(f"loop over layers {start} .. {stop - 1}, {times} times: outside the {len(layers)} layers")
+    rep = dataclasses.replace
+    out = [rep(l, weights=i) for i, l in enumerate(layers[:start])]
+    for t in range(times):
+        out += [rep(layers[i], weights=i, enter=t if i == start else None) for i in range(start, stop)]
+    return out + [rep(layers[i], weights=i) for i in range(stop, len(layers))]
+
+
+def _vizalix(name: str, vocab: int, width: int, layers: Sequence[LayerSpec], loop: Optional[Tuple[int, int, int]] = None,
+             eps: float = 1e-6) -> ModelConfig:
+    check_layers(layers)
+    runs = tuple(unroll(layers, *loop) if loop else layers)
+    first = layers[0]
+    return ModelConfig(
+        name=name, arch="vizalix", vocab_size=vocab, hidden=width, n_layers=len(runs), n_heads=first.mixer.heads,
+        n_kv_heads=getattr(first.mixer, "kv_heads", 1), ffn=first.mlp.ff if first.mlp else 0,
+        max_positions=1 << 20,  # rows of the rotation tables
+        norm_eps=eps, tie_embeddings=False, bos_token_id=0, eos_token_id=-1, layers=runs)
+
+
+def _vizalix_layers(ff: int, delta: dict, attention: dict, ssm: dict, repeat: int = 1) -> list:
+    """delta rule, attention, Mamba-2, `repeat` times."""
+    mixers = (ChannelDeltaSpec(**delta), AttentionSpec(**attention), SSMSpec(**ssm))
+    return [LayerSpec(m, DenseSpec(ff)) for m in mixers * repeat]
+
+
+_VIZALIX_ROPE = RopeSpec(64, 500000.0, RopeScaling(8.0, 1.0, 4.0, 8192))
+MODEL_PRESETS.update({
+    # Vizalix: small test sizes (none a multiple of the GEMM tiles), and two
+    # sizes that resemble the layers of models that are served today
+    "vizalix-test": _vizalix("vizalix-test", 300, 104, _vizalix_layers(
+        72, dict(heads=4, kv_heads=2, dim=24, vdim=20, conv=3, decay_rank=10, gate_rank=6),
+        dict(heads=6, kv_heads=3, dim=40, vdim=24, scale=0.2, window=90, softcap=20.0,
+             rope=RopeSpec(24, 10000.0, RopeScaling(4.0, 1.0, 4.0, 256))),
+        dict(heads=6, vdim=20, state=24, groups=2, norm_groups=2, conv=4)), loop=(0, 2, 2)),
+    "vizalix-2b": _vizalix("vizalix-2b", 32000, 2048, _vizalix_layers(
+        5632, dict(heads=16, kv_heads=16, dim=128, vdim=128, conv=4, decay_rank=128, gate_rank=128),
+        dict(heads=16, kv_heads=4, dim=128, vdim=128, scale=128 ** -0.5, window=1024, softcap=50.0, rope=_VIZALIX_ROPE),
+        dict(heads=64, vdim=64, state=128, groups=1, norm_groups=1, conv=4), repeat=2), loop=(0, 3, 2)),
+    "vizalix-8b": _vizalix("vizalix-8b", 32000, 4096, _vizalix_layers(
+        14336, dict(heads=32, kv_heads=32, dim=128, vdim=128, conv=4, decay_rank=128, gate_rank=128),
+        dict(heads=32, kv_heads=8, dim=128, vdim=128, scale=128 ** -0.5, window=1024, softcap=50.0, rope=_VIZALIX_ROPE),
+        dict(heads=128, vdim=64, state=128, groups=8, norm_groups=8, conv=4)), loop=(0, 3, 2)),
 })
 
 _ALIASES = {
@@ -299,11 +539,65 @@ def _timisun_from_json(c: dict, name: str) -> ModelConfig:
                     embed_scale=float(c["embedding"]["scale"]))
 
 
+def _vizalix_from_json(c: dict, name: str, shape) -> ModelConfig:
+    """The design's own config.json; `shape(tensor name)` gives the two sizes
+    that only the checkpoint's tensors have (ranks of the delta rule's decay
+    and gate projections)."""
+    layers = []
+    for i, l in enumerate(c["layers"]):
+        m, f = l["mixer"], l.get("mlp")
+        if l["type"] == "channel_delta":
+            mix = ChannelDeltaSpec(
+                heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"], conv=m["conv"],
+                decay_rank=shape(f"l{i}.mix.a1")[0], gate_rank=shape(f"l{i}.mix.g1")[0])
+        elif l["type"] == "attention":
+            r = m.get("rot") or {}
+            s = r.get("scaling")
+            rope = RopeSpec(r["dims"], float(r["base"]), RopeScaling(
+                float(s["factor"]), float(s["low"]), float(s["high"]), float(s["original"])) if s else None) if r else None
+            cap = m.get("softcap")
+            mix = AttentionSpec(
+                heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"], scale=float(m["scale"]),
+                window=(m.get("mask") or {}).get("size"), rope=rope, softcap=float(cap) if cap else None)
+        elif l["type"] == "mamba2":
+            mix = SSMSpec(heads=m["heads"], vdim=m["vdim"], state=m["state"], groups=m["groups"],
+                          norm_groups=m["norm_groups"], conv=m["conv"])
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {l['type']!r}")
+        if f and f.get("kind", "dense") != "dense":
+            raise ValueError(f"layer {i}: unknown feed-forward {f['kind']!r}")
+        layers.append(LayerSpec(mix, DenseSpec(f["ff"]) if f else None))
+    lp = c.get("loop")
+    return _vizalix(name, c["vocab"], c["width"], layers, loop=(lp["start"], lp["stop"], lp["times"]) if lp else None,
+                    eps=float(c["norm"]["eps"]))
+
+
+def _checkpoint_shapes(folder: str):
+    """name -> shape of the tensors in a folder's safetensors files (headers only)."""
+    import json
+
+    shapes = {}
+    for fn in sorted(os.listdir(folder)):
+        if fn.endswith(".safetensors"):
+            with open(os.path.join(folder, fn), "rb") as f:
+                n = int.from_bytes(f.read(8), "little")
+                shapes.update((k, tuple(v["shape"])) for k, v in json.loads(f.read(n)).items() if "shape" in v)
+
+    def shape(name: str) -> tuple:
+        if name not in shapes:
+            raise ValueError(f"{folder}: no tensor {name!r} beside config.json to read a size from")
+        return shapes[name]
+    return shape
+
+
 def model_config_from_hf_json(path: str) -> ModelConfig:
     import json
 
     with open(path) as f:
         c = json.load(f)
+    if c.get("architecture") == "Vizalix":
+        folder = os.path.dirname(os.path.abspath(path))
+        return _vizalix_from_json(c, os.path.basename(folder) or "vizalix", _checkpoint_shapes(folder))
     if c.get("architecture") == "Timisun":
         return _timisun_from_json(c, os.path.basename(os.path.dirname(os.path.abspath(path))) or "timisun")
     mt = c.get("model_type", "gpt2")

@@ -1,4 +1,4 @@
-"""One pipeline stage of a GPT-2, Llama or Timisun model.
+"""One pipeline stage of a GPT-2, Llama, Timisun or Vizalix model.
 
 Generalises the reference's two hard-wired shards (`server.py:51-105`):
   * ShardA (`server.py:68-86`): wte + wpe + blocks[0:split]   -> stage 0
@@ -25,8 +25,8 @@ import torch
 from ..config import ModelConfig
 from ..ops import Residual, get_backend
 from ..runtime.batch import BatchMeta
-from ..runtime.kv_cache import KVCache, LatentCache
-from .weights import layer_half, maybe_load
+from ..runtime.kv_cache import KVCache, LatentCache, PagedCache
+from .weights import layer_half, maybe_load, stage_tensor_shapes
 
 
 class StageModel:
@@ -75,6 +75,9 @@ class StageModel:
         self.backend = backend if backend is not None else get_backend(self.device)
         # columns of the residual rows (hidden, or padded by the backend)
         self.row_width = self.backend.row_width(cfg)
+        # columns that cross a stage boundary: where a loop's passes read the
+        # embedding output again, it travels beside the residual
+        self.wire_width = self.row_width * (2 if cfg.loop_times else 1)
         if cfg.parallel_block and (ua % 2 or ub % 2):
             raise ValueError(f"{cfg.name}: parallel layers cannot be cut in half (units {units})")
         if cfg.paged_cache:
@@ -86,8 +89,11 @@ class StageModel:
                     raise ValueError(f"layer {i} shares layer {j}'s cache: both must be on one stage")
             if pages is None:  # no page allocator in front: every slot owns its pages
                 pages, reserved_slots = 0, range(max_slots)
-            self.kv = LatentCache([self.backend.latent_width(cfg.layers[i].mixer.kv_rank) for i in own], max_slots,
-                                  pages, self.max_seq, dtype, self.device, reserved=reserved_slots)
+            args = (max_slots, pages, self.max_seq, dtype, self.device, reserved_slots)
+            if cfg.arch == "timisun":
+                self.kv = LatentCache([self.backend.latent_width(cfg.layers[i].mixer.kv_rank) for i in own], *args)
+            else:
+                self.kv = PagedCache([self.backend.layer_cache(cfg.layers[i].mixer) for i in own], *args)
         else:
             self.kv = KVCache(len(self.kv_layers), max_slots, cfg.n_kv_heads, self.max_seq,
                               cfg.head_dim, dtype, self.device)
@@ -95,6 +101,8 @@ class StageModel:
 
     def _owns(self, name: str) -> bool:
         """Is tensor `name` used by this stage (its units, embeddings, head)?"""
+        if self.cfg.arch == "vizalix":
+            return name in stage_tensor_shapes(self.cfg, self.layers, self.first, self.last)
         lh = layer_half(name)
         if lh is None:
             emb = name in ("wte", "wpe", "embed_tokens")
@@ -163,6 +171,33 @@ class StageModel:
         o = be.latent_attention(q, w, m, self.kv, pool, meta)
         be.parallel_residual(o, h, routing, w, spec.mlp, r)
 
+    # Vizalix: mixer and feed-forward of the same residual, each behind a norm
+    # with one number for a gain -- applied after the projections that follow,
+    # so both read the same normed rows
+    def _mixer_layer(self, i: int, r: Residual, x0, meta: BatchMeta) -> None:
+        be, c, spec = self.backend, self.cfg, self.cfg.layers[i]
+        if spec.enter is not None:  # a pass of the loop begins: x <- W_in [x; x0] + step
+            be.loop_enter(r, x0, self.w["loop.in"], self.w["loop.step"], spec.enter)
+        w = functools.partial(self._lw, c.weight_layer(i))
+        h = be.unit_rmsnorm(r, c)
+        o = be.mix(h, w, spec, self.kv, self.kv.entries[self._pool_index[i]], meta, c.norm_eps)
+        be.mixer_residual(o, h, w, spec, r)
+
+    # -- stage boundaries: [x | x0] where the loop's passes need x0, else x ------
+    def _unpack(self, rows: torch.Tensor):
+        if self.wire_width == self.row_width:
+            return rows, None
+        return rows[:, : self.row_width].contiguous(), rows[:, self.row_width:].contiguous()
+
+    def boundary_rows(self, rows: torch.Tensor) -> torch.Tensor:
+        """Rows as they leave the stage -> the model's own columns (compat forwards)."""
+        return torch.cat([p[:, : self.cfg.hidden] for p in rows.split(self.row_width, 1)], 1)
+
+    def wire_rows(self, rows: torch.Tensor) -> torch.Tensor:
+        """Inverse of boundary_rows: padded as the backend wants them."""
+        pad = (0, self.row_width - self.cfg.hidden)
+        return torch.cat([torch.nn.functional.pad(p, pad) for p in rows.split(self.cfg.hidden, 1)], 1)
+
     # ------------------------------------------------------------------
     def embed(self, ids: torch.Tensor, meta: BatchMeta) -> torch.Tensor:
         if self.cfg.arch == "gpt2":
@@ -184,7 +219,13 @@ class StageModel:
         `variant`: which of the stage's unit ranges to run (the microbatch
         group's parity under alternating splits; 0 otherwise).  `residuals`
         collects the residual rows after every parallel layer (debugging)."""
-        x = self.embed(inp, meta) if self.first else inp
+        x0 = None
+        if self.first:
+            x = self.embed(inp, meta)
+            if self.wire_width != self.row_width:
+                x0 = self.embed(inp, meta)  # the residual is updated in place
+        else:
+            x, x0 = self._unpack(inp)
         r = Residual(x)
         # decode-only routing rules (ops/hip.py); a mixed step's rows follow them up to 512
         self.backend.decode = getattr(meta, "routing_decode", meta.is_decode) and meta.num_tokens <= 512 \
@@ -197,7 +238,10 @@ class StageModel:
             i = u >> 1
             if self.cfg.parallel_block:  # a whole layer: its second unit is empty
                 if not u & 1:
-                    self._parallel_layer(i, r, meta)
+                    if self.cfg.arch == "timisun":
+                        self._parallel_layer(i, r, meta)
+                    else:
+                        self._mixer_layer(i, r, x0, meta)
                     if residuals is not None:
                         residuals.append(self.backend.flush(r)[:, : self.cfg.hidden].clone())
                 continue
@@ -207,7 +251,7 @@ class StageModel:
                 attn_fn(self._kv_index[i], i, r, meta)
         x = self.backend.flush(r)
         if not (self.last and head):
-            return x
+            return x if x0 is None or self.last else torch.cat([x, x0], 1)
         return self.head(x, meta, all_logits, head_rows)
 
     def head(self, x: torch.Tensor, meta: BatchMeta, all_logits: bool = False,
@@ -217,6 +261,8 @@ class StageModel:
             rows = None if (all_logits or meta.is_decode) else meta.last_idx  # last query per sequence
         if c.arch == "timisun":
             xn = be.norm_rows(x, self.w["norm.weight"], None, c.norm_eps, True, rows, offset=1.0, width=c.hidden)
+        elif c.arch == "vizalix":
+            xn = be.norm_rows(x, self.w["norm.weight"], None, c.norm_eps, True, rows, width=be.norm_width(c))
         elif c.arch == "gpt2":
             xn = be.norm_rows(x, self.w["ln_f.weight"], self.w["ln_f.bias"], c.norm_eps, False, rows)
         else:

@@ -25,7 +25,7 @@ from typing import Dict, Iterable, Optional, Tuple
 
 import torch
 
-from ..config import ModelConfig
+from ..config import ChannelDeltaSpec, ModelConfig, SSMSpec
 
 
 def _seed(seed: int, name: str) -> int:
@@ -95,7 +95,35 @@ def _timisun_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
     return out
 
 
-_ATTN_PARTS = ("ln_1.", "attn.", "input_layernorm.", "self_attn.")
+def _vizalix_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
+    """Tensors of layer i (named by the layer that owns them)."""
+    h, m, f = cfg.hidden, cfg.layers[i].mixer, cfg.layers[i].mlp
+    p = f"layers.{cfg.weight_layer(i)}."
+    out = {p + "input_layernorm.weight": ()}  # one number for all coordinates
+    if isinstance(m, ChannelDeltaSpec):
+        qk, v = m.kv_heads * m.dim, m.heads * m.vdim
+        mix = {"q": (qk, h), "k": (qk, h), "v": (v, h), "q.conv": (qk, m.conv), "k.conv": (qk, m.conv),
+               "v.conv": (v, m.conv), "b": (m.heads, h), "A_log": (m.heads,), "dt_bias": (m.heads * m.dim,),
+               "a1": (m.decay_rank, h), "a2": (m.heads * m.dim, m.decay_rank), "g1": (m.gate_rank, h),
+               "g2": (v, m.gate_rank), "norm": (m.vdim,), "o": (h, v)}
+    elif isinstance(m, SSMSpec):
+        mix = {"in": (m.inner + m.conv_channels + m.heads, h), "conv": (m.conv_channels, m.conv),
+               "conv.b": (m.conv_channels,), "dt_bias": (m.heads,), "A_log": (m.heads,), "D": (m.heads,),
+               "norm": (m.inner,), "o": (h, m.inner)}
+    else:
+        mix = {"q": (m.heads * m.dim, h), "k": (m.kv_heads * m.dim, h), "v": (m.kv_heads * m.vdim, h),
+               "o": (h, m.heads * m.vdim)}
+        if m.talking:
+            mix["talk"] = (m.heads, m.heads)
+    out.update((p + "mixer." + n, s) for n, s in mix.items())
+    if f is not None:
+        out[p + "post_attention_layernorm.weight"] = ()
+        out[p + "mlp.gate_up.weight"] = (2 * f.ff, h)  # gate rows | up rows
+        out[p + "mlp.down_proj.weight"] = (h, f.ff)
+    return out
+
+
+_ATTN_PARTS = ("ln_1.", "attn.", "input_layernorm.", "self_attn.", "mixer.")
 _MLP_PARTS = ("ln_2.", "mlp.", "post_attention_layernorm.")
 
 
@@ -129,6 +157,8 @@ def stage_tensor_shapes(cfg: ModelConfig, layers: Iterable[int], first: bool, la
                         units: Optional[Tuple[int, int]] = None):
     """Tensors a stage materialises; with `units` only the halves of the
     boundary layers that the stage runs."""
+    if cfg.arch == "vizalix":  # whole layers, several of which may share their tensors
+        return _stage_tensor_shapes(cfg, layers, first, last)
     return _filter_units(_stage_tensor_shapes(cfg, layers, first, last), units)
 
 
@@ -141,6 +171,17 @@ def _stage_tensor_shapes(cfg: ModelConfig, layers: Iterable[int], first: bool, l
             shapes.update(_timisun_shapes(cfg, i))
         if last:
             shapes["norm.weight"] = (cfg.hidden,)
+    elif cfg.arch == "vizalix":
+        if first:
+            shapes["embed_tokens"] = (cfg.vocab_size, cfg.hidden)
+        for i in layers:
+            shapes.update(_vizalix_shapes(cfg, i))
+            if cfg.layers[i].enter is not None:
+                shapes["loop.in"] = (cfg.hidden, 2 * cfg.hidden)
+                shapes["loop.step"] = (cfg.loop_times, cfg.hidden)
+        if last:
+            shapes["norm.weight"] = ()
+            shapes["lm_head"] = (cfg.vocab_size, cfg.hidden)
     elif cfg.arch == "gpt2":
         if first:
             shapes["wte"] = (cfg.vocab_size, cfg.hidden)
@@ -166,6 +207,8 @@ def _init_one(cfg: ModelConfig, name: str, shape, seed: int, device, dtype) -> t
     base = name.rsplit(".", 1)[-1]
     if cfg.arch == "timisun":
         return _timisun_init(cfg, name, shape, seed, device, dtype)
+    if cfg.arch == "vizalix":
+        return _vizalix_init(cfg, name, shape, seed, device, dtype)
     if name == "embed_tokens":
         # untied (Llama) input embeddings at unit scale (the T5 / muP
         # convention: the residual stream enters at the RMS its norms produce).
@@ -210,6 +253,32 @@ def _timisun_init(cfg: ModelConfig, name: str, shape, seed: int, device, dtype) 
         for e in range(shape[0]):
             out[e] = _randn(shape[1:], std, seed, f"{name}.{e}", device, dtype)
         return out
+    return _randn(shape, std, seed, name, device, dtype)
+
+
+def _vizalix_init(cfg: ModelConfig, name: str, shape, seed: int, device, dtype) -> torch.Tensor:
+    """Unit-variance projections, depth-scaled residual ones; decays between
+    slow and fast, head mixing near the identity."""
+    def around(mean, std):
+        return (mean + _randn(shape, std, seed, name, device, torch.float32)).to(dtype)
+
+    leaf = name.split(".", 2)[-1] if name.startswith("layers.") else name
+    if leaf == "embed_tokens":
+        return _randn(shape, 1.0, seed, name, device, dtype)
+    if leaf.endswith(("norm.weight", "layernorm.weight", "mixer.norm", "mixer.D")):
+        return around(1.0, 0.05)
+    if leaf == "mixer.A_log":
+        return around(0.5, 0.7)
+    if leaf == "mixer.dt_bias":
+        return around(-3.0, 1.0)
+    if leaf == "mixer.talk":
+        return (torch.eye(shape[0], device=device) + _randn(shape, 0.3 * shape[0] ** -0.5, seed, name, device,
+                                                            torch.float32)).to(dtype)
+    if leaf in ("mixer.conv.b", "loop.step"):
+        return _randn(shape, 0.1, seed, name, device, dtype)
+    std = shape[-1] ** -0.5
+    if leaf in ("mixer.o", "mlp.down_proj.weight"):
+        std /= (2 * cfg.n_layers) ** 0.5
     return _randn(shape, std, seed, name, device, dtype)
 
 
@@ -284,6 +353,21 @@ def _timisun_tensor(cfg: ModelConfig, name: str, get) -> torch.Tensor:
     return torch.stack([part(f"{p}e{e}.") for e in range(cfg.layers[int(i)].mlp.experts)])
 
 
+def _vizalix_tensor(name: str, get) -> torch.Tensor:
+    """One canonical tensor from a checkpoint in the design's own names."""
+    top = {"embed_tokens": "embed", "norm.weight": "final.norm", "lm_head": "head", "loop.in": "loop.in",
+           "loop.step": "loop.step"}
+    if name in top:
+        return get(top[name])
+    _, i, rest = name.split(".", 2)
+    if rest.startswith("mixer."):
+        return get(f"l{i}.mix." + rest[len("mixer."):])
+    if rest == "mlp.gate_up.weight":
+        return torch.cat([get(f"l{i}.mlp.gate"), get(f"l{i}.mlp.up")], 0)
+    return get(f"l{i}." + {"input_layernorm.weight": "norm1", "post_attention_layernorm.weight": "norm2",
+                           "mlp.down_proj.weight": "mlp.down"}[rest])
+
+
 def load_stage_weights(cfg: ModelConfig, path: str, layers, first: bool, last: bool,
                        device, dtype, units=None) -> Dict[str, torch.Tensor]:
     get, keys = _open_checkpoint(path)
@@ -299,6 +383,8 @@ def load_stage_weights(cfg: ModelConfig, path: str, layers, first: bool, last: b
     for name, shape in want.items():
         if cfg.arch == "timisun":
             t = _timisun_tensor(cfg, name, get)
+        elif cfg.arch == "vizalix":
+            t = _vizalix_tensor(name, get)
         elif cfg.arch == "gpt2":
             src = {"wte": "wte.weight", "wpe": "wpe.weight"}.get(name, name)
             t = find(src)

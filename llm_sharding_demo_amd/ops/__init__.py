@@ -23,6 +23,8 @@ from typing import List, Optional, Tuple
 
 import torch
 
+from ..config import AttentionSpec, ChannelDeltaSpec
+from ..runtime.kv_cache import LayerCache, layer_cache
 from . import reference as ref
 
 
@@ -49,6 +51,14 @@ class Backend:
     def latent_width(self, rank: int) -> int:
         """Columns of a cached latent row (>= rank; the rest stays zero)."""
         return rank
+
+    def layer_cache(self, mixer) -> LayerCache:
+        """What a layer keeps per page and per slot (runtime/kv_cache.py)."""
+        return layer_cache(mixer)
+
+    def norm_width(self, mcfg) -> int:
+        """`width` argument of the norms: the true row width where rows are padded, else 0."""
+        return mcfg.hidden if self.row_width(mcfg) != mcfg.hidden else 0
 
     def prepare_prefill(self, meta, mcfg) -> None:
         """Device-side helpers of a prefill batch, made before a graph capture."""
@@ -127,6 +137,83 @@ class ReferenceBackend(Backend):
             y = y + ref.expert(h, w("mlp.shared.gate_up.weight"), w("mlp.shared.down.weight"), spec.shared.limit,
                                GLU_ALPHA)
         r.x += y
+
+    # -- mixers of models/stage.py _mixer_layer --------------------------------
+    def loop_enter(self, r: Residual, x0, w_in, step, t: int) -> None:
+        """x <- W_in [x; x0] + step[t]: a pass of the looped layers begins."""
+        self._combine(r)
+        r.x.copy_(ref.linear(torch.cat([r.x, x0], 1), w_in) + step[t].float())
+
+    def unit_rmsnorm(self, r: Residual, mcfg):
+        self._combine(r)
+        return ref.rmsnorm(r.x, r.x.new_ones(r.x.shape[1]), mcfg.norm_eps)
+
+    def mix(self, h, w, spec, kv, entry, meta, eps):
+        """Mixer output before W_o [T, heads * vdim] fp32; `entry`: the layer's
+        cache tensors (kv.entries)."""
+        m = spec.mixer
+        h = h * w("input_layernorm.weight").float()
+        fn = (self._attend if isinstance(m, AttentionSpec) else
+              self._channel_delta if isinstance(m, ChannelDeltaSpec) else self._ssm)
+        return fn(h, w, m, kv, entry, meta, eps)
+
+    @staticmethod
+    def _parts(meta):
+        """(rows, meta) of a step's decode rows and prompt chunks."""
+        if getattr(meta, "dec", None) is not None:
+            return [(slice(0, meta.b), meta.dec), (slice(meta.b, meta.num_tokens), meta.pf)]
+        return [(slice(0, meta.num_tokens), meta)]
+
+    def _attend(self, h, w, m, kv, entry, meta, eps):
+        pos = meta.token_pos
+        q = ref.partial_rope(ref.linear(h, w("mixer.q")).reshape(-1, m.heads, m.dim), pos, m.rope)
+        k = ref.partial_rope(ref.linear(h, w("mixer.k")).reshape(-1, m.kv_heads, m.dim), pos, m.rope)
+        v = ref.linear(h, w("mixer.v")).reshape(-1, m.kv_heads, m.vdim)
+        for pool, x in zip(entry, (k, v)):
+            ref.paged_append(pool, kv.table, x, meta.token_slots, pos)
+        talk = w("mixer.talk") if m.talking else None
+        o = torch.cat([ref.talking_attention(q[s], entry[0], entry[1], kv.table, mt.seq_slots, mt.q_start, mt.cu_q,
+                                             talk, m.scale, m.softcap, m.window) for s, mt in self._parts(meta)])
+        return o.reshape(o.shape[0], -1)
+
+    def _channel_delta(self, h, w, m, kv, entry, meta, eps):
+        T, H, G, D, V = h.shape[0], m.heads, m.kv_heads, m.dim, m.vdim
+        x = torch.cat([ref.linear(h, w(f"mixer.{n}")) for n in "qkv"], 1)
+        taps = torch.cat([w(f"mixer.{n}.conv") for n in "qkv"])
+        dt = ref.linear(ref.linear(h, w("mixer.a1")), w("mixer.a2")) + w("mixer.dt_bias").float()
+        g = torch.exp(-torch.exp(w("mixer.A_log").float())[:, None] * torch.nn.functional.softplus(dt).view(T, H, D))
+        beta = torch.sigmoid(ref.linear(h, w("mixer.b")))
+        o = torch.empty(T, H, V)
+        for s, mt in self._parts(meta):
+            y = torch.nn.functional.silu(ref.ring_conv(x[s], taps, None, entry[1], mt))
+            q, k, v = y.split([G * D, G * D, H * V], 1)
+            q, k = (ref.unit(u.reshape(-1, G, D)).repeat_interleave(H // G, 1) for u in (q, k))
+            o[s] = ref.delta_rule(q * D ** -0.5, k, v.reshape(-1, H, V), g[s], beta[s], entry[0], mt)
+        o = ref.rmsnorm(o, w("mixer.norm"), eps)
+        return o.view(T, H * V) * torch.sigmoid(ref.linear(ref.linear(h, w("mixer.g1")), w("mixer.g2")))
+
+    def _ssm(self, h, w, m, kv, entry, meta, eps):
+        T, H, G, V, N = h.shape[0], m.heads, m.groups, m.vdim, m.state
+        z, x, dt = ref.linear(h, w("mixer.in")).split([m.inner, m.conv_channels, H], 1)
+        dt = torch.nn.functional.softplus(dt + w("mixer.dt_bias").float())
+        decay = torch.exp(-torch.exp(w("mixer.A_log").float()) * dt)
+        y = torch.empty(T, H, V)
+        for s, mt in self._parts(meta):
+            c = torch.nn.functional.silu(ref.ring_conv(x[s], w("mixer.conv"), w("mixer.conv.b"), entry[1], mt))
+            u, B, C = c.split([m.inner, G * N, G * N], 1)
+            B, C = (t.reshape(-1, G, N).repeat_interleave(H // G, 1) for t in (B, C))
+            u = u.reshape(-1, H, V)
+            y[s] = ref.ssd(u, B, C, dt[s], decay[s], entry[0], mt) + w("mixer.D").float()[:, None] * u
+        y = (y.view(T, -1) * torch.nn.functional.silu(z)).view(T, m.norm_groups, -1)
+        return ref.rmsnorm(y, y.new_ones(y.shape[-1]), eps).view(T, -1) * w("mixer.norm").float()
+
+    def mixer_residual(self, o, h, w, spec, r: Residual) -> None:
+        """x += o W_o^T + feed-forward(h): both halves of a parallel block."""
+        self.linear_residual(o, w("mixer.o"), None, r)
+        if spec.mlp is not None:
+            y = ref.linear(h * w("post_attention_layernorm.weight").float(), w("mlp.gate_up.weight"))
+            f = y.shape[1] // 2
+            self.linear_residual(ref.gelu_new(y[:, :f]) * y[:, f:], w("mlp.down_proj.weight"), None, r)
 
     def qkv_kv_append(self, xn, w, b, cache_k, cache_v, meta, mcfg):
         """QKV projection; K,V appended to the cache at (slot, pos); returns q [T, nh, hd]."""

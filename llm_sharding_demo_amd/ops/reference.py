@@ -21,6 +21,7 @@ from typing import Optional
 import torch
 import torch.nn.functional as F
 
+UNIT_EPS = 1e-6  # inside the root of a unit vector's length (fixed by the design)
 _GELU_C = math.sqrt(2.0 / math.pi)
 
 
@@ -150,6 +151,110 @@ def latent_attention(q: torch.Tensor, pool: torch.Tensor, table: torch.Tensor, s
         hide = d < 0 if window is None else (d < 0) | (d >= window)
         p = torch.softmax(s.masked_fill(hide, float("-inf")), dim=-1)
         out[a:b] = torch.matmul(p, c).transpose(0, 1)
+    return out
+
+
+def partial_rope(x: torch.Tensor, pos: torch.Tensor, rope) -> torch.Tensor:
+    """x [T, heads, dim]: pairs (i, i + dims / 2) of the first rope.dims dimensions turn."""
+    if rope is None or rope.dims == 0:
+        return x
+    half = rope.dims // 2
+    ang = pos.double()[:, None] * torch.tensor(rope.frequencies(), dtype=torch.float64, device=pos.device)
+    cos, sin = ang.cos().float()[:, None], ang.sin().float()[:, None]
+    a, b = x[..., :half].float(), x[..., half: 2 * half].float()
+    return torch.cat([a * cos - b * sin, b * cos + a * sin, x[..., 2 * half:].float()], -1)
+
+
+def paged_append(pool: torch.Tensor, table: torch.Tensor, x: torch.Tensor, slots, pos) -> None:
+    """pool [pages, heads, page, dim]; x [T, heads, dim]."""
+    page = pool.shape[2]
+    pg = table[slots.long(), pos.long() // page].long()
+    pool[pg, :, pos.long() % page] = x.to(pool.dtype)
+
+
+def talking_attention(q, k_pool, v_pool, table, seq_slots, q_start, cu_q, talk, scale: float,
+                      softcap: Optional[float], window: Optional[int]) -> torch.Tensor:
+    """q [T, heads, dim] over paged keys and values [pages, kv heads, page, .]:
+    scores are capped, mixed over the heads (talk [heads, heads]) and softmaxed
+    over i - window < j <= i.  Returns fp32 [T, heads, vdim]."""
+    T, H, _ = q.shape
+    page, grp = k_pool.shape[2], H // k_pool.shape[1]
+    out = torch.empty(T, H, v_pool.shape[3], dtype=torch.float32, device=q.device)
+    for i in range(seq_slots.numel()):
+        a, b = int(cu_q[i]), int(cu_q[i + 1])
+        if b == a:
+            continue
+        st, end = int(q_start[i]), int(q_start[i]) + b - a
+        lo = 0 if window is None else max(0, st - window + 1)
+        kpos = torch.arange(lo, end, device=q.device)
+        pg = table[int(seq_slots[i]), kpos // page].long()
+        k, v = (p[pg, :, kpos % page].float().transpose(0, 1).repeat_interleave(grp, 0) for p in (k_pool, v_pool))
+        s = torch.matmul(q[a:b].float().transpose(0, 1), k.transpose(1, 2)) * scale  # [heads, Lq, keys]
+        if softcap is not None:
+            s = softcap * torch.tanh(s / softcap)
+        if talk is not None:
+            s = torch.matmul(talk.float(), s.reshape(H, -1)).view_as(s)
+        d = torch.arange(st, end, device=q.device)[:, None] - kpos[None, :]
+        hide = d < 0 if window is None else (d < 0) | (d >= window)
+        out[a:b] = torch.matmul(torch.softmax(s.masked_fill(hide, float("-inf")), -1), v).transpose(0, 1)
+    return out
+
+
+def unit(x: torch.Tensor) -> torch.Tensor:
+    return x * torch.rsqrt((x * x).sum(-1, keepdim=True) + UNIT_EPS)
+
+
+def ring_conv(x: torch.Tensor, taps: torch.Tensor, bias, ring: torch.Tensor, meta) -> torch.Tensor:
+    """Causal convolution per channel of packed rows x [T, channels] (last
+    column of taps: the current token).  ring [slots, taps, channels] holds the
+    inputs of positions p at p % taps and is brought up to date."""
+    n = taps.shape[1]
+    out = torch.empty_like(x, dtype=torch.float32)
+    for i in range(meta.seq_slots.numel()):
+        a, b, st, slot = int(meta.cu_q[i]), int(meta.cu_q[i + 1]), int(meta.q_start[i]), int(meta.seq_slots[i])
+        past = [ring[slot, p % n].float() if p >= 0 else torch.zeros(x.shape[1]) for p in range(st - n + 1, st)]
+        rows = torch.cat([torch.stack(past), x[a:b].float()]) if past else x[a:b].float()
+        out[a:b] = sum(rows[j: j + b - a] * taps[:, j].float() for j in range(n))
+        for p in range(max(st, st + b - a - n), st + b - a):
+            ring[slot, p % n] = x[a + p - st].to(ring.dtype)
+    return out if bias is None else out + bias.float()
+
+
+def _scan(meta, state: torch.Tensor, step) -> None:
+    """step(t, S) -> S over every token of every sequence; a sequence's state
+    [heads, rows, vdim] starts at zero and is kept in state[slot]."""
+    for i in range(meta.seq_slots.numel()):
+        a, b, slot = int(meta.cu_q[i]), int(meta.cu_q[i + 1]), int(meta.seq_slots[i])
+        S = state[slot].clone() if int(meta.q_start[i]) > 0 else torch.zeros_like(state[slot])
+        for t in range(a, b):
+            S = step(t, S)
+        state[slot] = S
+
+
+def delta_rule(q, k, v, g, beta, state, meta) -> torch.Tensor:
+    """S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.
+    q, k, g [T, H, D], v [T, H, V], beta [T, H], state [slots, H, D, V]."""
+    out = torch.empty(v.shape, dtype=torch.float32)
+
+    def step(t, S):
+        S = g[t][..., None] * S
+        u = beta[t][:, None] * (v[t] - torch.matmul(k[t][:, None], S)[:, 0])
+        S = S + k[t][..., None] * u[:, None]
+        out[t] = torch.matmul(q[t][:, None], S)[:, 0]
+        return S
+    _scan(meta, state, step)
+    return out
+
+
+def ssd(x, B, C, dt, decay, state, meta) -> torch.Tensor:
+    """S <- decay S + dt B x^T; y = S^T C.  x [T, H, V], B, C [T, H, N]."""
+    out = torch.empty(x.shape, dtype=torch.float32)
+
+    def step(t, S):
+        S = decay[t][:, None, None] * S + B[t][..., None] * (dt[t][:, None] * x[t])[:, None]
+        out[t] = torch.matmul(C[t][:, None], S)[:, 0]
+        return S
+    _scan(meta, state, step)
     return out
 
 

@@ -169,6 +169,9 @@ def _layer_costs(cfg: ModelConfig, rows: int, avg_ctx: int):
     costs: List[float] = []
     for l in cfg.layers:
         m, f = l.mixer, l.mlp
+        if cfg.arch == "vizalix":
+            costs += [_mixer_cost(cfg, l, rows, avg_ctx), 0.0]
+            continue
         n_in = m.heads * m.dim + (m.kv_rank if m.kv_from is None else 0) + (f.experts if f else 0)
         ctx = min(avg_ctx, m.window or avg_ctx)
         c = 6.0 + _gemm_us(n_in, h, rows) + 4.0 + 3.0 + rows * ctx * m.kv_rank * 2 / 6.0e6
@@ -182,6 +185,24 @@ def _layer_costs(cfg: ModelConfig, rows: int, avg_ctx: int):
         costs += [c, 0.0]
     head = 6.0 + _gemm_us(cfg.vocab_padded, h, rows) + 8.0 + 0.37 * min(rows, 128)
     return costs, head, 4.0
+
+
+def _mixer_cost(cfg: ModelConfig, l, rows: int, avg_ctx: int) -> float:
+    """Decode step of one layer (attention or recurrence, dense feed-forward)."""
+    h, m, ff = cfg.hidden, l.mixer, l.mlp.ff if l.mlp else 0
+    ov = m.heads * m.vdim
+    if m.cached_per_token:
+        n_in = m.heads * m.dim + m.cached_per_token
+        moved = rows * min(avg_ctx, m.window or avg_ctx) * m.cached_per_token * 2
+    else:  # the state is read and written once
+        n_in = m.params(h) // h - ov
+        moved = rows * 8 * ov * (m.dim if hasattr(m, "dim") else m.state)
+    c = 6.0 + _gemm_us(n_in, h, rows) + 6.0 + moved / 5.0e6 + _gemm_us(h, ov + ff, rows)
+    if ff:
+        c += _gemm_us(2 * ff, h, rows)
+    if l.enter is not None:
+        c += 4.0 + _gemm_us(h, 2 * h, rows)
+    return c
 
 
 def layer_cuts(cfg: ModelConfig) -> List[int]:

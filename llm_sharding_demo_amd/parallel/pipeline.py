@@ -335,7 +335,7 @@ class StageWorker(racecheck.Shared):
         self.device = stage.device
         self.first = stage_idx == 0
         self.last = stage_idx == num_stages - 1
-        self.H = stage.row_width
+        self.H = stage.wire_width
         self.scratch_slot, self.compat_slot = scratch_slot, compat_slot
         self.use_graphs = True
         # Group "lanes": group g of this stage runs on lanes[g % L], so

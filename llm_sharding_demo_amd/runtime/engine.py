@@ -45,7 +45,7 @@ from ..parallel.comm import (DeviceLoopFabric, GlooPlanChannel, LocalFabric, Loc
                              open_data_plane, transport_chain)
 from ..parallel.partition import make_alt_unit_plans, make_unit_plan, union_plan, units_to_layers
 from ..parallel.pipeline import StageWorker
-from .kv_cache import PAGE, KVCache, LatentCache, SlotAllocator, pages_for, plan_pages, plan_slots
+from .kv_cache import PAGE, KVCache, SlotAllocator, layer_cache, pad_up, pages_for, plan_pages, plan_slots
 from .plan import GroupPlan, StepPlan
 from .scheduler import Request, Scheduler
 
@@ -299,20 +299,23 @@ class Engine(racecheck.Shared):
         return fits
 
     def _paged_budget(self, slots: int, per_dev: dict, share, devices, collective: bool) -> int:
-        """Paged caches: slots are only page-table rows, so all of them exist;
-        the pool takes kv_tokens (default: every slot at max_seq), capped by
-        the memory of the tightest device.  Sets kv_pages, returns the slots."""
+        """Paged caches: slots are page-table rows and the layers' recurrent
+        state; the pool takes kv_tokens (default: every slot at max_seq),
+        capped by the memory of the tightest device after the weights and the
+        states.  Sets kv_pages, returns the slots."""
         want = pages_for(self.cfg.kv_tokens) if self.cfg.kv_tokens > 0 else slots * pages_for(self.max_seq)
         elt = 4 if self.cfg.dtype == "fp32" else 2
         fits = want
         for dev, _, w_bytes in per_dev.values():
-            ranks = []
+            caches = []
             for i, d in enumerate(devices):
                 if str(d) == str(dev):
                     a, b = self.unit_plan[self.stage_idx if collective else i]
-                    ranks += [self.mcfg.layers[j].mixer.kv_rank + 63 for j in self.mcfg.cache_layers(range(a // 2, b // 2))]
-            fits = min(fits, plan_pages(want, LatentCache.bytes_per_page(ranks, elt), dev,
-                                        fraction=self.cfg.kv_fraction, reserve=w_bytes, mem_get_info=share))
+                    caches += [layer_cache(self.mcfg.layers[j].mixer, pad_up)
+                               for j in self.mcfg.cache_layers(range(a // 2, b // 2))]
+            states = (slots + 2) * sum(c.slot_bytes(elt) for c in caches)
+            fits = min(fits, plan_pages(want, sum(c.page_bytes(elt) for c in caches), dev, fraction=self.cfg.kv_fraction,
+                                        reserve=w_bytes + states, mem_get_info=share))
         if collective:
             import torch.distributed as dist
 
@@ -349,7 +352,7 @@ class Engine(racecheck.Shared):
         item's prefill rows (a group's chunk tokens, fp32) -- within 64 MiB to
         1 GiB, and never less than one such message plus 1 MiB."""
         per_seq = self.cfg.prefill_chunk if self.cfg.prefill_chunk > 0 else self.max_seq
-        big = self.group_cap * min(per_seq, self.max_seq) * ((self.mcfg.hidden + 63) // 64 * 64) * 4
+        big = self.group_cap * min(per_seq, self.max_seq) * ((self.mcfg.hidden + 63) // 64 * 64) * 4 * (2 if self.mcfg.loop_times else 1)
         ring = int(os.environ.get("LSD_LOOP_RING_MB", "0")) << 20 or min(1 << 30, max(64 << 20, 8 * big))
         return max(ring, big + (1 << 20))
 
@@ -358,8 +361,9 @@ class Engine(racecheck.Shared):
         a, b = self.unit_plan[i]
         if mc.layers:
             elt = 4 if self.cfg.dtype == "fp32" else 2
-            n = elt * sum(mc.layer_params(j) for j in range(a // 2, b // 2))
-            return n + elt * mc.embed_params() * (1 if i in (0, self.P - 1) else 0)
+            n = elt * mc.stage_params(range(a // 2, b // 2))
+            ends = (i in (0, self.P - 1)) if mc.tie_embeddings else (i == 0) + (i == self.P - 1)
+            return n + elt * mc.embed_params() * ends
         per_layer = mc.block_params() * 2
         n = per_layer * (b - a) // 2
         if i == 0:
@@ -825,7 +829,7 @@ class Engine(racecheck.Shared):
         with self._lock:
             ids = torch.tensor(input_ids, dtype=torch.int32, device=st.device)
             meta = BatchMeta.build([self.kv_slots + 1], [0], [len(input_ids)], st.device)
-            return st.forward(meta, ids)[:, : self.mcfg.hidden]
+            return st.boundary_rows(st.forward(meta, ids))
 
     def forward_b(self, hidden: torch.Tensor) -> torch.Tensor:
         """Remaining stages + ln_f + lm_head over all positions (ShardB,
@@ -837,10 +841,7 @@ class Engine(racecheck.Shared):
         if self.P < 2:
             raise RuntimeError("forward_b needs >= 2 pipeline stages")
         # a stage updates its input rows in place (the residual stream): copy
-        h = hidden.reshape(-1, self.mcfg.hidden).float().clone()
-        width = self.stages[0].row_width  # residual rows may be padded (ops/hip.py)
-        if width > h.shape[1]:
-            h = torch.nn.functional.pad(h, (0, width - h.shape[1]))
+        h = self.stages[0].wire_rows(hidden.reshape(-1, self.mcfg.boundary).float()).clone()
         T = h.shape[0]
         if T > self.max_seq:
             raise ValueError(f"sequence length {T} exceeds {self.max_seq}")

@@ -16,9 +16,12 @@ stage's weights (runtime/engine.py `_kv_slots`, reported on /health and
 """
 from __future__ import annotations
 
-from typing import List, Sequence
+from dataclasses import dataclass
+from typing import Callable, List, Sequence, Tuple
 
 import torch
+
+from ..config import AttentionSpec, ChannelDeltaSpec, SSMSpec
 
 PAGE = 64  # tokens per page of a paged cache (csrc/kernels/attention_latent.hip)
 
@@ -46,29 +49,68 @@ class KVCache:
         return n_layers * 2 * n_kv * max_seq * head_dim * elt
 
 
+def pad_up(n: int, m: int) -> int:
+    return -(-n // m) * m
+
+
 def pages_for(tokens: int) -> int:
     return -(-int(tokens) // PAGE)
 
 
-class LatentCache:
-    """Paged cache of latent rows (latent attention): one pool of PAGE-token
-    pages per layer that owns latents,
-        pools[k][page, token, rank]
-    and one page table for all of them, table[slot, position // PAGE].  Pages
+@dataclass(frozen=True)
+class LayerCache:
+    """What one layer keeps of a sequence: tensors of its PAGE-token pages
+    (their shapes), and tensors of its slot -- recurrent state in fp32, the
+    last inputs of a short convolution in the model's element type."""
+
+    pages: Tuple[tuple, ...] = ()
+    state: Tuple[tuple, ...] = ()   # fp32, per slot
+    ring: Tuple[tuple, ...] = ()    # element type, per slot
+
+    def page_bytes(self, elt: int = 2) -> int:
+        return elt * sum(torch.Size(s).numel() for s in self.pages)
+
+    def slot_bytes(self, elt: int = 2) -> int:
+        return sum(4 * torch.Size(s).numel() for s in self.state) + sum(elt * torch.Size(s).numel() for s in self.ring)
+
+
+def layer_cache(mixer, up: Callable[[int, int], int] = lambda n, m: n) -> LayerCache:
+    """Cache of one layer; up(n, m): the backend's padding of n to a multiple of m.
+      attention   K [kv head][token][dim], V [kv head][token][vdim] per page
+      delta rule  S [heads][dim][vdim] and the conv inputs of positions p % taps
+      Mamba-2     S [heads][state][vdim], and the same
+      latent      one row of `rank` per token"""
+    if isinstance(mixer, AttentionSpec):
+        g = mixer.kv_heads
+        return LayerCache(pages=((g, PAGE, up(mixer.dim, 32)), (g, PAGE, up(mixer.vdim, 16))))
+    if isinstance(mixer, (ChannelDeltaSpec, SSMSpec)):
+        rows = mixer.dim if isinstance(mixer, ChannelDeltaSpec) else mixer.state
+        return LayerCache(state=((mixer.heads, rows, up(mixer.vdim, 4)),), ring=((mixer.conv, mixer.conv_channels),))
+    return LayerCache(pages=((PAGE, up(mixer.kv_rank, 64)),))
+
+
+class PagedCache:
+    """Per-layer caches of models with per-layer specs: entries[k] holds layer
+    k's tensors, a pool of PAGE-token pages ([page, ...]) per LayerCache.pages
+    and per-slot tensors ([slot, ...]) per LayerCache.state / .ring, and one
+    page table serves all of them, table[slot, position // PAGE].  Pages
     belong to sequences, not to slots: the host's page allocator hands them out
     (the scheduler at admission, runtime/trace.py as a sequence grows) and
     `assign` writes a slot's table row.  Table entries without a page point at
-    the scratch page, which pad rows also write to.  `reserved` further slots
-    own a full row of pages each (compat forwards)."""
+    the scratch page, which pad rows also write to.  A slot's state needs no
+    clearing: whoever runs position 0 starts from zero.  `reserved` further
+    slots own a full row of pages each (compat forwards)."""
 
-    def __init__(self, ranks: Sequence[int], slots: int, pages: int, max_seq: int, dtype: torch.dtype, device,
+    def __init__(self, layers: Sequence[LayerCache], slots: int, pages: int, max_seq: int, dtype: torch.dtype, device,
                  reserved: Sequence[int] = ()):
         self.slots, self.pages, self.max_seq = slots, pages, max_seq
         self.width = pages_for(max_seq)
         extra = len(reserved) * self.width
         self.scratch = pages + extra
         # zeros: a masked key of a page's unused tail must be a finite number
-        self.pools = [torch.zeros(pages + extra + 1, PAGE, r, dtype=dtype, device=device) for r in ranks]
+        z = lambda n, s, dt: torch.zeros(n, *s, dtype=dt, device=device)  # noqa: E731
+        self.entries = [[z(pages + extra + 1, s, dtype) for s in l.pages] + [z(slots, s, torch.float32) for s in l.state] +
+                        [z(slots, s, dtype) for s in l.ring] for l in layers]
         self.table = torch.full((slots, self.width), self.scratch, dtype=torch.int32, device=device)
         for k, s in enumerate(reserved):
             self.table[s] = torch.arange(pages + k * self.width, pages + (k + 1) * self.width, dtype=torch.int32,
@@ -93,7 +135,17 @@ class LatentCache:
 
     @property
     def nbytes(self) -> int:
-        return sum(p.numel() * p.element_size() for p in self.pools) + self.table.numel() * 4
+        return sum(p.numel() * p.element_size() for e in self.entries for p in e) + self.table.numel() * 4
+
+
+class LatentCache(PagedCache):
+    """Paged cache of latent rows (latent attention): pools[k][page, token, rank]
+    per layer that owns latents."""
+
+    def __init__(self, ranks: Sequence[int], slots: int, pages: int, max_seq: int, dtype: torch.dtype, device,
+                 reserved: Sequence[int] = ()):
+        super().__init__([LayerCache(pages=((PAGE, r),)) for r in ranks], slots, pages, max_seq, dtype, device, reserved)
+        self.pools = [e[0] for e in self.entries]
 
     @staticmethod
     def bytes_per_page(ranks: Sequence[int], elt: int = 2) -> int:

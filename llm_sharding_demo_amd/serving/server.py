@@ -88,10 +88,10 @@ class ShardRunner:
         with self.lock:
             meta = BatchMeta.build([0], [0], [seq_len], st.device)
             x = x.to(st.device)
-            if not st.first and st.row_width > x.shape[1]:  # residual rows may be padded (ops/hip.py)
-                x = torch.nn.functional.pad(x, (0, st.row_width - x.shape[1]))
+            if not st.first:  # residual rows may be padded (ops/hip.py)
+                x = st.wire_rows(x)
             out = st.forward(meta, x, all_logits=True)
-        return out if st.last else out[:, : st.cfg.hidden]
+        return out if st.last else st.boundary_rows(out)
 
 
 def create_app(cfg: EngineConfig, engine=None, shard: Optional[ShardRunner] = None):
@@ -139,8 +139,8 @@ def create_app(cfg: EngineConfig, engine=None, shard: Optional[ShardRunner] = No
         if not _role_is("b"):
             return {"error": "This instance is not shard B."}
         hidden = torch.tensor(req.hidden_states, dtype=torch.float32)
-        if hidden.dim() != 3 or hidden.shape[-1] != mc.hidden:
-            raise HTTPException(422, f"hidden_states must be [B][S][{mc.hidden}]")
+        if hidden.dim() != 3 or hidden.shape[-1] != mc.boundary:
+            raise HTTPException(422, f"hidden_states must be [B][S][{mc.boundary}]")
         B, S, H = hidden.shape
         outs = []
         try:

@@ -1,0 +1,289 @@
+"""Vizalix on the CPU: config and weights, caches and states, portions of
+prompts, looped layers, stages, and greedy generation, against the plain model
+of vizalix_oracle.py."""
+from __future__ import annotations
+
+import math
+import random
+
+import pytest
+import torch
+
+import llm_sharding_demo_amd.runtime.trace as trace
+from llm_sharding_demo_amd.config import (AttentionSpec, ChannelDeltaSpec, EngineConfig, LayerSpec, RopeScaling, RopeSpec,
+                                          SamplingParams, SSMSpec, get_model_config, unroll)
+from llm_sharding_demo_amd.ops import reference as ref
+from llm_sharding_demo_amd.parallel.partition import layer_cuts, make_unit_plan, unit_costs
+from llm_sharding_demo_amd.runtime.batch import BatchMeta
+from llm_sharding_demo_amd.runtime.engine import Engine
+from llm_sharding_demo_amd.runtime.kv_cache import PAGE, PagedCache, layer_cache, pad_up
+
+from . import vizalix_oracle as orc
+
+F64 = torch.float64
+
+
+def model(tmp_path, layers, seed=0, **kw):
+    cfg = orc.config(layers, **kw)
+    w = orc.random_weights(cfg, seed)
+    orc.save(str(tmp_path), cfg, w)
+    return cfg, w
+
+
+def all_kinds():
+    """Every mixer twice with other sizes, one layer without a feed-forward."""
+    return [orc.delta(), orc.attn(), orc.ssm(), orc.delta(heads=3, kv_heads=3, dim=8, vdim=16, conv=1, ff=0, ranks=(3, 9)),
+            orc.attn(heads=3, kv_heads=1, dim=16, vdim=20, window=9, rot=16, scaling=None, ff=24),
+            orc.ssm(heads=2, vdim=24, state=5, groups=1, norm_groups=1, conv=2)]
+
+
+def engine(path, **kw):
+    kw = {"device": "cpu", "max_batch": 4, "max_seq_len": 320, "kv_tokens": 640, **kw}
+    return Engine(EngineConfig(model_id=str(path), weights=str(path), **kw))
+
+
+def ids_of(n, vocab=200, seed=0):
+    r = random.Random(seed)
+    return [r.randrange(vocab) for _ in range(n)]
+
+
+def close(got, want, tol=1e-4):
+    return float((got.double() - want).abs().max()) < tol * float(want.double().pow(2).mean().sqrt())
+
+
+# -- configuration and weights ------------------------------------------------
+
+def test_config_reader(tmp_path):
+    cfg, w = model(tmp_path, all_kinds(), eps=3e-6, loop=(1, 3, 3))
+    mc = get_model_config(str(tmp_path))
+    assert (mc.arch, mc.vocab_size, mc.hidden, mc.n_layers) == ("vizalix", 200, 88, 10)
+    assert mc.norm_eps == 3e-6 and mc.eos_token_id == -1 and mc.loop_times == 3 and mc.boundary == 176
+    assert [l.weights for l in mc.layers] == [0, 1, 2, 1, 2, 1, 2, 3, 4, 5]
+    assert [l.enter for l in mc.layers] == [None, 0, None, 1, None, 2, None, None, None, None]
+    assert [(i, t) for i, t in orc.passes(cfg)] == [(l.weights, l.enter) for l in mc.layers]
+    assert mc.layers[0].mixer == ChannelDeltaSpec(4, 2, 24, 20, 3, 10, 6)
+    assert mc.layers[1].mixer == AttentionSpec(6, 2, 40, 24, 0.2, 70, RopeSpec(24, 10000.0, RopeScaling(4, 1, 4, 96)), 6.0)
+    assert mc.layers[2].mixer == SSMSpec(6, 12, 20, 2, 3, 4) and mc.layers[7].mlp is None
+    assert mc.stage_params(range(10)) + 2 * mc.embed_params() + 1 == sum(torch.Size(s).numel()
+                                                                       for s in orc.shapes(cfg).values())
+
+
+@pytest.mark.parametrize("bad", [orc.attn(heads=5), orc.attn(rot=7), orc.attn(softcap=-1.0), orc.delta(heads=3),
+                                 orc.ssm(groups=4), orc.ssm(norm_groups=5), orc.ssm(state=0), {**orc.ssm(), "type": "x"},
+                                 {**orc.ssm(), "mlp": {"kind": "moe", "ff": 8}}])
+def test_config_rejects(tmp_path, bad):
+    orc.save(str(tmp_path), orc.config([orc.ssm(), bad]), {"l1.mix.a1": torch.zeros(2, 88), "l1.mix.g1": torch.zeros(2, 88)})
+    with pytest.raises(ValueError):
+        get_model_config(str(tmp_path))
+
+
+def test_ranks_come_from_the_checkpoint(tmp_path):
+    orc.save(str(tmp_path), orc.config([orc.delta()]), {"x": torch.zeros(1)})
+    with pytest.raises(ValueError, match="l0.mix.a1"):
+        get_model_config(str(tmp_path))
+
+
+def test_unroll_limits():
+    l = LayerSpec(SSMSpec(2, 4, 4, 1, 1, 2))
+    assert [x.weights for x in unroll([l] * 3, 2, 3, 2)] == [0, 1, 2, 2]
+    for bad in ((0, 4, 1), (1, 1, 2), (0, 1, 0)):
+        with pytest.raises(ValueError):
+            unroll([l] * 3, *bad)
+
+
+def test_presets_run():
+    eng = Engine(EngineConfig(model_id="vizalix-test", device="cpu", max_batch=2, max_seq_len=64))
+    out = eng.generate_ids([[3, 4, 5]], SamplingParams(greedy=True, max_new_tokens=4))
+    assert len(out[0]) == 4
+
+
+# -- mechanisms ----------------------------------------------------------------
+
+def test_rope_frequencies_and_partial_rotation():
+    """All three ranges of the scaling, and dimensions behind the rotated ones."""
+    rot = {"dims": 12, "base": 100.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 64}}
+    spec = RopeSpec(12, 100.0, RopeScaling(8.0, 1.0, 4.0, 64))
+    f, plain = spec.frequencies(), RopeSpec(12, 100.0).frequencies()
+    assert f == pytest.approx(orc.frequencies(rot), rel=1e-14)
+    kinds = {"kept" if a == b else "stretched" if a == pytest.approx(b / 8) else "between" for a, b in zip(f, plain)}
+    assert kinds == {"kept", "stretched", "between"}
+    x, pos = torch.randn(5, 3, 20, generator=torch.Generator().manual_seed(0)), torch.tensor([0, 1, 63, 64, 1000])
+    assert close(ref.partial_rope(x, pos, spec), orc.rotate(x.double(), pos.tolist(), rot), 1e-6)
+    assert torch.equal(ref.partial_rope(x, pos, spec)[..., 12:], x[..., 12:])
+
+
+def one_seq(T, slot=1, start=0):
+    return BatchMeta.build([slot], [start], [T], "cpu")
+
+
+@pytest.mark.parametrize("cut", [0, 1, 2, 3, 9])
+def test_delta_rule_and_conv_in_portions(cut):
+    g = torch.Generator().manual_seed(1)
+    T, H, D, V = 12, 2, 5, 4
+    q, k, v = torch.randn(T, H, D, generator=g), torch.randn(T, H, D, generator=g), torch.randn(T, H, V, generator=g)
+    d, beta = torch.rand(T, H, D, generator=g), torch.rand(T, H, generator=g)
+    d[3] = 0.0  # a channel may forget everything
+    state = torch.full((2, H, D, V), float("nan"))
+    parts = [(0, cut), (cut, T)] if cut else [(0, T)]
+    o = torch.cat([ref.delta_rule(q[a:b], k[a:b], v[a:b], d[a:b], beta[a:b], state, one_seq(b - a, start=a))
+                   for a, b in parts])
+    want, S = orc.delta_rule(*(t.double() for t in (q, k, v, d, beta)))
+    assert close(o, want) and close(state[1], S)
+    for n in (1, 2, 4):
+        x, taps = torch.randn(T, 6, generator=g), torch.randn(6, n, generator=g)
+        ring = torch.full((2, n, 6), float("nan"))
+        y = torch.cat([ref.ring_conv(x[a:b], taps, None, ring, one_seq(b - a, start=a)) for a, b in parts])
+        assert close(y, orc.short_conv(x.double(), taps.double()))
+
+
+@pytest.mark.parametrize("cut", [0, 1, 7])
+def test_ssd_in_portions(cut):
+    g = torch.Generator().manual_seed(2)
+    T, H, V, N = 11, 3, 4, 5
+    x, B, C = torch.randn(T, H, V, generator=g), torch.randn(T, H, N, generator=g), torch.randn(T, H, N, generator=g)
+    dt, A, D = torch.rand(T, H, generator=g), torch.randn(H, generator=g), torch.randn(H, generator=g)
+    state = torch.full((2, H, N, V), float("nan"))
+    decay = torch.exp(-torch.exp(A) * dt)
+    parts = [(0, cut), (cut, T)] if cut else [(0, T)]
+    y = torch.cat([ref.ssd(x[a:b], B[a:b], C[a:b], dt[a:b], decay[a:b], state, one_seq(b - a, start=a)) for a, b in parts])
+    want, S = orc.ssd(*(t.double() for t in (x, B, C, dt, A, D)))
+    assert close(y + D[:, None] * x, want) and close(state[1], S)
+
+
+def test_window_edges_and_head_mixing():
+    """A key whose score stands out is seen at the last place of the window and
+    not one place further, also at page borders, through any page order, and by
+    the heads that the mixing matrix sends it to."""
+    H, G, D, V, n, slot = 4, 2, 6, 5, 3 * PAGE, 1
+    kv = PagedCache([layer_cache(AttentionSpec(H, G, D, V, 1.0))], 2, 8, n, torch.float32, "cpu")
+    kv.assign([(slot, (5, 0, 3))])
+    g = torch.Generator().manual_seed(2)
+    pos, slots = torch.arange(n, dtype=torch.int32), torch.full((n,), slot)
+    k, v = torch.randn(n, G, D, generator=g) * 0.1, torch.randn(n, G, V, generator=g)
+    talk = torch.tensor([[1.0, 0, 0, 0], [0, 0, 1.0, 0], [0.5, -1.0, 0, 0], [0, 0, 0, 1.0]])
+    q = torch.ones(1, H, D)
+    for W in (1, 7, PAGE, PAGE + 1, 2 * PAGE, None):
+        for p in (PAGE - 1, PAGE, 2 * PAGE - 1, 2 * PAGE, n - 1):
+            for key in {p if W is None else max(0, p - W + 1), p if W is None else max(0, p - W), 0, p}:
+                kk, vv = k.clone(), v.clone()
+                kk[key, 0] = 8.0  # the heads of the first group
+                vv[key] = 100.0
+                for pool, x in zip(kv.entries[0], (kk, vv)):
+                    ref.paged_append(pool, kv.table, x, slots, pos)
+                i32 = dict(dtype=torch.int32)
+                o = ref.talking_attention(q, *kv.entries[0], kv.table, torch.tensor([slot], **i32),
+                                          torch.tensor([p], **i32), torch.tensor([0, 1], **i32), talk, 1.0, 30.0, W)
+                want = orc.talking_attention(q.double(), kk[: p + 1].double(), vv[: p + 1].double(), talk.double(), 1.0,
+                                             30.0, W, first=p)
+                assert close(o, want)
+                assert (float(o[0, 0].mean()) > 50) == orc.visible(p, key, W)
+                if W is None or W > 1:  # more than one key: head 2 turns away from it
+                    assert float(o[0, 2].mean()) < 50 or not orc.visible(p, key, W)
+
+
+def test_layer_caches():
+    c = layer_cache(AttentionSpec(6, 2, 40, 24, 1.0), pad_up)
+    assert c.pages == ((2, PAGE, 64), (2, PAGE, 32)) and c.page_bytes(2) == 2 * 2 * PAGE * 96 and c.slot_bytes() == 0
+    c = layer_cache(ChannelDeltaSpec(4, 2, 24, 21, 3, 10, 6), pad_up)
+    assert c.state == ((4, 24, 24),) and c.ring == ((3, 2 * 48 + 84),) and c.page_bytes() == 0
+    assert c.slot_bytes(2) == 4 * 4 * 24 * 24 + 2 * 3 * 180
+    assert layer_cache(SSMSpec(6, 12, 20, 2, 3, 4)).state == ((6, 20, 12),)
+
+
+# -- cache, portions, batches ---------------------------------------------------
+
+def run_portions(ses, rid, ids, sizes, end=True):
+    out, at, sizes = [], 0, list(sizes)
+    while at < len(ids):
+        n = min(sizes.pop(0) if sizes else 1, len(ids) - at)
+        out.append(ses.step([{"id": rid, "tokens": ids[at:at + n], "want": list(range(n))}],
+                            [rid] if end and at + n == len(ids) else []))
+        at += n
+    return torch.cat(out)
+
+
+@pytest.mark.parametrize("loop", [None, (0, 2, 2), (1, 4, 3)])
+def test_whole_prompts(tmp_path, loop):
+    cfg, w = model(tmp_path, all_kinds(), loop=loop, seed=3)
+    ids = ids_of(100)
+    got = run_portions(trace.TraceSession(engine(tmp_path)), "a", ids, [100])
+    assert close(got, orc.forward(cfg, w, ids))
+
+
+@pytest.mark.parametrize("sizes", [[2] * 75, [63, 1, 2, 60, 24], [1] * 150, [64, 64, 22], [7, 130, 13]])
+def test_portions(tmp_path, sizes):
+    cfg, w = model(tmp_path, all_kinds()[:3], loop=(0, 2, 2))
+    ids = ids_of(150)
+    assert close(run_portions(trace.TraceSession(engine(tmp_path)), "a", ids, sizes), orc.forward(cfg, w, ids))
+
+
+def test_mixed_batches_and_reused_slots(tmp_path):
+    """Unequal requests in one batch, finished ones' pages and slots used again."""
+    cfg, w = model(tmp_path, all_kinds()[:3], loop=(1, 3, 2))
+    eng = engine(tmp_path, kv_tokens=6 * PAGE)
+    ses = trace.TraceSession(eng)
+    seqs = {k: ids_of(n, seed=n) for k, n in (("a", 100), ("b", 5), ("c", 131), ("d", 66))}
+    want = {k: orc.forward(cfg, w, v) for k, v in seqs.items()}
+    steps = [[("a", 70), ("b", 1)], [("a", 1), ("b", 3), ("c", 2)], [("b", 1), ("c", 61), ("a", 1)],
+             [("c", 1), ("a", 28), ("d", 60)], [("d", 1), ("c", 2)], [("c", 65), ("d", 5)]]
+    at = dict.fromkeys(seqs, 0)
+    for _ in range(2):
+        for st in steps:
+            ent = [{"id": k, "tokens": seqs[k][at[k]:at[k] + n], "want": list(range(n))} for k, n in st]
+            rows = [want[k][at[k] + j] for k, n in st for j in range(n)]
+            for k, n in st:
+                at[k] += n
+            got = ses.step(ent, [k for k, _ in st if at[k] == len(seqs[k])])
+            assert close(got, torch.stack(rows))
+        assert not ses.live and eng.page_pools[0].available == 6 and eng.slots.available == 4
+        at = dict.fromkeys(seqs, 0)
+
+
+# -- scheduler and engine ---------------------------------------------------------
+
+@pytest.mark.parametrize("kw", [{}, {"num_microbatches": 2}, {"prefill_chunk": 7}, {"kv_tokens": 4 * PAGE}])
+def test_greedy_generation(tmp_path, kw):
+    cfg, w = model(tmp_path, all_kinds()[:3], loop=(0, 1, 2))
+    eng = engine(tmp_path, **kw)
+    prompts = [ids_of(n, seed=n) for n in (1, 70, 13, 40)]
+    sp = [SamplingParams(greedy=True, max_new_tokens=n) for n in (8, 5, 10, 3)]
+    for _ in range(2):  # the second session finds the first one's states in its slots
+        out = eng.generate_ids(prompts, sp)
+        assert [len(o) for o in out] == [s.max_new_tokens for s in sp]
+        assert all(orc.is_greedy(cfg, w, p, o) for p, o in zip(prompts, out))
+        assert eng.page_pools[0].available == eng.kv_pages and eng.slots.available == eng.kv_slots
+
+
+@pytest.mark.parametrize("split", [1, 2, 3, 4])
+def test_two_stages_and_compat_forwards(tmp_path, split):
+    """The cut may fall in front of, between and behind the loop's passes: the
+    embedding output crosses the boundary beside the residual."""
+    cfg, w = model(tmp_path, [orc.ssm(), orc.delta(), orc.attn()], loop=(1, 2, 2))
+    if split == 4:
+        with pytest.raises(ValueError):
+            engine(tmp_path, num_stages=2, split_points=[split], transport="strict")
+        return
+    eng = engine(tmp_path, num_stages=2, split_points=[split], transport="strict")
+    prompts = [ids_of(n, seed=n) for n in (30, 5, 66)]
+    out = eng.generate_ids(prompts, SamplingParams(greedy=True, max_new_tokens=4))
+    assert all(len(o) == 4 and orc.is_greedy(cfg, w, p, o) for p, o in zip(prompts, out))
+    hid = eng.forward_a(prompts[0])
+    assert hid.shape == (30, 2 * 88)
+    assert close(eng.forward_b(hid), orc.forward(cfg, w, prompts[0]))
+    eng.shutdown()
+
+
+def test_partition_and_memory_budget(tmp_path):
+    mc = get_model_config("vizalix-2b")
+    assert layer_cuts(mc) == list(range(1, mc.n_layers))
+    costs, head, _ = unit_costs(mc)
+    assert len(costs) == 2 * mc.n_layers and min(costs[::2]) > 0 and max(costs[1::2]) == 0 and head > 0
+    plan = make_unit_plan(mc, 3)
+    assert [u % 2 for p in plan for u in p] == [0] * 6
+    model(tmp_path, all_kinds(), loop=(1, 3, 2))
+    eng = engine(tmp_path)
+    slot = sum(layer_cache(l.mixer).slot_bytes(4) for l in eng.mcfg.layers)
+    page = sum(layer_cache(l.mixer).page_bytes(4) for l in eng.mcfg.layers)
+    kv = eng.stages[0].kv
+    assert kv.nbytes == (eng.kv_slots + 2) * slot + (eng.kv_pages + 1) * page + 4 * kv.table.numel()
+    assert eng._weight_bytes(0) == 2 * (eng.mcfg.stage_params(range(8)) + 2 * eng.mcfg.embed_params())
