@@ -138,6 +138,7 @@ GemmParams base_params(const torch::Tensor& a, const torch::Tensor& w, int64_t t
   p.W = bptr(w); p.ldw = w.stride(0);
   p.M = a.size(0); p.N = w.size(0); p.K = a.size(1);
   p.splits = 1;
+  p.act_scale = 1.f;
   TORCH_CHECK(p.N % 16 == 0, "N must be a multiple of 16 (pad the weight), got ", p.N);
   TORCH_CHECK(tiled >= 0 && tiled <= 3, "GEMM kind must be 0 (split-K), 1 (tiled), 2 / 3 (256-row), got ", tiled);
   if (tiled >= 2)
@@ -205,18 +206,30 @@ void run_gemm(GemmParams& p, int epi, int64_t tiled, int64_t splits,
 }
 
 
-// out = act(a @ w^T + bias), bf16
+// Output rows of a projection: the caller's (a column range of wider rows) or new ones.
+torch::Tensor out_rows(const c10::optional<torch::Tensor>& out, int64_t M, int64_t N, const torch::Tensor& like) {
+  if (!out.has_value()) return torch::empty({M, N}, like.options());
+  need(*out, like.scalar_type(), "out");
+  need_rows(*out, "out");
+  TORCH_CHECK(out->size(0) == M && out->size(1) == N, "out must be [", M, ", ", N, "]");
+  return *out;
+}
+
+// out = act(a @ w^T + bias), bf16.  act: 1 gelu, 2 silu(gate) up, 3 gelu(gate) up,
+// the gated ones with `scale` times both halves
 torch::Tensor linear(torch::Tensor a, torch::Tensor w, c10::optional<torch::Tensor> bias,
                      int64_t act, int64_t tiled, int64_t splits,
-                     c10::optional<torch::Tensor> counters) {
+                     c10::optional<torch::Tensor> counters, c10::optional<torch::Tensor> into, double scale) {
   GemmParams p = base_params(a, w, tiled);
   p.bias = opt_bias(bias, p.N);
-  int epi = act == 1 ? EPI_GELU : (act == 2 ? EPI_SILU_MUL : EPI_BF16);
+  int epi = act == 1 ? EPI_GELU : (act >= 2 ? EPI_SILU_MUL : EPI_BF16);
+  p.gelu = act == 3;
+  p.act_scale = (float)scale;
   if (epi == EPI_SILU_MUL) TORCH_CHECK(p.N % 32 == 0, "silu_mul needs N % 32 == 0");
   const int n_out = epi == EPI_SILU_MUL ? p.N / 2 : p.N;
-  auto out = torch::empty({p.M, n_out}, a.options());
+  auto out = out_rows(into, p.M, n_out, a);
   if (p.M == 0) return out;
-  p.out = out.data_ptr(); p.ldo = n_out;
+  p.out = out.data_ptr(); p.ldo = out.stride(0);
   run_gemm(p, epi, tiled, splits, counters, a, "linear");
   return out;
 }
@@ -337,13 +350,16 @@ c10::optional<torch::Tensor> gemv(torch::Tensor x, torch::Tensor w, c10::optiona
                                   c10::optional<torch::Tensor> tslot, c10::optional<torch::Tensor> tpos,
                                   int64_t q_size, int64_t kv_size, int64_t hd,
                                   c10::optional<torch::Tensor> rope,
-                                  c10::optional<torch::Tensor> segmax = c10::nullopt) {
+                                  c10::optional<torch::Tensor> segmax = c10::nullopt,
+                                  c10::optional<torch::Tensor> into = c10::nullopt, bool gelu = false,
+                                  double scale = 1.0) {
   need(w, torch::kBFloat16, "w");
   need_rows(w, "w");
   TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1, "x must be 2-D with unit last stride");
   TORCH_CHECK(reinterpret_cast<uintptr_t>(x.data_ptr()) % 16 == 0, "x must be 16-byte aligned");
   GemvParams p{};
   p.M = x.size(0); p.K = x.size(1); p.N = w.size(0);
+  p.gelu = gelu; p.act_scale = (float)scale;
   TORCH_CHECK(w.size(1) == p.K, "K mismatch: x ", x.sizes(), " w ", w.sizes());
   TORCH_CHECK(lsd_gemv_ok(p.M, p.K, (int)epi, (int)norm), "gemv: shape M=", p.M, " K=", p.K,
               " epi=", epi, " norm=", norm, " not supported");
@@ -391,12 +407,12 @@ c10::optional<torch::Tensor> gemv(torch::Tensor x, torch::Tensor w, c10::optiona
       p.segmax = segmax->data_ptr<float>(); p.ldseg = segmax->stride(0);
     }
   } else if (epi == EPI_BF16 || epi == EPI_GELU) {
-    ret = torch::empty({p.M, p.N}, bopt);
-    p.out = ret->data_ptr(); p.ldo = p.N;
+    ret = out_rows(into, p.M, p.N, w);
+    p.out = ret->data_ptr(); p.ldo = ret->stride(0);
   } else if (epi == EPI_SILU_MUL) {
     TORCH_CHECK(p.N % 32 == 0 && !bias.has_value(), "silu_mul needs N % 32 == 0 and no bias");
-    ret = torch::empty({p.M, p.N / 2}, bopt);
-    p.out = ret->data_ptr(); p.ldo = p.N / 2;
+    ret = out_rows(into, p.M, p.N / 2, w);
+    p.out = ret->data_ptr(); p.ldo = ret->stride(0);
   } else if (epi == EPI_QKV) {
     TORCH_CHECK(kc.has_value() && vc.has_value() && tslot.has_value() && tpos.has_value(),
                 "qkv needs caches and token slots/positions");
@@ -745,6 +761,7 @@ void lsd_register_comm(pybind11::module& m);  // csrc/comm.cpp
 void lsd_register_exec(pybind11::module& m);  // csrc/stage_exec.cpp
 void lsd_register_loopback(pybind11::module& m);  // csrc/loop_fabric.cpp
 void lsd_register_blaslt(pybind11::module& m);    // csrc/blaslt.cpp
+void lsd_register_mixers(pybind11::module& m);    // csrc/mixer_bindings.cpp
 void lsd_register_latent(pybind11::module& m);    // csrc/latent_bindings.cpp
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -754,7 +771,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   lsd_register_loopback(m);
   lsd_register_blaslt(m);
   lsd_register_latent(m);
-  m.def("linear", &linear);
+  lsd_register_mixers(m);
+  m.def("linear", &linear, py::arg("a"), py::arg("w"), py::arg("bias"), py::arg("act"), py::arg("tiled"),
+        py::arg("splits"), py::arg("counters"), py::arg("out") = py::none(), py::arg("scale") = 1.0);
   m.def("linear_f32", &linear_f32, py::arg("a"), py::arg("w"), py::arg("tiled"), py::arg("splits"),
         py::arg("counters"), py::arg("segmax") = py::none());
   m.def("linear_residual", &linear_residual, py::arg("a"), py::arg("w"), py::arg("bias"), py::arg("x"),
@@ -780,6 +799,14 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     return gemv(x, w, bias, epi, norm, gamma, beta, eps, resid, kc, vc, tslot, tpos, q_size, kv_size, hd, rope);
   });
   // fp32 logits GEMV that also writes the 8-column segment maxima (the sampler's threshold)
+  // bf16 outputs into the caller's rows, gated activations with a common factor
+  m.def("gemv_into", [](torch::Tensor x, torch::Tensor w, int64_t epi, int64_t norm,
+                        c10::optional<torch::Tensor> gamma, c10::optional<torch::Tensor> beta, double eps,
+                        c10::optional<torch::Tensor> out, bool gelu, double scale) {
+    return gemv(x, w, c10::nullopt, epi, norm, gamma, beta, eps, c10::nullopt, c10::nullopt, c10::nullopt,
+                c10::nullopt, c10::nullopt, 0, 0, 0, c10::nullopt, c10::nullopt, out, gelu, scale);
+  }, py::arg("x"), py::arg("w"), py::arg("epi"), py::arg("norm"), py::arg("gamma"), py::arg("beta"), py::arg("eps"),
+        py::arg("out") = py::none(), py::arg("gelu") = false, py::arg("scale") = 1.0);
   m.def("gemv_logits", [](torch::Tensor x, torch::Tensor w, int64_t norm, c10::optional<torch::Tensor> gamma,
                           c10::optional<torch::Tensor> beta, double eps, torch::Tensor segmax) {
     return gemv(x, w, c10::nullopt, EPI_F32, norm, gamma, beta, eps, c10::nullopt, c10::nullopt,

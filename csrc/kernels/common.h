@@ -202,6 +202,12 @@ __device__ __forceinline__ float silu(float x) {
   return x * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x));
 }
 
+// Gated activation of a gate / up projection whose rows miss a common factor
+// `s` (a norm's gain): silu(s g) (s u), or the tanh-GELU form.
+__device__ __forceinline__ float gated(float g, float u, int gelu, float s) {
+  return (gelu ? gelu_new(s * g) : silu(s * g)) * (s * u);
+}
+
 // Bijective XCD-aware remap of a 1-D workgroup id (guide §5.5 T1, "XCD
 // swizzle must be bijective"): consecutive logical tiles land on one XCD so
 // tiles sharing an operand panel share that XCD's L2.  Speed only.

@@ -1,0 +1,94 @@
+// Launch parameters of the recurrent mixers and of attention with mixed heads,
+// shared by csrc/kernels/recurrence.hip, attention_talk.hip and
+// csrc/mixer_bindings.cpp.  "Rows" are packed tokens; the element type T is
+// bf16 or fp32 (models served in fp32).
+#pragma once
+
+namespace lsd {
+
+// Short causal convolution of channels [0, channels), which are columns c0 ..
+// of the in-projection rows y [rows][ldy] (T).  `gain` (the norm in front of
+// the projection, one number) multiplies what the convolution sums.  The inputs
+// of position p are kept at ring[slot][p % taps].
+struct ConvParams {
+  const void* y; long ldy; int c0;
+  const float* w;      // [channels][taps], last column: the current token
+  const float* bias;   // [channels] or null
+  int taps, channels;
+  void* ring;          // [slots][taps][channels]
+  float gain;
+};
+
+// Sequences of a launch: slot, first position and packed rows of each.
+struct SeqParams {
+  int B; const int* slots; const int* start; const int* cu;
+};
+
+// Recurrence over a state S [rows D][V] per (sequence, head), fp32:
+//   delta rule   S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q
+//   Mamba-2      S <- a S + k (dt v)^T;                                o = S^T q + skip v
+// with q / k / v conv channels (Mamba-2: C / B / x).
+struct RecurParams {
+  ConvParams c;
+  SeqParams s;
+  int heads, groups, D, V, Vp;         // Vp: V padded to 4 (row pitch of S)
+  int q_ch, k_ch, v_ch;                // first conv channel of each
+  int gate_col;                        // y column of beta's logits / dt, one per head
+  float* S;                            // [slots][heads][D][Vp]
+  const float* A;                      // [heads], -exp(A_log)
+  const float* dt_bias;                // delta: [heads D], Mamba-2: [heads]
+  // delta: second projections of the decay [heads D] and output gate [heads V]
+  const void* low; long ldl; int gate_off;
+  const float* norm; float eps;        // delta: output norm [V]
+  const float* skip;                   // Mamba-2: [heads]
+  float* raw; long ldr;                // outputs before norm and gate [rows][heads V], or null:
+  void* out; long ldo; int out_cols;   // normed and gated rows (zeros up to out_cols)
+  int write_ring;                      // single-token portions: this kernel keeps the ring
+};
+
+// Output norms of the unfused forms.
+struct MixOutParams {
+  const float* raw; long ldr; int T;
+  int heads, V;                        // delta: per (row, head)
+  const void* low; long ldl; int gate_off;
+  int inner, groups;                   // Mamba-2: per (row, group), gate z = y[z_col ..]
+  const void* z; long ldz;
+  const float* norm; float eps, gain;
+  void* out; long ldo; int out_cols;
+};
+
+// Chunked prompt forms (bf16 models), chunks of RC_CHUNK tokens.  Chunk x of
+// the launch: sequence tiles[2 x], first token tiles[2 x + 1] within it.
+constexpr int RC_CHUNK = 64;
+
+// Attention over a paged cache, K [page][kv head][64][dim], V likewise with
+// vdim; scores capped, mixed over the heads, softmaxed.
+struct TalkParams {
+  const void* q;                       // [rows][H][dim]
+  const void* k; const void* v;        // pools
+  const int* table; int tw;            // [slots][pages of a sequence]
+  const float* talk;                   // [H][H] or null
+  const void* talk_frag;               // MFMA kernels: bf16 [HP][HP], zero padded (HP: H to 16 / 32 / 64)
+  void* out; long ldo; int out_cols;   // [rows][H][vdim], zeros up to out_cols
+  int H, G, dim, vdim, window;         // window: keys per query (INT_MAX: all)
+  float scale, cap;                    // cap 0: none
+  // one token alone: slot and position per row
+  const int* slots; const int* pos; int T;
+  // prompt tiles: (sequence, first query); sequences
+  const int* tiles; int n_tiles;
+  SeqParams s;
+  // decode, splits > 1
+  float* part_o; float* part_ml; int splits;
+};
+
+// Rotation and cache append behind the in-projection y [rows][H dim | G dim | G vdim].
+struct RopeAppendParams {
+  const void* y; long ldy; int T;
+  float gain;
+  const float* rope; int half;         // [positions][half][2] cos, sin; half 0: none
+  void* q; void* k; void* v;
+  const int* table; int tw; const int* tslot; const int* tpos;
+  int H, G, dim, vdim;
+};
+
+}  // namespace lsd

@@ -1,0 +1,291 @@
+// PyTorch bindings of the recurrent mixers and of attention with mixed heads
+// (csrc/kernels/recurrence.hip, attention_talk.hip).
+//
+// Every entry point checks dtypes, shapes, strides and alignment on the host
+// before launching; launches go on the current stream and are graph-capturable.
+// Element type: bf16 or fp32, that of the in-projection rows.
+#include <torch/extension.h>
+#include <c10/hip/HIPStream.h>
+
+#include <hip/hip_runtime.h>
+
+#include <climits>
+
+#include "kernels/mixer_params.h"
+
+using lsd::ConvParams;
+using lsd::MixOutParams;
+using lsd::RecurParams;
+using lsd::RopeAppendParams;
+using lsd::SeqParams;
+using lsd::TalkParams;
+
+extern "C" {
+int lsd_recur_block(int D, int V);
+hipError_t lsd_recur_seq(const RecurParams* p, int delta, int f32, hipStream_t st);
+hipError_t lsd_conv_tail(const ConvParams* c, const SeqParams* s, int f32, hipStream_t st);
+hipError_t lsd_head_norm_gate(const MixOutParams* p, int f32, hipStream_t st);
+hipError_t lsd_gated_group_norm(const MixOutParams* p, int f32, hipStream_t st);
+hipError_t lsd_loop_pack(float* x, const float* x0, const float* step, void* out, int T, int H, int f32, hipStream_t st);
+hipError_t lsd_gelu_mul_f32(const float* y, float* out, int T, int F, long ldo, float s, hipStream_t st);
+hipError_t lsd_rope_append(const RopeAppendParams* p, int f32, hipStream_t st);
+long lsd_talk_plain_lds(const TalkParams* p);
+hipError_t lsd_talk_plain(const TalkParams* p, int f32, hipStream_t st);
+}
+
+namespace {
+
+constexpr int PAGE = 64;
+constexpr long MAX_LDS = 160 * 1024;
+using Opt = c10::optional<torch::Tensor>;
+using torch::Tensor;
+
+hipStream_t cur_stream() { return c10::hip::getCurrentHIPStream().stream(); }
+
+void check_hip(hipError_t e, const char* what) { TORCH_CHECK(e == hipSuccess, what, ": ", hipGetErrorString(e)); }
+
+bool is_f32(const Tensor& t, const char* name) {
+  TORCH_CHECK(t.is_cuda() && (t.scalar_type() == torch::kBFloat16 || t.scalar_type() == torch::kFloat32), name,
+              " must be a bf16 or fp32 GPU tensor");
+  return t.scalar_type() == torch::kFloat32;
+}
+
+// contiguous fp32 with exactly n elements
+const float* fptr(const Tensor& t, int64_t n, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kFloat32 && t.is_contiguous() && t.numel() == n, name,
+              " must be a contiguous fp32 GPU tensor of ", n, " elements");
+  return t.data_ptr<float>();
+}
+
+const int* iptr(const Tensor& t, int64_t n, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kInt32 && t.is_contiguous() && t.numel() >= n, name,
+              " must be contiguous int32 on the GPU with >= ", n, " elements");
+  return t.data_ptr<int>();
+}
+
+// rows [T, >= cols] with unit last stride, 16-byte aligned
+void rows_of(const Tensor& t, c10::ScalarType dt, int64_t T, int64_t cols, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == dt && t.dim() == 2 && t.stride(1) == 1 && t.size(0) == T &&
+                  t.size(1) >= cols && t.stride(0) % (16 / t.element_size()) == 0 &&
+                  reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0,
+              name, " must be [", T, ", >= ", cols, "] rows of 16-byte aligned ", dt);
+}
+
+SeqParams seqs(const Tensor& slots, const Tensor& start, const Tensor& cu) {
+  SeqParams s{};
+  s.B = slots.numel();
+  s.slots = iptr(slots, s.B, "seq slots");
+  s.start = iptr(start, s.B, "seq starts");
+  s.cu = iptr(cu, s.B + 1, "row offsets");
+  return s;
+}
+
+// y [T, N]: conv channels are columns c0 ..; taps [channels, n], ring [slots, n, channels]
+ConvParams conv(const Tensor& y, int64_t c0, const Tensor& w, const Opt& bias, const Tensor& ring, double gain) {
+  is_f32(y, "y");
+  TORCH_CHECK(w.dim() == 2 && w.size(1) >= 1, "taps must be [channels, n]");
+  ConvParams c{};
+  c.channels = w.size(0);
+  c.taps = w.size(1);
+  rows_of(y, y.scalar_type(), y.size(0), c0 + c.channels, "y");
+  c.y = y.data_ptr(); c.ldy = y.stride(0); c.c0 = c0;
+  c.w = fptr(w, (int64_t)c.channels * c.taps, "taps");
+  if (bias.has_value()) c.bias = fptr(*bias, c.channels, "conv bias");
+  TORCH_CHECK(ring.is_cuda() && ring.scalar_type() == y.scalar_type() && ring.is_contiguous() && ring.dim() == 3 &&
+                  ring.size(1) == c.taps && ring.size(2) == c.channels, "ring must be [slots, taps, channels] like y");
+  c.ring = ring.data_ptr();
+  c.gain = (float)gain;
+  return c;
+}
+
+void state_of(RecurParams& p, const Tensor& state, int64_t heads, int64_t D, int64_t V) {
+  p.heads = heads; p.D = D; p.V = V; p.Vp = (V + 3) / 4 * 4;
+  TORCH_CHECK(state.is_cuda() && state.scalar_type() == torch::kFloat32 && state.is_contiguous() && state.dim() == 4 &&
+                  state.size(1) == heads && state.size(2) == D && state.size(3) == p.Vp,
+              "state must be contiguous fp32 [slots, heads, ", D, ", ", p.Vp, "]");
+  p.S = state.data_ptr<float>();
+}
+
+void out_rows(RecurParams& p, const Tensor& out, const Tensor& y) {
+  rows_of(out, y.scalar_type(), y.size(0), (int64_t)p.heads * p.V, "out");
+  p.out = out.data_ptr(); p.ldo = out.stride(0); p.out_cols = out.size(1);
+}
+
+// y [T, N] rows of q | k | v conv channels from column c0 and beta's logits from
+// gate_col; low [T, >= heads D at 0, heads V at gate_off].  Token by token.
+void delta_seq(Tensor y, int64_t c0, int64_t gate_col, Tensor low, int64_t gate_off, Tensor slots, Tensor start,
+               Tensor cu, int64_t heads, int64_t groups, int64_t D, int64_t V, Tensor taps, Tensor ring, Tensor state,
+               Tensor A, Tensor dt_bias, Tensor norm, double gain, double eps, Tensor out, bool single) {
+  const bool f32 = is_f32(y, "y");
+  RecurParams p{};
+  p.c = conv(y, c0, taps, c10::nullopt, ring, gain);
+  p.s = seqs(slots, start, cu);
+  TORCH_CHECK(groups >= 1 && heads % groups == 0 && D >= 1 && V >= 1, "delta_seq: heads / groups");
+  TORCH_CHECK(p.c.channels == 2 * groups * D + heads * V && gate_col + heads <= y.size(1), "delta_seq: y columns");
+  state_of(p, state, heads, D, V);
+  p.groups = groups;
+  p.q_ch = 0; p.k_ch = groups * D; p.v_ch = 2 * groups * D; p.gate_col = gate_col;
+  rows_of(low, y.scalar_type(), y.size(0), std::max(heads * D, gate_off + heads * V), "low");
+  p.low = low.data_ptr(); p.ldl = low.stride(0); p.gate_off = gate_off;
+  p.A = fptr(A, heads, "A"); p.dt_bias = fptr(dt_bias, heads * D, "dt_bias"); p.norm = fptr(norm, V, "norm");
+  p.eps = (float)eps;
+  out_rows(p, out, y);
+  p.write_ring = single;
+  TORCH_CHECK(!single || p.s.B == y.size(0), "delta_seq: one row per sequence");
+  const int vb = lsd_recur_block(D, V);
+  TORCH_CHECK(vb > 0, "delta_seq: no kernel for key dimension ", D);
+  Tensor raw;
+  if (p.Vp > vb) {
+    raw = torch::empty({y.size(0), heads * V}, y.options().dtype(torch::kFloat32));
+    p.raw = raw.data_ptr<float>(); p.ldr = heads * V;
+  }
+  check_hip(lsd_recur_seq(&p, 1, f32, cur_stream()), "delta_seq");
+  if (p.raw) {
+    MixOutParams o{};
+    o.raw = p.raw; o.ldr = p.ldr; o.T = y.size(0); o.heads = heads; o.V = V;
+    o.low = p.low; o.ldl = p.ldl; o.gate_off = gate_off; o.norm = p.norm; o.eps = p.eps; o.gain = p.c.gain;
+    o.out = p.out; o.ldo = p.ldo; o.out_cols = p.out_cols;
+    check_hip(lsd_head_norm_gate(&o, f32, cur_stream()), "head_norm_gate");
+  }
+  if (!single) check_hip(lsd_conv_tail(&p.c, &p.s, f32, cur_stream()), "conv_tail");
+}
+
+void group_norm_out(const Tensor& raw, const Tensor& y, int64_t inner, int64_t norm_groups, const Tensor& norm, double gain,
+                    double eps, const Tensor& out) {
+  const bool f32 = is_f32(y, "y");
+  MixOutParams o{};
+  o.raw = raw.data_ptr<float>(); o.ldr = inner; o.T = y.size(0); o.inner = inner; o.groups = norm_groups;
+  TORCH_CHECK(norm_groups >= 1 && inner % norm_groups == 0, "norm groups");
+  o.z = y.data_ptr(); o.ldz = y.stride(0);
+  o.norm = fptr(norm, inner, "norm"); o.eps = (float)eps; o.gain = (float)gain;
+  rows_of(out, y.scalar_type(), y.size(0), inner, "out");
+  o.out = out.data_ptr(); o.ldo = out.stride(0); o.out_cols = out.size(1);
+  check_hip(lsd_gated_group_norm(&o, f32, cur_stream()), "gated_group_norm");
+}
+
+// y [T, N]: z | x | B | C | dt.  Token by token.
+void ssm_seq(Tensor y, Tensor slots, Tensor start, Tensor cu, int64_t heads, int64_t groups, int64_t N, int64_t V,
+             int64_t norm_groups, Tensor taps, Tensor bias, Tensor ring, Tensor state, Tensor A, Tensor dt_bias,
+             Tensor skip, Tensor norm, double gain, double eps, Tensor out, bool single) {
+  const bool f32 = is_f32(y, "y");
+  const int64_t inner = heads * V;
+  RecurParams p{};
+  p.c = conv(y, inner, taps, bias, ring, gain);
+  p.s = seqs(slots, start, cu);
+  TORCH_CHECK(groups >= 1 && heads % groups == 0 && N >= 1 && V >= 1, "ssm_seq: heads / groups");
+  TORCH_CHECK(p.c.channels == inner + 2 * groups * N, "ssm_seq: channels");
+  p.gate_col = inner + p.c.channels;
+  TORCH_CHECK(p.gate_col + heads <= y.size(1), "ssm_seq: y columns");
+  state_of(p, state, heads, N, V);
+  p.groups = groups;
+  p.v_ch = 0; p.k_ch = inner; p.q_ch = inner + groups * N;
+  p.A = fptr(A, heads, "A"); p.dt_bias = fptr(dt_bias, heads, "dt_bias"); p.skip = fptr(skip, heads, "D");
+  auto raw = torch::empty({y.size(0), inner}, y.options().dtype(torch::kFloat32));
+  p.raw = raw.data_ptr<float>(); p.ldr = inner;
+  p.write_ring = single;
+  TORCH_CHECK(!single || p.s.B == y.size(0), "ssm_seq: one row per sequence");
+  TORCH_CHECK(lsd_recur_block(N, V) > 0, "ssm_seq: no kernel for state size ", N);
+  check_hip(lsd_recur_seq(&p, 0, f32, cur_stream()), "ssm_seq");
+  group_norm_out(raw, y, inner, norm_groups, norm, gain, eps, out);
+  if (!single) check_hip(lsd_conv_tail(&p.c, &p.s, f32, cur_stream()), "conv_tail");
+}
+
+// rows [x | x0] (fp32 or bf16) of a loop's entry; x <- step
+Tensor loop_pack(Tensor x, Tensor x0, Tensor step, bool f32) {
+  const int64_t T = x.size(0), H = x.size(1);
+  fptr(x0, T * H, "x0");
+  fptr(step, H, "step");
+  auto out = torch::empty({T, 2 * H}, x.options().dtype(f32 ? torch::kFloat32 : torch::kBFloat16));
+  check_hip(lsd_loop_pack(const_cast<float*>(fptr(x, T * H, "x")), x0.data_ptr<float>(), step.data_ptr<float>(),
+                          out.data_ptr(), T, H, f32, cur_stream()), "loop_pack");
+  return out;
+}
+
+// y fp32 [T, 2F] (gate / up in 16-row blocks) -> out [T, F]
+void gelu_mul_f32(Tensor y, Tensor out, double scale) {
+  const int64_t T = y.size(0), F = y.size(1) / 2;
+  fptr(y, T * F * 2, "y");
+  TORCH_CHECK(F % 16 == 0, "gelu_mul_f32: F % 16");
+  rows_of(out, torch::kFloat32, T, F, "out");
+  check_hip(lsd_gelu_mul_f32(y.data_ptr<float>(), out.data_ptr<float>(), T, F, out.stride(0), (float)scale,
+                             cur_stream()), "gelu_mul_f32");
+}
+
+void need_pools(const Tensor& k, const Tensor& v, const Tensor& table, c10::ScalarType dt) {
+  TORCH_CHECK(k.is_cuda() && k.scalar_type() == dt && v.scalar_type() == dt && k.dim() == 4 && v.dim() == 4 &&
+                  k.is_contiguous() && v.is_contiguous() && k.size(2) == PAGE && v.size(2) == PAGE &&
+                  k.size(0) == v.size(0) && k.size(1) == v.size(1), "pools must be [pages, kv heads, 64, dim]");
+  TORCH_CHECK(table.is_cuda() && table.scalar_type() == torch::kInt32 && table.dim() == 2 && table.is_contiguous(),
+              "table must be contiguous [slots, pages per sequence]");
+}
+
+// y [T, N]: q [heads dim] | k [G dim] | v [G vdim] -> rotated q [T, heads dim]; k, v appended
+Tensor rope_append(Tensor y, int64_t heads, Tensor k, Tensor v, Tensor table, Tensor tslot, Tensor tpos, Opt rope,
+                   double gain) {
+  const bool f32 = is_f32(y, "y");
+  need_pools(k, v, table, y.scalar_type());
+  RopeAppendParams p{};
+  p.T = y.size(0); p.H = heads; p.G = k.size(1); p.dim = k.size(3); p.vdim = v.size(3);
+  rows_of(y, y.scalar_type(), p.T, (p.H + p.G) * p.dim + p.G * p.vdim, "y");
+  p.y = y.data_ptr(); p.ldy = y.stride(0); p.gain = (float)gain;
+  if (rope.has_value()) {
+    TORCH_CHECK(rope->dim() == 3 && rope->size(2) == 2 && 2 * rope->size(1) <= p.dim &&
+                    rope->size(0) >= table.size(1) * (int64_t)PAGE, "rope must be [>= positions, half, 2]");
+    p.rope = fptr(*rope, rope->numel(), "rope"); p.half = rope->size(1);
+  }
+  auto q = torch::empty({p.T, heads * p.dim}, y.options());
+  p.q = q.data_ptr(); p.k = k.data_ptr(); p.v = v.data_ptr();
+  p.table = table.data_ptr<int>(); p.tw = table.size(1);
+  p.tslot = iptr(tslot, p.T, "tslot"); p.tpos = iptr(tpos, p.T, "tpos");
+  check_hip(lsd_rope_append(&p, f32, cur_stream()), "rope_append");
+  return q;
+}
+
+TalkParams talk_base(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& table, const Opt& talk, int64_t window,
+                     double scale, double cap, const Tensor& out) {
+  is_f32(q, "q");
+  need_pools(k, v, table, q.scalar_type());
+  TalkParams p{};
+  p.G = k.size(1); p.dim = k.size(3); p.vdim = v.size(3); p.H = q.size(1) / p.dim;
+  TORCH_CHECK(q.dim() == 2 && q.is_contiguous() && q.size(1) == (int64_t)p.H * p.dim && p.H % p.G == 0,
+              "q must be contiguous [T, heads dim]");
+  TORCH_CHECK(window >= 1, "window must be positive");
+  p.T = q.size(0);
+  p.q = q.data_ptr(); p.k = k.data_ptr(); p.v = v.data_ptr();
+  p.table = table.data_ptr<int>(); p.tw = table.size(1);
+  if (talk.has_value()) p.talk = fptr(*talk, (int64_t)p.H * p.H, "talk");
+  p.window = (int)std::min<int64_t>(window, INT_MAX);
+  p.scale = (float)scale; p.cap = (float)cap;
+  rows_of(out, q.scalar_type(), p.T, (int64_t)p.H * p.vdim, "out");
+  p.out = out.data_ptr(); p.ldo = out.stride(0); p.out_cols = out.size(1);
+  return p;
+}
+
+// every row is a query of its own: slots / pos [T]
+void talk_plain(Tensor q, Tensor k, Tensor v, Tensor table, Tensor slots, Tensor pos, Opt talk, int64_t window,
+                double scale, double cap, Tensor out) {
+  TalkParams p = talk_base(q, k, v, table, talk, window, scale, cap, out);
+  p.slots = iptr(slots, p.T, "slots"); p.pos = iptr(pos, p.T, "pos");
+  TORCH_CHECK(lsd_talk_plain_lds(&p) <= MAX_LDS, "talk_plain: ", p.H, " heads of ", p.dim, " / ", p.vdim,
+              " do not fit the LDS");
+  check_hip(lsd_talk_plain(&p, is_f32(q, "q"), cur_stream()), "talk_plain");
+}
+
+}  // namespace
+
+void lsd_register_mixers(pybind11::module& m) {
+  m.def("delta_seq", &delta_seq, py::arg("y"), py::arg("c0"), py::arg("gate_col"), py::arg("low"), py::arg("gate_off"),
+        py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("heads"), py::arg("groups"), py::arg("dim"),
+        py::arg("vdim"), py::arg("taps"), py::arg("ring"), py::arg("state"), py::arg("A"), py::arg("dt_bias"),
+        py::arg("norm"), py::arg("gain"), py::arg("eps"), py::arg("out"), py::arg("single"));
+  m.def("ssm_seq", &ssm_seq, py::arg("y"), py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("heads"),
+        py::arg("groups"), py::arg("state_dim"), py::arg("vdim"), py::arg("norm_groups"), py::arg("taps"), py::arg("bias"),
+        py::arg("ring"), py::arg("state"), py::arg("A"), py::arg("dt_bias"), py::arg("skip"), py::arg("norm"),
+        py::arg("gain"), py::arg("eps"), py::arg("out"), py::arg("single"));
+  m.def("loop_pack", &loop_pack, py::arg("x"), py::arg("x0"), py::arg("step"), py::arg("f32"));
+  m.def("gelu_mul_f32", &gelu_mul_f32, py::arg("y"), py::arg("out"), py::arg("scale"));
+  m.def("rope_append", &rope_append, py::arg("y"), py::arg("heads"), py::arg("k"), py::arg("v"), py::arg("table"),
+        py::arg("tslot"), py::arg("tpos"), py::arg("rope"), py::arg("gain"));
+  m.def("talk_plain", &talk_plain, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("slots"),
+        py::arg("pos"), py::arg("talk"), py::arg("window"), py::arg("scale"), py::arg("cap"), py::arg("out"));
+}

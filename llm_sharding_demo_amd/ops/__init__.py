@@ -60,6 +60,13 @@ class Backend:
         """`width` argument of the norms: the true row width where rows are padded, else 0."""
         return mcfg.hidden if self.row_width(mcfg) != mcfg.hidden else 0
 
+    @staticmethod
+    def _parts(meta):
+        """(rows, meta) of a step's decode rows and prompt chunks."""
+        if getattr(meta, "dec", None) is not None:
+            return [(slice(0, meta.b), meta.dec), (slice(meta.b, meta.num_tokens), meta.pf)]
+        return [(slice(0, meta.num_tokens), meta)]
+
     def prepare_prefill(self, meta, mcfg) -> None:
         """Device-side helpers of a prefill batch, made before a graph capture."""
 
@@ -156,13 +163,6 @@ class ReferenceBackend(Backend):
         fn = (self._attend if isinstance(m, AttentionSpec) else
               self._channel_delta if isinstance(m, ChannelDeltaSpec) else self._ssm)
         return fn(h, w, m, kv, entry, meta, eps)
-
-    @staticmethod
-    def _parts(meta):
-        """(rows, meta) of a step's decode rows and prompt chunks."""
-        if getattr(meta, "dec", None) is not None:
-            return [(slice(0, meta.b), meta.dec), (slice(meta.b, meta.num_tokens), meta.pf)]
-        return [(slice(0, meta.num_tokens), meta)]
 
     def _attend(self, h, w, m, kv, entry, meta, eps):
         pos = meta.token_pos

@@ -12,8 +12,9 @@ Device weight layout (set up once per stage by `prepare_stage`):
     q and the K cache simply live in that order.
   * Llama gate/up rows interleaved in 16-row blocks so one wave holds the gate
     and up value of the same output column (silu(gate)*up fused epilogue).
-  * Timisun: every width padded with zeros to what the MFMA tiles want, so a
-    model of any sizes runs (see _prepare_timisun); fp32 or bf16.
+  * Timisun, Vizalix: every width padded with zeros to what the MFMA tiles
+    want, so a model of any sizes runs (see _prepare_timisun and
+    _prepare_vizalix); fp32 or bf16.
 """
 from __future__ import annotations
 
@@ -24,6 +25,8 @@ from typing import Optional
 import numpy as np
 import torch
 
+from ..config import AttentionSpec, ChannelDeltaSpec, RopeSpec, SSMSpec
+from ..runtime.kv_cache import layer_cache
 from . import GLU_ALPHA, Backend, Residual
 from .routing import Routing
 
@@ -107,6 +110,12 @@ def rope_table(max_pos: int, hd: int, theta: float, device) -> torch.Tensor:
     return torch.stack([ang.cos(), ang.sin()], -1).float().contiguous().to(device)
 
 
+def rope_spec_table(rope: RopeSpec, max_pos: int, device) -> torch.Tensor:
+    """[max_pos, dims / 2, 2] cos, sin of a partial rotation, angles in fp64."""
+    ang = torch.arange(max_pos, dtype=torch.float64)[:, None] * torch.tensor(rope.frequencies(), dtype=torch.float64)
+    return torch.stack([ang.cos(), ang.sin()], -1).float().contiguous().to(device)
+
+
 def prefill_tiles(meta) -> torch.Tensor:
     """(sequence, query offset) of every 64-query tile of a packed batch."""
     qlens = meta.host_qlens
@@ -182,10 +191,12 @@ class HipBackend(Backend):
     def prepare_stage(self, stage) -> None:
         cfg, w, dev = stage.cfg, stage.w, stage.device
         self.fp32 = stage.dtype == torch.float32
-        if self.fp32 and cfg.arch != "timisun":
+        if self.fp32 and not cfg.layers:
             raise ValueError(f"{cfg.arch} has no fp32 kernels: serve it in bf16")
         if cfg.arch == "timisun":
             self._prepare_timisun(stage)
+        elif cfg.arch == "vizalix":
+            self._prepare_vizalix(stage)
         elif stage.last:
             # pad the head IN PLACE: the stage keeps one [vocab_padded, H]
             # tensor and its weight dict points at the first V rows (a
@@ -223,7 +234,10 @@ class HipBackend(Backend):
 
     # -- Timisun ---------------------------------------------------------------
     def row_width(self, mcfg) -> int:
-        return _up(mcfg.hidden, 64) if mcfg.arch == "timisun" else mcfg.hidden
+        return _up(mcfg.hidden, 64) if mcfg.layers else mcfg.hidden
+
+    def layer_cache(self, mixer):
+        return layer_cache(mixer, _up)
 
     def latent_width(self, rank: int) -> int:
         return _up(rank, 64)
@@ -282,6 +296,140 @@ class HipBackend(Backend):
             w[p + "attn.uv.weight"] = pad_to(t("attn.uv.weight").reshape(m.heads, m.vdim, m.kv_rank), m.heads, vp, rank)
             o = t("attn.o.weight").reshape(-1, m.heads, m.vdim)
             w[p + "attn.o.weight"] = pad_to(o, hp, m.heads, vp).reshape(hp, m.heads * vp)
+
+    def _prepare_vizalix(self, stage) -> None:
+        """Device layout per layer (zero padding everywhere):
+          mixer.in     rows of one in-projection
+                       attention   q | k | v, dims of a head padded
+                       delta rule  a1 | g1 (each to the same 64-multiple) | q | k | v | b
+                       Mamba-2     as stored: z | x | B | C | dt
+          mixer.low    [2][heads dim | heads vdim][rank]: the delta rule's a2 and g2
+          mixer.out    [W_o | W_down] side by side: one residual projection over
+                       the mixer's output and the feed-forward's inner row
+          mlp.gate_up  interleaved in 16-row blocks
+        Norm gains (one number each) stay on the host: they are factors of the
+        kernels behind the projections.  Decays, biases, taps and norm weights
+        of the recurrences, and the head mixing, are fp32."""
+        cfg, w, dev = stage.cfg, stage.w, stage.device
+        hp = self.row_width(cfg)
+        self._ones = torch.ones(hp, dtype=stage.dtype, device=dev)
+        self._ropes = {}
+        if "embed_tokens" in w:
+            w["embed_tokens"] = pad_to(w["embed_tokens"], cfg.vocab_size, hp)
+        if "lm_head" in w:
+            e = pad_to(w["lm_head"], cfg.vocab_padded, hp)
+            w["lm_head"], stage._lm_head_padded = e[: cfg.vocab_size], e
+            w["norm.weight"] = w["norm.weight"].expand(hp).contiguous()
+        if "loop.in" in w:
+            li = torch.stack(w["loop.in"].split(cfg.hidden, 1), 1)  # [H, 2, H]
+            w["loop.in"] = pad_to(li, hp, 2, hp).reshape(hp, 2 * hp)
+            w["loop.step"] = pad_to(w["loop.step"].float(), cfg.loop_times, hp)
+        for j, i in {cfg.weight_layer(i): i for i in stage.layers}.items():
+            m, f, p = cfg.layers[i].mixer, cfg.layers[i].mlp, f"layers.{j}."
+            t = lambda n: w.pop(p + n)  # noqa: E731
+            f32 = lambda n: w.__setitem__(p + n, w[p + n].float().contiguous())  # noqa: E731
+            w[p + "input_layernorm.weight"] = w[p + "input_layernorm.weight"].float().cpu()
+            o = t("mixer.o")
+            if isinstance(m, AttentionSpec):
+                dp, vp = _up(m.dim, 32), _up(m.vdim, 16)
+                rows = [pad_to(t(f"mixer.{n}").reshape(h, d, -1), h, dd, hp).reshape(h * dd, hp) for n, h, d, dd in (
+                    ("q", m.heads, m.dim, dp), ("k", m.kv_heads, m.dim, dp), ("v", m.kv_heads, m.vdim, vp))]
+                o = pad_to(o.reshape(-1, m.heads, m.vdim), o.shape[0], m.heads, vp).reshape(-1, m.heads * vp)
+                if m.talking:
+                    f32("mixer.talk")
+                if m.rope is not None and m.rope.dims and m.rope not in self._ropes:
+                    self._ropes[m.rope] = rope_spec_table(m.rope, _up(stage.max_seq, 64), dev)
+            elif isinstance(m, ChannelDeltaSpec):
+                kr, n = self._low_rank(m), self._low_cols(m)
+                rows = [pad_to(t("mixer.a1"), kr, hp), pad_to(t("mixer.g1"), kr, hp)]
+                rows += [pad_to(t(f"mixer.{x}"), s, hp) for x, s in (
+                    ("q", m.kv_heads * m.dim), ("k", m.kv_heads * m.dim), ("v", m.heads * m.vdim), ("b", m.heads))]
+                w[p + "mixer.low.weight"] = torch.stack([pad_to(t("mixer.a2"), n, kr), pad_to(t("mixer.g2"), n, kr)])
+                w[p + "mixer.taps"] = torch.cat([t(f"mixer.{x}.conv") for x in "qkv"]).float().contiguous()
+                w[p + "mixer.A"] = -torch.exp(t("mixer.A_log").float())
+                f32("mixer.dt_bias")
+                f32("mixer.norm")
+            else:
+                rows = [pad_to(t("mixer.in"), m.inner + m.conv_channels + m.heads, hp)]
+                w[p + "mixer.taps"] = t("mixer.conv").float().contiguous()
+                w[p + "mixer.A"] = -torch.exp(t("mixer.A_log").float())
+                for n in ("conv.b", "dt_bias", "D", "norm"):
+                    f32("mixer." + n)
+            n = sum(x.shape[0] for x in rows)
+            w[p + "mixer.in.weight"] = pad_to(torch.cat(rows), _up(n, 64), hp)
+            oc = _up(o.shape[1], 64)
+            out = [pad_to(o, hp, oc)]
+            if f is not None:
+                fp = _up(f.ff, 64)
+                w[p + "post_attention_layernorm.weight"] = w[p + "post_attention_layernorm.weight"].float().cpu()
+                w[p + "mlp.gate_up.weight"] = interleave_experts(t("mlp.gate_up.weight"), fp, hp)
+                out.append(pad_to(t("mlp.down_proj.weight"), hp, fp))
+            w[p + "mixer.out.weight"] = torch.cat(out, 1).contiguous()
+
+    @staticmethod
+    def _low_rank(m) -> int:
+        return _up(max(m.decay_rank, m.gate_rank), 64)
+
+    @staticmethod
+    def _low_cols(m) -> int:
+        return _up(max(m.heads * m.dim, m.heads * m.vdim), 16)
+
+    # -- mixers of models/stage.py _mixer_layer --------------------------------
+    def loop_enter(self, r: Residual, x0, w_in, step, t: int) -> None:
+        self.flush(r)
+        self.linear_residual(self.C.loop_pack(r.x, x0, step[t], self.fp32), w_in, None, r)
+
+    def unit_rmsnorm(self, r: Residual, mcfg):
+        return self.rmsnorm(r, self._ones, mcfg.norm_eps, width=self.norm_width(mcfg))
+
+    def _rows(self, h, w):
+        """In-projection rows in the element type."""
+        return self.C.linear_fp32(h, w) if self.fp32 else self.linear(h, w)
+
+    def mix(self, h, w, spec, kv, entry, meta, eps):
+        """Mixer output, and room for the feed-forward's inner row behind it:
+        [T, out columns + ff columns], the operand of the residual projection."""
+        m, gain = spec.mixer, float(w("input_layernorm.weight"))
+        y = self._rows(h, w("mixer.in.weight"))
+        buf = torch.empty(y.shape[0], w("mixer.out.weight").shape[1], dtype=y.dtype, device=y.device)
+        ff = _up(spec.mlp.ff, 64) if spec.mlp is not None else 0
+        out = buf[:, : buf.shape[1] - ff]
+        fn = (self._attend if isinstance(m, AttentionSpec) else
+              self._channel_delta if isinstance(m, ChannelDeltaSpec) else self._ssm)
+        fn(y, w, m, gain, kv, entry, meta, eps, out)
+        return buf
+
+    def mixer_residual(self, buf, h, w, spec, r: Residual) -> None:
+        if spec.mlp is not None:
+            gain, gu = float(w("post_attention_layernorm.weight")), w("mlp.gate_up.weight")
+            mid = buf[:, buf.shape[1] - gu.shape[0] // 2:]
+            if self.fp32:
+                self.C.gelu_mul_f32(self.C.linear_fp32(h, gu), mid, gain)
+            else:
+                self.linear(h, gu, act="gelu_mul", out=mid, scale=gain)
+        self.linear_residual(buf, w("mixer.out.weight"), None, r)
+
+    def _attend(self, y, w, m, gain, kv, entry, meta, eps, out):
+        k, v = entry
+        rope = self._ropes[m.rope] if m.rope is not None and m.rope.dims else None
+        q = self.C.rope_append(y, m.heads, k, v, kv.table, meta.token_slots, meta.token_pos, rope, gain)
+        for s, mt in self._parts(meta):
+            self.C.talk_plain(q[s], k, v, kv.table, mt.token_slots, mt.token_pos, w("mixer.talk") if m.talking else None,
+                              m.window or 1 << 30, m.scale, m.softcap or 0.0, out[s])
+
+    def _channel_delta(self, y, w, m, gain, kv, entry, meta, eps, out):
+        low = self._batch_linear(y, w("mixer.low.weight"))
+        c0, n = 2 * self._low_rank(m), self._low_cols(m)
+        for s, mt in self._parts(meta):
+            self.C.delta_seq(y[s], c0, c0 + m.conv_channels, low[s], n, mt.seq_slots, mt.q_start, mt.cu_q, m.heads,
+                             m.kv_heads, m.dim, m.vdim, w("mixer.taps"), entry[1], entry[0], w("mixer.A"),
+                             w("mixer.dt_bias"), w("mixer.norm"), gain, eps, out[s], mt.is_decode)
+
+    def _ssm(self, y, w, m, gain, kv, entry, meta, eps, out):
+        for s, mt in self._parts(meta):
+            self.C.ssm_seq(y[s], mt.seq_slots, mt.q_start, mt.cu_q, m.heads, m.groups, m.state, m.vdim, m.norm_groups,
+                           w("mixer.taps"), w("mixer.conv.b"), entry[1], entry[0], w("mixer.A"), w("mixer.dt_bias"),
+                           w("mixer.D"), w("mixer.norm"), gain, eps, out[s], mt.is_decode)
 
     def _tm(self, rows: float) -> int:
         return 64 if self.fp32 else self.R.group_tm(rows)
@@ -366,6 +514,8 @@ class HipBackend(Backend):
         return cache[heads]
 
     def prepare_prefill(self, meta, mcfg) -> None:
+        if mcfg.arch == "vizalix":
+            return
         if mcfg.arch != "timisun":
             meta._tiles = prefill_tiles(meta).to(meta.cu_q.device)
             return
@@ -459,7 +609,7 @@ class HipBackend(Backend):
         return self.C.embed(ids, pos, wte, wpe, scale)
 
     def _norm(self, r: Residual, w, b, eps, rms: bool, offset: float = 0.0, width: int = 0):
-        if not offset and not width and not r.pending and r.x.shape[0] <= self.R.gemv_norm_max_m and r.x.shape[1] % 8 == 0:
+        if not self.fp32 and not offset and not width and not r.pending and r.x.shape[0] <= self.R.gemv_norm_max_m and r.x.shape[1] % 8 == 0:
             return LazyNorm(r.x, w, b, eps, rms)
         self._flush_extra(r)
         slab, pb = (r.pending[0] if r.pending else (None, None))
@@ -552,7 +702,11 @@ class HipBackend(Backend):
         return self.C.attn_prefill(q, cache_k, cache_v, tiles, meta.seq_slots, meta.q_start,
                                    meta.cu_q, nh)
 
-    def linear(self, a, w, b=None, act: str = "none"):
+    def linear(self, a, w, b=None, act: str = "none", out=None, scale: float = 1.0):
+        """act(a w^T + b) in bf16; out: the caller's rows; scale: common factor
+        of a gated activation's halves."""
+        if act == "gelu_mul" or out is not None:
+            return self._linear_into(a, w, act, out, scale)
         code = _EPI[act]
         g = self._gemv_in(a, w.shape[1], code)
         if g is not None:
@@ -571,6 +725,17 @@ class HipBackend(Backend):
                 return self.C.silu_mul(y)
         tiled, splits = self._gemm_kw(a.shape[0], w.shape[0], w.shape[1], 2 if code == 2 else 1)
         return self.C.linear(a, w, b, code, tiled, splits, self.counters)
+
+    def _linear_into(self, a, w, act: str, out, scale: float):
+        gelu = act == "gelu_mul"
+        code = 2 if gelu else _EPI[act]
+        g = self._gemv_in(a, w.shape[1], code)
+        if g is not None:
+            x, nc, gw, gb, eps = g
+            return self.C.gemv_into(x, w, code, nc, gw, gb, eps, out, gelu, scale)
+        a = self.materialize(a)
+        tiled, splits = self._gemm_kw(a.shape[0], w.shape[0], w.shape[1], 2 if code == 2 else 1)
+        return self.C.linear(a, w, None, 3 if gelu else code, tiled, splits, self.counters, out, scale)
 
     def linear_residual(self, a, w, b, r: Residual, room=None) -> None:
         """x += a w^T + b; `room`: slab rows the caller owns and appends to
