@@ -4,10 +4,15 @@
 //
 //  * rope_append: behind the in-projection, rotates q and k, appends k and v to
 //    their page.
+//  * talk_prefill: MFMA, 16 queries of 4 heads per wave, all heads in a block.
+//  * talk_decode: MFMA, one token of all heads per block, keys split over blocks.
 //  * talk_plain: one token per block, any sizes, bf16 or fp32.
 //
 // Every head's score of a (query, key) pair is needed before any head's weight
-// of it is known, so a block works on all heads of its queries.
+// of it is known, so a block works on all heads of its queries.  Scores cross
+// the waves through LDS as two fp16 terms (value and remainder, 22 bits: the cap
+// bounds them) and are mixed by the matrix cores in fp32; softmax weights enter
+// the second product as two bf16 terms.
 #include "common.h"
 #include "mixer_params.h"
 
@@ -137,10 +142,543 @@ __global__ __launch_bounds__(256) void talk_plain_kernel(TalkParams p) {
   for (int i = tid; i < p.out_cols; i += 256) from_f(out + i, i < H * p.vdim ? acc[i] / l[i / p.vdim] : 0.f);
 }
 
+typedef _Float16 half8 __attribute__((ext_vector_type(8)));
+typedef _Float16 half4 __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ f32x4 mfma_f16(half8 a, half8 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0);
+}
+
+// Transposed read of 4 x 16 LDS blocks: k runs over rows, the result's lanes over columns.
+__device__ __forceinline__ bf16x4 ds_read_tr(const bf16* lds_ptr) {
+  typedef __attribute__((address_space(3))) bf16x4 lds_bf16x4;
+  return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds_bf16x4*)(lds_ptr));
+}
+
+// This wave's LDS accesses are done
+__device__ __forceinline__ void lds_fence() {
+  __builtin_amdgcn_s_waitcnt(0xC07F);  // lgkmcnt(0)
+  __builtin_amdgcn_wave_barrier();
+}
+
+// cap tanh(x): `two_over` is 2 log2(e) scale / cap, the factor of the raw product
+__device__ __forceinline__ float capped(float raw, float two_over, float cap) {
+  const float t = __builtin_amdgcn_exp2f(raw * two_over);
+  return cap - 2.f * cap * __builtin_amdgcn_rcpf(1.f + t);
+}
+
+// Two bf16 terms of eight weights
+__device__ __forceinline__ void split_p(const float* a, const float* b, u32x4& hi, u32x4& lo) {
+  bf16x8 h, l;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    h[j] = f2bf(a[j]);
+    l[j] = f2bf(a[j] - bf2f(h[j]));
+    h[4 + j] = f2bf(b[j]);
+    l[4 + j] = f2bf(b[j] - bf2f(h[4 + j]));
+  }
+  hi = __builtin_bit_cast(u32x4, h);
+  lo = __builtin_bit_cast(u32x4, l);
+}
+
+// x[k] of lane group g  ->  x[g] of lane group k (groups of 16 lanes)
+__device__ __forceinline__ void transpose_groups(u32x4 (&x)[4]) {
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const auto a = __builtin_amdgcn_permlane32_swap(x[0][e], x[2][e], false, false);
+    const auto b = __builtin_amdgcn_permlane32_swap(x[1][e], x[3][e], false, false);
+    const auto c = __builtin_amdgcn_permlane16_swap(a[0], b[0], false, false);
+    const auto d = __builtin_amdgcn_permlane16_swap(a[1], b[1], false, false);
+    x[0][e] = c[0];
+    x[1][e] = c[1];
+    x[2][e] = d[0];
+    x[3][e] = d[1];
+  }
+}
+
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr int VLD = 64 + 8;  // row pitch of 64 staged V columns
+
+// Prompt attention.  8 waves: HP / 4 of them share 16 queries, each owning 4
+// consecutive heads; 32 / HP query groups per block.  Per 32-key tile: scores of
+// the own heads -> LDS -> barrier -> every wave mixes the scores of all heads
+// into its own four (row 4 g of the product is head g, so lane (r, g) ends with
+// all keys of query r, head g) -> barrier -> softmax in the lane, weights
+// transposed between lane groups and registers, second product per head.
+template <int DKS, int VT, int HP>
+__global__ __launch_bounds__(512, 1) void talk_prefill_kernel(TalkParams p) {
+  constexpr int TK = 32, HW = HP / 4, QG = 8 / HW;
+  constexpr int PITCH = HP == 8 ? 8 : HP + 8;  // fp16 scores of one pair
+  constexpr int PLANE = TK * 16 * PITCH;
+  __shared__ __attribute__((aligned(16))) _Float16 ss[QG * 2 * PLANE];
+  __shared__ __attribute__((aligned(16))) bf16 vst[8][TK * VLD];
+  const int tile = xcd_remap(blockIdx.x, gridDim.x);
+  const int seq = p.tiles[2 * tile], off = p.tiles[2 * tile + 1];
+  const int cu = p.s.cu[seq], qlen = p.s.cu[seq + 1] - cu, st = p.s.start[seq];
+  const int* table = p.table + (long)p.s.slots[seq] * p.tw;
+  const bf16* K = static_cast<const bf16*>(p.k);
+  const bf16* V = static_cast<const bf16*>(p.v);
+  const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int hw = w % HW, qg = w / HW, H = p.H, G = p.G, rep = H / G, dim = p.dim, vdim = p.vdim;
+  _Float16* s_hi = ss + qg * 2 * PLANE;
+  _Float16* s_lo = s_hi + PLANE;
+  bf16* vs = vst[w];
+
+  const int qi = off + qg * 16 + r, qc = min(qi, qlen - 1);
+  const int my_pos = st + qc, my_lo = first_key(my_pos, p.window);
+  int kv[4];
+#pragma unroll
+  for (int hh = 0; hh < 4; ++hh) kv[hh] = min(hw * 4 + hh, H - 1) / rep;
+  const int q_at = (cu + qc) * H * dim + g * 8;
+  half8 tf = {};
+  if ((r & 3) == 0 && g * 8 < HP)
+    tf = *reinterpret_cast<const half8*>(static_cast<const _Float16*>(p.talk_frag) + (hw * 4 + (r >> 2)) * HP + g * 8);
+
+  f32x4 o[4][VT];
+#pragma unroll
+  for (int hh = 0; hh < 4; ++hh)
+#pragma unroll
+    for (int di = 0; di < VT; ++di) o[hh][di] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m = NEG, lsum = 0.f;
+  const float two_over = 2.f * LOG2E * p.scale / p.cap;
+  const int lo = first_key(st + off, p.window), hi = st + min(off + QG * 16, qlen);
+  const int kt0 = lo / TK, kt1 = (hi + TK - 1) / TK;
+
+  for (int kt = kt0; kt < kt1; ++kt) {
+    const long page = table[kt * TK / PAGE];
+    const int koff = (kt * TK) % PAGE;
+    // scores of the own heads; the queries are read again for every tile (from
+    // L1 / L2): the outputs take the registers
+    f32x4 s[4][2];
+    bf16x8 kf[2][DKS];
+    const bf16* qb = static_cast<const bf16*>(p.q);
+    asm volatile("" : "+s"(qb));  // not hoisted out of the loop
+#pragma unroll
+    for (int hh = 0; hh < 4; ++hh) {
+      const bf16x8 z = {};
+      if (hh == 0 || kv[hh] != kv[hh - 1]) {  // wave-uniform
+        const bf16* kp = K + ((page * G + kv[hh]) * PAGE + koff + r) * dim + g * 8;
+#pragma unroll
+        for (int ni = 0; ni < 2; ++ni)
+#pragma unroll
+          for (int ks = 0; ks < DKS; ++ks) kf[ni][ks] = ks * 32 < dim ? ld8(kp + ni * 16 * dim + ks * 32) : z;
+      }
+      bf16x8 qf[DKS];
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks)
+        qf[ks] = ks * 32 < dim ? ld8(qb + q_at + min(hw * 4 + hh, H - 1) * dim + ks * 32) : z;
+#pragma unroll
+      for (int ni = 0; ni < 2; ++ni) {
+        s[hh][ni] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < DKS; ++ks) s[hh][ni] = mfma16(kf[ni][ks], qf[ks], s[hh][ni]);
+      }
+    }
+#pragma unroll
+    for (int ni = 0; ni < 2; ++ni)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        half4 a, b;
+#pragma unroll
+        for (int hh = 0; hh < 4; ++hh) {
+          const float c = capped(s[hh][ni][i], two_over, p.cap);
+          a[hh] = (_Float16)c;
+          b[hh] = (_Float16)(c - (float)a[hh]);
+        }
+        const int at = ((ni * 16 + 4 * g + i) * 16 + r) * PITCH + hw * 4;
+        *reinterpret_cast<half4*>(s_hi + at) = a;
+        *reinterpret_cast<half4*>(s_lo + at) = b;
+      }
+    __syncthreads();
+    float e[TK];
+#pragma unroll
+    for (int key = 0; key < TK; ++key) {
+      half8 a = {}, b = {};
+      if (g * 8 < HP) {
+        a = *reinterpret_cast<const half8*>(s_hi + (key * 16 + r) * PITCH + g * 8);
+        b = *reinterpret_cast<const half8*>(s_lo + (key * 16 + r) * PITCH + g * 8);
+      }
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+      acc = mfma_f16(tf, a, acc);
+      acc = mfma_f16(tf, b, acc);
+      e[key] = acc[0] * LOG2E;
+    }
+    __syncthreads();  // the next tile's scores may be written
+    const bool whole = kt * TK >= my_lo && kt * TK + TK - 1 <= my_pos;
+    if (!__all(whole)) {
+#pragma unroll
+      for (int key = 0; key < TK; ++key) {
+        const int k = kt * TK + key;
+        e[key] = k >= my_lo && k <= my_pos ? e[key] : NEG;
+      }
+    }
+    float tmax = e[0];
+#pragma unroll
+    for (int key = 1; key < TK; ++key) tmax = fmaxf(tmax, e[key]);
+    // weights are taken relative to m, which follows the running maximum only
+    // when that is more than 2^6 ahead
+    if (__any(tmax > m + 6.f)) {
+      const float mn = fmaxf(m, tmax);
+      const float alpha = __builtin_amdgcn_exp2f(m - mn);
+      m = mn;
+      lsum *= alpha;
+#pragma unroll
+      for (int hh = 0; hh < 4; ++hh) {
+        const float ah = __shfl(alpha, hh * 16 + r, 64);
+#pragma unroll
+        for (int di = 0; di < VT; ++di) o[hh][di] *= ah;
+      }
+    }
+    const float off2 = m > 0.5f * NEG ? m : 0.f;  // no key seen yet: weights of zero
+    float ps = 0.f;
+#pragma unroll
+    for (int key = 0; key < TK; ++key) {
+      e[key] = __builtin_amdgcn_exp2f(e[key] - off2);
+      ps += e[key];
+    }
+    lsum += ps;
+    // k-slot j of group g <-> key 4 g + j (j < 4), 16 + 4 g + (j - 4) (j >= 4)
+    u32x4 ph[4], pl[4];
+#pragma unroll
+    for (int kg = 0; kg < 4; ++kg) split_p(e + 4 * kg, e + 16 + 4 * kg, ph[kg], pl[kg]);
+    transpose_groups(ph);
+    transpose_groups(pl);
+#pragma unroll
+    for (int hh = 0; hh < 4; ++hh) {
+      if (hh > 0 && kv[hh] == kv[hh - 1]) continue;  // done with the head before
+#pragma unroll
+      for (int vh = 0; vh < VT / 4; ++vh) {
+        if (vh * 64 >= vdim) continue;
+        const bf16* vp = V + ((page * G + kv[hh]) * PAGE + koff) * vdim + vh * 64;
+        bf16x8 vr[4];
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+          const int row = c * 8 + (lane >> 3), col = (lane & 7) * 8;
+          const bf16x8 z = {};
+          vr[c] = vh * 64 + col < vdim ? ld8(vp + (long)row * vdim + col) : z;
+        }
+        lds_fence();  // reads of what is staged now are done
+#pragma unroll
+        for (int c = 0; c < 4; ++c) st8(vs + (c * 8 + (lane >> 3)) * VLD + (lane & 7) * 8, vr[c]);
+        lds_fence();
+        const int r0 = 4 * g + (r >> 2);
+#pragma unroll
+        for (int dj = 0; dj < 4; ++dj) {
+          const int col = dj * 16 + 4 * (r & 3);
+          const bf16x4 a = ds_read_tr(vs + r0 * VLD + col);
+          const bf16x4 b = ds_read_tr(vs + (r0 + 16) * VLD + col);
+          const bf16x8 vf = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+#pragma unroll
+          for (int h2 = 0; h2 < 4; ++h2)
+            if (h2 >= hh && kv[h2] == kv[hh]) {  // wave-uniform
+              o[h2][vh * 4 + dj] = mfma16(vf, __builtin_bit_cast(bf16x8, ph[h2]), o[h2][vh * 4 + dj]);
+              o[h2][vh * 4 + dj] = mfma16(vf, __builtin_bit_cast(bf16x8, pl[h2]), o[h2][vh * 4 + dj]);
+            }
+        }
+      }
+    }
+  }
+  const float inv = 1.f / lsum;
+  bf16* out = static_cast<bf16*>(p.out) + (long)(cu + qc) * p.ldo;
+#pragma unroll
+  for (int hh = 0; hh < 4; ++hh) {
+    const float ih = __shfl(inv, hh * 16 + r, 64);
+    const int h = hw * 4 + hh;
+    if (h >= H || qi >= qlen) continue;
+#pragma unroll
+    for (int di = 0; di < VT; ++di) {
+      if (di * 16 >= vdim) continue;
+      st4(out + h * vdim + di * 16 + 4 * g, bf16x4{f2bf(o[hh][di][0] * ih), f2bf(o[hh][di][1] * ih),
+                                                   f2bf(o[hh][di][2] * ih), f2bf(o[hh][di][3] * ih)});
+    }
+  }
+  if (hw == HW - 1 && qi < qlen)
+    for (int c = H * vdim + g; c < p.out_cols; c += 4) out[c] = f2bf(0.f);
+}
+
+// Decode attention: one token of all heads, keys in 64-key tiles (pages).  Four
+// waves share the K / V heads; the columns of a score product are the query heads
+// of one K head.  Mixing: wave w takes keys 16 w .. of the tile, all heads.
+template <int DKS, int VT, int HP>
+__global__ __launch_bounds__(256, 2) void talk_decode_kernel(TalkParams p) {
+  constexpr int PITCH = HP + 8, MT = HP / 16, PLD = PAGE + 8;
+  constexpr int GW = HP / 4;  // K / V heads per wave at most
+  __shared__ __attribute__((aligned(16))) _Float16 s_hi[PAGE * PITCH], s_lo[PAGE * PITCH];
+  __shared__ __attribute__((aligned(16))) bf16 p_hi[HP * PLD], p_lo[HP * PLD];
+  __shared__ __attribute__((aligned(16))) bf16 vst[4][32 * VLD];
+  __shared__ float tmaxs[4][HP], alphas[HP], ms[HP], ls[4][HP];
+  const int b = blockIdx.x, H = p.H, G = p.G, rep = H / G, dim = p.dim, vdim = p.vdim;
+  const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int pos = p.pos[b], lo = first_key(pos, p.window);
+  const int* table = p.table + (long)p.slots[b] * p.tw;
+  const bf16* K = static_cast<const bf16*>(p.k);
+  const bf16* V = static_cast<const bf16*>(p.v);
+  const int t0 = lo / PAGE, nt = pos / PAGE + 1 - t0;
+  const int per = (nt + p.splits - 1) / p.splits;
+  const int ta = t0 + blockIdx.y * per, tb = min(ta + per, t0 + nt);
+  bf16* vs = vst[w];
+  const float two_over = 2.f * LOG2E * p.scale / p.cap;
+
+  half8 tf[MT];
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt) {
+    const half8 z = {};
+    tf[mt] = g * 8 < HP ? *reinterpret_cast<const half8*>(static_cast<const _Float16*>(p.talk_frag) +
+                                                           (mt * 16 + r) * HP + g * 8) : z;
+  }
+  // scores of heads that do not exist stay zero
+  for (int i = threadIdx.x; i < PAGE * PITCH; i += 256) s_hi[i] = s_lo[i] = (_Float16)0.f;
+  if (threadIdx.x < HP) ms[threadIdx.x] = NEG;
+  f32x4 o[GW / 4 > 0 ? GW / 4 : 1][VT];
+  constexpr int GMAX = GW / 4 > 0 ? GW / 4 : 1;  // heads per wave the accumulators hold: 4 GMAX >= G
+#pragma unroll
+  for (int c = 0; c < GMAX; ++c)
+#pragma unroll
+    for (int di = 0; di < VT; ++di) o[c][di] = f32x4{0.f, 0.f, 0.f, 0.f};
+  f32x4 lsum[MT];
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt) lsum[mt] = f32x4{0.f, 0.f, 0.f, 0.f};
+  __syncthreads();
+
+  for (int kt = ta; kt < tb; ++kt) {
+    const long page = table[kt];
+#pragma unroll
+    for (int c = 0; c < GMAX; ++c) {
+      const int kvh = w + 4 * c;
+      if (kvh >= G) continue;
+      bf16x8 qf[DKS], kf[4][DKS];
+      const bf16* q = static_cast<const bf16*>(p.q) + ((long)b * H + kvh * rep + min(r, rep - 1)) * dim + g * 8;
+      const bf16* kp = K + ((page * G + kvh) * PAGE + r) * dim + g * 8;
+      const bf16x8 z = {};
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks) qf[ks] = ks * 32 < dim ? ld8(q + ks * 32) : z;
+#pragma unroll
+      for (int ni = 0; ni < 4; ++ni)
+#pragma unroll
+        for (int ks = 0; ks < DKS; ++ks) kf[ni][ks] = ks * 32 < dim ? ld8(kp + (long)ni * 16 * dim + ks * 32) : z;
+#pragma unroll
+      for (int ni = 0; ni < 4; ++ni) {
+        f32x4 s = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < DKS; ++ks) s = mfma16(kf[ni][ks], qf[ks], s);
+        if (r < rep) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const float cv = capped(s[i], two_over, p.cap);
+            const _Float16 a = (_Float16)cv;
+            const int at = (ni * 16 + 4 * g + i) * PITCH + kvh * rep + r;
+            s_hi[at] = a;
+            s_lo[at] = (_Float16)(cv - (float)a);
+          }
+        }
+      }
+    }
+    __syncthreads();
+    // column r: key 16 w + r, rows: heads
+    f32x4 e[MT];
+    const int key = kt * PAGE + w * 16 + r;
+    const bool seen = key >= lo && key <= pos;
+    {
+      half8 a = {}, bq = {};
+      if (g * 8 < HP) {
+        a = *reinterpret_cast<const half8*>(s_hi + (w * 16 + r) * PITCH + g * 8);
+        bq = *reinterpret_cast<const half8*>(s_lo + (w * 16 + r) * PITCH + g * 8);
+      }
+#pragma unroll
+      for (int mt = 0; mt < MT; ++mt) {
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+        acc = mfma_f16(tf[mt], a, acc);
+        acc = mfma_f16(tf[mt], bq, acc);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          e[mt][i] = seen ? acc[i] * LOG2E : NEG;
+          float t = e[mt][i];
+          t = fmaxf(t, wave_xchg<1>(t));
+          t = fmaxf(t, wave_xchg<2>(t));
+          t = fmaxf(t, wave_xchg<4>(t));
+          t = fmaxf(t, wave_xchg<8>(t));
+          if (r == 0) tmaxs[w][mt * 16 + 4 * g + i] = t;
+        }
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int h = mt * 16 + 4 * g + i;
+        const float mo = ms[h];
+        const float t = fmaxf(fmaxf(tmaxs[0][h], tmaxs[1][h]), fmaxf(tmaxs[2][h], tmaxs[3][h]));
+        const float mn = t > mo + 6.f ? t : mo;  // every tile of the range holds a visible key
+        const float pw = __builtin_amdgcn_exp2f(e[mt][i] - mn);
+        const float al = __builtin_amdgcn_exp2f(mo - mn);
+        lsum[mt][i] = lsum[mt][i] * al + pw;
+        const bf16 ph = f2bf(pw);
+        p_hi[h * PLD + w * 16 + r] = ph;
+        p_lo[h * PLD + w * 16 + r] = f2bf(pw - bf2f(ph));
+        if (w == 0 && r == 0) alphas[h] = al;
+        e[mt][i] = mn;
+      }
+    }
+    __syncthreads();
+    if (w == 0 && r == 0) {
+#pragma unroll
+      for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) ms[mt * 16 + 4 * g + i] = e[mt][i];
+    }
+#pragma unroll
+    for (int c = 0; c < GMAX; ++c) {
+      const int kvh = w + 4 * c;
+      if (kvh >= G) continue;
+      const int h = kvh * rep + min(r, rep - 1);
+      const float al = alphas[h];
+      if (__any(al != 1.f)) {
+#pragma unroll
+        for (int di = 0; di < VT; ++di) o[c][di] *= al;
+      }
+#pragma unroll
+      for (int vh = 0; vh < VT / 4; ++vh) {
+        if (vh * 64 >= vdim) continue;
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+          const bf16* vp = V + ((page * G + kvh) * PAGE + kk * 32) * vdim + vh * 64;
+          bf16x8 vr[4];
+#pragma unroll
+          for (int q4 = 0; q4 < 4; ++q4) {
+            const int row = q4 * 8 + (lane >> 3), col = (lane & 7) * 8;
+            const bf16x8 z = {};
+            vr[q4] = vh * 64 + col < vdim ? ld8(vp + (long)row * vdim + col) : z;
+          }
+          const bf16* ph = p_hi + h * PLD + kk * 32 + 4 * g;
+          const bf16* pl = p_lo + h * PLD + kk * 32 + 4 * g;
+          const bf16x4 h0 = ld4(ph), h1 = ld4(ph + 16), l0 = ld4(pl), l1 = ld4(pl + 16);
+          const bf16x8 hf = {h0[0], h0[1], h0[2], h0[3], h1[0], h1[1], h1[2], h1[3]};
+          const bf16x8 lf = {l0[0], l0[1], l0[2], l0[3], l1[0], l1[1], l1[2], l1[3]};
+          lds_fence();
+#pragma unroll
+          for (int q4 = 0; q4 < 4; ++q4) st8(vs + (q4 * 8 + (lane >> 3)) * VLD + (lane & 7) * 8, vr[q4]);
+          lds_fence();
+          const int r0 = 4 * g + (r >> 2);
+#pragma unroll
+          for (int dj = 0; dj < 4; ++dj) {
+            const int col = dj * 16 + 4 * (r & 3);
+            const bf16x4 a = ds_read_tr(vs + r0 * VLD + col);
+            const bf16x4 d = ds_read_tr(vs + (r0 + 16) * VLD + col);
+            const bf16x8 vf = {a[0], a[1], a[2], a[3], d[0], d[1], d[2], d[3]};
+            o[c][vh * 4 + dj] = mfma16(vf, hf, o[c][vh * 4 + dj]);
+            o[c][vh * 4 + dj] = mfma16(vf, lf, o[c][vh * 4 + dj]);
+          }
+        }
+      }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float t = lsum[mt][i];
+      t += wave_xchg<1>(t);
+      t += wave_xchg<2>(t);
+      t += wave_xchg<4>(t);
+      t += wave_xchg<8>(t);
+      if (r == 0) ls[w][mt * 16 + 4 * g + i] = t;
+    }
+  __syncthreads();
+#pragma unroll
+  for (int c = 0; c < GMAX; ++c) {
+    const int kvh = w + 4 * c;
+    if (kvh >= G || r >= rep) continue;
+    const int h = kvh * rep + r;
+    const float l = ls[0][h] + ls[1][h] + ls[2][h] + ls[3][h];
+    if (p.splits > 1) {
+      const long pi = ((long)b * H + h) * p.splits + blockIdx.y;
+#pragma unroll
+      for (int di = 0; di < VT; ++di)
+        if (di * 16 < vdim) *reinterpret_cast<f32x4*>(p.part_o + pi * vdim + di * 16 + 4 * g) = o[c][di];
+      if (g == 0) {
+        p.part_ml[2 * pi] = ms[h];
+        p.part_ml[2 * pi + 1] = l;
+      }
+    } else {
+      const float inv = 1.f / l;
+      bf16* out = static_cast<bf16*>(p.out) + (long)b * p.ldo + h * vdim;
+#pragma unroll
+      for (int di = 0; di < VT; ++di)
+        if (di * 16 < vdim)
+          st4(out + di * 16 + 4 * g, bf16x4{f2bf(o[c][di][0] * inv), f2bf(o[c][di][1] * inv), f2bf(o[c][di][2] * inv),
+                                            f2bf(o[c][di][3] * inv)});
+    }
+  }
+  if (p.splits == 1)
+    for (int c = H * vdim + threadIdx.x; c < p.out_cols; c += 256) static_cast<bf16*>(p.out)[(long)b * p.ldo + c] = f2bf(0.f);
+}
+
+// One block per (token, head); the last head's also clears the pad columns.
+__global__ __launch_bounds__(64) void talk_combine_kernel(TalkParams p) {
+  const int b = blockIdx.x / p.H, h = blockIdx.x % p.H;
+  const long pi = (long)blockIdx.x * p.splits;
+  float M = NEG, L = 0.f;
+  for (int s = 0; s < p.splits; ++s) M = fmaxf(M, p.part_ml[2 * (pi + s)]);
+  for (int s = 0; s < p.splits; ++s) L += p.part_ml[2 * (pi + s) + 1] * exp2f(p.part_ml[2 * (pi + s)] - M);
+  const float inv = 1.f / L;
+  bf16* out = static_cast<bf16*>(p.out) + (long)b * p.ldo;
+  for (int d = threadIdx.x; d < p.vdim; d += 64) {
+    float v = 0.f;
+    for (int s = 0; s < p.splits; ++s) v += p.part_o[(pi + s) * p.vdim + d] * exp2f(p.part_ml[2 * (pi + s)] - M);
+    out[h * p.vdim + d] = f2bf(v * inv);
+  }
+  if (h == p.H - 1)
+    for (int c = p.H * p.vdim + threadIdx.x; c < p.out_cols; c += 64) out[c] = f2bf(0.f);
+}
+
 }  // namespace
 }  // namespace lsd
 
 using namespace lsd;
+
+// Head padding of the MFMA kernels, 0: sizes they do not take.
+extern "C" int lsd_talk_heads(int H, int G, int dim, int vdim, float cap) {
+  if (H > 32 || H / G > 16 || dim % 32 || dim > 128 || vdim % 16 || vdim > 128 || !(cap > 0.f) || cap > 3e4f) return 0;
+  return H <= 8 ? 8 : H <= 16 ? 16 : 32;
+}
+
+extern "C" int lsd_talk_tile(int hp) { return 16 * (32 / hp); }  // queries of a prefill tile
+
+#define LSD_TK_V(KERNEL, HP, GRID, NT)                                                                   \
+  if (p->dim <= 64 && p->vdim <= 64) hipLaunchKernelGGL((KERNEL<2, 4, HP>), GRID, dim3(NT), 0, st, *p); \
+  else if (p->dim <= 64) hipLaunchKernelGGL((KERNEL<2, 8, HP>), GRID, dim3(NT), 0, st, *p);              \
+  else if (p->vdim <= 64) hipLaunchKernelGGL((KERNEL<4, 4, HP>), GRID, dim3(NT), 0, st, *p);             \
+  else hipLaunchKernelGGL((KERNEL<4, 8, HP>), GRID, dim3(NT), 0, st, *p);
+
+extern "C" hipError_t lsd_talk_prefill(const TalkParams* p, int hp, hipStream_t st) {
+  if (p->n_tiles == 0) return hipSuccess;
+  const dim3 grid(p->n_tiles);
+  switch (hp) {
+    case 8: LSD_TK_V(talk_prefill_kernel, 8, grid, 512) break;
+    case 16: LSD_TK_V(talk_prefill_kernel, 16, grid, 512) break;
+    case 32: LSD_TK_V(talk_prefill_kernel, 32, grid, 512) break;
+    default: return hipErrorInvalidValue;
+  }
+  return hipGetLastError();
+}
+
+// hp: 16 or 32 (talk_frag padded to it); needs G <= hp
+extern "C" hipError_t lsd_talk_decode(const TalkParams* p, int hp, hipStream_t st) {
+  if (p->T == 0) return hipSuccess;
+  const dim3 grid(p->T, p->splits);
+  switch (hp) {
+    case 16: LSD_TK_V(talk_decode_kernel, 16, grid, 256) break;
+    case 32: LSD_TK_V(talk_decode_kernel, 32, grid, 256) break;
+    default: return hipErrorInvalidValue;
+  }
+  if (p->splits > 1) hipLaunchKernelGGL(talk_combine_kernel, dim3(p->T * p->H), dim3(64), 0, st, *p);
+  return hipGetLastError();
+}
+#undef LSD_TK_V
 
 extern "C" hipError_t lsd_rope_append(const RopeAppendParams* p, int f32, hipStream_t st) {
   if (p->T == 0) return hipSuccess;

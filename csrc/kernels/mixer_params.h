@@ -68,7 +68,7 @@ struct TalkParams {
   const void* k; const void* v;        // pools
   const int* table; int tw;            // [slots][pages of a sequence]
   const float* talk;                   // [H][H] or null
-  const void* talk_frag;               // MFMA kernels: bf16 [HP][HP], zero padded (HP: H to 16 / 32 / 64)
+  const void* talk_frag;               // MFMA kernels: fp16 [HP][HP], zero padded (HP: H to 8 / 16 / 32)
   void* out; long ldo; int out_cols;   // [rows][H][vdim], zeros up to out_cols
   int H, G, dim, vdim, window;         // window: keys per query (INT_MAX: all)
   float scale, cap;                    // cap 0: none

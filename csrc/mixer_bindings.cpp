@@ -31,6 +31,10 @@ hipError_t lsd_gelu_mul_f32(const float* y, float* out, int T, int F, long ldo, 
 hipError_t lsd_rope_append(const RopeAppendParams* p, int f32, hipStream_t st);
 long lsd_talk_plain_lds(const TalkParams* p);
 hipError_t lsd_talk_plain(const TalkParams* p, int f32, hipStream_t st);
+int lsd_talk_heads(int H, int G, int dim, int vdim, float cap);
+int lsd_talk_tile(int hp);
+hipError_t lsd_talk_prefill(const TalkParams* p, int hp, hipStream_t st);
+hipError_t lsd_talk_decode(const TalkParams* p, int hp, hipStream_t st);
 }
 
 namespace {
@@ -249,6 +253,7 @@ TalkParams talk_base(const Tensor& q, const Tensor& k, const Tensor& v, const Te
   p.G = k.size(1); p.dim = k.size(3); p.vdim = v.size(3); p.H = q.size(1) / p.dim;
   TORCH_CHECK(q.dim() == 2 && q.is_contiguous() && q.size(1) == (int64_t)p.H * p.dim && p.H % p.G == 0,
               "q must be contiguous [T, heads dim]");
+  TORCH_CHECK(q.numel() < (1L << 31), "q: at most 2^31 elements");
   TORCH_CHECK(window >= 1, "window must be positive");
   p.T = q.size(0);
   p.q = q.data_ptr(); p.k = k.data_ptr(); p.v = v.data_ptr();
@@ -271,6 +276,47 @@ void talk_plain(Tensor q, Tensor k, Tensor v, Tensor table, Tensor slots, Tensor
   check_hip(lsd_talk_plain(&p, is_f32(q, "q"), cur_stream()), "talk_plain");
 }
 
+int frag_of(TalkParams& p, const Tensor& q, const Tensor& frag) {
+  TORCH_CHECK(q.scalar_type() == torch::kBFloat16, "the MFMA kernels are bf16");
+  TORCH_CHECK(frag.is_cuda() && frag.scalar_type() == torch::kFloat16 && frag.is_contiguous() && frag.dim() == 2 &&
+                  frag.size(0) == frag.size(1), "talk must be a contiguous fp16 [HP, HP]");
+  p.talk_frag = frag.data_ptr();
+  const int hp = frag.size(0), need = lsd_talk_heads(p.H, p.G, p.dim, p.vdim, p.cap);
+  TORCH_CHECK(need > 0 && hp >= need && (hp == 8 || hp == 16 || hp == 32), "no MFMA kernel for ", p.H, " heads of ", p.dim,
+              " / ", p.vdim, " with talk padded to ", hp);
+  return hp;
+}
+
+// packed ragged queries; tiles [n, 2] = (sequence, first query) of talk_tile(hp) queries
+void talk_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tensor tiles, Tensor slots, Tensor start,
+                  Tensor cu, int64_t window, double scale, double cap, Tensor out) {
+  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, cap, out);
+  const int hp = frag_of(p, q, frag);
+  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2, "tiles must be [n, 2]");
+  p.tiles = iptr(tiles, 0, "tiles"); p.n_tiles = tiles.size(0);
+  p.s = seqs(slots, start, cu);
+  check_hip(lsd_talk_prefill(&p, hp, cur_stream()), "talk_prefill");
+}
+
+// one query per row; slots / pos [T]; hp (talk's padding) 16 or 32, G <= hp / 4
+void talk_decode(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tensor slots, Tensor pos, int64_t window,
+                 double scale, double cap, int64_t splits, Tensor out) {
+  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, cap, out);
+  const int hp = frag_of(p, q, frag);
+  TORCH_CHECK(hp >= 16 && 4 * p.G <= hp, "talk_decode: ", p.G, " K / V heads need talk padded to ", 4 * p.G);
+  p.slots = iptr(slots, p.T, "slots"); p.pos = iptr(pos, p.T, "pos");
+  TORCH_CHECK(splits >= 1 && splits <= 256, "splits");
+  p.splits = splits;
+  Tensor po, pml;
+  if (splits > 1) {
+    const int64_t n = (int64_t)p.T * p.H * splits;
+    po = torch::empty({n * p.vdim}, q.options().dtype(torch::kFloat32));
+    pml = torch::empty({n * 2}, q.options().dtype(torch::kFloat32));
+    p.part_o = po.data_ptr<float>(); p.part_ml = pml.data_ptr<float>();
+  }
+  check_hip(lsd_talk_decode(&p, hp, cur_stream()), "talk_decode");
+}
+
 }  // namespace
 
 void lsd_register_mixers(pybind11::module& m) {
@@ -286,6 +332,15 @@ void lsd_register_mixers(pybind11::module& m) {
   m.def("gelu_mul_f32", &gelu_mul_f32, py::arg("y"), py::arg("out"), py::arg("scale"));
   m.def("rope_append", &rope_append, py::arg("y"), py::arg("heads"), py::arg("k"), py::arg("v"), py::arg("table"),
         py::arg("tslot"), py::arg("tpos"), py::arg("rope"), py::arg("gain"));
+  m.def("talk_heads", [](int64_t H, int64_t G, int64_t dim, int64_t vdim, double cap) {
+    return lsd_talk_heads(H, G, dim, vdim, (float)cap); });
+  m.def("talk_tile", [](int64_t hp) { return lsd_talk_tile((int)hp); });
+  m.def("talk_prefill", &talk_prefill, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("frag"),
+        py::arg("tiles"), py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("window"), py::arg("scale"),
+        py::arg("cap"), py::arg("out"));
+  m.def("talk_decode", &talk_decode, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("frag"),
+        py::arg("slots"), py::arg("pos"), py::arg("window"), py::arg("scale"), py::arg("cap"), py::arg("splits"),
+        py::arg("out"));
   m.def("talk_plain", &talk_plain, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("slots"),
         py::arg("pos"), py::arg("talk"), py::arg("window"), py::arg("scale"), py::arg("cap"), py::arg("out"));
 }

@@ -112,9 +112,9 @@ class StageModel:
         return self.unit_start <= 2 * lh[0] + lh[1] < self.unit_end
 
     # ------------------------------------------------------------------
-    def _lw(self, i: int, name: str) -> torch.Tensor:
+    def _lw(self, i: int, name: str, *default) -> torch.Tensor:
         p = "h." if self.cfg.arch == "gpt2" else "layers."
-        return self.w[f"{p}{i}.{name}"]
+        return self.w.get(f"{p}{i}.{name}", *default) if default else self.w[f"{p}{i}.{name}"]
 
     # [tf5.15] modeling_gpt2.py:262-309 GPT2Block.forward, split at the residual
     def _gpt2_attn(self, li: int, i: int, r: Residual, meta: BatchMeta) -> None:

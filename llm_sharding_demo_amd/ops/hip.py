@@ -335,8 +335,15 @@ class HipBackend(Backend):
                 rows = [pad_to(t(f"mixer.{n}").reshape(h, d, -1), h, dd, hp).reshape(h * dd, hp) for n, h, d, dd in (
                     ("q", m.heads, m.dim, dp), ("k", m.kv_heads, m.dim, dp), ("v", m.kv_heads, m.vdim, vp))]
                 o = pad_to(o.reshape(-1, m.heads, m.vdim), o.shape[0], m.heads, vp).reshape(-1, m.heads * vp)
+                talk = w[p + "mixer.talk"] if m.talking else torch.eye(m.heads, dtype=stage.dtype, device=dev)
                 if m.talking:
                     f32("mixer.talk")
+                hq = 0 if self.fp32 else self.C.talk_heads(m.heads, m.kv_heads, dp, vp, m.softcap or 0.0)
+                if hq and float(talk.abs().max()) < 6e4:  # the mixing matrix in fp16, padded for each kernel
+                    w[p + "mixer.talk_prefill"] = pad_to(talk, hq, hq).half()
+                    hd = max(16, hq, 32 if m.kv_heads > 4 else 0)
+                    if 4 * m.kv_heads <= hd:
+                        w[p + "mixer.talk_decode"] = pad_to(talk, hd, hd).half()
                 if m.rope is not None and m.rope.dims and m.rope not in self._ropes:
                     self._ropes[m.rope] = rope_spec_table(m.rope, _up(stage.max_seq, 64), dev)
             elif isinstance(m, ChannelDeltaSpec):
@@ -413,9 +420,28 @@ class HipBackend(Backend):
         k, v = entry
         rope = self._ropes[m.rope] if m.rope is not None and m.rope.dims else None
         q = self.C.rope_append(y, m.heads, k, v, kv.table, meta.token_slots, meta.token_pos, rope, gain)
+        window, cap = m.window or 1 << 30, m.softcap or 0.0
         for s, mt in self._parts(meta):
-            self.C.talk_plain(q[s], k, v, kv.table, mt.token_slots, mt.token_pos, w("mixer.talk") if m.talking else None,
-                              m.window or 1 << 30, m.scale, m.softcap or 0.0, out[s])
+            tp, td = w("mixer.talk_prefill", None), w("mixer.talk_decode", None)
+            if tp is None:
+                self.C.talk_plain(q[s], k, v, kv.table, mt.token_slots, mt.token_pos,
+                                  w("mixer.talk") if m.talking else None, window, m.scale, cap, out[s])
+            elif mt.is_decode and td is not None:
+                splits = self.R.talk_splits(mt.num_seqs, min(window, mt.max_ctx))
+                self.C.talk_decode(q[s], k, v, kv.table, td, mt.token_slots, mt.token_pos, window, m.scale, cap, splits,
+                                   out[s])
+            else:
+                tiles = self._query_tiles(mt, self.C.talk_tile(tp.shape[0]), q.device)
+                self.C.talk_prefill(q[s], k, v, kv.table, tp, tiles, mt.seq_slots, mt.q_start, mt.cu_q, window, m.scale,
+                                    cap, out[s])
+
+    @staticmethod
+    def _query_tiles(meta, rows: int, device):
+        """(sequence, first query) of every `rows`-query tile, kept on the batch."""
+        cache = meta.__dict__.setdefault("_query_tiles", {})
+        if rows not in cache:
+            cache[rows] = latent_tiles(meta, 1, rows).to(device)
+        return cache[rows]
 
     def _channel_delta(self, y, w, m, gain, kv, entry, meta, eps, out):
         low = self._batch_linear(y, w("mixer.low.weight"))
@@ -515,6 +541,8 @@ class HipBackend(Backend):
 
     def prepare_prefill(self, meta, mcfg) -> None:
         if mcfg.arch == "vizalix":
+            for hp in (8, 16, 32):
+                self._query_tiles(meta, self.C.talk_tile(hp), meta.cu_q.device)
             return
         if mcfg.arch != "timisun":
             meta._tiles = prefill_tiles(meta).to(meta.cu_q.device)

@@ -124,6 +124,9 @@ class Routing:
     # prompts of at least latent_expand_t tokens attend over expanded keys and
     # values where that saves multiply-adds (latent_expand; 0 disables)
     latent_expand_t: int = 256
+    # decode attention with mixed heads: blocks a launch aims for, at least two
+    # 64-key tiles each
+    talk_target: int = 512
     # -- norms / head ------------------------------------------------------
     # one wave per row from norm_wave_min rows (prefill 32 K x 1600 97.7 ->
     # 53.7 us; r5_normwave.log) and from norm_wave_narrow_min rows when H <=
@@ -289,6 +292,11 @@ class Routing:
     def latent_splits(self, B: int, heads: int, keys: int) -> int:
         items = B * math.ceil(heads / 16)
         return max(1, min(math.ceil(self.latent_target / items), math.ceil((keys + 31) / 128), 64))
+
+    def talk_splits(self, B: int, keys: int) -> int:
+        """Context splits of a decode attention launch with mixed heads (one
+        block holds all heads of a token, 64 keys a step)."""
+        return max(1, min(math.ceil(self.talk_target / B), math.ceil((keys + 63) / 128), 64))
 
     def attn_splits(self, B: int, nh: int, n_kv: int, hd: int, max_ctx: int) -> int:
         """Context splits of a decode attention launch (a graph-captured
