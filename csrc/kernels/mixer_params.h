@@ -57,10 +57,6 @@ struct MixOutParams {
   void* out; long ldo; int out_cols;
 };
 
-// Chunked prompt forms (bf16 models), chunks of RC_CHUNK tokens.  Chunk x of
-// the launch: sequence tiles[2 x], first token tiles[2 x + 1] within it.
-constexpr int RC_CHUNK = 64;
-
 // Attention over a paged cache, K [page][kv head][64][dim], V likewise with
 // vdim; scores capped, mixed over the heads, softmaxed.
 struct TalkParams {

@@ -5,6 +5,12 @@
 //    convolution, SiLU, unit norms, decay, state update and read-out, and for
 //    the delta rule the output norm and gate.  Decode steps, and prompts of
 //    models served in fp32.
+//  * conv_silu, delta_chunk, ssd_chunk: prompts of bf16 models.  Chunks of 16
+//    (delta rule) or 32 tokens (Mamba-2) become matrix products around a state
+//    that stays in the accumulators of four waves, each owning columns of it; the
+//    accumulator layout of one product is the operand layout of the next, so
+//    state, pseudo-values and outputs never leave their wave.  fp32 operands
+//    enter the matrix cores as two bf16 terms (three products, 16 bits each).
 //  * conv_tail: keeps the convolution's last inputs after a prompt portion.
 //  * head_norm_gate / gated_group_norm: output norms of the unfused forms.
 //
@@ -190,6 +196,553 @@ __global__ __launch_bounds__(256) void recur_seq_kernel(RecurParams p) {
   }
 }
 
+// Rows of SiLU(convolution), bf16.  One block per row and 256 * VEC channels.
+template <int VEC>
+__global__ __launch_bounds__(256) void conv_silu_kernel(ConvParams c, SeqParams s, bf16* __restrict__ out, long ldo) {
+  const int row = blockIdx.x;
+  int a = 0, b = s.B;  // sequence: last one with cu <= row
+  while (b - a > 1) {
+    const int m = (a + b) >> 1;
+    if (s.cu[m] <= row) a = m;
+    else b = m;
+  }
+  const int t = row - s.cu[a], pos = s.start[a] + t, slot = s.slots[a];
+  const int ch = (blockIdx.y * 256 + threadIdx.x) * VEC;
+  if (ch >= c.channels) return;
+  if constexpr (VEC == 1) {
+    out[row * ldo + ch] = f2bf(silu_x(conv_at<bf16>(c, ch, row, t, pos, slot)));
+  } else {
+    const bf16* y = static_cast<const bf16*>(c.y) + c.c0 + ch;
+    const bf16* ring = static_cast<const bf16*>(c.ring) + (long)slot * c.taps * c.channels + ch;
+    float acc[8] = {};
+    for (int j = 0; j < c.taps; ++j) {
+      const int back = c.taps - 1 - j;
+      if (back > pos) continue;
+      const bf16x8 x = ld8(back <= t ? y + (row - back) * c.ldy : ring + (long)((pos - back) % c.taps) * c.channels);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[e] = fmaf(c.w[(long)(ch + e) * c.taps + j], bf2f(x[e]), acc[e]);
+    }
+    bf16x8 o;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float v = acc[e] * c.gain + (c.bias ? c.bias[ch + e] : 0.f);
+      o[e] = f2bf(silu(v));
+    }
+    st8(out + row * ldo + ch, o);
+  }
+}
+
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+
+// A[row r][k = 4 g + j] . B[k = 4 g + j][col r]
+__device__ __forceinline__ f32x4 mfma16k16(bf16x4 a, bf16x4 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(s16x4, a), __builtin_bit_cast(s16x4, b), c, 0, 0, 0);
+}
+
+__device__ __forceinline__ bf16x4 ds_read_tr(const bf16* lds_ptr) {
+  typedef __attribute__((address_space(3))) bf16x4 lds_bf16x4;
+  return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds_bf16x4*)(lds_ptr));
+}
+
+__device__ __forceinline__ void lds_fence() {
+  __builtin_amdgcn_s_waitcnt(0xC07F);  // lgkmcnt(0)
+  __builtin_amdgcn_wave_barrier();
+}
+
+__device__ __forceinline__ bf16x4 hi4(f32x4 v) { return bf16x4{f2bf(v[0]), f2bf(v[1]), f2bf(v[2]), f2bf(v[3])}; }
+__device__ __forceinline__ bf16x4 lo4(f32x4 v, bf16x4 h) {
+  return bf16x4{f2bf(v[0] - bf2f(h[0])), f2bf(v[1] - bf2f(h[1])), f2bf(v[2] - bf2f(h[2])), f2bf(v[3] - bf2f(h[3]))};
+}
+__device__ __forceinline__ bf16x8 cat(bf16x4 a, bf16x4 b) { return bf16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]}; }
+// two bf16 terms of eight values (two accumulator tiles: k-slots 4 g + j and 16 + 4 g + j)
+__device__ __forceinline__ void split8(f32x4 a, f32x4 b, bf16x8& hi, bf16x8& lo) {
+  const bf16x4 ha = hi4(a), hb = hi4(b);
+  hi = cat(ha, hb);
+  lo = cat(lo4(a, ha), lo4(b, hb));
+}
+// a (two terms) . b (two terms)
+__device__ __forceinline__ f32x4 mfma3(bf16x8 ah, bf16x8 al, bf16x8 bh, bf16x8 bl, f32x4 c) {
+  c = mfma16(ah, bh, c);
+  c = mfma16(ah, bl, c);
+  return mfma16(al, bh, c);
+}
+__device__ __forceinline__ f32x4 mfma3s(bf16x4 ah, bf16x4 al, bf16x4 bh, bf16x4 bl, f32x4 c) {
+  c = mfma16k16(ah, bh, c);
+  c = mfma16k16(ah, bl, c);
+  return mfma16k16(al, bh, c);
+}
+
+// Chunked delta rule.  With G_t the summed log decays of the chunk up to token t
+// (per key channel), S0 = diag(e^{G_0}) S and everything relative to G_0:
+//   X = V - K~ S0          K~_t = k_t e^{G_t - G_0}
+//   U = (I + A)^-1 diag(beta) X,   A_ts = beta_t sum_d K~_td k_sd e^{G_0 - G_s}  (s < t)
+//   O = Q~ S0 + P U        P_ts = sum_d Q~_td k_sd e^{G_0 - G_s}                 (s <= t)
+//   S = diag(e^{G_15 - G_0}) S0 + K^T U,   K^_s = k_s e^{G_15 - G_s}
+// Every factor is at most e^80 in size; channels that decay by more than that
+// within a chunk are left out of the two products over d and added term by term
+// (e^{G_t - G_s} <= 1 always).  One block per (sequence, head).
+template <int DKS, int VTW>
+__global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, const bf16* __restrict__ x, long ldx) {
+  constexpr int CT = 16, DP = DKS * 32, DT = DKS * 2, LDD = DP + 8, LDT = CT + 4;
+  constexpr float RANGE = 80.f;
+  __shared__ __attribute__((aligned(16))) bf16 kt_h[CT * LDD], kt_l[CT * LDD], qt_h[CT * LDD], qt_l[CT * LDD];
+  __shared__ __attribute__((aligned(16))) bf16 kc_h[CT * LDD], kc_l[CT * LDD];     // columns k_s e^{G_0 - G_s}
+  __shared__ __attribute__((aligned(16))) bf16 kh_h[DP * LDT], kh_l[DP * LDT];     // K^ transposed [d][s]
+  __shared__ __attribute__((aligned(16))) float Gs[CT][DP], Ks[CT][DP], Qs[CT][DP];
+  __shared__ __attribute__((aligned(16))) float e0[DP], er[DP];
+  __shared__ __attribute__((aligned(16))) bf16 tm_h[CT * LDT], tm_l[CT * LDT], pm_h[CT * LDT], pm_l[CT * LDT];
+  __shared__ float betas[CT], red[4][CT];
+  __shared__ int bad[DP], nbad;
+  const int h = blockIdx.x, b = blockIdx.y, D = p.D, V = p.V;
+  const int tid = threadIdx.x, lane = lane_id(), w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int kh = h / (p.heads / p.groups);
+  const int slot = p.s.slots[b], start = p.s.start[b], r0 = p.s.cu[b], n = p.s.cu[b + 1] - r0;
+  if (n <= 0) return;
+  float* Sg = p.S + ((long)slot * p.heads + h) * D * p.Vp;
+  const float A = p.A[h], gain = p.c.gain;
+  const bf16* y = static_cast<const bf16*>(p.c.y);
+  const bf16* low = static_cast<const bf16*>(p.low);
+
+  // state: rows d = 16 dt + 4 g + i, columns v = 16 (w VTW + j) + r
+  f32x4 S[DT][VTW];
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+    for (int j = 0; j < VTW; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
+        S[dt][j][i] = start > 0 && d < D && v < V ? Sg[(long)d * p.Vp + v] : 0.f;
+      }
+  // element work: token tid / 16, channels 8 (tid % 16) ..
+  const int et = tid >> 4, ed = (tid & 15) * 8;
+  const bool elive = ed < D;  // D % 8 == 0
+  float dtb[8] = {};
+  if (elive)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) dtb[e] = p.dt_bias[(long)h * D + ed + e];
+
+  for (int t0 = 0; t0 < n; t0 += CT) {
+    const int nt = min(CT, n - t0);
+    const long row = r0 + t0 + min(et, nt - 1);
+    const bool tlive = et < nt && elive;
+    float q8[8], k8[8], lg[8];
+    {
+      const bf16x8 z = {};
+      const bf16x8 xq = tlive ? ld8(x + row * ldx + p.q_ch + kh * D + ed) : z;
+      const bf16x8 xk = tlive ? ld8(x + row * ldx + p.k_ch + kh * D + ed) : z;
+      const bf16x8 xl = tlive ? ld8(low + row * p.ldl + (long)h * D + ed) : z;
+      float nq = 0.f, nk = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        q8[e] = bf2f(xq[e]);
+        k8[e] = bf2f(xk[e]);
+        nq = fmaf(q8[e], q8[e], nq);
+        nk = fmaf(k8[e], k8[e], nk);
+        lg[e] = tlive ? A * softplus_x(gain * bf2f(xl[e]) + dtb[e]) : 0.f;
+      }
+#pragma unroll
+      for (int off = 1; off < 16; off <<= 1) {
+        nq += wave_xchg_n(nq, off);
+        nk += wave_xchg_n(nk, off);
+      }
+      const float iq = rsqrtf((float)D) / sqrtf(nq + UNIT_EPS), ik = 1.f / sqrtf(nk + UNIT_EPS);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        q8[e] *= iq;
+        k8[e] *= ik;
+      }
+    }
+    if (ed < DP) {
+      *reinterpret_cast<f32x4*>(&Gs[et][ed]) = f32x4{lg[0], lg[1], lg[2], lg[3]};
+      *reinterpret_cast<f32x4*>(&Gs[et][ed + 4]) = f32x4{lg[4], lg[5], lg[6], lg[7]};
+    }
+    if (tid < CT)
+      betas[tid] = tid < nt ? sigmoid_x(gain * bf2f(y[(r0 + t0 + tid) * p.c.ldy + p.gate_col + h])) : 0.f;
+    if (tid == 0) nbad = 0;
+    __syncthreads();
+    f32x4 g0[2] = {}, gt[2] = {}, gc[2] = {};
+    if (ed < DP) {
+      g0[0] = *reinterpret_cast<const f32x4*>(&Gs[0][ed]);
+      g0[1] = *reinterpret_cast<const f32x4*>(&Gs[0][ed + 4]);
+#pragma unroll 4
+      for (int s = 0; s < CT; ++s)
+#pragma unroll
+        for (int q = 0; q < 2; ++q) {
+          const f32x4 v = *reinterpret_cast<const f32x4*>(&Gs[s][ed + 4 * q]);
+          gc[q] += v;
+          if (s == et) gt[q] = gc[q];
+        }
+    }
+    __syncthreads();  // the log decays have been read: Gs takes their sums
+    if (ed < DP) {
+      float kt[8], qt[8], kc[8], kf[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float G0 = g0[e >> 2][e & 3], Gt = gt[e >> 2][e & 3], Gc = gc[e >> 2][e & 3];
+        const float E = expf(Gt - G0);
+        const bool wide = G0 - Gc > RANGE;
+        kt[e] = k8[e] * E;
+        qt[e] = q8[e] * E;
+        kc[e] = wide ? 0.f : k8[e] * expf(G0 - Gt);
+        kf[e] = k8[e] * expf(Gc - Gt);
+        if (et == 0) {
+          e0[ed + e] = expf(G0);
+          er[ed + e] = expf(Gc - G0);
+          if (wide) bad[atomicAdd(&nbad, 1)] = ed + e;
+        }
+        Gs[et][ed + e] = Gt;
+        Ks[et][ed + e] = k8[e];
+        Qs[et][ed + e] = q8[e];
+      }
+      auto put = [&](bf16* hp, bf16* lp, const float* v) {
+        bf16x8 a, c;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          a[e] = f2bf(v[e]);
+          c[e] = f2bf(v[e] - bf2f(a[e]));
+        }
+        st8(hp + et * LDD + ed, a);
+        st8(lp + et * LDD + ed, c);
+      };
+      put(kt_h, kt_l, kt);
+      put(qt_h, qt_l, qt);
+      put(kc_h, kc_l, kc);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const bf16 a = f2bf(kf[e]);
+        kh_h[(ed + e) * LDT + et] = a;
+        kh_l[(ed + e) * LDT + et] = f2bf(kf[e] - bf2f(a));
+      }
+    }
+    // values of the chunk in the accumulator layout (tokens 4 g + i, columns r)
+    f32x4 vals[VTW];
+#pragma unroll
+    for (int j = 0; j < VTW; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 4 * g + i, v = (w * VTW + j) * 16 + r;
+        vals[j][i] = t < nt && v < V ? bf2f(x[(r0 + t0 + t) * ldx + p.v_ch + (long)h * V + v]) : 0.f;
+      }
+    __syncthreads();
+    // operand of row r: k-slots (g, j) <-> d = 32 ks + 4 g + j, 32 ks + 16 + 4 g + (j - 4)
+    auto opnd = [&](const bf16* a, int ks) {
+      return cat(ld4(a + r * LDD + ks * 32 + 4 * g), ld4(a + r * LDD + ks * 32 + 16 + 4 * g));
+    };
+    if (w < 2) {  // wave 0: A and (I + A)^-1, wave 1: P
+      const bf16 *ah = w == 0 ? kt_h : qt_h, *al = w == 0 ? kt_l : qt_l;
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks) {
+        asm volatile("" ::: "memory");  // operands of one step at a time
+        acc = mfma3(opnd(ah, ks), opnd(al, ks), opnd(kc_h, ks), opnd(kc_l, ks), acc);
+      }
+      const int nb = nbad;
+      for (int q = 0; q < nb; ++q) {
+        const int d = bad[q];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int t = 4 * g + i;
+          if (r <= t) acc[i] += (w == 0 ? Ks[t][d] : Qs[t][d]) * Ks[r][d] * expf(Gs[t][d] - Gs[r][d]);
+        }
+      }
+      if (w == 1) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int t = 4 * g + i;
+          const float v = r <= t ? acc[i] : 0.f;
+          const bf16 a = f2bf(v);
+          pm_h[t * LDT + r] = a;
+          pm_l[t * LDT + r] = f2bf(v - bf2f(a));
+        }
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[i] = r < 4 * g + i ? acc[i] * betas[4 * g + i] : 0.f;
+        // column r of the inverse by forward substitution (each lane group alike);
+        // A_ts is register t % 4 of lane 16 (t / 4) + s
+        float inv[CT];
+#pragma unroll
+        for (int t = 0; t < CT; ++t) {
+          float v = t == r ? 1.f : 0.f;
+#pragma unroll
+          for (int s = 0; s < t; ++s) {
+            // (a bit cast of a vector's element would take element 0)
+            const int a = __builtin_amdgcn_readlane(__float_as_int(acc[t & 3]), 16 * (t >> 2) + s);
+            v = fmaf(-__int_as_float(a), inv[s], v);
+          }
+          inv[t] = v;
+        }
+        const float bt = betas[r];
+        if (g == 0) {
+#pragma unroll
+          for (int t = 0; t < CT; ++t) {
+            const float v = inv[t] * bt;
+            const bf16 a = f2bf(v);
+            tm_h[t * LDT + r] = a;
+            tm_l[t * LDT + r] = f2bf(v - bf2f(a));
+          }
+        }
+      }
+    }
+    f32x4 ks_acc[VTW], o[VTW];
+#pragma unroll
+    for (int j = 0; j < VTW; ++j) ks_acc[j] = o[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < DKS; ++ks) {
+      const f32x4 da = *reinterpret_cast<const f32x4*>(&e0[ks * 32 + 4 * g]);
+      const f32x4 db = *reinterpret_cast<const f32x4*>(&e0[ks * 32 + 16 + 4 * g]);
+      const bf16x8 kah = opnd(kt_h, ks), kal = opnd(kt_l, ks), qah = opnd(qt_h, ks), qal = opnd(qt_l, ks);
+#pragma unroll
+      for (int j = 0; j < VTW; ++j) {
+        S[2 * ks][j] *= da;
+        S[2 * ks + 1][j] *= db;
+        bf16x8 sh, sl;
+        split8(S[2 * ks][j], S[2 * ks + 1][j], sh, sl);
+        ks_acc[j] = mfma3(kah, kal, sh, sl, ks_acc[j]);
+        o[j] = mfma3(qah, qal, sh, sl, o[j]);
+      }
+    }
+    __syncthreads();
+    const bf16x4 th = ld4(tm_h + r * LDT + 4 * g), tl = ld4(tm_l + r * LDT + 4 * g);
+    const bf16x4 ph = ld4(pm_h + r * LDT + 4 * g), pl = ld4(pm_l + r * LDT + 4 * g);
+    bf16x4 uh[VTW], ul[VTW];
+    f32x4 ss = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < VTW; ++j) {
+      const f32x4 xv = vals[j] - ks_acc[j];
+      const bf16x4 xh = hi4(xv), xl = lo4(xv, xh);
+      f32x4 u = {0.f, 0.f, 0.f, 0.f};
+      u = mfma3s(th, tl, xh, xl, u);
+      uh[j] = hi4(u);
+      ul[j] = lo4(u, uh[j]);
+      o[j] = mfma3s(ph, pl, uh[j], ul[j], o[j]);
+      ss += o[j] * o[j];  // columns beyond V are zero
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float v = ss[i];
+#pragma unroll
+      for (int off = 1; off < 16; off <<= 1) v += wave_xchg_n(v, off);
+      if (r == 0) red[w][4 * g + i] = v;
+    }
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      const f32x4 dec = *reinterpret_cast<const f32x4*>(&er[dt * 16 + 4 * g]);
+      const bf16x4 ah = ld4(kh_h + (dt * 16 + r) * LDT + 4 * g), al = ld4(kh_l + (dt * 16 + r) * LDT + 4 * g);
+#pragma unroll
+      for (int j = 0; j < VTW; ++j) S[dt][j] = mfma3s(ah, al, uh[j], ul[j], S[dt][j] * dec);
+    }
+    __syncthreads();
+    bf16* out = static_cast<bf16*>(p.out);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = 4 * g + i;
+      if (t >= nt) continue;
+      const long orow = r0 + t0 + t;
+      const float rs = rsqrtf((red[0][t] + red[1][t] + red[2][t] + red[3][t]) / V + p.eps);
+#pragma unroll
+      for (int j = 0; j < VTW; ++j) {
+        const int v = (w * VTW + j) * 16 + r;
+        if (v >= V) continue;
+        const float gate = gain * bf2f(low[orow * p.ldl + p.gate_off + (long)h * V + v]);
+        out[orow * p.ldo + (long)h * V + v] =
+            f2bf(o[j][i] * rs * p.norm[v] * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * gate)));
+      }
+    }
+    if (h == p.heads - 1)
+      for (int c = p.heads * V + (tid & 15); c < p.out_cols; c += 16)
+        if (et < nt) out[row * p.ldo + c] = f2bf(0.f);
+  }
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+    for (int j = 0; j < VTW; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
+        if (d < D && v < p.Vp) Sg[(long)d * p.Vp + v] = S[dt][j][i];
+      }
+}
+
+// Chunked Mamba-2 over x [rows][x | B | C] behind convolution and SiLU (bf16).
+// With a_t the summed log decays of the chunk up to token t:
+//   y = diag(e^{a}) C S + P x + D x,   P_ts = (C_t . B_s) e^{a_t - a_s} dt_s  (s <= t)
+//   S = e^{a_31} S + B^T diag(dt_s e^{a_31 - a_s}) x
+// One block per (sequence, head), wave w owns columns of the state.
+template <int NKS, int VTW>
+__global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const bf16* __restrict__ x, long ldx) {
+  constexpr int CT = 32, NP = NKS * 32, NT = NKS * 2, LDB = NP + 8;
+  __shared__ __attribute__((aligned(16))) bf16 bs[2][CT * LDB];
+  const int h = blockIdx.x, b = blockIdx.y, N = p.D, V = p.V;
+  const int tid = threadIdx.x, lane = lane_id(), w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int kg = h / (p.heads / p.groups);
+  const int slot = p.s.slots[b], start = p.s.start[b], r0 = p.s.cu[b], n = p.s.cu[b + 1] - r0;
+  if (n <= 0) return;
+  float* Sg = p.S + ((long)slot * p.heads + h) * N * p.Vp;
+  const float A = p.A[h], gain = p.c.gain, skip = p.skip[h], dtb = p.dt_bias[h];
+  const bf16* y = static_cast<const bf16*>(p.c.y);
+  const bf16* xb = x + p.k_ch + kg * N;
+  const bf16* xc = x + p.q_ch + kg * N;
+  const bf16* xv = x + p.v_ch + (long)h * V;
+
+  f32x4 S[NT][VTW];
+#pragma unroll
+  for (int dt = 0; dt < NT; ++dt)
+#pragma unroll
+    for (int j = 0; j < VTW; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
+        S[dt][j][i] = start > 0 && d < N && v < V ? Sg[(long)d * p.Vp + v] : 0.f;
+      }
+  for (int t0 = 0, buf = 0; t0 < n; t0 += CT, buf ^= 1) {
+    const int nt = min(CT, n - t0);
+    bf16* B = bs[buf];
+    for (int c = tid; c < CT * (NP / 4); c += 256) {
+      const int t = c / (NP / 4), d = (c % (NP / 4)) * 4;
+      const bf16x4 z = {};
+      st4(B + t * LDB + d, t < nt && d < N ? ld4(xb + (r0 + t0 + t) * ldx + d) : z);
+    }
+    // lane t (and t + 32): step size and summed log decay
+    const int tl = lane & 31;
+    float dt = 0.f;
+    if (tl < nt) dt = softplus_x(gain * bf2f(y[(r0 + t0 + tl) * p.c.ldy + p.gate_col + h]) + dtb);
+    float a = A * dt;
+#pragma unroll
+    for (int off = 1; off < 32; off <<= 1) {
+      const float u = __shfl_up(a, off, 32);
+      if (tl >= off) a += u;
+    }
+    const float a_end = __shfl(a, 31, 64);
+    const float wend = dt * expf(a_end - a);
+    // C as the operand of token r (two tiles), x as the operand of column r
+    bf16x8 cf[2][NKS];
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt)
+#pragma unroll
+      for (int ks = 0; ks < NKS; ++ks) {
+        const bf16x4 z = {};
+        const bf16* c = xc + (r0 + t0 + min(mt * 16 + r, nt - 1)) * ldx;
+        const int d = ks * 32 + 4 * g;
+        cf[mt][ks] = cat(d < N ? ld4(c + d) : z, d + 16 < N ? ld4(c + d + 16) : z);
+      }
+    bf16x8 xf[VTW];
+#pragma unroll
+    for (int j = 0; j < VTW; ++j) {
+      const int v = (w * VTW + j) * 16 + r;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int t = (e >> 2) * 16 + 4 * g + (e & 3);
+        xf[j][e] = t < nt && v < V ? xv[(r0 + t0 + t) * ldx + v] : f2bf(0.f);
+      }
+    }
+    __syncthreads();  // B is there; the buffer written next was last read before this
+    // scores transposed: rows s, column t = r -- the operand layout of P
+    f32x4 sc[2][2];  // [s tile][t tile]
+#pragma unroll
+    for (int st = 0; st < 2; ++st)
+#pragma unroll
+      for (int mt = 0; mt < 2; ++mt) sc[st][mt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks)
+#pragma unroll
+      for (int st = 0; st < 2; ++st) {
+        const bf16* bp = B + (st * 16 + r) * LDB + ks * 32 + 4 * g;
+        const bf16x8 bf = cat(ld4(bp), ld4(bp + 16));
+#pragma unroll
+        for (int mt = st; mt < 2; ++mt) sc[st][mt] = mfma16(bf, cf[mt][ks], sc[st][mt]);
+      }
+    f32x4 as[2], ds[2], wv[2];  // a, dt and the state weights of rows s = 16 st + 4 g + i
+#pragma unroll
+    for (int st = 0; st < 2; ++st)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        as[st][i] = __shfl(a, st * 16 + 4 * g + i, 64);
+        ds[st][i] = __shfl(dt, st * 16 + 4 * g + i, 64);
+        wv[st][i] = __shfl(wend, st * 16 + 4 * g + i, 64);
+      }
+    bf16x8 ph[2], pl[2];
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt) {
+      const float at = __shfl(a, mt * 16 + r, 64);
+      f32x4 pm[2];
+#pragma unroll
+      for (int st = 0; st < 2; ++st)
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          pm[st][i] = st * 16 + 4 * g + i <= mt * 16 + r
+                          ? sc[st][mt][i] * ds[st][i] * __builtin_amdgcn_exp2f(1.4426950408889634f * (at - as[st][i])) : 0.f;
+      split8(pm[0], pm[1], ph[mt], pl[mt]);
+    }
+    f32x4 o[2][VTW];
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt)
+#pragma unroll
+      for (int j = 0; j < VTW; ++j) o[mt][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks)
+#pragma unroll
+      for (int j = 0; j < VTW; ++j) {
+        bf16x8 sh, sl;
+        split8(S[2 * ks][j], S[2 * ks + 1][j], sh, sl);
+#pragma unroll
+        for (int mt = 0; mt < 2; ++mt) {
+          o[mt][j] = mfma16(cf[mt][ks], sh, o[mt][j]);
+          o[mt][j] = mfma16(cf[mt][ks], sl, o[mt][j]);
+        }
+      }
+    const float dec = expf(a_end);
+    bf16x8 uh[VTW], ul[VTW];
+#pragma unroll
+    for (int j = 0; j < VTW; ++j) {
+      f32x4 u[2];
+#pragma unroll
+      for (int st = 0; st < 2; ++st)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) u[st][i] = bf2f(xf[j][st * 4 + i]) * wv[st][i];
+      split8(u[0], u[1], uh[j], ul[j]);
+    }
+    // rows t = 16 mt + 4 g + i: the decays of rows s with the same index
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt)
+#pragma unroll
+      for (int j = 0; j < VTW; ++j) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[mt][j][i] *= __builtin_amdgcn_exp2f(1.4426950408889634f * as[mt][i]);
+        o[mt][j] = mfma16(ph[mt], xf[j], o[mt][j]);
+        o[mt][j] = mfma16(pl[mt], xf[j], o[mt][j]);
+        const int v = (w * VTW + j) * 16 + r;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int t = mt * 16 + 4 * g + i;
+          if (t < nt && v < V) p.raw[(r0 + t0 + t) * p.ldr + (long)h * V + v] = o[mt][j][i] + skip * bf2f(xf[j][mt * 4 + i]);
+        }
+      }
+#pragma unroll
+    for (int dt2 = 0; dt2 < NT; ++dt2) {
+      const bf16* bp = B + (4 * g + (r >> 2)) * LDB + dt2 * 16 + 4 * (r & 3);
+      const bf16x8 bf = cat(ds_read_tr(bp), ds_read_tr(bp + 16 * LDB));
+#pragma unroll
+      for (int j = 0; j < VTW; ++j) {
+        S[dt2][j] *= dec;
+        S[dt2][j] = mfma16(bf, uh[j], S[dt2][j]);
+        S[dt2][j] = mfma16(bf, ul[j], S[dt2][j]);
+      }
+    }
+  }
+#pragma unroll
+  for (int dt = 0; dt < NT; ++dt)
+#pragma unroll
+    for (int j = 0; j < VTW; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
+        if (d < N && v < p.Vp) Sg[(long)d * p.Vp + v] = S[dt][j][i];
+      }
+}
+
 // After a portion: the inputs of its last `taps` positions enter the ring.
 template <typename T>
 __global__ __launch_bounds__(256) void conv_tail_kernel(ConvParams c, SeqParams s) {
@@ -337,6 +890,42 @@ extern "C" hipError_t lsd_recur_seq(const RecurParams* p, int delta, int f32, hi
 #undef LSD_RS_V
 #undef LSD_RS_N
 #undef LSD_RS
+  return hipGetLastError();
+}
+
+// Can the chunked kernels take these sizes?
+extern "C" int lsd_chunk_ok(int delta, int D, int V, int groups, int heads) {
+  if (D > 128 || V > 128) return 0;
+  return delta ? D % 8 == 0 && V >= 1 : D % 4 == 0 && (heads * V) % 4 == 0;
+}
+
+extern "C" hipError_t lsd_conv_silu(const ConvParams* c, const SeqParams* s, int T, bf16* out, long ldo, hipStream_t st) {
+  if (T == 0) return hipSuccess;
+  if (c->c0 % 8 == 0 && c->channels % 8 == 0)
+    hipLaunchKernelGGL((conv_silu_kernel<8>), dim3(T, (c->channels + 2047) / 2048), dim3(256), 0, st, *c, *s, out, ldo);
+  else
+    hipLaunchKernelGGL((conv_silu_kernel<1>), dim3(T, (c->channels + 255) / 256), dim3(256), 0, st, *c, *s, out, ldo);
+  return hipGetLastError();
+}
+
+extern "C" hipError_t lsd_recur_chunk(const RecurParams* p, int delta, const bf16* x, long ldx, hipStream_t st) {
+  if (p->s.B == 0) return hipSuccess;
+  const dim3 grid(p->heads, p->s.B);
+#define LSD_CK(KERNEL, KS)                                                                               \
+  if (p->V <= 64) hipLaunchKernelGGL((KERNEL<KS, 1>), grid, dim3(256), 0, st, *p, x, ldx);                \
+  else hipLaunchKernelGGL((KERNEL<KS, 2>), grid, dim3(256), 0, st, *p, x, ldx);
+#define LSD_CK_D(KERNEL)                       \
+  if (p->D <= 32) { LSD_CK(KERNEL, 1) }        \
+  else if (p->D <= 64) { LSD_CK(KERNEL, 2) }   \
+  else if (p->D <= 128) { LSD_CK(KERNEL, 4) }  \
+  else return hipErrorInvalidValue;
+  if (delta) {
+    LSD_CK_D(delta_chunk_kernel)
+  } else {
+    LSD_CK_D(ssd_chunk_kernel)
+  }
+#undef LSD_CK_D
+#undef LSD_CK
   return hipGetLastError();
 }
 

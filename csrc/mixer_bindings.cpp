@@ -11,6 +11,7 @@
 
 #include <climits>
 
+#include "kernels/gemm_params.h"
 #include "kernels/mixer_params.h"
 
 using lsd::ConvParams;
@@ -23,6 +24,9 @@ using lsd::TalkParams;
 extern "C" {
 int lsd_recur_block(int D, int V);
 hipError_t lsd_recur_seq(const RecurParams* p, int delta, int f32, hipStream_t st);
+int lsd_chunk_ok(int delta, int D, int V, int groups, int heads);
+hipError_t lsd_conv_silu(const ConvParams* c, const SeqParams* s, int T, lsd_bf16_t* out, long ldo, hipStream_t st);
+hipError_t lsd_recur_chunk(const RecurParams* p, int delta, const lsd_bf16_t* x, long ldx, hipStream_t st);
 hipError_t lsd_conv_tail(const ConvParams* c, const SeqParams* s, int f32, hipStream_t st);
 hipError_t lsd_head_norm_gate(const MixOutParams* p, int f32, hipStream_t st);
 hipError_t lsd_gated_group_norm(const MixOutParams* p, int f32, hipStream_t st);
@@ -115,11 +119,20 @@ void out_rows(RecurParams& p, const Tensor& out, const Tensor& y) {
   p.out = out.data_ptr(); p.ldo = out.stride(0); p.out_cols = out.size(1);
 }
 
+// Rows of SiLU(convolution) (bf16) for the chunked forms, which then run.
+void run_chunks(const RecurParams& p, int delta, const Tensor& y) {
+  const int64_t T = y.size(0), ld = (p.c.channels + 7) / 8 * 8;
+  auto x = torch::empty({T, ld}, y.options());
+  auto* xp = reinterpret_cast<lsd_bf16_t*>(x.data_ptr());
+  check_hip(lsd_conv_silu(&p.c, &p.s, T, xp, ld, cur_stream()), "conv_silu");
+  check_hip(lsd_recur_chunk(&p, delta, xp, ld, cur_stream()), "recur_chunk");
+}
+
 // y [T, N] rows of q | k | v conv channels from column c0 and beta's logits from
 // gate_col; low [T, >= heads D at 0, heads V at gate_off].  Token by token.
 void delta_seq(Tensor y, int64_t c0, int64_t gate_col, Tensor low, int64_t gate_off, Tensor slots, Tensor start,
                Tensor cu, int64_t heads, int64_t groups, int64_t D, int64_t V, Tensor taps, Tensor ring, Tensor state,
-               Tensor A, Tensor dt_bias, Tensor norm, double gain, double eps, Tensor out, bool single) {
+               Tensor A, Tensor dt_bias, Tensor norm, double gain, double eps, Tensor out, bool single, bool chunked) {
   const bool f32 = is_f32(y, "y");
   RecurParams p{};
   p.c = conv(y, c0, taps, c10::nullopt, ring, gain);
@@ -136,6 +149,12 @@ void delta_seq(Tensor y, int64_t c0, int64_t gate_col, Tensor low, int64_t gate_
   out_rows(p, out, y);
   p.write_ring = single;
   TORCH_CHECK(!single || p.s.B == y.size(0), "delta_seq: one row per sequence");
+  if (chunked) {
+    TORCH_CHECK(!f32 && !single && lsd_chunk_ok(1, D, V, groups, heads), "delta_seq: no chunked kernel");
+    run_chunks(p, 1, y);
+    check_hip(lsd_conv_tail(&p.c, &p.s, f32, cur_stream()), "conv_tail");
+    return;
+  }
   const int vb = lsd_recur_block(D, V);
   TORCH_CHECK(vb > 0, "delta_seq: no kernel for key dimension ", D);
   Tensor raw;
@@ -167,10 +186,10 @@ void group_norm_out(const Tensor& raw, const Tensor& y, int64_t inner, int64_t n
   check_hip(lsd_gated_group_norm(&o, f32, cur_stream()), "gated_group_norm");
 }
 
-// y [T, N]: z | x | B | C | dt.  Token by token.
+// y [T, N]: z | x | B | C | dt.  `chunked`: prompts of bf16 models
 void ssm_seq(Tensor y, Tensor slots, Tensor start, Tensor cu, int64_t heads, int64_t groups, int64_t N, int64_t V,
              int64_t norm_groups, Tensor taps, Tensor bias, Tensor ring, Tensor state, Tensor A, Tensor dt_bias,
-             Tensor skip, Tensor norm, double gain, double eps, Tensor out, bool single) {
+             Tensor skip, Tensor norm, double gain, double eps, Tensor out, bool single, bool chunked) {
   const bool f32 = is_f32(y, "y");
   const int64_t inner = heads * V;
   RecurParams p{};
@@ -188,8 +207,13 @@ void ssm_seq(Tensor y, Tensor slots, Tensor start, Tensor cu, int64_t heads, int
   p.raw = raw.data_ptr<float>(); p.ldr = inner;
   p.write_ring = single;
   TORCH_CHECK(!single || p.s.B == y.size(0), "ssm_seq: one row per sequence");
-  TORCH_CHECK(lsd_recur_block(N, V) > 0, "ssm_seq: no kernel for state size ", N);
-  check_hip(lsd_recur_seq(&p, 0, f32, cur_stream()), "ssm_seq");
+  if (chunked) {
+    TORCH_CHECK(!f32 && !single && lsd_chunk_ok(0, N, V, groups, heads), "ssm_seq: no chunked kernel");
+    run_chunks(p, 0, y);
+  } else {
+    TORCH_CHECK(lsd_recur_block(N, V) > 0, "ssm_seq: no kernel for state size ", N);
+    check_hip(lsd_recur_seq(&p, 0, f32, cur_stream()), "ssm_seq");
+  }
   group_norm_out(raw, y, inner, norm_groups, norm, gain, eps, out);
   if (!single) check_hip(lsd_conv_tail(&p.c, &p.s, f32, cur_stream()), "conv_tail");
 }
@@ -320,14 +344,16 @@ void talk_decode(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tensor
 }  // namespace
 
 void lsd_register_mixers(pybind11::module& m) {
+  m.def("chunk_ok", [](bool delta, int64_t D, int64_t V, int64_t groups, int64_t heads) {
+    return lsd_chunk_ok(delta, (int)D, (int)V, (int)groups, (int)heads) != 0; });
   m.def("delta_seq", &delta_seq, py::arg("y"), py::arg("c0"), py::arg("gate_col"), py::arg("low"), py::arg("gate_off"),
         py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("heads"), py::arg("groups"), py::arg("dim"),
         py::arg("vdim"), py::arg("taps"), py::arg("ring"), py::arg("state"), py::arg("A"), py::arg("dt_bias"),
-        py::arg("norm"), py::arg("gain"), py::arg("eps"), py::arg("out"), py::arg("single"));
+        py::arg("norm"), py::arg("gain"), py::arg("eps"), py::arg("out"), py::arg("single"), py::arg("chunked") = false);
   m.def("ssm_seq", &ssm_seq, py::arg("y"), py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("heads"),
         py::arg("groups"), py::arg("state_dim"), py::arg("vdim"), py::arg("norm_groups"), py::arg("taps"), py::arg("bias"),
         py::arg("ring"), py::arg("state"), py::arg("A"), py::arg("dt_bias"), py::arg("skip"), py::arg("norm"),
-        py::arg("gain"), py::arg("eps"), py::arg("out"), py::arg("single"));
+        py::arg("gain"), py::arg("eps"), py::arg("out"), py::arg("single"), py::arg("chunked") = false);
   m.def("loop_pack", &loop_pack, py::arg("x"), py::arg("x0"), py::arg("step"), py::arg("f32"));
   m.def("gelu_mul_f32", &gelu_mul_f32, py::arg("y"), py::arg("out"), py::arg("scale"));
   m.def("rope_append", &rope_append, py::arg("y"), py::arg("heads"), py::arg("k"), py::arg("v"), py::arg("table"),

@@ -449,13 +449,19 @@ class HipBackend(Backend):
         for s, mt in self._parts(meta):
             self.C.delta_seq(y[s], c0, c0 + m.conv_channels, low[s], n, mt.seq_slots, mt.q_start, mt.cu_q, m.heads,
                              m.kv_heads, m.dim, m.vdim, w("mixer.taps"), entry[1], entry[0], w("mixer.A"),
-                             w("mixer.dt_bias"), w("mixer.norm"), gain, eps, out[s], mt.is_decode)
+                             w("mixer.dt_bias"), w("mixer.norm"), gain, eps, out[s], mt.is_decode,
+                             self._chunked(mt) and self.C.chunk_ok(True, m.dim, m.vdim, m.kv_heads, m.heads))
+
+    def _chunked(self, meta) -> bool:
+        """Prompts of bf16 models run in chunks (very short portions token by token)."""
+        return not self.fp32 and not meta.is_decode and meta.num_tokens > self.R.chunk_min * meta.num_seqs
 
     def _ssm(self, y, w, m, gain, kv, entry, meta, eps, out):
         for s, mt in self._parts(meta):
             self.C.ssm_seq(y[s], mt.seq_slots, mt.q_start, mt.cu_q, m.heads, m.groups, m.state, m.vdim, m.norm_groups,
                            w("mixer.taps"), w("mixer.conv.b"), entry[1], entry[0], w("mixer.A"), w("mixer.dt_bias"),
-                           w("mixer.D"), w("mixer.norm"), gain, eps, out[s], mt.is_decode)
+                           w("mixer.D"), w("mixer.norm"), gain, eps, out[s], mt.is_decode,
+                           self._chunked(mt) and self.C.chunk_ok(False, m.state, m.vdim, m.groups, m.heads))
 
     def _tm(self, rows: float) -> int:
         return 64 if self.fp32 else self.R.group_tm(rows)

@@ -124,6 +124,9 @@ class Routing:
     # prompts of at least latent_expand_t tokens attend over expanded keys and
     # values where that saves multiply-adds (latent_expand; 0 disables)
     latent_expand_t: int = 256
+    # recurrent layers: prompts of more than chunk_min tokens per sequence on
+    # average run in chunks, shorter ones token by token
+    chunk_min: int = 4
     # decode attention with mixed heads: blocks a launch aims for, at least two
     # 64-key tiles each
     talk_target: int = 512

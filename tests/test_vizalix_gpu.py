@@ -35,9 +35,9 @@ def i32(v):
 
 
 def err(got, want):
-    """Largest difference over the wanted rows' root mean square."""
+    """Largest difference, relative to the wanted value plus the root mean square of all."""
     want = want.double()
-    return float((got.double().cpu() - want).abs().max() / want.pow(2).mean().sqrt())
+    return float(((got.double().cpu() - want).abs() / (want.pow(2).mean().sqrt() + want.abs())).max())
 
 
 def rounded(t, dt):
@@ -231,3 +231,203 @@ def test_rope_append(C, H, G, D, V, rot, dt):
         pg = int(table[s, p // PAGE])
         assert err(K[pg, :, p % PAGE, :D], wk[t]) < tol and err(Vp[pg, :, p % PAGE, :V], x["v"][t] * gain) < tol
     assert int((Vp.abs().sum((1, 3)) > 0).sum()) == b.T
+
+
+# -- recurrences ------------------------------------------------------------------
+
+def portions(n, sizes):
+    out, at = [], 0
+    for s in sizes:
+        if at < n:
+            out.append((at, min(n, at + s)))
+            at += s
+    return out + ([(at, n)] if at < n else [])
+
+
+DELTA = [(2, 2, 8, 8, 1), (4, 2, 24, 20, 3), (3, 3, 64, 64, 4), (2, 1, 128, 128, 4), (4, 4, 32, 100, 2), (2, 2, 96, 40, 4)]
+
+
+class DeltaCase:
+    """In-projection and low-rank rows of one sequence, and what comes out of it."""
+
+    def __init__(self, C, H, G, D, V, n, T, dt, seed=0, decay=1.0, strong=0.0):
+        self.C, self.dims, self.dt = C, (H, G, D, V), dt
+        g = torch.Generator().manual_seed(seed)
+        R = lambda *s: torch.randn(*s, generator=g)  # noqa: E731
+        self.ch = 2 * G * D + H * V
+        self.c0, self.gain, self.eps = 64, 0.75, 1e-5
+        x, b = rounded(R(T, self.ch), dt), rounded(R(T, H), dt)
+        lowd, gate = rounded(R(T, H * D), dt), rounded(R(T, H * V), dt)
+        taps, A = R(self.ch, n) / n ** 0.5, R(H)
+        dtb, norm = R(H * D) - 2, 1 + 0.2 * R(V)
+        A = -torch.exp(A) * decay
+        if strong:  # some key channels forget nearly everything at every step
+            dtb[torch.rand(H * D, generator=g) < 0.2] += strong
+        self.y = torch.zeros(T, up(self.c0 + self.ch + H, 64), dtype=dt)
+        self.y[:, self.c0: self.c0 + self.ch], self.y[:, self.c0 + self.ch: self.c0 + self.ch + H] = x, b
+        self.nl = up(max(H * D, H * V), 16)
+        self.low = torch.zeros(T, 2 * self.nl, dtype=dt)
+        self.low[:, : H * D], self.low[:, self.nl: self.nl + H * V] = lowd, gate
+        self.par = [cuda(t, F32) for t in (taps, A, dtb, norm)]
+        A, taps, dtb, norm = A.double(), taps.double(), dtb.double(), norm.double()
+        q, k, v = torch.split(orc.silu(orc.short_conv(x * self.gain, taps)), [G * D, G * D, H * V], 1)
+        of = [h // (H // G) for h in range(H)]
+        q, k = (orc.unit(t.reshape(T, G, D))[:, of] for t in (q, k))
+        decays = torch.exp(A[:, None] * orc.softplus(lowd * self.gain + dtb).reshape(T, H, D))
+        o, self.S = orc.delta_rule(q * D ** -0.5, k, v.reshape(T, H, V), decays, orc.sigmoid(b * self.gain))
+        o = orc.rms(o, self.eps) * norm
+        self.want = o.reshape(T, H * V) * orc.sigmoid(gate * self.gain)
+        self.state = torch.full((3, H, D, up(V, 4)), float("nan"), device="cuda")
+        self.ring = torch.full((3, n, self.ch), float("nan"), dtype=dt, device="cuda")
+
+    def run(self, parts, chunked, slot=1):
+        H, G, D, V = self.dims
+        taps, A, dtb, norm = self.par
+        outs = []
+        for a, b in parts:
+            out = torch.full((b - a, up(H * V, 64)), float("nan"), dtype=self.dt, device="cuda")
+            single = b - a == 1 and not chunked
+            self.C.delta_seq(cuda(self.y[a:b]), self.c0, self.c0 + self.ch, cuda(self.low[a:b]), self.nl, i32([slot]),
+                             i32([a]), i32([0, b - a]), H, G, D, V, taps, self.ring, self.state, A, dtb, norm, self.gain,
+                             self.eps, out, single, chunked)
+            assert not out[:, H * V:].any()
+            outs.append(out[:, : H * V])
+        return torch.cat(outs)
+
+
+SPLITS = [[100], [1] * 100, [2] * 50, [16, 16, 1, 31, 2, 3, 5], [7, 33, 1, 1, 58]]
+
+
+@pytest.mark.parametrize("H,G,D,V,n", DELTA + [(2, 1, 200, 300, 5)])
+@pytest.mark.parametrize("sizes", SPLITS)
+@pytest.mark.parametrize("dt", [BF, F32])
+def test_delta_rule_by_tokens(C, H, G, D, V, n, sizes, dt):
+    c = DeltaCase(C, H, G, D, V, n, 60, dt)
+    out = c.run(portions(60, sizes), False)
+    assert err(out, c.want) < (3e-2 if dt == BF else 3e-5)
+    assert err(c.state[1, ..., :V], c.S) < 2e-5  # the state is fp32 in both
+
+
+@pytest.mark.parametrize("H,G,D,V,n", DELTA)
+@pytest.mark.parametrize("sizes", SPLITS)
+@pytest.mark.parametrize("decay,strong", [(1.0, 0.0), (0.01, 0.0), (8.0, 0.0), (4.0, 12.0)])
+def test_delta_rule_in_chunks(C, H, G, D, V, n, sizes, decay, strong):
+    """Slow decays, and some that outrun the range of a chunk's factors."""
+    c = DeltaCase(C, H, G, D, V, n, 100, BF, decay=decay, strong=strong)
+    out = c.run(portions(100, sizes), True)
+    assert err(out, c.want) < 8e-2
+    assert err(c.state[1, ..., :V], c.S) < 3e-2  # q, k and v are bf16 behind the convolution
+
+
+def test_delta_rule_chunks_between_tokens(C):
+    """A state passed between the two forms."""
+    c = DeltaCase(C, 3, 3, 64, 64, 4, 90, BF)
+    out = torch.cat([c.run([(0, 40)], True), c.run([(i, i + 1) for i in range(40, 60)], False), c.run([(60, 90)], True)])
+    assert err(out, c.want) < 8e-2
+
+
+SSM = [(2, 8, 8, 1, 1, 1), (6, 12, 20, 2, 3, 4), (4, 64, 128, 1, 1, 4), (3, 128, 64, 3, 3, 2), (8, 32, 16, 2, 4, 3),
+       (2, 100, 36, 1, 2, 4)]
+
+
+class SsmCase:
+    def __init__(self, C, H, V, N, G, NG, n, T, dt, seed=0, decay=1.0):
+        self.C, self.dims, self.dt = C, (H, V, N, G, NG), dt
+        g = torch.Generator().manual_seed(seed)
+        R = lambda *s: torch.randn(*s, generator=g)  # noqa: E731
+        inner, self.gain, self.eps = H * V, 0.75, 1e-5
+        ch = inner + 2 * G * N
+        z, x, d = rounded(R(T, inner), dt), rounded(R(T, ch), dt), rounded(R(T, H), dt)
+        taps, bias, A = R(ch, n) / n ** 0.5, 0.3 * R(ch), R(H)
+        dtb, skip, norm = R(H) - 1, 1 + 0.3 * R(H), 1 + 0.2 * R(inner)
+        A = A + float(np.log(decay))
+        self.y = torch.nn.functional.pad(torch.cat([z, x, d], 1), (0, up(inner + ch + H, 64) - inner - ch - H)).to(dt)
+        self.par = [cuda(t, F32) for t in (taps, bias, -torch.exp(A), dtb, skip, norm)]
+        taps, bias, A, dtb, skip, norm = (t.double() for t in (taps, bias, A, dtb, skip, norm))
+        xbc = orc.silu(orc.short_conv(x * self.gain, taps, bias))
+        u, B, Cc = torch.split(xbc, [inner, G * N, G * N], 1)
+        of = [h // (H // G) for h in range(H)]
+        yy, self.S = orc.ssd(u.reshape(T, H, V), B.reshape(T, G, N)[:, of], Cc.reshape(T, G, N)[:, of],
+                             orc.softplus(d * self.gain + dtb), A, skip)
+        yy = yy.reshape(T, inner) * orc.silu(z * self.gain)
+        self.want = orc.rms(yy.reshape(T, NG, -1), self.eps).reshape(T, inner) * norm
+        self.state = torch.full((3, H, N, up(V, 4)), float("nan"), device="cuda")
+        self.ring = torch.full((3, n, ch), float("nan"), dtype=dt, device="cuda")
+
+    def run(self, parts, chunked, slot=1):
+        H, V, N, G, NG = self.dims
+        taps, bias, A, dtb, skip, norm = self.par
+        outs = []
+        for a, b in parts:
+            out = torch.full((b - a, up(H * V, 64)), float("nan"), dtype=self.dt, device="cuda")
+            self.C.ssm_seq(cuda(self.y[a:b]), i32([slot]), i32([a]), i32([0, b - a]), H, G, N, V, NG, taps, bias, self.ring,
+                           self.state, A, dtb, skip, norm, self.gain, self.eps, out, b - a == 1 and not chunked, chunked)
+            assert not out[:, H * V:].any()
+            outs.append(out[:, : H * V])
+        return torch.cat(outs)
+
+
+@pytest.mark.parametrize("H,V,N,G,NG,n", SSM + [(2, 200, 300, 1, 1, 5)])
+@pytest.mark.parametrize("sizes", SPLITS)
+@pytest.mark.parametrize("dt", [BF, F32])
+def test_mamba2_by_tokens(C, H, V, N, G, NG, n, sizes, dt):
+    c = SsmCase(C, H, V, N, G, NG, n, 60, dt)
+    out = c.run(portions(60, sizes), False)
+    assert err(out, c.want) < (3e-2 if dt == BF else 3e-5)
+    assert err(c.state[1, ..., :V], c.S) < 2e-5
+
+
+@pytest.mark.parametrize("H,V,N,G,NG,n", SSM)
+@pytest.mark.parametrize("sizes", SPLITS)
+@pytest.mark.parametrize("decay", [1.0, 0.01, 30.0])
+def test_mamba2_in_chunks(C, H, V, N, G, NG, n, sizes, decay):
+    c = SsmCase(C, H, V, N, G, NG, n, 100, BF, decay=decay)
+    out = c.run(portions(100, sizes), True)
+    assert err(out, c.want) < 8e-2
+    assert err(c.state[1, ..., :V], c.S) < 3e-2
+
+
+def test_recurrences_of_many_sequences(C):
+    """Unequal sequences of one launch keep to their own slots."""
+    c = SsmCase(C, 4, 16, 32, 2, 2, 4, 70, BF)
+    H, V, N, G, NG = c.dims
+    taps, bias, A, dtb, skip, norm = c.par
+    lens, slots = [70, 3, 33, 1], [2, 0, 3, 1]
+    y = torch.cat([c.y[:n] for n in lens])
+    state = torch.full((4, H, N, V), float("nan"), device="cuda")
+    ring = torch.full((4, 4, H * V + 2 * G * N), float("nan"), dtype=BF, device="cuda")
+    out = torch.empty(sum(lens), H * V, dtype=BF, device="cuda")
+    cu = np.concatenate([[0], np.cumsum(lens)]).tolist()
+    C.ssm_seq(cuda(y), i32(slots), i32([0] * 4), i32(cu), H, G, N, V, NG, taps, bias, ring, state, A, dtb, skip, norm, c.gain,
+              c.eps, out, False, True)
+    for a, n in zip(cu, lens):
+        assert err(out[a: a + n], c.want[:n]) < 6e-2
+    assert err(state[2], c.S) < 3e-2
+    # one token each: all four sequences step together from there
+    pos = [n - 1 for n in lens]  # repeats each sequence's last token: other states, same for equal ones
+    out2 = torch.empty(4, H * V, dtype=BF, device="cuda")
+    before = state.clone()
+    C.ssm_seq(cuda(torch.stack([c.y[p] for p in pos])), i32(slots), i32(lens), i32([0, 1, 2, 3, 4]), H, G, N, V, NG, taps,
+              bias, ring, state, A, dtb, skip, norm, c.gain, c.eps, out2, True, False)
+    assert all(float((state[s] - before[s]).abs().max()) > 0 for s in slots)
+
+
+def test_gated_gemm_epilogue(C):
+    """gelu(s g) (s u) and the SiLU form, split-K, tiled and GEMV rows."""
+    from llm_sharding_demo_amd.ops.hip import HipBackend, interleave_experts
+
+    be = HipBackend()
+    be._counters = torch.zeros(8, 1 << 16, dtype=torch.int32, device="cuda")
+    g = torch.Generator().manual_seed(0)
+    for M in (1, 3, 8, 40, 200, 700):
+        h, w = rounded(torch.randn(M, 128, generator=g), BF), rounded(torch.randn(2 * 192, 128, generator=g) * 0.1, BF)
+        want = orc.gelu_tanh(h @ w[:192].T * 0.6) * (h @ w[192:].T * 0.6)
+        buf = torch.full((M, 256), 7.0, dtype=BF, device="cuda")
+        be.decode = M <= 200
+        be.linear(cuda(h, BF), interleave_experts(cuda(w, BF), 192, 128), act="gelu_mul", out=buf[:, 64:], scale=0.6)
+        assert err(buf[:, 64:], want) < 3e-2 and bool((buf[:, :64] == 7).all())
+    y = torch.randn(5, 64, generator=g)
+    out = torch.empty(5, 32, device="cuda")
+    C.gelu_mul_f32(cuda(y), out, 1.5)
+    gate, up_ = (torch.cat([y[:, i: i + 16], y[:, i + 32: i + 48]], 1).double() * 1.5 for i in (0, 16))
+    assert err(out, orc.gelu_tanh(gate) * up_) < 1e-5
