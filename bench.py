@@ -68,7 +68,7 @@ def parse():
                         "nothing measurable on one stage or in the 2/4-stage loopback rehearsal "
                         "(profiles/r2_prefill_chunk.log)")
     p.add_argument("--designs", default="",
-                   help="comma-separated presets with per-layer specs (timisun-2b, timisun-8b): instead of the "
+                   help="comma-separated presets with per-layer specs (timisun-2b, vizalix-2b, ...): instead of the "
                         "headline, prefill and decode throughput of each beside a Llama-family model of equal "
                         "width, depth, heads and active feed-forward (one GPU; one JSON line per model and batch)")
     p.add_argument("--design-batches", default="1,32,256")
@@ -107,14 +107,16 @@ def dense_twin(name: str) -> str:
     """Preset of the Llama-family model of a design's size: same width, depth,
     vocabulary and heads (4 query heads per KV head), and a feed-forward as
     wide as what one token activates.  Returns its name."""
-    from llm_sharding_demo_amd.config import MODEL_PRESETS, ModelConfig
+    from llm_sharding_demo_amd.config import MODEL_PRESETS, DenseSpec, ModelConfig
 
     mc = MODEL_PRESETS[name]
-    m, f = mc.layers[0].mixer, mc.layers[0].mlp
+    m = next((l.mixer for l in mc.layers if l.mixer.cached_per_token), mc.layers[0].mixer)
+    f = mc.layers[0].mlp
+    ffn = f.ff if isinstance(f, DenseSpec) else f.top * f.expert.ff + (f.shared.ff if f.shared else 0)
     twin = f"{name}-llama"
     MODEL_PRESETS[twin] = ModelConfig(
         name=twin, arch="llama", vocab_size=mc.vocab_size, hidden=m.heads * m.dim, n_layers=mc.n_layers,
-        n_heads=m.heads, n_kv_heads=max(1, m.heads // 4), ffn=f.top * f.expert.ff + (f.shared.ff if f.shared else 0),
+        n_heads=m.heads, n_kv_heads=max(1, m.heads // 4), ffn=ffn,
         max_positions=8192, norm_eps=mc.norm_eps, tie_embeddings=False, rope_theta=10000.0)
     return twin
 
@@ -152,7 +154,7 @@ def bench_designs(args) -> int:
                 print(json.dumps({
                     "metric": "prefill and decode throughput at equal size", "design": name, "model": model,
                     "batch": B, "prompt_len": args.prompt, "gen_tokens": args.gen, "layers": mc.n_layers,
-                    "params_m": round((mc.n_layers * mc.block_params() + mc.embed_params()) / 1e6, 1),
+                    "params_m": round((mc.stage_params(range(mc.n_layers)) + mc.embed_params()) / 1e6, 1),
                     "prefill_ms": round(p_ms, 3), "prefill_tok_s": round(B * args.prompt / p_ms * 1e3),
                     "decode_step_ms": round(d_ms, 4), "decode_tok_s": round(B / d_ms * 1e3), "dtype": "bf16",
                     "data": "synthetic prompts, random-init weights"}), flush=True)

@@ -57,6 +57,44 @@ __global__ __launch_bounds__(256) void rope_append_kernel(RopeAppendParams p) {
   }
 }
 
+// 8 columns per thread; dims and the rotation's half are multiples of 8.  One
+// block per four tokens, a wave each.
+__global__ __launch_bounds__(256) void rope_append_vec_kernel(RopeAppendParams p) {
+  const long row = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (row >= p.T) return;
+  const int pos = p.tpos[row], half = p.half;
+  const long page = p.table[(long)p.tslot[row] * p.tw + pos / PAGE];
+  const int nq = p.H * p.dim, nk = p.G * p.dim, nv = p.G * p.vdim;
+  const bf16* y = static_cast<const bf16*>(p.y) + row * p.ldy;
+  const float* cs = p.rope + (long)pos * half * 2;
+  for (int i = lane_id() * 8; i < nq + nk + nv; i += 512) {
+    const bf16x8 x = ld8(y + i);
+    float v[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = bf2f(x[e]) * p.gain;
+    const int d = i % p.dim;
+    if (i < nq + nk && d < 2 * half) {
+      const bool first = d < half;
+      const bf16x8 o = ld8(first ? y + i + half : y + i - half);
+      const float* c = cs + 2 * (first ? d : d - half);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float s = bf2f(o[e]) * p.gain * c[2 * e + 1];
+        v[e] = fmaf(v[e], c[2 * e], first ? -s : s);
+      }
+    }
+    bf16* dst;
+    if (i < nq) dst = static_cast<bf16*>(p.q) + row * nq + i;
+    else if (i < nq + nk) dst = static_cast<bf16*>(p.k) + ((page * p.G + (i - nq) / p.dim) * PAGE + pos % PAGE) * p.dim + d;
+    else dst = static_cast<bf16*>(p.v) + ((page * p.G + (i - nq - nk) / p.vdim) * PAGE + pos % PAGE) * p.vdim +
+               (i - nq - nk) % p.vdim;
+    bf16x8 r;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) r[e] = f2bf(v[e]);
+    st8(dst, r);
+  }
+}
+
 // One token per block, KT keys at a time.  Dynamic LDS: queries [H][dim], scores
 // before and after mixing [H][KT + 1], outputs [H][vdim], and per head the
 // running maximum, sum and rescaling factor.
@@ -683,6 +721,8 @@ extern "C" hipError_t lsd_talk_decode(const TalkParams* p, int hp, hipStream_t s
 extern "C" hipError_t lsd_rope_append(const RopeAppendParams* p, int f32, hipStream_t st) {
   if (p->T == 0) return hipSuccess;
   if (f32) hipLaunchKernelGGL((rope_append_kernel<float>), dim3(p->T), dim3(256), 0, st, *p);
+  else if (p->half % 8 == 0 && p->dim % 8 == 0 && p->vdim % 8 == 0)
+    hipLaunchKernelGGL(rope_append_vec_kernel, dim3((p->T + 3) / 4), dim3(256), 0, st, *p);
   else hipLaunchKernelGGL((rope_append_kernel<bf16>), dim3(p->T), dim3(256), 0, st, *p);
   return hipGetLastError();
 }

@@ -28,7 +28,29 @@ __device__ __forceinline__ void from_f(bf16* o, float v) { *o = f2bf(v); }
 
 __device__ __forceinline__ float sigmoid_x(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ float silu_x(float z) { return z / (1.f + expf(-z)); }
-__device__ __forceinline__ float softplus_x(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+// log(1 + e) = 2 atanh(s), s = e / (2 + e) <= 1/3 for e <= 1: the series is exact to fp32
+__device__ __forceinline__ float log1p_series(float s) {
+  const float q = s * s;
+  float t = fmaf(q, 2.f / 15.f, 2.f / 13.f);
+  t = fmaf(q, t, 2.f / 11.f);
+  t = fmaf(q, t, 2.f / 9.f);
+  t = fmaf(q, t, 2.f / 7.f);
+  t = fmaf(q, t, 2.f / 5.f);
+  t = fmaf(q, t, 2.f / 3.f);
+  return fmaf(q * t, s, 2.f * s);
+}
+// log(1 + exp(z)) = max(z, 0) + log(1 + exp(-|z|)), small values to full relative precision
+__device__ __forceinline__ float softplus_x(float z) {
+  const float e = expf(-fabsf(z));
+  return fmaxf(z, 0.f) + log1p_series(e / (2.f + e));
+}
+constexpr float LOG2E = 1.4426950408889634f;
+// hardware exp2 / reciprocal (about an ulp each) for the chunked forms
+__device__ __forceinline__ float exp_f(float z) { return __builtin_amdgcn_exp2f(z * LOG2E); }
+__device__ __forceinline__ float softplus_f(float z) {
+  const float e = exp_f(-fabsf(z));
+  return fmaxf(z, 0.f) + log1p_series(e * __builtin_amdgcn_rcpf(2.f + e));
+}
 constexpr float UNIT_EPS = 1e-6f;  // inside the root of a unit vector's length
 
 // Convolution of channel `ch` at packed row `row`, token t of its portion,
@@ -39,11 +61,27 @@ __device__ __forceinline__ float conv_at(const ConvParams& c, int ch, long row, 
   const T* ring = static_cast<const T*>(c.ring) + (long)slot * c.taps * c.channels + ch;
   const float* w = c.w + (long)ch * c.taps;
   float a = 0.f;
-  for (int j = 0; j < c.taps; ++j) {
-    const int back = c.taps - 1 - j;
-    if (back > pos) continue;
-    const float x = back <= t ? to_f(y[(row - back) * c.ldy]) : to_f(ring[(long)((pos - back) % c.taps) * c.channels]);
-    a = fmaf(w[j], x, a);
+  if (c.taps <= 4) {  // every load in flight at once
+    const int now = pos % c.taps;
+    float x[4], wv[4];
+#pragma unroll
+    for (int back = 0; back < 4; ++back) {
+      const bool live = back < c.taps && back <= pos;
+      const int at = now >= back ? now - back : now - back + c.taps;
+      const T* src = !live ? y + row * c.ldy : back <= t ? y + (row - back) * c.ldy : ring + (long)at * c.channels;
+      const float v = to_f(*src);
+      x[back] = live ? v : 0.f;
+      wv[back] = w[max(0, c.taps - 1 - back)];
+    }
+#pragma unroll
+    for (int back = 3; back >= 0; --back) a = fmaf(wv[back], x[back], a);
+  } else {
+    for (int j = 0; j < c.taps; ++j) {
+      const int back = c.taps - 1 - j;
+      if (back > pos) continue;
+      const float x = back <= t ? to_f(y[(row - back) * c.ldy]) : to_f(ring[(long)((pos - back) % c.taps) * c.channels]);
+      a = fmaf(w[j], x, a);
+    }
   }
   a *= c.gain;
   return c.bias ? a + c.bias[ch] : a;
@@ -70,7 +108,7 @@ __device__ __forceinline__ f32x4 column_sum(f32x4 v, float (*red)[LV * 4]) {
 // One (sequence, head, LV * 4 columns of the state) per block; thread (dg, lv)
 // holds rows dg + i * 256 / LV of four columns.  Dynamic LDS: q, k, decays [D].
 template <typename T, bool DELTA, int LV, int NR>
-__global__ __launch_bounds__(256) void recur_seq_kernel(RecurParams p) {
+__global__ __launch_bounds__(256, NR <= 8 ? 4 : 3) void recur_seq_kernel(RecurParams p) {
   constexpr int VB = LV * 4, DG = 256 / LV;
   extern __shared__ float dyn[];
   __shared__ __attribute__((aligned(16))) float red[4][LV * 4];
@@ -95,16 +133,43 @@ __global__ __launch_bounds__(256) void recur_seq_kernel(RecurParams p) {
   for (int t = 0; t < n; ++t) {
     const long row = r0 + t;
     const int pos = start + t;
-    for (int c = tid; c < 2 * D + VB; c += 256) {
+    // convolutions: q | k | v channels, a thread's first two together
+    auto channel = [&](int c, int& ch, float*& dst) -> bool {
       const int part = c < D ? 0 : c < 2 * D ? 1 : 2;
       const int i = part == 0 ? c : part == 1 ? c - D : c - 2 * D;
-      const int ch = part == 0 ? p.q_ch + kh * D + i : part == 1 ? p.k_ch + kh * D + i : p.v_ch + h * p.V + v0 + i;
-      const bool real = part < 2 || v0 + i < p.V;
-      const float a = real ? silu_x(conv_at<T>(p.c, ch, row, t, pos, slot)) : 0.f;
-      (part == 0 ? qs : part == 1 ? ks : vs)[i] = a;
-      if (p.write_ring && real && (part == 2 || (h % rep == 0 && v0 == 0)))
+      ch = part == 0 ? p.q_ch + kh * D + i : part == 1 ? p.k_ch + kh * D + i : p.v_ch + h * p.V + v0 + i;
+      dst = (part == 0 ? qs : part == 1 ? ks : vs) + i;
+      return part < 2 || v0 + i < p.V;
+    };
+    auto keep = [&](int c, int ch, bool real) {
+      if (p.write_ring && real && (c >= 2 * D || (h % rep == 0 && v0 == 0)))
         static_cast<T*>(p.c.ring)[((long)slot * p.c.taps + pos % p.c.taps) * p.c.channels + ch] =
             static_cast<const T*>(p.c.y)[row * p.c.ldy + p.c.c0 + ch];
+    };
+    {
+      int ch[2];
+      float* dst[2];
+      bool real[2];
+      float a[2];
+#pragma unroll
+      for (int q = 0; q < 2; ++q) {
+        const int c = min(tid + 256 * q, 2 * D + VB - 1);
+        real[q] = channel(c, ch[q], dst[q]);
+        a[q] = conv_at<T>(p.c, real[q] ? ch[q] : 0, row, t, pos, slot);
+      }
+#pragma unroll
+      for (int q = 0; q < 2; ++q) {
+        if (tid + 256 * q >= 2 * D + VB) continue;
+        *dst[q] = real[q] ? silu_x(a[q]) : 0.f;
+        keep(tid + 256 * q, ch[q], real[q]);
+      }
+    }
+    for (int c = tid + 512; c < 2 * D + VB; c += 256) {
+      int ch;
+      float* dst;
+      const bool real = channel(c, ch, dst);
+      *dst = real ? silu_x(conv_at<T>(p.c, ch, row, t, pos, slot)) : 0.f;
+      keep(c, ch, real);
     }
     const float gl = p.c.gain * to_f(static_cast<const T*>(p.c.y)[row * p.c.ldy + p.gate_col + h]);
     float beta = 0.f, a = 0.f, dt = 0.f;
@@ -196,9 +261,8 @@ __global__ __launch_bounds__(256) void recur_seq_kernel(RecurParams p) {
   }
 }
 
-// Rows of SiLU(convolution), bf16.  One block per row and 256 * VEC channels.
-template <int VEC>
-__global__ __launch_bounds__(256) void conv_silu_kernel(ConvParams c, SeqParams s, bf16* __restrict__ out, long ldo) {
+// Rows of SiLU(convolution), bf16, any tap count: one block per row and 256 channels.
+__global__ __launch_bounds__(256) void conv_silu_any_kernel(ConvParams c, SeqParams s, bf16* __restrict__ out, long ldo) {
   const int row = blockIdx.x;
   int a = 0, b = s.B;  // sequence: last one with cu <= row
   while (b - a > 1) {
@@ -206,29 +270,70 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvParams c, SeqParams 
     if (s.cu[m] <= row) a = m;
     else b = m;
   }
-  const int t = row - s.cu[a], pos = s.start[a] + t, slot = s.slots[a];
-  const int ch = (blockIdx.y * 256 + threadIdx.x) * VEC;
+  const int t = row - s.cu[a];
+  const int ch = blockIdx.y * 256 + threadIdx.x;
+  if (ch < c.channels) out[row * ldo + ch] = f2bf(silu_x(conv_at<bf16>(c, ch, row, t, s.start[a] + t, s.slots[a])));
+}
+
+// At most four taps, 8 channels per thread, CONV_RUN rows in turn: the taps and
+// the last three inputs stay in registers.
+constexpr int CONV_RUN = 16;
+__global__ __launch_bounds__(256) void conv_silu_kernel(ConvParams c, SeqParams s, int T, bf16* __restrict__ out, long ldo) {
+  const int row0 = blockIdx.x * CONV_RUN, row1 = min(T, row0 + CONV_RUN);
+  int seq = 0, hi = s.B;  // sequence of row0: last one with cu <= row0
+  while (hi - seq > 1) {
+    const int m = (seq + hi) >> 1;
+    if (s.cu[m] <= row0) seq = m;
+    else hi = m;
+  }
+  const int ch = (blockIdx.y * 256 + threadIdx.x) * 8;
   if (ch >= c.channels) return;
-  if constexpr (VEC == 1) {
-    out[row * ldo + ch] = f2bf(silu_x(conv_at<bf16>(c, ch, row, t, pos, slot)));
-  } else {
-    const bf16* y = static_cast<const bf16*>(c.y) + c.c0 + ch;
-    const bf16* ring = static_cast<const bf16*>(c.ring) + (long)slot * c.taps * c.channels + ch;
-    float acc[8] = {};
-    for (int j = 0; j < c.taps; ++j) {
-      const int back = c.taps - 1 - j;
-      if (back > pos) continue;
-      const bf16x8 x = ld8(back <= t ? y + (row - back) * c.ldy : ring + (long)((pos - back) % c.taps) * c.channels);
+  const bf16* y = static_cast<const bf16*>(c.y) + c.c0 + ch;
+  float w[4][8], bias[8];  // w[back]
 #pragma unroll
-      for (int e = 0; e < 8; ++e) acc[e] = fmaf(c.w[(long)(ch + e) * c.taps + j], bf2f(x[e]), acc[e]);
+  for (int e = 0; e < 8; ++e) {
+#pragma unroll
+    for (int back = 0; back < 4; ++back)
+      w[back][e] = back < c.taps ? c.w[(long)(ch + e) * c.taps + c.taps - 1 - back] * c.gain : 0.f;
+    bias[e] = c.bias ? c.bias[ch + e] : 0.f;
+  }
+  float past[3][8];
+  bool fresh = true;
+  int end = s.cu[seq + 1];
+  for (int row = row0; row < row1; ++row) {
+    while (row >= end) {
+      ++seq;
+      end = s.cu[seq + 1];
+      fresh = true;
     }
+    if (fresh) {  // inputs before this row: of this portion, or of earlier ones
+      const int t = row - s.cu[seq], pos = s.start[seq] + t;
+      const bf16* ring = static_cast<const bf16*>(c.ring) + (long)s.slots[seq] * c.taps * c.channels + ch;
+#pragma unroll
+      for (int back = 1; back < 4; ++back) {
+        bf16x8 v = {};
+        if (back < c.taps && back <= pos)
+          v = ld8(back <= t ? y + (long)(row - back) * c.ldy : ring + (long)((pos - back) % c.taps) * c.channels);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) past[back - 1][e] = bf2f(v[e]);
+      }
+      fresh = false;
+    }
+    const bf16x8 x = ld8(y + (long)row * c.ldy);
     bf16x8 o;
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-      const float v = acc[e] * c.gain + (c.bias ? c.bias[ch + e] : 0.f);
+      const float now = bf2f(x[e]);
+      float v = fmaf(w[0][e], now, bias[e]);
+      v = fmaf(w[1][e], past[0][e], v);
+      v = fmaf(w[2][e], past[1][e], v);
+      v = fmaf(w[3][e], past[2][e], v);
+      past[2][e] = past[1][e];
+      past[1][e] = past[0][e];
+      past[0][e] = now;
       o[e] = f2bf(silu(v));
     }
-    st8(out + row * ldo + ch, o);
+    st8(out + (long)row * ldo + ch, o);
   }
 }
 
@@ -315,6 +420,9 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
         S[dt][j][i] = start > 0 && d < D && v < V ? Sg[(long)d * p.Vp + v] : 0.f;
       }
+  float nrm[VTW];
+#pragma unroll
+  for (int j = 0; j < VTW; ++j) nrm[j] = p.norm[min((w * VTW + j) * 16 + r, V - 1)];
   // element work: token tid / 16, channels 8 (tid % 16) ..
   const int et = tid >> 4, ed = (tid & 15) * 8;
   const bool elive = ed < D;  // D % 8 == 0
@@ -323,16 +431,25 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
 #pragma unroll
     for (int e = 0; e < 8; ++e) dtb[e] = p.dt_bias[(long)h * D + ed + e];
 
+  // rows of the next chunk, in flight under this one
+  bf16x8 xq, xk, xl;
+  float rb = 0.f;
+  auto fetch = [&](int t0) {
+    const bf16x8 z = {};
+    const bool live = t0 + et < n && elive;
+    const long row = r0 + t0 + et;
+    xq = live ? ld8(x + row * ldx + p.q_ch + kh * D + ed) : z;
+    xk = live ? ld8(x + row * ldx + p.k_ch + kh * D + ed) : z;
+    xl = live ? ld8(low + row * p.ldl + (long)h * D + ed) : z;
+    if (tid < CT) rb = t0 + tid < n ? bf2f(y[(r0 + t0 + tid) * p.c.ldy + p.gate_col + h]) : 0.f;
+  };
+  fetch(0);
   for (int t0 = 0; t0 < n; t0 += CT) {
     const int nt = min(CT, n - t0);
     const long row = r0 + t0 + min(et, nt - 1);
     const bool tlive = et < nt && elive;
     float q8[8], k8[8], lg[8];
     {
-      const bf16x8 z = {};
-      const bf16x8 xq = tlive ? ld8(x + row * ldx + p.q_ch + kh * D + ed) : z;
-      const bf16x8 xk = tlive ? ld8(x + row * ldx + p.k_ch + kh * D + ed) : z;
-      const bf16x8 xl = tlive ? ld8(low + row * p.ldl + (long)h * D + ed) : z;
       float nq = 0.f, nk = 0.f;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
@@ -340,7 +457,7 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         k8[e] = bf2f(xk[e]);
         nq = fmaf(q8[e], q8[e], nq);
         nk = fmaf(k8[e], k8[e], nk);
-        lg[e] = tlive ? A * softplus_x(gain * bf2f(xl[e]) + dtb[e]) : 0.f;
+        lg[e] = tlive ? A * softplus_f(gain * bf2f(xl[e]) + dtb[e]) : 0.f;
       }
 #pragma unroll
       for (int off = 1; off < 16; off <<= 1) {
@@ -354,12 +471,24 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         k8[e] *= ik;
       }
     }
+    // values and gates of the chunk in the accumulator layout (tokens 4 g + i, columns r)
+    f32x4 vals[VTW], gates[VTW];
+#pragma unroll
+    for (int j = 0; j < VTW; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 4 * g + i, v = (w * VTW + j) * 16 + r;
+        const bool live = t < nt && v < V;
+        const long at = r0 + t0 + min(t, nt - 1);
+        vals[j][i] = live ? bf2f(x[at * ldx + p.v_ch + (long)h * V + v]) : 0.f;
+        gates[j][i] = live ? bf2f(low[at * p.ldl + p.gate_off + (long)h * V + v]) : 0.f;
+      }
     if (ed < DP) {
       *reinterpret_cast<f32x4*>(&Gs[et][ed]) = f32x4{lg[0], lg[1], lg[2], lg[3]};
       *reinterpret_cast<f32x4*>(&Gs[et][ed + 4]) = f32x4{lg[4], lg[5], lg[6], lg[7]};
     }
-    if (tid < CT)
-      betas[tid] = tid < nt ? sigmoid_x(gain * bf2f(y[(r0 + t0 + tid) * p.c.ldy + p.gate_col + h])) : 0.f;
+    if (tid < CT) betas[tid] = tid < nt ? sigmoid_x(gain * rb) : 0.f;
+    if (t0 + CT < n) fetch(t0 + CT);
     if (tid == 0) nbad = 0;
     __syncthreads();
     f32x4 g0[2] = {}, gt[2] = {}, gc[2] = {};
@@ -381,15 +510,15 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         const float G0 = g0[e >> 2][e & 3], Gt = gt[e >> 2][e & 3], Gc = gc[e >> 2][e & 3];
-        const float E = expf(Gt - G0);
+        const float E = exp_f(Gt - G0);
         const bool wide = G0 - Gc > RANGE;
         kt[e] = k8[e] * E;
         qt[e] = q8[e] * E;
-        kc[e] = wide ? 0.f : k8[e] * expf(G0 - Gt);
-        kf[e] = k8[e] * expf(Gc - Gt);
+        kc[e] = wide ? 0.f : k8[e] * exp_f(G0 - Gt);
+        kf[e] = k8[e] * exp_f(Gc - Gt);
         if (et == 0) {
-          e0[ed + e] = expf(G0);
-          er[ed + e] = expf(Gc - G0);
+          e0[ed + e] = exp_f(G0);
+          er[ed + e] = exp_f(Gc - G0);
           if (wide) bad[atomicAdd(&nbad, 1)] = ed + e;
         }
         Gs[et][ed + e] = Gt;
@@ -416,15 +545,6 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         kh_l[(ed + e) * LDT + et] = f2bf(kf[e] - bf2f(a));
       }
     }
-    // values of the chunk in the accumulator layout (tokens 4 g + i, columns r)
-    f32x4 vals[VTW];
-#pragma unroll
-    for (int j = 0; j < VTW; ++j)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = 4 * g + i, v = (w * VTW + j) * 16 + r;
-        vals[j][i] = t < nt && v < V ? bf2f(x[(r0 + t0 + t) * ldx + p.v_ch + (long)h * V + v]) : 0.f;
-      }
     __syncthreads();
     // operand of row r: k-slots (g, j) <-> d = 32 ks + 4 g + j, 32 ks + 16 + 4 g + (j - 4)
     auto opnd = [&](const bf16* a, int ks) {
@@ -444,7 +564,7 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int t = 4 * g + i;
-          if (r <= t) acc[i] += (w == 0 ? Ks[t][d] : Qs[t][d]) * Ks[r][d] * expf(Gs[t][d] - Gs[r][d]);
+          if (r <= t) acc[i] += (w == 0 ? Ks[t][d] : Qs[t][d]) * Ks[r][d] * exp_f(Gs[t][d] - Gs[r][d]);
         }
       }
       if (w == 1) {
@@ -545,9 +665,8 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
       for (int j = 0; j < VTW; ++j) {
         const int v = (w * VTW + j) * 16 + r;
         if (v >= V) continue;
-        const float gate = gain * bf2f(low[orow * p.ldl + p.gate_off + (long)h * V + v]);
         out[orow * p.ldo + (long)h * V + v] =
-            f2bf(o[j][i] * rs * p.norm[v] * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * gate)));
+            f2bf(o[j][i] * rs * nrm[j] * __builtin_amdgcn_rcpf(1.f + exp_f(-gain * gates[j][i])));
       }
     }
     if (h == p.heads - 1)
@@ -569,11 +688,12 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
 // With a_t the summed log decays of the chunk up to token t:
 //   y = diag(e^{a}) C S + P x + D x,   P_ts = (C_t . B_s) e^{a_t - a_s} dt_s  (s <= t)
 //   S = e^{a_31} S + B^T diag(dt_s e^{a_31 - a_s}) x
-// One block per (sequence, head), wave w owns columns of the state.
+// Rows y silu(z) leave in bf16 (z: the first columns of the in-projection).  One block per (sequence, head), wave w owns columns of the state.
 template <int NKS, int VTW>
 __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const bf16* __restrict__ x, long ldx) {
-  constexpr int CT = 32, NP = NKS * 32, NT = NKS * 2, LDB = NP + 8;
-  __shared__ __attribute__((aligned(16))) bf16 bs[2][CT * LDB];
+  constexpr int CT = 32, NP = NKS * 32, NT = NKS * 2, LDB = NP + 8, VP = VTW * 64, LDX = VP + 8;
+  constexpr int NB = CT * NP / 1024, NX = CT * VP / 1024;  // groups of four elements per thread
+  __shared__ __attribute__((aligned(16))) bf16 bs[2][CT * LDB], cs[2][CT * LDB], xs[2][CT * LDX];
   const int h = blockIdx.x, b = blockIdx.y, N = p.D, V = p.V;
   const int tid = threadIdx.x, lane = lane_id(), w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r = lane & 15, g = lane >> 4;
@@ -582,10 +702,10 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
   if (n <= 0) return;
   float* Sg = p.S + ((long)slot * p.heads + h) * N * p.Vp;
   const float A = p.A[h], gain = p.c.gain, skip = p.skip[h], dtb = p.dt_bias[h];
-  const bf16* y = static_cast<const bf16*>(p.c.y);
-  const bf16* xb = x + p.k_ch + kg * N;
-  const bf16* xc = x + p.q_ch + kg * N;
-  const bf16* xv = x + p.v_ch + (long)h * V;
+  const bf16* y = static_cast<const bf16*>(p.c.y) + (long)r0 * p.c.ldy;
+  const bf16* xb = x + r0 * ldx + p.k_ch + kg * N;
+  const bf16* xc = x + r0 * ldx + p.q_ch + kg * N;
+  const bf16* xv = x + r0 * ldx + p.v_ch + (long)h * V;
 
   f32x4 S[NT][VTW];
 #pragma unroll
@@ -597,18 +717,43 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
         const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
         S[dt][j][i] = start > 0 && d < N && v < V ? Sg[(long)d * p.Vp + v] : 0.f;
       }
+  // rows of the next chunk, in flight under this one's products
+  bf16x4 rb[NB], rc[NB], rx[NX];
+  float rdt = 0.f;
+  const int tl = lane & 31;
+  auto fetch = [&](int t0) {
+    const bf16x4 z = {};
+#pragma unroll
+    for (int q = 0; q < NB; ++q) {
+      const int c = tid + q * 256, t = c / (NP / 4), d = (c % (NP / 4)) * 4;
+      const bool live = t0 + t < n && d < N;
+      rb[q] = live ? ld4(xb + (t0 + t) * ldx + d) : z;
+      rc[q] = live ? ld4(xc + (t0 + t) * ldx + d) : z;
+    }
+#pragma unroll
+    for (int q = 0; q < NX; ++q) {
+      const int c = tid + q * 256, t = c / (VP / 4), v = (c % (VP / 4)) * 4;
+      rx[q] = t0 + t < n && v < V ? ld4(xv + (t0 + t) * ldx + v) : z;
+    }
+    rdt = t0 + tl < n ? bf2f(y[(long)(t0 + tl) * p.c.ldy + p.gate_col + h]) : 0.f;
+  };
+  fetch(0);
   for (int t0 = 0, buf = 0; t0 < n; t0 += CT, buf ^= 1) {
     const int nt = min(CT, n - t0);
-    bf16* B = bs[buf];
-    for (int c = tid; c < CT * (NP / 4); c += 256) {
-      const int t = c / (NP / 4), d = (c % (NP / 4)) * 4;
-      const bf16x4 z = {};
-      st4(B + t * LDB + d, t < nt && d < N ? ld4(xb + (r0 + t0 + t) * ldx + d) : z);
+    const bf16 *B = bs[buf], *C = cs[buf], *X = xs[buf];
+#pragma unroll
+    for (int q = 0; q < NB; ++q) {
+      const int c = tid + q * 256, at = c / (NP / 4) * LDB + (c % (NP / 4)) * 4;
+      st4(bs[buf] + at, rb[q]);
+      st4(cs[buf] + at, rc[q]);
+    }
+#pragma unroll
+    for (int q = 0; q < NX; ++q) {
+      const int c = tid + q * 256;
+      st4(xs[buf] + c / (VP / 4) * LDX + (c % (VP / 4)) * 4, rx[q]);
     }
     // lane t (and t + 32): step size and summed log decay
-    const int tl = lane & 31;
-    float dt = 0.f;
-    if (tl < nt) dt = softplus_x(gain * bf2f(y[(r0 + t0 + tl) * p.c.ldy + p.gate_col + h]) + dtb);
+    const float dt = tl < nt ? softplus_f(gain * rdt + dtb) : 0.f;
     float a = A * dt;
 #pragma unroll
     for (int off = 1; off < 32; off <<= 1) {
@@ -616,45 +761,20 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
       if (tl >= off) a += u;
     }
     const float a_end = __shfl(a, 31, 64);
-    const float wend = dt * expf(a_end - a);
-    // C as the operand of token r (two tiles), x as the operand of column r
-    bf16x8 cf[2][NKS];
+    const float wend = dt * exp_f(a_end - a);
+    __syncthreads();  // the rows are there; the buffers written next were last read before this
+    if (t0 + CT < n) fetch(t0 + CT);
+    float zg[2][VTW][4];  // the gate of the rows and columns this lane ends with
 #pragma unroll
     for (int mt = 0; mt < 2; ++mt)
 #pragma unroll
-      for (int ks = 0; ks < NKS; ++ks) {
-        const bf16x4 z = {};
-        const bf16* c = xc + (r0 + t0 + min(mt * 16 + r, nt - 1)) * ldx;
-        const int d = ks * 32 + 4 * g;
-        cf[mt][ks] = cat(d < N ? ld4(c + d) : z, d + 16 < N ? ld4(c + d + 16) : z);
-      }
-    bf16x8 xf[VTW];
+      for (int j = 0; j < VTW; ++j)
 #pragma unroll
-    for (int j = 0; j < VTW; ++j) {
-      const int v = (w * VTW + j) * 16 + r;
-#pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int t = (e >> 2) * 16 + 4 * g + (e & 3);
-        xf[j][e] = t < nt && v < V ? xv[(r0 + t0 + t) * ldx + v] : f2bf(0.f);
-      }
-    }
-    __syncthreads();  // B is there; the buffer written next was last read before this
-    // scores transposed: rows s, column t = r -- the operand layout of P
-    f32x4 sc[2][2];  // [s tile][t tile]
-#pragma unroll
-    for (int st = 0; st < 2; ++st)
-#pragma unroll
-      for (int mt = 0; mt < 2; ++mt) sc[st][mt] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int ks = 0; ks < NKS; ++ks)
-#pragma unroll
-      for (int st = 0; st < 2; ++st) {
-        const bf16* bp = B + (st * 16 + r) * LDB + ks * 32 + 4 * g;
-        const bf16x8 bf = cat(ld4(bp), ld4(bp + 16));
-#pragma unroll
-        for (int mt = st; mt < 2; ++mt) sc[st][mt] = mfma16(bf, cf[mt][ks], sc[st][mt]);
-      }
-    f32x4 as[2], ds[2], wv[2];  // a, dt and the state weights of rows s = 16 st + 4 g + i
+        for (int i = 0; i < 4; ++i) {
+          const int t = min(t0 + mt * 16 + 4 * g + i, n - 1), v = min((w * VTW + j) * 16 + r, V - 1);
+          zg[mt][j][i] = bf2f(y[(long)t * p.c.ldy + (long)h * V + v]);
+        }
+    f32x4 as[2], ds[2], wv[2];  // a, dt and the state weights of rows 16 st + 4 g + i
 #pragma unroll
     for (int st = 0; st < 2; ++st)
 #pragma unroll
@@ -663,7 +783,50 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
         ds[st][i] = __shfl(dt, st * 16 + 4 * g + i, 64);
         wv[st][i] = __shfl(wend, st * 16 + 4 * g + i, 64);
       }
-    bf16x8 ph[2], pl[2];
+    // scores transposed (rows s, column t = r: the operand layout of P), and C S
+    f32x4 sc[2][2], o[2][VTW];  // sc[s tile][t tile]
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt) {
+#pragma unroll
+      for (int st = 0; st < 2; ++st) sc[st][mt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < VTW; ++j) o[mt][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks) {
+      const int at = r * LDB + ks * 32 + 4 * g;
+      bf16x8 cf[2], bf[2];
+#pragma unroll
+      for (int q = 0; q < 2; ++q) {
+        cf[q] = cat(ld4(C + at + q * 16 * LDB), ld4(C + at + q * 16 * LDB + 16));
+        bf[q] = cat(ld4(B + at + q * 16 * LDB), ld4(B + at + q * 16 * LDB + 16));
+      }
+      sc[0][0] = mfma16(bf[0], cf[0], sc[0][0]);
+      sc[0][1] = mfma16(bf[0], cf[1], sc[0][1]);
+      sc[1][1] = mfma16(bf[1], cf[1], sc[1][1]);
+#pragma unroll
+      for (int j = 0; j < VTW; ++j) {
+        bf16x8 sh, sl;
+        split8(S[2 * ks][j], S[2 * ks + 1][j], sh, sl);
+#pragma unroll
+        for (int mt = 0; mt < 2; ++mt) {
+          o[mt][j] = mfma16(cf[mt], sh, o[mt][j]);
+          o[mt][j] = mfma16(cf[mt], sl, o[mt][j]);
+        }
+      }
+    }
+    bf16x8 xf[VTW], uh[VTW], ul[VTW];
+#pragma unroll
+    for (int j = 0; j < VTW; ++j) {
+      const bf16* xp = X + (4 * g + (r >> 2)) * LDX + (w * VTW + j) * 16 + 4 * (r & 3);
+      xf[j] = cat(ds_read_tr(xp), ds_read_tr(xp + 16 * LDX));
+      f32x4 u[2];
+#pragma unroll
+      for (int st = 0; st < 2; ++st)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) u[st][i] = bf2f(xf[j][st * 4 + i]) * wv[st][i];
+      split8(u[0], u[1], uh[j], ul[j]);
+    }
 #pragma unroll
     for (int mt = 0; mt < 2; ++mt) {
       const float at = __shfl(a, mt * 16 + r, 64);
@@ -672,54 +835,19 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
       for (int st = 0; st < 2; ++st)
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          pm[st][i] = st * 16 + 4 * g + i <= mt * 16 + r
-                          ? sc[st][mt][i] * ds[st][i] * __builtin_amdgcn_exp2f(1.4426950408889634f * (at - as[st][i])) : 0.f;
-      split8(pm[0], pm[1], ph[mt], pl[mt]);
-    }
-    f32x4 o[2][VTW];
-#pragma unroll
-    for (int mt = 0; mt < 2; ++mt)
-#pragma unroll
-      for (int j = 0; j < VTW; ++j) o[mt][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int ks = 0; ks < NKS; ++ks)
-#pragma unroll
-      for (int j = 0; j < VTW; ++j) {
-        bf16x8 sh, sl;
-        split8(S[2 * ks][j], S[2 * ks + 1][j], sh, sl);
-#pragma unroll
-        for (int mt = 0; mt < 2; ++mt) {
-          o[mt][j] = mfma16(cf[mt][ks], sh, o[mt][j]);
-          o[mt][j] = mfma16(cf[mt][ks], sl, o[mt][j]);
-        }
-      }
-    const float dec = expf(a_end);
-    bf16x8 uh[VTW], ul[VTW];
-#pragma unroll
-    for (int j = 0; j < VTW; ++j) {
-      f32x4 u[2];
-#pragma unroll
-      for (int st = 0; st < 2; ++st)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) u[st][i] = bf2f(xf[j][st * 4 + i]) * wv[st][i];
-      split8(u[0], u[1], uh[j], ul[j]);
-    }
-    // rows t = 16 mt + 4 g + i: the decays of rows s with the same index
-#pragma unroll
-    for (int mt = 0; mt < 2; ++mt)
+          pm[st][i] = st * 16 + 4 * g + i <= mt * 16 + r ? sc[st][mt][i] * ds[st][i] * exp_f(at - as[st][i]) : 0.f;
+      bf16x8 ph, pl;
+      split8(pm[0], pm[1], ph, pl);
+      // rows t = 16 mt + 4 g + i: the decays of rows s with the same index
 #pragma unroll
       for (int j = 0; j < VTW; ++j) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o[mt][j][i] *= __builtin_amdgcn_exp2f(1.4426950408889634f * as[mt][i]);
-        o[mt][j] = mfma16(ph[mt], xf[j], o[mt][j]);
-        o[mt][j] = mfma16(pl[mt], xf[j], o[mt][j]);
-        const int v = (w * VTW + j) * 16 + r;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int t = mt * 16 + 4 * g + i;
-          if (t < nt && v < V) p.raw[(r0 + t0 + t) * p.ldr + (long)h * V + v] = o[mt][j][i] + skip * bf2f(xf[j][mt * 4 + i]);
-        }
+        for (int i = 0; i < 4; ++i) o[mt][j][i] *= exp_f(as[mt][i]);
+        o[mt][j] = mfma16(ph, xf[j], o[mt][j]);
+        o[mt][j] = mfma16(pl, xf[j], o[mt][j]);
       }
+    }
+    const float dec = exp_f(a_end);
 #pragma unroll
     for (int dt2 = 0; dt2 < NT; ++dt2) {
       const bf16* bp = B + (4 * g + (r >> 2)) * LDB + dt2 * 16 + 4 * (r & 3);
@@ -731,6 +859,17 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
         S[dt2][j] = mfma16(bf, ul[j], S[dt2][j]);
       }
     }
+    bf16* out = static_cast<bf16*>(p.out) + (long)(r0 + t0) * p.ldo + (long)h * V;
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt)
+#pragma unroll
+      for (int j = 0; j < VTW; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int t = mt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
+          if (t < nt && v < V)
+            out[(long)t * p.ldo + v] = f2bf((o[mt][j][i] + skip * bf2f(xf[j][mt * 4 + i])) * silu(gain * zg[mt][j][i]));
+        }
   }
 #pragma unroll
   for (int dt = 0; dt < NT; ++dt)
@@ -774,41 +913,58 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(MixOutParams p) {
     for (int c = p.heads * p.V + lane; c < p.out_cols; c += 64) from_f(out + c, 0.f);
 }
 
-// One block per (row, norm group): y silu(z), rms over the group, times weight.
-template <typename T>
+// One block per (row, norm group): rms over the group, times weight.  GATED: the
+// rows are already y silu(z) (bf16, from out itself); else y (fp32) and z.
+template <typename T, bool GATED>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(MixOutParams p) {
   __shared__ float red[16];
   const long row = blockIdx.x;
   const int g = blockIdx.y, W = p.inner / p.groups;
-  const float* y = p.raw + row * p.ldr + (long)g * W;
-  const T* z = static_cast<const T*>(p.z) + row * p.ldz + (long)g * W;
-  constexpr int KEEP = 16;
-  float keep[KEEP];
-  float ss = 0.f;
-  for (int i = 0, c = threadIdx.x; c < W; ++i, c += 256) {
-    const float v = y[c] * silu_x(p.gain * to_f(z[c]));
-    if (i < KEEP) {
+  T* out = static_cast<T*>(p.out) + row * p.ldo + (long)g * W;
+  const float* wt = p.norm + (long)g * W;
+  constexpr int KEEP = 4;  // groups of four columns per thread
+  const bool vec = GATED && W % 4 == 0 && W <= KEEP * 1024 && p.ldo % 4 == 0;
+  if (vec) {
+    f32x4 v[KEEP];
+    float ss = 0.f;
 #pragma unroll
-      for (int j = 0; j < KEEP; ++j)
-        if (j == i) keep[j] = v;
+    for (int i = 0; i < KEEP; ++i) {
+      const int c = (threadIdx.x + i * 256) * 4;
+      v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if constexpr (GATED) {
+        if (c < W) {
+          const bf16x4 x = ld4(reinterpret_cast<const bf16*>(out) + c);
+          v[i] = f32x4{bf2f(x[0]), bf2f(x[1]), bf2f(x[2]), bf2f(x[3])};
+        }
+      }
+      ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
     }
-    ss += v * v;
-  }
-  const float rs = 1.f / sqrtf(block_sum(ss, red) / W + p.eps);
-  T* out = static_cast<T*>(p.out) + row * p.ldo;
-  for (int i = 0, c = threadIdx.x; c < W; ++i, c += 256) {
-    float v = 0.f;
-    if (i < KEEP) {
+    const float rs = rsqrtf(block_sum(ss, red) / W + p.eps);
 #pragma unroll
-      for (int j = 0; j < KEEP; ++j)
-        if (j == i) v = keep[j];
-    } else {
-      v = y[c] * silu_x(p.gain * to_f(z[c]));
+    for (int i = 0; i < KEEP; ++i) {
+      const int c = (threadIdx.x + i * 256) * 4;
+      if constexpr (GATED) {
+        if (c < W) {
+          const f32x4 w = f32x4{wt[c], wt[c + 1], wt[c + 2], wt[c + 3]};
+          const f32x4 o = v[i] * w * rs;
+          st4(reinterpret_cast<bf16*>(out) + c, bf16x4{f2bf(o[0]), f2bf(o[1]), f2bf(o[2]), f2bf(o[3])});
+        }
+      }
     }
-    from_f(out + (long)g * W + c, v * rs * p.norm[(long)g * W + c]);
+  } else {
+    const float* y = p.raw + row * p.ldr + (long)g * W;
+    const T* z = static_cast<const T*>(p.z) + row * p.ldz + (long)g * W;
+    auto value = [&](int c) { return GATED ? to_f(out[c]) : y[c] * silu_x(p.gain * to_f(z[c])); };
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < W; c += 256) {
+      const float v = value(c);
+      ss += v * v;
+    }
+    const float rs = 1.f / sqrtf(block_sum(ss, red) / W + p.eps);
+    for (int c = threadIdx.x; c < W; c += 256) from_f(out + c, value(c) * rs * wt[c]);
   }
   if (g == p.groups - 1)
-    for (int c = p.inner + threadIdx.x; c < p.out_cols; c += 256) from_f(out + c, 0.f);
+    for (int c = p.inner + threadIdx.x; c < p.out_cols; c += 256) from_f(static_cast<T*>(p.out) + row * p.ldo + c, 0.f);
 }
 
 // A loop's pass begins: rows [x | x0] for the projection, and x <- step.
@@ -896,15 +1052,16 @@ extern "C" hipError_t lsd_recur_seq(const RecurParams* p, int delta, int f32, hi
 // Can the chunked kernels take these sizes?
 extern "C" int lsd_chunk_ok(int delta, int D, int V, int groups, int heads) {
   if (D > 128 || V > 128) return 0;
-  return delta ? D % 8 == 0 && V >= 1 : D % 4 == 0 && (heads * V) % 4 == 0;
+  return delta ? D % 8 == 0 && V >= 1 : D % 4 == 0 && V % 4 == 0;
 }
 
 extern "C" hipError_t lsd_conv_silu(const ConvParams* c, const SeqParams* s, int T, bf16* out, long ldo, hipStream_t st) {
   if (T == 0) return hipSuccess;
-  if (c->c0 % 8 == 0 && c->channels % 8 == 0)
-    hipLaunchKernelGGL((conv_silu_kernel<8>), dim3(T, (c->channels + 2047) / 2048), dim3(256), 0, st, *c, *s, out, ldo);
+  if (c->taps <= 4 && c->c0 % 8 == 0 && c->channels % 8 == 0)
+    hipLaunchKernelGGL(conv_silu_kernel, dim3((T + CONV_RUN - 1) / CONV_RUN, (c->channels + 2047) / 2048), dim3(256), 0,
+                       st, *c, *s, T, out, ldo);
   else
-    hipLaunchKernelGGL((conv_silu_kernel<1>), dim3(T, (c->channels + 255) / 256), dim3(256), 0, st, *c, *s, out, ldo);
+    hipLaunchKernelGGL(conv_silu_any_kernel, dim3(T, (c->channels + 255) / 256), dim3(256), 0, st, *c, *s, out, ldo);
   return hipGetLastError();
 }
 
@@ -948,8 +1105,9 @@ extern "C" hipError_t lsd_head_norm_gate(const MixOutParams* p, int f32, hipStre
 extern "C" hipError_t lsd_gated_group_norm(const MixOutParams* p, int f32, hipStream_t st) {
   if (p->T == 0) return hipSuccess;
   const dim3 grid(p->T, p->groups);
-  if (f32) hipLaunchKernelGGL((gated_group_norm_kernel<float>), grid, dim3(256), 0, st, *p);
-  else hipLaunchKernelGGL((gated_group_norm_kernel<bf16>), grid, dim3(256), 0, st, *p);
+  if (f32) hipLaunchKernelGGL((gated_group_norm_kernel<float, false>), grid, dim3(256), 0, st, *p);
+  else if (p->raw) hipLaunchKernelGGL((gated_group_norm_kernel<bf16, false>), grid, dim3(256), 0, st, *p);
+  else hipLaunchKernelGGL((gated_group_norm_kernel<bf16, true>), grid, dim3(256), 0, st, *p);
   return hipGetLastError();
 }
 

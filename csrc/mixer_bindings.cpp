@@ -177,7 +177,10 @@ void group_norm_out(const Tensor& raw, const Tensor& y, int64_t inner, int64_t n
                     double eps, const Tensor& out) {
   const bool f32 = is_f32(y, "y");
   MixOutParams o{};
-  o.raw = raw.data_ptr<float>(); o.ldr = inner; o.T = y.size(0); o.inner = inner; o.groups = norm_groups;
+  if (raw.defined()) {  // else `out` holds y silu(z)
+    o.raw = raw.data_ptr<float>(); o.ldr = inner;
+  }
+  o.T = y.size(0); o.inner = inner; o.groups = norm_groups;
   TORCH_CHECK(norm_groups >= 1 && inner % norm_groups == 0, "norm groups");
   o.z = y.data_ptr(); o.ldz = y.stride(0);
   o.norm = fptr(norm, inner, "norm"); o.eps = (float)eps; o.gain = (float)gain;
@@ -203,14 +206,16 @@ void ssm_seq(Tensor y, Tensor slots, Tensor start, Tensor cu, int64_t heads, int
   p.groups = groups;
   p.v_ch = 0; p.k_ch = inner; p.q_ch = inner + groups * N;
   p.A = fptr(A, heads, "A"); p.dt_bias = fptr(dt_bias, heads, "dt_bias"); p.skip = fptr(skip, heads, "D");
-  auto raw = torch::empty({y.size(0), inner}, y.options().dtype(torch::kFloat32));
-  p.raw = raw.data_ptr<float>(); p.ldr = inner;
+  Tensor raw;
   p.write_ring = single;
   TORCH_CHECK(!single || p.s.B == y.size(0), "ssm_seq: one row per sequence");
   if (chunked) {
     TORCH_CHECK(!f32 && !single && lsd_chunk_ok(0, N, V, groups, heads), "ssm_seq: no chunked kernel");
+    out_rows(p, out, y);
     run_chunks(p, 0, y);
   } else {
+    raw = torch::empty({y.size(0), inner}, y.options().dtype(torch::kFloat32));
+    p.raw = raw.data_ptr<float>(); p.ldr = inner;
     TORCH_CHECK(lsd_recur_block(N, V) > 0, "ssm_seq: no kernel for state size ", N);
     check_hip(lsd_recur_seq(&p, 0, f32, cur_stream()), "ssm_seq");
   }
