@@ -108,7 +108,7 @@ __device__ __forceinline__ f32x4 column_sum(f32x4 v, float (*red)[LV * 4]) {
 // One (sequence, head, LV * 4 columns of the state) per block; thread (dg, lv)
 // holds rows dg + i * 256 / LV of four columns.  Dynamic LDS: q, k, decays [D].
 template <typename T, bool DELTA, int LV, int NR>
-__global__ __launch_bounds__(256, NR <= 8 ? 4 : 3) void recur_seq_kernel(RecurParams p) {
+__global__ __launch_bounds__(256, NR <= 8 ? 3 : 2) void recur_seq_kernel(RecurParams p) {
   constexpr int VB = LV * 4, DG = 256 / LV;
   extern __shared__ float dyn[];
   __shared__ __attribute__((aligned(16))) float red[4][LV * 4];
@@ -126,7 +126,10 @@ __global__ __launch_bounds__(256, NR <= 8 ? 4 : 3) void recur_seq_kernel(RecurPa
   float* Sg = p.S + ((long)slot * p.heads + h) * D * p.Vp + col;
   f32x4 s[NR];
 #pragma unroll
-  for (int i = 0; i < NR; ++i) s[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int i = 0; i < NR; ++i) {
+    s[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (start > 0 && live && dg + i * DG < D) s[i] = *reinterpret_cast<const f32x4*>(Sg + (long)(dg + i * DG) * p.Vp);
+  }
   const float A = p.A[h];
   const float inv_sqrt_d = rsqrtf((float)D);
 
@@ -181,11 +184,6 @@ __global__ __launch_bounds__(256, NR <= 8 ? 4 : 3) void recur_seq_kernel(RecurPa
     } else {
       dt = softplus_x(gl + p.dt_bias[h]);
       a = expf(A * dt);
-    }
-    if (t == 0 && start > 0 && live) {
-#pragma unroll
-      for (int i = 0; i < NR; ++i)
-        if (dg + i * DG < D) s[i] = *reinterpret_cast<const f32x4*>(Sg + (long)(dg + i * DG) * p.Vp);
     }
     __syncthreads();
     f32x4 v = f32x4{vs[lv * 4], vs[lv * 4 + 1], vs[lv * 4 + 2], vs[lv * 4 + 3]};
