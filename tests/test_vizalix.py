@@ -3,7 +3,6 @@ prompts, looped layers, stages, and greedy generation, against the plain model
 of vizalix_oracle.py."""
 from __future__ import annotations
 
-import math
 import random
 
 import pytest
@@ -19,8 +18,6 @@ from llm_sharding_demo_amd.runtime.engine import Engine
 from llm_sharding_demo_amd.runtime.kv_cache import PAGE, PagedCache, layer_cache, pad_up
 
 from . import vizalix_oracle as orc
-
-F64 = torch.float64
 
 
 def model(tmp_path, layers, seed=0, **kw):
