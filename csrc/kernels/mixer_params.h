@@ -41,18 +41,18 @@ struct RecurParams {
   const void* low; long ldl; int gate_off;
   const float* norm; float eps;        // delta: output norm [V]
   const float* skip;                   // Mamba-2: [heads]
-  float* raw; long ldr;                // outputs before norm and gate [rows][heads V], or null:
-  void* out; long ldo; int out_cols;   // normed and gated rows (zeros up to out_cols)
+  float* raw; long ldr;                // delta: outputs before norm and gate [rows][heads V], or null
+  void* out; long ldo; int out_cols;   // delta (raw null): normed and gated rows, zeros up to out_cols;
+                                       // Mamba-2: y silu(z) rows
   int write_ring;                      // single-token portions: this kernel keeps the ring
 };
 
-// Output norms of the unfused forms.
+// Output norms in a launch of their own.
 struct MixOutParams {
   const float* raw; long ldr; int T;
   int heads, V;                        // delta: per (row, head)
   const void* low; long ldl; int gate_off;
-  int inner, groups;                   // Mamba-2: per (row, group), gate z = y[z_col ..]
-  const void* z; long ldz;
+  int inner, groups;                   // Mamba-2: per (row, group), in place
   const float* norm; float eps, gain;
   void* out; long ldo; int out_cols;
 };

@@ -12,7 +12,8 @@
 //    state, pseudo-values and outputs never leave their wave.  fp32 operands
 //    enter the matrix cores as two bf16 terms (three products, 16 bits each).
 //  * conv_tail: keeps the convolution's last inputs after a prompt portion.
-//  * head_norm_gate / gated_group_norm: output norms of the unfused forms.
+//  * head_norm_gate: the delta rule's output norm and gate where a head's values
+//    take several blocks; group_norm: Mamba-2's output norm.
 //
 // State, decays, step sizes, gates of the recurrence and unit norms are fp32.
 #include "common.h"
@@ -227,13 +228,21 @@ __global__ __launch_bounds__(256, NR <= 8 ? 3 : 2) void recur_seq_kernel(RecurPa
     }
     o = column_sum<LV>(o, red);
     if constexpr (!DELTA) o += v * p.skip[h];
-    if (p.raw) {
+    if constexpr (!DELTA) {  // y silu(z): the group norm follows
+      if (dg == 0) {
+        const T* z = static_cast<const T*>(p.c.y) + row * p.c.ldy + (long)h * p.V;
+        T* out = static_cast<T*>(p.out) + row * p.ldo + (long)h * p.V;
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (col + i < p.V) from_f(out + col + i, o[i] * silu_x(p.c.gain * to_f(z[col + i])));
+      }
+    } else if (p.raw) {
       if (dg == 0 && live) {
 #pragma unroll
         for (int i = 0; i < 4; ++i)
           if (col + i < p.V) p.raw[row * p.ldr + (long)h * p.V + col + i] = o[i];
       }
-    } else {  // DELTA, one block holds all of V: norm and gate here
+    } else {  // one block holds all of V: norm and gate here
       float ss = 0.f;
 #pragma unroll
       for (int i = 0; i < 4; ++i) ss += dg == 0 && col + i < p.V ? o[i] * o[i] : 0.f;
@@ -275,7 +284,7 @@ __global__ __launch_bounds__(256) void conv_silu_any_kernel(ConvParams c, SeqPar
 
 // At most four taps, 8 channels per thread, CONV_RUN rows in turn: the taps and
 // the last three inputs stay in registers.
-constexpr int CONV_RUN = 16;
+constexpr int CONV_RUN = 32;
 __global__ __launch_bounds__(256) void conv_silu_kernel(ConvParams c, SeqParams s, int T, bf16* __restrict__ out, long ldo) {
   const int row0 = blockIdx.x * CONV_RUN, row1 = min(T, row0 + CONV_RUN);
   int seq = 0, hi = s.B;  // sequence of row0: last one with cu <= row0
@@ -298,7 +307,23 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvParams c, SeqParams 
   float past[3][8];
   bool fresh = true;
   int end = s.cu[seq + 1];
-  for (int row = row0; row < row1; ++row) {
+  auto emit = [&](const bf16x8& x, int row) {
+    bf16x8 o;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float now = bf2f(x[e]);
+      float v = fmaf(w[0][e], now, bias[e]);
+      v = fmaf(w[1][e], past[0][e], v);
+      v = fmaf(w[2][e], past[1][e], v);
+      v = fmaf(w[3][e], past[2][e], v);
+      past[2][e] = past[1][e];
+      past[1][e] = past[0][e];
+      past[0][e] = now;
+      o[e] = f2bf(silu(v));
+    }
+    st8(out + (long)row * ldo + ch, o);
+  };
+  for (int row = row0; row < row1;) {
     while (row >= end) {
       ++seq;
       end = s.cu[seq + 1];
@@ -317,21 +342,17 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvParams c, SeqParams 
       }
       fresh = false;
     }
-    const bf16x8 x = ld8(y + (long)row * c.ldy);
-    bf16x8 o;
+    if (row + 8 <= min(row1, end)) {  // eight rows of one sequence: their loads together
+      bf16x8 x[8];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const float now = bf2f(x[e]);
-      float v = fmaf(w[0][e], now, bias[e]);
-      v = fmaf(w[1][e], past[0][e], v);
-      v = fmaf(w[2][e], past[1][e], v);
-      v = fmaf(w[3][e], past[2][e], v);
-      past[2][e] = past[1][e];
-      past[1][e] = past[0][e];
-      past[0][e] = now;
-      o[e] = f2bf(silu(v));
+      for (int i = 0; i < 8; ++i) x[i] = ld8(y + (long)(row + i) * c.ldy);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) emit(x[i], row + i);
+      row += 8;
+    } else {
+      emit(ld8(y + (long)row * c.ldy), row);
+      ++row;
     }
-    st8(out + (long)row * ldo + ch, o);
   }
 }
 
@@ -911,55 +932,43 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(MixOutParams p) {
     for (int c = p.heads * p.V + lane; c < p.out_cols; c += 64) from_f(out + c, 0.f);
 }
 
-// One block per (row, norm group): rms over the group, times weight.  GATED: the
-// rows are already y silu(z) (bf16, from out itself); else y (fp32) and z.
-template <typename T, bool GATED>
-__global__ __launch_bounds__(256) void gated_group_norm_kernel(MixOutParams p) {
+// One block per (row, norm group) of rows y silu(z), in place: rms over the
+// group, times weight.
+template <typename T>
+__global__ __launch_bounds__(256) void group_norm_kernel(MixOutParams p) {
   __shared__ float red[16];
   const long row = blockIdx.x;
   const int g = blockIdx.y, W = p.inner / p.groups;
   T* out = static_cast<T*>(p.out) + row * p.ldo + (long)g * W;
   const float* wt = p.norm + (long)g * W;
   constexpr int KEEP = 4;  // groups of four columns per thread
-  const bool vec = GATED && W % 4 == 0 && W <= KEEP * 1024 && p.ldo % 4 == 0;
+  bool vec = false;
+  if constexpr (sizeof(T) == 2) vec = W % 4 == 0 && W <= KEEP * 1024;  // rows are 16-byte aligned
   if (vec) {
-    f32x4 v[KEEP];
+    bf16* ob = reinterpret_cast<bf16*>(out);
+    f32x4 v[KEEP], w[KEEP];
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < KEEP; ++i) {
-      const int c = (threadIdx.x + i * 256) * 4;
-      v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-      if constexpr (GATED) {
-        if (c < W) {
-          const bf16x4 x = ld4(reinterpret_cast<const bf16*>(out) + c);
-          v[i] = f32x4{bf2f(x[0]), bf2f(x[1]), bf2f(x[2]), bf2f(x[3])};
-        }
-      }
+      const int c = min((int)(threadIdx.x + i * 256) * 4, W - 4);
+      const bf16x4 x = ld4(ob + c);
+      w[i] = f32x4{wt[c], wt[c + 1], wt[c + 2], wt[c + 3]};
+      const float live = (threadIdx.x + i * 256) * 4 < W ? 1.f : 0.f;
+      v[i] = f32x4{bf2f(x[0]), bf2f(x[1]), bf2f(x[2]), bf2f(x[3])} * live;
       ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
     }
     const float rs = rsqrtf(block_sum(ss, red) / W + p.eps);
 #pragma unroll
     for (int i = 0; i < KEEP; ++i) {
       const int c = (threadIdx.x + i * 256) * 4;
-      if constexpr (GATED) {
-        if (c < W) {
-          const f32x4 w = f32x4{wt[c], wt[c + 1], wt[c + 2], wt[c + 3]};
-          const f32x4 o = v[i] * w * rs;
-          st4(reinterpret_cast<bf16*>(out) + c, bf16x4{f2bf(o[0]), f2bf(o[1]), f2bf(o[2]), f2bf(o[3])});
-        }
-      }
+      const f32x4 o = v[i] * w[i] * rs;
+      if (c < W) st4(ob + c, bf16x4{f2bf(o[0]), f2bf(o[1]), f2bf(o[2]), f2bf(o[3])});
     }
   } else {
-    const float* y = p.raw + row * p.ldr + (long)g * W;
-    const T* z = static_cast<const T*>(p.z) + row * p.ldz + (long)g * W;
-    auto value = [&](int c) { return GATED ? to_f(out[c]) : y[c] * silu_x(p.gain * to_f(z[c])); };
     float ss = 0.f;
-    for (int c = threadIdx.x; c < W; c += 256) {
-      const float v = value(c);
-      ss += v * v;
-    }
+    for (int c = threadIdx.x; c < W; c += 256) ss += to_f(out[c]) * to_f(out[c]);
     const float rs = 1.f / sqrtf(block_sum(ss, red) / W + p.eps);
-    for (int c = threadIdx.x; c < W; c += 256) from_f(out + c, value(c) * rs * wt[c]);
+    for (int c = threadIdx.x; c < W; c += 256) from_f(out + c, to_f(out[c]) * rs * wt[c]);
   }
   if (g == p.groups - 1)
     for (int c = p.inner + threadIdx.x; c < p.out_cols; c += 256) from_f(static_cast<T*>(p.out) + row * p.ldo + c, 0.f);
@@ -1008,7 +1017,7 @@ extern "C" hipError_t lsd_recur_seq(const RecurParams* p, int delta, int f32, hi
   const int vb = lsd_recur_block(p->D, p->V);
   if (vb == 0) return hipErrorInvalidValue;
   const int nvb = (p->Vp + vb - 1) / vb, dgs = 1024 / vb, nr = (p->D + dgs - 1) / dgs;
-  if (!p->raw && (nvb != 1 || !delta)) return hipErrorInvalidValue;
+  if (delta && !p->raw && nvb != 1) return hipErrorInvalidValue;
   const dim3 grid(p->heads * nvb, p->s.B);
   const size_t lds = 3 * p->D * sizeof(float);
 #define LSD_RS(T, DELTA, LV, NR) \
@@ -1100,12 +1109,11 @@ extern "C" hipError_t lsd_head_norm_gate(const MixOutParams* p, int f32, hipStre
   return hipGetLastError();
 }
 
-extern "C" hipError_t lsd_gated_group_norm(const MixOutParams* p, int f32, hipStream_t st) {
+extern "C" hipError_t lsd_group_norm(const MixOutParams* p, int f32, hipStream_t st) {
   if (p->T == 0) return hipSuccess;
   const dim3 grid(p->T, p->groups);
-  if (f32) hipLaunchKernelGGL((gated_group_norm_kernel<float, false>), grid, dim3(256), 0, st, *p);
-  else if (p->raw) hipLaunchKernelGGL((gated_group_norm_kernel<bf16, false>), grid, dim3(256), 0, st, *p);
-  else hipLaunchKernelGGL((gated_group_norm_kernel<bf16, true>), grid, dim3(256), 0, st, *p);
+  if (f32) hipLaunchKernelGGL((group_norm_kernel<float>), grid, dim3(256), 0, st, *p);
+  else hipLaunchKernelGGL((group_norm_kernel<bf16>), grid, dim3(256), 0, st, *p);
   return hipGetLastError();
 }
 

@@ -29,7 +29,7 @@ hipError_t lsd_conv_silu(const ConvParams* c, const SeqParams* s, int T, lsd_bf1
 hipError_t lsd_recur_chunk(const RecurParams* p, int delta, const lsd_bf16_t* x, long ldx, hipStream_t st);
 hipError_t lsd_conv_tail(const ConvParams* c, const SeqParams* s, int f32, hipStream_t st);
 hipError_t lsd_head_norm_gate(const MixOutParams* p, int f32, hipStream_t st);
-hipError_t lsd_gated_group_norm(const MixOutParams* p, int f32, hipStream_t st);
+hipError_t lsd_group_norm(const MixOutParams* p, int f32, hipStream_t st);
 hipError_t lsd_loop_pack(float* x, const float* x0, const float* step, void* out, int T, int H, int f32, hipStream_t st);
 hipError_t lsd_gelu_mul_f32(const float* y, float* out, int T, int F, long ldo, float s, hipStream_t st);
 hipError_t lsd_rope_append(const RopeAppendParams* p, int f32, hipStream_t st);
@@ -173,22 +173,6 @@ void delta_seq(Tensor y, int64_t c0, int64_t gate_col, Tensor low, int64_t gate_
   if (!single) check_hip(lsd_conv_tail(&p.c, &p.s, f32, cur_stream()), "conv_tail");
 }
 
-void group_norm_out(const Tensor& raw, const Tensor& y, int64_t inner, int64_t norm_groups, const Tensor& norm, double gain,
-                    double eps, const Tensor& out) {
-  const bool f32 = is_f32(y, "y");
-  MixOutParams o{};
-  if (raw.defined()) {  // else `out` holds y silu(z)
-    o.raw = raw.data_ptr<float>(); o.ldr = inner;
-  }
-  o.T = y.size(0); o.inner = inner; o.groups = norm_groups;
-  TORCH_CHECK(norm_groups >= 1 && inner % norm_groups == 0, "norm groups");
-  o.z = y.data_ptr(); o.ldz = y.stride(0);
-  o.norm = fptr(norm, inner, "norm"); o.eps = (float)eps; o.gain = (float)gain;
-  rows_of(out, y.scalar_type(), y.size(0), inner, "out");
-  o.out = out.data_ptr(); o.ldo = out.stride(0); o.out_cols = out.size(1);
-  check_hip(lsd_gated_group_norm(&o, f32, cur_stream()), "gated_group_norm");
-}
-
 // y [T, N]: z | x | B | C | dt.  `chunked`: prompts of bf16 models
 void ssm_seq(Tensor y, Tensor slots, Tensor start, Tensor cu, int64_t heads, int64_t groups, int64_t N, int64_t V,
              int64_t norm_groups, Tensor taps, Tensor bias, Tensor ring, Tensor state, Tensor A, Tensor dt_bias,
@@ -206,20 +190,22 @@ void ssm_seq(Tensor y, Tensor slots, Tensor start, Tensor cu, int64_t heads, int
   p.groups = groups;
   p.v_ch = 0; p.k_ch = inner; p.q_ch = inner + groups * N;
   p.A = fptr(A, heads, "A"); p.dt_bias = fptr(dt_bias, heads, "dt_bias"); p.skip = fptr(skip, heads, "D");
-  Tensor raw;
+  out_rows(p, out, y);
+  TORCH_CHECK(norm_groups >= 1 && inner % norm_groups == 0, "ssm_seq: norm groups");
   p.write_ring = single;
   TORCH_CHECK(!single || p.s.B == y.size(0), "ssm_seq: one row per sequence");
   if (chunked) {
     TORCH_CHECK(!f32 && !single && lsd_chunk_ok(0, N, V, groups, heads), "ssm_seq: no chunked kernel");
-    out_rows(p, out, y);
     run_chunks(p, 0, y);
   } else {
-    raw = torch::empty({y.size(0), inner}, y.options().dtype(torch::kFloat32));
-    p.raw = raw.data_ptr<float>(); p.ldr = inner;
     TORCH_CHECK(lsd_recur_block(N, V) > 0, "ssm_seq: no kernel for state size ", N);
     check_hip(lsd_recur_seq(&p, 0, f32, cur_stream()), "ssm_seq");
   }
-  group_norm_out(raw, y, inner, norm_groups, norm, gain, eps, out);
+  MixOutParams o{};
+  o.T = y.size(0); o.inner = inner; o.groups = norm_groups;
+  o.norm = fptr(norm, inner, "norm"); o.eps = (float)eps;
+  o.out = p.out; o.ldo = p.ldo; o.out_cols = p.out_cols;
+  check_hip(lsd_group_norm(&o, f32, cur_stream()), "group_norm");
   if (!single) check_hip(lsd_conv_tail(&p.c, &p.s, f32, cur_stream()), "conv_tail");
 }
 
