@@ -237,19 +237,21 @@ __device__ __forceinline__ void transpose_groups(u32x4 (&x)[4]) {
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr int VLD = 64 + 8;  // row pitch of 64 staged V columns
 
-// Prompt attention.  8 waves: HP / 4 of them share 16 queries, each owning 4
-// consecutive heads; 32 / HP query groups per block.  Per 32-key tile: scores of
+// Prompt attention.  HP / 4 waves share 16 queries, each owning 4 consecutive
+// heads; a block has at least 4 waves (one or more such groups of queries).  Per
+// 32-key tile: scores of
 // the own heads -> LDS -> barrier -> every wave mixes the scores of all heads
 // into its own four (row 4 g of the product is head g, so lane (r, g) ends with
 // all keys of query r, head g) -> barrier -> softmax in the lane, weights
-// transposed between lane groups and registers, second product per head.
+// transposed between lane groups and registers, second product per head.  Few
+// queries: the keys are split over blockIdx.y, partial outputs combined after.
 template <int DKS, int VT, int HP>
-__global__ __launch_bounds__(512, 1) void talk_prefill_kernel(TalkParams p) {
-  constexpr int TK = 32, HW = HP / 4, QG = 8 / HW;
+__global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_prefill_kernel(TalkParams p) {
+  constexpr int TK = 32, HW = HP / 4, NW = HW > 4 ? HW : 4, QG = NW / HW;
   constexpr int PITCH = HP == 8 ? 8 : HP + 8;  // fp16 scores of one pair
   constexpr int PLANE = TK * 16 * PITCH;
   __shared__ __attribute__((aligned(16))) _Float16 ss[QG * 2 * PLANE];
-  __shared__ __attribute__((aligned(16))) bf16 vst[8][TK * VLD];
+  __shared__ __attribute__((aligned(16))) bf16 vst[NW][TK * VLD];
   const int tile = xcd_remap(blockIdx.x, gridDim.x);
   const int seq = p.tiles[2 * tile], off = p.tiles[2 * tile + 1];
   const int cu = p.s.cu[seq], qlen = p.s.cu[seq + 1] - cu, st = p.s.start[seq];
@@ -281,7 +283,23 @@ __global__ __launch_bounds__(512, 1) void talk_prefill_kernel(TalkParams p) {
   float m = NEG, lsum = 0.f;
   const float two_over = 2.f * LOG2E * p.scale / p.cap;
   const int lo = first_key(st + off, p.window), hi = st + min(off + QG * 16, qlen);
-  const int kt0 = lo / TK, kt1 = (hi + TK - 1) / TK;
+  int kt0 = lo / TK, kt1 = (hi + TK - 1) / TK;
+  if (p.splits > 1) {
+    const int per = (kt1 - kt0 + p.splits - 1) / p.splits;
+    kt0 += blockIdx.y * per;
+    kt1 = min(kt1, kt0 + per);
+  }
+  // 64 columns of the tile's V rows, 16 bytes per lane and 8 rows
+  bf16x8 vr[4];
+  auto load_v = [&](long page, int koff, int kvh, int vh) {
+    const bf16* vp = V + ((page * G + kvh) * PAGE + koff) * vdim + vh * 64;
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      const int row = c * 8 + (lane >> 3), col = (lane & 7) * 8;
+      const bf16x8 z = {};
+      vr[c] = vh * 64 + col < vdim ? ld8(vp + (long)row * vdim + col) : z;
+    }
+  };
 
   for (int kt = kt0; kt < kt1; ++kt) {
     const long page = table[kt * TK / PAGE];
@@ -328,6 +346,7 @@ __global__ __launch_bounds__(512, 1) void talk_prefill_kernel(TalkParams p) {
         *reinterpret_cast<half4*>(s_hi + at) = a;
         *reinterpret_cast<half4*>(s_lo + at) = b;
       }
+    load_v(page, koff, kv[0], 0);  // in flight under the mixing and the softmax
     __syncthreads();
     float e[TK];
 #pragma unroll
@@ -388,17 +407,11 @@ __global__ __launch_bounds__(512, 1) void talk_prefill_kernel(TalkParams p) {
 #pragma unroll
       for (int vh = 0; vh < VT / 4; ++vh) {
         if (vh * 64 >= vdim) continue;
-        const bf16* vp = V + ((page * G + kv[hh]) * PAGE + koff) * vdim + vh * 64;
-        bf16x8 vr[4];
-#pragma unroll
-        for (int c = 0; c < 4; ++c) {
-          const int row = c * 8 + (lane >> 3), col = (lane & 7) * 8;
-          const bf16x8 z = {};
-          vr[c] = vh * 64 + col < vdim ? ld8(vp + (long)row * vdim + col) : z;
-        }
+        if (hh > 0 && vh == 0) load_v(page, koff, kv[hh], 0);
         lds_fence();  // reads of what is staged now are done
 #pragma unroll
         for (int c = 0; c < 4; ++c) st8(vs + (c * 8 + (lane >> 3)) * VLD + (lane & 7) * 8, vr[c]);
+        if ((vh + 1) * 64 < vdim) load_v(page, koff, kv[hh], vh + 1);
         lds_fence();
         const int r0 = 4 * g + (r >> 2);
 #pragma unroll
@@ -416,6 +429,24 @@ __global__ __launch_bounds__(512, 1) void talk_prefill_kernel(TalkParams p) {
         }
       }
     }
+  }
+  if (p.splits > 1) {
+#pragma unroll
+    for (int hh = 0; hh < 4; ++hh) {
+      const int h = hw * 4 + hh;
+      if (h >= H || qi >= qlen) continue;
+      const long pi = ((long)(cu + qi) * H + h) * p.splits + blockIdx.y;
+#pragma unroll
+      for (int di = 0; di < VT; ++di)
+        if (di * 16 < vdim) *reinterpret_cast<f32x4*>(p.part_o + pi * vdim + di * 16 + 4 * g) = o[hh][di];
+    }
+    const int h = hw * 4 + g;
+    if (h < H && qi < qlen) {
+      const long pi = ((long)(cu + qi) * H + h) * p.splits + blockIdx.y;
+      p.part_ml[2 * pi] = m;
+      p.part_ml[2 * pi + 1] = lsum;
+    }
+    return;
   }
   const float inv = 1.f / lsum;
   bf16* out = static_cast<bf16*>(p.out) + (long)(cu + qc) * p.ldo;
@@ -655,7 +686,7 @@ __global__ __launch_bounds__(256, 2) void talk_decode_kernel(TalkParams p) {
     for (int c = H * vdim + threadIdx.x; c < p.out_cols; c += 256) static_cast<bf16*>(p.out)[(long)b * p.ldo + c] = f2bf(0.f);
 }
 
-// One block per (token, head); the last head's also clears the pad columns.
+// One block per (query, head); the last head's also clears the pad columns.
 __global__ __launch_bounds__(64) void talk_combine_kernel(TalkParams p) {
   const int b = blockIdx.x / p.H, h = blockIdx.x % p.H;
   const long pi = (long)blockIdx.x * p.splits;
@@ -684,7 +715,7 @@ extern "C" int lsd_talk_heads(int H, int G, int dim, int vdim, float cap) {
   return H <= 8 ? 8 : H <= 16 ? 16 : 32;
 }
 
-extern "C" int lsd_talk_tile(int hp) { return 16 * (32 / hp); }  // queries of a prefill tile
+extern "C" int lsd_talk_tile(int hp) { return hp == 8 ? 32 : 16; }  // queries of a prefill tile
 
 #define LSD_TK_V(KERNEL, HP, GRID, NT)                                                                   \
   if (p->dim <= 64 && p->vdim <= 64) hipLaunchKernelGGL((KERNEL<2, 4, HP>), GRID, dim3(NT), 0, st, *p); \
@@ -694,13 +725,14 @@ extern "C" int lsd_talk_tile(int hp) { return 16 * (32 / hp); }  // queries of a
 
 extern "C" hipError_t lsd_talk_prefill(const TalkParams* p, int hp, hipStream_t st) {
   if (p->n_tiles == 0) return hipSuccess;
-  const dim3 grid(p->n_tiles);
+  const dim3 grid(p->n_tiles, p->splits);
   switch (hp) {
-    case 8: LSD_TK_V(talk_prefill_kernel, 8, grid, 512) break;
-    case 16: LSD_TK_V(talk_prefill_kernel, 16, grid, 512) break;
+    case 8: LSD_TK_V(talk_prefill_kernel, 8, grid, 256) break;
+    case 16: LSD_TK_V(talk_prefill_kernel, 16, grid, 256) break;
     case 32: LSD_TK_V(talk_prefill_kernel, 32, grid, 512) break;
     default: return hipErrorInvalidValue;
   }
+  if (p->splits > 1) hipLaunchKernelGGL(talk_combine_kernel, dim3(p->T * p->H), dim3(64), 0, st, *p);
   return hipGetLastError();
 }
 

@@ -302,11 +302,24 @@ int frag_of(TalkParams& p, const Tensor& q, const Tensor& frag) {
   return hp;
 }
 
+// fp32 outputs and (maximum, sum) of every key split
+void partials(TalkParams& p, int64_t splits, const Tensor& q, Tensor& po, Tensor& pml) {
+  TORCH_CHECK(splits >= 1 && splits <= 256, "splits");
+  p.splits = splits;
+  if (splits == 1) return;
+  const int64_t n = (int64_t)p.T * p.H * splits;
+  po = torch::empty({n * p.vdim}, q.options().dtype(torch::kFloat32));
+  pml = torch::empty({n * 2}, q.options().dtype(torch::kFloat32));
+  p.part_o = po.data_ptr<float>(); p.part_ml = pml.data_ptr<float>();
+}
+
 // packed ragged queries; tiles [n, 2] = (sequence, first query) of talk_tile(hp) queries
 void talk_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tensor tiles, Tensor slots, Tensor start,
-                  Tensor cu, int64_t window, double scale, double cap, Tensor out) {
+                  Tensor cu, int64_t window, double scale, double cap, int64_t splits, Tensor out) {
   TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, cap, out);
   const int hp = frag_of(p, q, frag);
+  Tensor po, pml;
+  partials(p, splits, q, po, pml);
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2, "tiles must be [n, 2]");
   p.tiles = iptr(tiles, 0, "tiles"); p.n_tiles = tiles.size(0);
   p.s = seqs(slots, start, cu);
@@ -320,15 +333,8 @@ void talk_decode(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tensor
   const int hp = frag_of(p, q, frag);
   TORCH_CHECK(hp >= 16 && 4 * p.G <= hp, "talk_decode: ", p.G, " K / V heads need talk padded to ", 4 * p.G);
   p.slots = iptr(slots, p.T, "slots"); p.pos = iptr(pos, p.T, "pos");
-  TORCH_CHECK(splits >= 1 && splits <= 256, "splits");
-  p.splits = splits;
   Tensor po, pml;
-  if (splits > 1) {
-    const int64_t n = (int64_t)p.T * p.H * splits;
-    po = torch::empty({n * p.vdim}, q.options().dtype(torch::kFloat32));
-    pml = torch::empty({n * 2}, q.options().dtype(torch::kFloat32));
-    p.part_o = po.data_ptr<float>(); p.part_ml = pml.data_ptr<float>();
-  }
+  partials(p, splits, q, po, pml);
   check_hip(lsd_talk_decode(&p, hp, cur_stream()), "talk_decode");
 }
 
@@ -354,7 +360,7 @@ void lsd_register_mixers(pybind11::module& m) {
   m.def("talk_tile", [](int64_t hp) { return lsd_talk_tile((int)hp); });
   m.def("talk_prefill", &talk_prefill, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("frag"),
         py::arg("tiles"), py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("window"), py::arg("scale"),
-        py::arg("cap"), py::arg("out"));
+        py::arg("cap"), py::arg("splits"), py::arg("out"));
   m.def("talk_decode", &talk_decode, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("frag"),
         py::arg("slots"), py::arg("pos"), py::arg("window"), py::arg("scale"), py::arg("cap"), py::arg("splits"),
         py::arg("out"));

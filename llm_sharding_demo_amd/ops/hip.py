@@ -432,8 +432,9 @@ class HipBackend(Backend):
                                    out[s])
             else:
                 tiles = self._query_tiles(mt, self.C.talk_tile(tp.shape[0]), q.device)
+                splits = self.R.talk_prefill_splits(tiles.shape[0], min(window, mt.max_ctx))
                 self.C.talk_prefill(q[s], k, v, kv.table, tp, tiles, mt.seq_slots, mt.q_start, mt.cu_q, window, m.scale,
-                                    cap, out[s])
+                                    cap, splits, out[s])
 
     @staticmethod
     def _query_tiles(meta, rows: int, device):

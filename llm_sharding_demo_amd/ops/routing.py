@@ -130,6 +130,8 @@ class Routing:
     # decode attention with mixed heads: blocks a launch aims for, at least two
     # 64-key tiles each
     talk_target: int = 512
+    # ... and prompt attention with few query tiles
+    talk_prefill_target: int = 512
     # -- norms / head ------------------------------------------------------
     # one wave per row from norm_wave_min rows (prefill 32 K x 1600 97.7 ->
     # 53.7 us; r5_normwave.log) and from norm_wave_narrow_min rows when H <=
@@ -300,6 +302,11 @@ class Routing:
         """Context splits of a decode attention launch with mixed heads (one
         block holds all heads of a token, 64 keys a step)."""
         return max(1, min(math.ceil(self.talk_target / B), math.ceil((keys + 63) / 128), 64))
+
+    def talk_prefill_splits(self, tiles: int, keys: int) -> int:
+        """Key splits of a prompt attention launch with mixed heads: few query
+        tiles over long contexts, at least four 32-key tiles each."""
+        return max(1, min(self.talk_prefill_target // max(1, tiles), keys // 128, 16))
 
     def attn_splits(self, B: int, nh: int, n_kv: int, hd: int, max_ctx: int) -> int:
         """Context splits of a decode attention launch (a graph-captured

@@ -134,13 +134,13 @@ def test_attention_plain(C, H, G, D, V, dt):
 
 
 @pytest.mark.parametrize("H,G,D,V", SIZES)
-@pytest.mark.parametrize("window", [1 << 30, 67, 1, 32])
-def test_attention_prefill(C, H, G, D, V, window):
+@pytest.mark.parametrize("window,splits", [(1 << 30, 1), (67, 1), (1, 1), (32, 1), (1 << 30, 3), (67, 2), (5, 4)])
+def test_attention_prefill(C, H, G, D, V, window, splits):
     b = Batch((1, 0, 75), (2, 70, 2), (0, 130, 33))
     q, K, Vp, table, talk, want, out, scale, cap = attention_case(H, G, D, V, BF, b, window)
     hp = C.talk_heads(H, G, up(D, 32), up(V, 16), cap)
     C.talk_prefill(q, K, Vp, table, frag(talk, hp), b.tiles(C.talk_tile(hp)), b.slots, b.start, b.cu, window, scale, cap,
-                   out)
+                   splits, out)
     assert err(unpad(out, H, V), want) < 3e-2
 
 
@@ -178,7 +178,7 @@ def test_attention_window_edges(C, window):
             outs = [out, out.clone(), out.clone()]
             C.talk_plain(q, K, Vp, table, b.tslot, b.tpos, cuda(eye, F32), window, scale, cap, outs[0])
             C.talk_prefill(q, K, Vp, table, frag(eye, hp), b.tiles(C.talk_tile(hp)), b.slots, b.start, b.cu, window,
-                           scale, cap, outs[1])
+                           scale, cap, 2, outs[1])
             C.talk_decode(q, K, Vp, table, frag(eye, 16), b.slots, b.tpos, window, scale, cap, 2, outs[2])
             for o in outs:
                 assert (float(o[0, : H * V].float().min()) > 10) == seen, (pos, key, window)
@@ -192,7 +192,7 @@ def test_attention_head_mixing(C):
     q, K, Vp, table, _, _, out, scale, cap = attention_case(H, G, D, V, BF, b, 1 << 30)
     perm = torch.roll(torch.eye(H), 1, 0)
     hp = C.talk_heads(H, G, D, V, cap)
-    rest = (b.slots, b.start, b.cu, 1 << 30, scale, cap)
+    rest = (b.slots, b.start, b.cu, 1 << 30, scale, cap, 1)
     C.talk_prefill(q, K, Vp, table, frag(perm, hp), b.tiles(C.talk_tile(hp)), *rest, out)
     other = torch.empty_like(out)
     C.talk_plain(q, K, Vp, table, b.tslot, b.tpos, cuda(perm, F32), 1 << 30, scale, cap, other)
