@@ -411,9 +411,9 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
   constexpr float RANGE = 80.f;
   __shared__ __attribute__((aligned(16))) bf16 kt_h[CT * LDD], kt_l[CT * LDD], qt_h[CT * LDD], qt_l[CT * LDD];
   __shared__ __attribute__((aligned(16))) bf16 kc_h[CT * LDD], kc_l[CT * LDD];     // columns k_s e^{G_0 - G_s}
-  __shared__ __attribute__((aligned(16))) bf16 kh_h[DP * LDT], kh_l[DP * LDT];     // K^ transposed [d][s]
+  __shared__ __attribute__((aligned(16))) bf16 kh_h[CT * LDD], kh_l[CT * LDD];     // K^
   __shared__ __attribute__((aligned(16))) float Gs[CT][DP], Ks[CT][DP], Qs[CT][DP];
-  __shared__ __attribute__((aligned(16))) float e0[DP], er[DP];
+  __shared__ __attribute__((aligned(16))) float e0[DP], s0[DP], er[DP], tot[4][DP], dtb[DP];
   __shared__ __attribute__((aligned(16))) bf16 tm_h[CT * LDT], tm_l[CT * LDT], pm_h[CT * LDT], pm_l[CT * LDT];
   __shared__ float betas[CT], red[4][CT];
   __shared__ int bad[DP], nbad;
@@ -445,10 +445,8 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
   // element work: token tid / 16, channels 8 (tid % 16) ..
   const int et = tid >> 4, ed = (tid & 15) * 8;
   const bool elive = ed < D;  // D % 8 == 0
-  float dtb[8] = {};
-  if (elive)
-#pragma unroll
-    for (int e = 0; e < 8; ++e) dtb[e] = p.dt_bias[(long)h * D + ed + e];
+  for (int d = tid; d < DP; d += 256) dtb[d] = d < D ? p.dt_bias[(long)h * D + d] : 0.f;
+  __syncthreads();
 
   // rows of the next chunk, in flight under this one
   bf16x8 xq, xk, xl;
@@ -476,7 +474,7 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         k8[e] = bf2f(xk[e]);
         nq = fmaf(q8[e], q8[e], nq);
         nk = fmaf(k8[e], k8[e], nk);
-        lg[e] = tlive ? A * softplus_f(gain * bf2f(xl[e]) + dtb[e]) : 0.f;
+        lg[e] = tlive ? A * softplus_f(gain * bf2f(xl[e]) + dtb[ed + e]) : 0.f;
       }
 #pragma unroll
       for (int off = 1; off < 16; off <<= 1) {
@@ -490,59 +488,70 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         k8[e] *= ik;
       }
     }
-    // values and gates of the chunk in the accumulator layout (tokens 4 g + i, columns r)
-    f32x4 vals[VTW], gates[VTW];
+    // log decays summed over the tokens: within the wave's four by lanes, across waves by LDS
+    float pre[8];
 #pragma unroll
-    for (int j = 0; j < VTW; ++j)
+    for (int e = 0; e < 8; ++e) {
+      pre[e] = lg[e];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = 4 * g + i, v = (w * VTW + j) * 16 + r;
-        const bool live = t < nt && v < V;
-        const long at = r0 + t0 + min(t, nt - 1);
-        vals[j][i] = live ? bf2f(x[at * ldx + p.v_ch + (long)h * V + v]) : 0.f;
-        gates[j][i] = live ? bf2f(low[at * p.ldl + p.gate_off + (long)h * V + v]) : 0.f;
+      for (int off = 16; off < 64; off <<= 1) {
+        const float u = __shfl_up(pre[e], off, 64);
+        if (lane >= off) pre[e] += u;
       }
+    }
     if (ed < DP) {
-      *reinterpret_cast<f32x4*>(&Gs[et][ed]) = f32x4{lg[0], lg[1], lg[2], lg[3]};
-      *reinterpret_cast<f32x4*>(&Gs[et][ed + 4]) = f32x4{lg[4], lg[5], lg[6], lg[7]};
+      if (lane >= 48) {
+        *reinterpret_cast<f32x4*>(&tot[w][ed]) = f32x4{pre[0], pre[1], pre[2], pre[3]};
+        *reinterpret_cast<f32x4*>(&tot[w][ed + 4]) = f32x4{pre[4], pre[5], pre[6], pre[7]};
+      }
+      if (et == 0) {
+        *reinterpret_cast<f32x4*>(&e0[ed]) = f32x4{lg[0], lg[1], lg[2], lg[3]};
+        *reinterpret_cast<f32x4*>(&e0[ed + 4]) = f32x4{lg[4], lg[5], lg[6], lg[7]};
+      }
     }
     if (tid < CT) betas[tid] = tid < nt ? sigmoid_x(gain * rb) : 0.f;
     if (t0 + CT < n) fetch(t0 + CT);
     if (tid == 0) nbad = 0;
     __syncthreads();
-    f32x4 g0[2] = {}, gt[2] = {}, gc[2] = {};
     if (ed < DP) {
-      g0[0] = *reinterpret_cast<const f32x4*>(&Gs[0][ed]);
-      g0[1] = *reinterpret_cast<const f32x4*>(&Gs[0][ed + 4]);
-#pragma unroll 4
-      for (int s = 0; s < CT; ++s)
+      float kt[8], qt[8], kc[8], kf[8], gt[8];
+      bool wides = false;
 #pragma unroll
-        for (int q = 0; q < 2; ++q) {
-          const f32x4 v = *reinterpret_cast<const f32x4*>(&Gs[s][ed + 4 * q]);
-          gc[q] += v;
-          if (s == et) gt[q] = gc[q];
-        }
-    }
-    __syncthreads();  // the log decays have been read: Gs takes their sums
-    if (ed < DP) {
-      float kt[8], qt[8], kc[8], kf[8];
+      for (int hf = 0; hf < 2; ++hf) {
+        const f32x4 g0 = *reinterpret_cast<const f32x4*>(&e0[ed + 4 * hf]);
+        f32x4 base = {0.f, 0.f, 0.f, 0.f}, all = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const float G0 = g0[e >> 2][e & 3], Gt = gt[e >> 2][e & 3], Gc = gc[e >> 2][e & 3];
-        const float E = exp_f(Gt - G0);
-        const bool wide = G0 - Gc > RANGE;
-        kt[e] = k8[e] * E;
-        qt[e] = q8[e] * E;
-        kc[e] = wide ? 0.f : k8[e] * exp_f(G0 - Gt);
-        kf[e] = k8[e] * exp_f(Gc - Gt);
-        if (et == 0) {
-          e0[ed + e] = exp_f(G0);
-          er[ed + e] = exp_f(Gc - G0);
-          if (wide) bad[atomicAdd(&nbad, 1)] = ed + e;
+        for (int q = 0; q < 4; ++q) {
+          const f32x4 v = *reinterpret_cast<const f32x4*>(&tot[q][ed + 4 * hf]);
+          if (q < w) base += v;  // wave-uniform
+          all += v;
         }
-        Gs[et][ed + e] = Gt;
-        Ks[et][ed + e] = k8[e];
-        Qs[et][ed + e] = q8[e];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int e = 4 * hf + i;
+          const float G0 = g0[i], Gt = base[i] + pre[e], Gc = all[i];
+          const float E = exp_f(Gt - G0);
+          const bool wide = G0 - Gc > RANGE;
+          gt[e] = Gt;
+          kt[e] = k8[e] * E;
+          qt[e] = q8[e] * E;
+          kc[e] = wide ? 0.f : k8[e] * exp_f(G0 - Gt);
+          kf[e] = k8[e] * exp_f(Gc - Gt);
+          wides |= wide;
+          if (et == 15) {
+            s0[ed + e] = exp_f(G0);
+            er[ed + e] = exp_f(Gc - G0);
+            if (wide) bad[atomicAdd(&nbad, 1)] = ed + e;
+          }
+        }
+      }
+      if (wides) {  // the same channels for every token
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          Gs[et][ed + e] = gt[e];
+          Ks[et][ed + e] = k8[e];
+          Qs[et][ed + e] = q8[e];
+        }
       }
       auto put = [&](bf16* hp, bf16* lp, const float* v) {
         bf16x8 a, c;
@@ -557,14 +566,21 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
       put(kt_h, kt_l, kt);
       put(qt_h, qt_l, qt);
       put(kc_h, kc_l, kc);
-#pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const bf16 a = f2bf(kf[e]);
-        kh_h[(ed + e) * LDT + et] = a;
-        kh_l[(ed + e) * LDT + et] = f2bf(kf[e] - bf2f(a));
-      }
+      put(kh_h, kh_l, kf);
     }
     __syncthreads();
+    // values and gates of the chunk in the accumulator layout (tokens 4 g + i, columns r)
+    f32x4 vals[VTW], gates[VTW];
+#pragma unroll
+    for (int j = 0; j < VTW; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 4 * g + i, v = (w * VTW + j) * 16 + r;
+        const bool live = t < nt && v < V;
+        const long at = r0 + t0 + min(t, nt - 1);
+        vals[j][i] = live ? bf2f(x[at * ldx + p.v_ch + (long)h * V + v]) : 0.f;
+        gates[j][i] = live ? bf2f(low[at * p.ldl + p.gate_off + (long)h * V + v]) : 0.f;
+      }
     // operand of row r: k-slots (g, j) <-> d = 32 ks + 4 g + j, 32 ks + 16 + 4 g + (j - 4)
     auto opnd = [&](const bf16* a, int ks) {
       return cat(ld4(a + r * LDD + ks * 32 + 4 * g), ld4(a + r * LDD + ks * 32 + 16 + 4 * g));
@@ -629,8 +645,8 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
     for (int j = 0; j < VTW; ++j) ks_acc[j] = o[j] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int ks = 0; ks < DKS; ++ks) {
-      const f32x4 da = *reinterpret_cast<const f32x4*>(&e0[ks * 32 + 4 * g]);
-      const f32x4 db = *reinterpret_cast<const f32x4*>(&e0[ks * 32 + 16 + 4 * g]);
+      const f32x4 da = *reinterpret_cast<const f32x4*>(&s0[ks * 32 + 4 * g]);
+      const f32x4 db = *reinterpret_cast<const f32x4*>(&s0[ks * 32 + 16 + 4 * g]);
       const bf16x8 kah = opnd(kt_h, ks), kal = opnd(kt_l, ks), qah = opnd(qt_h, ks), qal = opnd(qt_l, ks);
 #pragma unroll
       for (int j = 0; j < VTW; ++j) {
@@ -668,7 +684,8 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       const f32x4 dec = *reinterpret_cast<const f32x4*>(&er[dt * 16 + 4 * g]);
-      const bf16x4 ah = ld4(kh_h + (dt * 16 + r) * LDT + 4 * g), al = ld4(kh_l + (dt * 16 + r) * LDT + 4 * g);
+      const int at = (4 * g + (r >> 2)) * LDD + dt * 16 + 4 * (r & 3);
+      const bf16x4 ah = ds_read_tr(kh_h + at), al = ds_read_tr(kh_l + at);
 #pragma unroll
       for (int j = 0; j < VTW; ++j) S[dt][j] = mfma3s(ah, al, uh[j], ul[j], S[dt][j] * dec);
     }
