@@ -182,6 +182,11 @@ __global__ __launch_bounds__(256) void talk_plain_kernel(TalkParams p) {
 
 typedef _Float16 half8 __attribute__((ext_vector_type(8)));
 typedef _Float16 half4 __attribute__((ext_vector_type(4)));
+typedef _Float16 half2 __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ half2 pack_half(float a, float b) {  // rounds towards zero
+  const auto h = __builtin_amdgcn_cvt_pkrtz(a, b);
+  return __builtin_bit_cast(half2, h);
+}
 
 __device__ __forceinline__ f32x4 mfma_f16(half8 a, half8 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0);
@@ -207,16 +212,11 @@ __device__ __forceinline__ float capped(float raw, float two_over, float cap) {
 
 // Two bf16 terms of eight weights
 __device__ __forceinline__ void split_p(const float* a, const float* b, u32x4& hi, u32x4& lo) {
-  bf16x8 h, l;
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    h[j] = f2bf(a[j]);
-    l[j] = f2bf(a[j] - bf2f(h[j]));
-    h[4 + j] = f2bf(b[j]);
-    l[4 + j] = f2bf(b[j] - bf2f(h[4 + j]));
-  }
-  hi = __builtin_bit_cast(u32x4, h);
-  lo = __builtin_bit_cast(u32x4, l);
+  const bf16x4 ha = pack4(f32x4{a[0], a[1], a[2], a[3]}), hb = pack4(f32x4{b[0], b[1], b[2], b[3]});
+  const bf16x4 la = pack4(f32x4{a[0] - bf2f(ha[0]), a[1] - bf2f(ha[1]), a[2] - bf2f(ha[2]), a[3] - bf2f(ha[3])});
+  const bf16x4 lb = pack4(f32x4{b[0] - bf2f(hb[0]), b[1] - bf2f(hb[1]), b[2] - bf2f(hb[2]), b[3] - bf2f(hb[3])});
+  hi = __builtin_bit_cast(u32x4, (bf16x8{ha[0], ha[1], ha[2], ha[3], hb[0], hb[1], hb[2], hb[3]}));
+  lo = __builtin_bit_cast(u32x4, (bf16x8{la[0], la[1], la[2], la[3], lb[0], lb[1], lb[2], lb[3]}));
 }
 
 // x[k] of lane group g  ->  x[g] of lane group k (groups of 16 lanes)
@@ -337,10 +337,13 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
       for (int i = 0; i < 4; ++i) {
         half4 a, b;
 #pragma unroll
-        for (int hh = 0; hh < 4; ++hh) {
-          const float c = capped(s[hh][ni][i], two_over, p.cap);
-          a[hh] = (_Float16)c;
-          b[hh] = (_Float16)(c - (float)a[hh]);
+        for (int hh = 0; hh < 4; hh += 2) {  // the remainder makes up for the truncated first term
+          const float c = capped(s[hh][ni][i], two_over, p.cap), d = capped(s[hh + 1][ni][i], two_over, p.cap);
+          const half2 u = pack_half(c, d), v = pack_half(c - (float)u[0], d - (float)u[1]);
+          a[hh] = u[0];
+          a[hh + 1] = u[1];
+          b[hh] = v[0];
+          b[hh + 1] = v[1];
         }
         const int at = ((ni * 16 + 4 * g + i) * 16 + r) * PITCH + hw * 4;
         *reinterpret_cast<half4*>(s_hi + at) = a;

@@ -186,6 +186,14 @@ __device__ __forceinline__ float dot8(bf16x8 a, bf16x8 b, float acc) {
   return acc;
 }
 
+// Two values narrowed by one instruction (element-wise conversions take three)
+typedef float f32x2 __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ bf16x2 pack2(float a, float b) { return __builtin_convertvector((f32x2{a, b}), bf16x2); }
+__device__ __forceinline__ bf16x4 pack4(f32x4 v) {
+  const bf16x2 a = pack2(v[0], v[1]), b = pack2(v[2], v[3]);
+  return bf16x4{a[0], a[1], b[0], b[1]};
+}
+
 // gelu_new (tanh approximation) -- [tf5.15] activations.py:59-66
 //   0.5 x (1 + tanh(u)) = x * sigmoid(2u) = x / (1 + exp(-2u)),
 //   u = sqrt(2/pi) (x + 0.044715 x^3)

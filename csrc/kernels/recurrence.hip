@@ -373,9 +373,9 @@ __device__ __forceinline__ void lds_fence() {
   __builtin_amdgcn_wave_barrier();
 }
 
-__device__ __forceinline__ bf16x4 hi4(f32x4 v) { return bf16x4{f2bf(v[0]), f2bf(v[1]), f2bf(v[2]), f2bf(v[3])}; }
+__device__ __forceinline__ bf16x4 hi4(f32x4 v) { return pack4(v); }
 __device__ __forceinline__ bf16x4 lo4(f32x4 v, bf16x4 h) {
-  return bf16x4{f2bf(v[0] - bf2f(h[0])), f2bf(v[1] - bf2f(h[1])), f2bf(v[2] - bf2f(h[2])), f2bf(v[3] - bf2f(h[3]))};
+  return pack4(f32x4{v[0] - bf2f(h[0]), v[1] - bf2f(h[1]), v[2] - bf2f(h[2]), v[3] - bf2f(h[3])});
 }
 __device__ __forceinline__ bf16x8 cat(bf16x4 a, bf16x4 b) { return bf16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]}; }
 // two bf16 terms of eight values (two accumulator tiles: k-slots 4 g + j and 16 + 4 g + j)
@@ -425,8 +425,15 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
   if (n <= 0) return;
   float* Sg = p.S + ((long)slot * p.heads + h) * D * p.Vp;
   const float A = p.A[h], gain = p.c.gain;
-  const bf16* y = static_cast<const bf16*>(p.c.y);
-  const bf16* low = static_cast<const bf16*>(p.low);
+  // uniform bases of the sequence's rows; offsets within a chunk are 32-bit
+  const int ldxi = (int)ldx, ldl = (int)p.ldl, ldo = (int)p.ldo, ldy = (int)p.c.ldy;
+  const bf16* yb = static_cast<const bf16*>(p.c.y) + r0 * p.c.ldy + p.gate_col + h;
+  const bf16* xqb = x + r0 * ldx + p.q_ch + kh * D;
+  const bf16* xkb = x + r0 * ldx + p.k_ch + kh * D;
+  const bf16* xvb = x + r0 * ldx + p.v_ch + (long)h * V;
+  const bf16* lowb = static_cast<const bf16*>(p.low) + r0 * p.ldl + (long)h * D;
+  const bf16* gateb = static_cast<const bf16*>(p.low) + r0 * p.ldl + p.gate_off + (long)h * V;
+  bf16* outb = static_cast<bf16*>(p.out) + r0 * p.ldo;
 
   // state: rows d = 16 dt + 4 g + i, columns v = 16 (w VTW + j) + r
   f32x4 S[DT][VTW];
@@ -439,6 +446,7 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
         S[dt][j][i] = start > 0 && d < D && v < V ? Sg[(long)d * p.Vp + v] : 0.f;
       }
+  const float inv_sqrt_d = rsqrtf((float)D);
   float nrm[VTW];
 #pragma unroll
   for (int j = 0; j < VTW; ++j) nrm[j] = p.norm[min((w * VTW + j) * 16 + r, V - 1)];
@@ -454,16 +462,15 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
   auto fetch = [&](int t0) {
     const bf16x8 z = {};
     const bool live = t0 + et < n && elive;
-    const long row = r0 + t0 + et;
-    xq = live ? ld8(x + row * ldx + p.q_ch + kh * D + ed) : z;
-    xk = live ? ld8(x + row * ldx + p.k_ch + kh * D + ed) : z;
-    xl = live ? ld8(low + row * p.ldl + (long)h * D + ed) : z;
-    if (tid < CT) rb = t0 + tid < n ? bf2f(y[(r0 + t0 + tid) * p.c.ldy + p.gate_col + h]) : 0.f;
+    const int ox = et * ldxi + ed, ol = et * ldl + ed;
+    xq = live ? ld8(xqb + (long)t0 * ldx + ox) : z;
+    xk = live ? ld8(xkb + (long)t0 * ldx + ox) : z;
+    xl = live ? ld8(lowb + (long)t0 * p.ldl + ol) : z;
+    if (tid < CT) rb = t0 + tid < n ? bf2f((yb + (long)t0 * p.c.ldy)[tid * ldy]) : 0.f;
   };
   fetch(0);
   for (int t0 = 0; t0 < n; t0 += CT) {
     const int nt = min(CT, n - t0);
-    const long row = r0 + t0 + min(et, nt - 1);
     const bool tlive = et < nt && elive;
     float q8[8], k8[8], lg[8];
     {
@@ -481,7 +488,7 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         nq += wave_xchg_n(nq, off);
         nk += wave_xchg_n(nk, off);
       }
-      const float iq = rsqrtf((float)D) / sqrtf(nq + UNIT_EPS), ik = 1.f / sqrtf(nk + UNIT_EPS);
+      const float iq = inv_sqrt_d * rsqrtf(nq + UNIT_EPS), ik = rsqrtf(nk + UNIT_EPS);
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         q8[e] *= iq;
@@ -555,11 +562,7 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
       }
       auto put = [&](bf16* hp, bf16* lp, const float* v) {
         bf16x8 a, c;
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          a[e] = f2bf(v[e]);
-          c[e] = f2bf(v[e] - bf2f(a[e]));
-        }
+        split8(f32x4{v[0], v[1], v[2], v[3]}, f32x4{v[4], v[5], v[6], v[7]}, a, c);
         st8(hp + et * LDD + ed, a);
         st8(lp + et * LDD + ed, c);
       };
@@ -577,9 +580,9 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
       for (int i = 0; i < 4; ++i) {
         const int t = 4 * g + i, v = (w * VTW + j) * 16 + r;
         const bool live = t < nt && v < V;
-        const long at = r0 + t0 + min(t, nt - 1);
-        vals[j][i] = live ? bf2f(x[at * ldx + p.v_ch + (long)h * V + v]) : 0.f;
-        gates[j][i] = live ? bf2f(low[at * p.ldl + p.gate_off + (long)h * V + v]) : 0.f;
+        const int tc = min(t, nt - 1), vc = min(v, V - 1);
+        vals[j][i] = live ? bf2f((xvb + (long)t0 * ldx)[tc * ldxi + vc]) : 0.f;
+        gates[j][i] = bf2f((gateb + (long)t0 * p.ldl)[tc * ldl + vc]);
       }
     // operand of row r: k-slots (g, j) <-> d = 32 ks + 4 g + j, 32 ks + 16 + 4 g + (j - 4)
     auto opnd = [&](const bf16* a, int ks) {
@@ -645,6 +648,7 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
     for (int j = 0; j < VTW; ++j) ks_acc[j] = o[j] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int ks = 0; ks < DKS; ++ks) {
+      if constexpr (VTW > 1) asm volatile("" ::: "memory");  // operands of one step at a time
       const f32x4 da = *reinterpret_cast<const f32x4*>(&s0[ks * 32 + 4 * g]);
       const f32x4 db = *reinterpret_cast<const f32x4*>(&s0[ks * 32 + 16 + 4 * g]);
       const bf16x8 kah = opnd(kt_h, ks), kal = opnd(kt_l, ks), qah = opnd(qt_h, ks), qal = opnd(qt_l, ks);
@@ -690,24 +694,23 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
       for (int j = 0; j < VTW; ++j) S[dt][j] = mfma3s(ah, al, uh[j], ul[j], S[dt][j] * dec);
     }
     __syncthreads();
-    bf16* out = static_cast<bf16*>(p.out);
+    bf16* out = outb + (long)t0 * p.ldo;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int t = 4 * g + i;
       if (t >= nt) continue;
-      const long orow = r0 + t0 + t;
       const float rs = rsqrtf((red[0][t] + red[1][t] + red[2][t] + red[3][t]) / V + p.eps);
 #pragma unroll
       for (int j = 0; j < VTW; ++j) {
         const int v = (w * VTW + j) * 16 + r;
         if (v >= V) continue;
-        out[orow * p.ldo + (long)h * V + v] =
+        out[t * ldo + h * V + v] =
             f2bf(o[j][i] * rs * nrm[j] * __builtin_amdgcn_rcpf(1.f + exp_f(-gain * gates[j][i])));
       }
     }
     if (h == p.heads - 1)
       for (int c = p.heads * V + (tid & 15); c < p.out_cols; c += 16)
-        if (et < nt) out[row * p.ldo + c] = f2bf(0.f);
+        if (et < nt) out[et * ldo + c] = f2bf(0.f);
   }
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
@@ -739,6 +742,7 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
   float* Sg = p.S + ((long)slot * p.heads + h) * N * p.Vp;
   const float A = p.A[h], gain = p.c.gain, skip = p.skip[h], dtb = p.dt_bias[h];
   const bf16* y = static_cast<const bf16*>(p.c.y) + (long)r0 * p.c.ldy;
+  const int ldxi = (int)ldx, ldy = (int)p.c.ldy, ldo = (int)p.ldo;  // offsets within a chunk are 32-bit
   const bf16* xb = x + r0 * ldx + p.k_ch + kg * N;
   const bf16* xc = x + r0 * ldx + p.q_ch + kg * N;
   const bf16* xv = x + r0 * ldx + p.v_ch + (long)h * V;
@@ -763,13 +767,13 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
     for (int q = 0; q < NB; ++q) {
       const int c = tid + q * 256, t = c / (NP / 4), d = (c % (NP / 4)) * 4;
       const bool live = t0 + t < n && d < N;
-      rb[q] = live ? ld4(xb + (t0 + t) * ldx + d) : z;
-      rc[q] = live ? ld4(xc + (t0 + t) * ldx + d) : z;
+      rb[q] = live ? ld4(xb + (long)t0 * ldx + t * ldxi + d) : z;
+      rc[q] = live ? ld4(xc + (long)t0 * ldx + t * ldxi + d) : z;
     }
 #pragma unroll
     for (int q = 0; q < NX; ++q) {
       const int c = tid + q * 256, t = c / (VP / 4), v = (c % (VP / 4)) * 4;
-      rx[q] = t0 + t < n && v < V ? ld4(xv + (t0 + t) * ldx + v) : z;
+      rx[q] = t0 + t < n && v < V ? ld4(xv + (long)t0 * ldx + t * ldxi + v) : z;
     }
     rdt = t0 + tl < n ? bf2f(y[(long)(t0 + tl) * p.c.ldy + p.gate_col + h]) : 0.f;
   };
@@ -807,8 +811,8 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
       for (int j = 0; j < VTW; ++j)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const int t = min(t0 + mt * 16 + 4 * g + i, n - 1), v = min((w * VTW + j) * 16 + r, V - 1);
-          zg[mt][j][i] = bf2f(y[(long)t * p.c.ldy + (long)h * V + v]);
+          const int t = min(mt * 16 + 4 * g + i, nt - 1), v = min((w * VTW + j) * 16 + r, V - 1);
+          zg[mt][j][i] = bf2f((y + (long)t0 * p.c.ldy + (long)h * V)[t * ldy + v]);
         }
     f32x4 as[2], ds[2], wv[2];  // a, dt and the state weights of rows 16 st + 4 g + i
 #pragma unroll
@@ -904,7 +908,7 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
         for (int i = 0; i < 4; ++i) {
           const int t = mt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
           if (t < nt && v < V)
-            out[(long)t * p.ldo + v] = f2bf((o[mt][j][i] + skip * bf2f(xf[j][mt * 4 + i])) * silu(gain * zg[mt][j][i]));
+            out[t * ldo + v] = f2bf((o[mt][j][i] + skip * bf2f(xf[j][mt * 4 + i])) * silu(gain * zg[mt][j][i]));
         }
   }
 #pragma unroll
