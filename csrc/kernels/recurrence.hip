@@ -444,7 +444,7 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
-        S[dt][j][i] = start > 0 && d < D && v < V ? Sg[(long)d * p.Vp + v] : 0.f;
+        S[dt][j][i] = start > 0 && d < D && v < V ? Sg[d * p.Vp + v] : 0.f;
       }
   const float inv_sqrt_d = rsqrtf((float)D);
   float nrm[VTW];
@@ -460,13 +460,13 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
   bf16x8 xq, xk, xl;
   float rb = 0.f;
   auto fetch = [&](int t0) {
-    const bf16x8 z = {};
-    const bool live = t0 + et < n && elive;
-    const int ox = et * ldxi + ed, ol = et * ldl + ed;
-    xq = live ? ld8(xqb + (long)t0 * ldx + ox) : z;
-    xk = live ? ld8(xkb + (long)t0 * ldx + ox) : z;
-    xl = live ? ld8(lowb + (long)t0 * p.ldl + ol) : z;
-    if (tid < CT) rb = t0 + tid < n ? bf2f((yb + (long)t0 * p.c.ldy)[tid * ldy]) : 0.f;
+    // clamped to valid rows and channels; what is not live counts as zero where it is used
+    const int tr = min(et, n - 1 - t0), dc = elive ? ed : 0;
+    const int ox = tr * ldxi + dc, ol = tr * ldl + dc;
+    xq = ld8(xqb + (long)t0 * ldx + ox);
+    xk = ld8(xkb + (long)t0 * ldx + ox);
+    xl = ld8(lowb + (long)t0 * p.ldl + ol);
+    rb = bf2f((yb + (long)t0 * p.c.ldy)[min(tid & 15, n - 1 - t0) * ldy]);
   };
   fetch(0);
   for (int t0 = 0; t0 < n; t0 += CT) {
@@ -477,8 +477,8 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
       float nq = 0.f, nk = 0.f;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        q8[e] = bf2f(xq[e]);
-        k8[e] = bf2f(xk[e]);
+        q8[e] = elive ? bf2f(xq[e]) : 0.f;
+        k8[e] = elive ? bf2f(xk[e]) : 0.f;
         nq = fmaf(q8[e], q8[e], nq);
         nk = fmaf(k8[e], k8[e], nk);
         lg[e] = tlive ? A * softplus_f(gain * bf2f(xl[e]) + dtb[ed + e]) : 0.f;
@@ -488,7 +488,7 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         nq += wave_xchg_n(nq, off);
         nk += wave_xchg_n(nk, off);
       }
-      const float iq = inv_sqrt_d * rsqrtf(nq + UNIT_EPS), ik = rsqrtf(nk + UNIT_EPS);
+      const float iq = tlive ? inv_sqrt_d * rsqrtf(nq + UNIT_EPS) : 0.f, ik = tlive ? rsqrtf(nk + UNIT_EPS) : 0.f;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         q8[e] *= iq;
@@ -521,29 +521,31 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
     if (tid == 0) nbad = 0;
     __syncthreads();
     if (ed < DP) {
-      float kt[8], qt[8], kc[8], kf[8], gt[8];
-      bool wides = false;
 #pragma unroll
       for (int hf = 0; hf < 2; ++hf) {
-        const f32x4 g0 = *reinterpret_cast<const f32x4*>(&e0[ed + 4 * hf]);
-        f32x4 base = {0.f, 0.f, 0.f, 0.f}, all = {0.f, 0.f, 0.f, 0.f};
+        asm volatile("" ::: "memory");  // four channels at a time
+        const int d0 = ed + 4 * hf;
+        const f32x4 g0 = *reinterpret_cast<const f32x4*>(&e0[d0]);
+        f32x4 gt = {0.f, 0.f, 0.f, 0.f}, all = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int q = 0; q < 4; ++q) {
-          const f32x4 v = *reinterpret_cast<const f32x4*>(&tot[q][ed + 4 * hf]);
-          if (q < w) base += v;  // wave-uniform
+          const f32x4 v = *reinterpret_cast<const f32x4*>(&tot[q][d0]);
+          if (q < w) gt += v;  // wave-uniform
           all += v;
         }
+        f32x4 kt, qt, kc, kf;
+        bool wides = false;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int e = 4 * hf + i;
-          const float G0 = g0[i], Gt = base[i] + pre[e], Gc = all[i];
+          gt[i] += pre[e];
+          const float G0 = g0[i], Gt = gt[i], Gc = all[i];
           const float E = exp_f(Gt - G0);
           const bool wide = G0 - Gc > RANGE;
-          gt[e] = Gt;
-          kt[e] = k8[e] * E;
-          qt[e] = q8[e] * E;
-          kc[e] = wide ? 0.f : k8[e] * exp_f(G0 - Gt);
-          kf[e] = k8[e] * exp_f(Gc - Gt);
+          kt[i] = k8[e] * E;
+          qt[i] = q8[e] * E;
+          kc[i] = wide ? 0.f : k8[e] * exp_f(G0 - Gt);
+          kf[i] = k8[e] * exp_f(Gc - Gt);
           wides |= wide;
           if (et == 15) {
             s0[ed + e] = exp_f(G0);
@@ -551,25 +553,24 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
             if (wide) bad[atomicAdd(&nbad, 1)] = ed + e;
           }
         }
-      }
-      if (wides) {  // the same channels for every token
+        if (wides) {  // the same channels for every token
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          Gs[et][ed + e] = gt[e];
-          Ks[et][ed + e] = k8[e];
-          Qs[et][ed + e] = q8[e];
+          for (int i = 0; i < 4; ++i) {
+            Gs[et][d0 + i] = gt[i];
+            Ks[et][d0 + i] = k8[4 * hf + i];
+            Qs[et][d0 + i] = q8[4 * hf + i];
+          }
         }
+        auto put = [&](bf16* hp, bf16* lp, f32x4 v) {
+          const bf16x4 a = hi4(v);
+          st4(hp + et * LDD + d0, a);
+          st4(lp + et * LDD + d0, lo4(v, a));
+        };
+        put(kt_h, kt_l, kt);
+        put(qt_h, qt_l, qt);
+        put(kc_h, kc_l, kc);
+        put(kh_h, kh_l, kf);
       }
-      auto put = [&](bf16* hp, bf16* lp, const float* v) {
-        bf16x8 a, c;
-        split8(f32x4{v[0], v[1], v[2], v[3]}, f32x4{v[4], v[5], v[6], v[7]}, a, c);
-        st8(hp + et * LDD + ed, a);
-        st8(lp + et * LDD + ed, c);
-      };
-      put(kt_h, kt_l, kt);
-      put(qt_h, qt_l, qt);
-      put(kc_h, kc_l, kc);
-      put(kh_h, kh_l, kf);
     }
     __syncthreads();
     // values and gates of the chunk in the accumulator layout (tokens 4 g + i, columns r)
@@ -581,7 +582,8 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
         const int t = 4 * g + i, v = (w * VTW + j) * 16 + r;
         const bool live = t < nt && v < V;
         const int tc = min(t, nt - 1), vc = min(v, V - 1);
-        vals[j][i] = live ? bf2f((xvb + (long)t0 * ldx)[tc * ldxi + vc]) : 0.f;
+        const float xv = bf2f((xvb + (long)t0 * ldx)[tc * ldxi + vc]);
+        vals[j][i] = live ? xv : 0.f;
         gates[j][i] = bf2f((gateb + (long)t0 * p.ldl)[tc * ldl + vc]);
       }
     // operand of row r: k-slots (g, j) <-> d = 32 ks + 4 g + j, 32 ks + 16 + 4 g + (j - 4)
@@ -712,14 +714,16 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(RecurParams p, cons
       for (int c = p.heads * V + (tid & 15); c < p.out_cols; c += 16)
         if (et < nt) out[et * ldo + c] = f2bf(0.f);
   }
+  int g4 = 4 * g;
+  asm volatile("" : "+v"(g4));  // addresses are formed anew: none stays in a register through the loop
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
     for (int j = 0; j < VTW; ++j)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
-        if (d < D && v < p.Vp) Sg[(long)d * p.Vp + v] = S[dt][j][i];
+        const int d = dt * 16 + g4 + i, v = (w * VTW + j) * 16 + r;
+        if (d < D && v < p.Vp) Sg[d * p.Vp + v] = S[dt][j][i];
       }
 }
 
@@ -755,7 +759,7 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
-        S[dt][j][i] = start > 0 && d < N && v < V ? Sg[(long)d * p.Vp + v] : 0.f;
+        S[dt][j][i] = start > 0 && d < N && v < V ? Sg[d * p.Vp + v] : 0.f;
       }
   // rows of the next chunk, in flight under this one's products
   bf16x4 rb[NB], rc[NB], rx[NX];
@@ -765,17 +769,20 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
     const bf16x4 z = {};
 #pragma unroll
     for (int q = 0; q < NB; ++q) {
-      const int c = tid + q * 256, t = c / (NP / 4), d = (c % (NP / 4)) * 4;
-      const bool live = t0 + t < n && d < N;
-      rb[q] = live ? ld4(xb + (long)t0 * ldx + t * ldxi + d) : z;
-      rc[q] = live ? ld4(xc + (long)t0 * ldx + t * ldxi + d) : z;
+      // clamped to valid rows (their dt is zero) and columns (zeros)
+      const int c = tid + q * 256, t = min(c / (NP / 4), n - 1 - t0), d = (c % (NP / 4)) * 4;
+      const int at = t * ldxi + min(d, N - 4);
+      const bf16x4 vb = ld4(xb + (long)t0 * ldx + at), vc = ld4(xc + (long)t0 * ldx + at);
+      rb[q] = d < N ? vb : z;
+      rc[q] = d < N ? vc : z;
     }
 #pragma unroll
     for (int q = 0; q < NX; ++q) {
-      const int c = tid + q * 256, t = c / (VP / 4), v = (c % (VP / 4)) * 4;
-      rx[q] = t0 + t < n && v < V ? ld4(xv + (long)t0 * ldx + t * ldxi + v) : z;
+      const int c = tid + q * 256, t = min(c / (VP / 4), n - 1 - t0), v = (c % (VP / 4)) * 4;
+      const bf16x4 vx = ld4(xv + (long)t0 * ldx + t * ldxi + min(v, V - 4));
+      rx[q] = v < V ? vx : z;
     }
-    rdt = t0 + tl < n ? bf2f(y[(long)(t0 + tl) * p.c.ldy + p.gate_col + h]) : 0.f;
+    rdt = bf2f((y + (long)t0 * p.c.ldy + p.gate_col + h)[min(tl, n - 1 - t0) * ldy]);
   };
   fetch(0);
   for (int t0 = 0, buf = 0; t0 < n; t0 += CT, buf ^= 1) {
@@ -911,14 +918,16 @@ __global__ __launch_bounds__(256, 2) void ssd_chunk_kernel(RecurParams p, const 
             out[t * ldo + v] = f2bf((o[mt][j][i] + skip * bf2f(xf[j][mt * 4 + i])) * silu(gain * zg[mt][j][i]));
         }
   }
+  int g4 = 4 * g;
+  asm volatile("" : "+v"(g4));  // addresses are formed anew: none stays in a register through the loop
 #pragma unroll
   for (int dt = 0; dt < NT; ++dt)
 #pragma unroll
     for (int j = 0; j < VTW; ++j)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
-        if (d < N && v < p.Vp) Sg[(long)d * p.Vp + v] = S[dt][j][i];
+        const int d = dt * 16 + g4 + i, v = (w * VTW + j) * 16 + r;
+        if (d < N && v < p.Vp) Sg[d * p.Vp + v] = S[dt][j][i];
       }
 }
 
