@@ -689,22 +689,43 @@ __global__ __launch_bounds__(256, 2) void talk_decode_kernel(TalkParams p) {
     for (int c = H * vdim + threadIdx.x; c < p.out_cols; c += 256) static_cast<bf16*>(p.out)[(long)b * p.ldo + c] = f2bf(0.f);
 }
 
-// One block per (query, head); the last head's also clears the pad columns.
+// One wave per (query, head); the last head's also clears the pad columns.
 __global__ __launch_bounds__(64) void talk_combine_kernel(TalkParams p) {
-  const int b = blockIdx.x / p.H, h = blockIdx.x % p.H;
+  constexpr int RUN = 8;  // splits whose rows are loaded together
+  __shared__ float ws[256];
+  const int b = blockIdx.x / p.H, h = blockIdx.x % p.H, lane = threadIdx.x;
   const long pi = (long)blockIdx.x * p.splits;
-  float M = NEG, L = 0.f;
-  for (int s = 0; s < p.splits; ++s) M = fmaxf(M, p.part_ml[2 * (pi + s)]);
-  for (int s = 0; s < p.splits; ++s) L += p.part_ml[2 * (pi + s) + 1] * exp2f(p.part_ml[2 * (pi + s)] - M);
-  const float inv = 1.f / L;
+  float m[4], l[4], M = NEG, L = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int s = lane + 64 * i;
+    m[i] = s < p.splits ? p.part_ml[2 * (pi + s)] : NEG;
+    l[i] = s < p.splits ? p.part_ml[2 * (pi + s) + 1] : 0.f;
+    M = fmaxf(M, m[i]);
+  }
+  M = wave_max(M);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const float w = lane + 64 * i < p.splits ? exp2f(m[i] - M) : 0.f;
+    ws[lane + 64 * i] = w;
+    L += l[i] * w;
+  }
+  const float inv = 1.f / wave_sum(L);
+  __syncthreads();
   bf16* out = static_cast<bf16*>(p.out) + (long)b * p.ldo;
-  for (int d = threadIdx.x; d < p.vdim; d += 64) {
+  for (int d = lane; d < p.vdim; d += 64) {
     float v = 0.f;
-    for (int s = 0; s < p.splits; ++s) v += p.part_o[(pi + s) * p.vdim + d] * exp2f(p.part_ml[2 * (pi + s)] - M);
+    for (int s = 0; s < p.splits; s += RUN) {
+      float x[RUN];
+#pragma unroll
+      for (int i = 0; i < RUN; ++i) x[i] = p.part_o[(pi + min(s + i, p.splits - 1)) * p.vdim + d];
+#pragma unroll
+      for (int i = 0; i < RUN; ++i) v += x[i] * ws[s + i];
+    }
     out[h * p.vdim + d] = f2bf(v * inv);
   }
   if (h == p.H - 1)
-    for (int c = p.H * p.vdim + threadIdx.x; c < p.out_cols; c += 64) out[c] = f2bf(0.f);
+    for (int c = p.H * p.vdim + lane; c < p.out_cols; c += 64) out[c] = f2bf(0.f);
 }
 
 }  // namespace

@@ -962,8 +962,37 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(MixOutParams p) {
     for (int c = p.heads * p.V + lane; c < p.out_cols; c += 64) from_f(out + c, 0.f);
 }
 
-// One block per (row, norm group) of rows y silu(z), in place: rms over the
-// group, times weight.
+// One wave per (row, norm group) of at most 1024 columns (a multiple of 4) of
+// rows y silu(z), in place: rms over the group, times weight.
+__global__ __launch_bounds__(256) void group_norm_wave_kernel(MixOutParams p) {
+  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= (long)p.T * p.groups) return;
+  const int lane = lane_id(), g = (int)(item % p.groups), W = p.inner / p.groups;
+  bf16* row = static_cast<bf16*>(p.out) + item / p.groups * p.ldo;
+  bf16* out = row + (long)g * W;
+  const float* wt = p.norm + (long)g * W;
+  constexpr int KEEP = 4;  // groups of four columns per lane
+  f32x4 v[KEEP], w[KEEP];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int c = (lane + i * 64) * 4, at = min(c, W - 4);
+    const bf16x4 x = ld4(out + at);
+    w[i] = f32x4{wt[at], wt[at + 1], wt[at + 2], wt[at + 3]};
+    v[i] = f32x4{bf2f(x[0]), bf2f(x[1]), bf2f(x[2]), bf2f(x[3])} * (c < W ? 1.f : 0.f);
+    ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
+  }
+  const float rs = rsqrtf(wave_sum(ss) / W + p.eps);
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int c = (lane + i * 64) * 4;
+    if (c < W) st4(out + c, pack4(v[i] * w[i] * rs));
+  }
+  if (g == p.groups - 1)
+    for (int c = p.inner + lane; c < p.out_cols; c += 64) row[c] = f2bf(0.f);
+}
+
+// The same for any sizes, one block per (row, norm group).
 template <typename T>
 __global__ __launch_bounds__(256) void group_norm_kernel(MixOutParams p) {
   __shared__ float red[16];
@@ -1142,7 +1171,10 @@ extern "C" hipError_t lsd_head_norm_gate(const MixOutParams* p, int f32, hipStre
 extern "C" hipError_t lsd_group_norm(const MixOutParams* p, int f32, hipStream_t st) {
   if (p->T == 0) return hipSuccess;
   const dim3 grid(p->T, p->groups);
-  if (f32) hipLaunchKernelGGL((group_norm_kernel<float>), grid, dim3(256), 0, st, *p);
+  const int W = p->inner / p->groups;
+  if (!f32 && W % 4 == 0 && W <= 1024)
+    hipLaunchKernelGGL(group_norm_wave_kernel, dim3((unsigned)(((long)p->T * p->groups + 3) / 4)), dim3(256), 0, st, *p);
+  else if (f32) hipLaunchKernelGGL((group_norm_kernel<float>), grid, dim3(256), 0, st, *p);
   else hipLaunchKernelGGL((group_norm_kernel<bf16>), grid, dim3(256), 0, st, *p);
   return hipGetLastError();
 }

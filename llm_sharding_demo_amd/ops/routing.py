@@ -127,8 +127,8 @@ class Routing:
     # recurrent layers: prompts of more than chunk_min tokens per sequence on
     # average run in chunks, shorter ones token by token
     chunk_min: int = 4
-    # decode attention with mixed heads: blocks a launch aims for, at least two
-    # 64-key tiles each
+    # decode attention with mixed heads: blocks a launch aims for, two 64-key
+    # tiles each unless that leaves half of them idle
     talk_target: int = 512
     # ... and prompt attention with few query tiles
     talk_prefill_target: int = 512
@@ -301,7 +301,10 @@ class Routing:
     def talk_splits(self, B: int, keys: int) -> int:
         """Context splits of a decode attention launch with mixed heads (one
         block holds all heads of a token, 64 keys a step)."""
-        return max(1, min(math.ceil(self.talk_target / B), math.ceil((keys + 63) / 128), 64))
+        tiles = math.ceil((keys + 63) / 64)  # a window may begin inside one
+        if B * tiles > self.talk_target // 2:
+            tiles = math.ceil(tiles / 2)
+        return max(1, min(math.ceil(self.talk_target / B), tiles, 64))
 
     def talk_prefill_splits(self, tiles: int, keys: int) -> int:
         """Key splits of a prompt attention launch with mixed heads: few query

@@ -145,7 +145,7 @@ def test_attention_prefill(C, H, G, D, V, window, splits):
 
 
 @pytest.mark.parametrize("H,G,D,V", [s for s in SIZES if s[1] <= 8])
-@pytest.mark.parametrize("window,splits", [(1 << 30, 1), (67, 1), (1, 1), (1 << 30, 3), (100, 2)])
+@pytest.mark.parametrize("window,splits", [(1 << 30, 1), (67, 1), (1, 1), (1 << 30, 3), (100, 2), (1 << 30, 17)])
 def test_attention_decode(C, H, G, D, V, window, splits):
     b = Batch((1, 0, 1), (2, 63, 1), (0, 200, 1))
     q, K, Vp, table, talk, want, out, scale, cap = attention_case(H, G, D, V, BF, b, window)
@@ -325,7 +325,7 @@ def test_delta_rule_chunks_between_tokens(C):
 
 
 SSM = [(2, 8, 8, 1, 1, 1), (6, 12, 20, 2, 3, 4), (4, 64, 128, 1, 1, 4), (3, 128, 64, 3, 3, 2), (8, 32, 16, 2, 4, 3),
-       (2, 100, 36, 1, 2, 4)]
+       (2, 100, 36, 1, 2, 4), (20, 64, 16, 1, 1, 4)]
 
 
 class SsmCase:
@@ -365,7 +365,7 @@ class SsmCase:
         return torch.cat(outs)
 
 
-@pytest.mark.parametrize("H,V,N,G,NG,n", SSM + [(2, 200, 300, 1, 1, 5)])
+@pytest.mark.parametrize("H,V,N,G,NG,n", SSM + [(2, 200, 300, 1, 1, 5), (3, 10, 8, 1, 2, 2)])
 @pytest.mark.parametrize("sizes", SPLITS)
 @pytest.mark.parametrize("dt", [BF, F32])
 def test_mamba2_by_tokens(C, H, V, N, G, NG, n, sizes, dt):
