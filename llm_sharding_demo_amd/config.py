@@ -66,11 +66,13 @@ class RopeScaling:
 
 @dataclass(frozen=True)
 class RopeSpec:
-    """Rotation of the first `dims` dimensions of a head, pairs (i, i + dims / 2)."""
+    """Rotation of the first `dims` dimensions of a head, pairs (i, i + dims / 2)
+    or, interleaved, (2i, 2i + 1)."""
 
     dims: int
     base: float
     scaling: Optional[RopeScaling] = None
+    interleaved: bool = False
 
     def frequencies(self) -> list:
         out = []
@@ -90,9 +92,14 @@ class RopeSpec:
 
 @dataclass(frozen=True)
 class AttentionSpec:
-    """Grouped-query attention over a paged K/V cache: partial rotation, capped
-    scores (softcap tanh(s / softcap)), and scores mixed over the heads by a
-    learned [heads, heads] matrix before the softmax (`talking`)."""
+    """Grouped-query attention over a paged K/V cache.  In front of the scores:
+    projection biases, a short convolution of q, k and v over time, unit RMS
+    norms of q and k per head, partial rotation, and values mixed with those of
+    an earlier layer.  Scores: capped (softcap tanh(s / softcap)), less a
+    distance bias of the head's slope, a sliding window beside the first
+    `keep_first` tokens.  `talking`: a learned [heads, heads] matrix mixes the
+    scores over the heads before the softmax, or (talk_weights) the weights
+    behind it.  head_gate: a sigmoid gate per head on its output."""
 
     heads: int
     kv_heads: int
@@ -103,19 +110,38 @@ class AttentionSpec:
     rope: Optional[RopeSpec] = None
     softcap: Optional[float] = None
     talking: bool = True
+    talk_weights: bool = False
+    keep_first: int = 0
+    distance_bias: bool = False
+    conv: int = 0                   # taps (0: none)
+    qk_norm: bool = False
+    bias: bool = False              # of the projections in and out
+    head_gate: bool = False
+    mix_values: Optional[int] = None  # v <- (1 - l) v + l v of this layer (its own index: the values others mix in)
     kv_from: None = None
 
     @property
     def cached_per_token(self) -> int:
         return self.kv_heads * (self.dim + self.vdim)
 
+    @property
+    def conv_channels(self) -> int:
+        return self.heads * self.dim + self.cached_per_token
+
+    def slopes(self) -> list:
+        """Distance bias per head: slope (i - j) is taken off the score."""
+        return [2.0 ** (-8.0 * (h + 1) / self.heads) for h in range(self.heads)]
+
     def params(self, hidden: int) -> int:
-        n = hidden * (self.heads * (self.dim + self.vdim) + self.kv_heads * (self.dim + self.vdim))
-        return n + (self.heads ** 2 if self.talking else 0)
+        n = hidden * (self.conv_channels + self.heads * self.vdim) + self.conv_channels * self.conv
+        n += (self.conv_channels + hidden if self.bias else 0) + (self.heads * hidden if self.head_gate else 0)
+        return n + (self.heads ** 2 if self.talking else 0) + (self.mix_values is not None)
 
     def check(self) -> None:
         if min(self.heads, self.kv_heads, self.dim, self.vdim) < 1 or (self.window is not None and self.window < 1):
             raise ValueError("attention sizes must be positive")
+        if self.conv < 0 or self.keep_first < 0:
+            raise ValueError("convolution taps and kept tokens must not be negative")
         if self.heads % self.kv_heads:
             raise ValueError(f"{self.heads} heads cannot share {self.kv_heads} key / value heads evenly")
         if self.rope is not None and (self.rope.dims % 2 or not 0 <= self.rope.dims <= self.dim):
@@ -191,9 +217,11 @@ class SSMSpec:
 
 @dataclass(frozen=True)
 class DenseSpec:
-    """Gated feed-forward W_down(gelu_tanh(W_gate h) * W_up h)."""
+    """Gated feed-forward W_down(gelu_tanh(W_gate h) * W_up h), or with a
+    `limit` the clamped gate of the experts."""
 
     ff: int
+    limit: Optional[float] = None
 
     def params(self, hidden: int) -> int:
         return 3 * hidden * self.ff
@@ -243,10 +271,12 @@ class ModelConfig:
     Models whose layers differ list them in `layers` (arch "timisun": parallel
     blocks of latent attention and experts; "vizalix": parallel blocks of
     attention, delta rule or Mamba-2 and a dense feed-forward, some of them
-    looped); the scalar head / ffn fields then only describe the first layer."""
+    looped; "kedasun": attention and a dense feed-forward one after the other,
+    each between two norms); the scalar head / ffn fields then only describe the
+    first layer."""
 
     name: str
-    arch: str  # "gpt2" | "llama" | "timisun" | "vizalix"
+    arch: str  # "gpt2" | "llama" | "timisun" | "vizalix" | "kedasun"
     vocab_size: int
     hidden: int
     n_layers: int
@@ -261,11 +291,11 @@ class ModelConfig:
     eos_token_id: int = 50256
     embed_scale: float = 1.0
     layers: Tuple[LayerSpec, ...] = ()
+    norm_groups: int = 1  # equal parts of a row, each normed by itself
 
     @property
-    def parallel_block(self) -> bool:
-        """Attention and MLP read the same normed input and are added together:
-        a layer cannot be cut between them."""
+    def whole_layers(self) -> bool:
+        """A stage starts at a layer, never between its mixer and feed-forward."""
         return bool(self.layers)
 
     @property
@@ -280,10 +310,18 @@ class ModelConfig:
         return max((l.enter + 1 for l in self.layers if l.enter is not None), default=0)
 
     @property
+    def mixed_values(self) -> Optional[AttentionSpec]:
+        """The layer whose values later layers mix in (None: no layer does)."""
+        first = next((l.mixer.mix_values for l in self.layers if getattr(l.mixer, "mix_values", None) is not None), None)
+        return None if first is None else self.layers[first].mixer
+
+    @property
     def boundary(self) -> int:
-        """Columns a stage hands to the next: the residual, and the embedding
-        output where a loop's passes read it again."""
-        return self.hidden * (2 if self.loop_times else 1)
+        """Columns a stage hands to the next: the residual, the embedding
+        output where a loop's passes read it again, and the values that later
+        layers mix in."""
+        m = self.mixed_values
+        return self.hidden * (2 if self.loop_times else 1) + (m.kv_heads * m.vdim if m is not None else 0)
 
     def weight_layer(self, i: int) -> int:
         """The layer whose tensors layer i uses."""
@@ -328,7 +366,7 @@ class ModelConfig:
         if not self.layers:
             return self.block_params()
         h, m, f = self.hidden, self.layers[i].mixer, self.layers[i].mlp
-        norms = h if self.arch == "timisun" else 1 + (f is not None)
+        norms = {"timisun": h, "kedasun": 2 * h * (1 + (f is not None))}.get(self.arch, 1 + (f is not None))
         return norms + m.params(h) + (f.params(h) if f is not None else 0)
 
     def block_params(self) -> int:
@@ -419,6 +457,10 @@ def check_layers(layers: Sequence[LayerSpec]) -> None:
             raise ValueError(f"layer {i}: top must be in [1, experts]")
         if isinstance(f, DenseSpec) and f.ff < 1:
             raise ValueError(f"layer {i}: feed-forward width must be positive")
+        j = getattr(m, "mix_values", None)
+        if j is not None and not (0 <= j <= i and (layers[j].mixer.mix_values, layers[j].mixer.kv_heads, layers[j].mixer.vdim)
+                                  == (j, m.kv_heads, m.vdim)):
+            raise ValueError(f"layer {i}: cannot mix in the values of layer {j}")
 
 
 def _timisun_layers(n: int, share: int = 2, experts: int = 16, **kw) -> list:
@@ -489,6 +531,54 @@ MODEL_PRESETS.update({
         14336, dict(heads=32, kv_heads=32, dim=128, vdim=128, conv=4, decay_rank=128, gate_rank=128),
         dict(heads=32, kv_heads=8, dim=128, vdim=128, scale=128 ** -0.5, window=1024, softcap=50.0, rope=_VIZALIX_ROPE),
         dict(heads=128, vdim=64, state=128, groups=8, norm_groups=8, conv=4)), loop=(0, 3, 2)),
+})
+
+
+def _kedasun(name: str, vocab: int, width: int, layers: Sequence[LayerSpec], groups: int, eps: float = 1e-6,
+             embed_scale: float = 1.0) -> ModelConfig:
+    """The first attention layer with mix_values set is the one whose values the others mix in."""
+    rep = dataclasses.replace
+    first = next((i for i, l in enumerate(layers) if l.mixer.mix_values is not None), None)
+    layers = tuple(l if l.mixer.mix_values is None else rep(l, mixer=rep(l.mixer, mix_values=first)) for l in layers)
+    check_layers(layers)
+    if groups < 1 or width % groups:
+        raise ValueError(f"width {width} does not divide into {groups} norm groups")
+    m, f = layers[0].mixer, layers[0].mlp
+    return ModelConfig(
+        name=name, arch="kedasun", vocab_size=vocab, hidden=width, n_layers=len(layers), n_heads=m.heads,
+        n_kv_heads=m.kv_heads, ffn=f.ff if f else 0, max_positions=1 << 20,  # rows of the rotation tables
+        norm_eps=eps, tie_embeddings=False, bos_token_id=0, eos_token_id=-1, embed_scale=embed_scale, layers=layers,
+        norm_groups=groups)
+
+
+def _kedasun_full(rot: Tuple[int, float], v_mix: bool = True, **sizes) -> AttentionSpec:
+    return AttentionSpec(rope=RopeSpec(*rot, interleaved=True) if rot[0] else None, talking=False,
+                         mix_values=0 if v_mix else None, **sizes)
+
+
+def _kedasun_window(v_mix: bool = True, **sizes) -> AttentionSpec:
+    return AttentionSpec(talk_weights=True, distance_bias=True, qk_norm=True, bias=True, head_gate=True,
+                         mix_values=0 if v_mix else None, **sizes)
+
+
+def _kedasun_layers(ff: int, limit: float, rot: Tuple[int, float], window: dict, repeat: int, **sizes) -> list:
+    """A windowed layer and two full ones, `repeat` times."""
+    f = DenseSpec(ff, limit)
+    return [LayerSpec(m, f) for m in [_kedasun_window(**window, **sizes)] + [_kedasun_full(rot, **sizes)] * 2] * repeat
+
+
+MODEL_PRESETS.update({
+    # Kedasun: small test sizes (none a multiple of the GEMM tiles), and two
+    # sizes that resemble the layers of models that are served today
+    "kedasun-test": _kedasun("kedasun-test", 300, 104, _kedasun_layers(
+        72, 1.5, (24, 10000.0), dict(window=90, keep_first=3, conv=3), 1, heads=6, kv_heads=3, dim=40, vdim=24,
+        scale=0.2), groups=2, embed_scale=0.6),
+    "kedasun-2b": _kedasun("kedasun-2b", 32000, 2048, _kedasun_layers(
+        5632, 7.0, (64, 500000.0), dict(window=1024, keep_first=4, conv=4), 4, heads=16, kv_heads=4, dim=128, vdim=128,
+        scale=128 ** -0.5), groups=4),
+    "kedasun-8b": _kedasun("kedasun-8b", 32000, 4096, _kedasun_layers(
+        14336, 7.0, (64, 500000.0), dict(window=1024, keep_first=4, conv=4), 2, heads=32, kv_heads=8, dim=128, vdim=128,
+        scale=128 ** -0.5), groups=4),
 })
 
 _ALIASES = {
@@ -572,6 +662,29 @@ def _vizalix_from_json(c: dict, name: str, shape) -> ModelConfig:
                     eps=float(c["norm"]["eps"]))
 
 
+def _kedasun_from_json(c: dict, name: str) -> ModelConfig:
+    """The design's own config.json."""
+    layers = []
+    for i, l in enumerate(c["layers"]):
+        m, f = l["mixer"], l.get("mlp")
+        sizes = dict(heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"], scale=float(m["scale"]),
+                     v_mix=bool(m.get("v_mix")))
+        if l["type"] == "attention":
+            r = m.get("rot") or {"dims": 0, "base": 1.0}
+            mix = _kedasun_full((r["dims"], float(r["base"])), **sizes)
+        elif l["type"] == "attention_2":
+            mask = m.get("mask") or {}
+            mix = _kedasun_window(window=mask.get("size"), keep_first=mask.get("keep_first") or 0, conv=m.get("conv") or 0,
+                                  **sizes)
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {l['type']!r}")
+        if f and f.get("kind", "dense") != "dense":
+            raise ValueError(f"layer {i}: unknown feed-forward {f['kind']!r}")
+        layers.append(LayerSpec(mix, DenseSpec(f["ff"], float(f["limit"])) if f else None))
+    return _kedasun(name, c["vocab"], c["width"], layers, groups=c["norm"]["groups"], eps=float(c["norm"]["eps"]),
+                    embed_scale=float(c["embedding"]["scale"]))
+
+
 def _checkpoint_shapes(folder: str):
     """name -> shape of the tensors in a folder's safetensors files (headers only)."""
     import json
@@ -598,8 +711,9 @@ def model_config_from_hf_json(path: str) -> ModelConfig:
     if c.get("architecture") == "Vizalix":
         folder = os.path.dirname(os.path.abspath(path))
         return _vizalix_from_json(c, os.path.basename(folder) or "vizalix", _checkpoint_shapes(folder))
-    if c.get("architecture") == "Timisun":
-        return _timisun_from_json(c, os.path.basename(os.path.dirname(os.path.abspath(path))) or "timisun")
+    own = {"Timisun": _timisun_from_json, "Kedasun": _kedasun_from_json}.get(c.get("architecture"))
+    if own is not None:
+        return own(c, os.path.basename(os.path.dirname(os.path.abspath(path))) or c["architecture"].lower())
     mt = c.get("model_type", "gpt2")
     if mt == "gpt2":
         h = c["n_embd"]

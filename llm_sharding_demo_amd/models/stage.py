@@ -1,4 +1,4 @@
-"""One pipeline stage of a GPT-2, Llama, Timisun or Vizalix model.
+"""One pipeline stage of a GPT-2, Llama, Timisun, Vizalix or Kedasun model.
 
 Generalises the reference's two hard-wired shards (`server.py:51-105`):
   * ShardA (`server.py:68-86`): wte + wpe + blocks[0:split]   -> stage 0
@@ -75,11 +75,16 @@ class StageModel:
         self.backend = backend if backend is not None else get_backend(self.device)
         # columns of the residual rows (hidden, or padded by the backend)
         self.row_width = self.backend.row_width(cfg)
-        # columns that cross a stage boundary: where a loop's passes read the
-        # embedding output again, it travels beside the residual
-        self.wire_width = self.row_width * (2 if cfg.loop_times else 1)
-        if cfg.parallel_block and (ua % 2 or ub % 2):
-            raise ValueError(f"{cfg.name}: parallel layers cannot be cut in half (units {units})")
+        # rows that cross a stage boundary: the residual, beside it the embedding
+        # output where a loop's passes read it again, and the values that later
+        # layers mix in; (heads, columns of a head, the model's own of them) each
+        self.wire_parts = [(1, self.row_width, cfg.hidden)] * (2 if cfg.loop_times else 1)
+        m = cfg.mixed_values
+        if m is not None:
+            self.wire_parts = self.wire_parts + [(m.kv_heads, self.backend.value_width(m), m.vdim)]
+        self.wire_width = sum(n * c for n, c, _ in self.wire_parts)
+        if cfg.whole_layers and (ua % 2 or ub % 2):
+            raise ValueError(f"{cfg.name}: layers cannot be cut in half (units {units})")
         if cfg.paged_cache:
             own = cfg.cache_layers(self.kv_layers)
             self._pool_index = {i: k for k, i in enumerate(own)}
@@ -183,20 +188,56 @@ class StageModel:
         o = be.mix(h, w, spec, self.kv, self.kv.entries[self._pool_index[i]], meta, c.norm_eps)
         be.mixer_residual(o, h, w, spec, r)
 
-    # -- stage boundaries: [x | x0] where the loop's passes need x0, else x ------
+    # Kedasun: attention, then a feed-forward, each between a norm of the
+    # residual and a norm of its output
+    def _sandwich_layer(self, i: int, r: Residual, side: dict, meta: BatchMeta) -> None:
+        be, c, spec = self.backend, self.cfg, self.cfg.layers[i]
+        w, m = functools.partial(self._lw, i), spec.mixer
+        h = be.group_norm(r, w("input_layernorm.weight"), c)
+        first = side.get("values") if m.mix_values is not None and m.mix_values != i else None
+        o, values = be.attend(h, w, m, self.kv, self.kv.entries[self._pool_index[i]], meta, c.norm_eps, first,
+                              keep_values=m.mix_values == i)
+        if m.mix_values == i:
+            side["values"] = values
+        be.linear_post_norm(o, w("mixer.o"), w("mixer.o.b", None), w("mixer.out_norm.weight"), r, c)
+        if spec.mlp is not None:
+            h = be.group_norm(r, w("post_attention_layernorm.weight"), c)
+            h = be.clamped_glu(h, w("mlp.gate_up.weight"), spec.mlp.limit)
+            be.linear_post_norm(h, w("mlp.down_proj.weight"), None, w("mlp.out_norm.weight"), r, c)
+
+    # -- stage boundaries: the residual, and what travels beside it (wire_parts) --
     def _unpack(self, rows: torch.Tensor):
-        if self.wire_width == self.row_width:
-            return rows, None
-        return rows[:, : self.row_width].contiguous(), rows[:, self.row_width:].contiguous()
+        """Residual rows and the side rows {"x0": ..., "values": ...}."""
+        if len(self.wire_parts) == 1:
+            return rows, {}
+        parts = [p.contiguous() for p in rows.split([n * c for n, c, _ in self.wire_parts], 1)]
+        side = {"x0": parts[1]} if self.cfg.loop_times else {}
+        if self.cfg.mixed_values is not None:
+            side["values"] = parts[-1].to(self.dtype)
+        return parts[0], side
+
+    def _pack(self, x: torch.Tensor, side: dict) -> torch.Tensor:
+        if len(self.wire_parts) == 1:
+            return x
+        rows = [x] + ([side["x0"]] if self.cfg.loop_times else [])
+        if self.cfg.mixed_values is not None:
+            n, c, _ = self.wire_parts[-1]
+            v = side.get("values")  # not there yet: the first layer that has them comes later
+            rows.append(v.float() if v is not None else x.new_zeros(x.shape[0], n * c))
+        return torch.cat(rows, 1)
 
     def boundary_rows(self, rows: torch.Tensor) -> torch.Tensor:
         """Rows as they leave the stage -> the model's own columns (compat forwards)."""
-        return torch.cat([p[:, : self.cfg.hidden] for p in rows.split(self.row_width, 1)], 1)
+        parts = rows.split([n * c for n, c, _ in self.wire_parts], 1)
+        return torch.cat([p.reshape(-1, n, c)[..., :own].reshape(-1, n * own)
+                          for p, (n, c, own) in zip(parts, self.wire_parts)], 1)
 
     def wire_rows(self, rows: torch.Tensor) -> torch.Tensor:
         """Inverse of boundary_rows: padded as the backend wants them."""
-        pad = (0, self.row_width - self.cfg.hidden)
-        return torch.cat([torch.nn.functional.pad(p, pad) for p in rows.split(self.cfg.hidden, 1)], 1)
+        parts = rows.split([n * own for n, _, own in self.wire_parts], 1)
+        pad = torch.nn.functional.pad
+        return torch.cat([pad(p.reshape(-1, n, own), (0, c - own)).reshape(-1, n * c)
+                          for p, (n, c, own) in zip(parts, self.wire_parts)], 1)
 
     # ------------------------------------------------------------------
     def embed(self, ids: torch.Tensor, meta: BatchMeta) -> torch.Tensor:
@@ -218,14 +259,14 @@ class StageModel:
         batch when given -- e.g. only the prompts whose final chunk this is).
         `variant`: which of the stage's unit ranges to run (the microbatch
         group's parity under alternating splits; 0 otherwise).  `residuals`
-        collects the residual rows after every parallel layer (debugging)."""
-        x0 = None
+        collects the residual rows after every whole layer (debugging)."""
+        side: dict = {}
         if self.first:
             x = self.embed(inp, meta)
-            if self.wire_width != self.row_width:
-                x0 = self.embed(inp, meta)  # the residual is updated in place
+            if self.cfg.loop_times:
+                side["x0"] = self.embed(inp, meta)  # the residual is updated in place
         else:
-            x, x0 = self._unpack(inp)
+            x, side = self._unpack(inp)
         r = Residual(x)
         # decode-only routing rules (ops/hip.py); a mixed step's rows follow them up to 512
         self.backend.decode = getattr(meta, "routing_decode", meta.is_decode) and meta.num_tokens <= 512 \
@@ -236,12 +277,14 @@ class StageModel:
         ua, ub = self.variants[variant % len(self.variants)]
         for u in range(ua, ub):
             i = u >> 1
-            if self.cfg.parallel_block:  # a whole layer: its second unit is empty
+            if self.cfg.whole_layers:  # a whole layer: its second unit is empty
                 if not u & 1:
                     if self.cfg.arch == "timisun":
                         self._parallel_layer(i, r, meta)
+                    elif self.cfg.arch == "kedasun":
+                        self._sandwich_layer(i, r, side, meta)
                     else:
-                        self._mixer_layer(i, r, x0, meta)
+                        self._mixer_layer(i, r, side.get("x0"), meta)
                     if residuals is not None:
                         residuals.append(self.backend.flush(r)[:, : self.cfg.hidden].clone())
                 continue
@@ -251,7 +294,7 @@ class StageModel:
                 attn_fn(self._kv_index[i], i, r, meta)
         x = self.backend.flush(r)
         if not (self.last and head):
-            return x if x0 is None or self.last else torch.cat([x, x0], 1)
+            return x if self.last else self._pack(x, side)
         return self.head(x, meta, all_logits, head_rows)
 
     def head(self, x: torch.Tensor, meta: BatchMeta, all_logits: bool = False,
@@ -263,6 +306,8 @@ class StageModel:
             xn = be.norm_rows(x, self.w["norm.weight"], None, c.norm_eps, True, rows, offset=1.0, width=c.hidden)
         elif c.arch == "vizalix":
             xn = be.norm_rows(x, self.w["norm.weight"], None, c.norm_eps, True, rows, width=be.norm_width(c))
+        elif c.arch == "kedasun":
+            xn = be.group_norm_rows(x, self.w["norm.weight"], c, rows)
         elif c.arch == "gpt2":
             xn = be.norm_rows(x, self.w["ln_f.weight"], self.w["ln_f.bias"], c.norm_eps, False, rows)
         else:

@@ -123,6 +123,32 @@ def _vizalix_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
     return out
 
 
+def _kedasun_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
+    h, m, f = cfg.hidden, cfg.layers[i].mixer, cfg.layers[i].mlp
+    p = f"layers.{i}."
+    rows = {"q": m.heads * m.dim, "k": m.kv_heads * m.dim, "v": m.kv_heads * m.vdim}
+    mix: Dict[str, tuple] = {n: (r, h) for n, r in rows.items()}
+    mix["o"] = (h, m.heads * m.vdim)
+    if m.bias:
+        mix.update((n + ".b", (r,)) for n, r in rows.items())
+        mix["o.b"] = (h,)
+    if m.conv:
+        mix.update((n + ".conv", (r, m.conv)) for n, r in rows.items())
+    if m.mix_values is not None:
+        mix["vmix"] = ()
+    if m.talking:
+        mix["talk"] = (m.heads, m.heads)
+    if m.head_gate:
+        mix["g"] = (m.heads, h)
+    out = {p + "input_layernorm.weight": (h,), p + "mixer.out_norm.weight": (h,)}
+    out.update((p + "mixer." + n, s) for n, s in mix.items())
+    if f is not None:
+        out[p + "post_attention_layernorm.weight"] = out[p + "mlp.out_norm.weight"] = (h,)
+        out[p + "mlp.gate_up.weight"] = (2 * f.ff, h)  # gate rows | up rows
+        out[p + "mlp.down_proj.weight"] = (h, f.ff)
+    return out
+
+
 _ATTN_PARTS = ("ln_1.", "attn.", "input_layernorm.", "self_attn.", "mixer.")
 _MLP_PARTS = ("ln_2.", "mlp.", "post_attention_layernorm.")
 
@@ -182,6 +208,14 @@ def _stage_tensor_shapes(cfg: ModelConfig, layers: Iterable[int], first: bool, l
         if last:
             shapes["norm.weight"] = ()
             shapes["lm_head"] = (cfg.vocab_size, cfg.hidden)
+    elif cfg.arch == "kedasun":
+        if first:
+            shapes["embed_tokens"] = (cfg.vocab_size, cfg.hidden)
+        for i in layers:
+            shapes.update(_kedasun_shapes(cfg, i))
+        if last:
+            shapes["norm.weight"] = (cfg.hidden,)
+            shapes["lm_head"] = (cfg.vocab_size, cfg.hidden)
     elif cfg.arch == "gpt2":
         if first:
             shapes["wte"] = (cfg.vocab_size, cfg.hidden)
@@ -209,6 +243,8 @@ def _init_one(cfg: ModelConfig, name: str, shape, seed: int, device, dtype) -> t
         return _timisun_init(cfg, name, shape, seed, device, dtype)
     if cfg.arch == "vizalix":
         return _vizalix_init(cfg, name, shape, seed, device, dtype)
+    if cfg.arch == "kedasun":
+        return _kedasun_init(name, shape, seed, device, dtype)
     if name == "embed_tokens":
         # untied (Llama) input embeddings at unit scale (the T5 / muP
         # convention: the residual stream enters at the RMS its norms produce).
@@ -280,6 +316,29 @@ def _vizalix_init(cfg: ModelConfig, name: str, shape, seed: int, device, dtype) 
     if leaf in ("mixer.o", "mlp.down_proj.weight"):
         std /= (2 * cfg.n_layers) ** 0.5
     return _randn(shape, std, seed, name, device, dtype)
+
+
+def _kedasun_init(name: str, shape, seed: int, device, dtype) -> torch.Tensor:
+    """Unit-variance projections (the norms behind them set the residual's
+    scale), short convolutions that mostly pass the current token, head mixing
+    near the identity, half of the values mixed in."""
+    def around(mean, std):
+        return (mean + _randn(shape, std, seed, name, device, torch.float32)).to(dtype)
+
+    leaf = name.split(".", 2)[-1] if name.startswith("layers.") else name
+    if leaf == "embed_tokens":
+        return _randn(shape, 1.0, seed, name, device, dtype)
+    if leaf.endswith("norm.weight"):
+        return around(1.0, 0.05)
+    if leaf == "mixer.vmix":
+        return around(0.5, 0.05)
+    if leaf == "mixer.talk":
+        return around(torch.eye(shape[0], device=device), 0.3 * shape[0] ** -0.5)
+    if leaf.endswith(".conv"):
+        return around((torch.arange(shape[1], device=device) == shape[1] - 1).float(), 0.2)
+    if leaf.endswith(".b"):
+        return _randn(shape, 0.1, seed, name, device, dtype)
+    return _randn(shape, shape[-1] ** -0.5, seed, name, device, dtype)
 
 
 def init_stage_weights(cfg: ModelConfig, layers, first: bool, last: bool, seed: int,
@@ -368,6 +427,21 @@ def _vizalix_tensor(name: str, get) -> torch.Tensor:
                            "mlp.down_proj.weight": "mlp.down"}[rest])
 
 
+def _kedasun_tensor(name: str, get) -> torch.Tensor:
+    """One canonical tensor from a checkpoint in the design's own names."""
+    top = {"embed_tokens": "embed", "norm.weight": "final.norm", "lm_head": "head"}
+    if name in top:
+        return get(top[name])
+    _, i, rest = name.split(".", 2)
+    own = {"input_layernorm.weight": "norm1", "mixer.out_norm.weight": "norm1b",
+           "post_attention_layernorm.weight": "norm2", "mlp.out_norm.weight": "norm2b", "mlp.down_proj.weight": "mlp.down"}
+    if rest in own:
+        return get(f"l{i}.{own[rest]}")
+    if rest == "mlp.gate_up.weight":
+        return torch.cat([get(f"l{i}.mlp.gate"), get(f"l{i}.mlp.up")], 0)
+    return get(f"l{i}.mix." + rest[len("mixer."):])
+
+
 def load_stage_weights(cfg: ModelConfig, path: str, layers, first: bool, last: bool,
                        device, dtype, units=None) -> Dict[str, torch.Tensor]:
     get, keys = _open_checkpoint(path)
@@ -385,6 +459,8 @@ def load_stage_weights(cfg: ModelConfig, path: str, layers, first: bool, last: b
             t = _timisun_tensor(cfg, name, get)
         elif cfg.arch == "vizalix":
             t = _vizalix_tensor(name, get)
+        elif cfg.arch == "kedasun":
+            t = _kedasun_tensor(name, get)
         elif cfg.arch == "gpt2":
             src = {"wte": "wte.weight", "wpe": "wpe.weight"}.get(name, name)
             t = find(src)

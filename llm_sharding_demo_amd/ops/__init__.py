@@ -32,6 +32,9 @@ from . import reference as ref
 class Residual:
     x: torch.Tensor  # fp32 [T, H]
     pending: List[Tuple[torch.Tensor, Optional[torch.Tensor]]] = field(default_factory=list)
+    # output of a sublayer that is normed before it is added: (slabs [S, T, H],
+    # bias, norm weight, model config), folded in by the next group_norm or flush
+    post: Optional[tuple] = None
 
 
 # sigmoid slope of the experts' gated activation (fixed by the design)
@@ -51,6 +54,10 @@ class Backend:
     def latent_width(self, rank: int) -> int:
         """Columns of a cached latent row (>= rank; the rest stays zero)."""
         return rank
+
+    def value_width(self, mixer) -> int:
+        """Columns of a value head (>= vdim; the rest stays zero)."""
+        return mixer.vdim
 
     def layer_cache(self, mixer) -> LayerCache:
         """What a layer keeps per page and per slot (runtime/kv_cache.py)."""
@@ -165,16 +172,7 @@ class ReferenceBackend(Backend):
         return fn(h, w, m, kv, entry, meta, eps)
 
     def _attend(self, h, w, m, kv, entry, meta, eps):
-        pos = meta.token_pos
-        q = ref.partial_rope(ref.linear(h, w("mixer.q")).reshape(-1, m.heads, m.dim), pos, m.rope)
-        k = ref.partial_rope(ref.linear(h, w("mixer.k")).reshape(-1, m.kv_heads, m.dim), pos, m.rope)
-        v = ref.linear(h, w("mixer.v")).reshape(-1, m.kv_heads, m.vdim)
-        for pool, x in zip(entry, (k, v)):
-            ref.paged_append(pool, kv.table, x, meta.token_slots, pos)
-        talk = w("mixer.talk") if m.talking else None
-        o = torch.cat([ref.talking_attention(q[s], entry[0], entry[1], kv.table, mt.seq_slots, mt.q_start, mt.cu_q,
-                                             talk, m.scale, m.softcap, m.window) for s, mt in self._parts(meta)])
-        return o.reshape(o.shape[0], -1)
+        return self.attend(h, w, m, kv, entry, meta, eps, None)[0]
 
     def _channel_delta(self, h, w, m, kv, entry, meta, eps):
         T, H, G, D, V = h.shape[0], m.heads, m.kv_heads, m.dim, m.vdim
@@ -206,6 +204,57 @@ class ReferenceBackend(Backend):
             y[s] = ref.ssd(u, B, C, dt[s], decay[s], entry[0], mt) + w("mixer.D").float()[:, None] * u
         y = (y.view(T, -1) * torch.nn.functional.silu(z)).view(T, m.norm_groups, -1)
         return ref.rmsnorm(y, y.new_ones(y.shape[-1]), eps).view(T, -1) * w("mixer.norm").float()
+
+    # -- layers with norms around each sublayer (models/stage.py _sandwich_layer) ----
+    def group_norm(self, r: Residual, w, mcfg):
+        self._combine(r)
+        return ref.group_rmsnorm(r.x, w, mcfg.norm_eps, mcfg.norm_groups)
+
+    def group_norm_rows(self, x, w, mcfg, rows=None):
+        x = x if rows is None else x.index_select(0, rows.long())
+        return ref.group_rmsnorm(x, w, mcfg.norm_eps, mcfg.norm_groups)
+
+    def linear_post_norm(self, a, w, b, norm_w, r: Residual, mcfg) -> None:
+        """x += norm(a w^T + b)."""
+        self._combine(r)
+        r.x += ref.group_rmsnorm(ref.linear(a, w, b), norm_w, mcfg.norm_eps, mcfg.norm_groups)
+
+    def clamped_glu(self, h, w, limit: float):
+        y = ref.linear(h, w)
+        f = y.shape[1] // 2
+        return ref.clamped_glu(y[:, :f], y[:, f:], limit, GLU_ALPHA)
+
+    def attend(self, h, w, m: AttentionSpec, kv, entry, meta, eps, first_values, keep_values: bool = False):
+        """Attention before the output projection [T, heads * vdim], and with
+        keep_values this layer's values [T, kv heads * vdim].  first_values: rows
+        that are mixed into the values (None: they stay as they are)."""
+        qkv = torch.cat([ref.linear(h, w(f"mixer.{n}"), w(f"mixer.{n}.b", None)) for n in "qkv"], 1)
+        if m.conv:
+            taps, x = torch.cat([w(f"mixer.{n}.conv") for n in "qkv"]), qkv
+            qkv = torch.cat([ref.ring_conv(x[s], taps, None, entry[2], mt) for s, mt in self._parts(meta)])
+        G, pos = m.kv_heads, meta.token_pos
+        q, k, v = qkv.split([m.heads * m.dim, G * m.dim, G * m.vdim], 1)
+        q, k = q.reshape(-1, m.heads, m.dim), k.reshape(-1, G, m.dim)
+        if m.qk_norm:
+            q, k = (ref.rmsnorm(t, t.new_ones(m.dim), eps) for t in (q, k))
+        q, k = (ref.partial_rope(t, pos, m.rope) for t in (q, k))
+        values = v.contiguous() if keep_values else None
+        if first_values is not None:
+            lam = w("mixer.vmix").float()
+            v = (1 - lam) * v + lam * first_values.float()
+        for pool, x in zip(entry, (k, v.reshape(-1, G, m.vdim))):
+            ref.paged_append(pool, kv.table, x, meta.token_slots, pos)
+        o = self._attention_parts(q, w, m, kv, entry, meta)
+        if m.head_gate:
+            o = o * torch.sigmoid(ref.linear(h, w("mixer.g")))[..., None]
+        return o.reshape(o.shape[0], -1), values
+
+    def _attention_parts(self, q, w, m, kv, entry, meta):
+        talk = w("mixer.talk") if m.talking else None
+        slopes = torch.tensor(m.slopes()) if m.distance_bias else None
+        return torch.cat([ref.talking_attention(q[s], entry[0], entry[1], kv.table, mt.seq_slots, mt.q_start, mt.cu_q,
+                                                talk, m.scale, m.softcap, m.window, m.talk_weights, slopes, m.keep_first)
+                          for s, mt in self._parts(meta)])
 
     def mixer_residual(self, o, h, w, spec, r: Residual) -> None:
         """x += o W_o^T + feed-forward(h): both halves of a parallel block."""

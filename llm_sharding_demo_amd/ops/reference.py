@@ -49,6 +49,12 @@ def rmsnorm(x: torch.Tensor, w: torch.Tensor, eps: float, offset: float = 0.0) -
     return xf * torch.rsqrt(var + eps) * (w.float() + offset)
 
 
+def group_rmsnorm(x: torch.Tensor, w: torch.Tensor, eps: float, groups: int) -> torch.Tensor:
+    """`groups` equal consecutive parts of a row, each over its own root mean square."""
+    xf = x.float().view(*x.shape[:-1], groups, -1)
+    return (xf * torch.rsqrt(xf.pow(2).mean(-1, keepdim=True) + eps)).view(x.shape) * w.float()
+
+
 def linear(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """a [T, K] @ w[N, K]^T (+ bias) in fp32."""
     out = a.float() @ w.float().t()
@@ -155,12 +161,17 @@ def latent_attention(q: torch.Tensor, pool: torch.Tensor, table: torch.Tensor, s
 
 
 def partial_rope(x: torch.Tensor, pos: torch.Tensor, rope) -> torch.Tensor:
-    """x [T, heads, dim]: pairs (i, i + dims / 2) of the first rope.dims dimensions turn."""
+    """x [T, heads, dim]: pairs (i, i + dims / 2), or (2i, 2i + 1) where the
+    layout is interleaved, of the first rope.dims dimensions turn."""
     if rope is None or rope.dims == 0:
         return x
     half = rope.dims // 2
     ang = pos.double()[:, None] * torch.tensor(rope.frequencies(), dtype=torch.float64, device=pos.device)
     cos, sin = ang.cos().float()[:, None], ang.sin().float()[:, None]
+    if rope.interleaved:
+        a, b = x[..., 0: 2 * half: 2].float(), x[..., 1: 2 * half: 2].float()
+        turned = torch.stack([a * cos - b * sin, b * cos + a * sin], -1).flatten(-2)
+        return torch.cat([turned, x[..., 2 * half:].float()], -1)
     a, b = x[..., :half].float(), x[..., half: 2 * half].float()
     return torch.cat([a * cos - b * sin, b * cos + a * sin, x[..., 2 * half:].float()], -1)
 
@@ -173,10 +184,13 @@ def paged_append(pool: torch.Tensor, table: torch.Tensor, x: torch.Tensor, slots
 
 
 def talking_attention(q, k_pool, v_pool, table, seq_slots, q_start, cu_q, talk, scale: float,
-                      softcap: Optional[float], window: Optional[int]) -> torch.Tensor:
+                      softcap: Optional[float], window: Optional[int], talk_weights: bool = False,
+                      slopes: Optional[torch.Tensor] = None, keep_first: int = 0) -> torch.Tensor:
     """q [T, heads, dim] over paged keys and values [pages, kv heads, page, .]:
-    scores are capped, mixed over the heads (talk [heads, heads]) and softmaxed
-    over i - window < j <= i.  Returns fp32 [T, heads, vdim]."""
+    scores are capped, lessened by slopes [heads] times the distance, mixed over
+    the heads (talk [heads, heads]; talk_weights: behind the softmax) and
+    softmaxed over i - window < j <= i and j < keep_first.  Returns fp32
+    [T, heads, vdim]."""
     T, H, _ = q.shape
     page, grp = k_pool.shape[2], H // k_pool.shape[1]
     out = torch.empty(T, H, v_pool.shape[3], dtype=torch.float32, device=q.device)
@@ -187,16 +201,21 @@ def talking_attention(q, k_pool, v_pool, table, seq_slots, q_start, cu_q, talk, 
         st, end = int(q_start[i]), int(q_start[i]) + b - a
         lo = 0 if window is None else max(0, st - window + 1)
         kpos = torch.arange(lo, end, device=q.device)
+        kpos = torch.cat([torch.arange(min(lo, keep_first), device=q.device), kpos])
         pg = table[int(seq_slots[i]), kpos // page].long()
         k, v = (p[pg, :, kpos % page].float().transpose(0, 1).repeat_interleave(grp, 0) for p in (k_pool, v_pool))
         s = torch.matmul(q[a:b].float().transpose(0, 1), k.transpose(1, 2)) * scale  # [heads, Lq, keys]
         if softcap is not None:
             s = softcap * torch.tanh(s / softcap)
-        if talk is not None:
-            s = torch.matmul(talk.float(), s.reshape(H, -1)).view_as(s)
         d = torch.arange(st, end, device=q.device)[:, None] - kpos[None, :]
-        hide = d < 0 if window is None else (d < 0) | (d >= window)
-        out[a:b] = torch.matmul(torch.softmax(s.masked_fill(hide, float("-inf")), -1), v).transpose(0, 1)
+        if slopes is not None:
+            s = s - slopes[:, None, None] * d
+        mix = lambda x: x if talk is None else torch.matmul(talk.float(), x.reshape(H, -1)).view_as(x)  # noqa: E731
+        if not talk_weights:
+            s = mix(s)
+        hide = d < 0 if window is None else (d < 0) | ((d >= window) & (kpos >= keep_first))
+        p = torch.softmax(s.masked_fill(hide, float("-inf")), -1)
+        out[a:b] = torch.matmul(mix(p) if talk_weights else p, v).transpose(0, 1)
     return out
 
 

@@ -163,13 +163,13 @@ def unit_costs(cfg: ModelConfig, rows: int = 128, avg_ctx: int = 192) -> Tuple[L
 
 
 def _layer_costs(cfg: ModelConfig, rows: int, avg_ctx: int):
-    """unit_costs of models with per-layer specs (parallel blocks: a layer is
-    its first unit, the second costs nothing)."""
+    """unit_costs of models with per-layer specs (never cut within a layer: it
+    is its first unit, the second costs nothing)."""
     h = cfg.hidden
     costs: List[float] = []
     for l in cfg.layers:
         m, f = l.mixer, l.mlp
-        if cfg.arch == "vizalix":
+        if cfg.arch in ("vizalix", "kedasun"):
             costs += [_mixer_cost(cfg, l, rows, avg_ctx), 0.0]
             continue
         n_in = m.heads * m.dim + (m.kv_rank if m.kv_from is None else 0) + (f.experts if f else 0)
@@ -193,11 +193,15 @@ def _mixer_cost(cfg: ModelConfig, l, rows: int, avg_ctx: int) -> float:
     ov = m.heads * m.vdim
     if m.cached_per_token:
         n_in = m.heads * m.dim + m.cached_per_token
-        moved = rows * min(avg_ctx, m.window or avg_ctx) * m.cached_per_token * 2
+        moved = rows * min(avg_ctx, (m.window or avg_ctx) + m.keep_first) * m.cached_per_token * 2
     else:  # the state is read and written once
         n_in = m.params(h) // h - ov
         moved = rows * 8 * ov * (m.dim if hasattr(m, "dim") else m.state)
-    c = 6.0 + _gemm_us(n_in, h, rows) + 6.0 + moved / 5.0e6 + _gemm_us(h, ov + ff, rows)
+    c = 6.0 + _gemm_us(n_in, h, rows) + 6.0 + moved / 5.0e6
+    if cfg.arch == "kedasun":  # two sublayers, each with projections and norms of its own
+        c += _gemm_us(h, ov, rows) + (6.0 + _gemm_us(h, ff, rows) if ff else 0.0)
+    else:
+        c += _gemm_us(h, ov + ff, rows)
     if ff:
         c += _gemm_us(2 * ff, h, rows)
     if l.enter is not None:
@@ -218,7 +222,7 @@ def layer_cuts(cfg: ModelConfig) -> List[int]:
 def _check_cuts(cfg: ModelConfig, plan: UnitPlan) -> None:
     ok = {2 * b for b in layer_cuts(cfg)}
     for a, _ in plan[1:]:
-        if cfg.parallel_block and a not in ok:
+        if cfg.whole_layers and a not in ok:
             raise ValueError(f"a stage cannot start at unit {a}: stages of {cfg.name} start at layers "
                              f"{sorted(u // 2 for u in ok)} (whole layers, shared caches kept together)")
 
@@ -286,7 +290,7 @@ def make_unit_plan(cfg: ModelConfig, num_stages: int, split_points: Optional[Seq
         plan = [(0, 2 * L)]
     else:
         costs, head, embed = unit_costs(cfg, max(1, min(rows, 256)), avg_ctx)
-        if cfg.parallel_block:  # atoms: runs of layers between the allowed cuts
+        if cfg.whole_layers:  # atoms: runs of layers between the allowed cuts
             cuts = [0] + layer_cuts(cfg) + [L]
             if P > len(cuts) - 1:
                 raise ValueError(f"cannot split {cfg.name} into {P} stages: {len(cuts) - 1} groups of layers "

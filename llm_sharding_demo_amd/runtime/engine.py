@@ -96,7 +96,7 @@ class Engine(racecheck.Shared):
         # stage holds the union.  Needs an even group count and the
         # cost-model partition (no explicit split points).
         self.unit_plans = None
-        if (self.P > 1 and self.M % 2 == 0 and not self.mcfg.parallel_block and not cfg.split_points and not cfg.split_units
+        if (self.P > 1 and self.M % 2 == 0 and not self.mcfg.whole_layers and not cfg.split_points and not cfg.split_units
                 and cfg.half_layer_split and os.environ.get("LSD_ALT_SPLIT", "1") != "0"):
             pa, pb = make_alt_unit_plans(self.mcfg, self.P, rows=self.group_cap,
                                          avg_ctx=min(192, cfg.max_seq_len))
@@ -352,7 +352,9 @@ class Engine(racecheck.Shared):
         item's prefill rows (a group's chunk tokens, fp32) -- within 64 MiB to
         1 GiB, and never less than one such message plus 1 MiB."""
         per_seq = self.cfg.prefill_chunk if self.cfg.prefill_chunk > 0 else self.max_seq
-        big = self.group_cap * min(per_seq, self.max_seq) * ((self.mcfg.hidden + 63) // 64 * 64) * 4 * (2 if self.mcfg.loop_times else 1)
+        m = self.mcfg.mixed_values
+        cols = pad_up(self.mcfg.hidden, 64) * (2 if self.mcfg.loop_times else 1) + (m.kv_heads * pad_up(m.vdim, 16) if m else 0)
+        big = self.group_cap * min(per_seq, self.max_seq) * cols * 4
         ring = int(os.environ.get("LSD_LOOP_RING_MB", "0")) << 20 or min(1 << 30, max(64 << 20, 8 * big))
         return max(ring, big + (1 << 20))
 

@@ -76,13 +76,16 @@ class LayerCache:
 
 def layer_cache(mixer, up: Callable[[int, int], int] = lambda n, m: n) -> LayerCache:
     """Cache of one layer; up(n, m): the backend's padding of n to a multiple of m.
-      attention   K [kv head][token][dim], V [kv head][token][vdim] per page
+      attention   K [kv head][token][dim], V [kv head][token][vdim] per page, and the
+                  q | k | v rows of positions p % taps in front of a short convolution
       delta rule  S [heads][dim][vdim] and the conv inputs of positions p % taps
       Mamba-2     S [heads][state][vdim], and the same
       latent      one row of `rank` per token"""
     if isinstance(mixer, AttentionSpec):
         g = mixer.kv_heads
-        return LayerCache(pages=((g, PAGE, up(mixer.dim, 32)), (g, PAGE, up(mixer.vdim, 16))))
+        dp, vp = up(mixer.dim, 32), up(mixer.vdim, 16)
+        ring = ((mixer.conv, (mixer.heads + g) * dp + g * vp),) if mixer.conv else ()
+        return LayerCache(pages=((g, PAGE, dp), (g, PAGE, vp)), ring=ring)
     if isinstance(mixer, (ChannelDeltaSpec, SSMSpec)):
         rows = mixer.dim if isinstance(mixer, ChannelDeltaSpec) else mixer.state
         return LayerCache(state=((mixer.heads, rows, up(mixer.vdim, 4)),), ring=((mixer.conv, mixer.conv_channels),))
