@@ -216,14 +216,14 @@ torch::Tensor out_rows(const c10::optional<torch::Tensor>& out, int64_t M, int64
 }
 
 // out = act(a @ w^T + bias), bf16.  act: 1 gelu, 2 silu(gate) up, 3 gelu(gate) up,
-// the gated ones with `scale` times both halves
+// both with `scale` times both halves, 4 clamped gate with the limit `scale`
 torch::Tensor linear(torch::Tensor a, torch::Tensor w, c10::optional<torch::Tensor> bias,
                      int64_t act, int64_t tiled, int64_t splits,
                      c10::optional<torch::Tensor> counters, c10::optional<torch::Tensor> into, double scale) {
   GemmParams p = base_params(a, w, tiled);
   p.bias = opt_bias(bias, p.N);
   int epi = act == 1 ? EPI_GELU : (act >= 2 ? EPI_SILU_MUL : EPI_BF16);
-  p.gelu = act == 3;
+  p.glu = act >= 2 ? (int)act - 2 : 0;
   p.act_scale = (float)scale;
   if (epi == EPI_SILU_MUL) TORCH_CHECK(p.N % 32 == 0, "silu_mul needs N % 32 == 0");
   const int n_out = epi == EPI_SILU_MUL ? p.N / 2 : p.N;
@@ -351,7 +351,7 @@ c10::optional<torch::Tensor> gemv(torch::Tensor x, torch::Tensor w, c10::optiona
                                   int64_t q_size, int64_t kv_size, int64_t hd,
                                   c10::optional<torch::Tensor> rope,
                                   c10::optional<torch::Tensor> segmax = c10::nullopt,
-                                  c10::optional<torch::Tensor> into = c10::nullopt, bool gelu = false,
+                                  c10::optional<torch::Tensor> into = c10::nullopt, int64_t glu = 0,
                                   double scale = 1.0) {
   need(w, torch::kBFloat16, "w");
   need_rows(w, "w");
@@ -359,7 +359,8 @@ c10::optional<torch::Tensor> gemv(torch::Tensor x, torch::Tensor w, c10::optiona
   TORCH_CHECK(reinterpret_cast<uintptr_t>(x.data_ptr()) % 16 == 0, "x must be 16-byte aligned");
   GemvParams p{};
   p.M = x.size(0); p.K = x.size(1); p.N = w.size(0);
-  p.gelu = gelu; p.act_scale = (float)scale;
+  TORCH_CHECK(glu >= 0 && glu <= 2, "gated activation 0 to 2");
+  p.glu = (int)glu; p.act_scale = (float)scale;
   TORCH_CHECK(w.size(1) == p.K, "K mismatch: x ", x.sizes(), " w ", w.sizes());
   TORCH_CHECK(lsd_gemv_ok(p.M, p.K, (int)epi, (int)norm), "gemv: shape M=", p.M, " K=", p.K,
               " epi=", epi, " norm=", norm, " not supported");
@@ -802,11 +803,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   // bf16 outputs into the caller's rows, gated activations with a common factor
   m.def("gemv_into", [](torch::Tensor x, torch::Tensor w, int64_t epi, int64_t norm,
                         c10::optional<torch::Tensor> gamma, c10::optional<torch::Tensor> beta, double eps,
-                        c10::optional<torch::Tensor> out, bool gelu, double scale) {
+                        c10::optional<torch::Tensor> out, int64_t glu, double scale) {
     return gemv(x, w, c10::nullopt, epi, norm, gamma, beta, eps, c10::nullopt, c10::nullopt, c10::nullopt,
-                c10::nullopt, c10::nullopt, 0, 0, 0, c10::nullopt, c10::nullopt, out, gelu, scale);
+                c10::nullopt, c10::nullopt, 0, 0, 0, c10::nullopt, c10::nullopt, out, glu, scale);
   }, py::arg("x"), py::arg("w"), py::arg("epi"), py::arg("norm"), py::arg("gamma"), py::arg("beta"), py::arg("eps"),
-        py::arg("out") = py::none(), py::arg("gelu") = false, py::arg("scale") = 1.0);
+        py::arg("out") = py::none(), py::arg("glu") = 0, py::arg("scale") = 1.0);
   m.def("gemv_logits", [](torch::Tensor x, torch::Tensor w, int64_t norm, c10::optional<torch::Tensor> gamma,
                           c10::optional<torch::Tensor> beta, double eps, torch::Tensor segmax) {
     return gemv(x, w, c10::nullopt, EPI_F32, norm, gamma, beta, eps, c10::nullopt, c10::nullopt,

@@ -1,99 +1,23 @@
-// Attention over a paged K / V cache whose scores are capped and then mixed over
-// the heads by a learned [H][H] matrix before the softmax, with grouped K / V
-// heads, a sliding window, and rotation of part of a head's dimensions.
+// Attention over a paged K / V cache with a learned [H][H] matrix that mixes
+// over the heads: capped scores in front of the softmax, or the weights behind
+// it; grouped K / V heads and a sliding window.
 //
-//  * rope_append: behind the in-projection, rotates q and k, appends k and v to
-//    their page.
 //  * talk_prefill: MFMA, 16 queries of 4 heads per wave, all heads in a block.
-//  * talk_decode: MFMA, one token of all heads per block, keys split over blocks.
-//  * talk_plain: one token per block, any sizes, bf16 or fp32.
+//  * talk_decode: MFMA, one token of all heads per block, keys split over blocks
+//    (scores mixed; mixed weights: attention_paged.hip).
+//  * talk_plain: one token per block, any sizes, bf16 or fp32, and without mixing.
 //
 // Every head's score of a (query, key) pair is needed before any head's weight
-// of it is known, so a block works on all heads of its queries.  Scores cross
-// the waves through LDS as two fp16 terms (value and remainder, 22 bits: the cap
-// bounds them) and are mixed by the matrix cores in fp32; softmax weights enter
-// the second product as two bf16 terms.
-#include "common.h"
-#include "mixer_params.h"
+// of it is known, so a block works on all heads of its queries.  Scores (bounded
+// by the cap) or softmax weights cross the waves through LDS as two fp16 terms
+// (value and remainder, 22 bits) and are mixed by the matrix cores in fp32; what
+// multiplies the values enters the second product as two bf16 terms.  Weights
+// can be mixed once they are normalised: attention_paged.hip's prompt kernel
+// gives log2 of every softmax sum first.
+#include "attention_paged.h"
 
 namespace lsd {
 namespace {
-
-constexpr int PAGE = 64;
-constexpr float NEG = -1e30f;
-
-__device__ __forceinline__ float to_f(float v) { return v; }
-__device__ __forceinline__ float to_f(bf16 v) { return bf2f(v); }
-__device__ __forceinline__ void from_f(float* o, float v) { *o = v; }
-__device__ __forceinline__ void from_f(bf16* o, float v) { *o = f2bf(v); }
-
-__device__ __forceinline__ int first_key(int pos, int window) { return window > pos ? 0 : pos - window + 1; }
-
-// One block per token.
-template <typename T>
-__global__ __launch_bounds__(256) void rope_append_kernel(RopeAppendParams p) {
-  const long row = blockIdx.x;
-  const int pos = p.tpos[row], half = p.half;
-  const long page = p.table[(long)p.tslot[row] * p.tw + pos / PAGE];
-  const int nq = p.H * p.dim, nk = p.G * p.dim, nv = p.G * p.vdim;
-  const T* y = static_cast<const T*>(p.y) + row * p.ldy;
-  const float* cs = p.rope + (long)pos * half * 2;
-  for (int i = threadIdx.x; i < nq + nk + nv; i += 256) {
-    float v = to_f(y[i]) * p.gain;
-    if (i < nq + nk) {
-      const int d = i % p.dim;  // the k columns start at a multiple of dim
-      if (d < half) v = v * cs[2 * d] - to_f(y[i + half]) * p.gain * cs[2 * d + 1];
-      else if (d < 2 * half) v = v * cs[2 * (d - half)] + to_f(y[i - half]) * p.gain * cs[2 * (d - half) + 1];
-    }
-    if (i < nq) {
-      from_f(static_cast<T*>(p.q) + row * nq + i, v);
-    } else if (i < nq + nk) {
-      const int g = (i - nq) / p.dim, d = (i - nq) % p.dim;
-      from_f(static_cast<T*>(p.k) + ((page * p.G + g) * PAGE + pos % PAGE) * p.dim + d, v);
-    } else {
-      const int g = (i - nq - nk) / p.vdim, d = (i - nq - nk) % p.vdim;
-      from_f(static_cast<T*>(p.v) + ((page * p.G + g) * PAGE + pos % PAGE) * p.vdim + d, v);
-    }
-  }
-}
-
-// 8 columns per thread; dims and the rotation's half are multiples of 8.  One
-// block per four tokens, a wave each.
-__global__ __launch_bounds__(256) void rope_append_vec_kernel(RopeAppendParams p) {
-  const long row = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (row >= p.T) return;
-  const int pos = p.tpos[row], half = p.half;
-  const long page = p.table[(long)p.tslot[row] * p.tw + pos / PAGE];
-  const int nq = p.H * p.dim, nk = p.G * p.dim, nv = p.G * p.vdim;
-  const bf16* y = static_cast<const bf16*>(p.y) + row * p.ldy;
-  const float* cs = p.rope + (long)pos * half * 2;
-  for (int i = lane_id() * 8; i < nq + nk + nv; i += 512) {
-    const bf16x8 x = ld8(y + i);
-    float v[8];
-#pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = bf2f(x[e]) * p.gain;
-    const int d = i % p.dim;
-    if (i < nq + nk && d < 2 * half) {
-      const bool first = d < half;
-      const bf16x8 o = ld8(first ? y + i + half : y + i - half);
-      const float* c = cs + 2 * (first ? d : d - half);
-#pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const float s = bf2f(o[e]) * p.gain * c[2 * e + 1];
-        v[e] = fmaf(v[e], c[2 * e], first ? -s : s);
-      }
-    }
-    bf16* dst;
-    if (i < nq) dst = static_cast<bf16*>(p.q) + row * nq + i;
-    else if (i < nq + nk) dst = static_cast<bf16*>(p.k) + ((page * p.G + (i - nq) / p.dim) * PAGE + pos % PAGE) * p.dim + d;
-    else dst = static_cast<bf16*>(p.v) + ((page * p.G + (i - nq - nk) / p.vdim) * PAGE + pos % PAGE) * p.vdim +
-               (i - nq - nk) % p.vdim;
-    bf16x8 r;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) r[e] = f2bf(v[e]);
-    st8(dst, r);
-  }
-}
 
 // One token per block, KT keys at a time.  Dynamic LDS: queries [H][dim], scores
 // before and after mixing [H][KT + 1], outputs [H][vdim], and per head the
@@ -124,60 +48,75 @@ __global__ __launch_bounds__(256) void talk_plain_kernel(TalkParams p) {
     l[h] = 0.f;
   }
   __syncthreads();
-  for (int k0 = lo; k0 <= pos; k0 += KT) {
-    const int nk = min(KT, pos - k0 + 1);
-    for (int i = tid; i < H * KT; i += 256) {
-      const int h = i / KT, kk = i % KT, key = k0 + kk;
-      float s = 0.f;
-      if (kk < nk) {
-        const T* kp = K + (((long)table[key / PAGE] * p.G + h / rep) * PAGE + key % PAGE) * p.dim;
-        for (int d = 0; d < p.dim; ++d) s = fmaf(qs[h * p.dim + d], to_f(kp[d]), s);
-        s *= p.scale;
-        if (p.cap > 0.f) s = p.cap * tanhf(s / p.cap);
+  const int kept = min(p.keep, lo), n_keys = kept + pos - lo + 1;
+  auto key_at = [&](int i) { return i < kept ? i : i - kept + lo; };
+  // mixed weights: a first pass for the softmax sums, a second with the weights
+  for (int pass = p.mix_weights ? 0 : 1; pass < 2; ++pass) {
+    for (int k0 = 0; k0 < n_keys; k0 += KT) {
+      const int nk = min(KT, n_keys - k0);
+      for (int i = tid; i < H * KT; i += 256) {
+        const int h = i / KT, kk = i % KT, key = key_at(k0 + kk);
+        float s = 0.f;
+        if (kk < nk) {
+          const T* kp = K + (((long)table[key / PAGE] * p.G + h / rep) * PAGE + key % PAGE) * p.dim;
+          for (int d = 0; d < p.dim; ++d) s = fmaf(qs[h * p.dim + d], to_f(kp[d]), s);
+          s *= p.scale;
+          if (p.cap > 0.f) s = p.cap * tanhf(s / p.cap);
+          if (p.slopes) s -= p.slopes[h] * (float)(pos - key);
+          if (p.mix_weights && pass == 1) s = expf(s - m[h]) / l[h];
+        }
+        s0[h * LD + kk] = s;
       }
-      s0[h * LD + kk] = s;
-    }
-    __syncthreads();
-    for (int i = tid; i < H * KT; i += 256) {
-      const int h = i / KT, kk = i % KT;
-      float s = 0.f;
-      if (p.talk) {
-        for (int g = 0; g < H; ++g) s = fmaf(p.talk[h * H + g], s0[g * LD + kk], s);
-      } else {
-        s = s0[h * LD + kk];
+      __syncthreads();
+      const bool mix = p.talk && pass == 1;
+      for (int i = tid; i < H * KT; i += 256) {
+        const int h = i / KT, kk = i % KT;
+        float s = 0.f;
+        if (mix) {
+          for (int g = 0; g < H; ++g) s = fmaf(p.talk[h * H + g], s0[g * LD + kk], s);
+        } else {
+          s = s0[h * LD + kk];
+        }
+        s1[h * LD + kk] = kk < nk ? s : NEG;
       }
-      s1[h * LD + kk] = kk < nk ? s : NEG;
-    }
-    __syncthreads();
-    for (int h = tid >> 6; h < H; h += 4) {  // a wave per head; lanes past the tile are neutral
-      const int kk = lane_id();
-      const float s = kk < KT ? s1[h * LD + kk] : NEG;
-      const float mo = m[h], mn = fmaxf(mo, wave_max(s));
-      const float e = kk < nk ? expf(s - mn) : 0.f;
-      const float sum = wave_sum(e);
-      if (kk < KT) s1[h * LD + kk] = e;
-      if (kk == 0) {
-        const float alpha = expf(mo - mn);
-        m[h] = mn;
-        l[h] = l[h] * alpha + sum;
-        al[h] = alpha;
+      __syncthreads();
+      if (!p.mix_weights || pass == 0) {
+        for (int h = tid >> 6; h < H; h += 4) {  // a wave per head; lanes past the tile are neutral
+          const int kk = lane_id();
+          const float s = kk < KT ? s1[h * LD + kk] : NEG;
+          const float mo = m[h], mn = fmaxf(mo, wave_max(s));
+          const float e = kk < nk ? expf(s - mn) : 0.f;
+          const float sum = wave_sum(e);
+          if (kk < KT) s1[h * LD + kk] = e;
+          if (kk == 0) {
+            const float alpha = expf(mo - mn);
+            m[h] = mn;
+            l[h] = l[h] * alpha + sum;
+            al[h] = alpha;
+          }
+        }
+        __syncthreads();
+      }
+      if (pass == 1) {
+        for (int i = tid; i < H * p.vdim; i += 256) {
+          const int h = i / p.vdim, d = i % p.vdim;
+          float a = p.mix_weights ? acc[i] : acc[i] * al[h];
+          for (int kk = 0; kk < nk; ++kk) {
+            const int key = key_at(k0 + kk);
+            a = fmaf(s1[h * LD + kk],
+                     to_f(V[(((long)table[key / PAGE] * p.G + h / rep) * PAGE + key % PAGE) * p.vdim + d]), a);
+          }
+          acc[i] = a;
+        }
+        __syncthreads();
       }
     }
-    __syncthreads();
-    for (int i = tid; i < H * p.vdim; i += 256) {
-      const int h = i / p.vdim, d = i % p.vdim;
-      float a = acc[i] * al[h];
-      for (int kk = 0; kk < nk; ++kk) {
-        const int key = k0 + kk;
-        a = fmaf(s1[h * LD + kk],
-                 to_f(V[(((long)table[key / PAGE] * p.G + h / rep) * PAGE + key % PAGE) * p.vdim + d]), a);
-      }
-      acc[i] = a;
-    }
-    __syncthreads();
   }
   T* out = static_cast<T*>(p.out) + row * p.ldo;
-  for (int i = tid; i < p.out_cols; i += 256) from_f(out + i, i < H * p.vdim ? acc[i] / l[i / p.vdim] : 0.f);
+  for (int i = tid; i < p.out_cols; i += 256) {
+    const int h = i / p.vdim;
+    from_f(out + i, h < H ? acc[i] / (p.mix_weights ? 1.f : l[h]) * head_gate<T>(p, row, h) : 0.f);
+  }
 }
 
 typedef _Float16 half8 __attribute__((ext_vector_type(8)));
@@ -192,31 +131,10 @@ __device__ __forceinline__ f32x4 mfma_f16(half8 a, half8 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0);
 }
 
-// Transposed read of 4 x 16 LDS blocks: k runs over rows, the result's lanes over columns.
-__device__ __forceinline__ bf16x4 ds_read_tr(const bf16* lds_ptr) {
-  typedef __attribute__((address_space(3))) bf16x4 lds_bf16x4;
-  return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds_bf16x4*)(lds_ptr));
-}
-
-// This wave's LDS accesses are done
-__device__ __forceinline__ void lds_fence() {
-  __builtin_amdgcn_s_waitcnt(0xC07F);  // lgkmcnt(0)
-  __builtin_amdgcn_wave_barrier();
-}
-
 // cap tanh(x): `two_over` is 2 log2(e) scale / cap, the factor of the raw product
 __device__ __forceinline__ float capped(float raw, float two_over, float cap) {
   const float t = __builtin_amdgcn_exp2f(raw * two_over);
   return cap - 2.f * cap * __builtin_amdgcn_rcpf(1.f + t);
-}
-
-// Two bf16 terms of eight weights
-__device__ __forceinline__ void split_p(const float* a, const float* b, u32x4& hi, u32x4& lo) {
-  const bf16x4 ha = pack4(f32x4{a[0], a[1], a[2], a[3]}), hb = pack4(f32x4{b[0], b[1], b[2], b[3]});
-  const bf16x4 la = pack4(f32x4{a[0] - bf2f(ha[0]), a[1] - bf2f(ha[1]), a[2] - bf2f(ha[2]), a[3] - bf2f(ha[3])});
-  const bf16x4 lb = pack4(f32x4{b[0] - bf2f(hb[0]), b[1] - bf2f(hb[1]), b[2] - bf2f(hb[2]), b[3] - bf2f(hb[3])});
-  hi = __builtin_bit_cast(u32x4, (bf16x8{ha[0], ha[1], ha[2], ha[3], hb[0], hb[1], hb[2], hb[3]}));
-  lo = __builtin_bit_cast(u32x4, (bf16x8{la[0], la[1], la[2], la[3], lb[0], lb[1], lb[2], lb[3]}));
 }
 
 // x[k] of lane group g  ->  x[g] of lane group k (groups of 16 lanes)
@@ -234,9 +152,6 @@ __device__ __forceinline__ void transpose_groups(u32x4 (&x)[4]) {
   }
 }
 
-constexpr float LOG2E = 1.4426950408889634f;
-constexpr int VLD = 64 + 8;  // row pitch of 64 staged V columns
-
 // Prompt attention.  HP / 4 waves share 16 queries, each owning 4 consecutive
 // heads; a block has at least 4 waves (one or more such groups of queries).  Per
 // 32-key tile: scores of
@@ -245,7 +160,10 @@ constexpr int VLD = 64 + 8;  // row pitch of 64 staged V columns
 // all keys of query r, head g) -> barrier -> softmax in the lane, weights
 // transposed between lane groups and registers, second product per head.  Few
 // queries: the keys are split over blockIdx.y, partial outputs combined after.
-template <int DKS, int VT, int HP>
+// WTS: what crosses and is mixed are softmax weights (times 2^WSHIFT, which keeps
+// small ones within fp16), and the product with the values follows at once.
+constexpr float WSHIFT = 12.f, WUNIT = 1.f / 4096.f;
+template <int DKS, int VT, int HP, bool WTS>
 __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_prefill_kernel(TalkParams p) {
   constexpr int TK = 32, HW = HP / 4, NW = HW > 4 ? HW : 4, QG = NW / HW;
   constexpr int PITCH = HP == 8 ? 8 : HP + 8;  // fp16 scores of one pair
@@ -281,13 +199,22 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
 #pragma unroll
     for (int di = 0; di < VT; ++di) o[hh][di] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = NEG, lsum = 0.f;
-  const float two_over = 2.f * LOG2E * p.scale / p.cap;
-  const int lo = first_key(st + off, p.window), hi = st + min(off + QG * 16, qlen);
-  int kt0 = lo / TK, kt1 = (hi + TK - 1) / TK;
+  const float two_over = 2.f * LOG2E * p.scale / p.cap, scale2 = LOG2E * p.scale;
+  float lse[4], slope[4];
+  if constexpr (WTS) {
+#pragma unroll
+    for (int hh = 0; hh < 4; ++hh) {
+      const int h = min(hw * 4 + hh, H - 1);
+      lse[hh] = p.lse[(long)(cu + qc) * H + h] - WSHIFT;
+      slope[hh] = p.slopes ? p.slopes[h] * LOG2E : 0.f;
+    }
+  }
+  const KeyTiles kts = key_tiles<TK>(st + off, st + min(off + QG * 16, qlen) - 1, p.window, p.keep);
+  int it0 = 0, it1 = kts.count();
   if (p.splits > 1) {
-    const int per = (kt1 - kt0 + p.splits - 1) / p.splits;
-    kt0 += blockIdx.y * per;
-    kt1 = min(kt1, kt0 + per);
+    const int per = (it1 + p.splits - 1) / p.splits;
+    it0 = blockIdx.y * per;
+    it1 = min(it1, it0 + per);
   }
   // 64 columns of the tile's V rows, 16 bytes per lane and 8 rows
   bf16x8 vr[4];
@@ -301,9 +228,12 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
     }
   };
 
-  for (int kt = kt0; kt < kt1; ++kt) {
+  for (int it = it0; it < it1; ++it) {
+    const int kt = kts.at(it);
     const long page = table[kt * TK / PAGE];
     const int koff = (kt * TK) % PAGE;
+    const bool whole = (kt * TK >= my_lo || kt * TK + TK <= p.keep) && kt * TK + TK - 1 <= my_pos;
+    const bool all_whole = __all(whole);
     // scores of the own heads; the queries are read again for every tile (from
     // L1 / L2): the outputs take the registers
     f32x4 s[4][2];
@@ -336,9 +266,19 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         half4 a, b;
+        const int key = kt * TK + ni * 16 + 4 * g + i;
+        const bool hide = WTS && !all_whole && !seen(key, my_pos, my_lo, p.keep);
+        auto crossing = [&](int hh) {
+          if constexpr (WTS) {
+            const float x = fmaf(s[hh][ni][i], scale2, fmaf(slope[hh], (float)(key - my_pos), -lse[hh]));
+            return hide ? 0.f : __builtin_amdgcn_exp2f(x);
+          } else {
+            return capped(s[hh][ni][i], two_over, p.cap);
+          }
+        };
 #pragma unroll
         for (int hh = 0; hh < 4; hh += 2) {  // the remainder makes up for the truncated first term
-          const float c = capped(s[hh][ni][i], two_over, p.cap), d = capped(s[hh + 1][ni][i], two_over, p.cap);
+          const float c = crossing(hh), d = crossing(hh + 1);
           const half2 u = pack_half(c, d), v = pack_half(c - (float)u[0], d - (float)u[1]);
           a[hh] = u[0];
           a[hh + 1] = u[1];
@@ -362,42 +302,43 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
       acc = mfma_f16(tf, a, acc);
       acc = mfma_f16(tf, b, acc);
-      e[key] = acc[0] * LOG2E;
+      e[key] = WTS ? acc[0] : acc[0] * LOG2E;
     }
     __syncthreads();  // the next tile's scores may be written
-    const bool whole = kt * TK >= my_lo && kt * TK + TK - 1 <= my_pos;
-    if (!__all(whole)) {
+    if constexpr (!WTS) {
+      if (!all_whole) {
+#pragma unroll
+        for (int key = 0; key < TK; ++key) {
+          const int k = kt * TK + key;
+          e[key] = k >= my_lo && k <= my_pos ? e[key] : NEG;
+        }
+      }
+      float tmax = e[0];
+#pragma unroll
+      for (int key = 1; key < TK; ++key) tmax = fmaxf(tmax, e[key]);
+      // weights are taken relative to m, which follows the running maximum only
+      // when that is more than 2^6 ahead
+      if (__any(tmax > m + 6.f)) {
+        const float mn = fmaxf(m, tmax);
+        const float alpha = __builtin_amdgcn_exp2f(m - mn);
+        m = mn;
+        lsum *= alpha;
+#pragma unroll
+        for (int hh = 0; hh < 4; ++hh) {
+          const float ah = __shfl(alpha, hh * 16 + r, 64);
+#pragma unroll
+          for (int di = 0; di < VT; ++di) o[hh][di] *= ah;
+        }
+      }
+      const float off2 = m > 0.5f * NEG ? m : 0.f;  // no key seen yet: weights of zero
+      float ps = 0.f;
 #pragma unroll
       for (int key = 0; key < TK; ++key) {
-        const int k = kt * TK + key;
-        e[key] = k >= my_lo && k <= my_pos ? e[key] : NEG;
+        e[key] = __builtin_amdgcn_exp2f(e[key] - off2);
+        ps += e[key];
       }
+      lsum += ps;
     }
-    float tmax = e[0];
-#pragma unroll
-    for (int key = 1; key < TK; ++key) tmax = fmaxf(tmax, e[key]);
-    // weights are taken relative to m, which follows the running maximum only
-    // when that is more than 2^6 ahead
-    if (__any(tmax > m + 6.f)) {
-      const float mn = fmaxf(m, tmax);
-      const float alpha = __builtin_amdgcn_exp2f(m - mn);
-      m = mn;
-      lsum *= alpha;
-#pragma unroll
-      for (int hh = 0; hh < 4; ++hh) {
-        const float ah = __shfl(alpha, hh * 16 + r, 64);
-#pragma unroll
-        for (int di = 0; di < VT; ++di) o[hh][di] *= ah;
-      }
-    }
-    const float off2 = m > 0.5f * NEG ? m : 0.f;  // no key seen yet: weights of zero
-    float ps = 0.f;
-#pragma unroll
-    for (int key = 0; key < TK; ++key) {
-      e[key] = __builtin_amdgcn_exp2f(e[key] - off2);
-      ps += e[key];
-    }
-    lsum += ps;
     // k-slot j of group g <-> key 4 g + j (j < 4), 16 + 4 g + (j - 4) (j >= 4)
     u32x4 ph[4], pl[4];
 #pragma unroll
@@ -433,6 +374,14 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
       }
     }
   }
+  if constexpr (WTS) {  // the partial sums of key splits simply add up: equal maxima, sums of 1 in all
+    m = 0.f;
+    lsum = 1.f / p.splits;
+#pragma unroll
+    for (int hh = 0; hh < 4; ++hh)
+#pragma unroll
+      for (int di = 0; di < VT; ++di) o[hh][di] *= WUNIT;
+  }
   if (p.splits > 1) {
 #pragma unroll
     for (int hh = 0; hh < 4; ++hh) {
@@ -455,8 +404,8 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
   bf16* out = static_cast<bf16*>(p.out) + (long)(cu + qc) * p.ldo;
 #pragma unroll
   for (int hh = 0; hh < 4; ++hh) {
-    const float ih = __shfl(inv, hh * 16 + r, 64);
     const int h = hw * 4 + hh;
+    const float ih = __shfl(inv, hh * 16 + r, 64) * head_gate<bf16>(p, cu + qc, min(h, H - 1));
     if (h >= H || qi >= qlen) continue;
 #pragma unroll
     for (int di = 0; di < VT; ++di) {
@@ -710,7 +659,7 @@ __global__ __launch_bounds__(64) void talk_combine_kernel(TalkParams p) {
     ws[lane + 64 * i] = w;
     L += l[i] * w;
   }
-  const float inv = 1.f / wave_sum(L);
+  const float inv = 1.f / wave_sum(L), gate = head_gate<bf16>(p, b, h);
   __syncthreads();
   bf16* out = static_cast<bf16*>(p.out) + (long)b * p.ldo;
   for (int d = lane; d < p.vdim; d += 64) {
@@ -722,7 +671,7 @@ __global__ __launch_bounds__(64) void talk_combine_kernel(TalkParams p) {
 #pragma unroll
       for (int i = 0; i < RUN; ++i) v += x[i] * ws[s + i];
     }
-    out[h * p.vdim + d] = f2bf(v * inv);
+    out[h * p.vdim + d] = f2bf(v * inv * gate);
   }
   if (h == p.H - 1)
     for (int c = p.H * p.vdim + lane; c < p.out_cols; c += 64) out[c] = f2bf(0.f);
@@ -733,55 +682,57 @@ __global__ __launch_bounds__(64) void talk_combine_kernel(TalkParams p) {
 
 using namespace lsd;
 
-// Head padding of the MFMA kernels, 0: sizes they do not take.
+// Head padding of the MFMA kernels, 0: sizes they do not take.  cap: of the mixed
+// scores, < 0 where weights are mixed.
 extern "C" int lsd_talk_heads(int H, int G, int dim, int vdim, float cap) {
-  if (H > 32 || H / G > 16 || dim % 32 || dim > 128 || vdim % 16 || vdim > 128 || !(cap > 0.f) || cap > 3e4f) return 0;
+  if (H > 32 || H / G > 16 || dim % 32 || dim > 128 || vdim % 16 || vdim > 128 || cap == 0.f || cap > 3e4f) return 0;
   return H <= 8 ? 8 : H <= 16 ? 16 : 32;
 }
 
 extern "C" int lsd_talk_tile(int hp) { return hp == 8 ? 32 : 16; }  // queries of a prefill tile
 
-#define LSD_TK_V(KERNEL, HP, GRID, NT)                                                                   \
-  if (p->dim <= 64 && p->vdim <= 64) hipLaunchKernelGGL((KERNEL<2, 4, HP>), GRID, dim3(NT), 0, st, *p); \
-  else if (p->dim <= 64) hipLaunchKernelGGL((KERNEL<2, 8, HP>), GRID, dim3(NT), 0, st, *p);              \
-  else if (p->vdim <= 64) hipLaunchKernelGGL((KERNEL<4, 4, HP>), GRID, dim3(NT), 0, st, *p);             \
-  else hipLaunchKernelGGL((KERNEL<4, 8, HP>), GRID, dim3(NT), 0, st, *p);
+#define LSD_TK_V(KERNEL, GRID, NT, ...)                                                                           \
+  if (p->dim <= 64 && p->vdim <= 64) hipLaunchKernelGGL((KERNEL<2, 4, __VA_ARGS__>), GRID, dim3(NT), 0, st, *p); \
+  else if (p->dim <= 64) hipLaunchKernelGGL((KERNEL<2, 8, __VA_ARGS__>), GRID, dim3(NT), 0, st, *p);              \
+  else if (p->vdim <= 64) hipLaunchKernelGGL((KERNEL<4, 4, __VA_ARGS__>), GRID, dim3(NT), 0, st, *p);             \
+  else hipLaunchKernelGGL((KERNEL<4, 8, __VA_ARGS__>), GRID, dim3(NT), 0, st, *p);
+
+extern "C" hipError_t lsd_attention_combine(const TalkParams* p, hipStream_t st) {
+  if (p->T == 0) return hipSuccess;
+  hipLaunchKernelGGL(talk_combine_kernel, dim3(p->T * p->H), dim3(64), 0, st, *p);
+  return hipGetLastError();
+}
 
 extern "C" hipError_t lsd_talk_prefill(const TalkParams* p, int hp, hipStream_t st) {
   if (p->n_tiles == 0) return hipSuccess;
   const dim3 grid(p->n_tiles, p->splits);
-  switch (hp) {
-    case 8: LSD_TK_V(talk_prefill_kernel, 8, grid, 256) break;
-    case 16: LSD_TK_V(talk_prefill_kernel, 16, grid, 256) break;
-    case 32: LSD_TK_V(talk_prefill_kernel, 32, grid, 512) break;
+  switch (hp + (p->mix_weights ? 1 : 0)) {
+    case 8: LSD_TK_V(talk_prefill_kernel, grid, 256, 8, false) break;
+    case 16: LSD_TK_V(talk_prefill_kernel, grid, 256, 16, false) break;
+    case 32: LSD_TK_V(talk_prefill_kernel, grid, 512, 32, false) break;
+    case 9: LSD_TK_V(talk_prefill_kernel, grid, 256, 8, true) break;
+    case 17: LSD_TK_V(talk_prefill_kernel, grid, 256, 16, true) break;
+    case 33: LSD_TK_V(talk_prefill_kernel, grid, 512, 32, true) break;
     default: return hipErrorInvalidValue;
   }
-  if (p->splits > 1) hipLaunchKernelGGL(talk_combine_kernel, dim3(p->T * p->H), dim3(64), 0, st, *p);
+  if (p->splits > 1) return lsd_attention_combine(p, st);
   return hipGetLastError();
 }
 
 // hp: 16 or 32 (talk_frag padded to it); needs G <= hp
 extern "C" hipError_t lsd_talk_decode(const TalkParams* p, int hp, hipStream_t st) {
   if (p->T == 0) return hipSuccess;
+  if (p->mix_weights) return hipErrorInvalidValue;
   const dim3 grid(p->T, p->splits);
   switch (hp) {
-    case 16: LSD_TK_V(talk_decode_kernel, 16, grid, 256) break;
-    case 32: LSD_TK_V(talk_decode_kernel, 32, grid, 256) break;
+    case 16: LSD_TK_V(talk_decode_kernel, grid, 256, 16) break;
+    case 32: LSD_TK_V(talk_decode_kernel, grid, 256, 32) break;
     default: return hipErrorInvalidValue;
   }
-  if (p->splits > 1) hipLaunchKernelGGL(talk_combine_kernel, dim3(p->T * p->H), dim3(64), 0, st, *p);
+  if (p->splits > 1) return lsd_attention_combine(p, st);
   return hipGetLastError();
 }
 #undef LSD_TK_V
-
-extern "C" hipError_t lsd_rope_append(const RopeAppendParams* p, int f32, hipStream_t st) {
-  if (p->T == 0) return hipSuccess;
-  if (f32) hipLaunchKernelGGL((rope_append_kernel<float>), dim3(p->T), dim3(256), 0, st, *p);
-  else if (p->half % 8 == 0 && p->dim % 8 == 0 && p->vdim % 8 == 0)
-    hipLaunchKernelGGL(rope_append_vec_kernel, dim3((p->T + 3) / 4), dim3(256), 0, st, *p);
-  else hipLaunchKernelGGL((rope_append_kernel<bf16>), dim3(p->T), dim3(256), 0, st, *p);
-  return hipGetLastError();
-}
 
 extern "C" long lsd_talk_plain_lds(const TalkParams* p) {
   return 4L * (p->H * (p->dim + p->vdim + 2 * (PLAIN_KT + 1) + 3));

@@ -210,10 +210,18 @@ __device__ __forceinline__ float silu(float x) {
   return x * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x));
 }
 
-// Gated activation of a gate / up projection whose rows miss a common factor
-// `s` (a norm's gain): silu(s g) (s u), or the tanh-GELU form.
-__device__ __forceinline__ float gated(float g, float u, int gelu, float s) {
-  return (gelu ? gelu_new(s * g) : silu(s * g)) * (s * u);
+// Gated activation of a gate / up projection.  SiLU and tanh-GELU: rows miss a
+// common factor `s` (a norm's gain), silu(s g) (s u).  Clamped: `s` is the limit,
+// g' sigmoid(1.702 g') (u' + 1) with g' = min(g, s), u' = clamp(u, -s, s).
+enum Glu : int { GLU_SILU = 0, GLU_GELU = 1, GLU_CLAMPED = 2 };
+constexpr float GLU_ALPHA = 1.702f;
+__device__ __forceinline__ float gated(float g, float u, int glu, float s) {
+  if (glu == GLU_CLAMPED) {
+    g = fminf(g, s);
+    u = fminf(fmaxf(u, -s), s);
+    return g * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * GLU_ALPHA * g)) * (u + 1.f);
+  }
+  return (glu == GLU_GELU ? gelu_new(s * g) : silu(s * g)) * (s * u);
 }
 
 // Bijective XCD-aware remap of a 1-D workgroup id (guide §5.5 T1, "XCD

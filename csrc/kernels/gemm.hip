@@ -106,7 +106,7 @@ __device__ __forceinline__ void epilogue4(const GemmParams& p, int row0, int n, 
     const int col = (n >> 5) * 16 + (n & 15);
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (row0 + i < p.M) o[(long)(row0 + i) * p.ldo + col] = f2bf(gated(v[i], v2[i], p.gelu, p.act_scale));
+      if (row0 + i < p.M) o[(long)(row0 + i) * p.ldo + col] = f2bf(gated(v[i], v2[i], p.glu, p.act_scale));
     return;
   }
   if constexpr (EPI == EPI_QKV) {
@@ -723,7 +723,7 @@ __device__ __forceinline__ void ct_store(const GemmParams& p, const float* ct, i
       const float u[8] = {ulo[0], ulo[1], ulo[2], ulo[3], uhi[0], uhi[1], uhi[2], uhi[3]};
       bf16x8 o;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] = f2bf(gated(v[e], u[e], p.gelu, p.act_scale));
+      for (int e = 0; e < 8; ++e) o[e] = f2bf(gated(v[e], u[e], p.glu, p.act_scale));
       st8(reinterpret_cast<bf16*>(p.out) + (long)m * p.ldo + (n >> 5) * 16 + (n & 15), o);
     } else {
       epilogue8<EPI>(p, m, n, v, split);
@@ -1379,7 +1379,7 @@ __global__ __launch_bounds__(512) void gemm_big_kernel(GemmParams p, int tiles_m
         const float u[8] = {ulo[0], ulo[1], ulo[2], ulo[3], uhi[0], uhi[1], uhi[2], uhi[3]};
         bf16x8 o;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) o[e] = f2bf(gated(v[e], u[e], p.gelu, p.act_scale));
+        for (int e = 0; e < 8; ++e) o[e] = f2bf(gated(v[e], u[e], p.glu, p.act_scale));
         st8(reinterpret_cast<bf16*>(p.out) + (long)m * p.ldo + (n >> 5) * 16 + (n & 15), o);
       } else {
         epilogue8<EPI>(p, m, n, v, split);
@@ -1637,7 +1637,7 @@ __global__ __launch_bounds__(512) void gemm_p8_kernel(GemmParams p, int tiles_m,
         const float u[8] = {ulo[0], ulo[1], ulo[2], ulo[3], uhi[0], uhi[1], uhi[2], uhi[3]};
         bf16x8 o;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) o[e] = f2bf(gated(v[e], u[e], p.gelu, p.act_scale));
+        for (int e = 0; e < 8; ++e) o[e] = f2bf(gated(v[e], u[e], p.glu, p.act_scale));
         st8(reinterpret_cast<bf16*>(p.out) + (long)m * p.ldo + (n >> 5) * 16 + (n & 15), o);
       } else {
         epilogue8<EPI>(p, m, n, v, split);
@@ -1862,7 +1862,7 @@ __global__ __launch_bounds__(512) void gemm_d256_kernel(GemmParams p, int* __res
       const float u[8] = {ulo[0], ulo[1], ulo[2], ulo[3], uhi[0], uhi[1], uhi[2], uhi[3]};
       bf16x8 o;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] = f2bf(gated(v[e], u[e], p.gelu, p.act_scale));
+      for (int e = 0; e < 8; ++e) o[e] = f2bf(gated(v[e], u[e], p.glu, p.act_scale));
       st8(reinterpret_cast<bf16*>(p.out) + (long)m * p.ldo + (n >> 5) * 16 + (n & 15), o);
     } else {
       epilogue8<EPI>(p, m, n, v, split);

@@ -27,8 +27,8 @@ struct GemmParams {
   // EPI_F32 (tiled kernels): also the max of every 8-column segment,
   // segmax[m * ldseg + n / 8] -- the sampler's first pass, fused (sample.hip)
   float* segmax; long ldseg;
-  // EPI_SILU_MUL: GELU instead of SiLU, and the factor of both halves (common.h gated)
-  int gelu; float act_scale;
+  // EPI_SILU_MUL: which gated activation, and the factor of both halves or the limit (common.h gated)
+  int glu; float act_scale;
 };
 
 // Small-M (M <= 8) weight-streaming GEMV with an optional fused input norm
@@ -52,7 +52,7 @@ struct GemvParams {
   // fp32 logits epilogue: also the max of every 8-column segment (one
   // workgroup = 8 columns) per row, [M][ldseg] -- the sampler's top-k threshold
   float* segmax; long ldseg;
-  int gelu; float act_scale;          // SiLU epilogue: as in GemmParams
+  int glu; float act_scale;           // SiLU epilogue: as in GemmParams
 };
 
 }  // namespace lsd

@@ -281,7 +281,7 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvParams p) {
         const int col = gw2 * (CPW / 2) + jj;
         if (m < M && col < (p.N >> 1)) {
           const float g = rv[(2 * jj) * MR + m], u = rv[(2 * jj + 1) * MR + m];
-          reinterpret_cast<bf16*>(p.out)[(long)m * p.ldo + col] = f2bf(gated(g, u, p.gelu, p.act_scale));
+          reinterpret_cast<bf16*>(p.out)[(long)m * p.ldo + col] = f2bf(gated(g, u, p.glu, p.act_scale));
         }
       } else if (e_live) {
         const int j = e_j, m = e_m, n = e_n;

@@ -343,6 +343,7 @@ __global__ __launch_bounds__(256) void group_gemm_f32_kernel(GgParams p) {
       float* o = static_cast<float*>(t.out) + orow * t.ldo + n;
       if constexpr (MODE == GG_DOWN) *o = acc[i][j] * wt;
       else if constexpr (MODE == GG_ADD) *o += acc[i][j];
+      else if constexpr (MODE == GG_F32) *o = acc[i][j] + (p.bias ? p.bias[n] : 0.f);
       else *o = acc[i][j];
     }
   }

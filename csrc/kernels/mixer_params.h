@@ -1,6 +1,6 @@
-// Launch parameters of the recurrent mixers and of attention with mixed heads,
-// shared by csrc/kernels/recurrence.hip, attention_talk.hip and
-// csrc/mixer_bindings.cpp.  "Rows" are packed tokens; the element type T is
+// Launch parameters of the recurrent mixers, of attention over a paged cache and
+// of grouped norms, shared by csrc/kernels/recurrence.hip, attention_talk.hip,
+// attention_paged.hip, norm_group.hip and csrc/mixer_bindings.cpp.  "Rows" are packed tokens; the element type T is
 // bf16 or fp32 (models served in fp32).
 #pragma once
 
@@ -58,7 +58,9 @@ struct MixOutParams {
 };
 
 // Attention over a paged cache, K [page][kv head][64][dim], V likewise with
-// vdim; scores capped, mixed over the heads, softmaxed.
+// vdim.  Scores are capped, lessened by slope_h times the distance and mixed over
+// the heads, then softmaxed -- or mixed behind the softmax (mix_weights).  A
+// query at position i sees keys j <= i with i - j < window or j < keep.
 struct TalkParams {
   const void* q;                       // [rows][H][dim]
   const void* k; const void* v;        // pools
@@ -66,8 +68,12 @@ struct TalkParams {
   const float* talk;                   // [H][H] or null
   const void* talk_frag;               // MFMA kernels: fp16 [HP][HP], zero padded (HP: H to 8 / 16 / 32)
   void* out; long ldo; int out_cols;   // [rows][H][vdim], zeros up to out_cols
-  int H, G, dim, vdim, window;         // window: keys per query (INT_MAX: all)
+  int H, G, dim, vdim, window, keep;   // window: keys per query (INT_MAX: all)
   float scale, cap;                    // cap 0: none
+  const float* slopes;                 // [H] or null
+  int mix_weights;
+  const void* gate; long ldg;          // logits of a sigmoid gate per row and head, or null
+  float* lse;                          // [rows][H] log2 of the softmax' sum (mix_weights, prompts)
   // one token alone: slot and position per row
   const int* slots; const int* pos; int T;
   // prompt tiles: (sequence, first query); sequences
@@ -77,14 +83,34 @@ struct TalkParams {
   float* part_o; float* part_ml; int splits;
 };
 
-// Rotation and cache append behind the in-projection y [rows][H dim | G dim | G vdim].
+// Behind the in-projection y [rows][H dim | G dim | G vdim]: short convolution,
+// unit RMS norms of q and k, rotation, values mixed with earlier ones, and the
+// append to the cache.
 struct RopeAppendParams {
   const void* y; long ldy; int T;
   float gain;
+  const float* taps; int n_taps;       // [channels of y][n_taps], last: the current token; null: none
+  void* ring;                          // [slots][n_taps][channels], inputs of position p at p % n_taps
+  int write_ring;                      // one token per sequence: this kernel keeps the ring
+  float eps; int dim_own;              // norms over a head's dim_own columns (the rest is padding); eps < 0: none
+  const void* v_first; float lam;      // [rows][G vdim]: v <- (1 - lam) v + lam v_first, or null
+  void* v_out;                         // [rows][G vdim]: this layer's values, or null
   const float* rope; int half;         // [positions][half][2] cos, sin; half 0: none
   void* q; void* k; void* v;
   const int* table; int tw; const int* tslot; const int* tpos;
   int H, G, dim, vdim;
+};
+
+// Norms of a row's `groups` equal parts of `size` columns (rows of H columns, the
+// rest padding).  With slabs: x += norm(sum of slabs + bias) w_post, written
+// back.  With out: out = norm(x) w_pre, padding zeroed.
+struct GroupNormParams {
+  float* x; int T, H, groups, size;
+  float eps;
+  const void* slab; int splits, slab_bf16;   // [splits][T][H] or null
+  const void* bias; const void* w_post;      // [H], element type
+  const void* w_pre; void* out;              // [H], [rows][H], element type
+  const int* rows; int n_rows;               // rows of x that are normed into out (null: all)
 };
 
 }  // namespace lsd

@@ -20,6 +20,7 @@ struct GgParams {
   void* out; long ldo;
   int M, groups;                  // GG_BATCH rows / groups
   long a_gs, o_gs;
+  const float* bias;              // GG_F32: [N] added to every row, or null (fp32 kernels)
   // experts: the row-tile table of moe_group (expert, first sorted row, rows,
   // 0), the sorted (token, choice) entries and their weights
   const int* tiles; int n_tiles;

@@ -1045,14 +1045,19 @@ __global__ __launch_bounds__(256) void loop_pack_kernel(float* __restrict__ x, c
   }
 }
 
-// fp32 gated activation over [gate | up] rows in 16-row blocks: gelu(s g) (s u), exact
-__global__ __launch_bounds__(256) void gelu_mul_f32_kernel(const float* __restrict__ y, float* __restrict__ out, long n,
-                                                           int F, long ldo, float s) {
+// fp32 gated activation over [gate | up] rows in 16-row blocks (common.h gated), exact: tanh-GELU or clamped
+__global__ __launch_bounds__(256) void glu_f32_kernel(const float* __restrict__ y, float* __restrict__ out, long n, int F,
+                                                      long ldo, int glu, float s) {
   const long i = (long)blockIdx.x * 256 + threadIdx.x;
   if (i >= n) return;
   const long row = i / F;
   const int f = i % F;
   const float* yr = y + row * 2 * F + (f >> 4) * 32 + (f & 15);
+  if (glu == GLU_CLAMPED) {
+    const float g = fminf(yr[0], s), u = fminf(fmaxf(yr[16], -s), s);
+    out[row * ldo + f] = g / (1.f + expf(-GLU_ALPHA * g)) * (u + 1.f);
+    return;
+  }
   const float g = yr[0] * s, u = yr[16] * s;
   out[row * ldo + f] = 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
 }
@@ -1187,9 +1192,9 @@ extern "C" hipError_t lsd_loop_pack(float* x, const float* x0, const float* step
   return hipGetLastError();
 }
 
-extern "C" hipError_t lsd_gelu_mul_f32(const float* y, float* out, int T, int F, long ldo, float s, hipStream_t st) {
+extern "C" hipError_t lsd_glu_f32(const float* y, float* out, int T, int F, long ldo, int glu, float s, hipStream_t st) {
   const long n = (long)T * F;
   if (n == 0) return hipSuccess;
-  hipLaunchKernelGGL(gelu_mul_f32_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, y, out, n, F, ldo, s);
+  hipLaunchKernelGGL(glu_f32_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, y, out, n, F, ldo, glu, s);
   return hipGetLastError();
 }

@@ -108,8 +108,8 @@ torch::Tensor batch_linear(torch::Tensor a, torch::Tensor w, int64_t tm) {
   return out;
 }
 
-// fp32 linear: out = a w^T (a [M, >= K], w [N, K]), or x += a w^T in place.
-torch::Tensor linear_fp32(torch::Tensor a, torch::Tensor w, Opt x) {
+// fp32 linear: out = a w^T + bias (a [M, >= K], w [N, K]), or x += a w^T in place.
+torch::Tensor linear_fp32(torch::Tensor a, torch::Tensor w, Opt x, Opt bias) {
   need(a, torch::kFloat32, "a");
   need(w, torch::kFloat32, "w");
   need_rows(a, "a");
@@ -120,6 +120,11 @@ torch::Tensor linear_fp32(torch::Tensor a, torch::Tensor w, Opt x) {
   p.A = a.data_ptr(); p.lda = a.stride(0);
   p.W = w.data_ptr(); p.ldw = w.stride(0);
   p.N = N; p.K = K; p.M = a.size(0); p.groups = 1;
+  if (bias.has_value()) {
+    need(*bias, torch::kFloat32, "bias");
+    TORCH_CHECK(!x.has_value() && bias->is_contiguous() && bias->numel() == N, "bias must be [N], not into a residual");
+    p.bias = bias->data_ptr<float>();
+  }
   torch::Tensor out;
   if (x.has_value()) {
     need(*x, torch::kFloat32, "x");
@@ -454,7 +459,8 @@ torch::Tensor embed_fp32(torch::Tensor ids, torch::Tensor wte, double scale) {
 
 void lsd_register_latent(pybind11::module& m) {
   m.def("batch_linear", &batch_linear, py::arg("a"), py::arg("w"), py::arg("tm"));
-  m.def("linear_fp32", &linear_fp32, py::arg("a"), py::arg("w"), py::arg("x") = py::none());
+  m.def("linear_fp32", &linear_fp32, py::arg("a"), py::arg("w"), py::arg("x") = py::none(),
+        py::arg("bias") = py::none());
   m.def("moe_group", &moe_group, py::arg("ids"), py::arg("experts"), py::arg("tm"));
   m.def("moe_up", &moe_up, py::arg("h"), py::arg("perm"), py::arg("tiles"), py::arg("top"), py::arg("w"),
         py::arg("limit"), py::arg("alpha"), py::arg("ws"), py::arg("limit_s"), py::arg("tm"));

@@ -1,5 +1,6 @@
-// PyTorch bindings of the recurrent mixers and of attention with mixed heads
-// (csrc/kernels/recurrence.hip, attention_talk.hip).
+// PyTorch bindings of the recurrent mixers, of attention over a paged cache and
+// of grouped norms (csrc/kernels/recurrence.hip, attention_talk.hip,
+// attention_paged.hip, norm_group.hip).
 //
 // Every entry point checks dtypes, shapes, strides and alignment on the host
 // before launching; launches go on the current stream and are graph-capturable.
@@ -15,6 +16,7 @@
 #include "kernels/mixer_params.h"
 
 using lsd::ConvParams;
+using lsd::GroupNormParams;
 using lsd::MixOutParams;
 using lsd::RecurParams;
 using lsd::RopeAppendParams;
@@ -31,7 +33,7 @@ hipError_t lsd_conv_tail(const ConvParams* c, const SeqParams* s, int f32, hipSt
 hipError_t lsd_head_norm_gate(const MixOutParams* p, int f32, hipStream_t st);
 hipError_t lsd_group_norm(const MixOutParams* p, int f32, hipStream_t st);
 hipError_t lsd_loop_pack(float* x, const float* x0, const float* step, void* out, int T, int H, int f32, hipStream_t st);
-hipError_t lsd_gelu_mul_f32(const float* y, float* out, int T, int F, long ldo, float s, hipStream_t st);
+hipError_t lsd_glu_f32(const float* y, float* out, int T, int F, long ldo, int glu, float s, hipStream_t st);
 hipError_t lsd_rope_append(const RopeAppendParams* p, int f32, hipStream_t st);
 long lsd_talk_plain_lds(const TalkParams* p);
 hipError_t lsd_talk_plain(const TalkParams* p, int f32, hipStream_t st);
@@ -39,6 +41,14 @@ int lsd_talk_heads(int H, int G, int dim, int vdim, float cap);
 int lsd_talk_tile(int hp);
 hipError_t lsd_talk_prefill(const TalkParams* p, int hp, hipStream_t st);
 hipError_t lsd_talk_decode(const TalkParams* p, int hp, hipStream_t st);
+long lsd_append_lds(const RopeAppendParams* p);
+int lsd_paged_ok(int dim, int vdim);
+hipError_t lsd_paged_prefill(const TalkParams* p, int qt, int lse, hipStream_t st);
+hipError_t lsd_paged_decode(const TalkParams* p, hipStream_t st);
+int lsd_mix_decode_gc(int H, int G);
+long lsd_mix_combine_lds(const TalkParams* p);
+hipError_t lsd_mix_decode(const TalkParams* p, hipStream_t st);
+hipError_t lsd_group_rows_norm(const GroupNormParams* p, int f32, hipStream_t st);
 }
 
 namespace {
@@ -220,14 +230,14 @@ Tensor loop_pack(Tensor x, Tensor x0, Tensor step, bool f32) {
   return out;
 }
 
-// y fp32 [T, 2F] (gate / up in 16-row blocks) -> out [T, F]
-void gelu_mul_f32(Tensor y, Tensor out, double scale) {
+// y fp32 [T, 2F] (gate / up in 16-row blocks) -> out [T, F]; glu 1 tanh-GELU, 2 clamped
+void glu_f32(Tensor y, Tensor out, int64_t glu, double scale) {
   const int64_t T = y.size(0), F = y.size(1) / 2;
   fptr(y, T * F * 2, "y");
-  TORCH_CHECK(F % 16 == 0, "gelu_mul_f32: F % 16");
+  TORCH_CHECK(F % 16 == 0 && (glu == 1 || glu == 2), "glu_f32: F % 16, GELU or clamped");
   rows_of(out, torch::kFloat32, T, F, "out");
-  check_hip(lsd_gelu_mul_f32(y.data_ptr<float>(), out.data_ptr<float>(), T, F, out.stride(0), (float)scale,
-                             cur_stream()), "gelu_mul_f32");
+  check_hip(lsd_glu_f32(y.data_ptr<float>(), out.data_ptr<float>(), T, F, out.stride(0), (int)glu, (float)scale,
+                        cur_stream()), "glu_f32");
 }
 
 void need_pools(const Tensor& k, const Tensor& v, const Tensor& table, c10::ScalarType dt) {
@@ -238,20 +248,46 @@ void need_pools(const Tensor& k, const Tensor& v, const Tensor& table, c10::Scal
               "table must be contiguous [slots, pages per sequence]");
 }
 
-// y [T, N]: q [heads dim] | k [G dim] | v [G vdim] -> rotated q [T, heads dim]; k, v appended
+// [T, G vdim] rows of values, like y
+void* value_rows(const RopeAppendParams& p, const Tensor& t, const Tensor& y, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == y.scalar_type() && t.is_contiguous() && t.dim() == 2 && t.size(0) == p.T &&
+                  t.size(1) == (int64_t)p.G * p.vdim && reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0,
+              name, " must be contiguous [T, kv heads vdim] like y");
+  return t.data_ptr();
+}
+
+// y [T, N]: q [heads dim] | k [G dim] | v [G vdim] -> q [T, heads dim]; k, v appended.
+// taps [channels, n] and ring [slots, n, channels]: a short convolution of all three
+// (write_ring: one row per sequence); eps >= 0: unit norms of q and k over dim_own
+// columns; v_first: v <- (1 - lam) v + lam v_first; v_out: v as it was before that
 Tensor rope_append(Tensor y, int64_t heads, Tensor k, Tensor v, Tensor table, Tensor tslot, Tensor tpos, Opt rope,
-                   double gain) {
+                   double gain, Opt taps, Opt ring, bool write_ring, double eps, int64_t dim_own, Opt v_first, double lam,
+                   Opt v_out) {
   const bool f32 = is_f32(y, "y");
   need_pools(k, v, table, y.scalar_type());
   RopeAppendParams p{};
   p.T = y.size(0); p.H = heads; p.G = k.size(1); p.dim = k.size(3); p.vdim = v.size(3);
-  rows_of(y, y.scalar_type(), p.T, (p.H + p.G) * p.dim + p.G * p.vdim, "y");
+  const int64_t channels = (int64_t)(p.H + p.G) * p.dim + (int64_t)p.G * p.vdim;
+  rows_of(y, y.scalar_type(), p.T, channels, "y");
   p.y = y.data_ptr(); p.ldy = y.stride(0); p.gain = (float)gain;
   if (rope.has_value()) {
     TORCH_CHECK(rope->dim() == 3 && rope->size(2) == 2 && 2 * rope->size(1) <= p.dim &&
                     rope->size(0) >= table.size(1) * (int64_t)PAGE, "rope must be [>= positions, half, 2]");
     p.rope = fptr(*rope, rope->numel(), "rope"); p.half = rope->size(1);
   }
+  if (taps.has_value()) {
+    TORCH_CHECK(ring.has_value(), "a convolution needs its ring");
+    const ConvParams c = conv(y, 0, *taps, c10::nullopt, *ring, gain);
+    TORCH_CHECK(c.channels == channels, "taps must be [", channels, ", n]");
+    p.taps = c.w; p.n_taps = c.taps; p.ring = c.ring; p.write_ring = write_ring;
+  }
+  p.eps = (float)eps;
+  p.dim_own = dim_own > 0 ? (int)dim_own : p.dim;
+  TORCH_CHECK(p.dim_own <= p.dim, "dim_own");
+  if (v_first.has_value()) p.v_first = value_rows(p, *v_first, y, "v_first");
+  if (v_out.has_value()) p.v_out = value_rows(p, *v_out, y, "v_out");
+  p.lam = (float)lam;
+  TORCH_CHECK(lsd_append_lds(&p) <= MAX_LDS, "rope_append: ", channels, " channels do not fit the LDS");
   auto q = torch::empty({p.T, heads * p.dim}, y.options());
   p.q = q.data_ptr(); p.k = k.data_ptr(); p.v = v.data_ptr();
   p.table = table.data_ptr<int>(); p.tw = table.size(1);
@@ -260,8 +296,20 @@ Tensor rope_append(Tensor y, int64_t heads, Tensor k, Tensor v, Tensor table, Te
   return q;
 }
 
+// inputs of a portion's last positions enter the convolution's ring
+void conv_tail(Tensor y, Tensor taps, Tensor ring, Tensor slots, Tensor start, Tensor cu) {
+  const bool f32 = is_f32(y, "y");
+  const ConvParams c = conv(y, 0, taps, c10::nullopt, ring, 1.0);
+  const SeqParams s = seqs(slots, start, cu);
+  check_hip(lsd_conv_tail(&c, &s, f32, cur_stream()), "conv_tail");
+}
+
+// what is beside the scores of a head: kept first tokens, distance slopes [H], gate
+// logits [T, H] (a range of wider rows)
+struct Beside { int64_t keep; Opt slopes, gate; };
+
 TalkParams talk_base(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& table, const Opt& talk, int64_t window,
-                     double scale, double cap, const Tensor& out) {
+                     double scale, double cap, const Tensor& out, const Beside& b) {
   is_f32(q, "q");
   need_pools(k, v, table, q.scalar_type());
   TalkParams p{};
@@ -278,13 +326,24 @@ TalkParams talk_base(const Tensor& q, const Tensor& k, const Tensor& v, const Te
   p.scale = (float)scale; p.cap = (float)cap;
   rows_of(out, q.scalar_type(), p.T, (int64_t)p.H * p.vdim, "out");
   p.out = out.data_ptr(); p.ldo = out.stride(0); p.out_cols = out.size(1);
+  TORCH_CHECK(b.keep >= 0 && b.keep <= INT_MAX - 64, "kept tokens");
+  p.keep = (int)b.keep;
+  if (b.slopes.has_value()) p.slopes = fptr(*b.slopes, p.H, "slopes");
+  if (b.gate.has_value()) {
+    TORCH_CHECK(b.gate->is_cuda() && b.gate->scalar_type() == q.scalar_type() && b.gate->dim() == 2 &&
+                    b.gate->size(0) == p.T && b.gate->size(1) == p.H && (p.H == 1 || b.gate->stride(1) == 1),
+                "gate must be [T, heads] like q");
+    p.gate = b.gate->data_ptr(); p.ldg = b.gate->stride(0);
+  }
+  p.splits = 1;
   return p;
 }
 
 // every row is a query of its own: slots / pos [T]
 void talk_plain(Tensor q, Tensor k, Tensor v, Tensor table, Tensor slots, Tensor pos, Opt talk, int64_t window,
-                double scale, double cap, Tensor out) {
-  TalkParams p = talk_base(q, k, v, table, talk, window, scale, cap, out);
+                double scale, double cap, Tensor out, int64_t keep, Opt slopes, Opt gate, bool mix_weights) {
+  TalkParams p = talk_base(q, k, v, table, talk, window, scale, cap, out, {keep, slopes, gate});
+  p.mix_weights = mix_weights;
   p.slots = iptr(slots, p.T, "slots"); p.pos = iptr(pos, p.T, "pos");
   TORCH_CHECK(lsd_talk_plain_lds(&p) <= MAX_LDS, "talk_plain: ", p.H, " heads of ", p.dim, " / ", p.vdim,
               " do not fit the LDS");
@@ -296,7 +355,7 @@ int frag_of(TalkParams& p, const Tensor& q, const Tensor& frag) {
   TORCH_CHECK(frag.is_cuda() && frag.scalar_type() == torch::kFloat16 && frag.is_contiguous() && frag.dim() == 2 &&
                   frag.size(0) == frag.size(1), "talk must be a contiguous fp16 [HP, HP]");
   p.talk_frag = frag.data_ptr();
-  const int hp = frag.size(0), need = lsd_talk_heads(p.H, p.G, p.dim, p.vdim, p.cap);
+  const int hp = frag.size(0), need = lsd_talk_heads(p.H, p.G, p.dim, p.vdim, p.mix_weights ? -1.f : p.cap);
   TORCH_CHECK(need > 0 && hp >= need && (hp == 8 || hp == 16 || hp == 32), "no MFMA kernel for ", p.H, " heads of ", p.dim,
               " / ", p.vdim, " with talk padded to ", hp);
   return hp;
@@ -315,8 +374,15 @@ void partials(TalkParams& p, int64_t splits, const Tensor& q, Tensor& po, Tensor
 
 // packed ragged queries; tiles [n, 2] = (sequence, first query) of talk_tile(hp) queries
 void talk_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tensor tiles, Tensor slots, Tensor start,
-                  Tensor cu, int64_t window, double scale, double cap, int64_t splits, Tensor out) {
-  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, cap, out);
+                  Tensor cu, int64_t window, double scale, double cap, int64_t splits, Tensor out, int64_t keep, Opt slopes,
+                  Opt gate, Opt lse) {
+  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, cap, out, {keep, slopes, gate});
+  if (lse.has_value()) {  // mixed weights
+    p.mix_weights = 1;
+    p.lse = const_cast<float*>(fptr(*lse, (int64_t)p.T * p.H, "lse"));
+  } else {
+    TORCH_CHECK(keep == 0 && !slopes.has_value() && !gate.has_value(), "talk_prefill: mixed scores know a window only");
+  }
   const int hp = frag_of(p, q, frag);
   Tensor po, pml;
   partials(p, splits, q, po, pml);
@@ -329,13 +395,98 @@ void talk_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tenso
 // one query per row; slots / pos [T]; hp (talk's padding) 16 or 32, G <= hp / 4
 void talk_decode(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tensor slots, Tensor pos, int64_t window,
                  double scale, double cap, int64_t splits, Tensor out) {
-  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, cap, out);
+  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, cap, out, {0, c10::nullopt, c10::nullopt});
   const int hp = frag_of(p, q, frag);
   TORCH_CHECK(hp >= 16 && 4 * p.G <= hp, "talk_decode: ", p.G, " K / V heads need talk padded to ", 4 * p.G);
   p.slots = iptr(slots, p.T, "slots"); p.pos = iptr(pos, p.T, "pos");
   Tensor po, pml;
   partials(p, splits, q, po, pml);
   check_hip(lsd_talk_decode(&p, hp, cur_stream()), "talk_decode");
+}
+
+void need_paged(const TalkParams& p, const Tensor& q, const char* what) {
+  TORCH_CHECK(q.scalar_type() == torch::kBFloat16 && lsd_paged_ok(p.dim, p.vdim), what, ": bf16 heads up to 128 columns, got ",
+              p.dim, " / ", p.vdim);
+}
+
+// packed ragged queries; tiles [n, 2] = (sequence, first query) of 64 qt queries.
+// lse (fp32 [T, heads]): log2 of the softmax sums only, no output
+void paged_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor tiles, int64_t qt, Tensor slots, Tensor start,
+                   Tensor cu, int64_t window, double scale, int64_t keep, Opt slopes, Opt gate, Tensor out, Opt lse) {
+  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, 0.0, out, {keep, slopes, gate});
+  need_paged(p, q, "paged_prefill");
+  if (lse.has_value()) p.lse = const_cast<float*>(fptr(*lse, (int64_t)p.T * p.H, "lse"));
+  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2, "tiles must be [n, 2]");
+  p.tiles = iptr(tiles, 0, "tiles"); p.n_tiles = tiles.size(0);
+  p.s = seqs(slots, start, cu);
+  check_hip(lsd_paged_prefill(&p, (int)qt, lse.has_value(), cur_stream()), "paged_prefill");
+}
+
+// one query per row; slots / pos [T]; at most 16 query heads per K / V head
+void paged_decode(Tensor q, Tensor k, Tensor v, Tensor table, Tensor slots, Tensor pos, int64_t window, double scale,
+                  int64_t keep, Opt slopes, Opt gate, int64_t splits, Tensor out) {
+  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, 0.0, out, {keep, slopes, gate});
+  need_paged(p, q, "paged_decode");
+  TORCH_CHECK(p.H / p.G <= 16, "paged_decode: at most 16 query heads per K / V head");
+  p.slots = iptr(slots, p.T, "slots"); p.pos = iptr(pos, p.T, "pos");
+  Tensor po, pml;
+  partials(p, splits, q, po, pml);
+  check_hip(lsd_paged_decode(&p, cur_stream()), "paged_decode");
+}
+
+// the same with weights mixed over the heads by talk (fp32 [heads, heads])
+void mix_decode(Tensor q, Tensor k, Tensor v, Tensor table, Tensor talk, Tensor slots, Tensor pos, int64_t window,
+                double scale, int64_t keep, Opt slopes, Opt gate, int64_t splits, Tensor out) {
+  TalkParams p = talk_base(q, k, v, table, talk, window, scale, 0.0, out, {keep, slopes, gate});
+  need_paged(p, q, "mix_decode");
+  TORCH_CHECK(lsd_mix_decode_gc(p.H, p.G) > 0, "mix_decode: no kernel for ", p.H, " heads on ", p.G);
+  p.slots = iptr(slots, p.T, "slots"); p.pos = iptr(pos, p.T, "pos");
+  TORCH_CHECK(splits >= 1 && splits <= 64, "splits");
+  p.splits = splits;
+  const int64_t n = (int64_t)p.T * p.H * splits;
+  auto po = torch::empty({n * p.G * p.vdim}, q.options().dtype(torch::kFloat32));
+  auto pml = torch::empty({n * 2}, q.options().dtype(torch::kFloat32));
+  p.part_o = po.data_ptr<float>(); p.part_ml = pml.data_ptr<float>();
+  TORCH_CHECK(lsd_mix_combine_lds(&p) <= 64 * 1024, "mix_decode: heads do not fit the LDS");
+  check_hip(lsd_mix_decode(&p, cur_stream()), "mix_decode");
+}
+
+// x [T, H] fp32, groups parts over the first `width` columns.  slab [S, T, H]: x +=
+// norm(sum + bias) w_post; w_pre: returns norm(x) w_pre (rows of x, all by default)
+Opt group_norm(Tensor x, int64_t groups, int64_t width, double eps, Opt slab, Opt bias, Opt w_post, Opt w_pre, Opt rows,
+               bool f32) {
+  const auto dt = f32 ? torch::kFloat32 : torch::kBFloat16;
+  GroupNormParams p{};
+  TORCH_CHECK(x.dim() == 2, "x must be [T, H]");
+  p.T = x.size(0); p.H = x.size(1);
+  p.x = const_cast<float*>(fptr(x, (int64_t)p.T * p.H, "x"));
+  TORCH_CHECK(groups >= 1 && width >= 1 && width <= p.H && width % groups == 0 && p.H % 4 == 0, "group_norm: ", width,
+              " columns in ", groups, " parts");
+  p.groups = groups; p.size = width / groups; p.eps = (float)eps;
+  auto vec = [&](const Tensor& t, const char* name) -> const void* {
+    TORCH_CHECK(t.is_cuda() && t.scalar_type() == dt && t.is_contiguous() && t.numel() == p.H, name, " must be [H]");
+    return t.data_ptr();
+  };
+  if (slab.has_value()) {
+    const bool sf = is_f32(*slab, "slab");
+    TORCH_CHECK(slab->is_contiguous() && slab->dim() == 3 && slab->size(0) >= 1 && slab->size(1) == p.T &&
+                    slab->size(2) == p.H && w_post.has_value() && !rows.has_value(), "slab must be [S, T, H], with w_post");
+    p.slab = slab->data_ptr(); p.splits = slab->size(0); p.slab_bf16 = !sf;
+    p.w_post = vec(*w_post, "w_post");
+    if (bias.has_value()) p.bias = vec(*bias, "bias");
+  }
+  Opt out;
+  if (rows.has_value()) {
+    p.n_rows = rows->numel();
+    p.rows = iptr(*rows, p.n_rows, "rows");
+  }
+  if (w_pre.has_value()) {
+    p.w_pre = vec(*w_pre, "w_pre");
+    out = torch::empty({p.rows ? p.n_rows : p.T, p.H}, x.options().dtype(dt));
+    p.out = out->data_ptr();
+  }
+  check_hip(lsd_group_rows_norm(&p, f32, cur_stream()), "group_norm");
+  return out;
 }
 
 }  // namespace
@@ -352,18 +503,37 @@ void lsd_register_mixers(pybind11::module& m) {
         py::arg("ring"), py::arg("state"), py::arg("A"), py::arg("dt_bias"), py::arg("skip"), py::arg("norm"),
         py::arg("gain"), py::arg("eps"), py::arg("out"), py::arg("single"), py::arg("chunked") = false);
   m.def("loop_pack", &loop_pack, py::arg("x"), py::arg("x0"), py::arg("step"), py::arg("f32"));
-  m.def("gelu_mul_f32", &gelu_mul_f32, py::arg("y"), py::arg("out"), py::arg("scale"));
+  m.def("glu_f32", &glu_f32, py::arg("y"), py::arg("out"), py::arg("glu"), py::arg("scale"));
   m.def("rope_append", &rope_append, py::arg("y"), py::arg("heads"), py::arg("k"), py::arg("v"), py::arg("table"),
-        py::arg("tslot"), py::arg("tpos"), py::arg("rope"), py::arg("gain"));
+        py::arg("tslot"), py::arg("tpos"), py::arg("rope"), py::arg("gain"), py::arg("taps") = py::none(),
+        py::arg("ring") = py::none(), py::arg("write_ring") = false, py::arg("eps") = -1.0, py::arg("dim_own") = 0,
+        py::arg("v_first") = py::none(), py::arg("lam") = 0.0, py::arg("v_out") = py::none());
+  m.def("conv_tail", &conv_tail, py::arg("y"), py::arg("taps"), py::arg("ring"), py::arg("slots"), py::arg("start"),
+        py::arg("cu"));
   m.def("talk_heads", [](int64_t H, int64_t G, int64_t dim, int64_t vdim, double cap) {
     return lsd_talk_heads(H, G, dim, vdim, (float)cap); });
   m.def("talk_tile", [](int64_t hp) { return lsd_talk_tile((int)hp); });
   m.def("talk_prefill", &talk_prefill, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("frag"),
         py::arg("tiles"), py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("window"), py::arg("scale"),
-        py::arg("cap"), py::arg("splits"), py::arg("out"));
+        py::arg("cap"), py::arg("splits"), py::arg("out"), py::arg("keep") = 0, py::arg("slopes") = py::none(),
+        py::arg("gate") = py::none(), py::arg("lse") = py::none());
   m.def("talk_decode", &talk_decode, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("frag"),
         py::arg("slots"), py::arg("pos"), py::arg("window"), py::arg("scale"), py::arg("cap"), py::arg("splits"),
         py::arg("out"));
   m.def("talk_plain", &talk_plain, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("slots"),
-        py::arg("pos"), py::arg("talk"), py::arg("window"), py::arg("scale"), py::arg("cap"), py::arg("out"));
+        py::arg("pos"), py::arg("talk"), py::arg("window"), py::arg("scale"), py::arg("cap"), py::arg("out"),
+        py::arg("keep") = 0, py::arg("slopes") = py::none(), py::arg("gate") = py::none(), py::arg("mix_weights") = false);
+  m.def("paged_ok", [](int64_t dim, int64_t vdim) { return lsd_paged_ok((int)dim, (int)vdim) != 0; });
+  m.def("paged_prefill", &paged_prefill, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("tiles"),
+        py::arg("qt"), py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("window"), py::arg("scale"),
+        py::arg("keep"), py::arg("slopes"), py::arg("gate"), py::arg("out"), py::arg("lse") = py::none());
+  m.def("paged_decode", &paged_decode, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("slots"),
+        py::arg("pos"), py::arg("window"), py::arg("scale"), py::arg("keep"), py::arg("slopes"), py::arg("gate"),
+        py::arg("splits"), py::arg("out"));
+  m.def("mix_decode_ok", [](int64_t H, int64_t G) { return lsd_mix_decode_gc((int)H, (int)G) > 0; });
+  m.def("mix_decode", &mix_decode, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("talk"),
+        py::arg("slots"), py::arg("pos"), py::arg("window"), py::arg("scale"), py::arg("keep"), py::arg("slopes"),
+        py::arg("gate"), py::arg("splits"), py::arg("out"));
+  m.def("group_norm", &group_norm, py::arg("x"), py::arg("groups"), py::arg("width"), py::arg("eps"), py::arg("slab"),
+        py::arg("bias"), py::arg("w_post"), py::arg("w_pre"), py::arg("rows"), py::arg("f32"));
 }

@@ -12,9 +12,9 @@ Device weight layout (set up once per stage by `prepare_stage`):
     q and the K cache simply live in that order.
   * Llama gate/up rows interleaved in 16-row blocks so one wave holds the gate
     and up value of the same output column (silu(gate)*up fused epilogue).
-  * Timisun, Vizalix: every width padded with zeros to what the MFMA tiles
-    want, so a model of any sizes runs (see _prepare_timisun and
-    _prepare_vizalix); fp32 or bf16.
+  * Timisun, Vizalix, Kedasun: every width padded with zeros to what the MFMA
+    tiles want, so a model of any sizes runs (see _prepare_timisun,
+    _prepare_vizalix and _prepare_kedasun); fp32 or bf16.
 """
 from __future__ import annotations
 
@@ -95,6 +95,12 @@ def interleave_experts(w: torch.Tensor, fp: int, hp: int, blk: int = 16) -> torc
     return out.reshape(*lead, 2 * fp, hp)
 
 
+def split_pairs(dim: int, dims: int) -> torch.Tensor:
+    """Order of a head's dimensions that brings interleaved pairs (2i, 2i + 1) of
+    the first `dims` to places i and i + dims / 2."""
+    return torch.cat([torch.arange(0, dims, 2), torch.arange(1, dims, 2), torch.arange(dims, dim)])
+
+
 def latent_tiles(meta, heads: int, rows: int) -> torch.Tensor:
     """(sequence, first (token, head) row) of every prefill attention tile."""
     n = np.asarray(meta.host_qlens, dtype=np.int64) * heads
@@ -145,6 +151,7 @@ class LazyNorm:
 
 # gemv epilogue codes (csrc/kernels/gemm.hip Epi)
 _EPI = {"none": 0, "gelu": 1, "silu_mul": 2}
+_GLU = {"silu_mul": 0, "gelu_mul": 1, "clamped_glu": 2}  # gated activations (common.h Glu)
 EPI_F32, EPI_RESID, EPI_QKV = 3, 4, 6
 # longest row the sampler loads once into registers (sample.hip: CH x NT x 4)
 SAMPLER_ONE_LOAD = 13 * 1024 * 4
@@ -197,6 +204,8 @@ class HipBackend(Backend):
             self._prepare_timisun(stage)
         elif cfg.arch == "vizalix":
             self._prepare_vizalix(stage)
+        elif cfg.arch == "kedasun":
+            self._prepare_kedasun(stage)
         elif stage.last:
             # pad the head IN PLACE: the stage keeps one [vocab_padded, H]
             # tensor and its weight dict points at the first V rows (a
@@ -373,6 +382,79 @@ class HipBackend(Backend):
                 out.append(pad_to(t("mlp.down_proj.weight"), hp, fp))
             w[p + "mixer.out.weight"] = torch.cat(out, 1).contiguous()
 
+    def _prepare_kedasun(self, stage) -> None:
+        """Device layout per layer (zero padding everywhere):
+          mixer.in     q | k | v | gate rows of one in-projection, dims of a head
+                       padded, rotated pairs (2i, 2i + 1) moved to (i, i + dims / 2)
+                       -- scores do not change under a common order of q and k --
+                       with its bias
+          mixer.taps   of q | k | v, fp32
+          mixer.talk   fp32, and fp16 padded for the prompt kernel
+          mlp.gate_up  interleaved in 16-row blocks
+        The share of mixed-in values stays on the host."""
+        cfg, w, dev = stage.cfg, stage.w, stage.device
+        hp = self.row_width(cfg)
+        self._ropes = {}
+        if "embed_tokens" in w:
+            w["embed_tokens"] = pad_to(w["embed_tokens"], cfg.vocab_size, hp)
+        if "lm_head" in w:
+            e = pad_to(w["lm_head"], cfg.vocab_padded, hp)
+            w["lm_head"], stage._lm_head_padded = e[: cfg.vocab_size], e
+            w["norm.weight"] = pad_to(w["norm.weight"], hp)
+        for i in stage.layers:
+            m, f, p = cfg.layers[i].mixer, cfg.layers[i].mlp, f"layers.{i}."
+            t = lambda n: w.pop(p + n)  # noqa: E731
+            dp, vp = _up(m.dim, 32), _up(m.vdim, 16)
+            heads = {"q": (m.heads, m.dim, dp), "k": (m.kv_heads, m.dim, dp), "v": (m.kv_heads, m.vdim, vp)}
+            order = None
+            if m.rope is not None and m.rope.dims:
+                order = split_pairs(m.dim, m.rope.dims).to(dev) if m.rope.interleaved else None
+                if m.rope not in self._ropes:
+                    self._ropes[m.rope] = rope_spec_table(m.rope, _up(stage.max_seq, 64), dev)
+
+            def rows(suffix: str) -> torch.Tensor:
+                """q | k | v rows, one per padded channel."""
+                out = []
+                for n, (h, d, pad) in heads.items():
+                    x = t(f"mixer.{n}{suffix}").reshape(h, d, -1)
+                    if order is not None and n != "v":
+                        x = x.index_select(1, order)
+                    out.append(pad_to(x, h, pad, x.shape[2]).reshape(h * pad, -1))
+                return torch.cat(out)
+
+            w_in = rows("")
+            channels = w_in.shape[0]
+            if m.head_gate:
+                w_in = torch.cat([w_in, t("mixer.g")])
+            n = _up(w_in.shape[0], 64)
+            w[p + "mixer.in.weight"] = pad_to(w_in, n, hp)
+            if m.bias:
+                w[p + "mixer.in.bias"] = pad_to(rows(".b")[:, 0], n)
+                w[p + "mixer.o.b"] = pad_to(w[p + "mixer.o.b"], hp)
+            if m.conv:
+                w[p + "mixer.taps"] = rows(".conv").float().contiguous()
+                assert w[p + "mixer.taps"].shape[0] == channels
+            if m.mix_values is not None:
+                w[p + "mixer.vmix"] = w[p + "mixer.vmix"].float().cpu()
+            if m.distance_bias:
+                w[p + "mixer.slopes"] = torch.tensor(m.slopes(), dtype=torch.float32, device=dev)
+            if m.talking:
+                w[p + "mixer.talk"] = talk = w[p + "mixer.talk"].float().contiguous()
+                hq = 0 if self.fp32 else self.C.talk_heads(m.heads, m.kv_heads, dp, vp, -1.0)
+                if hq and float(talk.abs().max()) < 6e4:
+                    w[p + "mixer.talk_prefill"] = pad_to(talk, hq, hq).half()
+            o = t("mixer.o").reshape(-1, m.heads, m.vdim)
+            w[p + "mixer.o"] = pad_to(pad_to(o, o.shape[0], m.heads, vp).reshape(o.shape[0], -1), hp, _up(m.heads * vp, 64))
+            for name in ("input_layernorm", "mixer.out_norm") + (("post_attention_layernorm", "mlp.out_norm") if f else ()):
+                w[p + name + ".weight"] = pad_to(w[p + name + ".weight"], hp)
+            if f is not None:
+                fp = _up(f.ff, 64)
+                w[p + "mlp.gate_up.weight"] = interleave_experts(t("mlp.gate_up.weight"), fp, hp)
+                w[p + "mlp.down_proj.weight"] = pad_to(w[p + "mlp.down_proj.weight"], hp, fp)
+
+    def value_width(self, mixer) -> int:
+        return _up(mixer.vdim, 16)
+
     @staticmethod
     def _low_rank(m) -> int:
         return _up(max(m.decay_rank, m.gate_rank), 64)
@@ -389,9 +471,9 @@ class HipBackend(Backend):
     def unit_rmsnorm(self, r: Residual, mcfg):
         return self.rmsnorm(r, self._ones, mcfg.norm_eps, width=self.norm_width(mcfg))
 
-    def _rows(self, h, w):
+    def _rows(self, h, w, b=None):
         """In-projection rows in the element type."""
-        return self.C.linear_fp32(h, w) if self.fp32 else self.linear(h, w)
+        return self.C.linear_fp32(h, w, None, b) if self.fp32 else self.linear(h, w, b)
 
     def mix(self, h, w, spec, kv, entry, meta, eps):
         """Mixer output, and room for the feed-forward's inner row behind it:
@@ -411,37 +493,124 @@ class HipBackend(Backend):
             gain, gu = float(w("post_attention_layernorm.weight")), w("mlp.gate_up.weight")
             mid = buf[:, buf.shape[1] - gu.shape[0] // 2:]
             if self.fp32:
-                self.C.gelu_mul_f32(self.C.linear_fp32(h, gu), mid, gain)
+                self.C.glu_f32(self.C.linear_fp32(h, gu), mid, _GLU["gelu_mul"], gain)
             else:
                 self.linear(h, gu, act="gelu_mul", out=mid, scale=gain)
         self.linear_residual(buf, w("mixer.out.weight"), None, r)
 
     def _attend(self, y, w, m, gain, kv, entry, meta, eps, out):
         k, v = entry
-        rope = self._ropes[m.rope] if m.rope is not None and m.rope.dims else None
-        q = self.C.rope_append(y, m.heads, k, v, kv.table, meta.token_slots, meta.token_pos, rope, gain)
-        window, cap = m.window or 1 << 30, m.softcap or 0.0
+        q = self.C.rope_append(y, m.heads, k, v, kv.table, meta.token_slots, meta.token_pos, self._rope_of(m), gain)
         for s, mt in self._parts(meta):
-            tp, td = w("mixer.talk_prefill", None), w("mixer.talk_decode", None)
-            if tp is None:
-                self.C.talk_plain(q[s], k, v, kv.table, mt.token_slots, mt.token_pos,
-                                  w("mixer.talk") if m.talking else None, window, m.scale, cap, out[s])
-            elif mt.is_decode and td is not None:
-                splits = self.R.talk_splits(mt.num_seqs, min(window, mt.max_ctx))
-                self.C.talk_decode(q[s], k, v, kv.table, td, mt.token_slots, mt.token_pos, window, m.scale, cap, splits,
-                                   out[s])
+            self._attention(q[s], w, m, k, v, kv, mt, None, out[s])
+
+    def _rope_of(self, m):
+        return self._ropes[m.rope] if m.rope is not None and m.rope.dims else None
+
+    # -- layers with norms around each sublayer (models/stage.py _sandwich_layer) ----
+    def group_norm(self, r: Residual, w, mcfg):
+        slab, bias, w_post = r.post[:3] if r.post is not None else (None, None, None)
+        r.post = None
+        return self.C.group_norm(r.x, mcfg.norm_groups, mcfg.hidden, mcfg.norm_eps, slab, bias, w_post, w, None, self.fp32)
+
+    def group_norm_rows(self, x, w, mcfg, rows=None):
+        return self.C.group_norm(x, mcfg.norm_groups, mcfg.hidden, mcfg.norm_eps, None, None, None, w, rows, self.fp32)
+
+    def linear_post_norm(self, a, w, b, norm_w, r: Residual, mcfg) -> None:
+        """x += norm(a w^T + b), left to the next group_norm or flush as the
+        projection's slabs."""
+        (M, K), N = a.shape, w.shape[0]
+        if self.fp32 or self._gemv_in(a, K, EPI_F32) is not None or (
+                not self._tiled(M, N) and self._resid_splits(M, N, K) == 1):
+            slab = self._linear_f32(a, w)[None]
+        else:
+            slab = self.C.linear_residual(a, w, None, r.x, self._resid_splits(M, N, K), self._tiled(M, N), self.counters,
+                                          True, None)
+        r.post = (slab, b, norm_w, mcfg)
+
+    def clamped_glu(self, h, w, limit: float):
+        if self.fp32:
+            y = self.C.linear_fp32(h, w)
+            out = torch.empty(y.shape[0], y.shape[1] // 2, dtype=y.dtype, device=y.device)
+            self.C.glu_f32(y, out, _GLU["clamped_glu"], limit)
+            return out
+        return self.linear(h, w, act="clamped_glu", scale=limit)
+
+    def attend(self, h, w, m, kv, entry, meta, eps, first_values, keep_values: bool = False):
+        """Attention before the output projection (heads padded), and with
+        keep_values this layer's values.  first_values: rows that are mixed into
+        the values (None: they stay as they are)."""
+        y = self._rows(h, w("mixer.in.weight"), w("mixer.in.bias", None))
+        (k, v), ring = entry[:2], entry[2] if m.conv else None
+        G, vp = v.shape[1], v.shape[3]
+        values = torch.empty(y.shape[0], G * vp, dtype=y.dtype, device=y.device) if keep_values else None
+        taps = w("mixer.taps", None)
+        q = self.C.rope_append(y, m.heads, k, v, kv.table, meta.token_slots, meta.token_pos, self._rope_of(m), 1.0, taps,
+                               ring, meta.is_decode, eps if m.qk_norm else -1.0, m.dim, first_values,
+                               0.0 if first_values is None else float(w("mixer.vmix")), values)
+        out = torch.empty(y.shape[0], w("mixer.o").shape[1], dtype=y.dtype, device=y.device)
+        c = q.shape[1] + G * (k.shape[3] + vp)
+        gate = y[:, c: c + m.heads] if m.head_gate else None
+        for s, mt in self._parts(meta):
+            if m.conv and not meta.is_decode:
+                self.C.conv_tail(y[s], taps, ring, mt.seq_slots, mt.q_start, mt.cu_q)
+            self._attention(q[s], w, m, k, v, kv, mt, None if gate is None else gate[s], out[s])
+        return out, values
+
+    def _attention(self, q, w, m, k, v, kv, mt, gate, out) -> None:
+        """One part of a step (decode rows or prompt chunks) over the cache."""
+        C, R = self.C, self.R
+        H, G, dp, vp = m.heads, k.shape[1], k.shape[3], v.shape[3]
+        window, cap, keep, slopes = m.window or 1 << 30, m.softcap or 0.0, m.keep_first, w("mixer.slopes", None)
+        ctx = min(window + keep, mt.max_ctx)
+        tp = w("mixer.talk_prefill", None)
+        rows, seqs = (mt.token_slots, mt.token_pos), (mt.seq_slots, mt.q_start, mt.cu_q)
+        at = (q, k, v, kv.table)
+        beside = (keep, slopes, gate)
+        if m.talking and not m.talk_weights and tp is not None and not keep and slopes is None and gate is None:
+            td = w("mixer.talk_decode", None)
+            if mt.is_decode and td is not None:
+                C.talk_decode(*at, td, *rows, window, m.scale, cap, R.talk_splits(mt.num_seqs, ctx), out)
             else:
-                tiles = self._query_tiles(mt, self.C.talk_tile(tp.shape[0]), q.device)
-                splits = self.R.talk_prefill_splits(tiles.shape[0], min(window, mt.max_ctx))
-                self.C.talk_prefill(q[s], k, v, kv.table, tp, tiles, mt.seq_slots, mt.q_start, mt.cu_q, window, m.scale,
-                                    cap, splits, out[s])
+                tiles = self._query_tiles(mt, C.talk_tile(tp.shape[0]), q.device)
+                C.talk_prefill(*at, tp, tiles, *seqs, window, m.scale, cap, R.talk_prefill_splits(tiles.shape[0], ctx), out)
+            return
+        mfma = not self.fp32 and m.softcap is None and C.paged_ok(dp, vp)
+        if mfma and m.talking and m.talk_weights and tp is not None:
+            if mt.is_decode and C.mix_decode_ok(H, G):
+                C.mix_decode(*at, w("mixer.talk"), *rows, window, m.scale, *beside, R.mix_splits(mt.num_seqs, ctx, H, G), out)
+                return
+            lse = torch.empty(q.shape[0], H, dtype=torch.float32, device=q.device)
+            tiles, qt = self._paged_tiles(mt, H, q.device)
+            C.paged_prefill(*at, tiles, qt, *seqs, window, m.scale, *beside, out, lse)
+            tiles = self._query_tiles(mt, C.talk_tile(tp.shape[0]), q.device)
+            C.talk_prefill(*at, tp, tiles, *seqs, window, m.scale, 0.0, R.talk_prefill_splits(tiles.shape[0], ctx), out,
+                           *beside, lse)
+        elif mfma and not m.talking:
+            if mt.is_decode and H // G <= 16:
+                C.paged_decode(*at, *rows, window, m.scale, *beside, R.paged_splits(mt.num_seqs * G, ctx), out)
+            else:
+                tiles, qt = self._paged_tiles(mt, H, q.device)
+                C.paged_prefill(*at, tiles, qt, *seqs, window, m.scale, *beside, out)
+        else:
+            C.talk_plain(*at, *rows, w("mixer.talk") if m.talking else None, window, m.scale, cap, out, *beside,
+                         m.talk_weights)
+
+    def _paged_tiles(self, meta, heads: int, device):
+        """Query tiles of the per-head prompt kernel and their size in 64 queries."""
+        qt = 2 if self._query_tiles(meta, 128, device).shape[0] * heads >= self.R.paged_tile_min else 1
+        return self._query_tiles(meta, 64 * qt, device), qt
 
     @staticmethod
     def _query_tiles(meta, rows: int, device):
         """(sequence, first query) of every `rows`-query tile, kept on the batch."""
         cache = meta.__dict__.setdefault("_query_tiles", {})
         if rows not in cache:
-            cache[rows] = latent_tiles(meta, 1, rows).to(device)
+            if meta.is_decode:  # one each; made on the device (a captured decode step may ask)
+                first = torch.arange(meta.num_seqs, dtype=torch.int32, device=device)
+                cache[rows] = torch.stack([first, torch.zeros_like(first)], 1)
+            else:
+                cache[rows] = latent_tiles(meta, 1, rows).to(device)
         return cache[rows]
 
     def _channel_delta(self, y, w, m, gain, kv, entry, meta, eps, out):
@@ -547,9 +716,9 @@ class HipBackend(Backend):
         return cache[heads]
 
     def prepare_prefill(self, meta, mcfg) -> None:
-        if mcfg.arch == "vizalix":
-            for hp in (8, 16, 32):
-                self._query_tiles(meta, self.C.talk_tile(hp), meta.cu_q.device)
+        if mcfg.arch in ("vizalix", "kedasun"):
+            for rows in {self.C.talk_tile(hp) for hp in (8, 16, 32)} | {64, 128}:
+                self._query_tiles(meta, rows, meta.cu_q.device)
             return
         if mcfg.arch != "timisun":
             meta._tiles = prefill_tiles(meta).to(meta.cu_q.device)
@@ -667,6 +836,10 @@ class HipBackend(Backend):
             self.C.norm(x, slab, pb, None, None, 0.0, True, None, False)
 
     def flush(self, r: Residual):
+        if r.post is not None:
+            slab, bias, w_post, mcfg = r.post
+            r.post = None
+            self.C.group_norm(r.x, mcfg.norm_groups, mcfg.hidden, mcfg.norm_eps, slab, bias, w_post, None, None, self.fp32)
         for slab, pb in r.pending:
             self._fold(r.x, slab, pb)
         r.pending.clear()
@@ -739,8 +912,8 @@ class HipBackend(Backend):
 
     def linear(self, a, w, b=None, act: str = "none", out=None, scale: float = 1.0):
         """act(a w^T + b) in bf16; out: the caller's rows; scale: common factor
-        of a gated activation's halves."""
-        if act == "gelu_mul" or out is not None:
+        of a gated activation's halves, or the clamped one's limit."""
+        if act in ("gelu_mul", "clamped_glu") or out is not None:
             return self._linear_into(a, w, act, out, scale)
         code = _EPI[act]
         g = self._gemv_in(a, w.shape[1], code)
@@ -762,15 +935,15 @@ class HipBackend(Backend):
         return self.C.linear(a, w, b, code, tiled, splits, self.counters)
 
     def _linear_into(self, a, w, act: str, out, scale: float):
-        gelu = act == "gelu_mul"
-        code = 2 if gelu else _EPI[act]
+        glu = _GLU.get(act)
+        code = _EPI[act] if glu is None else _EPI["silu_mul"]
         g = self._gemv_in(a, w.shape[1], code)
         if g is not None:
             x, nc, gw, gb, eps = g
-            return self.C.gemv_into(x, w, code, nc, gw, gb, eps, out, gelu, scale)
+            return self.C.gemv_into(x, w, code, nc, gw, gb, eps, out, glu or 0, scale)
         a = self.materialize(a)
         tiled, splits = self._gemm_kw(a.shape[0], w.shape[0], w.shape[1], 2 if code == 2 else 1)
-        return self.C.linear(a, w, None, 3 if gelu else code, tiled, splits, self.counters, out, scale)
+        return self.C.linear(a, w, None, code + (glu or 0), tiled, splits, self.counters, out, scale)
 
     def linear_residual(self, a, w, b, r: Residual, room=None) -> None:
         """x += a w^T + b; `room`: slab rows the caller owns and appends to

@@ -132,6 +132,14 @@ class Routing:
     talk_target: int = 512
     # ... and prompt attention with few query tiles
     talk_prefill_target: int = 512
+    # attention over paged heads without mixing: query tiles of 128 (else 64) from
+    # paged_tile_min blocks; decode waves a launch aims for, at least paged_split_keys
+    # keys each
+    paged_tile_min: int = 512
+    paged_waves: int = 2048
+    paged_split_keys: int = 128
+    # decode attention with mixed weights: blocks a launch aims for
+    mix_target: int = 512
     # -- norms / head ------------------------------------------------------
     # one wave per row from norm_wave_min rows (prefill 32 K x 1600 97.7 ->
     # 53.7 us; r5_normwave.log) and from norm_wave_narrow_min rows when H <=
@@ -310,6 +318,18 @@ class Routing:
         """Key splits of a prompt attention launch with mixed heads: few query
         tiles over long contexts, at least four 32-key tiles each."""
         return max(1, min(self.talk_prefill_target // max(1, tiles), keys // 128, 16))
+
+    def paged_splits(self, items: int, keys: int) -> int:
+        """Context splits of decode attention, a wave per (token, K / V head)."""
+        return max(1, min(math.ceil(self.paged_waves / items), math.ceil(keys / self.paged_split_keys), 64))
+
+    def mix_splits(self, B: int, keys: int, heads: int, kv_heads: int) -> int:
+        """Context splits of decode attention with mixed weights (one block per
+        token, 64-key tiles).  A split leaves partial sums of every head and K /
+        V head: heads kv_heads rows against the 64 a tile holds per K / V head."""
+        tiles = math.ceil((keys + 63) / 64) + 1
+        per = 1 if B * tiles <= self.mix_target else max(1, min(4, heads // 16 * 2))
+        return max(1, min(math.ceil(self.mix_target / B), math.ceil(tiles / per), 64))
 
     def attn_splits(self, B: int, nh: int, n_kv: int, hd: int, max_ctx: int) -> int:
         """Context splits of a decode attention launch (a graph-captured
