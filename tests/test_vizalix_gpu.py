@@ -3,8 +3,6 @@ vizalix_oracle.py: bf16 kernels with inputs rounded to bf16 first, fp32 ones at
 fp32 accuracy."""
 from __future__ import annotations
 
-import random
-
 import numpy as np
 import pytest
 import torch
@@ -13,9 +11,10 @@ from llm_sharding_demo_amd.config import EngineConfig, SamplingParams
 from llm_sharding_demo_amd.runtime.kv_cache import PAGE
 
 from . import vizalix_oracle as orc
+from .paged_helpers import (BF, F32, Batch, cuda, err, i32, ids_of, logit_err, pools, portion_steps, portions, rounded,
+                            run_steps, up)
 
 pytestmark = pytest.mark.gpu
-BF, F32 = torch.bfloat16, torch.float32
 
 
 @pytest.fixture(scope="module")
@@ -25,69 +24,7 @@ def C():
     return _load()
 
 
-def cuda(t, dt=None):
-    return t.to(device="cuda", dtype=dt if dt is not None else t.dtype).contiguous()
-
-
-def i32(v):
-    return torch.tensor(v, dtype=torch.int32, device="cuda")
-
-
-def err(got, want):
-    """Largest difference, relative to the wanted value plus the root mean square of all."""
-    want = want.double()
-    return float(((got.double().cpu() - want).abs() / (want.pow(2).mean().sqrt() + want.abs())).max())
-
-
-def rounded(t, dt):
-    return t.to(dt).double()
-
-
-class Batch:
-    """Ragged sequences of a launch: (slot, first position, tokens)."""
-
-    def __init__(self, *seqs):
-        self.seqs = seqs
-        self.n = [s[2] for s in seqs]
-        self.T = sum(self.n)
-        self.cu_host = np.concatenate([[0], np.cumsum(self.n)]).tolist()
-        self.slots, self.start, self.cu = i32([s[0] for s in seqs]), i32([s[1] for s in seqs]), i32(self.cu_host)
-        self.tslot = i32([s[0] for s in seqs for _ in range(s[2])])
-        self.tpos = i32([s[1] + j for s in seqs for j in range(s[2])])
-
-    def tiles(self, rows):
-        return i32([[i, o] for i, n in enumerate(self.n) for o in range(0, n, rows)]).reshape(-1, 2)
-
-    def rows(self, i):
-        return slice(self.cu_host[i], self.cu_host[i + 1])
-
-
 # -- attention with mixed heads ---------------------------------------------------
-
-def pools(k, v, dt, dp, vp, slots=3, seed=0):
-    """Keys / values [slot][n, G, .] in shuffled pages of padded pools, and the table."""
-    g = random.Random(seed)
-    width = max(-(-len(x) // PAGE) for x in k.values()) + 1
-    ids = list(range(slots * width))
-    g.shuffle(ids)
-    G = next(iter(k.values())).shape[1]
-    K = torch.zeros(len(ids) + 1, G, PAGE, dp, dtype=dt)
-    V = torch.zeros(len(ids) + 1, G, PAGE, vp, dtype=dt)
-    table = torch.full((slots, width), len(ids), dtype=torch.int32)
-    for s, kk in k.items():
-        for j in range(-(-len(kk) // PAGE)):
-            pg = ids.pop()
-            table[s, j] = pg
-            part = slice(j * PAGE, min(len(kk), (j + 1) * PAGE))
-            n = part.stop - part.start
-            K[pg, :, :n, : kk.shape[2]] = kk[part].transpose(0, 1).to(dt)
-            V[pg, :, :n, : v[s].shape[2]] = v[s][part].transpose(0, 1).to(dt)
-    return cuda(K), cuda(V), cuda(table)
-
-
-def up(n, m):
-    return -(-n // m) * m
-
 
 SIZES = [(6, 2, 40, 24), (4, 4, 16, 20), (3, 1, 96, 72), (16, 4, 128, 128), (12, 12, 32, 64), (32, 8, 64, 128),
          (20, 5, 128, 48), (1, 1, 64, 16), (8, 1, 128, 128), (24, 3, 72, 96)]
@@ -232,15 +169,6 @@ def test_rope_append(C, H, G, D, V, rot, dt):
 
 
 # -- recurrences ------------------------------------------------------------------
-
-def portions(n, sizes):
-    out, at = [], 0
-    for s in sizes:
-        if at < n:
-            out.append((at, min(n, at + s)))
-            at += s
-    return out + ([(at, n)] if at < n else [])
-
 
 DELTA = [(2, 2, 8, 8, 1), (4, 2, 24, 20, 3), (3, 3, 64, 64, 4), (2, 1, 128, 128, 4), (4, 4, 32, 100, 2), (2, 2, 96, 40, 4)]
 
@@ -459,36 +387,7 @@ def open_model(tmp_path, cfg, dtype, seed=0, **kw):
     return w, Engine(EngineConfig(model_id=str(tmp_path), weights=str(tmp_path), dtype=dtype, device="cuda", **kw))
 
 
-def ids_of(n, vocab=200, seed=0):
-    r = random.Random(seed)
-    return [r.randrange(vocab) for _ in range(n)]
-
-
-def logit_err(got, want):
-    """Worst row's root mean square difference over the logits' own."""
-    d = got.double() - want
-    return float((d - d.mean(-1, keepdim=True)).pow(2).mean(-1).sqrt().max() / want.std())
-
-
 LIMIT = {"bf16": 0.08, "fp32": 5e-5}
-
-
-def run_steps(ses, seqs, steps):
-    """steps: [[(id, tokens), ...], ...] -> {id: logits of all its tokens}."""
-    at, out = dict.fromkeys(seqs, 0), {k: [] for k in seqs}
-    for st in steps:
-        ent = [{"id": k, "tokens": seqs[k][at[k]: at[k] + n], "want": list(range(n))} for k, n in st]
-        for k, n in st:
-            at[k] += n
-        got = ses.step(ent, [k for k, _ in st if at[k] == len(seqs[k])])
-        for k, n in st:
-            out[k].append(got[:n])
-            got = got[n:]
-    return {k: torch.cat(v) for k, v in out.items() if v}
-
-
-def portion_steps(rid, n, sizes):
-    return [[(rid, b - a)] for a, b in portions(n, list(sizes) + [1] * n)]
 
 
 @pytest.mark.parametrize("dtype", ["bf16", "fp32"])
