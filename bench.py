@@ -68,7 +68,7 @@ def parse():
                         "nothing measurable on one stage or in the 2/4-stage loopback rehearsal "
                         "(profiles/r2_prefill_chunk.log)")
     p.add_argument("--designs", default="",
-                   help="comma-separated presets with per-layer specs (timisun-2b, vizalix-2b, ...): instead of the "
+                   help="comma-separated presets with per-layer specs (timisun-2b, vizalix-2b, kedasun-2b, ...): instead of the "
                         "headline, prefill and decode throughput of each beside a Llama-family model of equal "
                         "width, depth, heads and active feed-forward (one GPU; one JSON line per model and batch)")
     p.add_argument("--design-batches", default="1,32,256")

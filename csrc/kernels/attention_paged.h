@@ -42,6 +42,18 @@ __device__ __forceinline__ float head_gate(const TalkParams& p, long row, int h)
   return p.gate ? sigmoid_x(to_f(static_cast<const T*>(p.gate)[row * p.ldg + h])) : 1.f;
 }
 
+typedef _Float16 half8 __attribute__((ext_vector_type(8)));
+typedef _Float16 half4 __attribute__((ext_vector_type(4)));
+typedef _Float16 half2 __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ half2 pack_half(float a, float b) {  // rounds towards zero
+  const auto h = __builtin_amdgcn_cvt_pkrtz(a, b);
+  return __builtin_bit_cast(half2, h);
+}
+
+__device__ __forceinline__ f32x4 mfma_f16(half8 a, half8 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0);
+}
+
 // Transposed read of 4 x 16 LDS blocks: k runs over rows, the result's lanes over columns.
 __device__ __forceinline__ bf16x4 ds_read_tr(const bf16* lds_ptr) {
   typedef __attribute__((address_space(3))) bf16x4 lds_bf16x4;

@@ -4,6 +4,8 @@
 //  * rope_append_vec, conv_append, append_plain: behind the in-projection.
 //  * paged_prefill: MFMA flash attention, 128 (64) queries of a head per block; or
 //    only log2 of the softmax sums, for weights that are mixed over the heads.
+//  * mix_prefill: MFMA, 16 queries of 4 heads per wave, all heads in a block, with
+//    weights mixed over the heads.
 //  * paged_decode: MFMA, a token's queries of one K / V head per wave.
 //  * mix_decode, mix_combine: MFMA, one token of all heads per block.  With
 //    W_g the unnormalised weights of head g over a block's keys,
@@ -37,7 +39,7 @@ __device__ __forceinline__ void mix_value(const RopeAppendParams& p, long row, i
 }
 
 // 8 columns per thread; dims and the rotation's half are multiples of 8.  One
-// block per four tokens, a wave each.
+// block per four tokens, a wave each (several where tokens are few: blockIdx.y).
 __global__ __launch_bounds__(256) void rope_append_vec_kernel(RopeAppendParams p) {
   const long row = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= p.T) return;
@@ -46,7 +48,7 @@ __global__ __launch_bounds__(256) void rope_append_vec_kernel(RopeAppendParams p
   const int nq = p.H * p.dim, nk = p.G * p.dim, nv = p.G * p.vdim;
   const bf16* y = static_cast<const bf16*>(p.y) + row * p.ldy;
   const float* cs = p.rope + (long)pos * half * 2;
-  for (int i = lane_id() * 8; i < nq + nk + nv; i += 512) {
+  for (int i = blockIdx.y * 512 + lane_id() * 8; i < nq + nk + nv; i += 512 * gridDim.y) {
     const bf16x8 x = ld8(y + i);
     float v[8];
 #pragma unroll
@@ -99,11 +101,10 @@ __global__ __launch_bounds__(256) void append_plain_kernel(RopeAppendParams p) {
   for (int i = tid; i < n; i += 256) {
     float v = to_f(y[i]) * p.gain;
     if (p.taps) {
-      const float* w = p.taps + (long)i * p.n_taps;
       v = 0.f;
       for (int j = 0; j < p.n_taps; ++j) {
         const T* src = conv_input<T>(p, row, slot, pos, p.n_taps - 1 - j, i, n);
-        if (src) v = fmaf(w[j], to_f(*src) * p.gain, v);
+        if (src) v = fmaf(p.taps[(long)j * n + i], to_f(*src) * p.gain, v);
       }
       if (p.write_ring) static_cast<T*>(p.ring)[((long)slot * p.n_taps + pos % p.n_taps) * n + i] = y[i];
     }
@@ -139,9 +140,9 @@ __global__ __launch_bounds__(256) void append_plain_kernel(RopeAppendParams p) {
 }
 
 // Convolution (at most four taps), unit norms, value mixing, append: LPH lanes of
-// 8 columns hold one head, `run` rows in turn; the taps and the last three inputs
-// stay in registers.
-template <int LPH>
+// 8 columns hold one head, `run` rows in turn, FLY of one portion together; the taps
+// and the last three inputs stay in registers.
+template <int LPH, int FLY>
 __global__ __launch_bounds__(256) void conv_append_kernel(RopeAppendParams p, int run) {
   const int units = p.H + 2 * p.G, lane = threadIdx.x % LPH;
   const long item = (long)blockIdx.x * (256 / LPH) + threadIdx.x / LPH;
@@ -157,41 +158,23 @@ __global__ __launch_bounds__(256) void conv_append_kernel(RopeAppendParams p, in
   const bool mine = d < width;  // lanes behind the head's columns repeat its last ones
   float w[4][8];                // w[back]
 #pragma unroll
-  for (int e = 0; e < 8; ++e)
+  for (int back = 0; back < 4; ++back) {
+    const f32x4* t = reinterpret_cast<const f32x4*>(p.taps + (long)max(0, p.n_taps - 1 - back) * channels + ch);
+    const f32x4 a = t[0], b = t[1];
+    const float f = back < p.n_taps ? p.gain : 0.f;
 #pragma unroll
-    for (int back = 0; back < 4; ++back)
-      w[back][e] = back < p.n_taps ? p.taps[(long)(ch + e) * p.n_taps + p.n_taps - 1 - back] * p.gain : 0.f;
-  float past[3][8];
-  int slot = -1, pos = -2;
-  long page = 0;
-  for (int i = 0; i < run; ++i) {  // equal trip counts: lanes exchange below
-    const bool on = i < n_rows;
-    const long row = row0 + (on ? i : 0);
-    const int sl = p.tslot[row], ps = p.tpos[row];
-    const bf16x8 x = ld8(static_cast<const bf16*>(p.y) + row * p.ldy + ch);
-    if (on && (sl != slot || ps != pos + 1)) {
-#pragma unroll
-      for (int back = 1; back < 4; ++back) {
-        bf16x8 z = {};
-        if (back < p.n_taps) {
-          const bf16* src = conv_input<bf16>(p, row, sl, ps, back, ch, channels);
-          if (src) z = ld8(src);
-        }
-#pragma unroll
-        for (int e = 0; e < 8; ++e) past[back - 1][e] = bf2f(z[e]);
-      }
+    for (int e = 0; e < 4; ++e) {
+      w[back][e] = a[e] * f;
+      w[back][4 + e] = b[e] * f;
     }
-    if (on && (sl != slot || ps / PAGE != pos / PAGE || pos < 0)) page = p.table[(long)sl * p.tw + ps / PAGE];
-    slot = sl;
-    pos = ps;
+  }
+  // convolution, norm and stores of one row; x[0] its input, x[1 ..] the ones before
+  auto emit = [&](const bf16x8& x0, const bf16x8& x1, const bf16x8& x2, const bf16x8& x3, bool on, long row, int slot, int pos,
+                  long page) {
     float v[8], ss = 0.f;
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-      const float now = bf2f(x[e]);
-      v[e] = fmaf(w[3][e], past[2][e], fmaf(w[2][e], past[1][e], fmaf(w[1][e], past[0][e], w[0][e] * now)));
-      past[2][e] = past[1][e];
-      past[1][e] = past[0][e];
-      past[0][e] = now;
+      v[e] = fmaf(w[3][e], bf2f(x3[e]), fmaf(w[2][e], bf2f(x2[e]), fmaf(w[1][e], bf2f(x1[e]), w[0][e] * bf2f(x0[e]))));
       ss = fmaf(v[e], mine ? v[e] : 0.f, ss);
     }
     if (p.eps >= 0.f) {
@@ -204,16 +187,60 @@ __global__ __launch_bounds__(256) void conv_append_kernel(RopeAppendParams p, in
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] *= rs;
     }
-    if (!on || !mine) continue;
-    if (p.write_ring) st8(static_cast<bf16*>(p.ring) + ((long)sl * p.n_taps + ps % p.n_taps) * channels + ch, x);
+    if (!on || !mine) return;
+    if (p.write_ring) st8(static_cast<bf16*>(p.ring) + ((long)slot * p.n_taps + pos % p.n_taps) * channels + ch, x0);
     if (is_v) mix_value(p, row, ch - nq - nk, v);
-    bf16x8 o;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) o[e] = f2bf(v[e]);
+    const bf16x4 lo = pack4(f32x4{v[0], v[1], v[2], v[3]}), hi = pack4(f32x4{v[4], v[5], v[6], v[7]});
     bf16* dst = is_q ? static_cast<bf16*>(p.q) + row * nq + ch
-                : is_v ? static_cast<bf16*>(p.v) + ((page * p.G + u - p.H - p.G) * PAGE + ps % PAGE) * p.vdim + d
-                       : static_cast<bf16*>(p.k) + ((page * p.G + u - p.H) * PAGE + ps % PAGE) * p.dim + d;
-    st8(dst, o);
+                : is_v ? static_cast<bf16*>(p.v) + ((page * p.G + u - p.H - p.G) * PAGE + pos % PAGE) * p.vdim + d
+                       : static_cast<bf16*>(p.k) + ((page * p.G + u - p.H) * PAGE + pos % PAGE) * p.dim + d;
+    st8(dst, bf16x8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
+  };
+  auto before = [&](long row, int slot, int pos, int back) {
+    const bf16x8 z = {};
+    if (back >= p.n_taps) return z;
+    const bf16* src = conv_input<bf16>(p, row, slot, pos, back, ch, channels);
+    return src ? ld8(src) : z;
+  };
+  const bf16* y = static_cast<const bf16*>(p.y) + ch;
+  bf16x8 x1, x2, x3;  // the inputs before the next row
+  int slot = -1, pos = -2;
+  for (int i = 0; i < run; i += FLY) {
+    const long row = row0 + i;
+    if (i + FLY <= n_rows && p.tslot[row + FLY - 1] == p.tslot[row] && p.tpos[row + FLY - 1] == p.tpos[row] + FLY - 1) {
+      // rows of one portion (equal for all lanes of a head)
+      bf16x8 x[FLY];
+#pragma unroll
+      for (int j = 0; j < FLY; ++j) x[j] = ld8(y + (row + j) * p.ldy);
+      const int sl = p.tslot[row], ps = p.tpos[row];
+      const int* table = p.table + (long)sl * p.tw;
+      const long page0 = table[ps / PAGE], page1 = table[(ps + FLY - 1) / PAGE];
+      if (sl != slot || ps != pos + 1) {
+        x1 = before(row, sl, ps, 1);
+        x2 = before(row, sl, ps, 2);
+        x3 = before(row, sl, ps, 3);
+      }
+#pragma unroll
+      for (int j = 0; j < FLY; ++j) {
+        emit(x[j], x1, x2, x3, true, row + j, sl, ps + j, (ps + j) / PAGE == ps / PAGE ? page0 : page1);
+        x3 = x2;
+        x2 = x1;
+        x1 = x[j];
+      }
+      slot = sl;
+      pos = ps + FLY - 1;
+    } else {
+#pragma unroll 1
+      for (int j = 0; j < FLY; ++j) {
+        const bool on = i + j < n_rows;
+        const long rw = on ? row + j : row0;
+        const int sl = p.tslot[rw], ps = p.tpos[rw];
+        emit(ld8(y + rw * p.ldy), before(rw, sl, ps, 1), before(rw, sl, ps, 2), before(rw, sl, ps, 3), on, rw, sl, ps,
+             p.table[(long)sl * p.tw + ps / PAGE]);
+      }
+      slot = -1;
+      pos = -2;
+    }
   }
 }
 
@@ -408,6 +435,229 @@ __global__ __launch_bounds__(256, 2) void paged_prefill_kernel(TalkParams p) {
   }
 }
 
+// Weights mixed over the heads, the softmax sums known (lse).  HP / 4 waves share 16
+// queries, each scores its 4 heads and writes their weights (times 2^WSHIFT, which
+// keeps small ones within fp16; two fp16 terms) to LDS.  Barrier.  Each wave then
+// mixes the weights of all heads for some of the tile's 32 keys -- a product
+// T [16 heads][heads] . weights [heads][16 queries] per key -- and writes the result
+// (two bf16 terms) as the operand fragments of the second product.  Barrier.  Each
+// wave multiplies its own heads' values.  Tile buffers:
+//   S  [key][(term, 8 heads) HP / 4][query 16]   16-byte chunks of 8 heads; the two
+//      4-head halves change places with bit 2 of the key, which spreads the banks
+//   P  [term][head][k-slot group 4][query 16]    16-byte chunks of 8 keys: slot j of
+//      group k <-> key 4 k + j (j < 4), 16 + 4 k + j - 4
+// Wave w of a group mixes the keys of k-slot group w % 4 (and w + 2 with two waves).
+constexpr float WSHIFT = 12.f, WUNIT = 1.f / 4096.f;
+template <int DKS, int VT, int HP>
+__global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void mix_prefill_kernel(TalkParams p) {
+  constexpr int TK = 32, HW = HP / 4, NW = HW > 4 ? HW : 4, QG = NW / HW;
+  constexpr int KCH = HP / 4 * 16;          // chunks of one key
+  constexpr int SETS = HW == 2 ? 2 : 1;     // k-slot groups a wave mixes
+  constexpr int VROW = 64;                  // staged V columns, 16-byte chunks swizzled by the row
+  __shared__ __attribute__((aligned(16))) _Float16 ss[QG][TK * KCH * 8];
+  __shared__ __attribute__((aligned(16))) bf16 pp[QG][2][HP * 64 * 8];
+  __shared__ __attribute__((aligned(16))) bf16 vst[NW][TK * VROW];
+  const int tile = xcd_remap(blockIdx.x, gridDim.x);
+  const int seq = p.tiles[2 * tile], off = p.tiles[2 * tile + 1];
+  const int cu = p.s.cu[seq], qlen = p.s.cu[seq + 1] - cu, st = p.s.start[seq];
+  const int* table = p.table + (long)p.s.slots[seq] * p.tw;
+  const bf16* K = static_cast<const bf16*>(p.k);
+  const bf16* V = static_cast<const bf16*>(p.v);
+  const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int hw = w % HW, qg = w / HW, H = p.H, G = p.G, rep = H / G, dim = p.dim, vdim = p.vdim;
+  _Float16* sb = ss[qg];
+  bf16* p_hi = pp[qg][0];
+  bf16* p_lo = pp[qg][1];
+  bf16* vs = vst[w];
+
+  const int qi = off + qg * 16 + r, qc = min(qi, qlen - 1);
+  const int my_pos = st + qc, my_lo = first_key(my_pos, p.window);
+  const float scale2 = LOG2E * p.scale;
+  int kv[4];
+  float lse[4], slope[4];
+#pragma unroll
+  for (int hh = 0; hh < 4; ++hh) {
+    const int h = min(hw * 4 + hh, H - 1);
+    kv[hh] = h / rep;
+    lse[hh] = p.lse[(long)(cu + qc) * H + h] - WSHIFT;
+    slope[hh] = p.slopes ? p.slopes[h] * LOG2E : 0.f;
+  }
+  const int q_at = (cu + qc) * H * dim + g * 8;
+  // rows of T for this wave's product: k-slots hold 8 heads of the chunk lane group g reads
+  const int set0 = hw % 4, mt = HP == 32 ? hw / 4 : 0;
+  half8 tf = {};
+  {
+    const int trow = mt * 16 + r, tcol = HP == 32 ? g * 8 : HP == 16 ? (g & 1) * 8 : 0;
+    if (trow < HP && (HP > 8 || g < 2))
+      tf = *reinterpret_cast<const half8*>(static_cast<const _Float16*>(p.talk_frag) + trow * HP + tcol);
+    if (set0 & 1) tf = half8{tf[4], tf[5], tf[6], tf[7], tf[0], tf[1], tf[2], tf[3]};
+  }
+
+  f32x4 o[4][VT];
+#pragma unroll
+  for (int hh = 0; hh < 4; ++hh)
+#pragma unroll
+    for (int di = 0; di < VT; ++di) o[hh][di] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const KeyTiles kts = key_tiles<TK>(st + off, st + min(off + QG * 16, qlen) - 1, p.window, p.keep);
+  int it0 = 0, it1 = kts.count();
+  if (p.splits > 1) {
+    const int per = (it1 + p.splits - 1) / p.splits;
+    it0 = blockIdx.y * per;
+    it1 = min(it1, it0 + per);
+  }
+  bf16x8 kf[2][DKS], vr[4];
+  auto load_k = [&](int kt, int kvh) {
+    const bf16* kp = K + (((long)table[kt * TK / PAGE] * G + kvh) * PAGE + kt * TK % PAGE + r) * dim + g * 8;
+    const bf16x8 z = {};
+#pragma unroll
+    for (int ni = 0; ni < 2; ++ni)
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks) kf[ni][ks] = ks * 32 < dim ? ld8(kp + ni * 16 * dim + ks * 32) : z;
+  };
+  auto load_v = [&](int kt, int kvh, int vh) {  // 64 columns of the tile's rows, 16 bytes per lane and 8 rows
+    const bf16* vp = V + (((long)table[kt * TK / PAGE] * G + kvh) * PAGE + kt * TK % PAGE) * vdim + vh * 64;
+    const int col = (lane & 7) * 8;
+    const bf16x8 z = {};
+#pragma unroll
+    for (int c = 0; c < 4; ++c) vr[c] = vh * 64 + col < vdim ? ld8(vp + (c * 8 + (lane >> 3)) * vdim + col) : z;
+  };
+  const int s_wr = (hw >> 1) * 128 + r * 8;        // + key, term, half
+  const int r0 = 4 * g + (r >> 2), sw = (r0 >> 1) & 7;
+  if (it0 < it1) load_k(kts.at(it0), kv[0]);
+  for (int it = it0; it < it1; ++it) {
+    const int kt = kts.at(it), next = kts.at(min(it + 1, it1 - 1));
+    // scores of the own heads; the queries are read again for every tile (from
+    // L1 / L2): the outputs take the registers
+    f32x4 s[4][2];
+    const bf16* qb = static_cast<const bf16*>(p.q);
+    asm volatile("" : "+s"(qb));  // not hoisted out of the loop
+#pragma unroll
+    for (int hh = 0; hh < 4; ++hh) {
+      if (hh > 0 && kv[hh] != kv[hh - 1]) load_k(kt, kv[hh]);  // wave-uniform
+      const bf16x8 z = {};
+      bf16x8 qf[DKS];
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks) qf[ks] = ks * 32 < dim ? ld8(qb + q_at + min(hw * 4 + hh, H - 1) * dim + ks * 32) : z;
+#pragma unroll
+      for (int ni = 0; ni < 2; ++ni) {
+        s[hh][ni] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < DKS; ++ks) s[hh][ni] = mfma16(kf[ni][ks], qf[ks], s[hh][ni]);
+      }
+    }
+    const bool whole = (kt * TK >= my_lo || kt * TK + TK <= p.keep) && kt * TK + TK - 1 <= my_pos;
+    const bool all_whole = __all(whole);
+#pragma unroll
+    for (int ni = 0; ni < 2; ++ni)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int in = ni * 16 + 4 * g + i, key = kt * TK + in;
+        const float dist = (float)(key - my_pos);
+        float e[4];
+#pragma unroll
+        for (int hh = 0; hh < 4; ++hh)
+          e[hh] = __builtin_amdgcn_exp2f(fmaf(s[hh][ni][i], scale2, fmaf(slope[hh], dist, -lse[hh])));
+        if (!all_whole && !seen(key, my_pos, my_lo, p.keep)) e[0] = e[1] = e[2] = e[3] = 0.f;
+        // the remainder makes up for the truncated first term
+        const half2 a = pack_half(e[0], e[1]), b = pack_half(e[2], e[3]);
+        const half2 c = pack_half(e[0] - (float)a[0], e[1] - (float)a[1]), d = pack_half(e[2] - (float)b[0], e[3] - (float)b[1]);
+        const int at = in * KCH * 8 + s_wr + ((hw ^ g) & 1) * 4;  // bit 2 of the key is g & 1
+        *reinterpret_cast<half4*>(sb + at) = half4{a[0], a[1], b[0], b[1]};
+        *reinterpret_cast<half4*>(sb + at + HP / 8 * 128) = half4{c[0], c[1], d[0], d[1]};
+      }
+    __syncthreads();
+#pragma unroll
+    for (int q = 0; q < SETS; ++q) {
+      const int set = set0 + 2 * q;
+      f32x4 acc[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const int in = (j < 4 ? 0 : 16) + 4 * set + (j & 3);
+        const _Float16* src = sb + (in * KCH + g * 16 + r) * 8;
+        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+        half8 a = {};
+        if (HP > 8 || g < 2) a = *reinterpret_cast<const half8*>(src);
+        acc[j] = mfma_f16(tf, a, zero);
+        if constexpr (HP == 32) acc[j] = mfma_f16(tf, *reinterpret_cast<const half8*>(src + 4 * 128), acc[j]);
+      }
+      if (q == SETS - 1) load_v(kt, kv[0], 0);  // in flight until the barrier
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int h = mt * 16 + 4 * g + i;
+        const float x[4] = {acc[0][i], acc[1][i], acc[2][i], acc[3][i]}, y[4] = {acc[4][i], acc[5][i], acc[6][i], acc[7][i]};
+        u32x4 hi, lo;
+        split_p(x, y, hi, lo);
+        if (HP > 8 || g < 2) {
+          *reinterpret_cast<u32x4*>(p_hi + ((h * 4 + set) * 16 + r) * 8) = hi;
+          *reinterpret_cast<u32x4*>(p_lo + ((h * 4 + set) * 16 + r) * 8) = lo;
+        }
+      }
+    }
+    __syncthreads();
+    load_k(next, kv[0]);  // in flight under the product
+#pragma unroll
+    for (int hh = 0; hh < 4; ++hh) {
+      if (hh > 0 && kv[hh] == kv[hh - 1]) continue;  // done with the head before
+      if (hh > 0) load_v(kt, kv[hh], 0);
+#pragma unroll
+      for (int vh = 0; vh < VT / 4; ++vh) {
+        if (vh * 64 >= vdim) continue;
+        lds_fence();  // reads of what is staged now are done
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+          const int row = c * 8 + (lane >> 3);
+          st8(vs + row * VROW + (((lane & 7) ^ ((row >> 1) & 7)) * 8), vr[c]);
+        }
+        if ((vh + 1) * 64 < vdim) load_v(kt, kv[hh], vh + 1);
+        lds_fence();
+        bf16x8 vf[4];
+#pragma unroll
+        for (int dj = 0; dj < 4; ++dj) {
+          const bf16* vp = vs + r0 * VROW + (((dj * 2 + ((r & 3) >> 1)) ^ sw) * 8) + (r & 1) * 4;
+          const bf16x4 a = ds_read_tr(vp);
+          const bf16x4 b = ds_read_tr(vp + 16 * VROW);
+          vf[dj] = bf16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+        }
+#pragma unroll
+        for (int h2 = 0; h2 < 4; ++h2)
+          if (h2 >= hh && kv[h2] == kv[hh]) {  // wave-uniform
+            const int at = (((hw * 4 + h2) * 4 + g) * 16 + r) * 8;
+            const bf16x8 ph = ld8(p_hi + at), pl = ld8(p_lo + at);
+#pragma unroll
+            for (int dj = 0; dj < 4; ++dj) {
+              o[h2][vh * 4 + dj] = mfma16(vf[dj], ph, o[h2][vh * 4 + dj]);
+              o[h2][vh * 4 + dj] = mfma16(vf[dj], pl, o[h2][vh * 4 + dj]);
+            }
+          }
+      }
+    }
+  }
+#pragma unroll
+  for (int hh = 0; hh < 4; ++hh) {
+    const int h = hw * 4 + hh;
+    if (h >= H || qi >= qlen) continue;
+    if (p.splits > 1) {  // the partial sums of key splits simply add up: equal maxima, sums of 1 in all
+      const long pi = ((long)(cu + qi) * H + h) * p.splits + blockIdx.y;
+#pragma unroll
+      for (int di = 0; di < VT; ++di)
+        if (di * 16 < vdim) *reinterpret_cast<f32x4*>(p.part_o + pi * vdim + di * 16 + 4 * g) = o[hh][di] * WUNIT;
+      if (g == 0) {
+        p.part_ml[2 * pi] = 0.f;
+        p.part_ml[2 * pi + 1] = 1.f / p.splits;
+      }
+      continue;
+    }
+    const float f = WUNIT * head_gate<bf16>(p, cu + qi, h);
+    bf16* out = static_cast<bf16*>(p.out) + (long)(cu + qi) * p.ldo + h * vdim;
+#pragma unroll
+    for (int di = 0; di < VT; ++di)
+      if (di * 16 < vdim) st4(out + di * 16 + 4 * g, pack4(o[hh][di] * f));
+  }
+  if (p.splits == 1 && hw == HW - 1 && qi < qlen)
+    for (int c = H * vdim + g; c < p.out_cols; c += 4) static_cast<bf16*>(p.out)[(long)(cu + qi) * p.ldo + c] = f2bf(0.f);
+}
+
 // -- decode ----------------------------------------------------------------------
 
 // One wave per (token, K / V head, key split): its rep <= 16 queries are the
@@ -551,16 +801,17 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(TalkParams p) {
     for (int c = p.H * p.vdim + lane; c < p.out_cols; c += 64) out[c] = f2bf(0.f);
 }
 
-// One token of all heads per block and key split, 64-key tiles (pages).  Wave w
-// owns K / V heads w, w + 4, ..: it scores their queries and writes the weights
+// One token of all heads per block and key split, 64-key tiles (pages).  Wave w of
+// NW owns K / V heads w, w + NW, ..: it scores their queries and writes the weights
 // (two bf16 terms) to LDS; behind the barrier it multiplies its heads' values by
 // the weights of all MT x 16 query heads.  LDS weights are double-buffered, so a
-// tile has one barrier.
-template <int DKS, int VT, int MT, int GC>
-__global__ __launch_bounds__(256, 2) void mix_decode_kernel(TalkParams p) {
-  constexpr int HP = MT * 16, PLD = PAGE + 8;
+// tile has one barrier.  In flight: the next K rows under the weights and their
+// product, the next V rows under a product with the ones before.
+template <int DKS, int VT, int MT, int GC, int NW>
+__global__ __launch_bounds__(NW * 64, 2) void mix_decode_kernel(TalkParams p) {
+  constexpr int HP = MT * 16, PLD = PAGE + 8, STEPS = VT / 4 * 2;
   __shared__ __attribute__((aligned(16))) bf16 p_hi[2][HP * PLD], p_lo[2][HP * PLD];
-  __shared__ __attribute__((aligned(16))) bf16 vst[4][32 * VLD];
+  __shared__ __attribute__((aligned(16))) bf16 vst[NW][32 * VLD];
   __shared__ float alphas[2][HP];
   const int b = blockIdx.x, H = p.H, G = p.G, rep = H / G, dim = p.dim, vdim = p.vdim;
   const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -581,14 +832,15 @@ __global__ __launch_bounds__(256, 2) void mix_decode_kernel(TalkParams p) {
   for (int c = 0; c < GC; ++c) {
     m[c] = NEG;
     lsum[c] = 0.f;
-    slope2[c] = p.slopes ? p.slopes[min((w + 4 * c) * rep + min(r, rep - 1), H - 1)] * LOG2E : 0.f;
+    slope2[c] = p.slopes ? p.slopes[min((w + NW * c) * rep + min(r, rep - 1), H - 1)] * LOG2E : 0.f;
 #pragma unroll
     for (int mt = 0; mt < MT; ++mt)
 #pragma unroll
       for (int di = 0; di < VT; ++di) o[c][mt][di] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
-  bf16x8 vr[4];
-  auto load_v = [&](long page, int kvh, int vh, int kk) {
+  bf16x8 vr[4], kf[4][DKS];
+  auto load_v = [&](long page, int kvh, int step) {
+    const int vh = step >> 1, kk = step & 1;
     const bf16* vp = V + ((page * G + kvh) * PAGE + kk * 32) * vdim + vh * 64;
     const bf16x8 z = {};
 #pragma unroll
@@ -597,22 +849,26 @@ __global__ __launch_bounds__(256, 2) void mix_decode_kernel(TalkParams p) {
       vr[q4] = vh * 64 + col < vdim ? ld8_nt(vp + (long)row * vdim + col) : z;
     }
   };
+  auto load_k = [&](long page, int kvh) {
+    const bf16* kp = K + ((page * G + kvh) * PAGE + r) * dim + g * 8;
+    const bf16x8 z = {};
+#pragma unroll
+    for (int ni = 0; ni < 4; ++ni)
+#pragma unroll
+      for (int ks = 0; ks < DKS; ++ks) kf[ni][ks] = ks * 32 < dim ? ld8_nt(kp + (long)ni * 16 * dim + ks * 32) : z;
+  };
+  if (it0 < it1 && w < G) load_k(table[kts.at(it0)], w);
   for (int it = it0; it < it1; ++it) {
     const int kt = kts.at(it), buf = it & 1;
-    const long page = table[kt];
+    const long page = table[kt], next = table[kts.at(min(it + 1, it1 - 1))];
 #pragma unroll
     for (int c = 0; c < GC; ++c) {
-      const int kvh = w + 4 * c;
+      const int kvh = w + NW * c;
       if (kvh >= G) continue;  // wave-uniform
       const int h = kvh * rep + min(r, rep - 1);
       const bf16* q = static_cast<const bf16*>(p.q) + ((long)b * H + h) * dim + g * 8;
-      const bf16* kp = K + ((page * G + kvh) * PAGE + r) * dim + g * 8;
       const bf16x8 z = {};
-      bf16x8 qf[DKS], kf[4][DKS];
-#pragma unroll
-      for (int ni = 0; ni < 4; ++ni)
-#pragma unroll
-        for (int ks = 0; ks < DKS; ++ks) kf[ni][ks] = ks * 32 < dim ? ld8_nt(kp + (long)ni * 16 * dim + ks * 32) : z;
+      bf16x8 qf[DKS];
 #pragma unroll
       for (int ks = 0; ks < DKS; ++ks) qf[ks] = ks * 32 < dim ? ld8(q + ks * 32) : z;
       f32x4 s[4];
@@ -630,7 +886,9 @@ __global__ __launch_bounds__(256, 2) void mix_decode_kernel(TalkParams p) {
           tmax = fmaxf(tmax, s[ni][i]);
         }
       }
-      if (c == 0) load_v(page, kvh, 0, 0);  // in flight under the softmax and the barrier
+      if (c == 0) load_v(page, kvh, 0);
+      if (c + 1 < GC && kvh + NW < G) load_k(page, kvh + NW);
+      else load_k(next, w);
       tmax = fmaxf(tmax, wave_xchg<16>(tmax));
       tmax = fmaxf(tmax, wave_xchg<32>(tmax));
       const float mn = tmax > m[c] + 6.f ? tmax : m[c];  // every tile holds a visible key
@@ -662,7 +920,7 @@ __global__ __launch_bounds__(256, 2) void mix_decode_kernel(TalkParams p) {
     for (int mt = 0; mt < MT; ++mt) al[mt] = mt * 16 + r < H ? alphas[buf][mt * 16 + r] : 1.f;
 #pragma unroll
     for (int c = 0; c < GC; ++c) {
-      const int kvh = w + 4 * c;
+      const int kvh = w + NW * c;
       if (kvh >= G) continue;
 #pragma unroll
       for (int mt = 0; mt < MT; ++mt)
@@ -671,13 +929,14 @@ __global__ __launch_bounds__(256, 2) void mix_decode_kernel(TalkParams p) {
           for (int di = 0; di < VT; ++di) o[c][mt][di] *= al[mt];
         }
 #pragma unroll
-      for (int step = 0; step < VT / 4 * 2; ++step) {
+      for (int step = 0; step < STEPS; ++step) {
         const int vh = step >> 1, kk = step & 1;
         if (vh * 64 >= vdim) continue;
-        if (c > 0 || step > 0) load_v(page, kvh, vh, kk);
         lds_fence();  // reads of what is staged now are done
 #pragma unroll
         for (int q4 = 0; q4 < 4; ++q4) st8(vs + (q4 * 8 + (lane >> 3)) * VLD + (lane & 7) * 8, vr[q4]);
+        if (step + 1 < STEPS && ((step + 1) >> 1) * 64 < vdim) load_v(page, kvh, step + 1);
+        else if (c + 1 < GC && kvh + NW < G) load_v(page, kvh + NW, 0);
         bf16x8 hf[MT], lf[MT];
 #pragma unroll
         for (int mt = 0; mt < MT; ++mt) {  // heads behind H read stale columns, which nobody stores
@@ -707,7 +966,7 @@ __global__ __launch_bounds__(256, 2) void mix_decode_kernel(TalkParams p) {
   const long part = (long)b * p.splits + blockIdx.y;
 #pragma unroll
   for (int c = 0; c < GC; ++c) {
-    const int kvh = w + 4 * c;
+    const int kvh = w + NW * c;
     if (kvh >= G) continue;
 #pragma unroll
     for (int mt = 0; mt < MT; ++mt) {
@@ -728,50 +987,57 @@ __global__ __launch_bounds__(256, 2) void mix_decode_kernel(TalkParams p) {
 }
 
 // out_h = gate_h sum_g T_hg sum_s e^{m_gs - M_g} / L_g  part_s[kv(h)][g], one block
-// per (token, K / V head).  Dynamic LDS: factors [H][splits], merged rows [H][vdim].
+// per (token, K / V head) and MIX_COLS columns.  Dynamic LDS: factors [H][splits],
+// merged rows [H][MIX_COLS].
+constexpr int MIX_COLS = 32;
 __global__ __launch_bounds__(256) void mix_combine_kernel(TalkParams p) {
   extern __shared__ float sh[];
+  constexpr int N4 = MIX_COLS / 4, FLY = 8;
   const int H = p.H, G = p.G, S = p.splits, vdim = p.vdim, rep = H / G, tid = threadIdx.x;
-  const int b = blockIdx.x / G, kvh = blockIdx.x % G;
-  float* rows = sh;            // [H][vdim]
-  float* cf = sh + H * vdim;   // [H][S]
-  for (int gq = tid; gq < H; gq += 256) {
+  const int b = blockIdx.x / G, kvh = blockIdx.x % G, col0 = blockIdx.y * MIX_COLS;
+  float* rows = sh;              // [H][MIX_COLS]
+  float* cf = sh + H * MIX_COLS; // [H][S]
+  for (int g0 = 0; g0 < H; g0 += 32) {  // eight lanes per head, all lanes stay
+    const int gq = min(g0 + (tid >> 3), H - 1), l8 = tid & 7;
     const float* ml = p.part_ml + 2 * ((long)b * S * H + gq);
     float M = NEG, L = 0.f;
-    for (int s = 0; s < S; ++s) M = fmaxf(M, ml[2L * s * H]);
-    for (int s = 0; s < S; ++s) {
-      const float e = exp2f(ml[2L * s * H] - M);
-      cf[gq * S + s] = e;
-      L += ml[2L * s * H + 1] * e;
-    }
-    for (int s = 0; s < S; ++s) cf[gq * S + s] /= L;
+    for (int s = l8; s < S; s += 8) M = fmaxf(M, ml[2L * s * H]);
+    M = fmaxf(M, wave_xchg<1>(M));
+    M = fmaxf(M, wave_xchg<2>(M));
+    M = fmaxf(M, wave_xchg<4>(M));
+    for (int s = l8; s < S; s += 8) L += ml[2L * s * H + 1] * exp2f(ml[2L * s * H] - M);
+    L += wave_xchg<1>(L);
+    L += wave_xchg<2>(L);
+    L += wave_xchg<4>(L);
+    if (g0 + (tid >> 3) < H)
+      for (int s = l8; s < S; s += 8) cf[gq * S + s] = exp2f(ml[2L * s * H] - M) / L;
   }
   __syncthreads();
-  const int n4 = vdim / 4;
-  for (int i = tid; i < H * n4; i += 256) {
-    const int gq = i / n4;
-    const float* po = p.part_o + (((long)b * S * G + kvh) * H) * vdim + 4L * i;
+  for (int i = tid; i < H * N4; i += 256) {
+    const int gq = i / N4, d = col0 + i % N4 * 4;
+    const float* po = p.part_o + (((long)b * S * G + kvh) * H + gq) * vdim + min(d, vdim - 4);
     f32x4 a = {0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < S; s += 4) {  // four loads in flight
-      f32x4 x[4];
+    for (int s = 0; s < S; s += FLY) {
+      f32x4 x[FLY];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) x[j] = *reinterpret_cast<const f32x4*>(po + (long)min(s + j, S - 1) * G * H * vdim);
+      for (int j = 0; j < FLY; ++j) x[j] = *reinterpret_cast<const f32x4*>(po + (long)min(s + j, S - 1) * G * H * vdim);
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
+      for (int j = 0; j < FLY; ++j)
         if (s + j < S) a += x[j] * cf[gq * S + s + j];
     }
     *reinterpret_cast<f32x4*>(rows + 4 * i) = a;
   }
   __syncthreads();
   bf16* out = static_cast<bf16*>(p.out) + (long)b * p.ldo;
-  for (int i = tid; i < rep * n4; i += 256) {
-    const int h = kvh * rep + i / n4, d = i % n4 * 4;
+  for (int i = tid; i < rep * N4; i += 256) {
+    const int h = kvh * rep + i / N4, c = i % N4 * 4, d = col0 + c;
+    if (d >= vdim) continue;
     const float* t = p.talk + (long)h * H;
     f32x4 a = {0.f, 0.f, 0.f, 0.f};
-    for (int gq = 0; gq < H; ++gq) a += *reinterpret_cast<const f32x4*>(rows + gq * vdim + d) * t[gq];
+    for (int gq = 0; gq < H; ++gq) a += *reinterpret_cast<const f32x4*>(rows + gq * MIX_COLS + c) * t[gq];
     st4(out + h * vdim + d, pack4(a * head_gate<bf16>(p, b, h)));
   }
-  if (kvh == G - 1)
+  if (kvh == G - 1 && blockIdx.y == 0)
     for (int c = H * vdim + tid; c < p.out_cols; c += 256) out[c] = f2bf(0.f);
 }
 
@@ -788,20 +1054,26 @@ extern "C" hipError_t lsd_rope_append(const RopeAppendParams* p, int f32, hipStr
   if (p->T == 0) return hipSuccess;
   const bool vec = !f32 && p->dim % 8 == 0 && p->vdim % 8 == 0;
   if (vec && !p->taps && p->eps < 0.f && p->half % 8 == 0) {
-    hipLaunchKernelGGL(rope_append_vec_kernel, dim3((p->T + 3) / 4), dim3(256), 0, st, *p);
+    const int cols = (p->H + p->G) * p->dim + p->G * p->vdim;
+    hipLaunchKernelGGL(rope_append_vec_kernel, dim3((p->T + 3) / 4, p->T <= 512 ? (cols + 511) / 512 : 1), dim3(256), 0, st, *p);
     return hipGetLastError();
   }
   const int wide = p->dim > p->vdim ? p->dim : p->vdim;
   if (vec && p->taps && p->n_taps <= 4 && p->half == 0 && wide <= 256) {
-    const int run = p->T >= 4096 ? 16 : p->T >= 512 ? 4 : 1, lph = wide <= 32 ? 4 : wide <= 64 ? 8 : wide <= 128 ? 16 : 32;
+    const int run = p->T >= 4096 ? 32 : p->T >= 512 ? 4 : 1, lph = wide <= 32 ? 4 : wide <= 64 ? 8 : wide <= 128 ? 16 : 32;
     const long items = (long)((p->T + run - 1) / run) * (p->H + 2 * p->G);
     const dim3 grid((unsigned)((items * lph + 255) / 256));
+#define LSD_CA(L)                                                                             \
+  if (run >= 32) hipLaunchKernelGGL((conv_append_kernel<L, 8>), grid, dim3(256), 0, st, *p, run); \
+  else if (run == 4) hipLaunchKernelGGL((conv_append_kernel<L, 4>), grid, dim3(256), 0, st, *p, run); \
+  else hipLaunchKernelGGL((conv_append_kernel<L, 1>), grid, dim3(256), 0, st, *p, run);
     switch (lph) {
-      case 4: hipLaunchKernelGGL((conv_append_kernel<4>), grid, dim3(256), 0, st, *p, run); break;
-      case 8: hipLaunchKernelGGL((conv_append_kernel<8>), grid, dim3(256), 0, st, *p, run); break;
-      case 16: hipLaunchKernelGGL((conv_append_kernel<16>), grid, dim3(256), 0, st, *p, run); break;
-      default: hipLaunchKernelGGL((conv_append_kernel<32>), grid, dim3(256), 0, st, *p, run);
+      case 4: LSD_CA(4) break;
+      case 8: LSD_CA(8) break;
+      case 16: LSD_CA(16) break;
+      default: LSD_CA(32)
     }
+#undef LSD_CA
     return hipGetLastError();
   }
   const size_t lds = lsd_append_lds(p);
@@ -846,6 +1118,26 @@ extern "C" hipError_t lsd_paged_prefill(const TalkParams* p, int qt, int lse, hi
   return hipGetLastError();
 }
 
+// hp: 8, 16 or 32 (talk_frag padded to it)
+extern "C" hipError_t lsd_mix_prefill(const TalkParams* p, int hp, hipStream_t st) {
+  if (p->n_tiles == 0) return hipSuccess;
+  const dim3 grid(p->n_tiles, p->splits);
+#define LSD_MP(HP, NT)                                                                                                 \
+  if (p->dim <= 64 && p->vdim <= 64) hipLaunchKernelGGL((mix_prefill_kernel<2, 4, HP>), grid, dim3(NT), 0, st, *p); \
+  else if (p->dim <= 64) hipLaunchKernelGGL((mix_prefill_kernel<2, 8, HP>), grid, dim3(NT), 0, st, *p);             \
+  else if (p->vdim <= 64) hipLaunchKernelGGL((mix_prefill_kernel<4, 4, HP>), grid, dim3(NT), 0, st, *p);            \
+  else hipLaunchKernelGGL((mix_prefill_kernel<4, 8, HP>), grid, dim3(NT), 0, st, *p);
+  switch (hp) {
+    case 8: LSD_MP(8, 256) break;
+    case 16: LSD_MP(16, 256) break;
+    case 32: LSD_MP(32, 512) break;
+    default: return hipErrorInvalidValue;
+  }
+#undef LSD_MP
+  if (p->splits > 1) return lsd_attention_combine(p, st);
+  return hipGetLastError();
+}
+
 extern "C" hipError_t lsd_paged_decode(const TalkParams* p, hipStream_t st) {
   if (p->T == 0) return hipSuccess;
   const dim3 grid((unsigned)(((long)p->T * p->G + 3) / 4), p->splits);
@@ -862,33 +1154,36 @@ extern "C" hipError_t lsd_paged_decode(const TalkParams* p, hipStream_t st) {
   return hipGetLastError();
 }
 
-// K / V heads per wave of mix_decode, 0: no kernel
+// Waves per block times K / V heads per wave of mix_decode cover G; 0: no kernel
+static int mix_waves(int G) { return G > 4 ? 8 : 4; }
 extern "C" int lsd_mix_decode_gc(int H, int G) {
   if (H > 32 || H / G > 16) return 0;
-  const int gc = (G + 3) / 4, mt = H <= 16 ? 1 : 2;
-  return gc * mt > 4 ? 0 : gc <= 2 ? gc : 4;
+  const int gc = (G + mix_waves(G) - 1) / mix_waves(G);
+  return gc * (H <= 16 ? 1 : 2) > 4 ? 0 : gc <= 2 ? gc : 4;
 }
 
-extern "C" long lsd_mix_combine_lds(const TalkParams* p) { return 4L * p->H * (p->vdim + p->splits); }
+extern "C" long lsd_mix_combine_lds(const TalkParams* p) { return 4L * p->H * (MIX_COLS + p->splits); }
 
 extern "C" hipError_t lsd_mix_decode(const TalkParams* p, hipStream_t st) {
   if (p->T == 0) return hipSuccess;
   const dim3 grid(p->T, p->splits);
-  const int gc = lsd_mix_decode_gc(p->H, p->G), mt = p->H <= 16 ? 1 : 2;
-#define LSD_MD(MT, GC)                                                                                              \
-  if (p->dim <= 64 && p->vdim <= 64) hipLaunchKernelGGL((mix_decode_kernel<2, 4, MT, GC>), grid, dim3(256), 0, st, *p); \
-  else if (p->dim <= 64) hipLaunchKernelGGL((mix_decode_kernel<2, 8, MT, GC>), grid, dim3(256), 0, st, *p);         \
-  else if (p->vdim <= 64) hipLaunchKernelGGL((mix_decode_kernel<4, 4, MT, GC>), grid, dim3(256), 0, st, *p);        \
-  else hipLaunchKernelGGL((mix_decode_kernel<4, 8, MT, GC>), grid, dim3(256), 0, st, *p);
-  switch (gc * 4 + mt) {
-    case 5: LSD_MD(1, 1) break;
-    case 9: LSD_MD(1, 2) break;
-    case 17: LSD_MD(1, 4) break;
-    case 6: LSD_MD(2, 1) break;
-    case 10: LSD_MD(2, 2) break;
+  const int gc = lsd_mix_decode_gc(p->H, p->G), mt = p->H <= 16 ? 1 : 2, nw = mix_waves(p->G);
+#define LSD_MD(MT, GC, NW)                                                                                                 \
+  if (p->dim <= 64 && p->vdim <= 64) hipLaunchKernelGGL((mix_decode_kernel<2, 4, MT, GC, NW>), grid, dim3(NW * 64), 0, st, *p); \
+  else if (p->dim <= 64) hipLaunchKernelGGL((mix_decode_kernel<2, 8, MT, GC, NW>), grid, dim3(NW * 64), 0, st, *p);         \
+  else if (p->vdim <= 64) hipLaunchKernelGGL((mix_decode_kernel<4, 4, MT, GC, NW>), grid, dim3(NW * 64), 0, st, *p);        \
+  else hipLaunchKernelGGL((mix_decode_kernel<4, 8, MT, GC, NW>), grid, dim3(NW * 64), 0, st, *p);
+  switch (nw * 16 + gc * 4 + mt) {
+    case 64 + 5: LSD_MD(1, 1, 4) break;
+    case 64 + 6: LSD_MD(2, 1, 4) break;
+    case 128 + 5: LSD_MD(1, 1, 8) break;
+    case 128 + 6: LSD_MD(2, 1, 8) break;
+    case 128 + 9: LSD_MD(1, 2, 8) break;
+    case 128 + 10: LSD_MD(2, 2, 8) break;
     default: return hipErrorInvalidValue;
   }
 #undef LSD_MD
-  hipLaunchKernelGGL(mix_combine_kernel, dim3(p->T * p->G), dim3(256), lsd_mix_combine_lds(p), st, *p);
+  hipLaunchKernelGGL(mix_combine_kernel, dim3(p->T * p->G, (p->vdim + MIX_COLS - 1) / MIX_COLS), dim3(256),
+                     lsd_mix_combine_lds(p), st, *p);
   return hipGetLastError();
 }

@@ -1,19 +1,17 @@
-// Attention over a paged K / V cache with a learned [H][H] matrix that mixes
-// over the heads: capped scores in front of the softmax, or the weights behind
-// it; grouped K / V heads and a sliding window.
+// Attention over a paged K / V cache whose capped scores are mixed over the heads by
+// a learned [H][H] matrix before the softmax, with grouped K / V heads and a sliding
+// window (mixed weights and no mixing: attention_paged.hip).
 //
 //  * talk_prefill: MFMA, 16 queries of 4 heads per wave, all heads in a block.
-//  * talk_decode: MFMA, one token of all heads per block, keys split over blocks
-//    (scores mixed; mixed weights: attention_paged.hip).
-//  * talk_plain: one token per block, any sizes, bf16 or fp32, and without mixing.
+//  * talk_decode: MFMA, one token of all heads per block, keys split over blocks.
+//  * talk_plain: one token per block, any sizes, bf16 or fp32, mixed scores, mixed
+//    weights or neither.
 //
 // Every head's score of a (query, key) pair is needed before any head's weight
-// of it is known, so a block works on all heads of its queries.  Scores (bounded
-// by the cap) or softmax weights cross the waves through LDS as two fp16 terms
-// (value and remainder, 22 bits) and are mixed by the matrix cores in fp32; what
-// multiplies the values enters the second product as two bf16 terms.  Weights
-// can be mixed once they are normalised: attention_paged.hip's prompt kernel
-// gives log2 of every softmax sum first.
+// of it is known, so a block works on all heads of its queries.  Scores cross
+// the waves through LDS as two fp16 terms (value and remainder, 22 bits: the cap
+// bounds them) and are mixed by the matrix cores in fp32; softmax weights enter
+// the second product as two bf16 terms.
 #include "attention_paged.h"
 
 namespace lsd {
@@ -119,18 +117,6 @@ __global__ __launch_bounds__(256) void talk_plain_kernel(TalkParams p) {
   }
 }
 
-typedef _Float16 half8 __attribute__((ext_vector_type(8)));
-typedef _Float16 half4 __attribute__((ext_vector_type(4)));
-typedef _Float16 half2 __attribute__((ext_vector_type(2)));
-__device__ __forceinline__ half2 pack_half(float a, float b) {  // rounds towards zero
-  const auto h = __builtin_amdgcn_cvt_pkrtz(a, b);
-  return __builtin_bit_cast(half2, h);
-}
-
-__device__ __forceinline__ f32x4 mfma_f16(half8 a, half8 b, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0);
-}
-
 // cap tanh(x): `two_over` is 2 log2(e) scale / cap, the factor of the raw product
 __device__ __forceinline__ float capped(float raw, float two_over, float cap) {
   const float t = __builtin_amdgcn_exp2f(raw * two_over);
@@ -160,10 +146,7 @@ __device__ __forceinline__ void transpose_groups(u32x4 (&x)[4]) {
 // all keys of query r, head g) -> barrier -> softmax in the lane, weights
 // transposed between lane groups and registers, second product per head.  Few
 // queries: the keys are split over blockIdx.y, partial outputs combined after.
-// WTS: what crosses and is mixed are softmax weights (times 2^WSHIFT, which keeps
-// small ones within fp16), and the product with the values follows at once.
-constexpr float WSHIFT = 12.f, WUNIT = 1.f / 4096.f;
-template <int DKS, int VT, int HP, bool WTS>
+template <int DKS, int VT, int HP>
 __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_prefill_kernel(TalkParams p) {
   constexpr int TK = 32, HW = HP / 4, NW = HW > 4 ? HW : 4, QG = NW / HW;
   constexpr int PITCH = HP == 8 ? 8 : HP + 8;  // fp16 scores of one pair
@@ -199,22 +182,13 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
 #pragma unroll
     for (int di = 0; di < VT; ++di) o[hh][di] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = NEG, lsum = 0.f;
-  const float two_over = 2.f * LOG2E * p.scale / p.cap, scale2 = LOG2E * p.scale;
-  float lse[4], slope[4];
-  if constexpr (WTS) {
-#pragma unroll
-    for (int hh = 0; hh < 4; ++hh) {
-      const int h = min(hw * 4 + hh, H - 1);
-      lse[hh] = p.lse[(long)(cu + qc) * H + h] - WSHIFT;
-      slope[hh] = p.slopes ? p.slopes[h] * LOG2E : 0.f;
-    }
-  }
-  const KeyTiles kts = key_tiles<TK>(st + off, st + min(off + QG * 16, qlen) - 1, p.window, p.keep);
-  int it0 = 0, it1 = kts.count();
+  const float two_over = 2.f * LOG2E * p.scale / p.cap;
+  const int lo = first_key(st + off, p.window), hi = st + min(off + QG * 16, qlen);
+  int kt0 = lo / TK, kt1 = (hi + TK - 1) / TK;
   if (p.splits > 1) {
-    const int per = (it1 + p.splits - 1) / p.splits;
-    it0 = blockIdx.y * per;
-    it1 = min(it1, it0 + per);
+    const int per = (kt1 - kt0 + p.splits - 1) / p.splits;
+    kt0 += blockIdx.y * per;
+    kt1 = min(kt1, kt0 + per);
   }
   // 64 columns of the tile's V rows, 16 bytes per lane and 8 rows
   bf16x8 vr[4];
@@ -228,12 +202,9 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
     }
   };
 
-  for (int it = it0; it < it1; ++it) {
-    const int kt = kts.at(it);
+  for (int kt = kt0; kt < kt1; ++kt) {
     const long page = table[kt * TK / PAGE];
     const int koff = (kt * TK) % PAGE;
-    const bool whole = (kt * TK >= my_lo || kt * TK + TK <= p.keep) && kt * TK + TK - 1 <= my_pos;
-    const bool all_whole = __all(whole);
     // scores of the own heads; the queries are read again for every tile (from
     // L1 / L2): the outputs take the registers
     f32x4 s[4][2];
@@ -266,19 +237,9 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         half4 a, b;
-        const int key = kt * TK + ni * 16 + 4 * g + i;
-        const bool hide = WTS && !all_whole && !seen(key, my_pos, my_lo, p.keep);
-        auto crossing = [&](int hh) {
-          if constexpr (WTS) {
-            const float x = fmaf(s[hh][ni][i], scale2, fmaf(slope[hh], (float)(key - my_pos), -lse[hh]));
-            return hide ? 0.f : __builtin_amdgcn_exp2f(x);
-          } else {
-            return capped(s[hh][ni][i], two_over, p.cap);
-          }
-        };
 #pragma unroll
         for (int hh = 0; hh < 4; hh += 2) {  // the remainder makes up for the truncated first term
-          const float c = crossing(hh), d = crossing(hh + 1);
+          const float c = capped(s[hh][ni][i], two_over, p.cap), d = capped(s[hh + 1][ni][i], two_over, p.cap);
           const half2 u = pack_half(c, d), v = pack_half(c - (float)u[0], d - (float)u[1]);
           a[hh] = u[0];
           a[hh + 1] = u[1];
@@ -302,43 +263,42 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
       acc = mfma_f16(tf, a, acc);
       acc = mfma_f16(tf, b, acc);
-      e[key] = WTS ? acc[0] : acc[0] * LOG2E;
+      e[key] = acc[0] * LOG2E;
     }
     __syncthreads();  // the next tile's scores may be written
-    if constexpr (!WTS) {
-      if (!all_whole) {
-#pragma unroll
-        for (int key = 0; key < TK; ++key) {
-          const int k = kt * TK + key;
-          e[key] = k >= my_lo && k <= my_pos ? e[key] : NEG;
-        }
-      }
-      float tmax = e[0];
-#pragma unroll
-      for (int key = 1; key < TK; ++key) tmax = fmaxf(tmax, e[key]);
-      // weights are taken relative to m, which follows the running maximum only
-      // when that is more than 2^6 ahead
-      if (__any(tmax > m + 6.f)) {
-        const float mn = fmaxf(m, tmax);
-        const float alpha = __builtin_amdgcn_exp2f(m - mn);
-        m = mn;
-        lsum *= alpha;
-#pragma unroll
-        for (int hh = 0; hh < 4; ++hh) {
-          const float ah = __shfl(alpha, hh * 16 + r, 64);
-#pragma unroll
-          for (int di = 0; di < VT; ++di) o[hh][di] *= ah;
-        }
-      }
-      const float off2 = m > 0.5f * NEG ? m : 0.f;  // no key seen yet: weights of zero
-      float ps = 0.f;
+    const bool whole = kt * TK >= my_lo && kt * TK + TK - 1 <= my_pos;
+    if (!__all(whole)) {
 #pragma unroll
       for (int key = 0; key < TK; ++key) {
-        e[key] = __builtin_amdgcn_exp2f(e[key] - off2);
-        ps += e[key];
+        const int k = kt * TK + key;
+        e[key] = k >= my_lo && k <= my_pos ? e[key] : NEG;
       }
-      lsum += ps;
     }
+    float tmax = e[0];
+#pragma unroll
+    for (int key = 1; key < TK; ++key) tmax = fmaxf(tmax, e[key]);
+    // weights are taken relative to m, which follows the running maximum only
+    // when that is more than 2^6 ahead
+    if (__any(tmax > m + 6.f)) {
+      const float mn = fmaxf(m, tmax);
+      const float alpha = __builtin_amdgcn_exp2f(m - mn);
+      m = mn;
+      lsum *= alpha;
+#pragma unroll
+      for (int hh = 0; hh < 4; ++hh) {
+        const float ah = __shfl(alpha, hh * 16 + r, 64);
+#pragma unroll
+        for (int di = 0; di < VT; ++di) o[hh][di] *= ah;
+      }
+    }
+    const float off2 = m > 0.5f * NEG ? m : 0.f;  // no key seen yet: weights of zero
+    float ps = 0.f;
+#pragma unroll
+    for (int key = 0; key < TK; ++key) {
+      e[key] = __builtin_amdgcn_exp2f(e[key] - off2);
+      ps += e[key];
+    }
+    lsum += ps;
     // k-slot j of group g <-> key 4 g + j (j < 4), 16 + 4 g + (j - 4) (j >= 4)
     u32x4 ph[4], pl[4];
 #pragma unroll
@@ -374,14 +334,6 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
       }
     }
   }
-  if constexpr (WTS) {  // the partial sums of key splits simply add up: equal maxima, sums of 1 in all
-    m = 0.f;
-    lsum = 1.f / p.splits;
-#pragma unroll
-    for (int hh = 0; hh < 4; ++hh)
-#pragma unroll
-      for (int di = 0; di < VT; ++di) o[hh][di] *= WUNIT;
-  }
   if (p.splits > 1) {
 #pragma unroll
     for (int hh = 0; hh < 4; ++hh) {
@@ -404,8 +356,8 @@ __global__ __launch_bounds__(HP == 32 ? 512 : 256, HP == 32 ? 1 : 2) void talk_p
   bf16* out = static_cast<bf16*>(p.out) + (long)(cu + qc) * p.ldo;
 #pragma unroll
   for (int hh = 0; hh < 4; ++hh) {
+    const float ih = __shfl(inv, hh * 16 + r, 64);
     const int h = hw * 4 + hh;
-    const float ih = __shfl(inv, hh * 16 + r, 64) * head_gate<bf16>(p, cu + qc, min(h, H - 1));
     if (h >= H || qi >= qlen) continue;
 #pragma unroll
     for (int di = 0; di < VT; ++di) {
@@ -706,13 +658,11 @@ extern "C" hipError_t lsd_attention_combine(const TalkParams* p, hipStream_t st)
 extern "C" hipError_t lsd_talk_prefill(const TalkParams* p, int hp, hipStream_t st) {
   if (p->n_tiles == 0) return hipSuccess;
   const dim3 grid(p->n_tiles, p->splits);
-  switch (hp + (p->mix_weights ? 1 : 0)) {
-    case 8: LSD_TK_V(talk_prefill_kernel, grid, 256, 8, false) break;
-    case 16: LSD_TK_V(talk_prefill_kernel, grid, 256, 16, false) break;
-    case 32: LSD_TK_V(talk_prefill_kernel, grid, 512, 32, false) break;
-    case 9: LSD_TK_V(talk_prefill_kernel, grid, 256, 8, true) break;
-    case 17: LSD_TK_V(talk_prefill_kernel, grid, 256, 16, true) break;
-    case 33: LSD_TK_V(talk_prefill_kernel, grid, 512, 32, true) break;
+  if (p->mix_weights) return hipErrorInvalidValue;
+  switch (hp) {
+    case 8: LSD_TK_V(talk_prefill_kernel, grid, 256, 8) break;
+    case 16: LSD_TK_V(talk_prefill_kernel, grid, 256, 16) break;
+    case 32: LSD_TK_V(talk_prefill_kernel, grid, 512, 32) break;
     default: return hipErrorInvalidValue;
   }
   if (p->splits > 1) return lsd_attention_combine(p, st);

@@ -89,7 +89,7 @@ struct TalkParams {
 struct RopeAppendParams {
   const void* y; long ldy; int T;
   float gain;
-  const float* taps; int n_taps;       // [channels of y][n_taps], last: the current token; null: none
+  const float* taps; int n_taps;       // [n_taps][channels of y], last: the current token; null: none
   void* ring;                          // [slots][n_taps][channels], inputs of position p at p % n_taps
   int write_ring;                      // one token per sequence: this kernel keeps the ring
   float eps; int dim_own;              // norms over a head's dim_own columns (the rest is padding); eps < 0: none

@@ -14,18 +14,17 @@ template <int N> struct Vec;
 template <> struct Vec<4> { typedef f32x4 type; };
 template <> struct Vec<1> { typedef f32x1 type; };
 
-template <int N>
-__device__ __forceinline__ typename Vec<N>::type load(const float* p) {
-  return *reinterpret_cast<const typename Vec<N>::type*>(p);
+// N elements as stored, and widened
+template <typename T, int N> struct Raw { typedef typename Vec<N>::type type; };
+template <int N> struct Raw<bf16, N> { typedef bf16 type __attribute__((ext_vector_type(N))); };
+template <int N, typename T>
+__device__ __forceinline__ typename Raw<T, N>::type load(const T* p) {
+  if constexpr (N == 4 && sizeof(T) == 2) return ld4(p);
+  else return *reinterpret_cast<const typename Raw<T, N>::type*>(p);
 }
-template <int N>
-__device__ __forceinline__ typename Vec<N>::type load(const bf16* p) {
-  if constexpr (N == 4) {
-    const bf16x4 v = ld4(p);
-    return f32x4{bf2f(v[0]), bf2f(v[1]), bf2f(v[2]), bf2f(v[3])};
-  } else {
-    return f32x1{bf2f(*p)};
-  }
+template <int N, typename R>
+__device__ __forceinline__ typename Vec<N>::type wide(R v) {
+  return __builtin_convertvector(v, typename Vec<N>::type);
 }
 template <int N>
 __device__ __forceinline__ void store(float* p, typename Vec<N>::type v) {
@@ -37,8 +36,8 @@ __device__ __forceinline__ void store(bf16* p, typename Vec<N>::type v) {
   else *p = f2bf(v[0]);
 }
 
-// LPI lanes per (row, part), MAXC chunks of N columns each.
-template <typename T, int N, int LPI, int MAXC>
+// LPI lanes per (row, part), MAXC chunks of N columns each; FLY slabs (of S) in flight.
+template <typename T, typename S, int N, int LPI, int MAXC, int FLY>
 __global__ __launch_bounds__(256) void part_norm_kernel(GroupNormParams p) {
   typedef typename Vec<N>::type V;
   __shared__ float red[16];
@@ -64,7 +63,8 @@ __global__ __launch_bounds__(256) void part_norm_kernel(GroupNormParams p) {
   };
   int col[MAXC];
   bool on[MAXC];
-  V v[MAXC], wp[MAXC];
+  V v[MAXC];
+  typename Raw<T, N>::type wp[MAXC];
 #pragma unroll
   for (int i = 0; i < MAXC; ++i) {
     const int c = (lane + i * LPI) * N;
@@ -74,30 +74,28 @@ __global__ __launch_bounds__(256) void part_norm_kernel(GroupNormParams p) {
     if (p.out) wp[i] = load<N>(static_cast<const T*>(p.w_pre) + c0 + col[i]);
   }
   if (p.slab) {
-    V y[MAXC], w[MAXC];
+    V y[MAXC];
+    typename Raw<T, N>::type w[MAXC];
 #pragma unroll
     for (int i = 0; i < MAXC; ++i) {
       w[i] = load<N>(static_cast<const T*>(p.w_post) + c0 + col[i]);
       y[i] = V(0.f);
-      if (p.bias) y[i] = load<N>(static_cast<const T*>(p.bias) + c0 + col[i]);
+      if (p.bias) y[i] = wide<N>(load<N>(static_cast<const T*>(p.bias) + c0 + col[i]));
     }
     const long step = (long)p.T * p.H, first = src * p.H + c0;
-    for (int s = 0; s < p.splits; s += 4) {  // four slabs in flight, added in order
-      V u[MAXC][4];
+    for (int s = 0; s < p.splits; s += FLY) {  // added in order
+      typename Raw<S, N>::type u[MAXC][FLY];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
+      for (int j = 0; j < FLY; ++j) {
         const long sl = min(s + j, p.splits - 1) * step + first;
 #pragma unroll
-        for (int i = 0; i < MAXC; ++i)
-          u[i][j] = p.slab_bf16 ? load<N>(static_cast<const bf16*>(p.slab) + sl + col[i])
-                                : load<N>(static_cast<const float*>(p.slab) + sl + col[i]);
-        if (p.splits == 1) break;
+        for (int i = 0; i < MAXC; ++i) u[i][j] = load<N>(static_cast<const S*>(p.slab) + sl + col[i]);
       }
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
+      for (int j = 0; j < FLY; ++j)
         if (s + j < p.splits) {
 #pragma unroll
-          for (int i = 0; i < MAXC; ++i) y[i] += u[i][j];
+          for (int i = 0; i < MAXC; ++i) y[i] += wide<N>(u[i][j]);
         }
     }
     float ss = 0.f;
@@ -108,7 +106,7 @@ __global__ __launch_bounds__(256) void part_norm_kernel(GroupNormParams p) {
     const float rs = 1.f / sqrtf(total(ss) / size + p.eps);
 #pragma unroll
     for (int i = 0; i < MAXC; ++i) {
-      v[i] += y[i] * rs * w[i];
+      v[i] += y[i] * rs * wide<N>(w[i]);
       if (live && on[i]) store<N>(x + col[i], v[i]);
     }
   }
@@ -122,7 +120,7 @@ __global__ __launch_bounds__(256) void part_norm_kernel(GroupNormParams p) {
   T* out = static_cast<T*>(p.out) + row * p.H;
 #pragma unroll
   for (int i = 0; i < MAXC; ++i)
-    if (live && on[i]) store<N>(out + c0 + col[i], v[i] * rs * wp[i]);
+    if (live && on[i]) store<N>(out + c0 + col[i], v[i] * rs * wide<N>(wp[i]));
   if (live && g == p.groups - 1)
     for (int c = p.groups * size + lane; c < p.H; c += LPI) out[c] = (T)0.f;
 }
@@ -132,14 +130,19 @@ __global__ __launch_bounds__(256) void part_norm_kernel(GroupNormParams p) {
 
 using namespace lsd;
 
-template <typename T>
+template <typename T, typename S>
 static hipError_t group_norm(const GroupNormParams& p, hipStream_t st) {
   const int vec = p.size % 4 == 0 ? 4 : 1;
   const long items = (long)(p.rows ? p.n_rows : p.T) * p.groups;
   const int chunks = (p.size + vec - 1) / vec;
   if (items == 0) return hipSuccess;
-#define LSD_GN(N, LPI, MAXC)                                                                                      \
-  hipLaunchKernelGGL((part_norm_kernel<T, N, LPI, MAXC>), dim3((unsigned)((items * LPI + 255) / 256)), dim3(256), 0, st, p)
+#define LSD_GN_F(N, LPI, MAXC, FLY) \
+  hipLaunchKernelGGL((part_norm_kernel<T, S, N, LPI, MAXC, FLY>), dim3((unsigned)((items * LPI + 255) / 256)), dim3(256), 0, st, p)
+#define LSD_GN(N, LPI, MAXC)                                 \
+  do {                                                       \
+    if (p.splits <= 1) LSD_GN_F(N, LPI, MAXC, 1);            \
+    else LSD_GN_F(N, LPI, MAXC, (MAXC > 4 ? 2 : 4));         \
+  } while (0)
 #define LSD_GN_N(N)                                         \
   if (chunks <= 16) LSD_GN(N, 16, 1);                       \
   else if (chunks <= 64) LSD_GN(N, 64, 1);                  \
@@ -158,9 +161,11 @@ static hipError_t group_norm(const GroupNormParams& p, hipStream_t st) {
   }
 #undef LSD_GN_N
 #undef LSD_GN
+#undef LSD_GN_F
   return hipGetLastError();
 }
 
 extern "C" hipError_t lsd_group_rows_norm(const GroupNormParams* p, int f32, hipStream_t st) {
-  return f32 ? group_norm<float>(*p, st) : group_norm<bf16>(*p, st);
+  if (f32) return p->slab && p->slab_bf16 ? hipErrorInvalidValue : group_norm<float, float>(*p, st);
+  return p->slab_bf16 ? group_norm<bf16, bf16>(*p, st) : group_norm<bf16, float>(*p, st);
 }

@@ -44,6 +44,7 @@ hipError_t lsd_talk_decode(const TalkParams* p, int hp, hipStream_t st);
 long lsd_append_lds(const RopeAppendParams* p);
 int lsd_paged_ok(int dim, int vdim);
 hipError_t lsd_paged_prefill(const TalkParams* p, int qt, int lse, hipStream_t st);
+hipError_t lsd_mix_prefill(const TalkParams* p, int hp, hipStream_t st);
 hipError_t lsd_paged_decode(const TalkParams* p, hipStream_t st);
 int lsd_mix_decode_gc(int H, int G);
 long lsd_mix_combine_lds(const TalkParams* p);
@@ -98,6 +99,13 @@ SeqParams seqs(const Tensor& slots, const Tensor& start, const Tensor& cu) {
   return s;
 }
 
+// [slots, taps, channels], like y
+void* ring_of(const Tensor& y, const Tensor& ring, int64_t taps, int64_t channels) {
+  TORCH_CHECK(ring.is_cuda() && ring.scalar_type() == y.scalar_type() && ring.is_contiguous() && ring.dim() == 3 &&
+                  ring.size(1) == taps && ring.size(2) == channels, "ring must be [slots, taps, channels] like y");
+  return ring.data_ptr();
+}
+
 // y [T, N]: conv channels are columns c0 ..; taps [channels, n], ring [slots, n, channels]
 ConvParams conv(const Tensor& y, int64_t c0, const Tensor& w, const Opt& bias, const Tensor& ring, double gain) {
   is_f32(y, "y");
@@ -109,9 +117,7 @@ ConvParams conv(const Tensor& y, int64_t c0, const Tensor& w, const Opt& bias, c
   c.y = y.data_ptr(); c.ldy = y.stride(0); c.c0 = c0;
   c.w = fptr(w, (int64_t)c.channels * c.taps, "taps");
   if (bias.has_value()) c.bias = fptr(*bias, c.channels, "conv bias");
-  TORCH_CHECK(ring.is_cuda() && ring.scalar_type() == y.scalar_type() && ring.is_contiguous() && ring.dim() == 3 &&
-                  ring.size(1) == c.taps && ring.size(2) == c.channels, "ring must be [slots, taps, channels] like y");
-  c.ring = ring.data_ptr();
+  c.ring = ring_of(y, ring, c.taps, c.channels);
   c.gain = (float)gain;
   return c;
 }
@@ -257,7 +263,7 @@ void* value_rows(const RopeAppendParams& p, const Tensor& t, const Tensor& y, co
 }
 
 // y [T, N]: q [heads dim] | k [G dim] | v [G vdim] -> q [T, heads dim]; k, v appended.
-// taps [channels, n] and ring [slots, n, channels]: a short convolution of all three
+// taps [n, channels] and ring [slots, n, channels]: a short convolution of all three
 // (write_ring: one row per sequence); eps >= 0: unit norms of q and k over dim_own
 // columns; v_first: v <- (1 - lam) v + lam v_first; v_out: v as it was before that
 Tensor rope_append(Tensor y, int64_t heads, Tensor k, Tensor v, Tensor table, Tensor tslot, Tensor tpos, Opt rope,
@@ -276,10 +282,12 @@ Tensor rope_append(Tensor y, int64_t heads, Tensor k, Tensor v, Tensor table, Te
     p.rope = fptr(*rope, rope->numel(), "rope"); p.half = rope->size(1);
   }
   if (taps.has_value()) {
-    TORCH_CHECK(ring.has_value(), "a convolution needs its ring");
-    const ConvParams c = conv(y, 0, *taps, c10::nullopt, *ring, gain);
-    TORCH_CHECK(c.channels == channels, "taps must be [", channels, ", n]");
-    p.taps = c.w; p.n_taps = c.taps; p.ring = c.ring; p.write_ring = write_ring;
+    TORCH_CHECK(ring.has_value() && taps->dim() == 2 && taps->size(0) >= 1 && taps->size(1) == channels,
+                "taps must be [n, ", channels, "], with a ring");
+    p.n_taps = taps->size(0);
+    p.taps = fptr(*taps, p.n_taps * channels, "taps");
+    p.ring = ring_of(y, *ring, p.n_taps, channels);
+    p.write_ring = write_ring;
   }
   p.eps = (float)eps;
   p.dim_own = dim_own > 0 ? (int)dim_own : p.dim;
@@ -296,10 +304,15 @@ Tensor rope_append(Tensor y, int64_t heads, Tensor k, Tensor v, Tensor table, Te
   return q;
 }
 
-// inputs of a portion's last positions enter the convolution's ring
-void conv_tail(Tensor y, Tensor taps, Tensor ring, Tensor slots, Tensor start, Tensor cu) {
+// inputs of a portion's last positions (the first columns of y) enter the convolution's ring
+void conv_tail(Tensor y, Tensor ring, Tensor slots, Tensor start, Tensor cu) {
   const bool f32 = is_f32(y, "y");
-  const ConvParams c = conv(y, 0, taps, c10::nullopt, ring, 1.0);
+  TORCH_CHECK(ring.dim() == 3, "ring must be [slots, taps, channels]");
+  ConvParams c{};
+  c.taps = ring.size(1); c.channels = ring.size(2);
+  rows_of(y, y.scalar_type(), y.size(0), c.channels, "y");
+  c.y = y.data_ptr(); c.ldy = y.stride(0);
+  c.ring = ring_of(y, ring, c.taps, c.channels);
   const SeqParams s = seqs(slots, start, cu);
   check_hip(lsd_conv_tail(&c, &s, f32, cur_stream()), "conv_tail");
 }
@@ -374,15 +387,8 @@ void partials(TalkParams& p, int64_t splits, const Tensor& q, Tensor& po, Tensor
 
 // packed ragged queries; tiles [n, 2] = (sequence, first query) of talk_tile(hp) queries
 void talk_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tensor tiles, Tensor slots, Tensor start,
-                  Tensor cu, int64_t window, double scale, double cap, int64_t splits, Tensor out, int64_t keep, Opt slopes,
-                  Opt gate, Opt lse) {
-  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, cap, out, {keep, slopes, gate});
-  if (lse.has_value()) {  // mixed weights
-    p.mix_weights = 1;
-    p.lse = const_cast<float*>(fptr(*lse, (int64_t)p.T * p.H, "lse"));
-  } else {
-    TORCH_CHECK(keep == 0 && !slopes.has_value() && !gate.has_value(), "talk_prefill: mixed scores know a window only");
-  }
+                  Tensor cu, int64_t window, double scale, double cap, int64_t splits, Tensor out) {
+  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, cap, out, {0, c10::nullopt, c10::nullopt});
   const int hp = frag_of(p, q, frag);
   Tensor po, pml;
   partials(p, splits, q, po, pml);
@@ -432,6 +438,24 @@ void paged_decode(Tensor q, Tensor k, Tensor v, Tensor table, Tensor slots, Tens
   Tensor po, pml;
   partials(p, splits, q, po, pml);
   check_hip(lsd_paged_decode(&p, cur_stream()), "paged_decode");
+}
+
+// prompts with weights mixed over the heads: lse (fp32 [T, heads]) from paged_prefill,
+// frag the mixing matrix in fp16, padded; tiles of mix_tile(hp) queries
+void mix_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor frag, Tensor tiles, Tensor slots, Tensor start,
+                 Tensor cu, int64_t window, double scale, int64_t keep, Opt slopes, Opt gate, Tensor lse, int64_t splits,
+                 Tensor out) {
+  TalkParams p = talk_base(q, k, v, table, c10::nullopt, window, scale, 0.0, out, {keep, slopes, gate});
+  need_paged(p, q, "mix_prefill");
+  p.mix_weights = 1;
+  p.lse = const_cast<float*>(fptr(lse, (int64_t)p.T * p.H, "lse"));
+  const int hp = frag_of(p, q, frag);
+  Tensor po, pml;
+  partials(p, splits, q, po, pml);
+  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2, "tiles must be [n, 2]");
+  p.tiles = iptr(tiles, 0, "tiles"); p.n_tiles = tiles.size(0);
+  p.s = seqs(slots, start, cu);
+  check_hip(lsd_mix_prefill(&p, hp, cur_stream()), "mix_prefill");
 }
 
 // the same with weights mixed over the heads by talk (fp32 [heads, heads])
@@ -508,15 +532,13 @@ void lsd_register_mixers(pybind11::module& m) {
         py::arg("tslot"), py::arg("tpos"), py::arg("rope"), py::arg("gain"), py::arg("taps") = py::none(),
         py::arg("ring") = py::none(), py::arg("write_ring") = false, py::arg("eps") = -1.0, py::arg("dim_own") = 0,
         py::arg("v_first") = py::none(), py::arg("lam") = 0.0, py::arg("v_out") = py::none());
-  m.def("conv_tail", &conv_tail, py::arg("y"), py::arg("taps"), py::arg("ring"), py::arg("slots"), py::arg("start"),
-        py::arg("cu"));
+  m.def("conv_tail", &conv_tail, py::arg("y"), py::arg("ring"), py::arg("slots"), py::arg("start"), py::arg("cu"));
   m.def("talk_heads", [](int64_t H, int64_t G, int64_t dim, int64_t vdim, double cap) {
     return lsd_talk_heads(H, G, dim, vdim, (float)cap); });
   m.def("talk_tile", [](int64_t hp) { return lsd_talk_tile((int)hp); });
   m.def("talk_prefill", &talk_prefill, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("frag"),
         py::arg("tiles"), py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("window"), py::arg("scale"),
-        py::arg("cap"), py::arg("splits"), py::arg("out"), py::arg("keep") = 0, py::arg("slopes") = py::none(),
-        py::arg("gate") = py::none(), py::arg("lse") = py::none());
+        py::arg("cap"), py::arg("splits"), py::arg("out"));
   m.def("talk_decode", &talk_decode, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("frag"),
         py::arg("slots"), py::arg("pos"), py::arg("window"), py::arg("scale"), py::arg("cap"), py::arg("splits"),
         py::arg("out"));
@@ -530,6 +552,9 @@ void lsd_register_mixers(pybind11::module& m) {
   m.def("paged_decode", &paged_decode, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("slots"),
         py::arg("pos"), py::arg("window"), py::arg("scale"), py::arg("keep"), py::arg("slopes"), py::arg("gate"),
         py::arg("splits"), py::arg("out"));
+  m.def("mix_prefill", &mix_prefill, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("frag"),
+        py::arg("tiles"), py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("window"), py::arg("scale"),
+        py::arg("keep"), py::arg("slopes"), py::arg("gate"), py::arg("lse"), py::arg("splits"), py::arg("out"));
   m.def("mix_decode_ok", [](int64_t H, int64_t G) { return lsd_mix_decode_gc((int)H, (int)G) > 0; });
   m.def("mix_decode", &mix_decode, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("talk"),
         py::arg("slots"), py::arg("pos"), py::arg("window"), py::arg("scale"), py::arg("keep"), py::arg("slopes"),

@@ -423,7 +423,6 @@ class HipBackend(Backend):
                 return torch.cat(out)
 
             w_in = rows("")
-            channels = w_in.shape[0]
             if m.head_gate:
                 w_in = torch.cat([w_in, t("mixer.g")])
             n = _up(w_in.shape[0], 64)
@@ -432,8 +431,7 @@ class HipBackend(Backend):
                 w[p + "mixer.in.bias"] = pad_to(rows(".b")[:, 0], n)
                 w[p + "mixer.o.b"] = pad_to(w[p + "mixer.o.b"], hp)
             if m.conv:
-                w[p + "mixer.taps"] = rows(".conv").float().contiguous()
-                assert w[p + "mixer.taps"].shape[0] == channels
+                w[p + "mixer.taps"] = rows(".conv").float().t().contiguous()  # [taps][channels]
             if m.mix_values is not None:
                 w[p + "mixer.vmix"] = w[p + "mixer.vmix"].float().cpu()
             if m.distance_bias:
@@ -553,7 +551,7 @@ class HipBackend(Backend):
         gate = y[:, c: c + m.heads] if m.head_gate else None
         for s, mt in self._parts(meta):
             if m.conv and not meta.is_decode:
-                self.C.conv_tail(y[s], taps, ring, mt.seq_slots, mt.q_start, mt.cu_q)
+                self.C.conv_tail(y[s], ring, mt.seq_slots, mt.q_start, mt.cu_q)
             self._attention(q[s], w, m, k, v, kv, mt, None if gate is None else gate[s], out[s])
         return out, values
 
@@ -584,8 +582,8 @@ class HipBackend(Backend):
             tiles, qt = self._paged_tiles(mt, H, q.device)
             C.paged_prefill(*at, tiles, qt, *seqs, window, m.scale, *beside, out, lse)
             tiles = self._query_tiles(mt, C.talk_tile(tp.shape[0]), q.device)
-            C.talk_prefill(*at, tp, tiles, *seqs, window, m.scale, 0.0, R.talk_prefill_splits(tiles.shape[0], ctx), out,
-                           *beside, lse)
+            C.mix_prefill(*at, tp, tiles, *seqs, window, m.scale, *beside, lse, R.talk_prefill_splits(tiles.shape[0], ctx),
+                          out)
         elif mfma and not m.talking:
             if mt.is_decode and H // G <= 16:
                 C.paged_decode(*at, *rows, window, m.scale, *beside, R.paged_splits(mt.num_seqs * G, ctx), out)

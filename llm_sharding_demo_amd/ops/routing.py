@@ -137,9 +137,9 @@ class Routing:
     # keys each
     paged_tile_min: int = 512
     paged_waves: int = 2048
-    paged_split_keys: int = 128
+    paged_split_keys: int = 64
     # decode attention with mixed weights: blocks a launch aims for
-    mix_target: int = 512
+    mix_target: int = 256
     # -- norms / head ------------------------------------------------------
     # one wave per row from norm_wave_min rows (prefill 32 K x 1600 97.7 ->
     # 53.7 us; r5_normwave.log) and from norm_wave_narrow_min rows when H <=

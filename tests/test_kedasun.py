@@ -258,3 +258,13 @@ def test_partition_and_memory_budget(tmp_path):
     kv = eng.stages[0].kv
     assert kv.nbytes == (eng.kv_slots + 2) * slot + (eng.kv_pages + 1) * page + 4 * kv.table.numel()
     assert eng._weight_bytes(0) == 2 * (eng.mcfg.stage_params(range(6)) + 2 * eng.mcfg.embed_params())
+
+
+def test_routing_of_the_attention_kernels():
+    """Splits fill the chip with few sequences and vanish with many; never more than there are tiles."""
+    from llm_sharding_demo_amd.ops.routing import Routing
+
+    r = Routing()
+    assert r.paged_splits(4, 1028) == 17 and r.paged_splits(4096, 1028) == 1 and r.paged_splits(1, 3) == 1
+    assert r.mix_splits(1, 1028, 16, 4) == 19 and r.mix_splits(256, 1028, 16, 4) == 1
+    assert r.mix_splits(128, 1028, 32, 8) == 2 and r.mix_splits(1, 1, 4, 4) <= 2

@@ -84,7 +84,7 @@ class AppendCase:
         w = {n: rounded(R(x[n].shape[1], x[n].shape[2], taps), F32) for n in "qkv"} if taps else None
         if taps:
             x = {n: orc.short_conv(x[n].reshape(T, -1), w[n].reshape(-1, taps)).reshape(x[n].shape) for n in "qkv"}
-            self.taps = cuda(torch.cat([pad(n, w[n].transpose(1, 2)).transpose(1, 2).reshape(-1, taps) for n in "qkv"]), F32)
+            self.taps = cuda(torch.cat([pad(n, w[n].transpose(1, 2)).transpose(1, 2).reshape(-1, taps) for n in "qkv"]).T, F32)
             self.ring = torch.full((3, taps, self.ch), float("nan"), dtype=dt, device="cuda")
         if norm:
             x["q"], x["k"] = orc.rms(x["q"], self.eps), orc.rms(x["k"], self.eps)
@@ -120,7 +120,7 @@ class AppendCase:
                                    self.rope, 1.0, self.taps if self.n else None, self.ring if self.n else None, single,
                                    self.eps, D, first, self.lam or 0.0, vout)
             if self.n and not single:
-                self.C.conv_tail(y, self.taps, self.ring, *seq)
+                self.C.conv_tail(y, self.ring, *seq)
             qs.append(q.reshape(-1, H, self.dp))
             vs.append(vout.reshape(-1, G, self.vp))
         return torch.cat(qs), torch.cat(vs)
@@ -170,12 +170,12 @@ def test_convolution_of_a_mixed_batch(C):
         b = Batch(*step)
         y = cuda(torch.cat([cases[s].y[a:a + n] for s, a, n in step]))
         q = C.rope_append(y, H, K, Vp, cuda(table), b.tslot, b.tpos, None, 1.0, w, ring, False, 1e-3, D, None, 0.0, None)
-        C.conv_tail(y, w, ring, b.slots, b.start, b.cu)
+        C.conv_tail(y, ring, b.slots, b.start, b.cu)
         for i, (s, _, _) in enumerate(step):
             out[s].append(q[b.rows(i)])
     for s, c in enumerate(cases):
         x = c.y[:, : H * D].double()
-        want = orc.rms(orc.short_conv(x, w[: H * D].double().cpu()).reshape(-1, H, D), 1e-3)
+        want = orc.rms(orc.short_conv(x, w[:, : H * D].T.double().cpu()).reshape(-1, H, D), 1e-3)
         assert err(torch.cat(out[s]).reshape(-1, H, D), want) < 3e-2
 
 
@@ -248,8 +248,8 @@ class AttentionCase:
         hp = C.talk_heads(H, G, self.at[1].shape[3], self.at[2].shape[3], -1.0)
         frag = torch.zeros(hp, hp, dtype=torch.float16, device="cuda")
         frag[:H, :H] = self.talk.half()
-        C.talk_prefill(*self.at, frag, b.tiles(C.talk_tile(hp)), *seqs, self.window, self.scale, 0.0, splits, out,
-                       *self.beside, lse)
+        C.mix_prefill(*self.at, frag, b.tiles(C.talk_tile(hp)), *seqs, self.window, self.scale, *self.beside, lse, splits,
+                      out)
         return out
 
     def decode(self, splits):
