@@ -24,36 +24,6 @@ from typing import Optional, Sequence, Tuple, Union
 # ---------------------------------------------------------------------------
 
 @dataclass(frozen=True)
-class LatentAttentionSpec:
-    """Attention whose keys and values are linear images of one cached latent
-    row per token (no positions); every size is the layer's own."""
-
-    heads: int
-    dim: int                       # query / key dimensions per head
-    vdim: int                      # value dimensions per head
-    kv_rank: int                   # latent dimensions: what the cache holds
-    scale: float                   # score = (q . k) * scale
-    window: Optional[int] = None   # keys per query, itself included (None: all)
-    kv_from: Optional[int] = None  # use this earlier layer's cached latents
-
-    @property
-    def params_per_hidden(self) -> int:
-        """Weight columns of `hidden` rows: q, out, and an own latent projection."""
-        return self.heads * (self.dim + self.vdim) + (self.kv_rank if self.kv_from is None else 0)
-
-    @property
-    def cached_per_token(self) -> int:
-        return self.kv_rank if self.kv_from is None else 0
-
-    def params(self, hidden: int) -> int:
-        return hidden * self.params_per_hidden + self.heads * (self.dim + self.vdim) * self.kv_rank + self.cached_per_token
-
-    def check(self) -> None:
-        if min(self.heads, self.dim, self.vdim, self.kv_rank) < 1 or (self.window is not None and self.window < 1):
-            raise ValueError("attention sizes must be positive")
-
-
-@dataclass(frozen=True)
 class RopeScaling:
     """Wavelengths above original / low are stretched by `factor`, those below
     original / high stay, a linear ramp lies between."""
@@ -88,6 +58,59 @@ class RopeSpec:
                     f = (1.0 - keep) * f / s.factor + keep * f
             out.append(f)
         return out
+
+
+@dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Attention whose keys and values are linear images of one cached latent
+    row per token; every size is the layer's own.  With `rope`, a head's queries
+    have rope.dims further dimensions that turn with the position, and all heads
+    share one turned key part, cached behind the latent.  q_rank: queries come
+    from a normed latent of their own.  sink: a learned score per head that
+    takes part in the softmax without a value.  gate: a sigmoid gate per output
+    channel."""
+
+    heads: int
+    dim: int                       # query / key dimensions per head (without positions)
+    vdim: int                      # value dimensions per head
+    kv_rank: int                   # latent dimensions: what the cache holds
+    scale: float                   # score = (q . k) * scale
+    window: Optional[int] = None   # keys per query, itself included (None: all)
+    kv_from: Optional[int] = None  # use this earlier layer's cached latents
+    rope: Optional[RopeSpec] = None
+    q_rank: Optional[int] = None
+    sink: bool = False
+    gate: bool = False
+
+    @property
+    def rot_dim(self) -> int:
+        return self.rope.dims if self.rope is not None else 0
+
+    @property
+    def q_dim(self) -> int:
+        """Query dimensions per head."""
+        return self.dim + self.rot_dim
+
+    @property
+    def cached_per_token(self) -> int:
+        return self.kv_rank + self.rot_dim if self.kv_from is None else 0
+
+    @property
+    def in_columns(self) -> int:
+        """Rows of the projections that read the layer's input."""
+        q = self.heads * self.q_dim if self.q_rank is None else self.q_rank
+        return q + self.cached_per_token + (self.heads * self.vdim if self.gate else 0)
+
+    def params(self, hidden: int) -> int:
+        n = hidden * (self.in_columns + self.heads * self.vdim) + self.heads * (self.dim + self.vdim) * self.kv_rank
+        n += (self.kv_rank if self.kv_from is None else 0) + (self.heads if self.sink else 0)
+        return n + (self.q_rank * (1 + self.heads * self.q_dim) if self.q_rank is not None else 0)
+
+    def check(self) -> None:
+        if min(self.heads, self.dim, self.vdim, self.kv_rank) < 1 or (self.window is not None and self.window < 1):
+            raise ValueError("attention sizes must be positive")
+        if self.rot_dim % 2 or (self.q_rank is not None and self.q_rank < 1):
+            raise ValueError(f"cannot rotate {self.rot_dim} dimensions, or no query latent of {self.q_rank}")
 
 
 @dataclass(frozen=True)
@@ -216,6 +239,26 @@ class SSMSpec:
 
 
 @dataclass(frozen=True)
+class ForgetSpec:
+    """Linear attention whose forget gate, per head and channel, also decides
+    what is written (HGRN2): a state [dim, vdim] per head, no keys."""
+
+    heads: int
+    dim: int
+    vdim: int
+    kv_from: None = None
+    cached_per_token = 0
+
+    def params(self, hidden: int) -> int:
+        n, v = self.heads * self.dim, self.heads * self.vdim
+        return hidden * 2 * (n + v) + 2 * n + self.vdim
+
+    def check(self) -> None:
+        if min(self.heads, self.dim, self.vdim) < 1:
+            raise ValueError("recurrence sizes must be positive")
+
+
+@dataclass(frozen=True)
 class DenseSpec:
     """Gated feed-forward W_down(gelu_tanh(W_gate h) * W_up h), or with a
     `limit` the clamped gate of the experts."""
@@ -229,25 +272,31 @@ class DenseSpec:
 
 @dataclass(frozen=True)
 class ExpertSpec:
-    """Gated feed-forward with clamped gate / up (`limit`)."""
+    """Gated feed-forward, SiLU or with clamped gate / up (`limit`)."""
 
     ff: int
-    limit: float
+    limit: Optional[float] = None
 
 
 @dataclass(frozen=True)
 class MoESpec:
+    """Experts chosen by corrected sigmoid scores, which weigh them too, or
+    (softmax) by their logits, with the softmax over the chosen ones as weights.
+    shared_gate: a sigmoid per token weighs the shared expert."""
+
     experts: int
     top: int
     expert: ExpertSpec
     shared: Optional[ExpertSpec] = None  # runs for every token
+    softmax: bool = False
+    shared_gate: bool = False
 
     def params(self, hidden: int) -> int:
-        n = self.experts * (hidden + 1 + 3 * hidden * self.expert.ff)
-        return n + (3 * hidden * self.shared.ff if self.shared is not None else 0)
+        n = self.experts * (hidden + (not self.softmax) + 3 * hidden * self.expert.ff)
+        return n + (3 * hidden * self.shared.ff + hidden * self.shared_gate if self.shared is not None else 0)
 
 
-MixerSpec = Union[LatentAttentionSpec, AttentionSpec, ChannelDeltaSpec, SSMSpec]
+MixerSpec = Union[LatentAttentionSpec, AttentionSpec, ChannelDeltaSpec, SSMSpec, ForgetSpec]
 
 
 @dataclass(frozen=True)
@@ -255,12 +304,17 @@ class LayerSpec:
     """One layer as it runs.  A loop over layers is written out: every pass has
     entries of its own (and so its own cache or state), `weights` names the
     layer whose tensors they share (None: its own), and `enter` is the pass
-    that begins in front of this entry (None: no pass begins here)."""
+    that begins in front of this entry with a step of its own (None: no such
+    step)."""
 
     mixer: MixerSpec
     mlp: Union[MoESpec, DenseSpec, None] = None
     weights: Optional[int] = None
     enter: Optional[int] = None
+
+
+# digits (base 256, exact in bf16) of a token id on the wire between stages
+ID_DIGITS = 3
 
 
 @dataclass(frozen=True)
@@ -272,11 +326,13 @@ class ModelConfig:
     blocks of latent attention and experts; "vizalix": parallel blocks of
     attention, delta rule or Mamba-2 and a dense feed-forward, some of them
     looped; "kedasun": attention and a dense feed-forward one after the other,
-    each between two norms); the scalar head / ffn fields then only describe the
-    first layer."""
+    each between two norms; "fagunex": latent attention or a recurrence, and
+    experts, each between two norms, behind a token shift and in front of rows of
+    the tokens' own, some of them looped); the scalar head / ffn fields then only
+    describe the first layer."""
 
     name: str
-    arch: str  # "gpt2" | "llama" | "timisun" | "vizalix" | "kedasun"
+    arch: str  # "gpt2" | "llama" | "timisun" | "vizalix" | "kedasun" | "fagunex"
     vocab_size: int
     hidden: int
     n_layers: int
@@ -292,6 +348,8 @@ class ModelConfig:
     embed_scale: float = 1.0
     layers: Tuple[LayerSpec, ...] = ()
     norm_groups: int = 1  # equal parts of a row, each normed by itself
+    token_shift: bool = False  # mixers read rows mixed with those of the previous token
+    token_side: int = 0  # width of the rows that tokens bring to every layer (0: none)
 
     @property
     def whole_layers(self) -> bool:
@@ -305,8 +363,18 @@ class ModelConfig:
         return bool(self.layers)
 
     @property
+    def shared_weights(self) -> bool:
+        """Several layer runs may use the tensors of one layer."""
+        return any(l.weights is not None for l in self.layers)
+
+    @property
+    def shift_width(self) -> int:
+        """Columns of the previous token's row that every layer keeps of a sequence."""
+        return self.hidden if self.token_shift else 0
+
+    @property
     def loop_times(self) -> int:
-        """Passes of the looped layers (0: no loop)."""
+        """Passes of the looped layers that begin with a step of their own (0: none)."""
         return max((l.enter + 1 for l in self.layers if l.enter is not None), default=0)
 
     @property
@@ -318,10 +386,11 @@ class ModelConfig:
     @property
     def boundary(self) -> int:
         """Columns a stage hands to the next: the residual, the embedding
-        output where a loop's passes read it again, and the values that later
-        layers mix in."""
+        output where a loop's passes read it again, the values that later
+        layers mix in, and the token ids where every layer looks them up."""
         m = self.mixed_values
-        return self.hidden * (2 if self.loop_times else 1) + (m.kv_heads * m.vdim if m is not None else 0)
+        n = self.hidden * (2 if self.loop_times else 1) + (m.kv_heads * m.vdim if m is not None else 0)
+        return n + (ID_DIGITS if self.token_side else 0)
 
     def weight_layer(self, i: int) -> int:
         """The layer whose tensors layer i uses."""
@@ -366,8 +435,10 @@ class ModelConfig:
         if not self.layers:
             return self.block_params()
         h, m, f = self.hidden, self.layers[i].mixer, self.layers[i].mlp
-        norms = {"timisun": h, "kedasun": 2 * h * (1 + (f is not None))}.get(self.arch, 1 + (f is not None))
-        return norms + m.params(h) + (f.params(h) if f is not None else 0)
+        subs = 1 + (f is not None)
+        norms = {"timisun": h, "kedasun": 2 * h * subs, "fagunex": 2 * (2 * h + 1) * subs}.get(self.arch, subs)
+        side = (2 * h + self.vocab_size) * self.token_side + h if self.token_side else 0
+        return norms + self.shift_width + side + m.params(h) + (f.params(h) if f is not None else 0)
 
     def block_params(self) -> int:
         """Parameters of a layer (of the mean layer when they differ)."""
@@ -485,14 +556,15 @@ MODEL_PRESETS.update({
         shared_ff=4096)),
 })
 
-def unroll(layers: Sequence[LayerSpec], start: int, stop: int, times: int) -> list:
-    """Layers start .. stop - 1 run `times` times in a row, written out."""
+def unroll(layers: Sequence[LayerSpec], start: int, stop: int, times: int, steps: bool = True) -> list:
+    """Layers start .. stop - 1 run `times` times in a row, written out; steps:
+    every pass begins with a step of its own."""
     if not (0 <= start < stop <= len(layers) and times >= 1):
         raise ValueError(f"loop over layers {start} .. {stop - 1}, {times} times: outside the {len(layers)} layers")
     rep = dataclasses.replace
     out = [rep(l, weights=i) for i, l in enumerate(layers[:start])]
     for t in range(times):
-        out += [rep(layers[i], weights=i, enter=t if i == start else None) for i in range(start, stop)]
+        out += [rep(layers[i], weights=i, enter=t if steps and i == start else None) for i in range(start, stop)]
     return out + [rep(layers[i], weights=i) for i in range(stop, len(layers))]
 
 
@@ -579,6 +651,56 @@ MODEL_PRESETS.update({
     "kedasun-8b": _kedasun("kedasun-8b", 32000, 4096, _kedasun_layers(
         14336, 7.0, (64, 500000.0), dict(window=1024, keep_first=4, conv=4), 2, heads=32, kv_heads=8, dim=128, vdim=128,
         scale=128 ** -0.5), groups=4),
+})
+
+
+def _fagunex(name: str, vocab: int, width: int, layers: Sequence[LayerSpec], loop: Optional[Tuple[int, int, int]] = None,
+             side: int = 0, eps: float = 1e-6) -> ModelConfig:
+    check_layers(layers)
+    if side < 0:
+        raise ValueError("the token-side rows need a positive width")
+    layers = tuple(unroll(layers, *loop, steps=False) if loop else layers)
+    m, f = layers[0].mixer, layers[0].mlp
+    return ModelConfig(
+        name=name, arch="fagunex", vocab_size=vocab, hidden=width, n_layers=len(layers), n_heads=m.heads, n_kv_heads=1,
+        ffn=f.expert.ff if f else 0, max_positions=1 << 20,  # rows of the rotation tables
+        norm_eps=eps, tie_embeddings=False, bos_token_id=0, eos_token_id=-1, layers=layers, token_shift=True,
+        token_side=side)
+
+
+def _fagunex_moe(experts: int, top: int, ff: int, shared_ff: Optional[int]) -> MoESpec:
+    return MoESpec(experts, top, ExpertSpec(ff), ExpertSpec(shared_ff) if shared_ff else None, softmax=True,
+                   shared_gate=bool(shared_ff))
+
+
+def _fagunex_windowed(rot: Tuple[int, float], **sizes) -> LatentAttentionSpec:
+    """The kind with a query latent, a sliding window, a sink and an output gate."""
+    return LatentAttentionSpec(rope=RopeSpec(*rot, interleaved=True), sink=True, gate=True, **sizes)
+
+
+def _fagunex_full(rot: Tuple[int, float], **sizes) -> LatentAttentionSpec:
+    return LatentAttentionSpec(rope=RopeSpec(*rot), **sizes)
+
+
+def _fagunex_layers(moe: MoESpec, attention: dict, windowed: dict, forget: dict) -> list:
+    """Full attention, recurrence, windowed attention, recurrence."""
+    r = ForgetSpec(**forget)
+    mixers = (_fagunex_full(**attention), r, _fagunex_windowed(**attention, **windowed), r)
+    return [LayerSpec(m, moe) for m in mixers]
+
+
+MODEL_PRESETS.update({
+    # Fagunex: small test sizes (none a multiple of the GEMM tiles), and two
+    # sizes that resemble the layers of models that are served today
+    "fagunex-test": _fagunex("fagunex-test", 300, 104, _fagunex_layers(
+        _fagunex_moe(6, 2, 48, 72), dict(heads=3, dim=24, vdim=40, kv_rank=56, scale=0.2, rot=(12, 10000.0)),
+        dict(q_rank=44, window=90), dict(heads=4, dim=20, vdim=28)), loop=(0, 2, 2), side=20),
+    "fagunex-2b": _fagunex("fagunex-2b", 32000, 2048, _fagunex_layers(
+        _fagunex_moe(32, 4, 1024, 2048), dict(heads=16, dim=128, vdim=128, kv_rank=512, scale=192 ** -0.5, rot=(64, 500000.0)),
+        dict(q_rank=1024, window=1024), dict(heads=16, dim=128, vdim=128)), loop=(0, 4, 2), side=256),
+    "fagunex-8b": _fagunex("fagunex-8b", 32000, 4096, _fagunex_layers(
+        _fagunex_moe(32, 4, 2048, 4096), dict(heads=32, dim=128, vdim=128, kv_rank=256, scale=192 ** -0.5, rot=(64, 500000.0)),
+        dict(q_rank=1536, window=1024), dict(heads=32, dim=128, vdim=128)), loop=(1, 3, 2), side=256),
 })
 
 _ALIASES = {
@@ -685,6 +807,34 @@ def _kedasun_from_json(c: dict, name: str) -> ModelConfig:
                     embed_scale=float(c["embedding"]["scale"]))
 
 
+def _fagunex_from_json(c: dict, name: str) -> ModelConfig:
+    """The design's own config.json."""
+    layers = []
+    for i, l in enumerate(c["layers"]):
+        m, f = l["mixer"], l.get("mlp")
+        if l["type"] == "hgrn2":
+            mix: MixerSpec = ForgetSpec(heads=m["heads"], dim=m["dim"], vdim=m["vdim"])
+        elif l["type"] in ("latent_attention", "latent_attention_2"):
+            sizes = dict(heads=m["heads"], dim=m["dim"], vdim=m["vdim"], kv_rank=m["kv_rank"], scale=float(m["scale"]),
+                         rot=(m["rot_dim"], float(m["rot"]["base"])))
+            if m["rot"].get("dims", m["rot_dim"]) != m["rot_dim"]:
+                raise ValueError(f"layer {i}: the whole rotated part turns")
+            mix = (_fagunex_full(**sizes) if l["type"] == "latent_attention_2" else
+                   _fagunex_windowed(q_rank=m["q_rank"], window=(m.get("mask") or {}).get("size"), **sizes))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {l['type']!r}")
+        moe = None
+        if f:
+            if f.get("kind", "moe") != "moe":
+                raise ValueError(f"layer {i}: unknown feed-forward {f['kind']!r}")
+            moe = _fagunex_moe(f["router"]["experts"], f["router"]["top"], f["expert"]["ff"],
+                               (f.get("shared") or {}).get("ff"))
+        layers.append(LayerSpec(mix, moe))
+    lp = c.get("loop")
+    return _fagunex(name, c["vocab"], c["width"], layers, loop=(lp["start"], lp["stop"], lp["times"]) if lp else None,
+                    side=(c.get("token_side") or {}).get("dim") or 0, eps=float(c["norm"]["eps"]))
+
+
 def _checkpoint_shapes(folder: str):
     """name -> shape of the tensors in a folder's safetensors files (headers only)."""
     import json
@@ -711,7 +861,8 @@ def model_config_from_hf_json(path: str) -> ModelConfig:
     if c.get("architecture") == "Vizalix":
         folder = os.path.dirname(os.path.abspath(path))
         return _vizalix_from_json(c, os.path.basename(folder) or "vizalix", _checkpoint_shapes(folder))
-    own = {"Timisun": _timisun_from_json, "Kedasun": _kedasun_from_json}.get(c.get("architecture"))
+    own = {"Timisun": _timisun_from_json, "Kedasun": _kedasun_from_json, "Fagunex": _fagunex_from_json}.get(
+        c.get("architecture"))
     if own is not None:
         return own(c, os.path.basename(os.path.dirname(os.path.abspath(path))) or c["architecture"].lower())
     mt = c.get("model_type", "gpt2")

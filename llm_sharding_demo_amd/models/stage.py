@@ -1,4 +1,4 @@
-"""One pipeline stage of a GPT-2, Llama, Timisun, Vizalix or Kedasun model.
+"""One pipeline stage of a GPT-2, Llama, Timisun, Vizalix, Kedasun or Fagunex model.
 
 Generalises the reference's two hard-wired shards (`server.py:51-105`):
   * ShardA (`server.py:68-86`): wte + wpe + blocks[0:split]   -> stage 0
@@ -22,7 +22,7 @@ from typing import Dict, Optional, Sequence, Tuple
 
 import torch
 
-from ..config import ModelConfig
+from ..config import ID_DIGITS, ForgetSpec, ModelConfig
 from ..ops import Residual, get_backend
 from ..runtime.batch import BatchMeta
 from ..runtime.kv_cache import KVCache, LatentCache, PagedCache
@@ -76,12 +76,18 @@ class StageModel:
         # columns of the residual rows (hidden, or padded by the backend)
         self.row_width = self.backend.row_width(cfg)
         # rows that cross a stage boundary: the residual, beside it the embedding
-        # output where a loop's passes read it again, and the values that later
-        # layers mix in; (heads, columns of a head, the model's own of them) each
-        self.wire_parts = [(1, self.row_width, cfg.hidden)] * (2 if cfg.loop_times else 1)
+        # output where a loop's passes read it again, the values that later layers
+        # mix in, and the digits of the token ids where every layer looks them up;
+        # (heads, columns of a head, the model's own of them) each
+        self.wire_names = ["x"] + (["x0"] if cfg.loop_times else [])
+        self.wire_parts = [(1, self.row_width, cfg.hidden)] * len(self.wire_names)
         m = cfg.mixed_values
         if m is not None:
-            self.wire_parts = self.wire_parts + [(m.kv_heads, self.backend.value_width(m), m.vdim)]
+            self.wire_names.append("values")
+            self.wire_parts.append((m.kv_heads, self.backend.value_width(m), m.vdim))
+        if cfg.token_side:
+            self.wire_names.append("ids")
+            self.wire_parts.append((1, 4, ID_DIGITS))
         self.wire_width = sum(n * c for n, c, _ in self.wire_parts)
         if cfg.whole_layers and (ua % 2 or ub % 2):
             raise ValueError(f"{cfg.name}: layers cannot be cut in half (units {units})")
@@ -98,7 +104,7 @@ class StageModel:
             if cfg.arch == "timisun":
                 self.kv = LatentCache([self.backend.latent_width(cfg.layers[i].mixer.kv_rank) for i in own], *args)
             else:
-                self.kv = PagedCache([self.backend.layer_cache(cfg.layers[i].mixer) for i in own], *args)
+                self.kv = PagedCache([self.backend.layer_cache(cfg.layers[i].mixer, cfg.shift_width) for i in own], *args)
         else:
             self.kv = KVCache(len(self.kv_layers), max_slots, cfg.n_kv_heads, self.max_seq,
                               cfg.head_dim, dtype, self.device)
@@ -106,7 +112,7 @@ class StageModel:
 
     def _owns(self, name: str) -> bool:
         """Is tensor `name` used by this stage (its units, embeddings, head)?"""
-        if self.cfg.arch == "vizalix":
+        if self.cfg.arch in ("vizalix", "fagunex"):
             return name in stage_tensor_shapes(self.cfg, self.layers, self.first, self.last)
         lh = layer_half(name)
         if lh is None:
@@ -172,8 +178,8 @@ class StageModel:
         m = spec.mixer
         pool = self.kv.pools[self._pool_index[i if m.kv_from is None else m.kv_from]]
         h = be.rmsnorm(r, w("input_layernorm.weight"), c.norm_eps, offset=1.0, width=c.hidden)
-        q, routing = be.latent_project(h, w, spec, self.kv, pool, meta, c.norm_eps)
-        o = be.latent_attention(q, w, m, self.kv, pool, meta)
+        q, gate, routing = be.latent_project(h, w, m, spec.mlp, self.kv, pool, meta, c.norm_eps)
+        o = be.latent_attention(q, gate, w, m, self.kv, pool, meta)
         be.parallel_residual(o, h, routing, w, spec.mlp, r)
 
     # Vizalix: mixer and feed-forward of the same residual, each behind a norm
@@ -205,25 +211,50 @@ class StageModel:
             h = be.clamped_glu(h, w("mlp.gate_up.weight"), spec.mlp.limit)
             be.linear_post_norm(h, w("mlp.down_proj.weight"), None, w("mlp.out_norm.weight"), r, c)
 
+    # Fagunex: the sandwich with elementwise norms; mixers read rows shifted towards
+    # the previous token's, the feed-forward is a mixture of experts, and rows of the
+    # tokens' own come last
+    def _token_layer(self, i: int, r: Residual, side: dict, meta: BatchMeta) -> None:
+        be, c, spec = self.backend, self.cfg, self.cfg.layers[i]
+        w, m = functools.partial(self._lw, c.weight_layer(i)), spec.mixer
+        entry = self.kv.entries[self._pool_index[i]]
+        h = be.shift_norm(r, w, entry[-1], meta, c)
+        if isinstance(m, ForgetSpec):
+            o, out = be.forget_mix(h, w, m, entry[0], meta, c.norm_eps), "mixer.o"
+        else:
+            q, gate, _ = be.latent_project(h, w, m, None, self.kv, entry[0], meta, c.norm_eps)
+            o, out = be.latent_attention(q, gate, w, m, self.kv, entry[0], meta), "attn.o.weight"
+        be.linear_tanh(o, w(out), lambda n: w("norm1b" + n), r)
+        if spec.mlp is not None:
+            h = be.tanh_norm(r, lambda n: w("norm2" + n))
+            be.experts_tanh(h, w, spec.mlp, lambda n: w("norm2b" + n), r)
+        if c.token_side:
+            be.token_side(r, side["ids"], w, c)
+
     # -- stage boundaries: the residual, and what travels beside it (wire_parts) --
     def _unpack(self, rows: torch.Tensor):
         """Residual rows and the side rows {"x0": ..., "values": ...}."""
         if len(self.wire_parts) == 1:
             return rows, {}
         parts = [p.contiguous() for p in rows.split([n * c for n, c, _ in self.wire_parts], 1)]
-        side = {"x0": parts[1]} if self.cfg.loop_times else {}
-        if self.cfg.mixed_values is not None:
-            side["values"] = parts[-1].to(self.dtype)
-        return parts[0], side
+        side = dict(zip(self.wire_names, parts))
+        if "values" in side:
+            side["values"] = side["values"].to(self.dtype)
+        if "ids" in side:
+            d = side["ids"].to(torch.int32)
+            side["ids"] = (d[:, 0] + 256 * d[:, 1] + 65536 * d[:, 2]).contiguous()
+        return side.pop("x"), side
 
     def _pack(self, x: torch.Tensor, side: dict) -> torch.Tensor:
         if len(self.wire_parts) == 1:
             return x
-        rows = [x] + ([side["x0"]] if self.cfg.loop_times else [])
-        if self.cfg.mixed_values is not None:
-            n, c, _ = self.wire_parts[-1]
-            v = side.get("values")  # not there yet: the first layer that has them comes later
-            rows.append(v.float() if v is not None else x.new_zeros(x.shape[0], n * c))
+        rows = [x]
+        for name, (n, c, _) in list(zip(self.wire_names, self.wire_parts))[1:]:
+            v = side.get(name)
+            if name == "ids":
+                rows.append(torch.stack([v % 256, v // 256 % 256, v // 65536, torch.zeros_like(v)], 1).float())
+            else:  # None: the first layer that has them comes later
+                rows.append(v.float() if v is not None else x.new_zeros(x.shape[0], n * c))
         return torch.cat(rows, 1)
 
     def boundary_rows(self, rows: torch.Tensor) -> torch.Tensor:
@@ -263,6 +294,7 @@ class StageModel:
         side: dict = {}
         if self.first:
             x = self.embed(inp, meta)
+            side["ids"] = inp
             if self.cfg.loop_times:
                 side["x0"] = self.embed(inp, meta)  # the residual is updated in place
         else:
@@ -283,6 +315,8 @@ class StageModel:
                         self._parallel_layer(i, r, meta)
                     elif self.cfg.arch == "kedasun":
                         self._sandwich_layer(i, r, side, meta)
+                    elif self.cfg.arch == "fagunex":
+                        self._token_layer(i, r, side, meta)
                     else:
                         self._mixer_layer(i, r, side.get("x0"), meta)
                     if residuals is not None:
@@ -308,6 +342,8 @@ class StageModel:
             xn = be.norm_rows(x, self.w["norm.weight"], None, c.norm_eps, True, rows, width=be.norm_width(c))
         elif c.arch == "kedasun":
             xn = be.group_norm_rows(x, self.w["norm.weight"], c, rows)
+        elif c.arch == "fagunex":
+            xn = be.tanh_norm_rows(x, lambda n: self.w["norm" + n], rows)
         elif c.arch == "gpt2":
             xn = be.norm_rows(x, self.w["ln_f.weight"], self.w["ln_f.bias"], c.norm_eps, False, rows)
         else:

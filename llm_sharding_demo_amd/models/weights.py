@@ -25,7 +25,7 @@ from typing import Dict, Iterable, Optional, Tuple
 
 import torch
 
-from ..config import ChannelDeltaSpec, ModelConfig, SSMSpec
+from ..config import ChannelDeltaSpec, ForgetSpec, ModelConfig, SSMSpec
 
 
 def _seed(seed: int, name: str) -> int:
@@ -149,6 +149,42 @@ def _kedasun_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
     return out
 
 
+def _fagunex_shapes(cfg: ModelConfig, i: int) -> Dict[str, tuple]:
+    """Tensors of layer i (named by the layer that owns them)."""
+    h, m, f, n = cfg.hidden, cfg.layers[i].mixer, cfg.layers[i].mlp, cfg.token_side
+    p = f"layers.{cfg.weight_layer(i)}."
+    out: Dict[str, tuple] = {"shift": (h,)}
+    for name in ("norm1", "norm1b") + (("norm2", "norm2b") if f is not None else ()):
+        out.update({name + ".weight": (h,), name + ".bias": (h,), name + ".alpha": ()})
+    if isinstance(m, ForgetSpec):
+        d, v = m.heads * m.dim, m.heads * m.vdim
+        out.update({"mixer.q": (d, h), "mixer.f": (d, h), "mixer.f.b": (d,), "mixer.lower": (d,), "mixer.v": (v, h),
+                    "mixer.norm": (m.vdim,), "mixer.o": (h, v)})
+    else:
+        q, v = m.heads * m.q_dim, m.heads * m.vdim
+        out.update({"attn.dkv.weight": (m.kv_rank + m.rot_dim, h), "attn.dkv_norm.weight": (m.kv_rank,),
+                    "attn.uk.weight": (m.heads * m.dim, m.kv_rank), "attn.uv.weight": (v, m.kv_rank), "attn.o.weight": (h, v)})
+        if m.q_rank is None:
+            out["attn.q.weight"] = (q, h)
+        else:
+            out.update({"attn.dq.weight": (m.q_rank, h), "attn.dq_norm.weight": (m.q_rank,), "attn.uq.weight": (q, m.q_rank)})
+        if m.sink:
+            out["attn.sink"] = (m.heads,)
+        if m.gate:
+            out["attn.g.weight"] = (v, h)
+    if f is not None:
+        out.update({"mlp.router.weight": (f.experts, h),
+                    "mlp.experts.gate_up.weight": (f.experts, 2 * f.expert.ff, h),  # gate rows | up rows
+                    "mlp.experts.down.weight": (f.experts, h, f.expert.ff)})
+        if f.shared is not None:
+            out.update({"mlp.shared.gate_up.weight": (2 * f.shared.ff, h), "mlp.shared.down.weight": (h, f.shared.ff)})
+            if f.shared_gate:
+                out["mlp.shared.sg"] = (1, h)
+    if n:
+        out.update({"side.embed": (cfg.vocab_size, n), "side.gate": (n, h), "side.proj": (h, n), "side.norm": (h,)})
+    return {p + k: s for k, s in out.items()}
+
+
 _ATTN_PARTS = ("ln_1.", "attn.", "input_layernorm.", "self_attn.", "mixer.")
 _MLP_PARTS = ("ln_2.", "mlp.", "post_attention_layernorm.")
 
@@ -183,7 +219,7 @@ def stage_tensor_shapes(cfg: ModelConfig, layers: Iterable[int], first: bool, la
                         units: Optional[Tuple[int, int]] = None):
     """Tensors a stage materialises; with `units` only the halves of the
     boundary layers that the stage runs."""
-    if cfg.arch == "vizalix":  # whole layers, several of which may share their tensors
+    if cfg.arch in ("vizalix", "fagunex"):  # whole layers, several of which may share their tensors
         return _stage_tensor_shapes(cfg, layers, first, last)
     return _filter_units(_stage_tensor_shapes(cfg, layers, first, last), units)
 
@@ -207,6 +243,14 @@ def _stage_tensor_shapes(cfg: ModelConfig, layers: Iterable[int], first: bool, l
                 shapes["loop.step"] = (cfg.loop_times, cfg.hidden)
         if last:
             shapes["norm.weight"] = ()
+            shapes["lm_head"] = (cfg.vocab_size, cfg.hidden)
+    elif cfg.arch == "fagunex":
+        if first:
+            shapes["embed_tokens"] = (cfg.vocab_size, cfg.hidden)
+        for i in layers:
+            shapes.update(_fagunex_shapes(cfg, i))
+        if last:
+            shapes.update({"norm.weight": (cfg.hidden,), "norm.bias": (cfg.hidden,), "norm.alpha": ()})
             shapes["lm_head"] = (cfg.vocab_size, cfg.hidden)
     elif cfg.arch == "kedasun":
         if first:
@@ -245,6 +289,8 @@ def _init_one(cfg: ModelConfig, name: str, shape, seed: int, device, dtype) -> t
         return _vizalix_init(cfg, name, shape, seed, device, dtype)
     if cfg.arch == "kedasun":
         return _kedasun_init(name, shape, seed, device, dtype)
+    if cfg.arch == "fagunex":
+        return _fagunex_init(name, shape, seed, device, dtype)
     if name == "embed_tokens":
         # untied (Llama) input embeddings at unit scale (the T5 / muP
         # convention: the residual stream enters at the RMS its norms produce).
@@ -284,12 +330,17 @@ def _timisun_init(cfg: ModelConfig, name: str, shape, seed: int, device, dtype) 
     std = shape[-1] ** -0.5
     if name.endswith(("attn.o.weight", "down.weight")):
         std /= (2 * cfg.n_layers) ** 0.5
-    if len(shape) == 3:  # experts one by one: no fp32 image of the whole stack
-        out = torch.empty(shape, device=device, dtype=dtype)
-        for e in range(shape[0]):
-            out[e] = _randn(shape[1:], std, seed, f"{name}.{e}", device, dtype)
-        return out
+    if len(shape) == 3:
+        return _stacked(shape, std, seed, name, device, dtype)
     return _randn(shape, std, seed, name, device, dtype)
+
+
+def _stacked(shape, std: float, seed: int, name: str, device, dtype) -> torch.Tensor:
+    """Experts one by one: no fp32 image of the whole stack."""
+    out = torch.empty(shape, device=device, dtype=dtype)
+    for e in range(shape[0]):
+        out[e] = _randn(shape[1:], std, seed, f"{name}.{e}", device, dtype)
+    return out
 
 
 def _vizalix_init(cfg: ModelConfig, name: str, shape, seed: int, device, dtype) -> torch.Tensor:
@@ -341,6 +392,33 @@ def _kedasun_init(name: str, shape, seed: int, device, dtype) -> torch.Tensor:
     return _randn(shape, shape[-1] ** -0.5, seed, name, device, dtype)
 
 
+def _fagunex_init(name: str, shape, seed: int, device, dtype) -> torch.Tensor:
+    """Unit-variance projections (the norms behind them bound what enters the
+    residual), forget gates between short and long memory, sinks near the
+    scores, half a token's shift."""
+    def around(mean, std):
+        return (mean + _randn(shape, std, seed, name, device, torch.float32)).to(dtype)
+
+    leaf = name.split(".", 2)[-1] if name.startswith("layers.") else name
+    if leaf == "embed_tokens" or leaf == "side.embed":
+        return _randn(shape, 1.0, seed, name, device, dtype)
+    if leaf.endswith("alpha") or leaf == "shift":
+        return around(0.5, 0.05)
+    if leaf.endswith(".bias"):
+        return _randn(shape, 0.02, seed, name, device, dtype)
+    if leaf.endswith(("norm.weight", "norm")) or (leaf.startswith("norm") and leaf.endswith("weight")):
+        return around(1.0, 0.05)
+    if leaf == "mixer.lower":
+        return around(0.0, 0.3).clamp(0.0, 0.9)
+    if leaf == "mixer.f.b":
+        return around(3.0, 1.5)
+    if leaf == "attn.sink":
+        return around(0.0, 1.0)
+    if len(shape) == 3:
+        return _stacked(shape, shape[-1] ** -0.5, seed, name, device, dtype)
+    return _randn(shape, shape[-1] ** -0.5, seed, name, device, dtype)
+
+
 def init_stage_weights(cfg: ModelConfig, layers, first: bool, last: bool, seed: int,
                        device, dtype, units=None) -> Dict[str, torch.Tensor]:
     shapes = stage_tensor_shapes(cfg, layers, first, last, units)
@@ -355,7 +433,8 @@ _GPT2_CONV1D = ("attn.c_attn.weight", "attn.c_proj.weight", "mlp.c_fc.weight", "
 
 
 def _open_checkpoint(path: str):
-    """Returns a callable name -> tensor that reads lazily where possible."""
+    """(name -> tensor, the names, (name, a, b) -> columns a .. b - 1 of a tensor);
+    reads lazily where possible."""
     files = []
     if os.path.isdir(path):
         for fn in sorted(os.listdir(path)):
@@ -377,11 +456,24 @@ def _open_checkpoint(path: str):
         for h in handles:
             for k in h.keys():
                 index[k] = h
-        return lambda k: index[k].get_tensor(k), set(index)
+        return lambda k: index[k].get_tensor(k), set(index), lambda k, a, b: index[k].get_slice(k)[:, a:b]
     sd = {}
     for f in files:
         sd.update(torch.load(f, map_location="cpu", weights_only=True))  # never unpickles code
-    return lambda k: sd[k], set(sd)
+    return lambda k: sd[k], set(sd), lambda k, a, b: sd[k][:, a:b]
+
+
+def _stack_experts(p: str, rest: str, experts: int, get) -> torch.Tensor:
+    """Expert tensors of the layer with checkpoint prefix p: gate and up joined,
+    routed experts stacked."""
+    def part(prefix: str) -> torch.Tensor:
+        if rest.endswith("gate_up.weight"):
+            return torch.cat([get(prefix + "gate"), get(prefix + "up")], 0)
+        return get(prefix + "down")
+
+    if rest.startswith("mlp.shared."):
+        return part(p + "mlp.shared.")
+    return torch.stack([part(f"{p}mlp.e{e}.") for e in range(experts)])
 
 
 def _timisun_tensor(cfg: ModelConfig, name: str, get) -> torch.Tensor:
@@ -398,18 +490,9 @@ def _timisun_tensor(cfg: ModelConfig, name: str, get) -> torch.Tensor:
     if rest.startswith("attn."):
         leaf = rest.split(".")[1]
         return get(p + "mix." + {"dkv_norm": "dkv.norm"}.get(leaf, leaf))
-    p += "mlp."
     if rest in ("mlp.router.weight", "mlp.correction"):
-        return get(p + rest.split(".")[1])
-
-    def part(prefix: str) -> torch.Tensor:
-        if rest.endswith("gate_up.weight"):
-            return torch.cat([get(prefix + "gate"), get(prefix + "up")], 0)
-        return get(prefix + "down")
-
-    if rest.startswith("mlp.shared."):
-        return part(p + "shared.")
-    return torch.stack([part(f"{p}e{e}.") for e in range(cfg.layers[int(i)].mlp.experts)])
+        return get(p + "mlp." + rest.split(".")[1])
+    return _stack_experts(p, rest, cfg.layers[int(i)].mlp.experts, get)
 
 
 def _vizalix_tensor(name: str, get) -> torch.Tensor:
@@ -442,9 +525,39 @@ def _kedasun_tensor(name: str, get) -> torch.Tensor:
     return get(f"l{i}.mix." + rest[len("mixer."):])
 
 
+def _fagunex_tensor(cfg: ModelConfig, name: str, get, get_columns) -> torch.Tensor:
+    """One canonical tensor from a checkpoint in the design's own names;
+    get_columns(name, a, b) reads some columns of a tensor."""
+    norm = {"weight": "", "bias": ".b", "alpha": ".alpha"}
+    top = {"embed_tokens": "embed", "lm_head": "head"}
+    if name in top:
+        return get(top[name])
+    if name.startswith("norm."):
+        return get("final.norm" + norm[name.split(".")[1]])
+    _, i, rest = name.split(".", 2)
+    p = f"l{i}."
+    if rest.startswith("norm"):
+        n, leaf = rest.split(".")
+        return get(p + n + norm[leaf])
+    if rest == "side.embed":  # one table for all layers, a layer's columns side by side
+        n = cfg.token_side
+        return get_columns("side.embed", int(i) * n, int(i) * n + n)
+    if rest.startswith(("side.", "shift")):
+        return get(p + rest)
+    if rest.startswith("mixer."):
+        return get(p + "mix." + rest[len("mixer."):])
+    if rest.startswith("attn."):
+        leaf = rest.split(".")[1]
+        return get(p + "mix." + {"dkv_norm": "dkv.norm", "dq_norm": "dq.norm"}.get(leaf, leaf))
+    if rest in ("mlp.router.weight", "mlp.shared.sg"):
+        return get(p + rest.removesuffix(".weight"))
+    run = next(l for j, l in enumerate(cfg.layers) if cfg.weight_layer(j) == int(i))
+    return _stack_experts(p, rest, run.mlp.experts, get)
+
+
 def load_stage_weights(cfg: ModelConfig, path: str, layers, first: bool, last: bool,
                        device, dtype, units=None) -> Dict[str, torch.Tensor]:
-    get, keys = _open_checkpoint(path)
+    get, keys, get_columns = _open_checkpoint(path)
     out: Dict[str, torch.Tensor] = {}
     want = stage_tensor_shapes(cfg, layers, first, last, units)
 
@@ -461,6 +574,8 @@ def load_stage_weights(cfg: ModelConfig, path: str, layers, first: bool, last: b
             t = _vizalix_tensor(name, get)
         elif cfg.arch == "kedasun":
             t = _kedasun_tensor(name, get)
+        elif cfg.arch == "fagunex":
+            t = _fagunex_tensor(cfg, name, get, get_columns)
         elif cfg.arch == "gpt2":
             src = {"wte": "wte.weight", "wpe": "wpe.weight"}.get(name, name)
             t = find(src)

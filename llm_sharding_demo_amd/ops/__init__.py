@@ -59,9 +59,9 @@ class Backend:
         """Columns of a value head (>= vdim; the rest stays zero)."""
         return mixer.vdim
 
-    def layer_cache(self, mixer) -> LayerCache:
+    def layer_cache(self, mixer, shift: int = 0) -> LayerCache:
         """What a layer keeps per page and per slot (runtime/kv_cache.py)."""
-        return layer_cache(mixer)
+        return layer_cache(mixer, shift=shift)
 
     def norm_width(self, mcfg) -> int:
         """`width` argument of the norms: the true row width where rows are padded, else 0."""
@@ -113,44 +113,97 @@ class ReferenceBackend(Backend):
 
     # -- latent attention and experts (models/stage.py _parallel_layer) -------
     # `w(name)`: the layer's tensors; `pool`: its cache layer (kv.pools)
-    def latent_project(self, h, w, spec, kv, pool, meta, eps):
-        """Queries [T, heads, rank] in the latent space and the routing (ids,
-        weights); a layer with its own latents appends them to the cache."""
-        m = spec.mixer
+    def latent_project(self, h, w, m, mlp, kv, pool, meta, eps):
+        """Queries [T, heads, rank + turned part] in the latent space, the output
+        gate's logits (None: no gate) and, for experts `mlp` that read the same
+        rows, the routing (ids, weights); a layer with its own latents appends
+        them to the cache."""
+        pos = meta.token_pos
         if m.kv_from is None:
-            c = ref.rmsnorm(ref.linear(h, w("attn.dkv.weight")), w("attn.dkv_norm.weight"), eps)
-            ref.latent_append(pool, kv.table, c, meta.token_slots, meta.token_pos)
-        q = ref.linear(h, w("attn.q.weight")).reshape(-1, m.heads, m.dim)
+            c, kr = ref.linear(h, w("attn.dkv.weight")).split([m.kv_rank, m.rot_dim], 1)
+            c = torch.cat([ref.rmsnorm(c, w("attn.dkv_norm.weight"), eps), ref.partial_rope(kr[:, None], pos, m.rope)[:, 0]], 1)
+            ref.latent_append(pool, kv.table, c, meta.token_slots, pos)
+        if m.q_rank is None:
+            q = ref.linear(h, w("attn.q.weight"))
+        else:
+            q = ref.linear(ref.rmsnorm(ref.linear(h, w("attn.dq.weight")), w("attn.dq_norm.weight"), eps), w("attn.uq.weight"))
+        q, qr = q.reshape(-1, m.heads, m.q_dim).split([m.dim, m.rot_dim], 2)
         uk = w("attn.uk.weight").float().reshape(m.heads, m.dim, m.kv_rank)
         q = torch.matmul(q.transpose(0, 1), uk).transpose(0, 1)
+        q = torch.cat([q, ref.partial_rope(qr, pos, m.rope)], 2)
+        gate = ref.linear(h, w("attn.g.weight")) if m.gate else None
         routing = None
-        if spec.mlp is not None:
+        if mlp is not None:
             z = ref.linear(h, w("mlp.router.weight"))
-            routing = ref.route(z, w("mlp.correction"), spec.mlp.top)
-        return q, routing
+            routing = ref.route(z, w("mlp.correction"), mlp.top)
+        return q, gate, routing
 
-    def latent_attention(self, q, w, m, kv, pool, meta):
-        parts = [(q, meta)]
-        if getattr(meta, "dec", None) is not None:
-            parts = [(q[: meta.b], meta.dec), (q[meta.b:], meta.pf)]
-        o = torch.cat([ref.latent_attention(x, pool, kv.table, mt.seq_slots, mt.q_start, mt.cu_q, m.scale, m.window)
-                       for x, mt in parts])
+    def latent_attention(self, q, gate, w, m, kv, pool, meta):
+        sink = w("attn.sink").float() if m.sink else None
+        o = torch.cat([ref.latent_attention(q[s], pool, kv.table, mt.seq_slots, mt.q_start, mt.cu_q, m.scale, m.window,
+                                            m.kv_rank, sink) for s, mt in self._parts(meta)])
         uv = w("attn.uv.weight").float().reshape(m.heads, m.vdim, m.kv_rank)
         o = torch.matmul(o.transpose(0, 1), uv.transpose(1, 2)).transpose(0, 1)
-        return o.reshape(o.shape[0], -1)
+        o = o.reshape(o.shape[0], -1)
+        return o if gate is None else o * torch.sigmoid(gate)
 
     def parallel_residual(self, o, h, routing, w, spec, r: Residual) -> None:
         """x += o W_o^T + experts(h): both halves of a parallel block."""
         self.linear_residual(o, w("attn.o.weight"), None, r)
         if spec is None:
             return
+        r.x += self._experts(h, routing, w, spec)
+
+    def _experts(self, h, routing, w, spec):
         ids, wts = routing
         y = ref.moe(h, ids, wts, w("mlp.experts.gate_up.weight"), w("mlp.experts.down.weight"), spec.expert.limit,
                     GLU_ALPHA)
         if spec.shared is not None:
-            y = y + ref.expert(h, w("mlp.shared.gate_up.weight"), w("mlp.shared.down.weight"), spec.shared.limit,
-                               GLU_ALPHA)
-        r.x += y
+            z = ref.expert(h, w("mlp.shared.gate_up.weight"), w("mlp.shared.down.weight"), spec.shared.limit, GLU_ALPHA)
+            y = y + (z * torch.sigmoid(ref.linear(h, w("mlp.shared.sg"))) if spec.shared_gate else z)
+        return y
+
+    # -- layers with elementwise norms (models/stage.py _token_layer); a norm is
+    # n(".weight"), n(".bias") and one number n(".alpha") --------------------------
+    def tanh_norm(self, r: Residual, n):
+        self._combine(r)
+        return ref.tanh_norm(r.x, n(".alpha"), n(".weight"), n(".bias"))
+
+    def tanh_norm_rows(self, x, n, rows=None):
+        return self.tanh_norm(Residual(x if rows is None else x.index_select(0, rows.long())), n)
+
+    def shift_norm(self, r: Residual, w, last, meta, mcfg):
+        """The layer's first norm, its rows moved towards the previous token's by
+        w("shift"); `last` [slots, hidden]: the previous portion's last row."""
+        h = self.tanh_norm(r, lambda n: w("norm1" + n))
+        return torch.cat([ref.token_shift(h[s], w("shift"), last, mt) for s, mt in self._parts(meta)])
+
+    def linear_tanh(self, a, wt, n, r: Residual) -> None:
+        """x += norm(a wt^T)."""
+        self._combine(r)
+        r.x += self.tanh_norm(Residual(ref.linear(a, wt)), n)
+
+    def experts_tanh(self, h, w, mlp, n, r: Residual) -> None:
+        """x += norm(experts(h))."""
+        self._combine(r)
+        routing = ref.route_softmax(ref.linear(h, w("mlp.router.weight")), mlp.top)
+        r.x += self.tanh_norm(Residual(self._experts(h, routing, w, mlp)), n)
+
+    def token_side(self, r: Residual, ids, w, mcfg) -> None:
+        """x += rms(proj(gelu(gate x) * e)) * norm, e the tokens' rows of the layer's table."""
+        self._combine(r)
+        g = ref.gelu_new(ref.linear(r.x, w("side.gate"))) * w("side.embed").index_select(0, ids.long()).float()
+        r.x += ref.rmsnorm(ref.linear(g, w("side.proj")), w("side.norm"), mcfg.norm_eps)
+
+    def forget_mix(self, h, w, m, state, meta, eps):
+        """Recurrence with forget gates before W_o [T, heads * vdim]."""
+        T, H, D, V = h.shape[0], m.heads, m.dim, m.vdim
+        q = torch.nn.functional.silu(ref.linear(h, w("mixer.q"))).view(T, H, D)
+        # 1 - f, formed without cancellation where f is close to one
+        k = (1 - w("mixer.lower").float()) * torch.sigmoid(-ref.linear(h, w("mixer.f"), w("mixer.f.b")))
+        k, v = k.view(T, H, D), ref.linear(h, w("mixer.v")).view(T, H, V)
+        o = torch.cat([ref.forget_rule(q[s], k[s], v[s], state, mt) for s, mt in self._parts(meta)])
+        return ref.rmsnorm(o, w("mixer.norm"), eps).view(T, H * V)
 
     # -- mixers of models/stage.py _mixer_layer --------------------------------
     def loop_enter(self, r: Residual, x0, w_in, step, t: int) -> None:

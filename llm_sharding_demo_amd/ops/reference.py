@@ -138,11 +138,14 @@ def latent_append(pool: torch.Tensor, table: torch.Tensor, c: torch.Tensor, slot
 
 
 def latent_attention(q: torch.Tensor, pool: torch.Tensor, table: torch.Tensor, seq_slots, q_start, cu_q,
-                     scale: float, window: Optional[int]) -> torch.Tensor:
-    """q [T, heads, rank] in the latent space; the cached latents are keys and
-    values of every head.  Query at position i sees i - window < j <= i.
-    Returns fp32 [T, heads, rank]."""
-    out = torch.empty(q.shape, dtype=torch.float32, device=q.device)
+                     scale: float, window: Optional[int], vdim: Optional[int] = None,
+                     sink: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """q [T, heads, columns] in the latent space; the cached rows are keys of every
+    head, their first vdim columns (None: all) the values.  Query at position i
+    sees i - window < j <= i; sink [heads]: a further score without a value.
+    Returns fp32 [T, heads, vdim]."""
+    vdim = q.shape[2] if vdim is None else vdim
+    out = torch.empty(*q.shape[:2], vdim, dtype=torch.float32, device=q.device)
     flat = pool.view(-1, pool.shape[2])
     for i in range(seq_slots.numel()):
         a, b = int(cu_q[i]), int(cu_q[i + 1])
@@ -151,12 +154,15 @@ def latent_attention(q: torch.Tensor, pool: torch.Tensor, table: torch.Tensor, s
         st, end = int(q_start[i]), int(q_start[i]) + b - a
         lo = 0 if window is None else max(0, st - window + 1)
         kpos = torch.arange(lo, end, device=q.device)
-        c = flat[paged_rows(table, seq_slots[i].expand_as(kpos), kpos, pool.shape[1])].float()
+        c = flat[paged_rows(table, seq_slots[i].expand_as(kpos), kpos, pool.shape[1])].float()[:, : q.shape[2]]
         s = torch.matmul(q[a:b].float().transpose(0, 1), c.t()) * scale  # [heads, Lq, keys]
         d = torch.arange(st, end, device=q.device)[:, None] - kpos[None, :]
         hide = d < 0 if window is None else (d < 0) | (d >= window)
-        p = torch.softmax(s.masked_fill(hide, float("-inf")), dim=-1)
-        out[a:b] = torch.matmul(p, c).transpose(0, 1)
+        s = s.masked_fill(hide, float("-inf"))
+        if sink is not None:
+            s = torch.cat([s, sink[:, None, None].expand(-1, b - a, 1)], 2)
+        p = torch.softmax(s, dim=-1)[..., : kpos.numel()]
+        out[a:b] = torch.matmul(p, c[:, :vdim]).transpose(0, 1)
     return out
 
 
@@ -277,6 +283,47 @@ def ssd(x, B, C, dt, decay, state, meta) -> torch.Tensor:
     return out
 
 
+def forget_rule(q, k, v, state, meta) -> torch.Tensor:
+    """S <- diag(1 - k) S + k v^T; o = S^T q.  q, k [T, H, D], v [T, H, V],
+    state [slots, H, D, V]."""
+    out = torch.empty(v.shape, dtype=torch.float32)
+
+    def step(t, S):
+        S = S + k[t][..., None] * (v[t][:, None] - S)
+        out[t] = torch.matmul(q[t][:, None], S)[:, 0]
+        return S
+    _scan(meta, state, step)
+    return out
+
+
+def tanh_norm(x: torch.Tensor, alpha: torch.Tensor, w: torch.Tensor, b: torch.Tensor) -> torch.Tensor:
+    """Dynamic tanh: no statistics of the row."""
+    return torch.tanh(alpha.float() * x.float()) * w.float() + b.float()
+
+
+def token_shift(h: torch.Tensor, amount: torch.Tensor, last: torch.Tensor, meta) -> torch.Tensor:
+    """Packed rows, each moved towards its sequence's previous one by `amount` per
+    column; last [slots, width] holds the row before a portion (zeros before
+    position 0) and is brought up to date."""
+    out = torch.empty_like(h)
+    for i in range(meta.seq_slots.numel()):
+        a, b, slot = int(meta.cu_q[i]), int(meta.cu_q[i + 1]), int(meta.seq_slots[i])
+        if b == a:
+            continue
+        first = last[slot: slot + 1] if int(meta.q_start[i]) > 0 else torch.zeros_like(h[:1])
+        before = torch.cat([first, h[a: b - 1]])
+        out[a:b] = h[a:b] + (before - h[a:b]) * amount.float()
+        last[slot] = h[b - 1]
+    return out
+
+
+def route_softmax(z: torch.Tensor, top: int):
+    """Router logits [T, E] -> (expert ids [T, top], weights [T, top]): the largest
+    logits choose, their softmax weighs."""
+    z, ids = torch.topk(z.float(), top, dim=-1)
+    return ids, torch.softmax(z, -1)
+
+
 def route(z: torch.Tensor, correction: torch.Tensor, top: int):
     """Router logits [T, E] -> (expert ids [T, top], weights [T, top]): the
     corrected sigmoid scores choose, the plain ones weigh."""
@@ -286,19 +333,22 @@ def route(z: torch.Tensor, correction: torch.Tensor, top: int):
     return ids, w / (w.sum(-1, keepdim=True) + 1e-20)
 
 
-def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
+def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: Optional[float], alpha: float) -> torch.Tensor:
+    """limit None: plain SiLU(gate) * up."""
+    if limit is None:
+        return silu_mul(gate, up)
     g = gate.clamp(max=limit)
     return g * torch.sigmoid(alpha * g) * (up.clamp(-limit, limit) + 1)
 
 
-def expert(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
+def expert(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, limit: Optional[float], alpha: float) -> torch.Tensor:
     y = linear(h, gate_up)
     f = y.shape[1] // 2
     return linear(clamped_glu(y[:, :f], y[:, f:], limit, alpha), down)
 
 
 def moe(h: torch.Tensor, ids: torch.Tensor, w: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
-        limit: float, alpha: float) -> torch.Tensor:
+        limit: Optional[float], alpha: float) -> torch.Tensor:
     out = torch.zeros(h.shape[0], down.shape[1], dtype=torch.float32, device=h.device)
     for e in ids.unique().tolist():
         t, k = (ids == e).nonzero(as_tuple=True)

@@ -21,7 +21,7 @@ from __future__ import annotations
 
 from typing import List, Optional, Sequence, Tuple
 
-from ..config import ModelConfig
+from ..config import ForgetSpec, ModelConfig
 
 Plan = List[Tuple[int, int]]
 
@@ -172,16 +172,26 @@ def _layer_costs(cfg: ModelConfig, rows: int, avg_ctx: int):
         if cfg.arch in ("vizalix", "kedasun"):
             costs += [_mixer_cost(cfg, l, rows, avg_ctx), 0.0]
             continue
-        n_in = m.heads * m.dim + (m.kv_rank if m.kv_from is None else 0) + (f.experts if f else 0)
-        ctx = min(avg_ctx, m.window or avg_ctx)
-        c = 6.0 + _gemm_us(n_in, h, rows) + 4.0 + 3.0 + rows * ctx * m.kv_rank * 2 / 6.0e6
-        c += _gemm_us(m.heads * m.dim, m.kv_rank, rows) + _gemm_us(m.heads * m.vdim, m.kv_rank, rows)
-        c += _gemm_us(h, m.heads * m.vdim, rows)
+        c = _gemm_us(h, m.heads * m.vdim, rows)
+        if isinstance(m, ForgetSpec):  # the state is read and written once
+            c += 6.0 + _gemm_us(2 * m.heads * (m.dim + m.vdim) - m.heads * m.vdim, h, rows)
+            c += 6.0 + rows * 8 * m.heads * m.dim * m.vdim / 5.0e6
+        else:
+            n_in = m.in_columns + (f.experts if f and cfg.arch == "timisun" else 0)
+            ctx = min(avg_ctx, m.window or avg_ctx)
+            c += 6.0 + _gemm_us(n_in, h, rows) + 4.0 + 3.0 + rows * ctx * (m.kv_rank + m.rot_dim) * 2 / 6.0e6
+            c += _gemm_us(m.heads * m.dim, m.kv_rank, rows) + _gemm_us(m.heads * m.vdim, m.kv_rank, rows)
+            if m.q_rank is not None:
+                c += 4.0 + _gemm_us(m.heads * m.q_dim, m.q_rank, rows)
         if f:
             used = min(f.experts, rows * f.top)  # experts whose weights a step reads
             params = 3 * h * (used * f.expert.ff + (f.shared.ff if f.shared else 0))
             flops = 6.0 * h * rows * (f.top * f.expert.ff + (f.shared.ff if f.shared else 0))
             c += 15.0 + 2 * params / 4.0e6 + flops / 0.45e9
+            if cfg.arch == "fagunex":  # norms and a router of its own
+                c += 14.0 + _gemm_us(f.experts, h, rows)
+        if cfg.token_side:
+            c += 14.0 + _gemm_us(cfg.token_side, h, rows) + _gemm_us(h, cfg.token_side, rows)
         costs += [c, 0.0]
     head = 6.0 + _gemm_us(cfg.vocab_padded, h, rows) + 8.0 + 0.37 * min(rows, 128)
     return costs, head, 4.0

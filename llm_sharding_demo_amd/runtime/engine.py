@@ -311,7 +311,7 @@ class Engine(racecheck.Shared):
             for i, d in enumerate(devices):
                 if str(d) == str(dev):
                     a, b = self.unit_plan[self.stage_idx if collective else i]
-                    caches += [layer_cache(self.mcfg.layers[j].mixer, pad_up)
+                    caches += [layer_cache(self.mcfg.layers[j].mixer, pad_up, self.mcfg.shift_width)
                                for j in self.mcfg.cache_layers(range(a // 2, b // 2))]
             states = (slots + 2) * sum(c.slot_bytes(elt) for c in caches)
             fits = min(fits, plan_pages(want, sum(c.page_bytes(elt) for c in caches), dev, fraction=self.cfg.kv_fraction,

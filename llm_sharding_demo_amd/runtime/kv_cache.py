@@ -21,7 +21,7 @@ from typing import Callable, List, Sequence, Tuple
 
 import torch
 
-from ..config import AttentionSpec, ChannelDeltaSpec, SSMSpec
+from ..config import AttentionSpec, ChannelDeltaSpec, ForgetSpec, SSMSpec
 
 PAGE = 64  # tokens per page of a paged cache (csrc/kernels/attention_latent.hip)
 
@@ -74,13 +74,18 @@ class LayerCache:
         return sum(4 * torch.Size(s).numel() for s in self.state) + sum(elt * torch.Size(s).numel() for s in self.ring)
 
 
-def layer_cache(mixer, up: Callable[[int, int], int] = lambda n, m: n) -> LayerCache:
+def layer_cache(mixer, up: Callable[[int, int], int] = lambda n, m: n, shift: int = 0) -> LayerCache:
     """Cache of one layer; up(n, m): the backend's padding of n to a multiple of m.
+    shift: columns of the last token's row that the layer keeps too, the last of its state.
       attention   K [kv head][token][dim], V [kv head][token][vdim] per page, and the
                   q | k | v rows of positions p % taps in front of a short convolution
       delta rule  S [heads][dim][vdim] and the conv inputs of positions p % taps
       Mamba-2     S [heads][state][vdim], and the same
-      latent      one row of `rank` per token"""
+      forget gate S [heads][dim][vdim]
+      latent      one row per token: `rank` columns and the turned key part"""
+    if shift:
+        c = layer_cache(mixer, up)
+        return LayerCache(c.pages, c.state + ((up(shift, 64),),), c.ring)
     if isinstance(mixer, AttentionSpec):
         g = mixer.kv_heads
         dp, vp = up(mixer.dim, 32), up(mixer.vdim, 16)
@@ -89,7 +94,9 @@ def layer_cache(mixer, up: Callable[[int, int], int] = lambda n, m: n) -> LayerC
     if isinstance(mixer, (ChannelDeltaSpec, SSMSpec)):
         rows = mixer.dim if isinstance(mixer, ChannelDeltaSpec) else mixer.state
         return LayerCache(state=((mixer.heads, rows, up(mixer.vdim, 4)),), ring=((mixer.conv, mixer.conv_channels),))
-    return LayerCache(pages=((PAGE, up(mixer.kv_rank, 64)),))
+    if isinstance(mixer, ForgetSpec):
+        return LayerCache(state=((mixer.heads, mixer.dim, up(mixer.vdim, 4)),))
+    return LayerCache(pages=((PAGE, up(mixer.kv_rank + mixer.rot_dim, 64)),))
 
 
 class PagedCache:
