@@ -7,6 +7,10 @@
 // serve as keys and as values.  One cached row per token, no per-head cache.
 // A window (`window` keys ending with the query itself) bounds the key range.
 //
+// A turned key part that all heads share is cached behind the latent: the way into
+// the latent space passes the queries' turned part on, and only the first columns
+// of a row are values.  A sink is one more score of the softmax, without a value.
+//
 // Cache: [page][64 tokens][rank], pages found through table[slot][pos / 64].
 // A 32- or 64-key tile never crosses a page.
 //
@@ -35,6 +39,7 @@ namespace {
 
 constexpr float NEG = -1e30f;
 constexpr int PAGE = 64;
+constexpr float LOG2E = 1.4426950408889634f;
 
 __device__ __forceinline__ bf16x4 ds_read_tr(const bf16* lds_ptr) {
   typedef __attribute__((address_space(3))) bf16x4 lds_bf16x4;
@@ -60,7 +65,7 @@ __device__ __forceinline__ void split_p(const f32x4& a, const f32x4& b, bf16x8& 
   }
 }
 
-template <int RANK, int QT, int NW, int KT>
+template <int RANK, int VR, int QT, int NW, int KT>
 __global__ __launch_bounds__(NW * 64) void latent_prefill_kernel(LatentAttnParams p) {
   constexpr int LDR = RANK + 8;
   constexpr int CPR = RANK / 8;
@@ -93,14 +98,15 @@ __global__ __launch_bounds__(NW * 64) void latent_prefill_kernel(LatentAttnParam
   const int hi = st + min(off + ROWS - 1, nrows - 1) / H + 1;  // keys [lo, hi)
   const int kt0 = lo / KT, kt1 = (hi + KT - 1) / KT;
 
-  f32x4 o[QT][RANK / 16];
+  f32x4 o[QT][VR / 16];
   float m[QT], lsum[QT];
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
-    m[t] = NEG;
-    lsum[t] = 0.f;
+    // a sink is a key that was seen first, without a value
+    m[t] = p.sink ? p.sink[min(row[t], nrows - 1) % H] * LOG2E : NEG;
+    lsum[t] = p.sink && g == 0 ? 1.f : 0.f;
 #pragma unroll
-    for (int di = 0; di < RANK / 16; ++di) o[t][di] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int di = 0; di < VR / 16; ++di) o[t][di] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   bf16x8 creg[CH];
   auto load_tile = [&](int kt) {
@@ -154,7 +160,7 @@ __global__ __launch_bounds__(NW * 64) void latent_prefill_kernel(LatentAttnParam
         m[t] = mn;
         lsum[t] *= alpha;
 #pragma unroll
-        for (int di = 0; di < RANK / 16; ++di) o[t][di] *= alpha;
+        for (int di = 0; di < VR / 16; ++di) o[t][di] *= alpha;
       }
       // a query whose window has not begun yet: nothing to weigh
       const float off2 = m[t] > 0.5f * NEG ? m[t] : 0.f;
@@ -178,7 +184,7 @@ __global__ __launch_bounds__(NW * 64) void latent_prefill_kernel(LatentAttnParam
       for (int t = 0; t < QT; ++t) split_p(s[t][2 * kk], s[t][2 * kk + 1], ph[t], pl[t]);
       const int r0 = kk * 32 + 4 * g + (r >> 2);
 #pragma unroll
-      for (int di = 0; di < RANK / 16; ++di) {
+      for (int di = 0; di < VR / 16; ++di) {
         const int col = di * 16 + 4 * (r & 3);
         const bf16x4 a = ds_read_tr(cs + r0 * LDR + col);
         const bf16x4 b = ds_read_tr(cs + (r0 + 16) * LDR + col);
@@ -191,7 +197,7 @@ __global__ __launch_bounds__(NW * 64) void latent_prefill_kernel(LatentAttnParam
       }
     }
   }
-  bf16* obase = static_cast<bf16*>(p.out) + (long)cu * H * RANK;
+  bf16* obase = static_cast<bf16*>(p.out) + (long)cu * H * VR;
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
     float l = lsum[t];
@@ -200,18 +206,18 @@ __global__ __launch_bounds__(NW * 64) void latent_prefill_kernel(LatentAttnParam
     if (row[t] >= nrows) continue;
     const float inv = 1.f / l;
 #pragma unroll
-    for (int di = 0; di < RANK / 16; ++di) {
+    for (int di = 0; di < VR / 16; ++di) {
       bf16x4 rr;
 #pragma unroll
       for (int i = 0; i < 4; ++i) rr[i] = f2bf(o[t][di][i] * inv);
-      st4(obase + (long)row[t] * RANK + di * 16 + 4 * g, rr);
+      st4(obase + (long)row[t] * VR + di * 16 + 4 * g, rr);
     }
   }
 }
 
 // 16 heads of one token per block; waves take the 32-key tiles in turn.
 // Two blocks per CU where the tiles leave the LDS for it.
-template <int RANK>
+template <int RANK, int VR>
 __global__ __launch_bounds__(256, RANK <= 256 ? 2 : 1) void latent_decode_kernel(LatentAttnParams p) {
   constexpr int KT = 32;
   constexpr int LDR = RANK + 8;
@@ -219,7 +225,7 @@ __global__ __launch_bounds__(256, RANK <= 256 ? 2 : 1) void latent_decode_kernel
   constexpr int CH = KT * CPR / 64;
   __shared__ __attribute__((aligned(16))) bf16 lds[4][KT * LDR];  // a wave's tile, then its O^T
   __shared__ float ml[4][16][2];
-  static_assert(KT * LDR * 2 >= RANK * 16 * 4, "the partial output fits the key tile");
+  static_assert(KT * LDR * 2 >= VR * 16 * 4, "the partial output fits the key tile");
   const int H = p.H, HG = (H + 15) / 16;
   const int item = xcd_remap(blockIdx.x, gridDim.x);  // a token's head groups on one XCD
   const int b = item / HG, h0 = (item % HG) * 16;
@@ -237,10 +243,14 @@ __global__ __launch_bounds__(256, RANK <= 256 ? 2 : 1) void latent_decode_kernel
   const bf16* q = static_cast<const bf16*>(p.q) + ((long)b * H + min(h0 + r, H - 1)) * RANK;
 #pragma unroll
   for (int kk = 0; kk < RANK / 32; ++kk) qf[kk] = ld8(q + kk * 32 + g * 8);
-  f32x4 o[RANK / 16];
+  f32x4 o[VR / 16];
 #pragma unroll
-  for (int di = 0; di < RANK / 16; ++di) o[di] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int di = 0; di < VR / 16; ++di) o[di] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = NEG, lsum = 0.f;
+  if (p.sink && w == 0 && blockIdx.y == 0) {  // a key that was seen first, without a value
+    m = p.sink[min(h0 + r, H - 1)] * LOG2E;
+    lsum = g == 0 ? 1.f : 0.f;
+  }
 
   bf16x8 creg[CH];
   auto page_of = [&](int kt) { return table[min(kt, tb - 1) * KT / PAGE]; };
@@ -300,7 +310,7 @@ __global__ __launch_bounds__(256, RANK <= 256 ? 2 : 1) void latent_decode_kernel
       m = mn;
       lsum *= alpha;
 #pragma unroll
-      for (int di = 0; di < RANK / 16; ++di) o[di] *= alpha;
+      for (int di = 0; di < VR / 16; ++di) o[di] *= alpha;
     }
     float ps = 0.f;
 #pragma unroll
@@ -317,7 +327,7 @@ __global__ __launch_bounds__(256, RANK <= 256 ? 2 : 1) void latent_decode_kernel
     split_p(s[0], s[1], ph, pl);
     const int r0 = 4 * g + (r >> 2);
 #pragma unroll
-    for (int di = 0; di < RANK / 16; ++di) {
+    for (int di = 0; di < VR / 16; ++di) {
       const int col = di * 16 + 4 * (r & 3);
       const bf16x4 a = ds_read_tr(cs + r0 * LDR + col);
       const bf16x4 c = ds_read_tr(cs + (r0 + 16) * LDR + col);
@@ -341,12 +351,12 @@ __global__ __launch_bounds__(256, RANK <= 256 ? 2 : 1) void latent_decode_kernel
   const float f = exp2f(m - M);
   float* ow = reinterpret_cast<float*>(cs);  // [di][g][r][4]
 #pragma unroll
-  for (int di = 0; di < RANK / 16; ++di)
+  for (int di = 0; di < VR / 16; ++di)
     *reinterpret_cast<f32x4*>(ow + ((di * 4 + g) * 16 + r) * 4) = o[di] * f;
   __syncthreads();
   // thread -> (dimension group, head): its head is r again (256 % 16 == 0)
   const int h = h0 + r;
-  for (int u = threadIdx.x; u < RANK * 4; u += 256) {
+  for (int u = threadIdx.x; u < VR * 4; u += 256) {
     f32x4 v = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int i = 0; i < 4; ++i) v += *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(lds[i]) + u * 4);
@@ -354,14 +364,14 @@ __global__ __launch_bounds__(256, RANK <= 256 ? 2 : 1) void latent_decode_kernel
     const int d = (u >> 4) * 4;
     if (p.splits > 1) {
       const long pi = ((long)b * H + h) * p.splits + blockIdx.y;
-      *reinterpret_cast<f32x4*>(p.part_o + pi * RANK + d) = v;
+      *reinterpret_cast<f32x4*>(p.part_o + pi * VR + d) = v;
       if (d == 0) {
         p.part_ml[2 * pi] = M;
         p.part_ml[2 * pi + 1] = L;
       }
     } else {
       const float inv = 1.f / L;
-      st4(static_cast<bf16*>(p.out) + ((long)b * H + h) * RANK + d,
+      st4(static_cast<bf16*>(p.out) + ((long)b * H + h) * VR + d,
           bf16x4{f2bf(v[0] * inv), f2bf(v[1] * inv), f2bf(v[2] * inv), f2bf(v[3] * inv)});
     }
   }
@@ -435,8 +445,8 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentExpandedP
   float m[QT], lsum[QT];
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
-    m[t] = NEG;
-    lsum[t] = 0.f;
+    m[t] = p.sink ? p.sink[h] * LOG2E : NEG;  // a key that was seen first, without a value
+    lsum[t] = p.sink && g == 0 ? 1.f : 0.f;
 #pragma unroll
     for (int di = 0; di < VP / 16; ++di) o[t][di] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
@@ -554,10 +564,13 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentExpandedP
 #pragma unroll
     for (int di = 0; di < VP / 16; ++di) {
       if (di * 16 >= p.vdim) continue;
-      bf16x4 rr;
+      f32x4 v = o[t][di] * inv;
+      if (p.gate) {
+        const f32x4 z = *reinterpret_cast<const f32x4*>(p.gate + (cu + qi[t]) * p.ldg + (long)h * p.vdim + di * 16 + 4 * g);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) rr[i] = f2bf(o[t][di][i] * inv);
-      st4(op + di * 16 + 4 * g, rr);
+        for (int i = 0; i < 4; ++i) v[i] *= __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-LOG2E * z[i]));
+      }
+      st4(op + di * 16 + 4 * g, pack4(v));
     }
   }
 }
@@ -598,7 +611,8 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(LatentAttnParams p) {
   const T* q = static_cast<const T*>(p.q) + ((long)t * p.H + h) * R;
   for (int i = tid; i < R; i += 256) qs[i] = to_f(q[i]) * p.scale_log2;
   float o[OPT] = {};
-  float m = NEG, l = 0.f;
+  float m = p.sink ? p.sink[h] * LOG2E : NEG, l = p.sink ? 1.f : 0.f;
+  const int V = p.v_pad;
   __syncthreads();
   for (int k0 = lo; k0 <= pos; k0 += 256) {
     const int key = k0 + tid;
@@ -628,15 +642,15 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(LatentAttnParams p) {
       const float pv = ps[i];
 #pragma unroll
       for (int j = 0; j < OPT; ++j)
-        if (tid + 256 * j < R) o[j] = fmaf(pv, to_f(c[tid + 256 * j]), o[j]);
+        if (tid + 256 * j < V) o[j] = fmaf(pv, to_f(c[tid + 256 * j]), o[j]);
     }
     __syncthreads();
   }
-  T* out = static_cast<T*>(p.out) + ((long)t * p.H + h) * R;
+  T* out = static_cast<T*>(p.out) + ((long)t * p.H + h) * V;
   const float inv = 1.f / l;
 #pragma unroll
   for (int j = 0; j < OPT; ++j)
-    if (tid + 256 * j < R) from_f(out + tid + 256 * j, o[j] * inv);
+    if (tid + 256 * j < V) from_f(out + tid + 256 * j, o[j] * inv);
 }
 
 }  // namespace
@@ -646,15 +660,27 @@ using namespace lsd;
 
 // Query rows of one prefill tile for this rank, 0: no MFMA kernel.
 extern "C" int lsd_latent_tile_rows(int rank) {
-  if (rank % 64 || rank > 512 || rank == 0) return 0;
+  if (rank % 64 || rank > 576 || rank == 0) return 0;
   return 128;
+}
+
+// Value columns the kernels weigh for cached rows of `rank_pad` columns, the first
+// `rank` of which are values: as many, or 64 fewer.
+extern "C" int lsd_latent_value_cols(int rank_pad, int rank) {
+  return rank <= rank_pad - 64 ? rank_pad - 64 : rank_pad;
 }
 
 extern "C" hipError_t lsd_latent_prefill(const LatentAttnParams* p, hipStream_t st) {
   const dim3 grid(p->n_tiles);
   if (p->n_tiles == 0) return hipSuccess;
-#define LSD_LP(R, QT, NW, KT)                                                                            \
-  case R: hipLaunchKernelGGL((latent_prefill_kernel<R, QT, NW, KT>), grid, dim3(NW * 64), 0, st, *p); break;
+#define LSD_LP_V(R, V, QT, NW, KT) \
+  hipLaunchKernelGGL((latent_prefill_kernel<R, V, QT, NW, KT>), grid, dim3(NW * 64), 0, st, *p)
+#define LSD_LP(R, QT, NW, KT)                                                \
+  case R:                                                                    \
+    if (p->v_pad == R) LSD_LP_V(R, R, QT, NW, KT);                           \
+    else LSD_LP_V(R, (R > 64 ? R - 64 : R), QT, NW, KT);                     \
+    break;
+  if (p->v_pad != p->rank_pad && (p->rank_pad == 64 || p->v_pad != p->rank_pad - 64)) return hipErrorInvalidValue;
   switch (p->rank_pad) {
     LSD_LP(64, 2, 4, 64)
     LSD_LP(128, 2, 4, 64)
@@ -664,8 +690,10 @@ extern "C" hipError_t lsd_latent_prefill(const LatentAttnParams* p, hipStream_t 
     LSD_LP(384, 1, 8, 32)
     LSD_LP(448, 1, 8, 32)
     LSD_LP(512, 1, 8, 32)
+    LSD_LP(576, 1, 8, 32)
     default: return hipErrorInvalidValue;
   }
+#undef LSD_LP_V
 #undef LSD_LP
   return hipGetLastError();
 }
@@ -673,8 +701,13 @@ extern "C" hipError_t lsd_latent_prefill(const LatentAttnParams* p, hipStream_t 
 extern "C" hipError_t lsd_latent_decode(const LatentAttnParams* p, hipStream_t st) {
   if (p->B == 0) return hipSuccess;
   const dim3 grid(p->B * ((p->H + 15) / 16), p->splits);
-#define LSD_LD(R) \
-  case R: hipLaunchKernelGGL((latent_decode_kernel<R>), grid, dim3(256), 0, st, *p); break;
+#define LSD_LD_V(R, V) hipLaunchKernelGGL((latent_decode_kernel<R, V>), grid, dim3(256), 0, st, *p)
+#define LSD_LD(R)                                         \
+  case R:                                                 \
+    if (p->v_pad == R) LSD_LD_V(R, R);                    \
+    else LSD_LD_V(R, (R > 64 ? R - 64 : R));              \
+    break;
+  if (p->v_pad != p->rank_pad && (p->rank_pad == 64 || p->v_pad != p->rank_pad - 64)) return hipErrorInvalidValue;
   switch (p->rank_pad) {
     LSD_LD(64)
     LSD_LD(128)
@@ -684,12 +717,14 @@ extern "C" hipError_t lsd_latent_decode(const LatentAttnParams* p, hipStream_t s
     LSD_LD(384)
     LSD_LD(448)
     LSD_LD(512)
+    LSD_LD(576)
     default: return hipErrorInvalidValue;
   }
+#undef LSD_LD_V
 #undef LSD_LD
   if (p->splits > 1)
     hipLaunchKernelGGL(latent_combine_kernel, dim3(p->B * p->H), dim3(256), 0, st, p->part_o, p->part_ml,
-                       static_cast<bf16*>(p->out), p->rank_pad, p->splits);
+                       static_cast<bf16*>(p->out), p->v_pad, p->splits);
   return hipGetLastError();
 }
 
@@ -700,7 +735,7 @@ extern "C" hipError_t lsd_latent_plain(const LatentAttnParams* p, int f32, hipSt
   const dim3 grid(p->B, p->H);
   const size_t lds = (p->rank_pad + 256) * sizeof(float);
 #define LSD_PL(T, OPT) hipLaunchKernelGGL((latent_plain_kernel<T, OPT>), grid, dim3(256), lds, st, *p)
-  const int opt = (p->rank_pad + 255) / 256;
+  const int opt = (p->v_pad + 255) / 256;
   if (f32) {
     if (opt <= 1) LSD_PL(float, 1);
     else if (opt <= 4) LSD_PL(float, 4);
@@ -730,6 +765,8 @@ extern "C" hipError_t lsd_latent_expanded(const LatentExpandedParams* p, hipStre
   else if (p->dim == 64 && p->vdim <= 128) LSD_LE(64, 128);
   else if (p->dim == 128 && p->vdim <= 64) LSD_LE(128, 64);
   else if (p->dim == 128 && p->vdim <= 128) LSD_LE(128, 128);
+  else if (p->dim == 192 && p->vdim <= 64) LSD_LE(192, 64);
+  else if (p->dim == 192 && p->vdim <= 128) LSD_LE(192, 128);
   else return hipErrorInvalidValue;
 #undef LSD_LE
   return hipGetLastError();

@@ -112,16 +112,20 @@ __device__ __forceinline__ long a_row(const GgParams& p, const Tile& t, int i) {
   return r;
 }
 
-// g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + 1)
-__device__ __forceinline__ float glu_fast(float g, float u, float limit, float alpha) {
+// g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + one).  SiLU
+// gates have limit = infinity, alpha = 1 and one = 0.
+__device__ __forceinline__ float glu_fast(float g, float u, float limit, float alpha, float one) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * alpha * g)) * (u + 1.f);
+  return g * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * alpha * g)) * (u + one);
 }
-__device__ __forceinline__ float glu_exact(float g, float u, float limit, float alpha) {
+__device__ __forceinline__ float glu_exact(float g, float u, float limit, float alpha, float one) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.f + expf(-alpha * g)) * (u + 1.f);
+  return g / (1.f + expf(-alpha * g)) * (u + one);
+}
+__device__ __forceinline__ float sigmoid_fast(float z) {
+  return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
 }
 }  // namespace gg
 
@@ -183,6 +187,8 @@ __global__ __launch_bounds__(256) void group_gemm_kernel(GgParams p) {
         const int ent = p.perm[m];
         wt = p.wts[ent];
         row = (ent % p.top) * p.T + ent / p.top;  // < top * T, checked on the host to fit
+      } else if (p.wts_s) {
+        wt = p.wts_s[m];
       }
       s_row[threadIdx.x] = row;
       s_wt[threadIdx.x] = wt;
@@ -246,7 +252,7 @@ __global__ __launch_bounds__(256) void group_gemm_kernel(GgParams p) {
       if ((ch & 3) >= 2) continue;
       bf16x8 o;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] = f2bf(glu_fast(src[e], src[16 + e], t.limit, p.alpha));
+      for (int e = 0; e < 8; ++e) o[e] = f2bf(glu_fast(src[e], src[16 + e], t.limit, p.alpha, p.up_one));
       st8(static_cast<bf16*>(t.out) + (long)m * t.ldo + (n >> 5) * 16 + (n & 15), o);
     } else if constexpr (MODE == GG_DOWN) {
       const long orow = s_row[row];
@@ -263,8 +269,15 @@ __global__ __launch_bounds__(256) void group_gemm_kernel(GgParams p) {
       }
     } else {
       bf16x8 o;
+      if (p.gate) {
+        const float* gt = p.gate + m * p.ldg + t.group * p.o_gs + n;
+        const f32x4 ga = *reinterpret_cast<const f32x4*>(gt), gb = *reinterpret_cast<const f32x4*>(gt + 4);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] = f2bf(src[e]);
+        for (int e = 0; e < 8; ++e) o[e] = f2bf(src[e] * sigmoid_fast(e < 4 ? ga[e & 3] : gb[e & 3]));
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o[e] = f2bf(src[e]);
+      }
       st8(static_cast<bf16*>(t.out) + (long)m * t.ldo + n, o);
     }
   }
@@ -323,7 +336,7 @@ __global__ __launch_bounds__(256) void group_gemm_f32_kernel(GgParams p) {
         const int n = t.n0 + tx + 16 * j;
         if (n < t.N)
           static_cast<float*>(t.out)[(long)m * t.ldo + (n >> 5) * 16 + (n & 15)] =
-              glu_exact(acc[i][j], acc[i][j + 1], t.limit, p.alpha);
+              glu_exact(acc[i][j], acc[i][j + 1], t.limit, p.alpha, p.up_one);
       }
       continue;
     }
@@ -334,6 +347,8 @@ __global__ __launch_bounds__(256) void group_gemm_f32_kernel(GgParams p) {
         const int ent = p.perm[m];
         wt = p.wts[ent];
         orow = (long)(ent % p.top) * p.T + ent / p.top;
+      } else if (p.wts_s) {
+        wt = p.wts_s[m];
       }
     }
 #pragma unroll
@@ -343,7 +358,10 @@ __global__ __launch_bounds__(256) void group_gemm_f32_kernel(GgParams p) {
       float* o = static_cast<float*>(t.out) + orow * t.ldo + n;
       if constexpr (MODE == GG_DOWN) *o = acc[i][j] * wt;
       else if constexpr (MODE == GG_ADD) *o += acc[i][j];
-      else if constexpr (MODE == GG_F32) *o = acc[i][j] + (p.bias ? p.bias[n] : 0.f);
+      else if constexpr (MODE == GG_F32) {
+        const float gt = p.gate ? 1.f / (1.f + expf(-p.gate[m * p.ldg + t.group * p.o_gs + n])) : 1.f;
+        *o = (acc[i][j] + (p.bias ? p.bias[n] : 0.f)) * gt;
+      }
       else *o = acc[i][j];
     }
   }
@@ -401,7 +419,7 @@ __global__ __launch_bounds__(256) void moe_gemv_up_kernel(MoeGemvParams p) {
   for (int j = 0; j < 2 * C; ++j) acc[j] = wave_sum(acc[j]);
 #pragma unroll
   for (int j = 0; j < C; ++j)
-    if (lane == j && c0 + j < F) out[c0 + j] = f2bf(gg::glu_fast(acc[2 * j], acc[2 * j + 1], limit, p.alpha));
+    if (lane == j && c0 + j < F) out[c0 + j] = f2bf(gg::glu_fast(acc[2 * j], acc[2 * j + 1], limit, p.alpha, p.up_one));
 }
 
 // One wave: one column of one token's residual += all its experts.
@@ -411,7 +429,7 @@ __global__ __launch_bounds__(256) void moe_gemv_down_kernel(MoeGemvParams p) {
   if (n >= p.K) return;  // K: the residual's width here
   const int ck = (p.F + 511) / 512, cs = (p.Fs + 511) / 512;
   float* x = p.x + (long)t * p.K + n;
-  const float x0 = *x;
+  const float x0 = p.add ? *x : 0.f;
   float acc = 0.f;
   const int items = p.top * ck;
 #pragma unroll 8
@@ -428,7 +446,7 @@ __global__ __launch_bounds__(256) void moe_gemv_down_kernel(MoeGemvParams p) {
     const int c = i * 512 + lane * 8, cc = min(c, p.Fs - 8);
     const bf16x8 a = ld8(static_cast<const bf16*>(p.mids) + (long)t * p.Fs + cc);
     const bf16x8 v = ld8(static_cast<const bf16*>(p.ws) + (long)n * p.Fs + cc);
-    const float d = dot8(a, v, 0.f);
+    const float d = dot8(a, v, 0.f) * (p.wts_s ? p.wts_s[t] : 1.f);
     acc += c < p.Fs ? d : 0.f;
   }
   acc = wave_sum(acc);

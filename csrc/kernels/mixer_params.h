@@ -47,10 +47,30 @@ struct RecurParams {
   int write_ring;                      // single-token portions: this kernel keeps the ring
 };
 
+// Recurrence whose forget gate f also decides what is written:
+//   S <- diag(f) S + (1 - f) v^T;  o = S^T q;  out = rms(o) norm
+// with q = silu, f = l + (1 - l) sigmoid(z + bias) of the in-projection's columns
+// q [heads D] | z [heads D] | v [heads V].
+struct ForgetParams {
+  const void* y; long ldy;
+  SeqParams s;
+  int heads, D, V, Vp;                 // Vp: V padded to 4 (row pitch of S)
+  float* S;                            // [slots][heads][D][Vp]
+  const float* bias; const float* lower;  // [heads D]
+  const float* norm; float eps;        // [V]
+  float* raw; long ldr;                // outputs before the norm [rows][heads V], or null
+  void* out; long ldo; int out_cols;   // zeros behind heads V
+  // prompts in `segs` segments of each sequence, run together: what a segment
+  // starts from (the first two, as it is; of later ones without the segments before
+  // them) [seq][head][seg][D][Vp], and the summed log gates of a segment [..][D]
+  int segs;
+  float* part; float* decay;
+};
+
 // Output norms in a launch of their own.
 struct MixOutParams {
   const float* raw; long ldr; int T;
-  int heads, V;                        // delta: per (row, head)
+  int heads, V;                        // delta, forget: per (row, head); low null: no gate
   const void* low; long ldl; int gate_off;
   int inner, groups;                   // Mamba-2: per (row, group), in place
   const float* norm; float eps, gain;
@@ -111,6 +131,38 @@ struct GroupNormParams {
   const void* bias; const void* w_post;      // [H], element type
   const void* w_pre; void* out;              // [H], [rows][H], element type
   const int* rows; int n_rows;               // rows of x that are normed into out (null: all)
+};
+
+// Elementwise norm tanh(alpha x) w + b; w, b [H] in the element type.
+struct TanhNorm {
+  float alpha;
+  const void* w; const void* b;
+};
+
+// Rows of H columns.  With slabs: x += post(sum of slabs), written back.  With out:
+// out = pre(x), or x in the element type (pre.w null).
+struct TanhStepParams {
+  float* x; int T, H;
+  const void* slab; int splits, slab_bf16;   // [splits][T][H] or null
+  TanhNorm post, pre;
+  void* out;                                 // [rows][H] or null
+  const int* rows; int n_rows;               // rows of x that go into out (null: all)
+};
+
+// In front of a mixer: x_new = x + rms(sum of slabs) w_side over `size` columns (no
+// slabs: x stays), h = pre(x), out = h + (h of the token before - h) mix.  last
+// [slots][H] holds the row before a portion.  Rows whose slot is the previous
+// row's and whose position follows continue a portion.
+struct ShiftNormParams {
+  const float* x; float* x_new; int T, H, size;
+  const void* slab; int splits, slab_bf16;
+  const void* w_side; float eps;
+  TanhNorm pre;
+  const void* mix;
+  float* last;
+  const int* tslot; const int* tpos;
+  void* out;
+  const int* tail; int n_tail;               // rows whose h enters `last` (shift_tail)
 };
 
 }  // namespace lsd

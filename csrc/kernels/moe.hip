@@ -1,12 +1,15 @@
 // Expert routing and the per-token work behind a latent-attention layer's
 // input projection.
 //
-//  * latent_post: one block per token over the fp32 projection row
-//    [queries | latent | router]: RMS norm of the latent and its append to the
-//    paged cache, bf16 queries for the MFMA projections, router scores
-//    (sigmoid), the `top` experts with the largest corrected score and their
-//    normalised uncorrected scores.  A model whose layers have only some of
-//    the three passes the others as absent.
+//  * latent_post: one block per token over the fp32 projection row: RMS norm of
+//    the latent and its append to the paged cache with the turned key part, bf16
+//    queries for the MFMA projections (turned, or normed where they are a latent of
+//    their own), and the routing where the router reads the same row.  A model
+//    whose layers have only some of these passes the others as absent.
+//  * route: a wave per row of router logits; the `top` experts with the largest
+//    corrected sigmoid score and their normalised uncorrected scores, or with the
+//    largest logits and their softmax.
+//  * side_mul: gated rows times the tokens' own rows of a table.
 //  * moe_group: sorts the (token, choice) entries by expert and cuts every
 //    expert's rows into tiles for the grouped GEMMs (group_gemm.hip) -- all on
 //    the device, so a captured decode graph follows the routing of each replay.
@@ -25,25 +28,127 @@ __device__ __forceinline__ float narrow<float>(float v) { return v; }
 constexpr int LATENT_PAGE = 64;  // tokens per cache page
 constexpr int MAX_EXPERTS = 1024;
 
-template <typename T, int EPL>  // EPL: experts per lane
-__global__ __launch_bounds__(256) void latent_post_kernel(LatentPostParams p) {
-  // the three parts are independent: wave 0 routes, wave 1 appends, waves 2
-  // and 3 narrow (no block barrier)
-  const int lane = lane_id(), w = threadIdx.x >> 6, t = blockIdx.x;
-  const float* y = p.y + (long)t * p.ldy;
-  if (p.q != nullptr && w >= 2) {
-    T* q = static_cast<T*>(p.q) + (long)t * p.nq;
-    const int id = threadIdx.x - 128;
-    if constexpr (sizeof(T) == 2) {
-      for (int c = id * 4; c < p.nq; c += 512) {
-        const f32x4 v = *reinterpret_cast<const f32x4*>(y + c);
-        st4(reinterpret_cast<bf16*>(q) + c, bf16x4{f2bf(v[0]), f2bf(v[1]), f2bf(v[2]), f2bf(v[3])});
+// One row's routing by one wave; EPL: experts per lane.
+template <int EPL>
+__device__ __forceinline__ void route_row(const RouteParams& p, const float* z, int t) {
+  const int lane = lane_id();
+  float sc[EPL], ch[EPL];
+#pragma unroll
+  for (int j = 0; j < EPL; ++j) {
+    const int e = lane + 64 * j;
+    const bool ok = e < p.experts;
+    const float v = ok ? z[e] : 0.f;
+    sc[j] = p.correction ? 1.f / (1.f + expf(-v)) : v;
+    ch[j] = !ok ? -INFINITY : p.correction ? sc[j] + p.correction[e] : sc[j];
+  }
+  if (p.shared && lane == 0) p.shared[t] = 1.f / (1.f + expf(-z[p.experts]));
+  float sum = 0.f, mine = 0.f, best = 0.f;
+  for (int k = 0; k < p.top; ++k) {
+    // best corrected score of the wave; the lower expert wins a tie
+    float b = -INFINITY;
+    int be = 0x7fffffff;
+#pragma unroll
+    for (int j = 0; j < EPL; ++j)
+      if (ch[j] > b) {
+        b = ch[j];
+        be = lane + 64 * j;
       }
-    } else {
-      for (int c = id; c < p.nq; c += 128) q[c] = narrow<T>(y[c]);
+#pragma unroll
+    for (int m = 32; m >= 1; m >>= 1) {
+      const float ob = __shfl_xor(b, m, 64);
+      const int oe = __shfl_xor(be, m, 64);
+      if (ob > b || (ob == b && oe < be)) {
+        b = ob;
+        be = oe;
+      }
+    }
+    // scores that are not numbers never win: keep the ids in range
+    if (be >= p.experts) be = k;
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < EPL; ++j)
+      if (be == lane + 64 * j) {
+        s = sc[j];
+        ch[j] = -INFINITY;
+      }
+    s = __shfl(s, be & 63, 64);
+    if (!p.correction) {  // softmax over the chosen logits, the first the largest
+      if (k == 0) best = s;
+      s = expf(s - best);
+    }
+    sum += s;
+    if (lane == (k & 63)) {
+      if (k >= 64) {  // more choices than lanes: park the earlier ones
+        p.wts[(long)t * p.top + k - 64] = mine;
+      }
+      mine = s;
+      p.ids[(long)t * p.top + k] = be;
     }
   }
-  if (p.cache != nullptr && w == 1) {
+  // divide by the sum: lane l holds choice k = l (+ 64 when top > 64)
+  const float inv = 1.f / (sum + 1e-20f);
+  for (int k = lane; k < p.top; k += 64) {
+    const bool held = k + 64 >= p.top;
+    p.wts[(long)t * p.top + k] = (held ? mine : p.wts[(long)t * p.top + k]) * inv;
+  }
+}
+
+// One wave per row of router logits that stand alone
+template <int EPL>
+__global__ __launch_bounds__(256) void route_kernel(RouteParams p) {
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (t < p.T) route_row<EPL>(p, p.z + (long)t * p.ldz, t);
+}
+
+// Column c of a head turned: pairs (rot + i, rot + i + half)
+__device__ __forceinline__ float turned(const float* head, int c, int rot, int half, const float* cs) {
+  const int j = c - rot;
+  const float v = head[c];
+  if (j < 0 || j >= 2 * half) return v;
+  const int i = j < half ? j : j - half;
+  const float co = cs[2 * i], si = cs[2 * i + 1];
+  return j < half ? v * co - head[c + half] * si : v * co + head[c - half] * si;
+}
+
+template <typename T, int EPL>  // EPL: experts per lane
+__global__ __launch_bounds__(256) void latent_post_kernel(LatentPostParams p) {
+  // the parts are independent (no block barrier): wave 0 routes, wave 1 appends, and
+  // those that have neither, at least the last two, see to the queries
+  const int lane = lane_id(), w = threadIdx.x >> 6, t = blockIdx.x;
+  const float* y = p.y + (long)t * p.ldy;
+  const float* cs = p.half ? p.rope + (long)p.tpos[t] * 2 * p.half : nullptr;
+  const int w0 = p.r.experts > 0 ? 2 : p.cache != nullptr ? 1 : 0;  // first wave that may be free
+  const bool appends = p.cache != nullptr && w == (w0 == 1 ? 0 : 1);
+  if (p.q != nullptr && w >= w0) {
+    T* q = static_cast<T*>(p.q) + (long)t * p.nq;
+    const int id = threadIdx.x - 64 * w0, step = 256 - 64 * w0;
+    if (p.q_gain) {
+      if (w == 3) {
+        float s = 0.f;
+#pragma unroll 8
+        for (int i = lane; i < p.q_rank; i += 64) s += y[i] * y[i];
+        const float rstd = 1.f / sqrtf(wave_sum(s) / p.q_rank + p.eps);
+#pragma unroll 8
+        for (int i = lane; i < p.nq; i += 64) q[i] = narrow<T>(i < p.q_rank ? y[i] * rstd * p.q_gain[i] : 0.f);
+      }
+    } else if constexpr (sizeof(T) == 2) {
+      for (int c = id * 4; c < p.nq; c += step * 4) {
+        f32x4 v = *reinterpret_cast<const f32x4*>(y + c);
+        if (p.half) {  // heads are a multiple of four columns wide
+          const int at = c % p.q_head;
+          if (at + 3 >= p.q_rot && at < p.q_rot + 2 * p.half) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = turned(y + c - at, at + e, p.q_rot, p.half, cs);
+          }
+        }
+        st4(reinterpret_cast<bf16*>(q) + c, pack4(v));
+      }
+    } else {
+      for (int c = id; c < p.nq; c += step)
+        q[c] = narrow<T>(p.half ? turned(y + c - c % p.q_head, c % p.q_head, p.q_rot, p.half, cs) : y[c]);
+    }
+  }
+  if (appends) {
     const float* c = y + p.c_off;
     const int pos = p.tpos[t];
     const int page = p.table[(long)p.tslot[t] * p.tw + pos / LATENT_PAGE];
@@ -54,64 +159,13 @@ __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostParams p) {
     const float rstd = 1.f / sqrtf(s / p.rank + p.eps);
     T* o = static_cast<T*>(p.cache) + ((long)page * LATENT_PAGE + pos % LATENT_PAGE) * p.rank_pad;
 #pragma unroll 8
-    for (int i = lane; i < p.rank_pad; i += 64) o[i] = narrow<T>(i < p.rank ? c[i] * rstd * p.gain[i] : 0.f);
-  }
-  if (p.experts > 0 && w == 0) {
-    const float* z = y + p.r_off;
-    float sc[EPL], ch[EPL];
-#pragma unroll
-    for (int j = 0; j < EPL; ++j) {
-      const int e = lane + 64 * j;
-      const bool ok = e < p.experts;
-      sc[j] = ok ? 1.f / (1.f + expf(-z[e])) : 0.f;
-      ch[j] = ok ? sc[j] + p.correction[e] : -INFINITY;
-    }
-    float sum = 0.f, mine = 0.f;
-    for (int k = 0; k < p.top; ++k) {
-      // best corrected score of the wave; the lower expert wins a tie
-      float b = -INFINITY;
-      int be = 0x7fffffff;
-#pragma unroll
-      for (int j = 0; j < EPL; ++j)
-        if (ch[j] > b) {
-          b = ch[j];
-          be = lane + 64 * j;
-        }
-#pragma unroll
-      for (int m = 32; m >= 1; m >>= 1) {
-        const float ob = __shfl_xor(b, m, 64);
-        const int oe = __shfl_xor(be, m, 64);
-        if (ob > b || (ob == b && oe < be)) {
-          b = ob;
-          be = oe;
-        }
-      }
-      // scores that are not numbers never win: keep the ids in range
-      if (be >= p.experts) be = k;
-      float s = 0.f;
-#pragma unroll
-      for (int j = 0; j < EPL; ++j)
-        if (be == lane + 64 * j) {
-          s = sc[j];
-          ch[j] = -INFINITY;
-        }
-      s = __shfl(s, be & 63, 64);
-      sum += s;
-      if (lane == (k & 63)) {
-        if (k >= 64) {  // more choices than lanes: park the earlier ones
-          p.wts[(long)t * p.top + k - 64] = mine;
-        }
-        mine = s;
-        p.ids[(long)t * p.top + k] = be;
-      }
-    }
-    // divide by the sum: lane l holds choice k = l (+ 64 when top > 64)
-    const float inv = 1.f / (sum + 1e-20f);
-    for (int k = lane; k < p.top; k += 64) {
-      const bool held = k + 64 >= p.top;
-      p.wts[(long)t * p.top + k] = (held ? mine : p.wts[(long)t * p.top + k]) * inv;
+    for (int i = lane; i < p.rank_pad; i += 64) {
+      float v = i < p.rank ? c[i] * rstd * p.gain[i] : 0.f;
+      if (i >= p.rank && i < p.rank + 2 * p.half) v = turned(c, i, p.rank, p.half, cs);
+      o[i] = narrow<T>(v);
     }
   }
+  if (p.r.experts > 0 && w == 0) route_row<EPL>(p.r, y + p.r_off, t);
 }
 
 // One block.  ids [n] -> perm [n] (entries sorted by expert), tiles
@@ -196,6 +250,30 @@ __global__ __launch_bounds__(256) void embed_f32_kernel(const int* __restrict__ 
   for (int c = threadIdx.x; c < H; c += 256) out[(long)blockIdx.x * H + c] = wte[(long)id * H + c] * scale;
 }
 
+// out[t] = g[t] * table[ids[t]], rows of n columns (fp32: gelu(g[t]) * table[ids[t]])
+template <typename T>
+__global__ __launch_bounds__(256) void side_mul_kernel(const T* g, const int* __restrict__ ids,
+                                                       const T* __restrict__ table, T* out, long items, int n, int vocab) {
+  const long at = (long)blockIdx.x * 256 + threadIdx.x;
+  if (at >= items) return;
+  const long row = at / (n / 4);
+  const int c = (int)(at % (n / 4)) * 4;
+  int id = ids[row];
+  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  if constexpr (sizeof(T) == 2) {
+    const bf16x4 a = ld4(g + row * n + c), e = ld4(table + (long)id * n + c);
+    st4(out + row * n + c, pack4(f32x4{bf2f(a[0]) * bf2f(e[0]), bf2f(a[1]) * bf2f(e[1]), bf2f(a[2]) * bf2f(e[2]),
+                                       bf2f(a[3]) * bf2f(e[3])}));
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float z = g[row * n + c + i];
+      out[row * n + c + i] =
+          0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))) * table[(long)id * n + c + i];
+    }
+  }
+}
+
 }  // namespace lsd
 
 using namespace lsd;
@@ -203,7 +281,7 @@ using namespace lsd;
 template <typename T>
 static hipError_t post(const LatentPostParams& p, hipStream_t st) {
   const dim3 grid(p.T), blk(256);
-  const int epl = (p.experts + 63) / 64;
+  const int epl = (p.r.experts + 63) / 64;
   if (epl <= 1) hipLaunchKernelGGL((latent_post_kernel<T, 1>), grid, blk, 0, st, p);
   else if (epl <= 4) hipLaunchKernelGGL((latent_post_kernel<T, 4>), grid, blk, 0, st, p);
   else if (epl <= 16) hipLaunchKernelGGL((latent_post_kernel<T, 16>), grid, blk, 0, st, p);
@@ -213,8 +291,34 @@ static hipError_t post(const LatentPostParams& p, hipStream_t st) {
 
 extern "C" hipError_t lsd_latent_post(const LatentPostParams* p, int f32, hipStream_t st) {
   if (p->T == 0) return hipSuccess;
-  if (p->top > 128 || p->top > p->experts) return hipErrorInvalidValue;
+  if (p->r.top > 128 || p->r.top > p->r.experts) return hipErrorInvalidValue;
   return f32 ? post<float>(*p, st) : post<bf16>(*p, st);
+}
+
+extern "C" hipError_t lsd_route(const RouteParams* p, hipStream_t st) {
+  if (p->T == 0) return hipSuccess;
+  if (p->top > 128 || p->top > p->experts) return hipErrorInvalidValue;
+  const dim3 grid((p->T + 3) / 4), blk(256);
+  const int epl = (p->experts + 63) / 64;
+  if (epl <= 1) hipLaunchKernelGGL((route_kernel<1>), grid, blk, 0, st, *p);
+  else if (epl <= 4) hipLaunchKernelGGL((route_kernel<4>), grid, blk, 0, st, *p);
+  else if (epl <= 16) hipLaunchKernelGGL((route_kernel<16>), grid, blk, 0, st, *p);
+  else return hipErrorInvalidValue;
+  return hipGetLastError();
+}
+
+extern "C" hipError_t lsd_side_mul(const void* g, const int* ids, const void* table, void* out, int T, int n, int vocab,
+                                   int f32, hipStream_t st) {
+  if (T == 0) return hipSuccess;
+  const long items = (long)T * n / 4;
+  const dim3 grid((unsigned)((items + 255) / 256));
+  if (f32)
+    hipLaunchKernelGGL((side_mul_kernel<float>), grid, dim3(256), 0, st, static_cast<const float*>(g), ids,
+                       static_cast<const float*>(table), static_cast<float*>(out), items, n, vocab);
+  else
+    hipLaunchKernelGGL((side_mul_kernel<bf16>), grid, dim3(256), 0, st, static_cast<const bf16*>(g), ids,
+                       static_cast<const bf16*>(table), static_cast<bf16*>(out), items, n, vocab);
+  return hipGetLastError();
 }
 
 extern "C" hipError_t lsd_moe_group(const int* ids, int n, int E, int tm, int* perm, int* tiles, int n_tiles,

@@ -25,7 +25,7 @@ struct GgParams {
   // 0), the sorted (token, choice) entries and their weights
   const int* tiles; int n_tiles;
   const int* perm; const float* wts; int top, T;
-  float limit, alpha;             // clamp and sigmoid slope of the gated activation
+  float limit, alpha, up_one;     // g sigmoid(alpha g) (u + up_one), g and u clamped at limit
   int slab_bf16;                  // GG_DOWN output dtype (0: fp32)
   // shared expert: one more group over every token (Ns == 0: none)
   const void* As; long ldas;
@@ -33,6 +33,8 @@ struct GgParams {
   int Ns, Ks;
   void* outs; long ldos;
   float limit_s;
+  const float* wts_s;             // GG_DOWN: its weight per token, or null (1)
+  const float* gate; long ldg;    // GG_BATCH / GG_F32: out *= sigmoid(gate[m][o_gs g + n]), or null
   int gr, gr_s;                   // row tiles per group of the tile order (experts, shared)
 };
 
@@ -44,32 +46,50 @@ struct MoeGemvParams {
   const void* w;             // up [E][2F][K] interleaved, down [E][K][F]
   const void* ws;            // up [2Fs][K], down [K][Fs]
   void* mid; void* mids;     // [T top][F], [T][Fs]
-  float limit, limit_s, alpha;
-  float* x;                  // down: fp32 residual [T][K], added to
+  float limit, limit_s, alpha, up_one;
+  const float* wts_s;        // down: weight of the shared expert per token, or null (1)
+  float* x; int add;         // down: fp32 rows [T][K], added to or written
+};
+
+// A router's logits of one row and what becomes of them: the `top` experts with
+// the largest corrected sigmoid scores and their normalised scores, or (no
+// correction) with the largest logits and the softmax over these.
+struct RouteParams {
+  const float* z; long ldz;                         // logits [T][experts]
+  int T, experts, top;
+  const float* correction;                          // [experts] or null
+  int* ids; float* wts;                             // [T][top]
+  float* shared;                                    // [T] sigmoid of the column behind the logits, or null
 };
 
 // One token row behind a layer's input projection y (fp32): the latent columns
-// are normed and appended to the paged cache, the query columns narrowed, the
-// router columns scored and the experts chosen.
+// are normed and appended to the paged cache with the turned key part behind them,
+// the query columns narrowed and their last `rot` columns per head turned -- or
+// normed, where they are a latent of their own -- and the experts chosen.
 struct LatentPostParams {
   const float* y; long ldy; int T;
   void* q; int nq;                                  // null: queries stay in y
+  const float* q_gain; int q_rank;                  // not null: q = norm of the first q_rank of nq columns
+  int q_head, q_rot;                                // columns per head and the first turned one
+  const float* rope; int half;                      // [positions][half][2] cos, sin; pairs (i, i + half); half 0: none
   void* cache; int c_off, rank, rank_pad;           // null cache: another layer's latent is used
   const float* gain; float eps;
   const int* table; int tw; const int* tslot; const int* tpos;
-  int r_off, experts, top;                          // experts == 0: no router
-  const float* correction; int* ids; float* wts;
+  int r_off;                                        // first router column (r.experts == 0: no router)
+  RouteParams r;
 };
 
 // Attention over the paged latent cache, in the latent space: query row
-// (t, head) of `rank_pad` columns, keys and values both the cached latents.
+// (t, head) of `rank_pad` columns, keys the cached rows, values their first
+// `v_pad` columns.
 struct LatentAttnParams {
-  const void* q; void* out;                         // [T][H][rank_pad]
+  const void* q; void* out;                         // [T][H][rank_pad], [T][H][v_pad]
   const void* cache; const int* table; int tw;      // [pages][64][rank_pad], [slots][tw]
   const int* seq_slots; const int* pos;             // decode: [B] positions; prefill: q_start
   const int* cu_q; const int* tiles; int n_tiles;   // prefill tiles (sequence, first row)
-  int B, H, rank_pad, window;                       // window: keys per query (INT_MAX: all)
+  int B, H, rank_pad, v_pad, window;                // window: keys per query (INT_MAX: all)
   float scale_log2;
+  const float* sink;                                // [H] a further score without a value, or null
   float* part_o; float* part_ml; int splits;        // decode, splits > 1
 };
 
@@ -82,6 +102,8 @@ struct LatentExpandedParams {
   const int* cu_q; const int* q_start; const int* k_lo; const int* cu_k;
   int H, dim, vdim, window;
   float scale_log2;
+  const float* sink;                                // [H] or null
+  const float* gate; long ldg;                      // out *= sigmoid(gate[T][H vdim]), or null
 };
 
 }  // namespace lsd

@@ -18,6 +18,7 @@ using lsd::GgParams;
 using lsd::LatentAttnParams;
 using lsd::LatentPostParams;
 using lsd::MoeGemvParams;
+using lsd::RouteParams;
 
 extern "C" {
 hipError_t lsd_group_gemm(const GgParams* p, int mode, int tm, hipStream_t st);
@@ -25,6 +26,10 @@ hipError_t lsd_group_gemm_f32(const GgParams* p, int mode, hipStream_t st);
 hipError_t lsd_moe_gemv_up(const MoeGemvParams* p, hipStream_t st);
 hipError_t lsd_moe_gemv_down(const MoeGemvParams* p, hipStream_t st);
 hipError_t lsd_latent_post(const LatentPostParams* p, int f32, hipStream_t st);
+hipError_t lsd_route(const RouteParams* p, hipStream_t st);
+hipError_t lsd_side_mul(const void* g, const int* ids, const void* table, void* out, int T, int n, int vocab, int f32,
+                        hipStream_t st);
+int lsd_latent_value_cols(int rank_pad, int rank);
 hipError_t lsd_moe_group(const int* ids, int n, int E, int tm, int* perm, int* tiles, int n_tiles, hipStream_t st);
 hipError_t lsd_norm_f32(float* x, const float* slab, int splits, const float* w, float* out, int T, int H, float eps,
                         const int* rows, int nrows, int Hn, float woff, hipStream_t st);
@@ -89,9 +94,30 @@ int tile_rows(int64_t tm, bool f32) {
   return (int)tm;
 }
 
-// Per-group projection: out[m][g N + n] = a[m][g K : g K + K] . w[g][n].
-// a [M, groups K], w [groups, N, K]; bf16 -> bf16, fp32 -> fp32.
-torch::Tensor batch_linear(torch::Tensor a, torch::Tensor w, int64_t tm) {
+// fp32 gate logits [M, N] (rows of a wider tensor)
+const float* gate_rows(const torch::Tensor& t, int64_t M, int64_t N, long& ld) {
+  need(t, torch::kFloat32, "gate");
+  TORCH_CHECK(t.dim() == 2 && t.size(0) == M && t.size(1) == N && t.stride(1) == 1 && (M <= 1 || t.stride(0) % 4 == 0) &&
+                  reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0, "gate must be [", M, ", ", N, "] 16-byte rows");
+  ld = t.stride(0);
+  return t.data_ptr<float>();
+}
+
+// per-head scores of the softmax without values
+const float* sink_of(const Opt& sink, int64_t H) {
+  if (!sink.has_value()) return nullptr;
+  need(*sink, torch::kFloat32, "sink");
+  TORCH_CHECK(sink->is_contiguous() && sink->numel() == H, "sink must be [heads]");
+  return sink->data_ptr<float>();
+}
+
+// Clamped gates have a limit; SiLU ones (limit 0) none.
+float glu_limit(double limit) { return limit > 0 ? (float)limit : INFINITY; }
+
+// Per-group projection: out[m][g N + n] = a[m][g K : g K + K] . w[g][n], times the
+// sigmoid of gate [M, groups N].  a [M, groups K], w [groups, N, K]; bf16 -> bf16,
+// fp32 -> fp32.
+torch::Tensor batch_linear(torch::Tensor a, torch::Tensor w, int64_t tm, Opt gate) {
   const bool f32 = is_f32(a, "a");
   need(w, a.scalar_type(), "w");
   need_rows(a, "a");
@@ -104,6 +130,7 @@ torch::Tensor batch_linear(torch::Tensor a, torch::Tensor w, int64_t tm) {
   p.W = w.data_ptr(); p.ldw = K; p.w_gs = N * K;
   p.N = N; p.K = K; p.M = a.size(0); p.groups = G;
   p.out = out.data_ptr(); p.ldo = G * N; p.o_gs = N;
+  if (gate.has_value()) p.gate = gate_rows(*gate, p.M, G * N, p.ldg);
   if (p.M) run(p, f32 ? lsd::GG_F32 : lsd::GG_BATCH, tile_rows(tm, f32), f32, "batch_linear");
   return out;
 }
@@ -176,7 +203,7 @@ std::vector<torch::Tensor> moe_up(torch::Tensor h, torch::Tensor perm, torch::Te
   p.perm = iptr(perm, n, "perm");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 4, "tiles must be [n, 4]");
   p.tiles = iptr(tiles, 0, "tiles"); p.n_tiles = tiles.size(0);
-  p.limit = limit; p.alpha = alpha;
+  p.limit = glu_limit(limit); p.alpha = limit > 0 ? alpha : 1.f; p.up_one = limit > 0 ? 1.f : 0.f;
   auto mid = torch::empty({n, w.size(1) / 2}, h.options());
   p.out = mid.data_ptr(); p.ldo = mid.size(1);
   torch::Tensor mids;
@@ -185,7 +212,8 @@ std::vector<torch::Tensor> moe_up(torch::Tensor h, torch::Tensor perm, torch::Te
     TORCH_CHECK(ws->size(1) == K && ws->size(0) % 32 == 0, "moe_up: ws must be [2Fs, K], Fs % 16 == 0");
     mids = torch::empty({T, ws->size(0) / 2}, h.options());
     p.As = p.A; p.ldas = p.lda; p.Ws = ws->data_ptr(); p.ldws = K;
-    p.Ns = ws->size(0); p.Ks = K; p.outs = mids.data_ptr(); p.ldos = mids.size(1); p.limit_s = limit_s;
+    p.Ns = ws->size(0); p.Ks = K; p.outs = mids.data_ptr(); p.ldos = mids.size(1); p.limit_s = glu_limit(limit_s);
+    TORCH_CHECK((limit > 0) == (limit_s > 0), "moe_up: experts and shared expert have gates of one kind");
   } else {
     mids = torch::empty({0}, h.options());
   }
@@ -193,10 +221,16 @@ std::vector<torch::Tensor> moe_up(torch::Tensor h, torch::Tensor perm, torch::Te
   return {mid, mids};
 }
 
+const float* token_weights(const torch::Tensor& t, int64_t T) {
+  need(t, torch::kFloat32, "wts_s");
+  TORCH_CHECK(t.is_contiguous() && t.numel() == T, "wts_s must be [T]");
+  return t.data_ptr<float>();
+}
+
 // Down projections: slab[k][t] = wts[t][k] * (expert k of token t), and
-// slab[top][t] the shared expert's.  slab [>= top (+ 1), T, N], bf16 or fp32.
+// slab[top][t] the shared expert's (times wts_s[t]).  slab [>= top (+ 1), T, N], bf16 or fp32.
 void moe_down(torch::Tensor mid, Opt mids, torch::Tensor perm, torch::Tensor tiles, torch::Tensor wts,
-              torch::Tensor w, Opt ws, torch::Tensor slab, int64_t tm) {
+              torch::Tensor w, Opt ws, torch::Tensor slab, int64_t tm, Opt wts_s) {
   const bool f32 = is_f32(mid, "mid");
   need_rows(mid, "mid");
   expert_weight(w, mid.scalar_type(), 3, "w");
@@ -229,14 +263,15 @@ void moe_down(torch::Tensor mid, Opt mids, torch::Tensor perm, torch::Tensor til
     p.As = mids->data_ptr(); p.ldas = mids->size(1);
     p.Ws = ws->data_ptr(); p.ldws = ws->size(1); p.Ns = N; p.Ks = ws->size(1);
     p.outs = static_cast<char*>(slab.data_ptr()) + top * T * N * slab.element_size(); p.ldos = N;
+    if (wts_s.has_value()) p.wts_s = token_weights(*wts_s, T);
   }
   if (T) run(p, lsd::GG_DOWN, tile_rows(tm, f32), f32, "moe_down");
 }
 
-// x += the experts of a few tokens, weights streamed per (token, choice):
+// x += (add) or = the experts of a few tokens, weights streamed per (token, choice):
 // h [T, K] bf16, w_up [E, 2F, K], w_down [E, K, F] (+ shared), x [T, K] fp32.
 void moe_few(torch::Tensor h, torch::Tensor ids, torch::Tensor wts, torch::Tensor w_up, torch::Tensor w_down,
-             double limit, double alpha, Opt ws_up, Opt ws_down, double limit_s, torch::Tensor x) {
+             double limit, double alpha, Opt ws_up, Opt ws_down, double limit_s, torch::Tensor x, Opt wts_s, bool add) {
   need(h, torch::kBFloat16, "h");
   TORCH_CHECK(h.dim() == 2 && h.is_contiguous(), "h must be contiguous [T, K]");
   const int64_t T = h.size(0), K = h.size(1), top = ids.size(1);
@@ -266,7 +301,11 @@ void moe_few(torch::Tensor h, torch::Tensor ids, torch::Tensor wts, torch::Tenso
     p.ws = ws_up->data_ptr();
   }
   p.h = h.data_ptr(); p.w = w_up.data_ptr(); p.mid = mid.data_ptr();
-  p.limit = limit; p.limit_s = limit_s; p.alpha = alpha;
+  p.limit = glu_limit(limit); p.limit_s = glu_limit(limit_s);
+  p.alpha = limit > 0 ? alpha : 1.f; p.up_one = limit > 0 ? 1.f : 0.f;
+  TORCH_CHECK(!ws_up.has_value() || (limit > 0) == (limit_s > 0), "moe_few: gates of one kind");
+  if (wts_s.has_value()) p.wts_s = token_weights(*wts_s, T);
+  p.add = add;
   check_hip(lsd_moe_gemv_up(&p, cur_stream()), "moe_few up");
   p.w = w_down.data_ptr();
   if (ws_down.has_value()) p.ws = ws_down->data_ptr();
@@ -281,17 +320,37 @@ void need_cache(const torch::Tensor& cache, const torch::Tensor& table, c10::Sca
   TORCH_CHECK(table.dim() == 2 && table.is_contiguous(), "table must be contiguous [slots, pages per slot]");
 }
 
-// See LatentPostParams: -> (q or empty, expert ids, expert weights)
+// See LatentPostParams: -> (q or empty, expert ids, expert weights).  c_off: first
+// latent column (-1: behind the queries); rope [positions, half, 2] turns columns
+// q_rot .. of every q_head query columns and those behind the latent's rank; q_gain
+// [<= nq]: the first columns are normed into q
 std::vector<torch::Tensor> latent_post(torch::Tensor y, int64_t nq, bool want_q, bool f32, Opt cache, int64_t rank,
                                        Opt gain, double eps, Opt table, Opt tslot, Opt tpos, Opt correction,
-                                       int64_t top) {
+                                       int64_t top, int64_t c_off, Opt rope, int64_t q_head, int64_t q_rot, Opt q_gain) {
   need(y, torch::kFloat32, "y");
   need_rows(y, "y");
   const int64_t T = y.size(0);
   const auto dt = f32 ? torch::kFloat32 : torch::kBFloat16;
   LatentPostParams p{};
   p.y = y.data_ptr<float>(); p.ldy = y.stride(0); p.T = T; p.nq = nq; p.eps = eps;
-  int64_t off = nq;
+  int64_t off = c_off >= 0 ? c_off : nq;
+  TORCH_CHECK(nq <= y.size(1) && off >= nq, "latent_post: queries come first");
+  if (rope.has_value()) {
+    need(*rope, torch::kFloat32, "rope");
+    TORCH_CHECK(rope->dim() == 3 && rope->size(2) == 2 && rope->is_contiguous() && tpos.has_value(), "rope [positions, half, 2]");
+    TORCH_CHECK(!table.has_value() || rope->size(0) >= table->size(1) * (int64_t)PAGE, "rope: too few positions");
+    p.rope = rope->data_ptr<float>(); p.half = rope->size(1);
+    p.tpos = iptr(*tpos, T, "tpos");
+    if (want_q && !q_gain.has_value())
+      TORCH_CHECK(q_head >= 4 && q_head % 4 == 0 && nq % q_head == 0 && q_rot >= 0 && q_rot + 2 * p.half <= q_head,
+                  "latent_post: turned columns of a head");
+    p.q_head = q_head; p.q_rot = q_rot;
+  }
+  if (q_gain.has_value()) {
+    need(*q_gain, torch::kFloat32, "q_gain");
+    TORCH_CHECK(want_q && q_gain->is_contiguous() && q_gain->numel() >= 1 && q_gain->numel() <= nq, "q_gain [<= nq]");
+    p.q_gain = q_gain->data_ptr<float>(); p.q_rank = q_gain->numel();
+  }
   torch::Tensor q = torch::empty({want_q ? T : 0, nq}, y.options().dtype(dt));
   TORCH_CHECK(nq % 4 == 0, "query columns must be a multiple of 4");
   if (want_q) p.q = q.data_ptr();
@@ -299,12 +358,13 @@ std::vector<torch::Tensor> latent_post(torch::Tensor y, int64_t nq, bool want_q,
     TORCH_CHECK(table.has_value() && tslot.has_value() && tpos.has_value() && gain.has_value(), "latent_post: cache");
     need_cache(*cache, *table, dt);
     need(*gain, torch::kFloat32, "gain");
-    TORCH_CHECK(gain->is_contiguous() && gain->numel() == rank && rank >= 1 && rank <= cache->size(2), "gain [rank]");
+    TORCH_CHECK(gain->is_contiguous() && gain->numel() == rank && rank >= 1 && rank + 2 * p.half <= cache->size(2),
+                "gain [rank], and room for the turned part");
     p.cache = cache->data_ptr(); p.c_off = off; p.rank = rank; p.rank_pad = cache->size(2);
     p.gain = gain->data_ptr<float>();
     p.table = table->data_ptr<int>(); p.tw = table->size(1);
     p.tslot = iptr(*tslot, T, "tslot"); p.tpos = iptr(*tpos, T, "tpos");
-    off += rank;
+    off += rank + 2 * p.half;
   }
   const int64_t E = correction.has_value() ? correction->numel() : 0;
   auto ids = torch::empty({T, E ? top : 0}, y.options().dtype(torch::kInt32));
@@ -312,8 +372,8 @@ std::vector<torch::Tensor> latent_post(torch::Tensor y, int64_t nq, bool want_q,
   if (E) {
     need(*correction, torch::kFloat32, "correction");
     TORCH_CHECK(correction->is_contiguous() && top >= 1 && top <= E && top <= 128 && E <= 1024, "router sizes");
-    p.r_off = off; p.experts = E; p.top = top; p.correction = correction->data_ptr<float>();
-    p.ids = ids.data_ptr<int>(); p.wts = wts.data_ptr<float>();
+    p.r_off = off; p.r.experts = E; p.r.top = top; p.r.correction = correction->data_ptr<float>();
+    p.r.ids = ids.data_ptr<int>(); p.r.wts = wts.data_ptr<float>();
     off += E;
   }
   TORCH_CHECK(off <= y.size(1), "latent_post: y has ", y.size(1), " columns, needs ", off);
@@ -321,15 +381,50 @@ std::vector<torch::Tensor> latent_post(torch::Tensor y, int64_t nq, bool want_q,
   return {q, ids, wts};
 }
 
+// z [T, >= experts (+ 1 with a shared gate)] fp32 logits -> (ids [T, top], weights
+// [T, top], [T] weights of the shared expert or empty): softmax over the chosen
+std::vector<torch::Tensor> route_softmax(torch::Tensor z, int64_t experts, int64_t top, bool shared) {
+  need(z, torch::kFloat32, "z");
+  const int64_t T = z.size(0);
+  TORCH_CHECK(z.dim() == 2 && z.stride(1) == 1 && z.size(1) >= experts + (shared ? 1 : 0), "z [T, experts (+ 1)]");
+  TORCH_CHECK(top >= 1 && top <= experts && top <= 128 && experts <= 1024, "router sizes");
+  auto ids = torch::empty({T, top}, z.options().dtype(torch::kInt32));
+  auto wts = torch::empty({T, top}, z.options());
+  auto sh = torch::empty({shared ? T : 0}, z.options());
+  RouteParams p{};
+  p.z = z.data_ptr<float>(); p.ldz = z.stride(0); p.T = T; p.experts = experts; p.top = top;
+  p.ids = ids.data_ptr<int>(); p.wts = wts.data_ptr<float>();
+  if (shared) p.shared = sh.data_ptr<float>();
+  check_hip(lsd_route(&p, cur_stream()), "route");
+  return {ids, wts, sh};
+}
+
+// rows g [T, n] times rows ids of table [vocab, n] (fp32: gelu(g) times them)
+torch::Tensor side_mul(torch::Tensor g, torch::Tensor ids, torch::Tensor table) {
+  const bool f32 = is_f32(g, "g");
+  need(table, g.scalar_type(), "table");
+  const int64_t T = g.size(0), n = g.size(1);
+  TORCH_CHECK(g.dim() == 2 && g.is_contiguous() && table.dim() == 2 && table.is_contiguous() && table.size(1) == n &&
+                  n % 4 == 0, "side_mul: g [T, n], table [vocab, n], n % 4");
+  auto out = torch::empty_like(g);
+  check_hip(lsd_side_mul(g.data_ptr(), iptr(ids, T, "ids"), table.data_ptr(), out.data_ptr(), T, n, table.size(0), f32,
+                         cur_stream()), "side_mul");
+  return out;
+}
+
+// rank: value columns of a cached row (0: all)
 LatentAttnParams attn_base(const torch::Tensor& q, const torch::Tensor& cache, const torch::Tensor& table,
-                           torch::Tensor& out, int64_t H, int64_t window, double scale) {
+                           torch::Tensor& out, int64_t H, int64_t window, double scale, int64_t rank, const Opt& sink) {
   is_f32(q, "q");
   need_rows(q, "q");
   need_cache(cache, table, q.scalar_type());
   TORCH_CHECK(q.is_contiguous() && q.size(1) == H * cache.size(2), "q must be contiguous [T, H rank]");
   TORCH_CHECK(window >= 1, "window must be positive");
-  out = torch::empty_like(q);
+  const int64_t cols = lsd_latent_value_cols(cache.size(2), rank > 0 ? rank : cache.size(2));
+  out = torch::empty({q.size(0), H * cols}, q.options());
   LatentAttnParams p{};
+  p.v_pad = cols;
+  p.sink = sink_of(sink, H);
   p.q = q.data_ptr(); p.out = out.data_ptr();
   p.cache = cache.data_ptr(); p.table = table.data_ptr<int>(); p.tw = table.size(1);
   p.H = H; p.rank_pad = cache.size(2); p.window = (int)std::min<int64_t>(window, INT_MAX);
@@ -339,9 +434,10 @@ LatentAttnParams attn_base(const torch::Tensor& q, const torch::Tensor& cache, c
 
 // one query token per sequence; slots / pos [B]
 torch::Tensor latent_decode(torch::Tensor q, torch::Tensor cache, torch::Tensor table, torch::Tensor slots,
-                            torch::Tensor pos, int64_t H, int64_t window, double scale, int64_t splits) {
+                            torch::Tensor pos, int64_t H, int64_t window, double scale, int64_t splits, int64_t rank,
+                            Opt sink) {
   torch::Tensor out, po, pml;
-  LatentAttnParams p = attn_base(q, cache, table, out, H, window, scale);
+  LatentAttnParams p = attn_base(q, cache, table, out, H, window, scale, rank, sink);
   p.B = q.size(0);
   p.seq_slots = iptr(slots, p.B, "slots"); p.pos = iptr(pos, p.B, "pos");
   if (is_f32(q, "q") || lsd_latent_tile_rows(p.rank_pad) == 0) {
@@ -351,7 +447,7 @@ torch::Tensor latent_decode(torch::Tensor q, torch::Tensor cache, torch::Tensor 
   TORCH_CHECK(splits >= 1 && splits <= 1024, "splits");
   p.splits = splits;
   if (splits > 1) {
-    po = torch::empty({p.B * H * splits * p.rank_pad}, q.options().dtype(torch::kFloat32));
+    po = torch::empty({p.B * H * splits * p.v_pad}, q.options().dtype(torch::kFloat32));
     pml = torch::empty({p.B * H * splits * 2}, q.options().dtype(torch::kFloat32));
     p.part_o = po.data_ptr<float>(); p.part_ml = pml.data_ptr<float>();
   }
@@ -362,9 +458,9 @@ torch::Tensor latent_decode(torch::Tensor q, torch::Tensor cache, torch::Tensor 
 // packed ragged queries; tiles [n, 2] = (sequence, first (token, head) row)
 torch::Tensor latent_prefill(torch::Tensor q, torch::Tensor cache, torch::Tensor table, torch::Tensor tiles,
                              torch::Tensor seq_slots, torch::Tensor q_start, torch::Tensor cu_q, int64_t H,
-                             int64_t window, double scale) {
+                             int64_t window, double scale, int64_t rank, Opt sink) {
   torch::Tensor out;
-  LatentAttnParams p = attn_base(q, cache, table, out, H, window, scale);
+  LatentAttnParams p = attn_base(q, cache, table, out, H, window, scale, rank, sink);
   TORCH_CHECK(!is_f32(q, "q") && lsd_latent_tile_rows(p.rank_pad) > 0, "latent_prefill: no kernel for this rank");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2, "tiles must be [n, 2]");
   p.tiles = iptr(tiles, 0, "tiles"); p.n_tiles = tiles.size(0);
@@ -389,18 +485,20 @@ torch::Tensor latent_gather(torch::Tensor cache, torch::Tensor table, torch::Ten
   return out;
 }
 
-// q [T, H dim] over expanded k [rows, H dim], v [rows, H vdim] -> [T, H vdim]
+// q [T, H dim] over expanded k [rows, H dim], v [rows, H vdim] -> [T, H vdim], times
+// the sigmoid of gate [T, H vdim]
 torch::Tensor latent_expanded(torch::Tensor q, torch::Tensor k, torch::Tensor v, torch::Tensor tiles,
                               torch::Tensor cu_q, torch::Tensor q_start, torch::Tensor k_lo, torch::Tensor cu_k,
-                              int64_t H, int64_t window, double scale) {
+                              int64_t H, int64_t window, double scale, Opt sink, Opt gate) {
   need(q, torch::kBFloat16, "q");
   need(k, torch::kBFloat16, "k");
   need(v, torch::kBFloat16, "v");
   TORCH_CHECK(q.dim() == 2 && q.is_contiguous() && k.dim() == 2 && k.is_contiguous() && v.dim() == 2 &&
                   v.is_contiguous() && k.size(1) == q.size(1) && v.size(0) == k.size(0), "latent_expanded: shapes");
   const int64_t B = q_start.numel(), dim = q.size(1) / H, vdim = v.size(1) / H;
-  TORCH_CHECK(q.size(1) == H * dim && v.size(1) == H * vdim && (dim == 64 || dim == 128) && vdim % 16 == 0 &&
-                  vdim >= 16 && vdim <= 128 && window >= 1, "latent_expanded: dim 64 / 128, vdim % 16, vdim <= 128");
+  TORCH_CHECK(q.size(1) == H * dim && v.size(1) == H * vdim && (dim == 64 || dim == 128 || dim == 192) &&
+                  vdim % 16 == 0 && vdim >= 16 && vdim <= 128 && window >= 1,
+              "latent_expanded: dim 64 / 128 / 192, vdim % 16, vdim <= 128");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2, "tiles must be [n, 2]");
   auto out = torch::empty({q.size(0), v.size(1)}, q.options());
   lsd::LatentExpandedParams p{};
@@ -408,6 +506,8 @@ torch::Tensor latent_expanded(torch::Tensor q, torch::Tensor k, torch::Tensor v,
   p.tiles = iptr(tiles, 0, "tiles"); p.n_tiles = tiles.size(0);
   p.cu_q = iptr(cu_q, B + 1, "cu_q"); p.q_start = iptr(q_start, B, "q_start");
   p.k_lo = iptr(k_lo, B, "k_lo"); p.cu_k = iptr(cu_k, B + 1, "cu_k");
+  p.sink = sink_of(sink, H);
+  if (gate.has_value()) p.gate = gate_rows(*gate, q.size(0), H * vdim, p.ldg);
   p.H = H; p.dim = dim; p.vdim = vdim; p.window = (int)std::min<int64_t>(window, INT_MAX);
   p.scale_log2 = (float)(scale * 1.4426950408889634);
   check_hip(lsd_latent_expanded(&p, cur_stream()), "latent_expanded");
@@ -458,31 +558,37 @@ torch::Tensor embed_fp32(torch::Tensor ids, torch::Tensor wte, double scale) {
 }  // namespace
 
 void lsd_register_latent(pybind11::module& m) {
-  m.def("batch_linear", &batch_linear, py::arg("a"), py::arg("w"), py::arg("tm"));
+  m.def("batch_linear", &batch_linear, py::arg("a"), py::arg("w"), py::arg("tm"), py::arg("gate") = py::none());
   m.def("linear_fp32", &linear_fp32, py::arg("a"), py::arg("w"), py::arg("x") = py::none(),
         py::arg("bias") = py::none());
   m.def("moe_group", &moe_group, py::arg("ids"), py::arg("experts"), py::arg("tm"));
   m.def("moe_up", &moe_up, py::arg("h"), py::arg("perm"), py::arg("tiles"), py::arg("top"), py::arg("w"),
         py::arg("limit"), py::arg("alpha"), py::arg("ws"), py::arg("limit_s"), py::arg("tm"));
   m.def("moe_down", &moe_down, py::arg("mid"), py::arg("mids"), py::arg("perm"), py::arg("tiles"), py::arg("wts"),
-        py::arg("w"), py::arg("ws"), py::arg("slab"), py::arg("tm"));
+        py::arg("w"), py::arg("ws"), py::arg("slab"), py::arg("tm"), py::arg("wts_s") = py::none());
   m.def("moe_set_group_rows", [](int64_t v) { g_group_rows = v < 1 ? 1 : (int)v; });
   m.def("moe_few", &moe_few, py::arg("h"), py::arg("ids"), py::arg("wts"), py::arg("w_up"), py::arg("w_down"),
-        py::arg("limit"), py::arg("alpha"), py::arg("ws_up"), py::arg("ws_down"), py::arg("limit_s"), py::arg("x"));
+        py::arg("limit"), py::arg("alpha"), py::arg("ws_up"), py::arg("ws_down"), py::arg("limit_s"), py::arg("x"),
+        py::arg("wts_s") = py::none(), py::arg("add") = true);
   m.def("latent_post", &latent_post, py::arg("y"), py::arg("nq"), py::arg("want_q"), py::arg("f32"), py::arg("cache"),
         py::arg("rank"), py::arg("gain"), py::arg("eps"), py::arg("table"), py::arg("tslot"), py::arg("tpos"),
-        py::arg("correction"), py::arg("top"));
+        py::arg("correction"), py::arg("top"), py::arg("c_off") = -1, py::arg("rope") = py::none(), py::arg("q_head") = 0,
+        py::arg("q_rot") = 0, py::arg("q_gain") = py::none());
+  m.def("route_softmax", &route_softmax, py::arg("z"), py::arg("experts"), py::arg("top"), py::arg("shared"));
+  m.def("side_mul", &side_mul, py::arg("g"), py::arg("ids"), py::arg("table"));
+  m.def("latent_value_cols", [](int64_t rank_pad, int64_t rank) { return lsd_latent_value_cols((int)rank_pad, (int)rank); });
   m.def("latent_tile_rows", [](int64_t rank) { return lsd_latent_tile_rows((int)rank); });
   m.def("latent_decode", &latent_decode, py::arg("q"), py::arg("cache"), py::arg("table"), py::arg("slots"),
-        py::arg("pos"), py::arg("heads"), py::arg("window"), py::arg("scale"), py::arg("splits"));
+        py::arg("pos"), py::arg("heads"), py::arg("window"), py::arg("scale"), py::arg("splits"), py::arg("rank") = 0,
+        py::arg("sink") = py::none());
   m.def("latent_prefill", &latent_prefill, py::arg("q"), py::arg("cache"), py::arg("table"), py::arg("tiles"),
         py::arg("seq_slots"), py::arg("q_start"), py::arg("cu_q"), py::arg("heads"), py::arg("window"),
-        py::arg("scale"));
+        py::arg("scale"), py::arg("rank") = 0, py::arg("sink") = py::none());
   m.def("latent_gather", &latent_gather, py::arg("cache"), py::arg("table"), py::arg("seq_slots"), py::arg("k_lo"),
         py::arg("cu_k"), py::arg("rows"));
   m.def("latent_expanded", &latent_expanded, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("tiles"),
         py::arg("cu_q"), py::arg("q_start"), py::arg("k_lo"), py::arg("cu_k"), py::arg("heads"), py::arg("window"),
-        py::arg("scale"));
+        py::arg("scale"), py::arg("sink") = py::none(), py::arg("gate") = py::none());
   m.def("norm_fp32", &norm_fp32, py::arg("x"), py::arg("slab"), py::arg("w"), py::arg("eps"), py::arg("rows"),
         py::arg("want_out"), py::arg("width"), py::arg("woff"));
   m.def("embed_fp32", &embed_fp32, py::arg("ids"), py::arg("wte"), py::arg("scale"));

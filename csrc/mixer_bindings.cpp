@@ -16,11 +16,15 @@
 #include "kernels/mixer_params.h"
 
 using lsd::ConvParams;
+using lsd::ForgetParams;
 using lsd::GroupNormParams;
 using lsd::MixOutParams;
 using lsd::RecurParams;
 using lsd::RopeAppendParams;
 using lsd::SeqParams;
+using lsd::ShiftNormParams;
+using lsd::TanhNorm;
+using lsd::TanhStepParams;
 using lsd::TalkParams;
 
 extern "C" {
@@ -49,6 +53,12 @@ hipError_t lsd_paged_decode(const TalkParams* p, hipStream_t st);
 int lsd_mix_decode_gc(int H, int G);
 long lsd_mix_combine_lds(const TalkParams* p);
 hipError_t lsd_mix_decode(const TalkParams* p, hipStream_t st);
+int lsd_forget_ok(int D, int V);
+hipError_t lsd_forget_seq(const ForgetParams* p, int vb, int f32, hipStream_t st);
+hipError_t lsd_forget_chunk(const ForgetParams* p, hipStream_t st);
+hipError_t lsd_tanh_step(const TanhStepParams* p, int f32, hipStream_t st);
+hipError_t lsd_shift_norm(const ShiftNormParams* p, int f32, hipStream_t st);
+hipError_t lsd_shift_tail(const ShiftNormParams* p, int f32, hipStream_t st);
 hipError_t lsd_group_rows_norm(const GroupNormParams* p, int f32, hipStream_t st);
 }
 
@@ -122,7 +132,8 @@ ConvParams conv(const Tensor& y, int64_t c0, const Tensor& w, const Opt& bias, c
   return c;
 }
 
-void state_of(RecurParams& p, const Tensor& state, int64_t heads, int64_t D, int64_t V) {
+template <typename P>
+void state_of(P& p, const Tensor& state, int64_t heads, int64_t D, int64_t V) {
   p.heads = heads; p.D = D; p.V = V; p.Vp = (V + 3) / 4 * 4;
   TORCH_CHECK(state.is_cuda() && state.scalar_type() == torch::kFloat32 && state.is_contiguous() && state.dim() == 4 &&
                   state.size(1) == heads && state.size(2) == D && state.size(3) == p.Vp,
@@ -130,7 +141,8 @@ void state_of(RecurParams& p, const Tensor& state, int64_t heads, int64_t D, int
   p.S = state.data_ptr<float>();
 }
 
-void out_rows(RecurParams& p, const Tensor& out, const Tensor& y) {
+template <typename P>
+void out_rows(P& p, const Tensor& out, const Tensor& y) {
   rows_of(out, y.scalar_type(), y.size(0), (int64_t)p.heads * p.V, "out");
   p.out = out.data_ptr(); p.ldo = out.stride(0); p.out_cols = out.size(1);
 }
@@ -223,6 +235,49 @@ void ssm_seq(Tensor y, Tensor slots, Tensor start, Tensor cu, int64_t heads, int
   o.out = p.out; o.ldo = p.ldo; o.out_cols = p.out_cols;
   check_hip(lsd_group_norm(&o, f32, cur_stream()), "group_norm");
   if (!single) check_hip(lsd_conv_tail(&p.c, &p.s, f32, cur_stream()), "conv_tail");
+}
+
+// y [T, N]: q [heads D] | forget gate's logits [heads D] | v [heads V].  chunked:
+// prompts of bf16 models, each sequence in `segs` segments that run together
+void forget_seq(Tensor y, Tensor slots, Tensor start, Tensor cu, int64_t heads, int64_t D, int64_t V, Tensor bias,
+                Tensor lower, Tensor norm, double eps, Tensor state, Tensor out, bool chunked, int64_t segs) {
+  const bool f32 = is_f32(y, "y");
+  TORCH_CHECK(heads >= 1 && D >= 1 && V >= 1, "forget_seq: sizes");
+  ForgetParams p{};
+  rows_of(y, y.scalar_type(), y.size(0), heads * (2 * D + V), "y");
+  p.y = y.data_ptr(); p.ldy = y.stride(0);
+  p.s = seqs(slots, start, cu);
+  state_of(p, state, heads, D, V);
+  p.bias = fptr(bias, heads * D, "bias"); p.lower = fptr(lower, heads * D, "lower"); p.norm = fptr(norm, V, "norm");
+  p.eps = (float)eps;
+  out_rows(p, out, y);
+  if (chunked) {
+    TORCH_CHECK(!f32 && lsd_forget_ok(D, V) && segs >= 1 && segs <= 64, "forget_seq: no chunked kernel");
+    p.segs = segs;
+    Tensor part, decay;
+    if (segs > 1) {
+      const int64_t n = p.s.B * heads * segs;
+      part = torch::empty({n * D * p.Vp}, y.options().dtype(torch::kFloat32));
+      decay = torch::empty({n * D}, y.options().dtype(torch::kFloat32));
+      p.part = part.data_ptr<float>(); p.decay = decay.data_ptr<float>();
+    }
+    check_hip(lsd_forget_chunk(&p, cur_stream()), "forget_chunk");
+    return;
+  }
+  const int vb = lsd_recur_block(D, V);
+  TORCH_CHECK(vb > 0 && 2 * D * sizeof(float) <= 48 * 1024, "forget_seq: no kernel for dimension ", D);
+  Tensor raw;
+  if (p.Vp > vb) {
+    raw = torch::empty({y.size(0), heads * V}, y.options().dtype(torch::kFloat32));
+    p.raw = raw.data_ptr<float>(); p.ldr = heads * V;
+  }
+  check_hip(lsd_forget_seq(&p, vb, f32, cur_stream()), "forget_seq");
+  if (p.raw) {
+    MixOutParams o{};
+    o.raw = p.raw; o.ldr = p.ldr; o.T = y.size(0); o.heads = heads; o.V = V; o.norm = p.norm; o.eps = p.eps;
+    o.out = p.out; o.ldo = p.ldo; o.out_cols = p.out_cols;
+    check_hip(lsd_head_norm_gate(&o, f32, cur_stream()), "head_norm_gate");
+  }
 }
 
 // rows [x | x0] (fp32 or bf16) of a loop's entry; x <- step
@@ -513,6 +568,92 @@ Opt group_norm(Tensor x, int64_t groups, int64_t width, double eps, Opt slab, Op
   return out;
 }
 
+// weight and bias [H] of an elementwise norm in the element type
+TanhNorm tanh_norm(double alpha, const Tensor& w, const Tensor& b, int64_t H, c10::ScalarType dt) {
+  for (const Tensor* t : {&w, &b})
+    TORCH_CHECK(t->is_cuda() && t->scalar_type() == dt && t->is_contiguous() && t->numel() == H, "norm vectors must be [H]");
+  return {(float)alpha, w.data_ptr(), b.data_ptr()};
+}
+
+// slabs [S, T, H] (bf16 or fp32)
+template <typename P>
+void slabs_of(P& p, const Tensor& slab) {
+  const bool sf = is_f32(slab, "slab");
+  TORCH_CHECK(slab.is_contiguous() && slab.dim() == 3 && slab.size(0) >= 1 && slab.size(1) == p.T && slab.size(2) == p.H,
+              "slab must be [S, T, H]");
+  p.slab = slab.data_ptr(); p.splits = slab.size(0); p.slab_bf16 = !sf;
+}
+
+// x [T, H] fp32.  slab, post: x += tanh(alpha sum) w + b; want_out: returns
+// tanh(alpha x) w + b (pre), or x in the element type; rows of x (no slab), all by default
+Opt tanh_step(Tensor x, Opt slab, double a_post, Opt w_post, Opt b_post, bool want_out, double a_pre, Opt w_pre, Opt b_pre,
+              Opt rows, bool f32) {
+  const auto dt = f32 ? torch::kFloat32 : torch::kBFloat16;
+  TORCH_CHECK(x.dim() == 2 && x.size(1) % 4 == 0, "x must be [T, H], H % 4");
+  TanhStepParams p{};
+  p.T = x.size(0); p.H = x.size(1);
+  p.x = const_cast<float*>(fptr(x, (int64_t)p.T * p.H, "x"));
+  if (slab.has_value()) {
+    TORCH_CHECK(w_post.has_value() && b_post.has_value() && !rows.has_value(), "slabs need a norm, and all rows");
+    slabs_of(p, *slab);
+    p.post = tanh_norm(a_post, *w_post, *b_post, p.H, dt);
+  }
+  if (rows.has_value()) {
+    p.n_rows = rows->numel();
+    p.rows = iptr(*rows, p.n_rows, "rows");
+  }
+  Opt out;
+  if (want_out) {
+    if (w_pre.has_value()) p.pre = tanh_norm(a_pre, *w_pre, *b_pre, p.H, dt);
+    out = torch::empty({p.rows ? p.n_rows : p.T, p.H}, x.options().dtype(dt));
+    p.out = out->data_ptr();
+  }
+  check_hip(lsd_tanh_step(&p, f32, cur_stream()), "tanh_step");
+  return out;
+}
+
+// x [T, H] fp32 -> (residual, shifted norm rows).  slab, w_side: residual = x + rms(sum
+// of slabs) w_side over `width` columns, else x itself; last [slots, H]
+std::vector<Tensor> shift_norm(Tensor x, Opt slab, Opt w_side, int64_t width, double eps, double alpha, Tensor w, Tensor b,
+                               Tensor mix, Tensor last, Tensor tslot, Tensor tpos, bool f32) {
+  const auto dt = f32 ? torch::kFloat32 : torch::kBFloat16;
+  TORCH_CHECK(x.dim() == 2 && x.size(1) % 4 == 0, "x must be [T, H], H % 4");
+  ShiftNormParams p{};
+  p.T = x.size(0); p.H = x.size(1); p.size = width; p.eps = (float)eps;
+  p.x = fptr(x, (int64_t)p.T * p.H, "x");
+  p.pre = tanh_norm(alpha, w, b, p.H, dt);
+  p.mix = tanh_norm(0.0, mix, mix, p.H, dt).w;
+  TORCH_CHECK(last.dim() == 2 && last.size(1) == p.H, "last must be [slots, H]");
+  p.last = const_cast<float*>(fptr(last, last.numel(), "last"));
+  p.tslot = iptr(tslot, p.T, "tslot"); p.tpos = iptr(tpos, p.T, "tpos");
+  Tensor x_new = x;
+  if (slab.has_value()) {
+    TORCH_CHECK(w_side.has_value() && width >= 1 && width <= p.H, "slabs need a norm");
+    slabs_of(p, *slab);
+    p.w_side = tanh_norm(0.0, *w_side, *w_side, p.H, dt).w;
+    x_new = torch::empty_like(x);
+    p.x_new = x_new.data_ptr<float>();
+  }
+  auto out = torch::empty({p.T, p.H}, x.options().dtype(dt));
+  p.out = out.data_ptr();
+  check_hip(lsd_shift_norm(&p, f32, cur_stream()), "shift_norm");
+  return {x_new, out};
+}
+
+// last[slot of row] = norm(x[row]) for `rows` of x
+void shift_tail(Tensor x, double alpha, Tensor w, Tensor b, Tensor last, Tensor tslot, Tensor rows, bool f32) {
+  ShiftNormParams p{};
+  p.T = x.size(0); p.H = x.size(1);
+  p.x = fptr(x, (int64_t)p.T * p.H, "x");
+  p.pre = tanh_norm(alpha, w, b, p.H, f32 ? torch::kFloat32 : torch::kBFloat16);
+  TORCH_CHECK(last.dim() == 2 && last.size(1) == p.H && p.H % 4 == 0, "last must be [slots, H]");
+  p.last = const_cast<float*>(fptr(last, last.numel(), "last"));
+  p.tslot = iptr(tslot, p.T, "tslot");
+  p.n_tail = rows.numel();
+  p.tail = iptr(rows, p.n_tail, "rows");
+  check_hip(lsd_shift_tail(&p, f32, cur_stream()), "shift_tail");
+}
+
 }  // namespace
 
 void lsd_register_mixers(pybind11::module& m) {
@@ -526,6 +667,17 @@ void lsd_register_mixers(pybind11::module& m) {
         py::arg("groups"), py::arg("state_dim"), py::arg("vdim"), py::arg("norm_groups"), py::arg("taps"), py::arg("bias"),
         py::arg("ring"), py::arg("state"), py::arg("A"), py::arg("dt_bias"), py::arg("skip"), py::arg("norm"),
         py::arg("gain"), py::arg("eps"), py::arg("out"), py::arg("single"), py::arg("chunked") = false);
+  m.def("forget_ok", [](int64_t D, int64_t V) { return lsd_forget_ok((int)D, (int)V) != 0; });
+  m.def("forget_seq", &forget_seq, py::arg("y"), py::arg("slots"), py::arg("start"), py::arg("cu"), py::arg("heads"),
+        py::arg("dim"), py::arg("vdim"), py::arg("bias"), py::arg("lower"), py::arg("norm"), py::arg("eps"),
+        py::arg("state"), py::arg("out"), py::arg("chunked"), py::arg("segs"));
+  m.def("tanh_step", &tanh_step, py::arg("x"), py::arg("slab"), py::arg("a_post"), py::arg("w_post"), py::arg("b_post"),
+        py::arg("want_out"), py::arg("a_pre"), py::arg("w_pre"), py::arg("b_pre"), py::arg("rows"), py::arg("f32"));
+  m.def("shift_norm", &shift_norm, py::arg("x"), py::arg("slab"), py::arg("w_side"), py::arg("width"), py::arg("eps"),
+        py::arg("alpha"), py::arg("w"), py::arg("b"), py::arg("mix"), py::arg("last"), py::arg("tslot"), py::arg("tpos"),
+        py::arg("f32"));
+  m.def("shift_tail", &shift_tail, py::arg("x"), py::arg("alpha"), py::arg("w"), py::arg("b"), py::arg("last"),
+        py::arg("tslot"), py::arg("rows"), py::arg("f32"));
   m.def("loop_pack", &loop_pack, py::arg("x"), py::arg("x0"), py::arg("step"), py::arg("f32"));
   m.def("glu_f32", &glu_f32, py::arg("y"), py::arg("out"), py::arg("glu"), py::arg("scale"));
   m.def("rope_append", &rope_append, py::arg("y"), py::arg("heads"), py::arg("k"), py::arg("v"), py::arg("table"),

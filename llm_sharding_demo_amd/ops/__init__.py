@@ -32,9 +32,21 @@ from . import reference as ref
 class Residual:
     x: torch.Tensor  # fp32 [T, H]
     pending: List[Tuple[torch.Tensor, Optional[torch.Tensor]]] = field(default_factory=list)
-    # output of a sublayer that is normed before it is added: (slabs [S, T, H],
-    # bias, norm weight, model config), folded in by the next group_norm or flush
-    post: Optional[tuple] = None
+    # output of a sublayer that is normed before it is added, folded in by the
+    # next norm or flush
+    post: Optional["PostNorm"] = None
+
+
+@dataclass
+class PostNorm:
+    """A sublayer's output [S, T, H] (split-K slabs) on its way through a norm
+    into the residual: RMS in equal parts (weight, model config), or elementwise
+    (alpha, weight, bias)."""
+
+    slab: torch.Tensor
+    bias: Optional[torch.Tensor] = None
+    rms: Optional[tuple] = None   # (weight, parts, columns, eps)
+    tanh: Optional[tuple] = None  # (alpha, weight, bias)
 
 
 # sigmoid slope of the experts' gated activation (fixed by the design)

@@ -12,9 +12,9 @@ Device weight layout (set up once per stage by `prepare_stage`):
     q and the K cache simply live in that order.
   * Llama gate/up rows interleaved in 16-row blocks so one wave holds the gate
     and up value of the same output column (silu(gate)*up fused epilogue).
-  * Timisun, Vizalix, Kedasun: every width padded with zeros to what the MFMA
-    tiles want, so a model of any sizes runs (see _prepare_timisun,
-    _prepare_vizalix and _prepare_kedasun); fp32 or bf16.
+  * Timisun, Vizalix, Kedasun, Fagunex: every width padded with zeros to what the
+    MFMA tiles want, so a model of any sizes runs (see _prepare_timisun,
+    _prepare_vizalix, _prepare_kedasun and _prepare_fagunex); fp32 or bf16.
 """
 from __future__ import annotations
 
@@ -25,9 +25,9 @@ from typing import Optional
 import numpy as np
 import torch
 
-from ..config import AttentionSpec, ChannelDeltaSpec, RopeSpec, SSMSpec
+from ..config import AttentionSpec, ChannelDeltaSpec, ForgetSpec, LatentAttentionSpec, RopeSpec, SSMSpec
 from ..runtime.kv_cache import layer_cache
-from . import GLU_ALPHA, Backend, Residual
+from . import GLU_ALPHA, Backend, PostNorm, Residual
 from .routing import Routing
 
 _C = None
@@ -206,6 +206,8 @@ class HipBackend(Backend):
             self._prepare_vizalix(stage)
         elif cfg.arch == "kedasun":
             self._prepare_kedasun(stage)
+        elif cfg.arch == "fagunex":
+            self._prepare_fagunex(stage)
         elif stage.last:
             # pad the head IN PLACE: the stage keeps one [vocab_padded, H]
             # tensor and its weight dict points at the first V rows (a
@@ -245,8 +247,8 @@ class HipBackend(Backend):
     def row_width(self, mcfg) -> int:
         return _up(mcfg.hidden, 64) if mcfg.layers else mcfg.hidden
 
-    def layer_cache(self, mixer):
-        return layer_cache(mixer, _up)
+    def layer_cache(self, mixer, shift: int = 0):
+        return layer_cache(mixer, _up, shift)
 
     def latent_width(self, rank: int) -> int:
         return _up(rank, 64)
@@ -276,9 +278,7 @@ class HipBackend(Backend):
             m, f, p = cfg.layers[i].mixer, cfg.layers[i].mlp, f"layers.{i}."
             t = lambda n: w.pop(p + n)  # noqa: E731
             rank, dp = self.latent_width(m.kv_rank), _up(m.dim, 64)
-            vp = _up(m.vdim, 16)
-            while m.heads * vp % 64:
-                vp += 16
+            vp = self._latent_vcols(m)
             w[p + "input_layernorm.weight"] = pad_to(w[p + "input_layernorm.weight"], hp)
             q = pad_to(t("attn.q.weight").reshape(m.heads, m.dim, -1), m.heads, dp, hp).reshape(m.heads * dp, hp)
             rows = [q]
@@ -288,14 +288,7 @@ class HipBackend(Backend):
             if f is not None:
                 rows.append(pad_to(t("mlp.router.weight"), f.experts, hp))
                 w[p + "mlp.correction"] = w[p + "mlp.correction"].float().contiguous()
-                w[p + "mlp.experts.gate_up.weight"] = interleave_experts(
-                    t("mlp.experts.gate_up.weight"), _up(f.expert.ff, 64), hp)
-                w[p + "mlp.experts.down.weight"] = pad_to(t("mlp.experts.down.weight"), f.experts, hp,
-                                                          _up(f.expert.ff, 64))
-                if f.shared is not None:
-                    w[p + "mlp.shared.gate_up.weight"] = interleave_experts(
-                        t("mlp.shared.gate_up.weight"), _up(f.shared.ff, 64), hp)
-                    w[p + "mlp.shared.down.weight"] = pad_to(t("mlp.shared.down.weight"), hp, _up(f.shared.ff, 64))
+                self._prepare_experts(w, p, f, hp)
             n = sum(x.shape[0] for x in rows)
             w[p + "attn.in.weight"] = pad_to(torch.cat(rows), _up(n, 64), hp)
             uk = t("attn.uk.weight").reshape(m.heads, m.dim, m.kv_rank)
@@ -305,6 +298,129 @@ class HipBackend(Backend):
             w[p + "attn.uv.weight"] = pad_to(t("attn.uv.weight").reshape(m.heads, m.vdim, m.kv_rank), m.heads, vp, rank)
             o = t("attn.o.weight").reshape(-1, m.heads, m.vdim)
             w[p + "attn.o.weight"] = pad_to(o, hp, m.heads, vp).reshape(hp, m.heads * vp)
+
+    @staticmethod
+    def _latent_vcols(m) -> int:
+        """Columns of a value head: padded so that all heads together fill the
+        out-projection's K tiles."""
+        vp = _up(m.vdim, 16)
+        while m.heads * vp % 64:
+            vp += 16
+        return vp
+
+    @staticmethod
+    def _prepare_experts(w, p: str, f, hp: int) -> None:
+        """Gate / up rows interleaved in 16-row blocks, widths padded."""
+        t = lambda n: w.pop(p + n)  # noqa: E731
+        w[p + "mlp.experts.gate_up.weight"] = interleave_experts(t("mlp.experts.gate_up.weight"), _up(f.expert.ff, 64), hp)
+        w[p + "mlp.experts.down.weight"] = pad_to(t("mlp.experts.down.weight"), f.experts, hp, _up(f.expert.ff, 64))
+        if f.shared is not None:
+            w[p + "mlp.shared.gate_up.weight"] = interleave_experts(t("mlp.shared.gate_up.weight"), _up(f.shared.ff, 64), hp)
+            w[p + "mlp.shared.down.weight"] = pad_to(t("mlp.shared.down.weight"), hp, _up(f.shared.ff, 64))
+
+    def _prepare_fagunex(self, stage) -> None:
+        """Device layout per layer (zero padding everywhere):
+          attn.in      [queries, or their latent | output gate | latent | turned key part] x H;
+                       heads padded, turned pairs (2i, 2i + 1) moved to (i, i + dims / 2) --
+                       scores do not change under a common order of q and k
+          attn.uq      queries from their latent
+          attn.uk      [heads][rank + turned][dim + turned]: queries into the latent space,
+                       the turned part passed on by an identity block
+          attn.uk_rows [heads dim][rank + turned]: cached rows to keys (expanded prefill)
+          attn.uv      [heads][vdim][value columns of the attention kernels]
+          mixer.in     q | forget gate | v of a recurrence
+          mlp.router   router rows, behind them the shared expert's gate
+          side.*       width of the tokens' rows padded
+        The norms' alphas stay on the host; gains of latents, gate biases and bounds,
+        sinks and the recurrence's norm are fp32."""
+        cfg, w, dev = stage.cfg, stage.w, stage.device
+        hp = self.row_width(cfg)
+        self._ropes = {}
+
+        def norm(name: str) -> None:
+            w[name + ".weight"], w[name + ".bias"] = (pad_to(w[name + s], hp) for s in (".weight", ".bias"))
+            w[name + ".alpha"] = w[name + ".alpha"].float().cpu()
+
+        if "embed_tokens" in w:
+            w["embed_tokens"] = pad_to(w["embed_tokens"], cfg.vocab_size, hp)
+        if "lm_head" in w:
+            e = pad_to(w["lm_head"], cfg.vocab_padded, hp)
+            w["lm_head"], stage._lm_head_padded = e[: cfg.vocab_size], e
+            norm("norm")
+        for j, i in {cfg.weight_layer(i): i for i in stage.layers}.items():
+            m, f, p = cfg.layers[i].mixer, cfg.layers[i].mlp, f"layers.{j}."
+            t = lambda n: w.pop(p + n)  # noqa: E731
+            f32 = lambda n: w.__setitem__(p + n, w[p + n].float().contiguous())  # noqa: E731
+            for n in ("norm1", "norm1b") + (("norm2", "norm2b") if f is not None else ()):
+                norm(p + n)
+            w[p + "shift"] = pad_to(w[p + "shift"], hp)
+            if isinstance(m, ForgetSpec):
+                rows = torch.cat([t("mixer.q"), t("mixer.f"), t("mixer.v")])
+                w[p + "mixer.in.weight"] = pad_to(rows, _up(rows.shape[0], 64), hp)
+                for n in ("mixer.f.b", "mixer.lower", "mixer.norm"):
+                    f32(n)
+                o = t("mixer.o")
+                w[p + "mixer.o"] = pad_to(o, hp, _up(o.shape[1], 64))
+            else:
+                self._prepare_latent(stage, m, p, hp)
+            if f is not None:
+                rows = [t("mlp.router.weight")] + ([t("mlp.shared.sg")] if f.shared_gate else [])
+                rows = torch.cat(rows)
+                w[p + "mlp.router.weight"] = pad_to(rows, _up(rows.shape[0], 64), hp)
+                self._prepare_experts(w, p, f, hp)
+            if cfg.token_side:
+                n = _up(cfg.token_side, 64)
+                w[p + "side.embed"] = pad_to(w[p + "side.embed"], cfg.vocab_size, n)
+                w[p + "side.gate"], w[p + "side.proj"] = pad_to(w[p + "side.gate"], n, hp), pad_to(w[p + "side.proj"], hp, n)
+                w[p + "side.norm"] = pad_to(w[p + "side.norm"], hp)
+
+    def _prepare_latent(self, stage, m, p: str, hp: int) -> None:
+        """Latent attention with a turned part (the layout is _prepare_fagunex')."""
+        w, dev = stage.w, stage.device
+        t = lambda n: w.pop(p + n)  # noqa: E731
+        rot, rank, H = m.rot_dim, m.kv_rank, m.heads
+        dp, cols, vp = _up(m.q_dim, 64), self.latent_width(rank + rot), self._latent_vcols(m)
+        order = torch.arange(rot, device=dev)
+        if rot and m.rope.interleaved:
+            order = split_pairs(rot, rot).to(dev)
+        if rot and m.rope not in self._ropes:
+            self._ropes[m.rope] = rope_spec_table(m.rope, _up(stage.max_seq, 64), dev)
+
+        def q_rows(x):  # [H (dim + rot), n] -> padded heads
+            x = x.reshape(H, m.q_dim, -1)
+            x = torch.cat([x[:, : m.dim], x[:, m.dim:].index_select(1, order)], 1)
+            return pad_to(x, H, dp, x.shape[2])
+
+        rows = []
+        if m.q_rank is None:
+            q = q_rows(t("attn.q.weight"))
+            rows.append(pad_to(q, H, dp, hp).reshape(H * dp, hp))
+        else:
+            qr = _up(m.q_rank, 64)
+            rows.append(pad_to(t("attn.dq.weight"), qr, hp))
+            q = q_rows(t("attn.uq.weight"))
+            w[p + "attn.uq.weight"] = pad_to(q, H, dp, qr).reshape(H * dp, qr)
+            w[p + "attn.dq_norm.weight"] = w[p + "attn.dq_norm.weight"].float().contiguous()
+        if m.gate:
+            g = t("attn.g.weight").reshape(H, m.vdim, -1)
+            rows.append(pad_to(g, H, vp, hp).reshape(H * vp, hp))
+        d = t("attn.dkv.weight")
+        rows.append(pad_to(torch.cat([d[:rank], d[rank:].index_select(0, order)]), rank + rot, hp))
+        n = sum(x.shape[0] for x in rows)
+        w[p + "attn.in.weight"] = pad_to(torch.cat(rows), _up(n, 64), hp)
+        w[p + "attn.dkv_norm.weight"] = w[p + "attn.dkv_norm.weight"].float().contiguous()
+        uk = torch.zeros(H, cols, dp, dtype=stage.dtype, device=dev)
+        uk[:, :rank, : m.dim] = t("attn.uk.weight").reshape(H, m.dim, rank).transpose(1, 2)
+        uk[:, rank: rank + rot, m.dim: m.q_dim] = torch.eye(rot, dtype=stage.dtype, device=dev)
+        w[p + "attn.uk.weight"] = uk
+        if not self.fp32:
+            w[p + "attn.uk_rows.weight"] = uk.transpose(1, 2).reshape(H * dp, cols).contiguous()
+        vc = self.C.latent_value_cols(cols, rank)
+        w[p + "attn.uv.weight"] = pad_to(t("attn.uv.weight").reshape(H, m.vdim, rank), H, vp, vc)
+        o = t("attn.o.weight").reshape(-1, H, m.vdim)
+        w[p + "attn.o.weight"] = pad_to(o, hp, H, vp).reshape(hp, H * vp)
+        if m.sink:
+            w[p + "attn.sink"] = w[p + "attn.sink"].float().contiguous()
 
     def _prepare_vizalix(self, stage) -> None:
         """Device layout per layer (zero padding everywhere):
@@ -507,7 +623,7 @@ class HipBackend(Backend):
 
     # -- layers with norms around each sublayer (models/stage.py _sandwich_layer) ----
     def group_norm(self, r: Residual, w, mcfg):
-        slab, bias, w_post = r.post[:3] if r.post is not None else (None, None, None)
+        slab, bias, w_post = (r.post.slab, r.post.bias, r.post.rms[0]) if r.post is not None else (None, None, None)
         r.post = None
         return self.C.group_norm(r.x, mcfg.norm_groups, mcfg.hidden, mcfg.norm_eps, slab, bias, w_post, w, None, self.fp32)
 
@@ -517,14 +633,89 @@ class HipBackend(Backend):
     def linear_post_norm(self, a, w, b, norm_w, r: Residual, mcfg) -> None:
         """x += norm(a w^T + b), left to the next group_norm or flush as the
         projection's slabs."""
+        r.post = PostNorm(self._slabs(a, w, r.x), b, rms=(norm_w, mcfg.norm_groups, mcfg.hidden, mcfg.norm_eps))
+
+    def _slabs(self, a, w, x):
+        """a w^T as slabs [S, T, H] (their sum); x: rows of the same shape."""
         (M, K), N = a.shape, w.shape[0]
         if self.fp32 or self._gemv_in(a, K, EPI_F32) is not None or (
                 not self._tiled(M, N) and self._resid_splits(M, N, K) == 1):
-            slab = self._linear_f32(a, w)[None]
+            return self._linear_f32(a, w)[None]
+        return self.C.linear_residual(a, w, None, x, self._resid_splits(M, N, K), self._tiled(M, N), self.counters, True, None)
+
+    # -- layers with elementwise norms (models/stage.py _token_layer) ----------------
+    @staticmethod
+    def _tanh(n):
+        return float(n(".alpha")), n(".weight"), n(".bias")
+
+    def _tanh_step(self, r: Residual, out: bool, pre=(0.0, None, None), rows=None):
+        """Folds a pending elementwise norm; with `out` the residual normed by
+        `pre`, or in the element type."""
+        post = r.post if r.post is not None and r.post.tanh else None
+        if r.post is not None and post is None:
+            self.flush(r)
+        r.post = None
+        slab, args = (post.slab, post.tanh) if post is not None else (None, (0.0, None, None))
+        return self.C.tanh_step(r.x, slab, *args, out, *pre, rows, self.fp32)
+
+    def tanh_norm(self, r: Residual, n):
+        return self._tanh_step(r, True, self._tanh(n))
+
+    def tanh_norm_rows(self, x, n, rows=None):
+        return self._tanh_step(Residual(x), True, self._tanh(n), rows)
+
+    def shift_norm(self, r: Residual, w, last, meta, mcfg):
+        """The layer's first norm, its rows moved towards the previous token's by
+        w("shift"); `last` [slots, H]: the previous portion's last row."""
+        if r.post is not None and r.post.tanh:
+            self.flush(r)
+        slab, gain = (r.post.slab, r.post.rms[0]) if r.post is not None else (None, None)
+        r.post = None
+        norm = self._tanh(lambda n: w("norm1" + n))
+        r.x, h = self.C.shift_norm(r.x, slab, gain, mcfg.hidden, mcfg.norm_eps, *norm, w("shift"), last, meta.token_slots,
+                                   meta.token_pos, self.fp32)
+        for s, mt in self._parts(meta):
+            if not mt.is_decode:
+                self.C.shift_tail(r.x[s], *norm, last, mt.token_slots, mt.last_idx, self.fp32)
+        return h
+
+    def linear_tanh(self, a, wt, n, r: Residual) -> None:
+        """x += norm(a wt^T), left to the next norm as the projection's slabs."""
+        r.post = PostNorm(self._slabs(a, wt, r.x), tanh=self._tanh(n))
+
+    def experts_tanh(self, h, w, mlp, n, r: Residual) -> None:
+        """x += norm(experts(h)), left to the next norm: one slab per choice and the
+        shared expert's."""
+        ids, wts, shared = self.C.route_softmax(self._linear_f32(h, w("mlp.router.weight")), mlp.experts, mlp.top,
+                                                mlp.shared_gate)
+        shared = shared if mlp.shared_gate else None
+        T, H = h.shape
+        if not self.fp32 and T <= self.R.moe_few_t:
+            slab = torch.empty(1, T, H, dtype=torch.float32, device=h.device)
+            self._moe_few(h, ids, wts, w, mlp, slab[0], shared, False)
         else:
-            slab = self.C.linear_residual(a, w, None, r.x, self._resid_splits(M, N, K), self._tiled(M, N), self.counters,
-                                          True, None)
-        r.post = (slab, b, norm_w, mcfg)
+            slab = torch.empty(mlp.top + (mlp.shared is not None), T, H, dtype=h.dtype, device=h.device)
+            self._moe(h, ids, wts, w, mlp, slab, shared)
+        r.post = PostNorm(slab, tanh=self._tanh(n))
+
+    def token_side(self, r: Residual, ids, w, mcfg) -> None:
+        """x += rms(proj(gelu(gate x) * e)) * norm, e the tokens' rows of the layer's
+        table; the norm is left to the next layer."""
+        x = self._tanh_step(r, True)
+        g = self._linear_f32(x, w("side.gate")) if self.fp32 else self.linear(x, w("side.gate"), act="gelu")
+        g = self.C.side_mul(g, ids, w("side.embed"))
+        r.post = PostNorm(self._slabs(g, w("side.proj"), r.x), rms=(w("side.norm"), 1, mcfg.hidden, mcfg.norm_eps))
+
+    def forget_mix(self, h, w, m, state, meta, eps):
+        """Recurrence with forget gates in front of the out-projection (rows padded)."""
+        y = self._rows(h, w("mixer.in.weight"))
+        out = torch.empty(y.shape[0], w("mixer.o").shape[1], dtype=y.dtype, device=y.device)
+        for s, mt in self._parts(meta):
+            chunked = self._chunked(mt) and self.C.forget_ok(m.dim, m.vdim)
+            segs = self.R.forget_segments(mt.num_seqs * m.heads, mt.max_q) if chunked else 1
+            self.C.forget_seq(y[s], mt.seq_slots, mt.q_start, mt.cu_q, m.heads, m.dim, m.vdim, w("mixer.f.b"),
+                              w("mixer.lower"), w("mixer.norm"), eps, state, out[s], chunked, segs)
+        return out
 
     def clamped_glu(self, h, w, limit: float):
         if self.fp32:
@@ -634,54 +825,65 @@ class HipBackend(Backend):
     def _tm(self, rows: float) -> int:
         return 64 if self.fp32 else self.R.group_tm(rows)
 
-    def _batch_linear(self, a, w):
-        return self.C.batch_linear(a, w, 64 if self.fp32 else self.R.batch_tm(a.shape[0], w.shape[0], w.shape[1]))
+    def _batch_linear(self, a, w, gate=None):
+        return self.C.batch_linear(a, w, 64 if self.fp32 else self.R.batch_tm(a.shape[0], w.shape[0], w.shape[1]), gate)
 
-    def latent_project(self, h, w, spec, kv, pool, meta, eps):
-        m, f = spec.mixer, spec.mlp
+    def latent_project(self, h, w, m, mlp, kv, pool, meta, eps):
+        """Queries per head, turned; the output gate's logits; the routing of experts
+        `mlp` that read the same rows."""
         y = self._linear_f32(h, w("attn.in.weight"))
-        own = m.kv_from is None
+        own, dp = m.kv_from is None, w("attn.uk.weight").shape[2]
+        nq = m.heads * dp if m.q_rank is None else w("attn.uq.weight").shape[1]
+        ng = m.heads * self._latent_vcols(m) if m.gate else 0
+        rope = self._ropes[m.rope] if m.rot_dim else None
+        where = (meta.token_slots, meta.token_pos)
+        turn = dict(rope=rope, q_head=dp, q_rot=m.dim)
+        gains = w("attn.dkv_norm.weight") if own else None
+        keep = self.fp32 and rope is None and m.q_rank is None  # the queries are read where they are
         q, ids, wts = self.C.latent_post(
-            y, m.heads * w("attn.uk.weight").shape[2], not self.fp32, self.fp32, pool if own else None, m.kv_rank,
-            w("attn.dkv_norm.weight") if own else None, eps, kv.table, meta.token_slots, meta.token_pos,
-            w("mlp.correction") if f is not None else None, f.top if f is not None else 0)
-        return (y if self.fp32 else q), (ids, wts)
+            y, nq, not keep, self.fp32, pool if own else None, m.kv_rank, gains, eps, kv.table, *where,
+            w("mlp.correction") if mlp is not None else None, mlp.top if mlp is not None else 0, c_off=nq + ng,
+            q_gain=None if m.q_rank is None else w("attn.dq_norm.weight"), **turn)
+        if m.q_rank is not None:
+            q = self._linear_f32(q, w("attn.uq.weight"))
+            if rope is not None or not self.fp32:
+                q = self.C.latent_post(q, m.heads * dp, True, self.fp32, None, 0, None, eps, None, *where, None, 0, **turn)[0]
+        return (y if keep else q), (y[:, nq: nq + ng] if m.gate else None), (ids, wts)
 
-    def latent_attention(self, q, w, m, kv, pool, meta):
-        if getattr(meta, "dec", None) is not None:  # mixed step: each part its own kernel
-            return torch.cat([self._latent_part(q[: meta.b], w, m, kv, pool, meta.dec),
-                              self._latent_part(q[meta.b:], w, m, kv, pool, meta.pf)])
-        return self._latent_part(q, w, m, kv, pool, meta)
+    def latent_attention(self, q, gate, w, m, kv, pool, meta):
+        o = [self._latent_part(q[s], None if gate is None else gate[s], w, m, kv, pool, mt) for s, mt in self._parts(meta)]
+        return o[0] if len(o) == 1 else torch.cat(o)  # mixed step: each part its own kernel
 
-    def _latent_part(self, q, w, m, kv, pool, meta):
+    def _latent_part(self, q, gate, w, m, kv, pool, meta):
         window = m.window or 1 << 30
+        beside = (m.kv_rank, w("attn.sink") if m.sink else None)
         uk, uv = w("attn.uk.weight"), w("attn.uv.weight")
         rows = self.C.latent_tile_rows(pool.shape[2])
         if not self.fp32 and not meta.is_decode and q.shape[0] >= self.R.latent_expand_t:
             reach = self._latent_reach(meta, m.window)
-            if reach is not None and uk.shape[2] <= 128 and uv.shape[1] <= 128 and self.R.latent_expand(
+            if reach is not None and uk.shape[2] <= 192 and uv.shape[1] <= 128 and self.R.latent_expand(
                     q.shape[0], reach[3], reach[2], uk.shape[2], uv.shape[1], pool.shape[2]):
-                return self._latent_expanded(q, w, m, kv, pool, meta, window, reach)
+                return self._latent_expanded(q, gate, w, m, kv, pool, meta, window, reach)
         q = self._batch_linear(q, uk)
         if meta.is_decode or self.fp32 or rows == 0:
             # one query per sequence, or the kernel that takes any token alone
             splits = self.R.latent_splits(q.shape[0], m.heads, min(window, meta.max_ctx))
             o = self.C.latent_decode(q, pool, kv.table, meta.token_slots, meta.token_pos, m.heads, window, m.scale,
-                                     splits)
+                                     splits, *beside)
         else:
             o = self.C.latent_prefill(q, pool, kv.table, self._latent_tiles(meta, m.heads, rows, q.device),
-                                      meta.seq_slots, meta.q_start, meta.cu_q, m.heads, window, m.scale)
-        return self._batch_linear(o, uv)
+                                      meta.seq_slots, meta.q_start, meta.cu_q, m.heads, window, m.scale, *beside)
+        return self._batch_linear(o, uv, gate)
 
-    def _latent_expanded(self, q, w, m, kv, pool, meta, window, reach):
+    def _latent_expanded(self, q, gate, w, m, kv, pool, meta, window, reach):
         """Keys and values of every row in reach made once, then per-head attention."""
         k_lo, cu_k, rows, _ = reach
         c = self.C.latent_gather(pool, kv.table, meta.seq_slots, k_lo, cu_k, rows)
         k = self.linear(c, w("attn.uk_rows.weight"))
         uv = w("attn.uv.weight")
-        v = self.linear(c, uv.reshape(-1, uv.shape[2]))
+        v = self.linear(c[:, : uv.shape[2]], uv.reshape(-1, uv.shape[2]))
         return self.C.latent_expanded(q, k, v, self._latent_tiles(meta, 1, 128, q.device), meta.cu_q, meta.q_start,
-                                      k_lo, cu_k, m.heads, window, m.scale)
+                                      k_lo, cu_k, m.heads, window, m.scale, w("attn.sink") if m.sink else None, gate)
 
     @staticmethod
     def _latent_reach(meta, window):
@@ -718,10 +920,10 @@ class HipBackend(Backend):
             for rows in {self.C.talk_tile(hp) for hp in (8, 16, 32)} | {64, 128}:
                 self._query_tiles(meta, rows, meta.cu_q.device)
             return
-        if mcfg.arch != "timisun":
+        if not mcfg.layers:
             meta._tiles = prefill_tiles(meta).to(meta.cu_q.device)
             return
-        for heads in {l.mixer.heads for l in mcfg.layers}:
+        for heads in {l.mixer.heads for l in mcfg.layers if isinstance(l.mixer, LatentAttentionSpec)}:
             self._latent_tiles(meta, heads, 128, meta.cu_q.device)
 
     def parallel_residual(self, o, h, routing, w, mlp, r: Residual) -> None:
@@ -736,25 +938,34 @@ class HipBackend(Backend):
         T, H = h.shape
         if not self.fp32 and T <= self.R.moe_few_t:
             self.linear_residual(o, wo, None, r)
-            sh = mlp.shared
-            self.C.moe_few(h, ids, wts, w("mlp.experts.gate_up.weight"), w("mlp.experts.down.weight"),
-                           mlp.expert.limit, GLU_ALPHA, w("mlp.shared.gate_up.weight") if sh else None,
-                           w("mlp.shared.down.weight") if sh else None, sh.limit if sh else 0.0, r.x)
+            self._moe_few(h, ids, wts, w, mlp, r.x, None, True)
             return
-        tm = self._tm(T * mlp.top / mlp.experts)
         shared = mlp.shared is not None
         so = self._slab_splits(o, wo)
         if so and bool(self.C.gemm_slab_bf16()) != (h.dtype == torch.bfloat16):
             so = 0  # slabs of two element types: the out-projection keeps its own
         slab = torch.empty(so + mlp.top + shared, T, H, dtype=h.dtype, device=h.device)
         self.linear_residual(o, wo, None, r, slab[:so] if so else None)
-        perm, tiles = self.C.moe_group(ids, mlp.experts, tm)
-        mid, mids = self.C.moe_up(h, perm, tiles, mlp.top, w("mlp.experts.gate_up.weight"), mlp.expert.limit,
-                                  GLU_ALPHA, w("mlp.shared.gate_up.weight") if shared else None,
-                                  mlp.shared.limit if shared else 0.0, tm)
-        self.C.moe_down(mid, mids if shared else None, perm, tiles, wts, w("mlp.experts.down.weight"),
-                        w("mlp.shared.down.weight") if shared else None, slab[so:], tm)
+        self._moe(h, ids, wts, w, mlp, slab[so:], None)
         r.pending.append((slab, None))
+
+    def _moe_few(self, h, ids, wts, w, mlp, x, shared_wts, add: bool) -> None:
+        """x (+)= experts of a few tokens, weights streamed."""
+        sh = mlp.shared
+        self.C.moe_few(h, ids, wts, w("mlp.experts.gate_up.weight"), w("mlp.experts.down.weight"), mlp.expert.limit or 0.0,
+                       GLU_ALPHA, w("mlp.shared.gate_up.weight") if sh else None, w("mlp.shared.down.weight") if sh else None,
+                       (sh.limit or 0.0) if sh else 0.0, x, shared_wts, add)
+
+    def _moe(self, h, ids, wts, w, mlp, slab, shared_wts) -> None:
+        """slab[k] = choice k's expert, slab[top] the shared one, weighed per token."""
+        tm = self._tm(h.shape[0] * mlp.top / mlp.experts)
+        shared = mlp.shared is not None
+        perm, tiles = self.C.moe_group(ids, mlp.experts, tm)
+        mid, mids = self.C.moe_up(h, perm, tiles, mlp.top, w("mlp.experts.gate_up.weight"), mlp.expert.limit or 0.0,
+                                  GLU_ALPHA, w("mlp.shared.gate_up.weight") if shared else None,
+                                  (mlp.shared.limit or 0.0) if shared else 0.0, tm)
+        self.C.moe_down(mid, mids if shared else None, perm, tiles, wts, w("mlp.experts.down.weight"),
+                        w("mlp.shared.down.weight") if shared else None, slab, tm, shared_wts)
 
     def _slab_splits(self, a, w) -> int:
         """Partial slabs linear_residual(a, w) leaves for the next norm (0: it
@@ -834,10 +1045,12 @@ class HipBackend(Backend):
             self.C.norm(x, slab, pb, None, None, 0.0, True, None, False)
 
     def flush(self, r: Residual):
-        if r.post is not None:
-            slab, bias, w_post, mcfg = r.post
-            r.post = None
-            self.C.group_norm(r.x, mcfg.norm_groups, mcfg.hidden, mcfg.norm_eps, slab, bias, w_post, None, None, self.fp32)
+        if r.post is not None and r.post.tanh:
+            self._tanh_step(r, False)
+        elif r.post is not None:
+            post, r.post = r.post, None
+            w_post, *parts = post.rms
+            self.C.group_norm(r.x, *parts, post.slab, post.bias, w_post, None, None, self.fp32)
         for slab, pb in r.pending:
             self._fold(r.x, slab, pb)
         r.pending.clear()

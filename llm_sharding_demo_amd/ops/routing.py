@@ -127,6 +127,10 @@ class Routing:
     # recurrent layers: prompts of more than chunk_min tokens per sequence on
     # average run in chunks, shorter ones token by token
     chunk_min: int = 4
+    # recurrences with forget gates: blocks a prompt launch aims for, segments of a
+    # sequence at least forget_tokens long
+    forget_target: int = 512
+    forget_tokens: int = 64
     # decode attention with mixed heads: blocks a launch aims for, two 64-key
     # tiles each unless that leaves half of them idle
     talk_target: int = 512
@@ -305,6 +309,12 @@ class Routing:
     def latent_splits(self, B: int, heads: int, keys: int) -> int:
         items = B * math.ceil(heads / 16)
         return max(1, min(math.ceil(self.latent_target / items), math.ceil((keys + 31) / 128), 64))
+
+    def forget_segments(self, items: int, tokens: int) -> int:
+        """Segments of every sequence in a chunked recurrence (items: sequences x
+        heads): two launches over all of them where that fills the chip."""
+        n = min(self.forget_target // max(1, items), math.ceil(tokens / self.forget_tokens), 16)
+        return n if n > 2 else 1
 
     def talk_splits(self, B: int, keys: int) -> int:
         """Context splits of a decode attention launch with mixed heads (one
