@@ -131,9 +131,9 @@ def latent_tokens(C, q, pool, table, pos, H, window, scale, splits=1):
 
 
 @DTYPES
-@pytest.mark.parametrize("rank", [64, 128, 192, 256, 320, 384, 448, 512, 576])
+@pytest.mark.parametrize("rank", [64, 128, 192, 256, 320, 384, 448, 512, 576, 640])
 def test_latent_attention_ranks(C, dtype, rank):
-    """Prefill and decode kernels on every instantiated rank (576: the kernel
+    """Prefill and decode kernels on every instantiated rank (640: the kernel
     without MFMA), heads over one 16-head group."""
     from llm_sharding_demo_amd.ops.hip import latent_tiles
 
