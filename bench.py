@@ -68,9 +68,10 @@ def parse():
                         "nothing measurable on one stage or in the 2/4-stage loopback rehearsal "
                         "(profiles/r2_prefill_chunk.log)")
     p.add_argument("--designs", default="",
-                   help="comma-separated presets with per-layer specs (timisun-2b, vizalix-2b, kedasun-2b, ...): instead of the "
-                        "headline, prefill and decode throughput of each beside a Llama-family model of equal "
-                        "width, depth, heads and active feed-forward (one GPU; one JSON line per model and batch)")
+                   help="comma-separated presets with per-layer specs (timisun-2b, vizalix-2b, kedasun-2b, fagunex-2b, ...): "
+                        "instead of the headline, prefill and decode throughput of each beside a Llama-family model of equal "
+                        "width, depth, heads and active feed-forward -- fagunex beside a Timisun model of equal width, "
+                        "depth, heads, latents and experts (one GPU; one JSON line per model and batch)")
     p.add_argument("--design-batches", default="1,32,256")
     p.add_argument("--device", default="cuda",
                    help="cuda (MI355X); cpu only to rehearse the multi-rank contract with gloo")
@@ -121,6 +122,22 @@ def dense_twin(name: str) -> str:
     return twin
 
 
+def latent_twin(name: str) -> str:
+    """Preset of the Timisun model of a design's size: same width, depth,
+    vocabulary, heads, latent rank, window and experts."""
+    from llm_sharding_demo_amd.config import MODEL_PRESETS, _timisun, _timisun_layers
+
+    mc = MODEL_PRESETS[name]
+    m = next(l.mixer for l in mc.layers if l.mixer.cached_per_token)
+    window = next((l.mixer.window for l in mc.layers if getattr(l.mixer, "window", None)), None)
+    f = mc.layers[0].mlp
+    twin = f"{name}-timisun"
+    MODEL_PRESETS[twin] = _timisun(twin, mc.vocab_size, mc.hidden, _timisun_layers(
+        mc.n_layers, heads=m.heads, dim=m.dim, vdim=m.vdim, kv_rank=m.kv_rank, scale=m.dim ** -0.5, window=window,
+        experts=f.experts, top=f.top, ff=f.expert.ff, shared_ff=f.shared.ff))
+    return twin
+
+
 def bench_designs(args) -> int:
     """--designs: one generation session per (model, batch) after a warm-up:
     prefill of batch x --prompt tokens, then --gen greedy decode steps."""
@@ -128,11 +145,12 @@ def bench_designs(args) -> int:
 
     import torch
 
-    from llm_sharding_demo_amd.config import EngineConfig, SamplingParams
+    from llm_sharding_demo_amd.config import EngineConfig, SamplingParams, get_model_config
     from llm_sharding_demo_amd.runtime.engine import Engine
 
     for name in args.designs.split(","):
-        for model in (name, dense_twin(name)):
+        twin = latent_twin if get_model_config(name).arch == "fagunex" else dense_twin
+        for model in (name, twin(name)):
             for B in (int(b) for b in args.design_batches.split(",")):
                 cfg = EngineConfig(model_id=model, max_batch=B, max_seq_len=args.prompt + args.gen,
                                    device=args.device, use_graphs=not args.no_graphs, num_microbatches=1,

@@ -377,6 +377,138 @@ __global__ __launch_bounds__(256, RANK <= 256 ? 2 : 1) void latent_decode_kernel
   }
 }
 
+// The same for wide rows: the four waves share a 64-key tile.  Each scores 16 of its
+// keys, the scores cross LDS, and each weighs a quarter of the value columns, so
+// that no wave holds a whole output row and two blocks fit a CU.
+template <int RANK, int VR>
+__global__ __launch_bounds__(256, 2) void latent_decode_wide_kernel(LatentAttnParams p) {
+  constexpr int KT = 64;
+  constexpr int LDR = RANK + 8;
+  constexpr int CPR = RANK / 8;
+  constexpr int CH = KT * CPR / 256;
+  constexpr int DW = VR / 64;  // 16-column tiles per wave
+  constexpr int LDSC = KT + 4;
+  __shared__ __attribute__((aligned(16))) bf16 cs[KT * LDR];
+  __shared__ __attribute__((aligned(16))) float sc[16 * LDSC];  // [head][key]
+  const int H = p.H, HG = (H + 15) / 16;
+  const int item = xcd_remap(blockIdx.x, gridDim.x);  // a token's head groups on one XCD
+  const int b = item / HG, h0 = (item % HG) * 16;
+  const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int pos = p.pos[b], lo = first_key(pos, p.window);
+  const int* table = p.table + (long)p.seq_slots[b] * p.tw;
+  const bf16* cache = static_cast<const bf16*>(p.cache);
+  const int t0 = lo / KT, nt = pos / KT + 1 - t0;
+  const int per = (nt + p.splits - 1) / p.splits;
+  const int ta = t0 + blockIdx.y * per, tb = min(ta + per, t0 + nt);
+
+  bf16x8 qf[RANK / 32];
+  const bf16* q = static_cast<const bf16*>(p.q) + ((long)b * H + min(h0 + r, H - 1)) * RANK;
+#pragma unroll
+  for (int kk = 0; kk < RANK / 32; ++kk) qf[kk] = ld8(q + kk * 32 + g * 8);
+  f32x4 o[DW];
+#pragma unroll
+  for (int di = 0; di < DW; ++di) o[di] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m = NEG, lsum = 0.f;
+  if (p.sink && blockIdx.y == 0) {  // a key that was seen first, without a value
+    m = p.sink[min(h0 + r, H - 1)] * LOG2E;
+    lsum = g == 0 ? 1.f : 0.f;
+  }
+  bf16x8 creg[CH];
+  auto load_tile = [&](int kt) {  // a tile is a page
+    const bf16* src = cache + (long)table[kt] * PAGE * RANK;
+#pragma unroll
+    for (int c = 0; c < CH; ++c) creg[c] = ld8(src + (threadIdx.x + c * 256) * 8);
+  };
+  if (ta < tb) load_tile(ta);
+  for (int kt = ta; kt < tb; ++kt) {
+    __syncthreads();  // the previous tile's readers are done
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+      const int idx = threadIdx.x + c * 256;
+      st8(cs + (idx / CPR) * LDR + (idx % CPR) * 8, creg[c]);
+    }
+    __syncthreads();
+    if (kt + 1 < tb) load_tile(kt + 1);  // in flight under this tile's math
+
+    f32x4 s = {0.f, 0.f, 0.f, 0.f}, s2 = s;  // two chains
+    const bf16* row = cs + (w * 16 + r) * LDR + g * 8;
+#pragma unroll
+    for (int kk = 0; kk < RANK / 32; kk += 2) {
+      s = mfma16(*reinterpret_cast<const bf16x8*>(row + kk * 32), qf[kk], s);
+      s2 = mfma16(*reinterpret_cast<const bf16x8*>(row + kk * 32 + 32), qf[kk + 1], s2);
+    }
+    s += s2;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int key = kt * KT + w * 16 + 4 * g + i;
+      s[i] = key <= pos && key >= lo ? s[i] * p.scale_log2 : NEG;
+    }
+    *reinterpret_cast<f32x4*>(sc + r * LDSC + w * 16 + 4 * g) = s;
+    __syncthreads();
+    // k-slot j of group g <-> key 32 kk + 4 g + j (j < 4), 32 kk + 16 + 4 g + (j - 4)
+    f32x4 e[4];
+    float tmax = NEG;
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      e[c] = *reinterpret_cast<const f32x4*>(sc + r * LDSC + c * 16 + 4 * g);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) tmax = fmaxf(tmax, e[c][i]);
+    }
+    tmax = fmaxf(tmax, wave_xchg<16>(tmax));
+    tmax = fmaxf(tmax, wave_xchg<32>(tmax));
+    if (grew(tmax, m)) {
+      const float mn = fmaxf(m, tmax);
+      const float alpha = exp2f(m - mn);
+      m = mn;
+      lsum *= alpha;
+#pragma unroll
+      for (int di = 0; di < DW; ++di) o[di] *= alpha;
+    }
+#pragma unroll
+    for (int c = 0; c < 4; ++c)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        // every tile of the range holds a visible key, so m is a real score
+        e[c][i] = exp2f(e[c][i] - m);
+        lsum += e[c][i];
+      }
+    bf16x8 ph[2], pl[2];
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) split_p(e[2 * kk], e[2 * kk + 1], ph[kk], pl[kk]);
+    const int r0 = 4 * g + (r >> 2);
+#pragma unroll
+    for (int di = 0; di < DW; ++di) {
+      const int col = (w * DW + di) * 16 + 4 * (r & 3);
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk) {
+        const bf16x4 a = ds_read_tr(cs + (kk * 32 + r0) * LDR + col);
+        const bf16x4 c = ds_read_tr(cs + (kk * 32 + r0 + 16) * LDR + col);
+        const bf16x8 vf = {a[0], a[1], a[2], a[3], c[0], c[1], c[2], c[3]};
+        o[di] = mfma16(vf, ph[kk], o[di]);
+        o[di] = mfma16(vf, pl[kk], o[di]);
+      }
+    }
+  }
+  lsum += wave_xchg<16>(lsum);
+  lsum += wave_xchg<32>(lsum);
+  const int h = h0 + r;
+  if (h >= H) return;
+  // column tile 16 (w DW + di): rows 4 g + i of O^T are its columns, lane r the head
+  const float inv = 1.f / lsum;
+  const long pi = ((long)b * H + h) * p.splits + blockIdx.y;
+#pragma unroll
+  for (int di = 0; di < DW; ++di) {
+    const int d = (w * DW + di) * 16 + 4 * g;
+    if (p.splits > 1) *reinterpret_cast<f32x4*>(p.part_o + pi * VR + d) = o[di];
+    else st4(static_cast<bf16*>(p.out) + ((long)b * H + h) * VR + d, pack4(o[di] * inv));
+  }
+  if (p.splits > 1 && w == 0 && g == 0) {
+    p.part_ml[2 * pi] = m;
+    p.part_ml[2 * pi + 1] = lsum;
+  }
+}
+
 // Latent rows of every sequence's reach, packed: row cu_k[i] + j of the output is
 // position k_lo[i] + j of sequence i (zeros before position 0).  One wave a row.
 __global__ __launch_bounds__(256) void latent_gather_kernel(const bf16* __restrict__ cache,
@@ -698,10 +830,18 @@ extern "C" hipError_t lsd_latent_prefill(const LatentAttnParams* p, hipStream_t 
   return hipGetLastError();
 }
 
+// rows from this width on are shared by the four waves of a block
+#ifndef WIDE_DECODE
+#define WIDE_DECODE 320
+#endif
 extern "C" hipError_t lsd_latent_decode(const LatentAttnParams* p, hipStream_t st) {
   if (p->B == 0) return hipSuccess;
   const dim3 grid(p->B * ((p->H + 15) / 16), p->splits);
-#define LSD_LD_V(R, V) hipLaunchKernelGGL((latent_decode_kernel<R, V>), grid, dim3(256), 0, st, *p)
+#define LSD_LD_V(R, V)                                                                                    \
+  do {                                                                                                     \
+    if constexpr (R >= WIDE_DECODE) hipLaunchKernelGGL((latent_decode_wide_kernel<R, V>), grid, dim3(256), 0, st, *p); \
+    else hipLaunchKernelGGL((latent_decode_kernel<R, V>), grid, dim3(256), 0, st, *p);                     \
+  } while (0)
 #define LSD_LD(R)                                         \
   case R:                                                 \
     if (p->v_pad == R) LSD_LD_V(R, R);                    \

@@ -15,6 +15,7 @@
 //    the device, so a captured decode graph follows the routing of each replay.
 #include "common.h"
 #include "moe_params.h"
+#include "route.h"
 
 namespace lsd {
 
@@ -28,76 +29,13 @@ __device__ __forceinline__ float narrow<float>(float v) { return v; }
 constexpr int LATENT_PAGE = 64;  // tokens per cache page
 constexpr int MAX_EXPERTS = 1024;
 
-// One row's routing by one wave; EPL: experts per lane.
-template <int EPL>
-__device__ __forceinline__ void route_row(const RouteParams& p, const float* z, int t) {
-  const int lane = lane_id();
-  float sc[EPL], ch[EPL];
-#pragma unroll
-  for (int j = 0; j < EPL; ++j) {
-    const int e = lane + 64 * j;
-    const bool ok = e < p.experts;
-    const float v = ok ? z[e] : 0.f;
-    sc[j] = p.correction ? 1.f / (1.f + expf(-v)) : v;
-    ch[j] = !ok ? -INFINITY : p.correction ? sc[j] + p.correction[e] : sc[j];
-  }
-  if (p.shared && lane == 0) p.shared[t] = 1.f / (1.f + expf(-z[p.experts]));
-  float sum = 0.f, mine = 0.f, best = 0.f;
-  for (int k = 0; k < p.top; ++k) {
-    // best corrected score of the wave; the lower expert wins a tie
-    float b = -INFINITY;
-    int be = 0x7fffffff;
-#pragma unroll
-    for (int j = 0; j < EPL; ++j)
-      if (ch[j] > b) {
-        b = ch[j];
-        be = lane + 64 * j;
-      }
-#pragma unroll
-    for (int m = 32; m >= 1; m >>= 1) {
-      const float ob = __shfl_xor(b, m, 64);
-      const int oe = __shfl_xor(be, m, 64);
-      if (ob > b || (ob == b && oe < be)) {
-        b = ob;
-        be = oe;
-      }
-    }
-    // scores that are not numbers never win: keep the ids in range
-    if (be >= p.experts) be = k;
-    float s = 0.f;
-#pragma unroll
-    for (int j = 0; j < EPL; ++j)
-      if (be == lane + 64 * j) {
-        s = sc[j];
-        ch[j] = -INFINITY;
-      }
-    s = __shfl(s, be & 63, 64);
-    if (!p.correction) {  // softmax over the chosen logits, the first the largest
-      if (k == 0) best = s;
-      s = expf(s - best);
-    }
-    sum += s;
-    if (lane == (k & 63)) {
-      if (k >= 64) {  // more choices than lanes: park the earlier ones
-        p.wts[(long)t * p.top + k - 64] = mine;
-      }
-      mine = s;
-      p.ids[(long)t * p.top + k] = be;
-    }
-  }
-  // divide by the sum: lane l holds choice k = l (+ 64 when top > 64)
-  const float inv = 1.f / (sum + 1e-20f);
-  for (int k = lane; k < p.top; k += 64) {
-    const bool held = k + 64 >= p.top;
-    p.wts[(long)t * p.top + k] = (held ? mine : p.wts[(long)t * p.top + k]) * inv;
-  }
-}
-
 // One wave per row of router logits that stand alone
 template <int EPL>
 __global__ __launch_bounds__(256) void route_kernel(RouteParams p) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (t < p.T) route_row<EPL>(p, p.z + (long)t * p.ldz, t);
+  if (t >= p.T) return;
+  if (EPL == 1 && !p.correction) route_few(p, p.z + (long)t * p.ldz, t);
+  else route_row<EPL>(p, p.z + (long)t * p.ldz, t);
 }
 
 // Column c of a head turned: pairs (rot + i, rot + i + half)
@@ -131,17 +69,38 @@ __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostParams p) {
 #pragma unroll 8
         for (int i = lane; i < p.nq; i += 64) q[i] = narrow<T>(i < p.q_rank ? y[i] * rstd * p.q_gain[i] : 0.f);
       }
-    } else if constexpr (sizeof(T) == 2) {
-      for (int c = id * 4; c < p.nq; c += step * 4) {
-        f32x4 v = *reinterpret_cast<const f32x4*>(y + c);
-        if (p.half) {  // heads are a multiple of four columns wide
-          const int at = c % p.q_head;
-          if (at + 3 >= p.q_rot && at < p.q_rot + 2 * p.half) {
+    } else if (sizeof(T) == 2 && (p.half == 0 || (p.q_rot % 4 == 0 && p.half % 4 == 0))) {
+      // a wave takes a head (or 256 columns where nothing turns) at a time: what a lane
+      // turns, and by how much, is the same for all of them
+      const int span = p.half ? p.q_head : 256, nh = (p.nq + span - 1) / span, nw = 4 - w0;
+      for (int at = lane * 4; at < span; at += 256) {
+        const int j = at - p.q_rot;
+        const bool in = p.half && j >= 0 && j < 2 * p.half;
+        const int other = !in ? 0 : j < p.half ? p.half : -p.half;
+        f32x4 co = {1.f, 1.f, 1.f, 1.f}, si = {0.f, 0.f, 0.f, 0.f};
+        if (in) {
+          const float* c = cs + 2 * (j < p.half ? j : j - p.half);
 #pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] = turned(y + c - at, at + e, p.q_rot, p.half, cs);
+          for (int e = 0; e < 4; ++e) {
+            co[e] = c[2 * e];
+            si[e] = j < p.half ? -c[2 * e + 1] : c[2 * e + 1];
           }
         }
-        st4(reinterpret_cast<bf16*>(q) + c, pack4(v));
+        constexpr int FLY = 4;
+        for (int h = w - w0; h < nh; h += FLY * nw) {
+          f32x4 v[FLY], u[FLY];
+#pragma unroll
+          for (int i = 0; i < FLY; ++i) {
+            const int c = min(min(h + i * nw, nh - 1) * span + at, p.nq - 4);
+            v[i] = *reinterpret_cast<const f32x4*>(y + c);
+            u[i] = p.half ? *reinterpret_cast<const f32x4*>(y + c + other) : v[i];
+          }
+#pragma unroll
+          for (int i = 0; i < FLY; ++i) {
+            const int c = (h + i * nw) * span + at;
+            if (h + i * nw < nh && c < p.nq) st4(reinterpret_cast<bf16*>(q) + c, pack4(p.half ? v[i] * co + u[i] * si : v[i]));
+          }
+        }
       }
     } else {
       for (int c = id; c < p.nq; c += step)

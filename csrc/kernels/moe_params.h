@@ -62,6 +62,19 @@ struct RouteParams {
   float* shared;                                    // [T] sigmoid of the column behind the logits, or null
 };
 
+// Narrow projections with what follows them: a w^T of rows a [T][K] (bf16), then the
+// routing of the logits (r.experts > 0, all columns in one block), or
+// out = gelu(.) * table[ids[t]].
+struct RowsParams {
+  const void* a; long lda;
+  const void* w; long ldw;                          // [N][K]
+  int T, N, K;                                      // K % 64 == 0, N % 16 == 0
+  RouteParams r;                                    // z unused
+  int splits; float* part; int* counters;           // router: K splits, [row tiles][splits][16][columns], tickets (zero)
+  const int* ids; const void* table; int vocab;     // [vocab][N]
+  void* out; long ldo;
+};
+
 // One token row behind a layer's input projection y (fp32): the latent columns
 // are normed and appended to the paged cache with the turned key part behind them,
 // the query columns narrowed and their last `rot` columns per head turned -- or

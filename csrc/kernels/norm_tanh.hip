@@ -102,9 +102,10 @@ __global__ __launch_bounds__(256) void tanh_step_kernel(TanhStepParams p) {
 }
 
 // One block per `run` rows; MAXC groups of four columns per thread.
-template <typename T, typename S, int MAXC, int FLY>
-__global__ __launch_bounds__(256) void shift_norm_kernel(ShiftNormParams p, int run) {
-  __shared__ float red[2][4];
+template <typename T, typename S, int NT, int MAXC, int FLY>
+__global__ __launch_bounds__(NT) void shift_norm_kernel(ShiftNormParams p, int run) {
+  constexpr int NW = NT / 64;
+  __shared__ float red[2][NW];
   const int row0 = blockIdx.x * run, row1 = min(p.T, row0 + run);
   const int tid = threadIdx.x, w = tid >> 6;
   typedef typename Quad<T>::type Q;
@@ -113,7 +114,7 @@ __global__ __launch_bounds__(256) void shift_norm_kernel(ShiftNormParams p, int 
   Q ws[MAXC], wn[MAXC], bn[MAXC], mx[MAXC];
 #pragma unroll
   for (int i = 0; i < MAXC; ++i) {
-    const int c = (tid + i * 256) * 4;
+    const int c = (tid + i * NT) * 4;
     on[i] = c < p.H;
     col[i] = min(c, p.H - 4);
     if (p.slab) ws[i] = vec4<T>(p.w_side, col[i]);
@@ -121,17 +122,27 @@ __global__ __launch_bounds__(256) void shift_norm_kernel(ShiftNormParams p, int 
     bn[i] = vec4<T>(p.pre.b, col[i]);
     mx[i] = vec4<T>(p.mix, col[i]);
   }
-  f32x4 x[MAXC], y[MAXC], prev[MAXC];
+  // bit i: row row0 - 1 + i continues the row before it
+  const int lane = lane_id(), at_row = row0 - 1 + lane;
+  const bool cont = lane <= run + 1 && at_row > 0 && at_row < p.T && p.tslot[at_row] == p.tslot[at_row - 1] &&
+                    p.tpos[at_row] == p.tpos[at_row - 1] + 1;
+  const unsigned long long conts = __ballot(cont);
+  auto follows = [&](int row) { return (conts >> (row - row0 + 1)) & 1; };
+  f32x4 x[MAXC], y[MAXC], prev[MAXC], kept[MAXC];
+  int slot = 0;
   auto load = [&](int row) {
     const long at = (long)row * p.H;
+    if (row >= row0 && !follows(row)) {  // a portion begins: the row in front of it is kept, or zero
+      slot = p.tslot[row];
+      const bool zero = p.tpos[row] == 0;
+#pragma unroll
+      for (int i = 0; i < MAXC; ++i) kept[i] = zero ? f32x4{0.f, 0.f, 0.f, 0.f} : get4(p.last + (long)slot * p.H + col[i]);
+    }
 #pragma unroll
     for (int i = 0; i < MAXC; ++i) {
       x[i] = get4(p.x + at + col[i]);
       if (p.slab) y[i] = slab_sum<S, FLY>(p.slab, p.splits, (long)p.T * p.H, at + col[i]);
     }
-  };
-  auto follows = [&](int row) {  // does this row continue the one before?
-    return row > 0 && row < p.T && p.tslot[row] == p.tslot[row - 1] && p.tpos[row] == p.tpos[row - 1] + 1;
   };
   const bool inside = follows(row0);
   const int first = inside ? row0 - 1 : row0;
@@ -139,10 +150,13 @@ __global__ __launch_bounds__(256) void shift_norm_kernel(ShiftNormParams p, int 
   bool own = false;  // the current portion began in this run
   for (int row = first; row < row1; ++row) {
     f32x4 v[MAXC], z[MAXC];
+    const bool begins = row >= row0 && !follows(row);
+    const int mine = slot;
 #pragma unroll
     for (int i = 0; i < MAXC; ++i) {
       v[i] = x[i];
       z[i] = y[i];
+      if (begins) prev[i] = kept[i];
     }
     if (row + 1 < row1) load(row + 1);  // in flight under the sum
     if (p.slab) {
@@ -155,7 +169,10 @@ __global__ __launch_bounds__(256) void shift_norm_kernel(ShiftNormParams p, int 
       float* rd = red[(row - first) & 1];  // alternating: one barrier a row
       if (lane_id() == 0) rd[w] = ss;
       __syncthreads();
-      const float rs = 1.f / sqrtf((rd[0] + rd[1] + rd[2] + rd[3]) / p.size + p.eps);
+      float all = 0.f;
+#pragma unroll
+      for (int i = 0; i < NW; ++i) all += rd[i];
+      const float rs = 1.f / sqrtf(all / p.size + p.eps);
 #pragma unroll
       for (int i = 0; i < MAXC; ++i) v[i] += z[i] * rs * wide4(ws[i]);
     }
@@ -163,13 +180,7 @@ __global__ __launch_bounds__(256) void shift_norm_kernel(ShiftNormParams p, int 
 #pragma unroll
     for (int i = 0; i < MAXC; ++i) h[i] = norm4<T>(p.pre.alpha, v[i], wide4(wn[i]), wide4(bn[i]));
     if (row >= row0) {
-      if (!follows(row)) {  // a portion begins: the row in front of it is kept, or zero
-        own = true;
-        const long at = (long)p.tslot[row] * p.H;
-        const bool zero = p.tpos[row] == 0;
-#pragma unroll
-        for (int i = 0; i < MAXC; ++i) prev[i] = zero ? f32x4{0.f, 0.f, 0.f, 0.f} : get4(p.last + at + col[i]);
-      }
+      own |= begins;
       const bool ends = own && !follows(row + 1);
 #pragma unroll
       for (int i = 0; i < MAXC; ++i) {
@@ -177,7 +188,7 @@ __global__ __launch_bounds__(256) void shift_norm_kernel(ShiftNormParams p, int 
         if (p.slab) put4(p.x_new + (long)row * p.H + col[i], v[i]);
         put4(static_cast<T*>(p.out) + (long)row * p.H + col[i], h[i] + (prev[i] - h[i]) * wide4(mx[i]));
         // read by this thread alone, above
-        if (ends) put4(p.last + (long)p.tslot[row] * p.H + col[i], h[i]);
+        if (ends) put4(p.last + (long)mine * p.H + col[i], h[i]);
       }
     }
 #pragma unroll
@@ -216,18 +227,21 @@ template <typename T, typename S>
 hipError_t shift_norm(const ShiftNormParams& p, hipStream_t st) {
   if (p.T == 0) return hipSuccess;
   const int run = p.T <= 1024 ? 1 : p.T <= 16384 ? 8 : 16;
-  const int chunks = (p.H + 1023) / 1024;
-#define LSD_SN(MAXC)                                                                                                    \
-  do {                                                                                                                  \
-    if (p.splits <= 1) hipLaunchKernelGGL((shift_norm_kernel<T, S, MAXC, 1>), dim3((p.T + run - 1) / run), dim3(256), 0, st, p, run); \
-    else hipLaunchKernelGGL((shift_norm_kernel<T, S, MAXC, 2>), dim3((p.T + run - 1) / run), dim3(256), 0, st, p, run);  \
+#define LSD_SN_F(NT, MAXC, FLY) \
+  hipLaunchKernelGGL((shift_norm_kernel<T, S, NT, MAXC, FLY>), dim3((p.T + run - 1) / run), dim3(NT), 0, st, p, run)
+#define LSD_SN(NT, MAXC)                      \
+  do {                                        \
+    if (p.splits <= 1) LSD_SN_F(NT, MAXC, 1); \
+    else LSD_SN_F(NT, MAXC, 2);               \
   } while (0)
-  if (chunks <= 1) LSD_SN(1);
-  else if (chunks <= 2) LSD_SN(2);
-  else if (chunks <= 4) LSD_SN(4);
-  else if (chunks <= 8) LSD_SN(8);
-  else if (chunks <= 16) LSD_SN(16);
+  const int chunks = (p.H + 2047) / 2048;  // of 512 threads
+  if (p.H <= 1024) LSD_SN(256, 1);
+  else if (chunks <= 1) LSD_SN(512, 1);
+  else if (chunks <= 2) LSD_SN(512, 2);
+  else if (chunks <= 4) LSD_SN(512, 4);
+  else if (chunks <= 8) LSD_SN(512, 8);
   else return hipErrorInvalidValue;
+#undef LSD_SN_F
 #undef LSD_SN
   return hipGetLastError();
 }

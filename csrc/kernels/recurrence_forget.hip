@@ -6,8 +6,8 @@
 //  * forget_chunk: prompts of bf16 models, up to 32 tokens at a time as matrix
 //    products around a state that stays in the accumulators of four waves, each
 //    owning columns of it.  Few sequences are cut in segments that run together:
-//    one launch leaves each segment's own state and decay, the next starts every
-//    segment from the sum of those before it.
+//    one launch leaves each segment's own state and decay, forget_join sums up what
+//    every segment starts from, and the segments run from there.
 //
 // Gates, their logarithms, decays and the state are fp32; fp32 operands enter the
 // matrix cores as two bf16 terms (16 bits).
@@ -140,13 +140,15 @@ __global__ __launch_bounds__(256, 2) void forget_chunk_kernel(ForgetParams p) {
   // state: rows d = 16 dt + 4 g + i, columns v = 16 (w VTW + j) + r
   f32x4 S[DT][VTW];
   auto save = [&](float* dst) {
+    int g4 = 4 * g;
+    asm volatile("" : "+v"(g4));  // addresses are formed anew: none stays in a register through the loop
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
       for (int j = 0; j < VTW; ++j)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const int d = dt * 16 + 4 * g + i, v = (w * VTW + j) * 16 + r;
+          const int d = dt * 16 + g4 + i, v = (w * VTW + j) * 16 + r;
           if (d < D && v < V) dst[d * p.Vp + v] = S[dt][j][i];
         }
   };
@@ -162,15 +164,8 @@ __global__ __launch_bounds__(256, 2) void forget_chunk_kernel(ForgetParams p) {
         }
   };
   if constexpr (MODE == FORGET_SEGMENT) {
-    const float* src = part(min(seg, 1));
+    const float* src = part(seg);
     each([&](float, int d, int v, bool in) { return in ? src[d * p.Vp + v] : 0.f; });
-    for (int k = 2; k <= seg; ++k) {
-      const float* own = part(k);
-      const float* dec = p.decay + (part0 + k) * D;
-      each([&](float s, int d, int v, bool in) {
-        return in ? s * __builtin_amdgcn_exp2f(dec[d]) + own[d * p.Vp + v] : 0.f;
-      });
-    }
   } else {
     const bool old = start > 0 && seg == 0;
     each([&](float, int d, int v, bool in) { return old && in ? Sg[d * p.Vp + v] : 0.f; });
@@ -440,6 +435,39 @@ __global__ __launch_bounds__(256, 2) void forget_chunk_kernel(ForgetParams p) {
   }
 }
 
+// What segments 2 .. start from: the state of the segment before, less its decay,
+// and that one's own.  A thread takes four columns of one row.
+__global__ __launch_bounds__(256) void forget_join_kernel(ForgetParams p) {
+  constexpr int FLY = 4;
+  const int q = p.Vp / 4, at = blockIdx.x * 256 + threadIdx.x;
+  if (at >= p.D * q) return;
+  const long part0 = ((long)blockIdx.z * p.heads + blockIdx.y) * p.segs;
+  const int n = p.s.cu[blockIdx.z + 1] - p.s.cu[blockIdx.z];
+  const int len = ((n + p.segs - 1) / p.segs + 31) / 32 * 32;  // as in forget_chunk
+  const int segs = n > 0 ? (n + len - 1) / len : 0;            // those that hold tokens
+  const long size = (long)p.D * p.Vp;
+  float* s = p.part + part0 * size + (at / q) * p.Vp + (at % q) * 4;
+  const float* dec = p.decay + part0 * p.D + at / q;
+  if (segs <= 2) return;
+  f32x4 acc = *reinterpret_cast<const f32x4*>(s + size);
+  for (int k = 2; k < segs; k += FLY) {
+    f32x4 own[FLY];
+    float d[FLY];
+#pragma unroll
+    for (int i = 0; i < FLY; ++i) {
+      const int c = min(k + i, segs - 1);
+      own[i] = *reinterpret_cast<const f32x4*>(s + c * size);
+      d[i] = dec[(long)c * p.D];
+    }
+#pragma unroll
+    for (int i = 0; i < FLY; ++i)
+      if (k + i < segs) {
+        acc = acc * __builtin_amdgcn_exp2f(d[i]) + own[i];
+        *reinterpret_cast<f32x4*>(s + (k + i) * size) = acc;
+      }
+  }
+}
+
 }  // namespace
 }  // namespace lsd
 
@@ -492,6 +520,8 @@ extern "C" hipError_t lsd_forget_chunk(const ForgetParams* p, hipStream_t st) {
   if (p->segs == 1) LSD_FC(DKS, VTW, FORGET_WHOLE, 1);       \
   else {                                                     \
     LSD_FC(DKS, VTW, FORGET_STATES, p->segs - 1);            \
+    if (p->segs > 2)                                         \
+      hipLaunchKernelGGL(forget_join_kernel, dim3((p->D * p->Vp / 4 + 255) / 256, p->heads, p->s.B), dim3(256), 0, st, *p); \
     LSD_FC(DKS, VTW, FORGET_SEGMENT, p->segs);               \
   }
 #define LSD_FC_V(DKS)                       \

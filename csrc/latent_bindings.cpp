@@ -19,6 +19,7 @@ using lsd::LatentAttnParams;
 using lsd::LatentPostParams;
 using lsd::MoeGemvParams;
 using lsd::RouteParams;
+using lsd::RowsParams;
 
 extern "C" {
 hipError_t lsd_group_gemm(const GgParams* p, int mode, int tm, hipStream_t st);
@@ -27,6 +28,8 @@ hipError_t lsd_moe_gemv_up(const MoeGemvParams* p, hipStream_t st);
 hipError_t lsd_moe_gemv_down(const MoeGemvParams* p, hipStream_t st);
 hipError_t lsd_latent_post(const LatentPostParams* p, int f32, hipStream_t st);
 hipError_t lsd_route(const RouteParams* p, hipStream_t st);
+hipError_t lsd_router(const RowsParams* p, hipStream_t st);
+hipError_t lsd_side_gate(const RowsParams* p, hipStream_t st);
 hipError_t lsd_side_mul(const void* g, const int* ids, const void* table, void* out, int T, int n, int vocab, int f32,
                         hipStream_t st);
 int lsd_latent_value_cols(int rank_pad, int rank);
@@ -399,6 +402,56 @@ std::vector<torch::Tensor> route_softmax(torch::Tensor z, int64_t experts, int64
   return {ids, wts, sh};
 }
 
+// rows a [T, K], w [N, K] of a narrow projection (bf16)
+RowsParams rows_of(const torch::Tensor& a, const torch::Tensor& w) {
+  need(a, torch::kBFloat16, "a");
+  need(w, torch::kBFloat16, "w");
+  need_rows(a, "a");
+  need_rows(w, "w");
+  RowsParams p{};
+  p.a = a.data_ptr(); p.lda = a.stride(0); p.w = w.data_ptr(); p.ldw = w.stride(0);
+  p.T = a.size(0); p.N = w.size(0); p.K = w.size(1);
+  TORCH_CHECK(a.size(1) == p.K && p.K % 64 == 0 && p.N % 16 == 0, "narrow projection: a [T, K], w [N, K], K % 64, N % 16");
+  return p;
+}
+
+// route_softmax of a w^T in one launch (at most 64 columns); splits of K; counters:
+// int32 tickets, zero at rest
+std::vector<torch::Tensor> router(torch::Tensor a, torch::Tensor w, int64_t experts, int64_t top, bool shared,
+                                  int64_t splits, torch::Tensor counters) {
+  RowsParams p = rows_of(a, w);
+  TORCH_CHECK(p.N <= 64 && experts >= 1 && experts + (shared ? 1 : 0) <= p.N && top >= 1 && top <= experts, "router sizes");
+  auto f32 = a.options().dtype(torch::kFloat32);
+  auto ids = torch::empty({p.T, top}, a.options().dtype(torch::kInt32));
+  auto wts = torch::empty({p.T, top}, f32);
+  auto sh = torch::empty({shared ? p.T : 0}, f32);
+  p.r.T = p.T; p.r.experts = experts; p.r.top = top;
+  p.r.ids = ids.data_ptr<int>(); p.r.wts = wts.data_ptr<float>();
+  if (shared) p.r.shared = sh.data_ptr<float>();
+  torch::Tensor part;
+  p.splits = std::max<int64_t>(1, std::min<int64_t>(splits, p.K / 64));
+  if (p.splits > 1) {
+    const int64_t tiles = (p.T + 15) / 16, cols = p.N <= 16 ? 16 : p.N <= 32 ? 32 : 64;
+    part = torch::empty({tiles * p.splits * 16 * cols}, f32);
+    p.part = part.data_ptr<float>();
+    p.counters = const_cast<int*>(iptr(counters, tiles, "counters"));
+  }
+  check_hip(lsd_router(&p, cur_stream()), "router");
+  return {ids, wts, sh};
+}
+
+// gelu(a w^T) times rows ids of table [vocab, N] in one launch
+torch::Tensor side_gate(torch::Tensor a, torch::Tensor w, torch::Tensor ids, torch::Tensor table) {
+  RowsParams p = rows_of(a, w);
+  need(table, torch::kBFloat16, "table");
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && table.size(1) == p.N, "table must be [vocab, N]");
+  auto out = torch::empty({p.T, p.N}, a.options());
+  p.ids = iptr(ids, p.T, "ids"); p.table = table.data_ptr(); p.vocab = table.size(0);
+  p.out = out.data_ptr(); p.ldo = p.N;
+  check_hip(lsd_side_gate(&p, cur_stream()), "side_gate");
+  return out;
+}
+
 // rows g [T, n] times rows ids of table [vocab, n] (fp32: gelu(g) times them)
 torch::Tensor side_mul(torch::Tensor g, torch::Tensor ids, torch::Tensor table) {
   const bool f32 = is_f32(g, "g");
@@ -575,6 +628,9 @@ void lsd_register_latent(pybind11::module& m) {
         py::arg("correction"), py::arg("top"), py::arg("c_off") = -1, py::arg("rope") = py::none(), py::arg("q_head") = 0,
         py::arg("q_rot") = 0, py::arg("q_gain") = py::none());
   m.def("route_softmax", &route_softmax, py::arg("z"), py::arg("experts"), py::arg("top"), py::arg("shared"));
+  m.def("router", &router, py::arg("a"), py::arg("w"), py::arg("experts"), py::arg("top"), py::arg("shared"),
+        py::arg("splits"), py::arg("counters"));
+  m.def("side_gate", &side_gate, py::arg("a"), py::arg("w"), py::arg("ids"), py::arg("table"));
   m.def("side_mul", &side_mul, py::arg("g"), py::arg("ids"), py::arg("table"));
   m.def("latent_value_cols", [](int64_t rank_pad, int64_t rank) { return lsd_latent_value_cols((int)rank_pad, (int)rank); });
   m.def("latent_tile_rows", [](int64_t rank) { return lsd_latent_tile_rows((int)rank); });

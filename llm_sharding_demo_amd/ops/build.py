@@ -28,7 +28,7 @@ ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 
 KERNELS = ["gemm.hip", "gemv.hip", "norm.hip", "attention.hip", "sample.hip", "loopback.hip", "elementwise.hip",
-           "group_gemm.hip", "moe.hip", "attention_latent.hip", "attention_talk.hip", "attention_paged.hip", "recurrence.hip",
+           "group_gemm.hip", "gemm_rows.hip", "moe.hip", "attention_latent.hip", "attention_talk.hip", "attention_paged.hip", "recurrence.hip",
            "recurrence_forget.hip", "norm_group.hip", "norm_tanh.hip"]
 # host code of the extension: kernel bindings, native RCCL communicator, native stage
 # executor, device loopback channels (single-GPU rehearsal of the RCCL edges),

@@ -686,10 +686,13 @@ class HipBackend(Backend):
     def experts_tanh(self, h, w, mlp, n, r: Residual) -> None:
         """x += norm(experts(h)), left to the next norm: one slab per choice and the
         shared expert's."""
-        ids, wts, shared = self.C.route_softmax(self._linear_f32(h, w("mlp.router.weight")), mlp.experts, mlp.top,
-                                                mlp.shared_gate)
+        wr, (T, H) = w("mlp.router.weight"), h.shape
+        args = (mlp.experts, mlp.top, mlp.shared_gate)
+        if not self.fp32 and wr.shape[0] <= 64 and T <= self.R.rows_few_t:
+            ids, wts, shared = self.C.router(h, wr, *args, self.R.router_splits(T, wr.shape[1]), self.counters)
+        else:
+            ids, wts, shared = self.C.route_softmax(self._linear_f32(h, wr), *args)
         shared = shared if mlp.shared_gate else None
-        T, H = h.shape
         if not self.fp32 and T <= self.R.moe_few_t:
             slab = torch.empty(1, T, H, dtype=torch.float32, device=h.device)
             self._moe_few(h, ids, wts, w, mlp, slab[0], shared, False)
@@ -702,8 +705,11 @@ class HipBackend(Backend):
         """x += rms(proj(gelu(gate x) * e)) * norm, e the tokens' rows of the layer's
         table; the norm is left to the next layer."""
         x = self._tanh_step(r, True)
-        g = self._linear_f32(x, w("side.gate")) if self.fp32 else self.linear(x, w("side.gate"), act="gelu")
-        g = self.C.side_mul(g, ids, w("side.embed"))
+        wg, e = w("side.gate"), w("side.embed")
+        if not self.fp32 and x.shape[0] <= self.R.rows_few_t:
+            g = self.C.side_gate(x, wg, ids, e)
+        else:
+            g = self.C.side_mul(self._linear_f32(x, wg) if self.fp32 else self.linear(x, wg, act="gelu"), ids, e)
         r.post = PostNorm(self._slabs(g, w("side.proj"), r.x), rms=(w("side.norm"), 1, mcfg.hidden, mcfg.norm_eps))
 
     def forget_mix(self, h, w, m, state, meta, eps):

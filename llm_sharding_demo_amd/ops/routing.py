@@ -116,6 +116,11 @@ class Routing:
     # row tiles that walk an expert's columns together in a long prompt (8: down
     # projection 702 -> 787 TF/s over 4)
     moe_group_rows: int = 8
+    # up to this many tokens, narrow projections (routers, token-side gates) take 16
+    # rows a block; a router's K in splits of at least router_k, towards router_target blocks
+    rows_few_t: int = 1024
+    router_k: int = 256
+    router_target: int = 256
     # up to this many tokens, experts stream their weights per (token, choice)
     moe_few_t: int = 4
     # latent decode attention: workgroups (16 heads of a sequence x splits) a
@@ -315,6 +320,9 @@ class Routing:
         heads): two launches over all of them where that fills the chip."""
         n = min(self.forget_target // max(1, items), math.ceil(tokens / self.forget_tokens), 16)
         return n if n > 2 else 1
+
+    def router_splits(self, T: int, K: int) -> int:
+        return max(1, min(self.router_target // math.ceil(T / 16), K // self.router_k, 16))
 
     def talk_splits(self, B: int, keys: int) -> int:
         """Context splits of a decode attention launch with mixed heads (one

@@ -127,6 +127,25 @@ def test_softmax_routing(C, E, top, shared):
     assert err(sh, orc.sigmoid(z[:, E])) < 1e-5 if shared else sh.numel() == 0
 
 
+@pytest.mark.parametrize("T,K,N", [(1, 64, 16), (16, 128, 32), (17, 512, 64), (130, 2048, 64), (40, 4160, 48)])
+def test_narrow_projections(C, T, K, N):
+    """Router and token-side gate in one launch each, rows and K shared among the waves."""
+    g = torch.Generator().manual_seed(T)
+    a, w = randn(g, T, K, dt=BF), rounded(torch.randn(N, K, generator=g) * 2 / K ** 0.5, BF)
+    z, tickets = a @ w.T, i32([0] * 16)
+    for E, top, shared in ((N, 1, False), (N - 1, 3, True), (5, 5, True)):
+        for splits in (1, 2, 5, 16):
+            ids, wts, sh = C.router(cuda(a, BF), cuda(w, BF), E, top, shared, splits, tickets)
+            for t in range(T):
+                order, want = orc.route(torch.ones(1, dtype=z.dtype), z[t, :E, None], top)
+                assert ids[t].tolist() == order and err(wts[t], want) < 1e-4
+            assert not shared or err(sh, orc.sigmoid(z[:, E])) < 1e-4
+            assert not tickets.any()
+    table, ids = randn(g, 11, N, dt=BF), [(7 * i) % 11 for i in range(T)]
+    out = C.side_gate(cuda(a, BF), cuda(w, BF), i32(ids), cuda(table, BF))
+    assert err(out, orc.gelu_tanh(z) * table[ids]) < 1e-2
+
+
 @pytest.mark.parametrize("T,E,top,ff,shared", [(1, 4, 2, 40, 24), (3, 6, 1, 64, 0), (4, 5, 5, 24, 72), (9, 4, 2, 40, 24),
                                                (70, 6, 3, 64, 96), (300, 5, 2, 48, 0), (700, 8, 2, 64, 40)])
 @pytest.mark.parametrize("dtype", ["bf16", "fp32"])
