@@ -22,8 +22,9 @@
 //    GEMMs) and a per-head flash kernel runs over them: (dim + vdim) / (2 rank)
 //    of the multiply-adds per score.
 //  * decode: a block takes 16 heads of one token; its 4 waves take key tiles
-//    in turn, each with a private LDS tile, merged at the end; long ranges are
-//    split over blocks (latent_combine).
+//    in turn, each with a private LDS tile, merged at the end, or (wide rows)
+//    share a tile and divide the value columns; long ranges are split over
+//    blocks (latent_combine).
 //  * plain: one (token, head) per block on the VALU -- fp32 models, and ranks
 //    without an MFMA instantiation.
 //
@@ -831,9 +832,7 @@ extern "C" hipError_t lsd_latent_prefill(const LatentAttnParams* p, hipStream_t 
 }
 
 // rows from this width on are shared by the four waves of a block
-#ifndef WIDE_DECODE
-#define WIDE_DECODE 320
-#endif
+constexpr int WIDE_DECODE = 320;
 extern "C" hipError_t lsd_latent_decode(const LatentAttnParams* p, hipStream_t st) {
   if (p->B == 0) return hipSuccess;
   const dim3 grid(p->B * ((p->H + 15) / 16), p->splits);
